@@ -7,6 +7,7 @@
   mcp        MCP tool server (stdio; --http for streamable HTTP)
   bridge     HTTP bridge (:3333)
   telemetry  alert loop
+  trace      replay a token trace through an engine (engine/trace.py)
   build      compile the native extensions in-tree
   config     print every environment setting (typed, defaults, current)
 
@@ -358,6 +359,7 @@ def main(argv=None):
             p.add_argument("--engine", action="append", default=[])
     sub.add_parser("worker", add_help=False)
     sub.add_parser("mcp", add_help=False)
+    sub.add_parser("trace", add_help=False)
     sub.add_parser("bridge")
     sub.add_parser("telemetry")
     sub.add_parser("build")
@@ -373,6 +375,9 @@ def main(argv=None):
     elif args.cmd == "worker":
         from .worker.main import main as wm
         wm(rest)
+    elif args.cmd == "trace":
+        from .engine.trace import main as tm
+        sys.exit(tm(rest))
     elif args.cmd == "mcp":
         from .mcp.server import main as mm
         sys.argv = [sys.argv[0]] + rest

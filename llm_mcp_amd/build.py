@@ -30,7 +30,7 @@ EXT = sysconfig.get_config_var("EXT_SUFFIX") or ".so"
 
 KERNEL_SOURCES = ["norm.hip", "rope_cache.hip", "attention.hip", "sampling.hip",
                   "elementwise.hip", "gemm.hip", "dgemm.hip", "pgemm.hip",
-                  "rsgemm.hip", "allreduce.hip"]
+                  "rsgemm.hip", "allreduce.hip", "conv.hip", "linscan.hip"]
 RUNTIME_SOURCES = ["job_queue.cpp", "block_manager.cpp", "scheduler.cpp", "bindings.cpp"]
 
 
@@ -130,8 +130,11 @@ def build_kernels(force: bool = False, verbose: bool = False) -> Path:
     objdir = BUILD / "kernels"
     objdir.mkdir(parents=True, exist_ok=True)
     hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
+    # no packed fp32 instructions: hipcc forms them from ordinary float code and
+    # some of their forms have given wrong results on this hardware
     common = [hipcc, f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC",
-              "-munsafe-fp-atomics", f"-I{kdir}"]
+              "-munsafe-fp-atomics", "-Xclang", "-target-feature", "-Xclang",
+              "-packed-fp32-ops", f"-I{kdir}"]
     objs = []
     jobs = []
     audit_file = objdir / "resource_usage.json"

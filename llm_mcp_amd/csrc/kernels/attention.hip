@@ -111,7 +111,18 @@ __device__ __forceinline__ bf16x8_t kv_frag_2x8B(const bf16_t* p0, const bf16_t*
   }
 }
 
-template <int HD, bool NTL = false>
+// fp32 softmax weights as a bf16 pair: p = hi + lo to within 2^-17, so a PV
+// product of both parts keeps the weights' precision (SPLIT forms)
+__device__ __forceinline__ void split_weights(const float (&p)[8], bf16x8_t& hi, bf16x8_t& lo) {
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const uint16_t h = f2bf(p[j]);
+    hi[j] = (short)h;
+    lo[j] = (short)f2bf(p[j] - bf2f(h));
+  }
+}
+
+template <int HD, bool NTL = false, bool SPLIT = false>
 __device__ __forceinline__ void process_page(PageState<HD>& st, const bf16x8_t (&qf)[HD / 32],
                                              const bf16_t* __restrict__ kpage,
                                              const bf16_t* __restrict__ vpage, int page_pos0,
@@ -157,13 +168,18 @@ __device__ __forceinline__ void process_page(PageState<HD>& st, const bf16x8_t (
   rs = col4_sum(rs);
   st.l = st.l * alpha + rs;
   st.m = m_new;
-  bf16x8_t pf;
+  bf16x8_t pf, pl;
+  if constexpr (SPLIT) {
+    split_weights(p, pf, pl);
+  } else {
 #pragma unroll
-  for (int j = 0; j < 8; ++j) pf[j] = (short)f2bf(p[j]);
+    for (int j = 0; j < 8; ++j) pf[j] = (short)f2bf(p[j]);
+  }
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
     st.acc[i] *= alpha;
     st.acc[i] = mfma16(vf[i], pf, st.acc[i]);
+    if constexpr (SPLIT) st.acc[i] = mfma16(vf[i], pl, st.acc[i]);
   }
 }
 
@@ -477,6 +493,17 @@ __device__ __forceinline__ void rope_write_kv(const bf16_t* __restrict__ krow,
   }
 }
 
+// Optional output gate (ptr == nullptr: off): the finished output element is
+// multiplied by sigmoid(gate), gate rows laid out like the output rows.
+struct GateIn {
+  const bf16_t* ptr;
+  long stride;
+};
+__device__ __forceinline__ float gate_mul(const GateIn& gt, long row, long col, float o) {
+  if (!gt.ptr) return o;
+  return o / (1.f + __expf(-bf2f(gt.ptr[row * gt.stride + col])));
+}
+
 // Partition length used for a sequence: the requested split-K granule, grown
 // (in 128-token steps) when the context would need more than max_parts
 // partitions, so the grid baked into a captured graph always covers it.
@@ -493,7 +520,8 @@ __device__ __forceinline__ int effective_part(int ctx, int part_tokens, int max_
 // (two pages in flight per wave); MODE 2: loads only (diagnostic ceiling);
 // MODE 3: loads only, every instruction one contiguous 1 KB (diagnostic);
 // MODE 5: MODE 0 with non-temporal K/V loads; MODE 6: MODE 0 with a
-// block-table load per page.  MODE 0 / 5 read the segment's block ids once
+// block-table load per page; MODE 16: MODE 0 with fp32-precise softmax weights
+// (split_weights).  MODE 0 / 5 / 16 read the segment's block ids once
 // into a VGPR (lane i: page pg0 + i) and take them by readlane, so a page's
 // K/V loads do not wait on its block-table load.
 template <int HD>
@@ -509,7 +537,7 @@ __device__ __forceinline__ void decode_segment(
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ context_lens,
     bf16_t* __restrict__ out, long out_stride, float* __restrict__ part_o,
     float* __restrict__ part_ml, int Hq, int Hkv, float scale, int part_tokens, int max_parts,
-    const RopeIn rp) {
+    const RopeIn rp, const GateIn gt) {
   float (&sm_ml)[4][16][2] = sm.ml;
   float (&sm_o)[4][16][HD + 4] = sm.o;
   const int ctx = context_lens[b];
@@ -522,7 +550,7 @@ __device__ __forceinline__ void decode_segment(
   // page-loop control stay scalar (s_load / s_cbranch, no exec masking)
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int t0 = p * part_tokens, t1 = min(t0 + part_tokens, ctx);
-  constexpr bool kOnePage = MODE == 0 || MODE == 5 || MODE == 6;
+  constexpr bool kOnePage = MODE == 0 || MODE == 5 || MODE == 6 || MODE == 16;
   constexpr bool kRing = MODE == 9;
 
   bf16x8_t qf[HD / 32];
@@ -648,7 +676,7 @@ __device__ __forceinline__ void decode_segment(
       const long blk = blk_of(pg);
       const bf16_t* kp = k_cache + (blk * Hkv + kvh) * (BS * HD);
       const bf16_t* vp = v_cache + (blk * Hkv + kvh) * (BS * HD);
-      process_page<HD, MODE == 5>(st, qf, kp, vp, pg * BS, t1 - 1, scale_log2);
+      process_page<HD, MODE == 5, MODE == 16>(st, qf, kp, vp, pg * BS, t1 - 1, scale_log2);
     }
   } else {
     int pg = pg0 + wave;
@@ -715,7 +743,8 @@ __device__ __forceinline__ void decode_segment(
     }
     const int head = kvh * G + h;
     if (nparts == 1) {
-      out[(long)b * out_stride + (long)head * HD + d] = f2bf(O / L);
+      const long col = (long)head * HD + d;
+      out[(long)b * out_stride + col] = f2bf(gate_mul(gt, b, col, O / L));
     } else {
       const long idx = ((long)b * Hq + head) * max_parts + p;
       part_o[idx * HD + d] = O;
@@ -735,12 +764,12 @@ __global__ void __launch_bounds__(256) paged_decode_kernel(
     const int* __restrict__ context_lens, const int* __restrict__ order,
     bf16_t* __restrict__ out, long out_stride,
     float* __restrict__ part_o, float* __restrict__ part_ml, int Hq, int Hkv, float scale,
-    int part_tokens, int max_parts, RopeIn rp) {
+    int part_tokens, int max_parts, RopeIn rp, GateIn gt) {
   __shared__ DecodeSmem<HD> sm;
   decode_segment<HD, MODE>(sm, blockIdx.x, blockIdx.y, order ? order[blockIdx.z] : blockIdx.z, q,
                            q_stride, k_cache, v_cache, block_tables, bt_stride, context_lens,
                            out, out_stride, part_o, part_ml, Hq, Hkv, scale, part_tokens,
-                           max_parts, rp);
+                           max_parts, rp, gt);
 }
 
 // Persistent form (one partition per sequence): a fixed grid of about the
@@ -754,14 +783,14 @@ __global__ void __launch_bounds__(256, OCC) paged_decode_persist_kernel(
     const bf16_t* __restrict__ v_cache, const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ context_lens, const int* __restrict__ order,
     bf16_t* __restrict__ out, long out_stride, int B, int Hq, int Hkv, float scale,
-    int part_tokens, RopeIn rp) {
+    int part_tokens, RopeIn rp, GateIn gt) {
   __shared__ DecodeSmem<HD> sm;
   const int nseg = B * Hkv;
   for (int seg = blockIdx.x; seg < nseg; seg += gridDim.x) {
     const int r = seg / Hkv, kvh = seg - r * Hkv;
     decode_segment<HD, MODE>(sm, 0, kvh, order ? order[r] : r, q, q_stride, k_cache, v_cache,
                           block_tables, bt_stride, context_lens, out, out_stride, nullptr,
-                          nullptr, Hq, Hkv, scale, part_tokens, 1, rp);
+                          nullptr, Hq, Hkv, scale, part_tokens, 1, rp, gt);
     __syncthreads();            // the segment's LDS combine is read before the next reuses it
   }
 }
@@ -771,7 +800,7 @@ template <int HD>
 __global__ void __launch_bounds__(128) paged_decode_reduce_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     const int* __restrict__ context_lens, bf16_t* __restrict__ out, long out_stride, int Hq,
-    int part_tokens, int max_parts) {
+    int part_tokens, int max_parts, GateIn gt) {
   const int head = blockIdx.x, b = blockIdx.y, d = threadIdx.x;
   const int ctx = context_lens[b];
   part_tokens = effective_part(ctx, part_tokens, max_parts);
@@ -786,7 +815,8 @@ __global__ void __launch_bounds__(128) paged_decode_reduce_kernel(
     L += part_ml[(base + p) * 2 + 1] * f;
     O += part_o[(base + p) * HD + d] * f;
   }
-  out[(long)b * out_stride + (long)head * HD + d] = f2bf(O / L);
+  const long col = (long)head * HD + d;
+  out[(long)b * out_stride + col] = f2bf(gate_mul(gt, b, col, O / L));
 }
 
 // loop form (probe / A-B knob): 0 default -- the persistent grid when every
@@ -816,8 +846,10 @@ int paged_decode(const void* q, long q_stride, const void* k_cache, const void* 
                  long out_stride, float* part_o, float* part_ml, int B, int Hq, int Hkv, int D,
                  int block_size, float scale, int part_tokens, int max_parts,
                  const int* rope_positions, const float* cos_sin, const int* slots,
-                 hipStream_t stream) {
+                 const void* gate, long gate_stride, int split_p, hipStream_t stream) {
   if (B <= 0) return 0;
+  if (split_p && cos_sin) return -6;     // the split form has no rotary variant
+  const GateIn gt{(const bf16_t*)gate, gate_stride};
   if (cos_sin && (!rope_positions || !slots)) return -5;
   const RopeIn rp{rope_positions, cos_sin, slots};
   if ((D != 128 && D != 64) || block_size != BS) return -1;
@@ -828,27 +860,30 @@ int paged_decode(const void* q, long q_stride, const void* k_cache, const void* 
   paged_decode_kernel<HDV, MODE><<<dim3(max_parts, Hkv, B), dim3(256), 0, stream>>>(          \
       (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, \
       bt_stride, context_lens, order, (bf16_t*)out, out_stride, part_o, part_ml, Hq, Hkv,     \
-      scale, part_tokens, max_parts, rp);
+      scale, part_tokens, max_parts, rp, gt);
 #define LMX_DEC_P(HDV, MODE)                                                                  \
   paged_decode_persist_kernel<HDV, MODE><<<dim3(std::min(B * Hkv, decode_resident_wgs())), dim3(256), \
                                       0, stream>>>(                                           \
       (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, \
       bt_stride, context_lens, order, (bf16_t*)out, out_stride, B, Hq, Hkv, scale, part_tokens, \
-      rp);
+      rp, gt);
 #define LMX_DEC_R(HDV, OCC)                                                                   \
   paged_decode_persist_kernel<HDV, 9, OCC>                                                    \
       <<<dim3(std::min(B * Hkv, decode_resident_wgs(OCC))), dim3(256), 0, stream>>>(          \
       (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, \
       bt_stride, context_lens, order, (bf16_t*)out, out_stride, B, Hq, Hkv, scale, part_tokens, \
-      rp);
+      rp, gt);
   // mode 0 with no more segments than CUs (a TP rank's single kv head, e.g.
   // 256 rows x 1 kv head): one workgroup per segment, the grid form -- the
   // persistent form walks one segment per workgroup there anyway and measured
   // 22.2 vs 19.6 us (profiles/r5_proxy70.md)
-  const int mode = (g_decode_mode == 0 && max_parts == 1 && B * Hkv <= decode_resident_wgs(1))
+  const int mode = split_p ? (max_parts == 1 && B * Hkv > decode_resident_wgs(1) ? 16 : 17)
+                   : (g_decode_mode == 0 && max_parts == 1 && B * Hkv <= decode_resident_wgs(1))
                        ? 4 : g_decode_mode;
 #define LMX_DEC(HDV)                                                                          \
-  if (mode == 9 && max_parts == 1) { LMX_DEC_R(HDV, 2) }                                      \
+  if (mode == 16) { LMX_DEC_P(HDV, 16) }                                                      \
+  else if (mode == 17) { LMX_DEC_K(HDV, 16) }                                                 \
+  else if (mode == 9 && max_parts == 1) { LMX_DEC_R(HDV, 2) }                                      \
   else if (mode == 10 && max_parts == 1) { LMX_DEC_R(HDV, 3) }                       \
   else if ((mode == 9 || mode == 10)) { LMX_DEC_K(HDV, 9) }                 \
   else if (mode == 0 && max_parts == 1) { LMX_DEC_P(HDV, 0) }                        \
@@ -862,7 +897,7 @@ int paged_decode(const void* q, long q_stride, const void* k_cache, const void* 
   else { LMX_DEC_K(HDV, 0) }                                                                  \
   if (max_parts > 1)                                                                          \
     paged_decode_reduce_kernel<HDV><<<dim3(Hq, B), dim3(HDV), 0, stream>>>(                   \
-        part_o, part_ml, context_lens, (bf16_t*)out, out_stride, Hq, part_tokens, max_parts);
+        part_o, part_ml, context_lens, (bf16_t*)out, out_stride, Hq, part_tokens, max_parts, gt);
   if (D == 128) { LMX_DEC(128) } else { LMX_DEC(64) }
 #undef LMX_DEC
 #undef LMX_DEC_K
@@ -961,14 +996,16 @@ __device__ __forceinline__ void pf_vmwait() {
 // L2 / HBM into LDS are moved half as often -- the short causal walks of a
 // GQA prefill chunk (32 queries per 4-wave workgroup at G = 4) are bound by
 // that tile latency, not by the MFMAs.
-template <int HD, int NST, int PW = 4, int PF_NG = pf_groups<HD>()>
+// SPLIT: the softmax weights enter the PV product as a bf16 pair (high part +
+// remainder), i.e. with fp32 precision to within 2^-17.
+template <int HD, int NST, int PW = 4, bool SPLIT = false, int PF_NG = pf_groups<HD>()>
 __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
     const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ context_lens,
     const int* __restrict__ tiles, bf16_t* __restrict__ out, long out_stride, int Hq, int Hkv,
     float scale, int causal, float rescale_thr, int xcd, const int* __restrict__ rope_pos,
-    const float* __restrict__ rope_cs) {
+    const float* __restrict__ rope_cs, GateIn gt) {
   extern __shared__ __attribute__((aligned(16))) char pf_smem[];
   constexpr int PAGE = BS * HD;
   // buffer b: K pages at b*4*PAGE + {0, PAGE}, V pages at b*4*PAGE + 2*PAGE + {0, PAGE}
@@ -1131,7 +1168,7 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
     auto tile_body = [&](auto mask_tag) {
       constexpr bool MASK = decltype(mask_tag)::value;
       f32x4_t s[PF_NG][4];
-      bf16x8_t pf[PF_NG][2];
+      bf16x8_t pf[PF_NG][2], pl[SPLIT ? PF_NG : 1][2];
       bool need[PF_NG];
       float alpha[PF_NG];
       bf16x8_t kf[4][KS];
@@ -1205,6 +1242,12 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
             const uint32_t w = pack_bf16x2(x[4 * pp + j].x, x[4 * pp + j].y);
             pf[n][pp][2 * j] = (short)(w & 0xffff);
             pf[n][pp][2 * j + 1] = (short)(w >> 16);
+            if constexpr (SPLIT) {
+              const uint32_t r = pack_bf16x2(x[4 * pp + j].x - __uint_as_float(w << 16),
+                                             x[4 * pp + j].y - __uint_as_float(w & 0xffff0000u));
+              pl[n][pp][2 * j] = (short)(r & 0xffff);
+              pl[n][pp][2 * j + 1] = (short)(r >> 16);
+            }
           }
       };
       auto rescale = [&](int n) {
@@ -1244,11 +1287,14 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
 #pragma unroll
         for (int pp = 0; pp < 2; ++pp)
 #pragma unroll
-          for (int i = 0; i < NT; ++i) acc[n][i] = mfma16(vf[pp][i], pf[n][pp], acc[n][i]);
+          for (int i = 0; i < NT; ++i) {
+            acc[n][i] = mfma16(vf[pp][i], pf[n][pp], acc[n][i]);
+            if constexpr (SPLIT) acc[n][i] = mfma16(vf[pp][i], pl[n][pp], acc[n][i]);
+          }
       };
       pv(0);
       softmax(PF_NG - 1);
-      interleave(2 * NT);
+      interleave((SPLIT ? 4 : 2) * NT);
       __builtin_amdgcn_sched_barrier(0);
       rescale(PF_NG - 1);
       __builtin_amdgcn_sched_barrier(0);
@@ -1291,9 +1337,17 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
         *reinterpret_cast<const bf16x8_t*>(oimg + col * ROWB + 16 * (j ^ (col & (CH - 1))));
     const int n = col / 16, cc = col % 16;
     const int qq = q_start + (wave * PF_NG + n) * QG + cc / G;
-    if (cc < QG * G && qq < qlen)
-      *reinterpret_cast<bf16x8_t*>(out + (long)(qbeg + qq) * out_stride +
-                                   (long)(kvh * G + cc % G) * HD + 8 * j) = v;
+    if (cc < QG * G && qq < qlen) {
+      const long row = qbeg + qq, col = (long)(kvh * G + cc % G) * HD + 8 * j;
+      bf16x8_t ov = v;
+      if (gt.ptr) {
+        const bf16x8_t gv = load_frag16B(gt.ptr + row * gt.stride + col);
+#pragma unroll
+        for (int t = 0; t < 8; ++t)
+          ov[t] = (short)f2bf(bf2f((uint16_t)v[t]) / (1.f + __expf(-bf2f((uint16_t)gv[t]))));
+      }
+      *reinterpret_cast<bf16x8_t*>(out + row * out_stride + col) = ov;
+    }
   }
 }
 
@@ -1319,7 +1373,8 @@ int paged_prefill(const void* q, long q_stride, const void* k_cache, const void*
                   const int* context_lens, const int* tiles, int num_tiles, void* out,
                   long out_stride, int Hq, int Hkv, int D, int block_size, float scale,
                   int causal, int q_per_tile, const int* rope_pos, const float* rope_cs,
-                  hipStream_t stream) {
+                  const void* gate, long gate_stride, int split_p, hipStream_t stream) {
+  const GateIn gt{(const bf16_t*)gate, gate_stride};
   if ((rope_pos == nullptr) != (rope_cs == nullptr)) return -4;
   if (num_tiles <= 0) return 0;
   if ((D != 128 && D != 64) || block_size != BS) return -1;
@@ -1327,35 +1382,129 @@ int paged_prefill(const void* q, long q_stride, const void* k_cache, const void*
   const int per_wave = (D == 128 ? pf_groups<128>() : pf_groups<64>()) * (16 / (Hq / Hkv));
   const int pw = q_per_tile / per_wave;
   if (q_per_tile % per_wave != 0 || (pw != 4 && pw != 8) || (pw == 8 && D != 128)) return -3;
-#define LMX_PRE(HDV, NSTV, PWV)                                                               \
+#define LMX_PRE(HDV, NSTV, PWV, SPL)                                                          \
   {                                                                                           \
     constexpr int smem = NSTV * 4 * BS * HDV * 2;                                             \
     static bool attr = false;                                                                 \
     if (smem > 65536 && !attr) {                                                              \
-      (void)hipFuncSetAttribute((const void*)paged_prefill_kernel<HDV, NSTV, PWV>,            \
+      (void)hipFuncSetAttribute((const void*)paged_prefill_kernel<HDV, NSTV, PWV, SPL>,       \
                                 hipFuncAttributeMaxDynamicSharedMemorySize, smem);            \
       attr = true;                                                                            \
     }                                                                                         \
-    paged_prefill_kernel<HDV, NSTV, PWV><<<dim3(num_tiles, Hkv), dim3(64 * PWV), smem,        \
-                                           stream>>>(                                         \
+    paged_prefill_kernel<HDV, NSTV, PWV, SPL><<<dim3(num_tiles, Hkv), dim3(64 * PWV), smem,   \
+                                                stream>>>(                                         \
         (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,           \
         block_tables, bt_stride, cu_q, context_lens, tiles, (bf16_t*)out, out_stride, Hq, Hkv, \
-        scale, causal, g_prefill_rescale_thr, g_prefill_xcd, rope_pos, rope_cs);              \
+        scale, causal, g_prefill_rescale_thr, g_prefill_xcd, rope_pos, rope_cs, gt);              \
   }
   // 2 slots by default: 3 measured equal at D = 64 and 1.55x slower at D = 128
   // with 4-wave workgroups (96 KB of LDS leaves one workgroup per CU) --
   // tools/prefill_attn_probe.py; the 8-wave form is one workgroup per CU anyway
   const int nst = g_prefill_stages ? g_prefill_stages : 2;
-  if (D == 128) {
+  if (split_p) {
+    if (pw != 4) return -5;
+    if (D == 128) LMX_PRE(128, 2, 4, true) else LMX_PRE(64, 2, 4, true)
+  } else if (D == 128) {
     if (pw == 8) {
-      if (nst == 3) LMX_PRE(128, 3, 8) else LMX_PRE(128, 2, 8)
+      if (nst == 3) LMX_PRE(128, 3, 8, false) else LMX_PRE(128, 2, 8, false)
     } else {
-      if (nst == 3) LMX_PRE(128, 3, 4) else LMX_PRE(128, 2, 4)
+      if (nst == 3) LMX_PRE(128, 3, 4, false) else LMX_PRE(128, 2, 4, false)
     }
   } else {
-    if (nst == 3) LMX_PRE(64, 3, 4) else LMX_PRE(64, 2, 4)
+    if (nst == 3) LMX_PRE(64, 3, 4, false) else LMX_PRE(64, 2, 4, false)
   }
 #undef LMX_PRE
+  return (int)hipGetLastError();
+}
+
+// ------------------------------------------------------ any head geometry ----
+// Paged causal attention for what K3 / K4 do not cover: fp32 caches, head
+// sizes above 128, more than 16 query heads per kv head.  One wave per (row,
+// query head), all arithmetic fp32; a lane scores one key of a 64-key block
+// (q from LDS), then owns every 64th output channel of the weighted sum.
+// grid (rows, ceil(Hq / 4)), block 256 = 4 heads.  D <= 512, a multiple of 64.
+template <typename T, int ND>
+__global__ void __launch_bounds__(256) attention_any_kernel(
+    const T* __restrict__ q, long q_stride, const T* __restrict__ kc, const T* __restrict__ vc,
+    const int* __restrict__ bt, int bt_stride, const int* __restrict__ cu_q, int S,
+    const int* __restrict__ positions, T* __restrict__ out, long out_stride,
+    const T* __restrict__ gate, long gate_stride, int Hq, int Hkv, float scale) {
+  constexpr int D = ND * 64;
+  __shared__ float sq[4][D];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int row = blockIdx.x, h = blockIdx.y * 4 + wave;
+  const bool on = h < Hq;
+  if (on)
+    for (int d = lane; d < D; d += 64) sq[wave][d] = ld1(q + row * q_stride + (long)h * D + d);
+  __syncthreads();
+  if (!on) return;
+  int lo = 0, hi = S - 1;                     // the sequence of this row
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (cu_q[mid] <= row) lo = mid; else hi = mid - 1;
+  }
+  const int* tab = bt + (long)lo * bt_stride;
+  const int n = positions[row] + 1;
+  const long kvh = h / (Hq / Hkv);
+  float m = -INFINITY, l = 0.f, acc[ND];
+#pragma unroll
+  for (int i = 0; i < ND; ++i) acc[i] = 0.f;
+  for (int k0 = 0; k0 < n; k0 += 64) {
+    const int key = k0 + lane;
+    float s = -INFINITY;
+    if (key < n) {
+      const T* kp = kc + (((long)tab[key / BS] * Hkv + kvh) * BS + key % BS) * D;
+      float t = 0.f;
+      for (int d = 0; d < D; d += 8) {
+        float x[8];
+        ldv<8>(x, kp + d);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) t += x[e] * sq[wave][d + e];
+      }
+      s = t * scale;
+    }
+    const float mn = fmaxf(m, wave_max(s));
+    const float al = expf(m - mn), p = expf(s - mn);   // exp(-inf) = 0
+    l = l * al + wave_sum(p);
+    m = mn;
+#pragma unroll
+    for (int i = 0; i < ND; ++i) acc[i] *= al;
+    const int cnt = min(64, n - k0);
+    for (int j = 0; j < cnt; ++j) {
+      const float pj = __shfl(p, j, 64);
+      const int kj = k0 + j, off = kj % BS;
+      const T* vp = vc + ((long)tab[kj / BS] * Hkv + kvh) * BS * D;
+#pragma unroll
+      for (int i = 0; i < ND; ++i) acc[i] += pj * ld1(vp + vq_off(i * 64 + lane, off, D));
+    }
+  }
+  const float inv = 1.f / l;
+#pragma unroll
+  for (int i = 0; i < ND; ++i) {
+    const long col = (long)h * D + i * 64 + lane;
+    float o = acc[i] * inv;
+    if (gate) o *= sigmoid_t<T>(ld1(gate + row * gate_stride + col));
+    st1(out + row * out_stride + col, o);
+  }
+}
+
+int attention_any(const void* q, long q_stride, const void* kc, const void* vc, const int* bt,
+                  int bt_stride, const int* cu_q, int S, const int* positions, int rows, void* out,
+                  long out_stride, const void* gate, long gate_stride, int Hq, int Hkv, int D,
+                  int block_size, float scale, int is_bf16, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (block_size != BS || S < 1 || Hq % Hkv != 0) return -1;
+  const dim3 grid(rows, (Hq + 3) / 4);
+#define LMX_ANY(T, ND)                                                                           \
+  attention_any_kernel<T, ND><<<grid, dim3(256), 0, stream>>>(                                   \
+      (const T*)q, q_stride, (const T*)kc, (const T*)vc, bt, bt_stride, cu_q, S, positions,      \
+      (T*)out, out_stride, (const T*)gate, gate_stride, Hq, Hkv, scale)
+#define LMX_ANY_D(T)                                                                             \
+  if (D == 64) LMX_ANY(T, 1); else if (D == 128) LMX_ANY(T, 2); else if (D == 256) LMX_ANY(T, 4); \
+  else if (D == 512) LMX_ANY(T, 8); else return -2;
+  if (is_bf16) { LMX_ANY_D(bf16_t) } else { LMX_ANY_D(float) }
+#undef LMX_ANY_D
+#undef LMX_ANY
   return (int)hipGetLastError();
 }
 

@@ -28,15 +28,31 @@ void set_prefill_xcd(int);
 int paged_decode(const void*, long, const void*, const void*, const int*, int, const int*,
                  const int*, void*,
                  long, float*, float*, int, int, int, int, int, float, int, int, const int*,
-                 const float*, const int*, hipStream_t);
+                 const float*, const int*, const void*, long, int, hipStream_t);
 int paged_prefill(const void*, long, const void*, const void*, const int*, int, const int*,
                   const int*, const int*, int, void*, long, int, int, int, int, float, int, int,
-                  const int*, const float*, hipStream_t);
+                  const int*, const float*, const void*, long, int, hipStream_t);
+int attention_any(const void*, long, const void*, const void*, const int*, int, const int*, int,
+                  const int*, int, void*, long, const void*, long, int, int, int, int, float, int,
+                  hipStream_t);
+int sandwich_norm(void*, float*, const void*, long, int, long, const int*, const void*,
+                  const float*, const float*, const long*, int, int, float, int, hipStream_t);
+int gated_norm(void*, long, const void*, long, const void*, long, const float*, int, int, int, int,
+               float, int, hipStream_t);
+int short_conv(const void*, long, const float*, const float*, void*, const int*, int, int,
+               const int*, const int*, const int*, int, int, void*, long, int, int, hipStream_t);
+int conv_qkv_cache(const void*, long, const float*, const float*, void*, const int*, int, int, const int*,
+                   const int*, const int*, int, void*, long, void*, void*, const int*, const int*,
+                   int, int, int, int, int, float, float, float, int, hipStream_t);
+int linear_scan(const void*, long, const void*, long, const void*, long, const void*, long,
+                const float*, const float*, const float*, const float*, const float*, void*, long,
+                float*, const int*, const int*, const int*, int, int, int, int, int, int, int, int,
+                const int*, int, const int*, int, float*, float*, hipStream_t);
 int sample(const void*, int, long, int, int, const float*, const int*, const float*,
            const uint64_t*, const int*, int*, float*, int, hipStream_t);
-int glu(void*, const void*, long, int, int, int, hipStream_t);
-int apply_penalties(void*, long, int, int, const int*, const int*, const float*, const int*, int,
-                    int, hipStream_t);
+int glu(void*, const void*, long, int, int, int, int, hipStream_t);
+int apply_penalties(void*, int, long, int, int, const int*, const int*, const float*, const int*,
+                    int, int, hipStream_t);
 int race_sample_phase(int, int, int, const void*, int, long, int, int, int, int, const float*,
                       const int*, const float*, const uint64_t*, const int*, const float*, int,
                       float*, float*, int*, float*, hipStream_t);
@@ -126,11 +142,12 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                            uptr ctx, uptr order, uptr out, long out_stride, uptr part_o,
                            uptr part_ml, int B, int Hq, int Hkv, int D, int BS, float scale,
                            int part_tokens, int max_parts, uptr positions, uptr cos_sin,
-                           uptr slots, uptr stream) {
+                           uptr slots, uptr gate, long gate_stride, int split_p, uptr stream) {
     check(lmx::paged_decode(P<void>(q), q_stride, P<void>(kc), P<void>(vc), P<int>(bt), bt_stride,
                             P<int>(ctx), P<int>(order), P<void>(out), out_stride, P<float>(part_o),
                             P<float>(part_ml), B, Hq, Hkv, D, BS, scale, part_tokens, max_parts,
-                            P<int>(positions), P<float>(cos_sin), P<int>(slots), S(stream)),
+                            P<int>(positions), P<float>(cos_sin), P<int>(slots), P<void>(gate),
+                            gate_stride, split_p, S(stream)),
           "paged_decode");
   });
   m.def("set_slab_norm_threads", [](int t) { lmx::set_slab_norm_threads(t); },
@@ -146,13 +163,77 @@ PYBIND11_MODULE(_lmx_kernels, m) {
   m.def("paged_prefill", [](uptr q, long q_stride, uptr kc, uptr vc, uptr bt, int bt_stride,
                             uptr cu_q, uptr ctx, uptr tiles, int num_tiles, uptr out,
                             long out_stride, int Hq, int Hkv, int D, int BS, float scale,
-                            int causal, int q_per_tile, uptr rope_pos, uptr rope_cs,
-                            uptr stream) {
+                            int causal, int q_per_tile, uptr rope_pos, uptr rope_cs, uptr gate,
+                            long gate_stride, int split_p, uptr stream) {
     check(lmx::paged_prefill(P<void>(q), q_stride, P<void>(kc), P<void>(vc), P<int>(bt),
                              bt_stride, P<int>(cu_q), P<int>(ctx), P<int>(tiles), num_tiles,
                              P<void>(out), out_stride, Hq, Hkv, D, BS, scale, causal, q_per_tile,
-                             P<int>(rope_pos), P<float>(rope_cs), S(stream)),
+                             P<int>(rope_pos), P<float>(rope_cs), P<void>(gate), gate_stride,
+                             split_p, S(stream)),
           "paged_prefill");
+  });
+  m.def("attention_any", [](uptr q, long q_stride, uptr kc, uptr vc, uptr bt, int bt_stride,
+                            uptr cu_q, int nseq, uptr positions, int rows, uptr out,
+                            long out_stride, uptr gate, long gate_stride, int Hq, int Hkv, int D,
+                            int BS, float scale, int is_bf16, uptr stream) {
+    check(lmx::attention_any(P<void>(q), q_stride, P<void>(kc), P<void>(vc), P<int>(bt), bt_stride,
+                             P<int>(cu_q), nseq, P<int>(positions), rows, P<void>(out), out_stride,
+                             P<void>(gate), gate_stride, Hq, Hkv, D, BS, scale, is_bf16, S(stream)),
+          "attention_any");
+  });
+  // ---- sandwich / gated norms (norm.hip) ----
+  m.def("sandwich_norm", [](uptr out, uptr residual, uptr y, long y_ld, int slabs,
+                            long slab_stride, uptr ids, uptr table, uptr w_post, uptr w_pre,
+                            uptr rows_idx, int rows, int cols, float eps, int is_bf16,
+                            uptr stream) {
+    check(lmx::sandwich_norm(P<void>(out), P<float>(residual), P<void>(y), y_ld, slabs,
+                             slab_stride, P<int>(ids), P<void>(table), P<float>(w_post),
+                             P<float>(w_pre), P<long>(rows_idx), rows, cols, eps, is_bf16,
+                             S(stream)),
+          "sandwich_norm");
+  });
+  m.def("gated_norm", [](uptr out, long out_ld, uptr x, long x_ld, uptr g, long g_ld, uptr w,
+                         int rows, int cols, int groups, int gate_first, float eps, int is_bf16,
+                         uptr stream) {
+    check(lmx::gated_norm(P<void>(out), out_ld, P<void>(x), x_ld, P<void>(g), g_ld, P<float>(w),
+                          rows, cols, groups, gate_first, eps, is_bf16, S(stream)),
+          "gated_norm");
+  });
+  // ---- K16 short causal convolution (conv.hip) ----
+  m.def("short_conv", [](uptr u, long u_ld, uptr w, uptr bias, uptr state, uptr tiles, int ntiles,
+                         int tile, uptr cu_q, uptr ctx, uptr slots, int C, int taps, uptr out,
+                         long out_ld, int act, int is_bf16, uptr stream) {
+    check(lmx::short_conv(P<void>(u), u_ld, P<float>(w), P<float>(bias), P<void>(state),
+                          P<int>(tiles), ntiles, tile, P<int>(cu_q), P<int>(ctx), P<int>(slots), C,
+                          taps, P<void>(out), out_ld, act, is_bf16, S(stream)),
+          "short_conv");
+  });
+  m.def("conv_qkv_cache", [](uptr u, long u_ld, uptr w, uptr in_bias, uptr state, uptr tiles,
+                             int ntiles, int tile, uptr cu_q, uptr ctx, uptr state_slots, int taps, uptr q,
+                             long q_ld, uptr kc, uptr vc, uptr positions, uptr slots, int Hq,
+                             int Hkv, int D, int dk, int BS, float eps, float coef, float every,
+                             int is_bf16, uptr stream) {
+    check(lmx::conv_qkv_cache(P<void>(u), u_ld, P<float>(w), P<float>(in_bias), P<void>(state),
+                              P<int>(tiles), ntiles, tile, P<int>(cu_q), P<int>(ctx), P<int>(state_slots), taps,
+                              P<void>(q), q_ld, P<void>(kc), P<void>(vc), P<int>(positions),
+                              P<int>(slots), Hq, Hkv, D, dk, BS, eps, coef, every, is_bf16,
+                              S(stream)),
+          "conv_qkv_cache");
+  });
+  // ---- K15 linear-attention / state-space scan (linscan.hip) ----
+  m.def("linear_scan", [](uptr q, long q_ld, uptr k, long k_ld, uptr v, long v_ld, uptr dt,
+                          long dt_ld, uptr dt_bias, uptr neg_a, uptr decay, uptr log_decay,
+                          uptr skip, uptr out, long out_ld, uptr state, uptr cu_q, uptr ctx,
+                          uptr slots, int H, int N, int Pd, int hpg, int act, int is_bf16, int seq0,
+                          int nseq, uptr segs, int nseg, uptr first, int one_pass, uptr ws,
+                          uptr ws_log, uptr stream) {
+    check(lmx::linear_scan(P<void>(q), q_ld, P<void>(k), k_ld, P<void>(v), v_ld, P<void>(dt),
+                           dt_ld, P<float>(dt_bias), P<float>(neg_a), P<float>(decay),
+                           P<float>(log_decay), P<float>(skip), P<void>(out), out_ld,
+                           P<float>(state), P<int>(cu_q), P<int>(ctx), P<int>(slots), H, N, Pd, hpg,
+                           act, is_bf16, seq0, nseq, P<int>(segs), nseg, P<int>(first), one_pass,
+                           P<float>(ws), P<float>(ws_log), S(stream)),
+          "linear_scan");
   });
   m.def("sample", [](uptr logits, int is_bf16, long stride, int B, int V, uptr temp, uptr topk,
                      uptr topp, uptr seeds, uptr offsets, uptr out_tok, uptr out_lp,
@@ -162,8 +243,9 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                       P<float>(out_lp), max_rounds, S(stream)),
           "sample");
   });
-  m.def("glu", [](uptr out, uptr x, long rows, int I, int act, int block, uptr stream) {
-    check(lmx::glu(P<void>(out), P<void>(x), rows, I, act, block, S(stream)), "glu");
+  m.def("glu", [](uptr out, uptr x, long rows, int I, int act, int block, int is_bf16,
+                  uptr stream) {
+    check(lmx::glu(P<void>(out), P<void>(x), rows, I, act, block, is_bf16, S(stream)), "glu");
   });
   m.def("ids_from_prev", [](uptr ids, uptr src, uptr prev, int n, uptr stream) {
     check(lmx::ids_from_prev(P<int>(ids), P<int>(src), P<int>(prev), n, S(stream)),
@@ -293,9 +375,9 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                          two_shot, blocks, spin_max, S(stream)),
           "allreduce");
   });
-  m.def("apply_penalties", [](uptr logits, long ld, int B, int V, uptr win, uptr ngen, uptr pen,
+  m.def("apply_penalties", [](uptr logits, int is_bf16, long ld, int B, int V, uptr win, uptr ngen, uptr pen,
                               uptr on, int W, int v0, uptr stream) {
-    check(lmx::apply_penalties(P<void>(logits), ld, B, V, P<const int>(win), P<const int>(ngen),
+    check(lmx::apply_penalties(P<void>(logits), is_bf16, ld, B, V, P<const int>(win), P<const int>(ngen),
                                P<const float>(pen), P<const int>(on), W, v0, S(stream)),
           "apply_penalties");
   });

@@ -108,6 +108,61 @@ __device__ __forceinline__ bf16x8_t load_frag_2x8B(const bf16_t* p0, const bf16_
   return r;
 }
 
+// Element access of kernels that run on bf16 or fp32 rows (arithmetic fp32).
+__device__ __forceinline__ float ld1(const bf16_t* p) { return bf2f(*p); }
+__device__ __forceinline__ float ld1(const float* p) { return *p; }
+__device__ __forceinline__ void st1(bf16_t* p, float v) { *p = f2bf(v); }
+__device__ __forceinline__ void st1(float* p, float v) { *p = v; }
+
+// V = 8 (16-B aligned rows) or 1 consecutive elements
+template <int V>
+__device__ __forceinline__ void ldv(float (&f)[V], const bf16_t* p) {
+  if constexpr (V == 8) {
+    const u16x8 x = *reinterpret_cast<const u16x8*>(p);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) f[j] = bf2f(x.v[j]);
+  } else {
+    f[0] = bf2f(*p);
+  }
+}
+template <int V>
+__device__ __forceinline__ void ldv(float (&f)[V], const float* p) {
+  if constexpr (V == 8) {
+    const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+    f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+  } else {
+    f[0] = *p;
+  }
+}
+template <int V>
+__device__ __forceinline__ void stv(bf16_t* p, const float (&f)[V]) {
+  if constexpr (V == 8) {
+    u16x8 x;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x.v[j] = f2bf(f[j]);
+    *reinterpret_cast<u16x8*>(p) = x;
+  } else {
+    *p = f2bf(f[0]);
+  }
+}
+template <int V>
+__device__ __forceinline__ void stv(float* p, const float (&f)[V]) {
+  if constexpr (V == 8) {
+    *reinterpret_cast<float4*>(p) = make_float4(f[0], f[1], f[2], f[3]);
+    *reinterpret_cast<float4*>(p + 4) = make_float4(f[4], f[5], f[6], f[7]);
+  } else {
+    *p = f[0];
+  }
+}
+
+// exp-based activations: fp32 rows use the accurate exponential, bf16 rows the
+// hardware one (its error is far below a bf16 rounding)
+template <typename T> __device__ __forceinline__ float sigmoid_t(float x) {
+  if constexpr (sizeof(T) == 4) return 1.f / (1.f + expf(-x));
+  else return 1.f / (1.f + __expf(-x));
+}
+
 // XCD-aware bijective remap of a linear workgroup id (cdna guide §5, T1):
 // consecutive logical tiles land on the same XCD so neighbouring tiles share L2.
 __device__ __forceinline__ int xcd_remap(int orig, int nwg) {

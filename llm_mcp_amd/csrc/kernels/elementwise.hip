@@ -25,39 +25,41 @@ __device__ __forceinline__ float gelu_tanh(float x) {
 // ``block`` > 0: the gate|up columns are interleaved per block (the layout of
 // the fused-SwiGLU decode GEMM weights, dgemm.hip): gate channel i sits at
 // column (i / block) * 2 * block + i % block and its up partner block later.
-template <int ACT>
-__global__ void __launch_bounds__(256) glu_kernel(bf16_t* __restrict__ out,
-                                                  const bf16_t* __restrict__ x, int I,
-                                                  int block) {
+// ACT: 0 SiLU, 1 tanh-GELU, 2 ReLU.
+template <typename T, int ACT>
+__global__ void __launch_bounds__(256) glu_kernel(T* __restrict__ out, const T* __restrict__ x,
+                                                  int I, int block) {
   const int c = blockIdx.y * 256 + threadIdx.x;
   if (c >= I / 8) return;
   const long r = blockIdx.x;
-  const bf16_t* xr = x + r * (2L * I);
+  const T* xr = x + r * (2L * I);
   const int gi = c * 8;
   const int go = block > 0 ? (gi / block) * 2 * block + gi % block : gi;
   const int uo = block > 0 ? go + block : I + gi;
-  const u16x8 g = *reinterpret_cast<const u16x8*>(xr + go);
-  const u16x8 u = *reinterpret_cast<const u16x8*>(xr + uo);
-  u16x8 o;
+  float g[8], u[8];
+  ldv<8>(g, xr + go);
+  ldv<8>(u, xr + uo);
 #pragma unroll
-  for (int j = 0; j < 8; ++j) {
-    const float gv = bf2f(g.v[j]);
-    const float a = ACT == 0 ? silu(gv) : gelu_tanh(gv);
-    o.v[j] = f2bf(a * bf2f(u.v[j]));
-  }
-  *reinterpret_cast<u16x8*>(out + r * I + c * 8) = o;
+  for (int j = 0; j < 8; ++j)
+    u[j] *= ACT == 0 ? g[j] * sigmoid_t<T>(g[j]) : ACT == 1 ? gelu_tanh(g[j]) : fmaxf(g[j], 0.f);
+  stv<8>(out + r * I + c * 8, u);
 }
 
-int glu(void* out, const void* x, long rows, int I, int act, int block, hipStream_t stream) {
+int glu(void* out, const void* x, long rows, int I, int act, int block, int is_bf16,
+        hipStream_t stream) {
   if (rows <= 0) return 0;
-  if (I % 8 != 0 || rows > 0x7fffffffL || block < 0 || block % 8 != 0 ||
+  if (I % 8 != 0 || rows > 0x7fffffffL || block < 0 || block % 8 != 0 || act < 0 || act > 2 ||
       (block > 0 && I % block != 0))
     return -1;
   const dim3 grid((unsigned)rows, (unsigned)((I / 8 + 255) / 256));
-  if (act == 0)
-    glu_kernel<0><<<grid, dim3(256), 0, stream>>>((bf16_t*)out, (const bf16_t*)x, I, block);
-  else
-    glu_kernel<1><<<grid, dim3(256), 0, stream>>>((bf16_t*)out, (const bf16_t*)x, I, block);
+#define LMX_GLU(T, A) \
+  glu_kernel<T, A><<<grid, dim3(256), 0, stream>>>((T*)out, (const T*)x, I, block)
+  if (is_bf16) {
+    if (act == 0) LMX_GLU(bf16_t, 0); else if (act == 1) LMX_GLU(bf16_t, 1); else LMX_GLU(bf16_t, 2);
+  } else {
+    if (act == 0) LMX_GLU(float, 0); else if (act == 1) LMX_GLU(float, 1); else LMX_GLU(float, 2);
+  }
+#undef LMX_GLU
   return (int)hipGetLastError();
 }
 

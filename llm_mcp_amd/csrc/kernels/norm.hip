@@ -345,4 +345,203 @@ int layernorm(void* out, const void* x, const void* residual, const void* w, con
   return (int)hipGetLastError();
 }
 
+// Sandwich norm: the norm after a sublayer, the residual add and the norm
+// before the next sublayer in one pass, over an fp32 residual stream.
+//
+//   r   = ids ? table[ids[row]] : residual[row]
+//   r  += norm(y[row]) * w_post              (y: the sublayer's output; optional)
+//   out = norm(r) * w_pre                    (optional)
+//
+// norm(x) = x / sqrt(mean(x^2) + eps); the gains are fp32 (a weight stored
+// around zero arrives as 1 + w).  y is T rows, or S fp32 split-K slabs
+// [S][rows][cols] summed here.  rows_idx (optional): out row i is source row
+// rows_idx[i] and the residual is left as it is (the final norm of the sampled
+// rows); otherwise the residual row is written when it changed.
+struct SandwichArgs {
+  void* out;
+  float* residual;
+  const void* y;
+  long y_ld, slab_stride;
+  int slabs;                  // 0: y is T rows
+  const int* ids;
+  const void* table;
+  const float *w_post, *w_pre;
+  const long* rows_idx;
+  int cols;
+  float eps;
+};
+
+template <typename T, int V, int VPT>
+__global__ void __launch_bounds__(256) sandwich_norm_kernel(SandwichArgs a) {
+  __shared__ float scratch[16];
+  const long src = a.rows_idx ? a.rows_idx[blockIdx.x] : blockIdx.x;
+  const int cols = a.cols, nchunk = cols / V;
+  float* rr = a.residual + src * cols;
+  float r[VPT][V], y[VPT][V];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c >= nchunk) continue;
+    if (a.ids) ldv<V>(r[i], (const T*)a.table + (long)a.ids[src] * cols + c * V);
+    else ldv<V>(r[i], rr + c * V);
+    if (a.y) {
+      if (a.slabs) {
+        const float* p = (const float*)a.y + src * cols + c * V;
+        ldv<V>(y[i], p);
+        for (int s = 1; s < a.slabs; ++s) {
+          float t[V];
+          ldv<V>(t, p + s * a.slab_stride);
+#pragma unroll
+          for (int e = 0; e < V; ++e) y[i][e] += t[e];
+        }
+      } else {
+        ldv<V>(y[i], (const T*)a.y + src * a.y_ld + c * V);
+      }
+#pragma unroll
+      for (int e = 0; e < V; ++e) ss += y[i][e] * y[i][e];
+    }
+  }
+  if (a.y) {
+    ss = block_sum(ss, scratch);
+    const float inv = rsqrtf(ss / (float)cols + a.eps);
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c >= nchunk) continue;
+      float w[V];
+      ldv<V>(w, a.w_post + c * V);
+#pragma unroll
+      for (int e = 0; e < V; ++e) r[i][e] += y[i][e] * inv * w[e];
+    }
+  }
+  if (!a.rows_idx && (a.y || a.ids)) {
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c < nchunk) stv<V>(rr + c * V, r[i]);
+    }
+  }
+  if (!a.w_pre) return;
+  ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c < nchunk)
+#pragma unroll
+      for (int e = 0; e < V; ++e) ss += r[i][e] * r[i][e];
+  }
+  ss = block_sum(ss, scratch);
+  const float inv = rsqrtf(ss / (float)cols + a.eps);
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c >= nchunk) continue;
+    float w[V];
+    ldv<V>(w, a.w_pre + c * V);
+#pragma unroll
+    for (int e = 0; e < V; ++e) w[e] *= r[i][e] * inv;
+    stv<V>((T*)a.out + (long)blockIdx.x * cols + c * V, w);
+  }
+}
+
+int sandwich_norm(void* out, float* residual, const void* y, long y_ld, int slabs, long slab_stride,
+                  const int* ids, const void* table, const float* w_post, const float* w_pre,
+                  const long* rows_idx, int rows, int cols, float eps, int is_bf16,
+                  hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (cols <= 0 || !residual || (y && !w_post) || (w_pre && !out)) return -1;
+  const SandwichArgs a{out, residual, y, y_ld, slab_stride, slabs, ids, table,
+                       w_post, w_pre, rows_idx, cols, eps};
+  const bool vec = cols % 8 == 0 && y_ld % 8 == 0;
+  const int nchunk = vec ? cols / 8 : cols;
+  const int vpt = (nchunk + 255) / 256;
+  if (vpt > 8) return -2;
+  const int threads = nchunk >= 256 ? 256 : (nchunk + 63) / 64 * 64;
+#define LMX_SW(T, V, P) sandwich_norm_kernel<T, V, P><<<dim3(rows), dim3(threads), 0, stream>>>(a)
+#define LMX_SWT(T)                                                            \
+  if (vec) {                                                                  \
+    if (vpt == 1) LMX_SW(T, 8, 1); else if (vpt == 2) LMX_SW(T, 8, 2);        \
+    else if (vpt <= 4) LMX_SW(T, 8, 4); else LMX_SW(T, 8, 8);                 \
+  } else {                                                                    \
+    if (vpt == 1) LMX_SW(T, 1, 1); else LMX_SW(T, 1, 8);                      \
+  }
+  if (is_bf16) { LMX_SWT(bf16_t) } else { LMX_SWT(float) }
+#undef LMX_SWT
+#undef LMX_SW
+  return (int)hipGetLastError();
+}
+
+// Gated RMS norm of a mixer's output, in `groups` equal parts of a row, each
+// divided by its own root mean square:
+//   gate_first 0: out = norm(x) * w * sigmoid(g)      (linear attention)
+//   gate_first 1: out = norm(x * silu(g)) * w         (state-space mixer)
+// grid (rows, groups), one workgroup per part.
+template <typename T, int V, int VPT>
+__global__ void __launch_bounds__(256) gated_norm_kernel(T* out, long out_ld, const T* x, long x_ld,
+                                                         const T* g, long g_ld,
+                                                         const float* __restrict__ w, int part,
+                                                         int gate_first, float eps) {
+  __shared__ float scratch[16];
+  const long row = blockIdx.x, off = (long)blockIdx.y * part;
+  const T* xr = x + row * x_ld + off;
+  const T* gr = g + row * g_ld + off;
+  const int nchunk = part / V;
+  float v[VPT][V], gt[VPT][V];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c >= nchunk) continue;
+    ldv<V>(v[i], xr + c * V);
+    ldv<V>(gt[i], gr + c * V);
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      const float s = sigmoid_t<T>(gt[i][e]);
+      if (gate_first) v[i][e] *= gt[i][e] * s;
+      gt[i][e] = gate_first ? 1.f : s;
+      ss += v[i][e] * v[i][e];
+    }
+  }
+  ss = block_sum(ss, scratch);
+  const float inv = rsqrtf(ss / (float)part + eps);
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c >= nchunk) continue;
+    float wv[V];
+    ldv<V>(wv, w + off + c * V);
+#pragma unroll
+    for (int e = 0; e < V; ++e) wv[e] *= v[i][e] * inv * gt[i][e];
+    stv<V>(out + row * out_ld + off + c * V, wv);
+  }
+}
+
+int gated_norm(void* out, long out_ld, const void* x, long x_ld, const void* g, long g_ld,
+               const float* w, int rows, int cols, int groups, int gate_first, float eps,
+               int is_bf16, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (groups < 1 || cols % groups != 0) return -1;
+  const int part = cols / groups;
+  const bool vec = part % 8 == 0 && out_ld % 8 == 0 && x_ld % 8 == 0 && g_ld % 8 == 0 &&
+                   (((uintptr_t)x | (uintptr_t)g | (uintptr_t)out) & 15) == 0;
+  const int nchunk = vec ? part / 8 : part, vpt = (nchunk + 255) / 256;
+  if (vpt > (vec ? 8 : 16)) return -2;
+  const int threads = nchunk >= 256 ? 256 : (nchunk + 63) / 64 * 64;
+  const dim3 grid(rows, groups);
+#define LMX_GN(T, V, P)                                                                         \
+  gated_norm_kernel<T, V, P><<<grid, dim3(threads), 0, stream>>>(                               \
+      (T*)out, out_ld, (const T*)x, x_ld, (const T*)g, g_ld, w, part, gate_first, eps)
+#define LMX_GNT(T)                                                                              \
+  if (vec) {                                                                                    \
+    if (vpt == 1) LMX_GN(T, 8, 1); else if (vpt == 2) LMX_GN(T, 8, 2); else LMX_GN(T, 8, 8);    \
+  } else {                                                                                      \
+    if (vpt == 1) LMX_GN(T, 1, 1); else LMX_GN(T, 1, 16);                                       \
+  }
+  if (is_bf16) { LMX_GNT(bf16_t) } else { LMX_GNT(float) }
+#undef LMX_GNT
+#undef LMX_GN
+  return (int)hipGetLastError();
+}
+
 }  // namespace lmx

@@ -527,7 +527,8 @@ int race_sample_phase(int phase, int round, int max_rounds, const void* logits, 
 //       l -= frequency * count + presence * (count > 0)
 // `on` (device flag, may be null) lets a captured graph skip the kernel for
 // steps without penalised rows.
-__global__ void __launch_bounds__(64) penalty_kernel(bf16_t* __restrict__ logits, long ld, int V,
+template <typename T>
+__global__ void __launch_bounds__(64) penalty_kernel(T* __restrict__ logits, long ld, int V,
                                                      const int* __restrict__ win,
                                                      const int* __restrict__ ngen,
                                                      const float* __restrict__ pen,
@@ -545,19 +546,24 @@ __global__ void __launch_bounds__(64) penalty_kernel(bf16_t* __restrict__ logits
   int cnt = 0;
   for (int j = lane > g0 ? lane : g0; j < W; ++j) cnt += ids[j] == t;
   const float rep = pen[3 * row], pres = pen[3 * row + 1], freq = pen[3 * row + 2];
-  bf16_t* p = logits + (long)row * ld + (t - v0);
-  float l = bf2f(*p);
+  T* p = logits + (long)row * ld + (t - v0);
+  float l = ld1(p);
   if (rep != 1.f) l = l > 0.f ? l / rep : l * rep;
   l -= freq * (float)cnt + (cnt > 0 ? pres : 0.f);
-  *p = f2bf(l);
+  st1(p, l);
 }
 
-int apply_penalties(void* logits, long ld, int B, int V, const int* win, const int* ngen,
-                    const float* pen, const int* on, int W, int v0, hipStream_t stream) {
+int apply_penalties(void* logits, int is_bf16, long ld, int B, int V, const int* win,
+                    const int* ngen, const float* pen, const int* on, int W, int v0,
+                    hipStream_t stream) {
   if (B <= 0) return 0;
   if (W <= 0 || W > 64) return -1;
-  penalty_kernel<<<dim3(B), dim3(64), 0, stream>>>((bf16_t*)logits, ld, V, win, ngen, pen, on, W,
-                                                    v0);
+  if (is_bf16)
+    penalty_kernel<bf16_t><<<dim3(B), dim3(64), 0, stream>>>((bf16_t*)logits, ld, V, win, ngen, pen,
+                                                             on, W, v0);
+  else
+    penalty_kernel<float><<<dim3(B), dim3(64), 0, stream>>>((float*)logits, ld, V, win, ngen, pen,
+                                                            on, W, v0);
   return (int)hipGetLastError();
 }
 

@@ -98,6 +98,7 @@ PYBIND11_MODULE(_lmx_runtime, m) {
            py::arg("stop_ids"), py::arg("ignore_eos") = false, py::arg("priority") = 0,
            py::arg("temperature") = 1.f, py::arg("top_k") = 0, py::arg("top_p") = 1.f,
            py::arg("seed") = 0)
+      .def("feed", &Scheduler::feed, py::arg("id"), py::arg("tokens"))
       .def("abort", &Scheduler::abort)
       .def("set_mixed_prefill_cap", &Scheduler::set_mixed_prefill_cap, py::arg("tokens"),
            py::arg("min_decodes"), py::arg("later_steps") = 0)
@@ -115,6 +116,7 @@ PYBIND11_MODULE(_lmx_runtime, m) {
         d["seq_ids"] = to_np(p.seq_ids);
         d["qlens"] = to_np(p.qlens);
         d["context_lens"] = to_np(p.context_lens);
+        d["state_slots"] = to_np(p.state_slots);
         d["cu_q"] = to_np(p.cu_q);
         d["block_tables"] = to_np(p.block_tables);
         d["sample_rows"] = to_np(p.sample_rows);

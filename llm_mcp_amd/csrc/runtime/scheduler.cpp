@@ -3,6 +3,7 @@
 #include <climits>
 
 #include <algorithm>
+#include <functional>
 #include <stdexcept>
 
 namespace lmxrt {
@@ -16,6 +17,14 @@ Scheduler::Scheduler(int num_blocks, int block_size, int max_num_seqs, int max_b
   if (max_num_seqs <= 0 || max_batched_tokens <= 0 || max_model_len <= 0)
     throw std::invalid_argument("bad scheduler limits");
   max_blocks_ = (max_model_len + block_size - 1) / block_size;
+  for (int i = 0; i < max_num_seqs; ++i) free_slots_.push_back(i);  // ascending = a min-heap
+}
+
+void Scheduler::release_slot(Seq* s) {
+  if (s->slot < 0) return;
+  free_slots_.push_back(s->slot);
+  std::push_heap(free_slots_.begin(), free_slots_.end(), std::greater<int32_t>());
+  s->slot = -1;
 }
 
 void Scheduler::add(int64_t id, const std::vector<int32_t>& prompt, int max_new,
@@ -62,6 +71,29 @@ bool Scheduler::set_penalties(int64_t id, float repetition, float presence, floa
   return true;
 }
 
+void Scheduler::feed(int64_t id, const std::vector<int32_t>& tokens) {
+  if (tokens.empty()) throw std::invalid_argument("feed without tokens");
+  auto it = seqs_.find(id);
+  if (it != seqs_.end() && !it->second->fed)
+    throw std::invalid_argument("feed of a sequence that is sampled");
+  const size_t len = (it == seqs_.end() ? 0 : it->second->tokens.size()) + tokens.size();
+  if ((int)len > max_model_len_) throw std::invalid_argument("fed tokens exceed max_model_len");
+  if ((int)len > bm_.num_blocks() * bm_.block_size())
+    throw std::invalid_argument("fed tokens exceed the KV cache");
+  if (it == seqs_.end()) {
+    auto s = std::make_unique<Seq>();
+    s->id = id;
+    s->fed = true;
+    s->arrival = arrival_++;
+    s->arrival_step = steps_;
+    waiting_.push_back(s.get());
+    it = seqs_.emplace(id, std::move(s)).first;
+  }
+  Seq* s = it->second.get();
+  s->tokens.insert(s->tokens.end(), tokens.begin(), tokens.end());
+  s->prompt_len = (int)s->tokens.size();
+}
+
 const Seq* Scheduler::get(int64_t id) const {
   auto it = seqs_.find(id);
   return it == seqs_.end() ? nullptr : it->second.get();
@@ -77,6 +109,7 @@ bool Scheduler::abort(int64_t id) {
   auto r = std::find(running_.begin(), running_.end(), s);
   if (r != running_.end()) running_.erase(r);
   bm_.free_seq(id);
+  release_slot(s);
   // lookahead: a sample of it awaiting patch() is dropped; a row of it in the
   // plan in flight keeps the object alive until update_lookahead() consumes it
   for (Seq*& q : inflight_)
@@ -103,6 +136,7 @@ bool Scheduler::length_done(const Seq* s) const {
 
 void Scheduler::preempt(Seq* s) {
   bm_.free_seq(s->id);
+  release_slot(s);
   s->num_computed = 0;
   s->scheduled = 0;
   s->status = WAITING;
@@ -117,6 +151,7 @@ void Scheduler::finish(Seq* s, int reason) {
   s->status = FINISHED;
   s->finish = reason;
   bm_.free_seq(s->id);
+  release_slot(s);
   auto r = std::find(running_.begin(), running_.end(), s);
   if (r != running_.end()) running_.erase(r);
   // lookahead: a sequence preempted by the plan after the one that sampled
@@ -131,7 +166,7 @@ const StepPlan& Scheduler::schedule(int q_per_tile) {
   StepPlan& p = plan_;
   p.input_ids.clear(); p.positions.clear(); p.slots.clear(); p.input_src.clear();
   p.num_pending_inputs = 0;
-  p.seq_ids.clear(); p.qlens.clear(); p.context_lens.clear(); p.cu_q.clear();
+  p.seq_ids.clear(); p.qlens.clear(); p.state_slots.clear(); p.context_lens.clear(); p.cu_q.clear();
   p.block_tables.clear(); p.sample_rows.clear(); p.sample_seq.clear();
   p.sample_temp.clear(); p.sample_topp.clear(); p.sample_topk.clear(); p.sample_off.clear();
   p.sample_seed.clear();
@@ -188,7 +223,7 @@ const StepPlan& Scheduler::schedule(int q_per_tile) {
   // 2. admit waiting sequences
   while (!waiting_.empty() && budget > 0 && (int)running_.size() < max_num_seqs_) {
     Seq* s = waiting_.front();
-    if (s->num_computed == 0 && !bm_.has(s->id))
+    if (s->num_computed == 0 && !s->fed && !bm_.has(s->id))
       s->num_computed = bm_.match_prefix(s->id, s->tokens.data(), (int)s->tokens.size());
     const int remaining = (int)s->tokens.size() - s->num_computed;
     int n = std::min(remaining, budget);
@@ -203,6 +238,10 @@ const StepPlan& Scheduler::schedule(int q_per_tile) {
       break;
     }
     waiting_.pop_front();
+    // one slot per running sequence: running_ < max_num_seqs leaves one free
+    std::pop_heap(free_slots_.begin(), free_slots_.end(), std::greater<int32_t>());
+    s->slot = free_slots_.back();
+    free_slots_.pop_back();
     s->status = RUNNING;
     running_.push_back(s);
     s->scheduled = n;
@@ -241,13 +280,14 @@ const StepPlan& Scheduler::schedule(int q_per_tile) {
     const int ctx = s->num_computed + n;
     p.seq_ids.push_back(s->id);
     p.qlens.push_back(n);
+    p.state_slots.push_back(s->slot);
     p.context_lens.push_back(ctx);
     p.cu_q.push_back(p.num_tokens);
     p.max_context = std::max(p.max_context, ctx);
     const size_t off = p.block_tables.size();
     p.block_tables.resize(off + width, 0);
     std::copy(tab.begin(), tab.end(), p.block_tables.begin() + off);
-    if (ctx == (int)s->tokens.size()) {
+    if (!s->fed && ctx == (int)s->tokens.size()) {
       p.sample_rows.push_back(row0 + n - 1);
       p.sample_seq.push_back((int)plan_seqs_.size());
       p.sample_temp.push_back(s->temperature);

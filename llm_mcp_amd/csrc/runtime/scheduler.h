@@ -61,6 +61,13 @@ struct Seq {
   // finished (stop token / abort) while the plan in flight still holds a row
   // of it: the object lives until that plan is consumed
   bool zombie = false;
+  // recurrent-state slot while running (-1 otherwise): layers with a state of
+  // fixed size per sequence (linear attention, state-space, short
+  // convolutions) keep it there.  A slot is handed out uncleared: a row at
+  // position 0 starts from the zero state.
+  int slot = -1;
+  // tokens come from outside (feed()); nothing of it is sampled
+  bool fed = false;
 };
 
 constexpr int kPenWindow = 64;   // token window of the penalty kernel (one wave per row)
@@ -75,6 +82,7 @@ struct StepPlan {
   // per scheduled sequence (S), decode sequences first
   std::vector<int64_t> seq_ids;
   std::vector<int32_t> qlens, context_lens, cu_q;  // cu_q has S+1 entries
+  std::vector<int32_t> state_slots;                // recurrent-state slot per sequence
   std::vector<int32_t> block_tables;               // S x max_blocks (0-padded)
   std::vector<int32_t> sample_rows;                // token rows whose logits are sampled
   std::vector<int32_t> sample_seq;                 // index into seq_ids for each sample row
@@ -104,6 +112,11 @@ class Scheduler {
   void add(int64_t id, const std::vector<int32_t>& prompt, int max_new,
            const std::vector<int32_t>& stop_ids, bool ignore_eos, int priority,
            float temperature = 1.f, int top_k = 0, float top_p = 1.f, int64_t seed = 0);
+  // Teacher-forced sequences: feed() opens the sequence at its first call and
+  // appends tokens; each schedule() takes what is pending (a sequence with
+  // nothing pending keeps its pages and slot and is left out of the plan), no
+  // row of it is sampled, and abort() ends it.
+  void feed(int64_t id, const std::vector<int32_t>& tokens);
   bool abort(int64_t id);
   bool set_penalties(int64_t id, float repetition, float presence, float frequency, int last_n);
   // q_per_tile: queries per prefill workgroup (64 / G for the paged prefill kernel)
@@ -153,6 +166,7 @@ class Scheduler {
  private:
   void preempt(Seq* s);
   void finish(Seq* s, int reason);
+  void release_slot(Seq* s);
   bool in_plan(const Seq* s) const;
   bool length_done(const Seq* s) const;
 
@@ -164,6 +178,7 @@ class Scheduler {
   std::deque<Seq*> waiting_;
   std::vector<Seq*> running_;
   std::vector<Seq*> plan_seqs_;
+  std::vector<int32_t> free_slots_;   // min-heap: the lowest free slot first
   std::vector<Seq*> inflight_;   // samples awaiting patch() (nullptr: dropped)
   StepPlan plan_;
   int64_t arrival_ = 0;

@@ -31,8 +31,8 @@ import numpy as np
 import torch
 
 from .. import ops
-from ..models.config import LlamaConfig
-from ..models.llama import LlamaModel, StepInputs, TPContext
+from ..models.llama import StepInputs, TPContext
+from ..models.registry import build_model
 from ..utils.faults import faults
 
 log = logging.getLogger("lmx.engine")
@@ -130,6 +130,12 @@ class EngineConfig:
     use_graphs: bool = True
     part_tokens: int = 512
     seed: int = 0
+    # a KV pool of this many tokens (whole pages) instead of a share of HBM
+    kv_cache_tokens: int | None = None
+    dtype: str = "bfloat16"         # or "float32" (families that run in it)
+
+
+_DTYPES = {"bfloat16": torch.bfloat16, "float32": torch.float32}
 
 
 class _Packer:
@@ -255,7 +261,7 @@ def _load_gemm_tuning() -> None:
 
 class LLMEngine:
     def __init__(self, ecfg: EngineConfig, device: str | torch.device = "cuda",
-                 model_cfg: LlamaConfig | None = None, tp: TPContext | None = None,
+                 model_cfg=None, tp: TPContext | None = None,
                  event_sink: Callable[[list[TokenEvent]], None] | None = None,
                  weights: dict | None = None, plan_channel=None):
         """``tp`` + ``plan_channel``: member of a tensor-parallel group.  The
@@ -273,7 +279,10 @@ class LLMEngine:
         self.max_model_len = min(ecfg.max_model_len, self.cfg.max_position)
         if self.device.type == "cuda":
             _load_gemm_tuning()
-        self.model = LlamaModel(self.cfg, self.device, tp=tp, seed=ecfg.seed, weights=weights)
+        if ecfg.dtype not in _DTYPES:
+            raise ValueError(f"dtype {ecfg.dtype!r}: one of {sorted(_DTYPES)}")
+        self.model = build_model(self.cfg, self.device, dtype=_DTYPES[ecfg.dtype], tp=tp,
+                                 seed=ecfg.seed, weights=weights)
         self.tp = self.model.tp
         self.is_leader = self.tp.rank == 0
         self.chan = plan_channel
@@ -282,11 +291,12 @@ class LLMEngine:
         self.tp_comm_live: dict = {}
         self._upload_ev = None
         self.Hq, self.Hkv, self.D = self.model.Hq, self.model.Hkv, self.model.D
-        self.q_per_tile = ops.prefill_q_per_tile(self.Hq, self.Hkv, self.D)
+        self.q_per_tile = self.model.q_per_tile
+        self._alloc_states()
         self._alloc_kv()
         self.sched = _runtime.Scheduler(self.num_blocks, BLOCK_SIZE, ecfg.max_num_seqs,
                                         ecfg.max_batched_tokens, self.max_model_len,
-                                        ecfg.prefix_cache)
+                                        ecfg.prefix_cache and self.model.prefix_cache_ok)
         if ecfg.mixed_prefill_tokens and ecfg.mixed_prefill_tokens < ecfg.max_batched_tokens:
             self.sched.set_mixed_prefill_cap(ecfg.mixed_prefill_tokens, ecfg.mixed_min_decodes,
                                              ecfg.mixed_later_steps)
@@ -298,6 +308,8 @@ class LLMEngine:
         cap = 4 * (4 * T + ecfg.max_num_seqs * (self.max_blocks + 8) + 2 * T) + 16 * 64 + \
             8 * ecfg.max_num_seqs * 4 + 4 * ecfg.max_num_seqs * (PEN_WINDOW + 4) + \
             4 * ecfg.max_num_seqs + 16          # decode dispatch order
+        if self.states:      # state slots and the model's host plan
+            cap += 4 * (3 * ecfg.max_num_seqs) + 64 * (T + 16 * ecfg.max_num_seqs)
         self.packer = _Packer(cap, self.device)
         self.event_sink = event_sink
         self._intake: queue.SimpleQueue = queue.SimpleQueue()
@@ -387,17 +399,36 @@ class LLMEngine:
         self._bucket_list = sorted(self.graphs)
 
     # ------------------------------------------------------------ memory ----
+    def _alloc_states(self):
+        """One slot per running sequence of every state tensor the model keeps
+        beside the KV pages (recurrent states, convolution tails)."""
+        self.states = [torch.zeros((self.ecfg.max_num_seqs,) + tuple(shape), dtype=dt,
+                                   device=self.device)
+                       for shape, dt in self.model.state_shapes()]
+        if self.states:
+            log.info("state slots: %d x %.2f MB", self.ecfg.max_num_seqs,
+                     sum(t[0].numel() * t.element_size() for t in self.states) / 1e6)
+
     def _alloc_kv(self):
-        cfg = self.cfg
-        per_block = cfg.num_layers * 2 * self.Hkv * BLOCK_SIZE * self.D * 2
-        if self.ecfg.kv_cache_gb is not None:
+        layers = self.model.kv_layers            # (kv heads, head size) per cache layer
+        es = torch.empty((), dtype=self.model.dtype).element_size()
+        sizes = [Hkv * BLOCK_SIZE * D for Hkv, D in layers]     # elements per page of K (or V)
+        per_block = max(1, 2 * sum(sizes) * es)
+        if self.ecfg.kv_cache_tokens is not None:
+            kv_bytes = -(-self.ecfg.kv_cache_tokens // BLOCK_SIZE) * per_block
+        elif self.ecfg.kv_cache_gb is not None:
             kv_bytes = int(self.ecfg.kv_cache_gb * (1 << 30))
         elif self.device.type == "cuda":
             free, _ = torch.cuda.mem_get_info(self.device)
             kv_bytes = int(free * self.ecfg.kv_fraction)
         else:
             kv_bytes = 64 * per_block
-        self.num_blocks = max(16, kv_bytes // per_block)
+        if not layers and self.ecfg.kv_cache_tokens is None:
+            # no paged layer: pages only count tokens
+            kv_bytes = self.ecfg.max_num_seqs * math.ceil(self.max_model_len / BLOCK_SIZE)
+        self.num_blocks = kv_bytes // per_block
+        if self.ecfg.kv_cache_tokens is None:
+            self.num_blocks = max(16, self.num_blocks)
         if self.tp.size > 1:
             # the leader's scheduler hands out page ids for every rank
             gloo = torch.distributed.get_backend(self.tp.group) == "gloo"
@@ -407,14 +438,16 @@ class LLMEngine:
                                          group=self.tp.group)
             self.num_blocks = int(t.item())
         # zero-filled: masked keys multiply P = 0 with V, which must be finite
-        self.kv = torch.zeros((cfg.num_layers, 2, self.num_blocks, self.Hkv, BLOCK_SIZE * self.D),
-                              dtype=torch.bfloat16, device=self.device)
-        self.k_caches = [self.kv[l, 0].view(self.num_blocks, self.Hkv, BLOCK_SIZE, self.D)
-                         for l in range(cfg.num_layers)]
-        self.v_caches = [self.kv[l, 1].view(self.num_blocks, self.Hkv, BLOCK_SIZE // 4, self.D, 4)
-                         for l in range(cfg.num_layers)]
-        log.info("KV cache: %d blocks x %d tokens (%.1f GB)", self.num_blocks, BLOCK_SIZE,
-                 self.kv.numel() * 2 / 1e9)
+        NB = self.num_blocks
+        self.kv = torch.zeros(2 * NB * sum(sizes), dtype=self.model.dtype, device=self.device)
+        self.k_caches, self.v_caches, off = [], [], 0
+        for (Hkv, D), n in zip(layers, sizes):
+            self.k_caches.append(self.kv[off:off + NB * n].view(NB, Hkv, BLOCK_SIZE, D))
+            off += NB * n
+            self.v_caches.append(self.kv[off:off + NB * n].view(NB, Hkv, BLOCK_SIZE // 4, D, 4))
+            off += NB * n
+        log.info("KV cache: %d blocks x %d tokens (%.1f GB)", NB, BLOCK_SIZE,
+                 self.kv.numel() * es / 1e9)
 
     # ----------------------------------------------------------- sampling ---
     def _sample(self, logits, temp, topk, topp, seeds, offs, out_tok=None, out_lp=None):
@@ -469,7 +502,7 @@ class LLMEngine:
             ("temp", np.float32, (Bmax,)), ("topk", np.int32, (Bmax,)),
             ("topp", np.float32, (Bmax,)), ("seeds", np.int64, (Bmax,)),
             ("offs", np.int32, (Bmax,)), ("order", np.int32, (Bmax,)),
-            ("src", np.int32, (Bmax,))], dev)
+            ("src", np.int32, (Bmax,)), ("sslots", np.int32, (Bmax,))], dev)
         # penalty inputs: uploaded only on steps with penalised rows, read by
         # the lazily captured penalty variants of the decode graphs
         pmeta = _FixedMeta([("win", np.int32, (Bmax, PEN_WINDOW)), ("ngen", np.int32, (Bmax,)),
@@ -482,7 +515,7 @@ class LLMEngine:
         h["ids"][:] = 0; h["pos"][:] = 0; h["slots"][:] = -1; h["ctx"][:] = 1; h["bt"][:] = 0
         h["temp"][:] = 0; h["topk"][:] = 0; h["topp"][:] = 1; h["seeds"][:] = 0; h["offs"][:] = 0
         h["order"][:] = np.arange(Bmax, dtype=np.int32)
-        h["src"][:] = -1
+        h["src"][:] = -1; h["sslots"][:] = -1
         meta.mirror_all()
         meta.upload()
         self._gmeta = meta
@@ -511,7 +544,8 @@ class LLMEngine:
         g, dev, stream = self._gbuf, self.device, self._gstream
         inp = StepInputs(g["ids"][:B], g["pos"][:B], g["slots"][:B], B, g["bt"][:B],
                          g["ctx"][:B], g["cu"][:B + 1], g["tiles"], g["rows"][:B], B, B,
-                         decode_order=g["order"][:B])
+                         decode_order=g["order"][:B], state_slots=g["sslots"][:B],
+                         states=self.states)
         ws = self._decode_ws(B)
         out = {}
 
@@ -1032,35 +1066,48 @@ class LLMEngine:
         if evs and self.event_sink:
             self.event_sink(evs)
 
-    def _run_eager(self, plan):
+    def _forward_plan(self, plan, rows, extra=()):
+        """Upload a plan's metadata and run the model on it: (logits of the
+        token rows ``rows``, the uploaded tensors)."""
         T = plan["num_tokens"]
         S = len(plan["seq_ids"])
         mb = plan["max_blocks"]
-        rows = plan["sample_rows"].astype(np.int64)
         items = [
             ("ids", plan["input_ids"]), ("pos", plan["positions"]), ("slots", plan["slots"]),
             ("ctx", plan["context_lens"]), ("cu", plan["cu_q"]),
             ("bt", plan["block_tables"].reshape(S, mb)),
             ("tiles", plan["prefill_tiles"] if len(plan["prefill_tiles"]) else
-             np.zeros(2, np.int32)),
-            ("rows", rows), ("temp", plan["temp"]), ("topk", plan["topk"]),
-            ("topp", plan["topp"]), ("seeds", plan["seeds"]), ("offs", plan["offs"])]
+             np.zeros(2, np.int32)), ("rows", rows)]
         nd = plan["num_decode"]
         if nd > 1:
             items.append(("order", ops.decode_order(plan["context_lens"][:nd])))
+        host = None
+        if self.states:
+            more, host = self.model.host_plan(plan)
+            items += [("sslots", plan["state_slots"])] + more
+        d = self.packer.pack(items + list(extra))
+        self._mark_upload()
+        inp = StepInputs(d["ids"], d["pos"], d["slots"], nd, d["bt"], d["ctx"],
+                         d["cu"], d["tiles"], d["rows"], T, S, decode_order=d.get("order"),
+                         host={"cu_q": plan["cu_q"], "tiles": plan["prefill_tiles"], "rows": rows})
+        if self.states:
+            inp.state_slots, inp.states = d["sslots"], self.states
+            inp.aux = self.model.bind_plan(d, host)
+        ws = self._decode_ws(nd) if nd else self.decode_ws
+        return self.model.forward(inp, self.k_caches, self.v_caches, ws,
+                                  self.ecfg.part_tokens), d
+
+    def _run_eager(self, plan):
+        rows = plan["sample_rows"].astype(np.int64)
+        extra = [("temp", plan["temp"]), ("topk", plan["topk"]), ("topp", plan["topp"]),
+                 ("seeds", plan["seeds"]), ("offs", plan["offs"])]
         samples = self.is_leader or self.sample_all
         pen = bool(plan.get("any_penalty")) and samples
         if pen:   # one pack, one upload: the pinned staging buffer is reused per call
             N = len(plan["sample_rows"])
-            items += [("win", plan["pen_window"].reshape(N, PEN_WINDOW)),
+            extra += [("win", plan["pen_window"].reshape(N, PEN_WINDOW)),
                       ("ngen", plan["pen_ngen"]), ("pen", plan["pen_params"].reshape(N, 3))]
-        d = self.packer.pack(items)
-        self._mark_upload()
-        inp = StepInputs(d["ids"], d["pos"], d["slots"], plan["num_decode"], d["bt"], d["ctx"],
-                         d["cu"], d["tiles"], d["rows"], T, S, decode_order=d.get("order"),
-                         host={"cu_q": plan["cu_q"], "tiles": plan["prefill_tiles"], "rows": rows})
-        ws = self._decode_ws(plan["num_decode"]) if plan["num_decode"] else self.decode_ws
-        logits = self.model.forward(inp, self.k_caches, self.v_caches, ws, self.ecfg.part_tokens)
+        logits, d = self._forward_plan(plan, rows, extra)
         self._peer_check()
         if not samples:
             return None, None
@@ -1085,6 +1132,9 @@ class LLMEngine:
             a = h[k]
             a[:n] = plan[_PLAN_KEY.get(k, k)]
             a[n:B] = fill
+        if self.states:
+            h["sslots"][:n] = plan["state_slots"]
+            h["sslots"][n:B] = -1
         src = plan.get("input_src")
         if src is not None and plan.get("num_pending_inputs"):
             h["src"][:n] = src
@@ -1163,6 +1213,62 @@ class LLMEngine:
         self._peer_raise()      # this step's collectives were sound (see _peer_check)
         h = self._hout_np[k]
         return h[0, :n].copy(), h[1, :n].view(np.float32).copy()
+
+    # ------------------------------------------------- teacher forcing ------
+    def feed(self, entries: list[tuple[int, list[int], list[int]]],
+             end: list[int] = ()) -> torch.Tensor:
+        """One step over given tokens: ``entries`` are (sequence id, its next
+        tokens, places among them whose logits are wanted).  A sequence is
+        admitted at its first entry, runs on from the cache and state its
+        earlier entries left, and may be left out of a step; ``end`` gives
+        back what finished sequences hold.  All entries run as one batch (more
+        than one step only when they exceed ``max_batched_tokens``); nothing
+        is sampled.  Returns fp32 logits [wanted, vocab], in the order of the
+        entries and their places.  Must not be mixed with submitted requests."""
+        if self._reqs or self.chan is not None:
+            raise RuntimeError("feed: an engine without requests, alone on its GPU")
+        where: dict[int, dict[int, list[int]]] = {}    # id -> position -> output rows
+        n_out = 0
+        for sid, toks, want in entries:
+            base = len(self.sched.seq_tokens(sid))
+            bad = [t for t in toks if not 0 <= t < self.cfg.vocab_size]
+            if bad or any(not 0 <= w < len(toks) for w in want):
+                raise ValueError(f"feed: token or place out of range in sequence {sid}")
+            if sid in where:
+                raise ValueError(f"feed: sequence {sid} twice in a step")
+            where[sid] = {}
+            for w in want:
+                where[sid].setdefault(base + w, []).append(n_out)
+                n_out += 1
+        for sid, toks, _ in entries:
+            self.sched.feed(sid, list(toks))
+        out = torch.empty((n_out, self.cfg.vocab_size), dtype=torch.float32)
+        while True:
+            plan = self.sched.schedule(self.q_per_tile)
+            if plan["num_tokens"] == 0:
+                break
+            rows, dst = [], []
+            for i, sid in enumerate(plan["seq_ids"].tolist()):
+                r0, r1 = int(plan["cu_q"][i]), int(plan["cu_q"][i + 1])
+                p0 = int(plan["positions"][r0])
+                for pos in sorted(p for p in where.get(sid, {}) if p0 <= p < p0 + r1 - r0):
+                    for k in where[sid].pop(pos):
+                        rows.append(r0 + pos - p0)
+                        dst.append(k)
+            # a step without wanted rows still runs every layer
+            logits, _ = self._forward_plan(plan, np.asarray(rows or [0], np.int64))
+            if rows:
+                out[dst] = logits.float().cpu()
+            elif self.device.type == "cuda":
+                torch.cuda.synchronize(self.device)   # the pinned staging buffer is reused
+            self.sched.update(np.zeros(0, np.int32))
+            self.stats["steps"] += 1
+            self.stats["prefill_tokens"] += plan["num_prefill_tokens"]
+        if any(where.values()):
+            raise RuntimeError("feed: out of KV pages")
+        for sid in end:
+            self.sched.abort(sid)
+        return out
 
     # ----------------------------------------------------- offline helper ---
     def generate(self, prompts: list[list[int]], params: SamplingParams,

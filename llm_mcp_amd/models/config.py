@@ -8,6 +8,7 @@ are kept only for foreign names (policy/inference.py)."""
 from __future__ import annotations
 
 import json
+import math
 from dataclasses import asdict, dataclass, field
 from pathlib import Path
 
@@ -142,6 +143,84 @@ class BertConfig:
         return asdict(self)
 
 
+@dataclass
+class ZegopelConfig:
+    """Zegopel: a decoder whose layers each name their own token mixer
+    (``lightning`` linear attention, ``mamba2`` state-space, or ``attention``
+    with short convolutions) and feed-forward, with their own sizes.
+
+    ``layers`` holds one dict per layer, as in the checkpoint's config.json:
+    ``{"type": ..., "mixer": {sizes and constants}, "mlp": {"kind", "ff"} | None}``."""
+    name: str = "zegopel"
+    vocab_size: int = 512
+    hidden_size: int = 256
+    layers: list = field(default_factory=list)
+    rms_eps: float = 1e-5
+    # positions enter only through the query temperature: no table bounds them
+    max_position: int = 1 << 20
+    bos_token_id: int | None = None
+    eos_token_ids: tuple = ()
+    family: str = "zegopel"
+    kind: str = "chat"
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def params(self) -> int:
+        from .zegopel import tensor_shapes
+        return sum(math.prod(s) for s in tensor_shapes(self).values())
+
+    @property
+    def params_b(self) -> float:
+        return round(self.params / 1e9, 3)
+
+    @property
+    def context_k(self) -> int:
+        return self.max_position // 1024
+
+    def to_dict(self) -> dict:
+        return asdict(self)
+
+
+def zegopel_stack(pattern: str, ff: int, lightning: dict, mamba2: dict,
+                  attention: dict) -> list:
+    """Layer list from a pattern of L (lightning), M (mamba2), A (attention):
+    attention layers carry the feed-forward."""
+    kinds = {"L": ("lightning", lightning), "M": ("mamba2", mamba2), "A": ("attention", attention)}
+    return [{"type": kinds[c][0], "mixer": dict(kinds[c][1]),
+             "mlp": {"kind": "dense", "ff": ff} if c == "A" else None} for c in pattern]
+
+
+def _slopes(heads: int) -> list:
+    """Per-head decays exp(-2^(-8 (h + 1) / heads)): from fast to slow."""
+    return [math.exp(-2.0 ** (-8.0 * (h + 1) / heads)) for h in range(heads)]
+
+
+def _zegopel_tiny() -> ZegopelConfig:
+    return ZegopelConfig(
+        name="tiny-zegopel", vocab_size=512, hidden_size=192, bos_token_id=506,
+        eos_token_ids=(510,), layers=zegopel_stack(
+            "LMALA", 256,
+            dict(heads=3, dim=32, vdim=48, decay=[0.5, 0.9, 0.995]),
+            dict(heads=6, vdim=32, state=40, groups=3, conv=4, norm_groups=2),
+            dict(heads=4, kv_heads=2, dim=64, vdim=64, conv=3, scale=0.125,
+                 q_temp=dict(coef=0.3, every=64))))
+
+
+def _zegopel_8b() -> ZegopelConfig:
+    """Llama-3-8B's width, head layout and size (random weights: benchmarks)."""
+    return ZegopelConfig(
+        name="zegopel-8b", vocab_size=128256, hidden_size=4096, bos_token_id=128000,
+        eos_token_ids=(128001, 128009), layers=zegopel_stack(
+            "LMA" * 16, 14336,
+            dict(heads=32, dim=128, vdim=128, decay=_slopes(32)),
+            dict(heads=64, vdim=128, state=128, groups=8, conv=4, norm_groups=8),
+            dict(heads=32, kv_heads=8, dim=128, vdim=128, conv=4, scale=128 ** -0.5,
+                 q_temp=dict(coef=0.1, every=8192))))
+
+
 _LLAMA32_ROPE = {"rope_type": "llama3", "factor": 32.0, "low_freq_factor": 1.0,
                  "high_freq_factor": 4.0, "original_max_position_embeddings": 8192}
 
@@ -233,6 +312,8 @@ PRESETS: dict[str, object] = {
     "tiny-bert-mean": BertConfig(name="tiny-bert-mean", vocab_size=512, hidden_size=256,
                                  intermediate_size=512, num_layers=2, num_heads=2, head_dim=128,
                                  embed_dim=256, max_position=256, pooling="mean"),
+    "tiny-zegopel": _zegopel_tiny(),
+    "zegopel-8b": _zegopel_8b(),
     "tiny-nomic": NomicBertConfig(name="tiny-nomic", vocab_size=512, hidden_size=256,
                                   intermediate_size=512, num_layers=2, num_heads=2, head_dim=128,
                                   embed_dim=256, max_position=2048),
@@ -259,7 +340,10 @@ ALIASES = {
 def resolve(name: str):
     """Preset by name or alias.  ``<name>@L<n>`` keeps the preset's shapes
     with only n layers (e.g. ``llama-3-70b@L8``: one-GPU rehearsals of the
-    70B TP layout; never a number for the full model)."""
+    70B TP layout; never a number for the full model).  A directory with a
+    config.json is a checkpoint: its own configuration."""
+    if is_checkpoint_dir(name):
+        return from_hf_config(Path(name) / "config.json")
     base, _, layers = name.partition("@L")
     key = ALIASES.get(base, base)
     if key not in PRESETS:
@@ -270,13 +354,34 @@ def resolve(name: str):
         n = int(layers)
         if n < 1 or n > cfg.num_layers:
             raise KeyError(f"{name!r}: layer count must be 1..{cfg.num_layers}")
+        if isinstance(cfg, ZegopelConfig):
+            return dataclasses.replace(cfg, name=name, layers=cfg.layers[:n])
         cfg = dataclasses.replace(cfg, name=name, num_layers=n)
     return cfg
+
+
+def is_checkpoint_dir(name: str) -> bool:
+    return (Path(name) / "config.json").is_file()
+
+
+def _zegopel_from_json(cfg: dict, name: str) -> ZegopelConfig:
+    for i, L in enumerate(cfg["layers"]):
+        if L["type"] not in ("lightning", "mamba2", "attention"):
+            raise ValueError(f"layer {i}: unknown mixer {L['type']!r}")
+        if L.get("mlp") is not None and L["mlp"].get("kind") != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward {L['mlp'].get('kind')!r}")
+    eos = cfg.get("eos_token_id", ())
+    return ZegopelConfig(
+        name=name, vocab_size=cfg["vocab"], hidden_size=cfg["width"], layers=cfg["layers"],
+        rms_eps=cfg["norm"]["eps"], bos_token_id=cfg.get("bos_token_id"),
+        eos_token_ids=tuple(eos) if isinstance(eos, (list, tuple)) else (eos,))
 
 
 def from_hf_config(path: str | Path):
     """Build a config from a HF config.json (local file; no network)."""
     cfg = json.loads(Path(path).read_text())
+    if cfg.get("architecture") == "Zegopel":
+        return _zegopel_from_json(cfg, Path(path).resolve().parent.name)
     arch = (cfg.get("architectures") or [""])[0]
     if "Llama" in arch or "Qwen2" in arch or "Qwen3" in arch or "Mistral" in arch:
         qwen = "Qwen2" in arch

@@ -55,6 +55,13 @@ class StepInputs:
     # host copies of the plan's cu_q / prefill_tiles / sample_rows (numpy), when
     # the caller has them: lets the model split a step without a device sync
     host: dict | None = None
+    # models with per-sequence state (``state_shapes``): each sequence's slot,
+    # the state tensors, the host plan's extra index tensors (``host_plan``)
+    state_slots: torch.Tensor | None = None    # int32 [S], -1 = padding row
+    states: list | None = None
+    aux: dict | None = None
+    decode_ws: object = None
+    part_tokens: int = 512
 
 
 class TPContext:
@@ -246,12 +253,36 @@ class _Done:
 
 
 class LlamaModel:
+    # what the engine allocates and plans for a model (see ZegopelModel for one
+    # that uses all of it)
+    prefix_cache_ok = True        # a cached prefix page is all a sequence needs of it
+
+    def state_shapes(self) -> list:
+        """Per-slot state tensors: [(shape, dtype)]."""
+        return []
+
+    def host_plan(self, plan: dict) -> tuple[list, dict]:
+        """Extra index arrays of an eager step [(name, int32 array)] and the
+        host values that go with them."""
+        return [], {}
+
+    @property
+    def kv_layers(self) -> list:
+        """(kv heads, head size) of each paged-cache layer."""
+        return [(self.Hkv, self.D)] * self.cfg.num_layers
+
+    @property
+    def q_per_tile(self) -> int:
+        return ops.prefill_q_per_tile(self.Hq, self.Hkv, self.D)
+
     def __init__(self, cfg: LlamaConfig, device: torch.device | str = "cuda",
                  dtype=torch.bfloat16, tp: TPContext | None = None, seed: int = 0,
                  weights: dict | None = None):
         self.cfg = cfg
         self.device = torch.device(device)
         self.dtype = dtype
+        if dtype != torch.bfloat16 and self.device.type == "cuda":
+            raise ValueError(f"{cfg.family}: served in bfloat16 only")
         self.tp = tp or TPContext()
         T = self.tp.size
         if cfg.num_heads % T or cfg.intermediate_size % T:

@@ -243,3 +243,42 @@ def save_hf_llama(full: dict, cfg: LlamaConfig, path: str) -> None:
           "_name_or_path": cfg.name}
     with open(os.path.join(path, "config.json"), "w") as f:
         json.dump(hf, f)
+
+
+def load_tensors(path: str, shapes: dict[str, tuple]) -> dict:
+    """Named tensors of a safetensors checkpoint directory (host memory, the
+    checkpoint's own dtypes), each checked against its expected shape."""
+    rd = _Reader(path)
+    out = {}
+    for name, shape in shapes.items():
+        t = rd.rows(name)
+        if tuple(t.shape) != tuple(shape):
+            raise ValueError(f"{name}: checkpoint shape {tuple(t.shape)}, expected {tuple(shape)}")
+        out[name] = t
+    return out
+
+
+def load_weights(path: str, cfg, device, rank: int = 0, size: int = 1) -> dict:
+    """This rank's weights of a chat model's checkpoint directory, by family."""
+    if cfg.family == "zegopel":
+        from .zegopel import tensor_shapes
+        if size > 1:
+            raise ValueError("zegopel: no tensor-parallel form")
+        return load_tensors(path, tensor_shapes(cfg))
+    return load_llama_weights(path, cfg, device, rank, size)
+
+
+def save_zegopel(weights: dict, cfg, path: str) -> None:
+    """Write named tensors and the configuration as a checkpoint directory."""
+    from safetensors.torch import save_file
+    os.makedirs(path, exist_ok=True)
+    save_file({k: v.detach().to("cpu").contiguous() for k, v in weights.items()},
+              os.path.join(path, "model.safetensors"))
+    js = {"architecture": "Zegopel", "layers": cfg.layers, "norm": {"eps": cfg.rms_eps},
+          "vocab": cfg.vocab_size, "width": cfg.hidden_size}
+    if cfg.eos_token_ids:
+        js["eos_token_id"] = list(cfg.eos_token_ids)
+    if cfg.bos_token_id is not None:
+        js["bos_token_id"] = cfg.bos_token_id
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(js, f)

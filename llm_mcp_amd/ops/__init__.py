@@ -230,7 +230,8 @@ class DecodeWorkspace:
 def paged_decode_attention(q: torch.Tensor, k_cache, v_cache, block_tables, context_lens,
                            scale: float, out: torch.Tensor, ws: DecodeWorkspace | None = None,
                            part_tokens: int = 512, Hq: int | None = None,
-                           order: torch.Tensor | None = None, rope: tuple | None = None
+                           order: torch.Tensor | None = None, rope: tuple | None = None,
+                           gate: torch.Tensor | None = None, precise: bool = False
                            ) -> torch.Tensor:
     """q: [B, Hq*D] rows (row stride = q.stride(0)); out: [B, Hq*D].
     ``order`` (int32 [B], optional): a permutation of the rows, longest
@@ -239,7 +240,9 @@ def paged_decode_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cont
     the UNROTATED fused QKV row ([q | k | v] heads); the kernel rotates q in
     registers and writes the step's rotated k and v into the cache at
     ``slots`` itself (K2 + K5 fused into K4: ``rope_and_cache`` is skipped for
-    these rows; no q/k-norm models)."""
+    these rows; no q/k-norm models).  ``gate`` ([B, Hq*D] rows): the output is
+    multiplied by sigmoid(gate).  ``precise``: softmax weights enter the PV
+    product with fp32 precision (a bf16 pair) instead of one bf16."""
     B = q.shape[0]
     NB, Hkv, BS, D = k_cache.shape
     Hq = Hq or (q.shape[1] // D)
@@ -250,9 +253,12 @@ def paged_decode_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cont
     if not q.is_cuda:
         o = ref.paged_decode(q[:, : Hq * D].reshape(B, Hq, D), k_cache, v_cache, block_tables,
                              context_lens, scale)
-        out.copy_(o.reshape(B, Hq * D))
+        out.copy_(ref.gate_rows(o.reshape(B, Hq * D), gate))
         return out
     _bf16(q, "q")
+    _chk(gate is None or (gate.stride(1) == 1 and gate.dtype == torch.bfloat16
+                          and gate.shape[0] >= B and gate.shape[1] >= Hq * D), "gate rows")
+    _chk(not (precise and rope is not None), "precise weights: no fused-rotary form")
     _chk(D in (64, 128) and BS == 32, "paged decode kernel needs D in (64,128), BS=32")
     _chk(Hq % Hkv == 0 and Hq // Hkv <= 16, "GQA group must be <= 16")
     _chk(block_tables.dtype == torch.int32 and context_lens.dtype == torch.int32, "int32 meta")
@@ -274,7 +280,8 @@ def paged_decode_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cont
                           out.stride(0),
                           _ptr(ws.part_o) if ws else 0, _ptr(ws.part_ml) if ws else 0, B, Hq, Hkv,
                           D, BS, float(scale), part_tokens, max_parts, _ptr(pos), _ptr(cs),
-                          _ptr(slots), _stream())
+                          _ptr(slots), _ptr(gate), gate.stride(0) if gate is not None else 0,
+                          int(precise), _stream())
     return out
 
 
@@ -290,13 +297,16 @@ def decode_order(context_lens) -> "np.ndarray":
 def paged_prefill_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q,
                             context_lens, tiles, scale: float, out: torch.Tensor,
                             causal: bool = True, Hq: int | None = None,
-                            q_per_tile: int | None = None, rope=None) -> torch.Tensor:
+                            q_per_tile: int | None = None, rope=None,
+                            gate: torch.Tensor | None = None,
+                            precise: bool = False) -> torch.Tensor:
     """Varlen prefill. q/out: [T, Hq*D] rows; tiles: int32 [(seq, q_start)]
     built with ``q_per_tile`` queries per tile (default
     ``prefill_q_per_tile(Hq, Hkv, D)``; the kernel's workgroup width follows
     from it).  ``rope`` = (positions int32 [rows], cos_sin fp32 [P, D]): q is
     unrotated and the kernel applies the rotary embedding (the rope/cache
-    kernel ran with ``skip_q``)."""
+    kernel ran with ``skip_q``).  ``gate`` / ``precise``: as in
+    ``paged_decode_attention``."""
     NB, Hkv, BS, D = k_cache.shape
     T = q.shape[0]
     Hq = Hq or (q.shape[1] // D)
@@ -308,9 +318,12 @@ def paged_prefill_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_
         o = ref.paged_prefill(q[:, : Hq * D].reshape(T, Hq, D), k_cache, v_cache, block_tables,
                               cu_q, context_lens, scale, causal)
         a, b = int(cu_q[0]), int(cu_q[len(context_lens)])
-        out[a:b].copy_(o.reshape(T, Hq * D)[a:b])
+        out[a:b].copy_(ref.gate_rows(o.reshape(T, Hq * D), gate)[a:b])
         return out
     _bf16(q, "q")
+    _chk(gate is None or (gate.stride(1) == 1 and gate.dtype == torch.bfloat16
+                          and gate.shape[1] >= Hq * D and gate.stride(0) % 8 == 0
+                          and gate.data_ptr() % 16 == 0), "gate rows")
     _chk(D in (64, 128) and BS == 32, "paged prefill kernel needs D in (64,128), BS=32")
     _chk(Hq % Hkv == 0 and Hq // Hkv <= 16, "GQA group must be <= 16")
     _chk(tiles.dtype == torch.int32 and cu_q.dtype == torch.int32, "int32 meta")
@@ -321,7 +334,8 @@ def paged_prefill_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_
                            Hq, Hkv, D, BS, float(scale), int(causal),
                            q_per_tile or prefill_q_per_tile(Hq, Hkv, D),
                            _ptr(rope[0]) if rope is not None else 0,
-                           _ptr(rope[1]) if rope is not None else 0, _stream())
+                           _ptr(rope[1]) if rope is not None else 0, _ptr(gate),
+                           gate.stride(0) if gate is not None else 0, int(precise), _stream())
     return out
 
 
@@ -437,13 +451,15 @@ def apply_penalties(logits: torch.Tensor, window: torch.Tensor, ngen: torch.Tens
         if on is not None and int(on[0]) == 0:
             return logits
         return ref.apply_penalties(logits, window, ngen, pen, v0)
-    _chk(logits.dtype == torch.bfloat16 and logits.stride(1) == 1, "bf16 logits rows")
+    _chk(logits.dtype in (torch.bfloat16, torch.float32) and logits.stride(1) == 1,
+         "bf16 / fp32 logits rows")
     _chk(window.dtype == torch.int32 and window.is_contiguous() and window.shape[0] >= B
          and window.shape[1] <= 64, "penalty window")
     _chk(ngen.dtype == torch.int32 and pen.dtype == torch.float32 and pen.is_contiguous(),
          "penalty params")
-    native().apply_penalties(_ptr(logits), logits.stride(0), B, V, _ptr(window), _ptr(ngen),
-                             _ptr(pen), _ptr(on), window.shape[1], v0, _stream())
+    native().apply_penalties(_ptr(logits), int(logits.dtype == torch.bfloat16), logits.stride(0),
+                             B, V, _ptr(window), _ptr(ngen), _ptr(pen), _ptr(on),
+                             window.shape[1], v0, _stream())
     return logits
 
 
@@ -470,7 +486,7 @@ def silu_mul(x: torch.Tensor, out: torch.Tensor | None = None, block: int = 0) -
     rows = x.numel() // x.shape[-1]
     if out is None:
         out = torch.empty(x.shape[:-1] + (I,), dtype=x.dtype, device=x.device)
-    native().glu(_ptr(out), _ptr(x), rows, I, 0, block, _stream())
+    native().glu(_ptr(out), _ptr(x), rows, I, 0, block, 1, _stream())
     return out
 
 
@@ -481,7 +497,20 @@ def gelu_mul(x: torch.Tensor) -> torch.Tensor:
     I = x.shape[-1] // 2
     rows = x.numel() // x.shape[-1]
     out = torch.empty(x.shape[:-1] + (I,), dtype=x.dtype, device=x.device)
-    native().glu(_ptr(out), _ptr(x), rows, I, 1, 0, _stream())
+    native().glu(_ptr(out), _ptr(x), rows, I, 1, 0, 1, _stream())
+    return out
+
+
+def relu_mul(x: torch.Tensor) -> torch.Tensor:
+    """relu(gate) * up of a fused gate|up projection output (bf16 or fp32)."""
+    if not x.is_cuda:
+        return ref.relu_mul(x)
+    _chk(x.dtype in (torch.bfloat16, torch.float32) and x.is_contiguous()
+         and x.shape[-1] % 16 == 0, "relu_mul shape")
+    I = x.shape[-1] // 2
+    rows = x.numel() // x.shape[-1]
+    out = torch.empty(x.shape[:-1] + (I,), dtype=x.dtype, device=x.device)
+    native().glu(_ptr(out), _ptr(x), rows, I, 2, 0, int(x.dtype == torch.bfloat16), _stream())
     return out
 
 
@@ -757,7 +786,10 @@ def linear(x: torch.Tensor, w: torch.Tensor, defer: bool = False,
     hipBLASLt (bias in its epilogue).  ``defer``: the caller feeds the result to
     ``rms_norm(..., residual=)``, so a table entry for the partials-only form
     (epi 2) may return ``Partials`` and leave the K reduction to the norm.
-    ``out``: a bf16 [M, N] destination (plain products only, not with defer)."""
+    ``out``: a bf16 [M, N] destination (plain products only, not with defer).
+    fp32 operands: the library's true-fp32 product."""
+    if x.dtype == torch.float32:
+        return _into(out, torch.nn.functional.linear(x, w, bias))
     _chk(out is None or not defer, "linear: out= is for the plain product")
     if x.is_cuda and x.dim() == 2 and (piece := rows_split(x.shape[0], w.shape[0], w.shape[1], 0, w)):
         return _by_rows(x, piece, w.shape[0], lambda xs, o: linear(xs, w, bias=bias, out=o))
@@ -1722,3 +1754,7 @@ def pgemm_sk(a: torch.Tensor, w: torch.Tensor, splits: int, act: int = 0, epi: i
     native().pgemm_sk(_ptr(out), _ptr(a), _ptr(w), _ptr(slabs), _ptr(cnt), _PG_CNT, M, N, K,
                       a.stride(0), w.stride(0), out.stride(0), act, splits, 0, _stream())
     return out
+
+
+from .mixers import (ScanSegments, attention_any, conv_qkv_cache, gated_norm,  # noqa: E402,F401
+                     linear_scan, sandwich_norm, scan_segments, short_conv)

@@ -1,0 +1,315 @@
+"""Ops of the token mixers beyond plain attention: linear-attention /
+state-space scans, short causal convolutions, sandwich and gated norms, and
+paged attention for any head geometry.
+
+Same conventions as the package: GPU tensors run the kernels of
+``csrc/kernels`` (bf16 or fp32 rows), CPU tensors the references in
+``ops.ref``, and every shape is checked on the host before a launch.
+
+Per-sequence state (recurrent state, convolution inputs) is a tensor
+[slots, ...]; a step names each sequence's slot.  Rows that start at position 0
+(``ctx == rows of the sequence in this step``) start from the zero state, so
+slots are never cleared.
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+
+import numpy as np
+import torch
+
+from . import Partials, _chk, _ptr, _stream, native, ref
+
+CONV_TILE = 64        # tokens per convolution workgroup
+SCAN_CHUNK = 64       # SC in csrc/kernels/linscan.hip
+SCAN_VT = 64          # v columns per workgroup (SVT)
+SCAN_FILL = 512       # workgroups wanted before a sequence is cut into segments
+
+
+def _rows_dtype(t: torch.Tensor, name: str) -> int:
+    """1 for bf16 rows, 0 for fp32 rows."""
+    _chk(t.dtype in (torch.bfloat16, torch.float32), f"{name}: bf16 or fp32, got {t.dtype}")
+    return int(t.dtype == torch.bfloat16)
+
+
+def _f32(t: torch.Tensor | None, n: int, name: str) -> None:
+    _chk(t is None or (t.dtype == torch.float32 and t.numel() == n and t.is_contiguous()),
+         f"{name}: fp32 [{n}]")
+
+
+def _meta(S: int, **ts) -> None:
+    for name, t in ts.items():
+        _chk(t.dtype == torch.int32 and t.is_cuda and t.is_contiguous()
+             and t.numel() >= S + (name == "cu_q"), f"{name}: int32[{S}]")
+
+
+# -------------------------------------------------------------------- norms --
+def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tensor | None = None,
+                  w_pre: torch.Tensor | None = None, ids: torch.Tensor | None = None,
+                  table: torch.Tensor | None = None, rows: torch.Tensor | None = None,
+                  dtype: torch.dtype = torch.bfloat16) -> torch.Tensor | None:
+    """One pass over the fp32 residual stream between two sublayers:
+
+        r = table[ids] (if given) else residual
+        r += rms(y) * w_post         (y: sublayer output rows or ``Partials``)
+        residual = r                 (unless ``rows`` is given)
+        return rms(r) * w_pre        (``dtype`` rows; None without w_pre)
+
+    ``rows`` (int64): only these rows are normed, the residual stays as it is.
+    The gains are fp32 vectors."""
+    T, d = residual.shape
+    if not residual.is_cuda:
+        return ref.sandwich_norm(residual, eps, y, w_post, w_pre, ids, table, rows, dtype)
+    _chk(residual.dtype == torch.float32 and residual.is_contiguous(), "residual: fp32 rows")
+    _f32(w_post, d, "w_post"); _f32(w_pre, d, "w_pre")
+    bf = int(dtype == torch.bfloat16)
+    yp, y_ld, slabs, sstride = 0, 0, 0, 0
+    if isinstance(y, Partials):
+        _chk((y.M, y.N) == (T, d), "sandwich_norm partials shape")
+        yp, y_ld, slabs, sstride = _ptr(y.slabs), d, y.S, y.M * y.N
+    elif y is not None:
+        _chk(y.shape == (T, d) and y.stride(1) == 1 and y.dtype == dtype, "sandwich_norm y rows")
+        yp, y_ld = _ptr(y), y.stride(0)
+    _chk((y is None) == (w_post is None), "w_post goes with y")
+    if ids is not None:
+        _chk(ids.dtype == torch.int32 and ids.numel() >= T and table.dtype == dtype
+             and table.is_contiguous() and table.shape[1] == d, "embedding rows")
+    n = T
+    if rows is not None:
+        _chk(rows.dtype == torch.int64 and rows.is_contiguous(), "rows: int64")
+        n = rows.numel()
+    out = torch.empty((n, d), dtype=dtype, device=residual.device) if w_pre is not None else None
+    native().sandwich_norm(_ptr(out), _ptr(residual), yp, y_ld, slabs, sstride, _ptr(ids),
+                           _ptr(table), _ptr(w_post), _ptr(w_pre), _ptr(rows), n, d, float(eps),
+                           bf, _stream())
+    return out
+
+
+def gated_norm(x: torch.Tensor, gate: torch.Tensor, w: torch.Tensor, groups: int, eps: float,
+               gate_first: bool) -> torch.Tensor:
+    """RMS norm of x in ``groups`` equal parts of a row, gain w (fp32), gated:
+    rms(x) * w * sigmoid(gate), or with ``gate_first`` rms(x * silu(gate)) * w."""
+    T, C = x.shape
+    _chk(C % groups == 0, "gated_norm groups")
+    if not x.is_cuda:
+        return ref.gated_norm(x, gate, w, groups, eps, gate_first)
+    bf = _rows_dtype(x, "x")
+    _f32(w, C, "w")
+    _chk(gate.dtype == x.dtype and gate.shape[0] == T and gate.shape[1] >= C
+         and gate.stride(1) == 1 and x.stride(1) == 1, "gated_norm rows")
+    out = torch.empty((T, C), dtype=x.dtype, device=x.device)
+    native().gated_norm(_ptr(out), out.stride(0), _ptr(x), x.stride(0), _ptr(gate),
+                        gate.stride(0), _ptr(w), T, C, groups, int(gate_first), float(eps), bf,
+                        _stream())
+    return out
+
+
+# -------------------------------------------------------------- convolution --
+def row_tiles(qlens, tile: int) -> np.ndarray:
+    """int32 [n, 2] (sequence, first row in it): every sequence's rows in tiles."""
+    nt = -(-np.asarray(qlens, dtype=np.int64) // tile)
+    seq = np.repeat(np.arange(len(nt)), nt)
+    base = np.repeat(np.cumsum(nt) - nt, nt)
+    start = (np.arange(len(seq)) - base) * tile
+    return np.stack([seq, start], 1).astype(np.int32)
+
+
+def conv_tiles(cu_q) -> np.ndarray:
+    """``row_tiles`` of a step's convolutions (all its sequences)."""
+    return row_tiles(np.diff(np.asarray(cu_q)), CONV_TILE)
+
+
+def _conv_meta(u, w, state, tiles, cu_q, ctx, slots):
+    taps, C = w.shape
+    S = ctx.numel()
+    _chk(w.dtype == torch.float32 and w.is_contiguous(), "conv weights: fp32 [taps, C]")
+    _chk(u.stride(1) == 1 and u.shape[1] >= C, "conv rows")
+    _chk(1 <= taps <= 32, "conv taps 1..32")
+    _chk(taps == 1 or (state is not None and state.dtype == u.dtype and state.is_contiguous()
+                       and tuple(state.shape[1:]) == (taps - 1, C)),
+         "conv state [slots, taps - 1, C]")
+    _meta(S, cu_q=cu_q, ctx=ctx, slots=slots)
+    if tiles is not None:
+        _chk(tiles.dtype == torch.int32 and tiles.is_contiguous(), "conv tiles int32")
+    else:
+        _chk(u.shape[0] == S, "conv without tiles: one row per sequence")
+    return taps, C, (S if tiles is None else tiles.numel() // 2)
+
+
+def short_conv(u: torch.Tensor, w: torch.Tensor, state: torch.Tensor | None, cu_q, ctx, slots,
+               bias: torch.Tensor | None = None, silu: bool = False,
+               tiles: torch.Tensor | None = None) -> torch.Tensor:
+    """Causal convolution over time of each channel (w fp32 [taps, C], last
+    tap = the current token), optionally SiLU; ``state`` [slots, taps - 1, C]
+    carries the last inputs.  ``tiles`` (``conv_tiles``): needed when a
+    sequence has more than one row."""
+    taps, C = w.shape
+    out = torch.empty((u.shape[0], C), dtype=u.dtype, device=u.device)
+    if not u.is_cuda:
+        ref.short_conv(u, w, bias, state, cu_q, ctx, slots, out, silu)
+        return out
+    bf = _rows_dtype(u, "u")
+    taps, C, n = _conv_meta(u, w, state, tiles, cu_q, ctx, slots)
+    _f32(bias, C, "conv bias")
+    native().short_conv(_ptr(u), u.stride(0), _ptr(w), _ptr(bias), _ptr(state), _ptr(tiles), n,
+                        CONV_TILE, _ptr(cu_q), _ptr(ctx), _ptr(slots), C, taps, _ptr(out),
+                        out.stride(0), int(silu), bf, _stream())
+    return out
+
+
+def conv_qkv_cache(u: torch.Tensor, w: torch.Tensor, in_bias: torch.Tensor | None,
+                   state: torch.Tensor | None, cu_q, ctx, state_slots, positions, slots,
+                   k_cache, v_cache, Hq: int, dk: int, eps: float, temp: tuple[float, float],
+                   tiles: torch.Tensor | None = None) -> torch.Tensor:
+    """The projection rows' q | k | v heads (each padded to D channels) through
+    a short convolution; q and k divided by their root mean square over the
+    ``dk`` true channels; q times 1 + temp[0] ln(floor((p + 1) / temp[1]) + 1);
+    k and v written to the paged cache at ``slots``.  ``in_bias``: the
+    projection's bias (fp32 [C]).  Returns q rows [T, Hq * D]."""
+    _, Hkv, BS, D = k_cache.shape
+    T = u.shape[0]
+    q = torch.empty((T, Hq * D), dtype=u.dtype, device=u.device)
+    if not u.is_cuda:
+        ref.conv_qkv_cache(u, w, in_bias, state, cu_q, ctx, state_slots, q, k_cache, v_cache,
+                           positions, slots, Hq, Hkv, D, dk, eps, temp)
+        return q
+    bf = _rows_dtype(u, "u")
+    taps, C, n = _conv_meta(u, w, state, tiles, cu_q, ctx, state_slots)
+    _f32(in_bias, C, "projection bias")
+    _chk(C == (Hq + 2 * Hkv) * D and k_cache.dtype == u.dtype and v_cache.dtype == u.dtype
+         and k_cache.is_contiguous() and v_cache.is_contiguous(), "q | k | v heads / caches")
+    _meta(T, positions=positions, rows=slots)
+    native().conv_qkv_cache(_ptr(u), u.stride(0), _ptr(w), _ptr(in_bias), _ptr(state),
+                            _ptr(tiles), n, CONV_TILE, _ptr(cu_q), _ptr(ctx), _ptr(state_slots),
+                            taps, _ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache),
+                            _ptr(positions), _ptr(slots), Hq, Hkv, D, dk, BS, float(eps),
+                            float(temp[0]), float(temp[1]), bf, _stream())
+    return q
+
+
+# --------------------------------------------------------------------- scan --
+@dataclass
+class ScanSegments:
+    """Row segments of a step's multi-token sequences for the chunked scan."""
+    segs: torch.Tensor      # int32 [n, 4]: sequence, first row, end row, last of its sequence
+    first: torch.Tensor     # int32 [sequences + 1]: each sequence's first segment
+    n: int
+    one_pass: bool
+
+
+def scan_segments(qlens, seq0: int, H: int, P: int) -> tuple[np.ndarray, np.ndarray, bool]:
+    """Host plan of ``ScanSegments`` for sequences seq0, seq0 + 1, ... with
+    ``qlens`` rows: one segment each when (sequences x heads x column tiles)
+    fills the chip, else whole-chunk cuts until it does (at least 4 chunks per
+    segment: a segment's start state costs a pass over its k and v)."""
+    wgs = max(1, len(qlens) * H * -(-P // SCAN_VT))
+    parts = -(-SCAN_FILL // wgs)
+    segs, first = [], [0]
+    for i, n in enumerate(qlens):
+        chunks = -(-int(n) // SCAN_CHUNK)
+        p = max(1, min(parts, chunks // 4))
+        step = -(-chunks // p) * SCAN_CHUNK
+        starts = range(0, int(n), step)
+        segs += [(seq0 + i, b, min(b + step, int(n)), int(b + step >= n)) for b in starts]
+        first.append(len(segs))
+    one_pass = len(segs) == len(qlens)
+    return (np.asarray(segs, np.int32).reshape(-1, 4), np.asarray(first, np.int32), one_pass)
+
+
+def _chunk_ok(N: int, P: int, *rows) -> bool:
+    return (N % 8 == 0 and P % 8 == 0 and N <= 256 and
+            all(t.dtype == torch.bfloat16 and t.data_ptr() % 16 == 0 and t.stride(0) % 8 == 0
+                for t in rows))
+
+
+def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, cu_q, ctx,
+                slots, heads_per_group: int = 1,
+                decay: tuple[torch.Tensor, torch.Tensor] | None = None,
+                dt: tuple[torch.Tensor, torch.Tensor, torch.Tensor] | None = None,
+                skip: torch.Tensor | None = None, silu: bool = False, num_decode: int = 0,
+                segments: ScanSegments | None = None) -> torch.Tensor:
+    """Per head S <- a S + s k v^T, o = S^T q + skip v over each sequence's rows,
+    from and to ``state`` (fp32 [slots, H, N, P]).
+
+    q, k: rows of (H / heads_per_group) x N channels shared by the heads of a
+    group; v: rows of H x P channels; ``silu`` applies SiLU to all three first.
+    ``decay`` = (a, ln a) fp32 [H]: constant, s = 1.  ``dt`` = (rows [T, H],
+    bias fp32 [H], neg_a fp32 [H]): s = softplus(dt + bias), a = exp(neg_a s).
+    Sequences before ``num_decode`` (one row each) take the recurrent kernel;
+    the others the chunked MFMA kernel when ``segments`` is given and the shape
+    allows it, the recurrent one otherwise.  Returns rows [T, H * P]."""
+    _, H, N, P = state.shape
+    T, S = q.shape[0], ctx.numel()
+    _chk((decay is None) != (dt is None), "linear_scan: decay or dt")
+    _chk(H % heads_per_group == 0, "linear_scan: heads per group")
+    out = torch.empty((T, H * P), dtype=q.dtype, device=q.device)
+    if not q.is_cuda:
+        ref.linear_scan(q, k, v, out, state, cu_q, ctx, slots, heads_per_group, decay, dt, skip,
+                        silu, range(S))
+        return out
+    bf = _rows_dtype(q, "q")
+    gn = H // heads_per_group * N
+    for t, c, name in ((q, gn, "q"), (k, gn, "k"), (v, H * P, "v")):
+        _chk(t.dtype == q.dtype and t.shape[0] == T and t.shape[1] >= c and t.stride(1) == 1,
+             f"linear_scan {name} rows")
+    _chk(state.dtype == torch.float32 and state.is_contiguous(), "scan state: fp32")
+    _meta(S, cu_q=cu_q, ctx=ctx, slots=slots)
+    _f32(skip, H, "skip")
+    if dt is not None:
+        _chk(dt[0].dtype == q.dtype and dt[0].shape[0] == T and dt[0].shape[1] >= H
+             and dt[0].stride(1) == 1, "dt rows")
+        _f32(dt[1], H, "dt bias"); _f32(dt[2], H, "neg_a")
+        scal = (_ptr(dt[0]), dt[0].stride(0), _ptr(dt[1]), _ptr(dt[2]), 0, 0)
+    else:
+        _f32(decay[0], H, "decay"); _f32(decay[1], H, "log decay")
+        scal = (0, 0, 0, 0, _ptr(decay[0]), _ptr(decay[1]))
+    args = (_ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), *scal, _ptr(skip),
+            _ptr(out), out.stride(0), _ptr(state), _ptr(cu_q), _ptr(ctx), _ptr(slots), H, N, P,
+            heads_per_group, int(silu), bf)
+    chunked = segments is not None and S > num_decode and _chunk_ok(N, P, q, k, v)
+    n_rec = num_decode if chunked else S
+    if n_rec:
+        native().linear_scan(*args, 0, n_rec, 0, 0, 0, 0, 0, 0, _stream())
+    if chunked:
+        g = segments
+        _chk(g.segs.dtype == torch.int32 and g.segs.numel() >= 4 * g.n
+             and g.first.dtype == torch.int32 and g.first.numel() == S - num_decode + 1,
+             "scan segments")
+        ws = wl = None
+        if not g.one_pass:
+            ws = torch.empty((g.n, H, N, P), dtype=torch.float32, device=q.device)
+            wl = torch.empty((g.n, H), dtype=torch.float32, device=q.device)
+        native().linear_scan(*args, num_decode, S - num_decode, _ptr(g.segs), g.n, _ptr(g.first),
+                             int(g.one_pass), _ptr(ws), _ptr(wl), _stream())
+    return out
+
+
+# ---------------------------------------------------------------- attention --
+def attention_any(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, ctx, positions,
+                  scale: float, Hq: int, gate: torch.Tensor | None = None) -> torch.Tensor:
+    """Causal paged attention of every row (decode and prompt rows alike), fp32
+    arithmetic, for what the MFMA kernels do not cover: fp32 caches, head sizes
+    256 / 512, more than 16 query heads per kv head.  Output times
+    sigmoid(gate) when given."""
+    _, Hkv, BS, D = k_cache.shape
+    T, S = q.shape[0], ctx.numel()
+    out = torch.empty((T, Hq * D), dtype=q.dtype, device=q.device)
+    if not q.is_cuda:
+        o = ref.paged_prefill(q.reshape(T, Hq, D), k_cache, v_cache, block_tables, cu_q, ctx, scale)
+        out.copy_(ref.gate_rows(o.reshape(T, Hq * D), gate))
+        return out
+    bf = _rows_dtype(q, "q")
+    _chk(q.shape[1] == Hq * D and q.stride(1) == 1 and k_cache.dtype == q.dtype
+         and v_cache.dtype == q.dtype and BS == 32 and D in (64, 128, 256, 512), "attention_any")
+    _meta(S, cu_q=cu_q, ctx=ctx)
+    _meta(T, positions=positions)
+    _chk(block_tables.dtype == torch.int32 and block_tables.shape[0] >= S
+         and block_tables.stride(1) == 1, "block tables")
+    _chk(gate is None or (gate.dtype == q.dtype and gate.shape[0] == T
+                          and gate.shape[1] >= Hq * D and gate.stride(1) == 1), "gate rows")
+    native().attention_any(_ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache),
+                           _ptr(block_tables), block_tables.stride(0), _ptr(cu_q), S,
+                           _ptr(positions), T, _ptr(out), out.stride(0), _ptr(gate),
+                           gate.stride(0) if gate is not None else 0, Hq, Hkv, D, BS,
+                           float(scale), bf, _stream())
+    return out

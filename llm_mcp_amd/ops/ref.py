@@ -384,3 +384,110 @@ def apply_penalties(logits, window, ngen, pen, v0: int = 0):
             x -= freq * cnt + (pres if cnt > 0 else 0.0)
             logits[b, t - v0] = x
     return logits
+
+
+# ------------------------------------- gated / recurrent token mixers ------
+def relu_mul(x):
+    I = x.shape[-1] // 2
+    return (torch.relu(x[..., :I].float()) * x[..., I:].float()).to(x.dtype)
+
+
+def gate_rows(o, gate):
+    """o * sigmoid(gate) (gate None: o)."""
+    if gate is None:
+        return o
+    return (o.float() * torch.sigmoid(gate[:, :o.shape[1]].float())).to(o.dtype)
+
+
+def _unit(x, eps):
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def sandwich_norm(residual, eps, y=None, w_post=None, w_pre=None, ids=None, table=None,
+                  rows=None, dtype=torch.bfloat16):
+    r = table[ids.long()].float() if ids is not None else residual
+    if rows is not None:
+        r, y = r[rows], None if y is None else y[rows]
+    if y is not None:
+        r = r + _unit(y.float(), eps) * w_post
+    if rows is None:
+        residual.copy_(r)
+    return None if w_pre is None else (_unit(r, eps) * w_pre).to(dtype)
+
+
+def gated_norm(x, gate, w, groups, eps, gate_first):
+    T, C = x.shape
+    v, g = x.float(), gate[:, :C].float()
+    if gate_first:
+        v = v * torch.nn.functional.silu(g)
+    v = _unit(v.reshape(T, groups, C // groups), eps).reshape(T, C) * w
+    if not gate_first:
+        v = v * torch.sigmoid(g)
+    return v.to(x.dtype)
+
+
+def _conv_rows(u, w, bias, in_bias, state, cu_q, ctx, slots):
+    """fp32 conv output of every row; advances ``state`` in place."""
+    taps, C = w.shape
+    y = torch.zeros((u.shape[0], C), dtype=torch.float32, device=u.device)
+    for s in range(len(ctx)):
+        a, b, slot = int(cu_q[s]), int(cu_q[s + 1]), int(slots[s])
+        if slot < 0:
+            continue
+        x = u[a:b, :C].float()
+        if in_bias is not None:
+            x = x + in_bias
+        old = torch.zeros((taps - 1, C)) if taps == 1 or int(ctx[s]) == b - a \
+            else state[slot].float()
+        full = torch.cat([old.to(x.device), x])
+        for j in range(taps):
+            y[a:b] += full[j:j + b - a] * w[j]
+        if taps > 1:
+            state[slot] = full[b - a:].to(state.dtype)
+    return y if bias is None else y + bias
+
+
+def short_conv(u, w, bias, state, cu_q, ctx, slots, out, silu):
+    y = _conv_rows(u, w, bias, None, state, cu_q, ctx, slots)
+    out.copy_(torch.nn.functional.silu(y) if silu else y)
+
+
+def conv_qkv_cache(u, w, in_bias, state, cu_q, ctx, state_slots, q_out, k_cache, v_cache,
+                   positions, slots, Hq, Hkv, D, dk, eps, temp):
+    T = u.shape[0]
+    y = _conv_rows(u, w, None, in_bias, state, cu_q, ctx, state_slots).view(T, -1, D)
+    inv = torch.rsqrt(y.pow(2).sum(-1, keepdim=True) / dk + eps)
+    coef, every = temp
+    t = 1.0 + coef * torch.log(torch.floor((positions.float() + 1.0) / every) + 1.0)
+    q_out.copy_((y[:, :Hq] * inv[:, :Hq] * t[:, None, None]).reshape(T, Hq * D))
+    write_cache((y * inv)[:, Hq:Hq + Hkv], y[:, Hq + Hkv:Hq + 2 * Hkv], slots, k_cache, v_cache)
+
+
+def linear_scan(q, k, v, out, state, cu_q, ctx, slots, hpg, decay, dt, skip, silu, seqs):
+    """See ops.linear_scan; one token after the other, fp32."""
+    _, H, N, P = state.shape
+    G = H // hpg
+    act = (lambda x: torch.nn.functional.silu(x.float()).to(q.dtype).float()) if silu \
+        else (lambda x: x.float())
+    for s in seqs:
+        a, b, slot = int(cu_q[s]), int(cu_q[s + 1]), int(slots[s])
+        if slot < 0:
+            continue
+        n = b - a
+        qs = act(q[a:b, :G * N]).view(n, G, N).repeat_interleave(hpg, 1)
+        ks = act(k[a:b, :G * N]).view(n, G, N).repeat_interleave(hpg, 1)
+        vs = act(v[a:b, :H * P]).view(n, H, P)
+        if dt is not None:
+            rows, bias, neg_a = dt
+            st = torch.nn.functional.softplus(rows[a:b, :H].float() + bias)
+            dec = torch.exp(neg_a * st)
+        else:
+            st, dec = torch.ones(n, H), decay[0].expand(n, H)
+        S = torch.zeros(H, N, P) if int(ctx[s]) == n else state[slot].clone()
+        for t in range(n):
+            S = dec[t][:, None, None] * S + ks[t][:, :, None] * (vs[t] * st[t][:, None])[:, None, :]
+            o = torch.einsum("hn,hnp->hp", qs[t], S)
+            if skip is not None:
+                o = o + skip[:, None] * vs[t]
+            out[a + t, :H * P] = o.reshape(-1).to(out.dtype)
+        state[slot] = S

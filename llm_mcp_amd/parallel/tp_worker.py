@@ -165,8 +165,8 @@ def build_tp_engine(ecfg, device, tp: TPContext, tag: str, weights_path: str = "
     cfg = model_cfg or mc.resolve(ecfg.model)
     weights = None
     if weights_path:
-        from ..models.weights import load_llama_weights
-        weights = load_llama_weights(weights_path, cfg, device, tp.rank, tp.size)
+        from ..models.weights import load_weights
+        weights = load_weights(weights_path, cfg, device, tp.rank, tp.size)
     dev = torch.device(device)
     comm = {}
     selftest = group_self_test(tp, dev) if tp.size > 1 else {}

@@ -78,9 +78,11 @@ def main(argv=None):
     if a.chat_model:
         cfg = mc.resolve(a.chat_model)
         weights = None
+        if not a.weights and mc.is_checkpoint_dir(a.chat_model):
+            a.weights = a.chat_model
         if a.weights:
-            from ..models.weights import load_llama_weights
-            weights = load_llama_weights(a.weights, cfg, dev)
+            from ..models.weights import load_weights
+            weights = load_weights(a.weights, cfg, dev)
         ecfg = EngineConfig(model=a.chat_model, max_num_seqs=a.max_num_seqs,
                             max_model_len=a.max_model_len, kv_fraction=a.kv_fraction)
         if a.max_batched_tokens:
