@@ -90,6 +90,10 @@ def parse(argv=None):
                     help="--load poisson: arrivals per second per GPU")
     ap.add_argument("--duration", type=float, default=30.0)
     ap.add_argument("--closed-warmup", type=float, default=10.0)
+    ap.add_argument("--compare", default="", metavar="MODEL",
+                    help="instead of the headline: engine-only prefill and decode throughput of "
+                         "MODEL (e.g. zegopel-8b) beside --model at a few sizes, one JSON line "
+                         "(bench/model_compare.py)")
     ap.add_argument("--cpu", action="store_true",
                     help="plumbing mode for tests: every rank runs its engine on the CPU (gloo; "
                          "use a tiny model such as tiny-llama); never a reported number")
@@ -161,8 +165,23 @@ def start_front_door(a, world: int, tag: str, socks: list[str]):
     return apis, lgs, url, ready_files
 
 
+def compare(a) -> None:
+    """--compare MODEL: MODEL beside --model, engine only, one GPU."""
+    import torch
+    from llm_mcp_amd.bench import model_compare
+    torch.cuda.set_device(0)
+    res = model_compare.compare([a.compare, a.model], torch.device("cuda", 0), say=log)
+    print(json.dumps({"metric": f"engine prefill / decode tokens/s, {a.compare} beside {a.model}",
+                      "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16",
+                      "data": "synthetic prompts, random-init weights", **res}), flush=True)
+
+
 def main() -> None:
     a = parse()
+    if a.compare:
+        if a.gpus != 1 or a.tp != 1:
+            sys.exit("bench.py: --compare is a one-GPU measurement")
+        return compare(a)
     if "WORLD_SIZE" not in os.environ and a.gpus > 1:
         self_launch(a)
     world = int(os.environ.get("WORLD_SIZE", "1"))
