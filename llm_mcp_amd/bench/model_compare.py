@@ -5,7 +5,7 @@ from __future__ import annotations
 
 import time
 
-PREFILL = ((1, 2048), (1, 8192), (16, 2048))          # (prompts, tokens each)
+PREFILL = ((1, 2048), (1, 7680), (16, 2048))          # (prompts, tokens each)
 DECODE = ((1, 1024), (16, 1024), (64, 1024), (256, 512))   # (streams, context)
 NEW_TOKENS = 48
 

@@ -207,55 +207,83 @@ int scan_recurrent(const ScanArgs& a, int is_bf16, int seq0, int nseq, hipStream
 
 // --------------------------------------------------------------- chunked ----
 constexpr int SC = 64;     // tokens per chunk
-constexpr int SCP = 72;    // padded row of the [.][64] LDS images (16-B aligned rows)
-constexpr int SVT = 64;    // v columns per workgroup (16 per wave)
+constexpr int SCP = 72;    // padded row of the score images (16-B aligned)
+constexpr float SCAN_LOG2E = 1.4426950408889634f;
 
 struct SegArgs {
   const int* segs;         // [nseg][4]: sequence, first row, last row (in the sequence), last-of-sequence
   float* ws;               // [nseg][H][N][P] segment states (modes 1, 2)
-  float* ws_log;           // [nseg][H] log of the segment's total decay (mode 1)
+  float* ws_log;           // [nseg][H] log2 of the segment's total decay (mode 1)
 };
 
-__device__ __forceinline__ void split_bf16(float x, short& hi, short& lo) {
-  const uint16_t h = f2bf(x);
-  hi = (short)h;
-  lo = (short)f2bf(x - bf2f(h));
+typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x2_t __attribute__((ext_vector_type(2)));
+
+// (a, b) as packed bf16 pairs: hi + lo = the values to within 2^-17
+__device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
+  hi = pack_bf16x2(a, b);
+  lo = pack_bf16x2(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
 }
 
-__device__ __forceinline__ bf16x8_t frag_2x8(const bf16_t* p0, const bf16_t* p1) {
-  return load_frag_2x8B(p0, p1);
+__device__ __forceinline__ float silu_fast(float x) {
+  return x * __builtin_amdgcn_rcpf(1.f + fast_exp2(-x * SCAN_LOG2E));
 }
 
-// NK: N / 32 rounded up.  MODE 0: one segment per sequence, from and to the
-// state slot; 1: segment end states only (start zero); 2: outputs from the
-// chained segment states, the last segment writes the slot.
+__device__ __forceinline__ void silu_words(u32x4_t& w) {
+#pragma unroll
+  for (int m = 0; m < 4; ++m)
+    w[m] = pack_bf16x2(silu_fast(__uint_as_float(w[m] << 16)),
+                       silu_fast(__uint_as_float(w[m] & 0xffff0000u)));
+}
+
+// Transposed LDS image [rows][64 tokens]: 16-B pieces (8 tokens) of a row are
+// XOR-permuted by the row so that both the 8-B transposing stores (16 row
+// groups x 4 token quads per wave) and the 16-B fragment reads (16 rows x 4
+// pieces) spread evenly over the banks.
+__device__ __forceinline__ int tr_swz(int row) {
+  return ((row & 3) | ((row >> 1) & 4)) ^ ((row >> 4) & 7);
+}
+
+// Barrier over LDS only: __syncthreads would also wait for every global load
+// in flight, i.e. for the next chunk's rows.
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
+// NK: N / 32 rounded up; NV: 16-column tiles per wave (a workgroup covers 64
+// NV columns of v).  MODE 0: one segment per sequence, from and to the state
+// slot; 1: segment end states only (start zero); 2: outputs from the chained
+// segment states, the last segment writes the slot.
 //
-// LDS images (bf16): q [64][NK*32+8], k the same (later overlaid by the score
-// images hi/lo [64][SCP]), k^T [NK*32][SCP], v^T [SVT][SCP]; fp32: cum[64],
-// s[64], exp(cum)[64].
+// LDS images (bf16): q [64][32 NK + 8], k the same (overlaid by the score
+// images hi / lo [64][SCP] once the scores exist), k^T [32 NK][64] and v^T
+// [64 NV][64] swizzled; fp32 per token: log2 decay prefix, s, 2^prefix, and
+// the weight of the token in the end state.
 //
-// Wave w computes the scores of query rows 16w..16w+15 and owns v columns
-// 16w..16w+15 of outputs and state.  The state tile t of a wave sits in MFMA
-// C layout (row = state channel 16t + 4g + r, col = v column), which is the
-// B-operand layout of a product whose k index is permuted within 32: k slot
-// (g, j) = channel 4g + j (j < 4) or 16 + 4g + j - 4.  q is read with the same
-// permutation, so the state needs no transposition.
-template <int NK, int MODE>
+// Wave w computes the scores of query rows 16w..16w+15 and owns 16 NV columns
+// of outputs and state.  A state tile pair (2 ks, 2 ks + 1) keeps channels
+// 32 ks + 8 g + j in lane group g (tile j >> 2, register j & 3) of its column:
+// that is the operand layout of the products with q, so the state is split
+// into bf16 pairs in place, with no exchange.  Outputs are computed transposed
+// (MFMA row = v column): a lane ends up with 4 consecutive columns of a row.
+template <int NK, int NV, int MODE>
 __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanArgs a, SegArgs sg) {
   extern __shared__ __attribute__((aligned(16))) char chunk_sm[];
-  constexpr int DK = NK * 32, LQ = DK + 8;
-  constexpr int KBYTES = SC * LQ * 2 > 2 * SC * SCP * 2 ? SC * LQ * 2 : 2 * SC * SCP * 2;
+  constexpr int DK = NK * 32, LQ = DK + 8, VT = 64 * NV, NP = 4 * NK;
+  constexpr int KEL = MODE == 1 ? 0 : (SC * LQ > 2 * SC * SCP ? SC * LQ : 2 * SC * SCP);
   bf16_t* const sQ = reinterpret_cast<bf16_t*>(chunk_sm);
   bf16_t* const sK = sQ + (MODE == 1 ? 0 : SC * LQ);
   bf16_t* const sP = sK;                                   // hi [64][SCP], lo [64][SCP]
-  bf16_t* const sKT = reinterpret_cast<bf16_t*>(reinterpret_cast<char*>(sK) +
-                                                (MODE == 1 ? 0 : KBYTES));
-  bf16_t* const sVT = sKT + DK * SCP;
-  float* const cum = reinterpret_cast<float*>(sVT + SVT * SCP);
+  bf16_t* const sKT = sK + KEL;
+  bf16_t* const sVT = sKT + DK * SC;
+  float* const cum = reinterpret_cast<float*>(sVT + VT * SC);
   float* const sdt = cum + SC;
   float* const ecum = sdt + SC;
+  float* const wend = ecum + SC;
 
-  const int seg = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * SVT;
+  const int seg = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VT;
   const int seq = sg.segs[4 * seg], b = sg.segs[4 * seg + 1], e = sg.segs[4 * seg + 2];
   const bool last = sg.segs[4 * seg + 3] != 0;
   const int N = a.N, P = a.P;
@@ -264,97 +292,127 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
   const bool fresh = a.ctx[seq] == a.cu_q[seq + 1] - qrow;
   const long row0 = qrow + b;
   const int n = e - b;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
-  const int vcol = v0 + wave * 16 + c;
-  const bool vok = vcol < P;
+  const int tid = threadIdx.x, lane = tid & 63, c = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int vw = v0 + wave * 16 * NV;                      // this wave's first column
   const int grp = h / a.hpg;
   const bf16_t* q = (const bf16_t*)a.q + row0 * a.q_ld + (long)grp * N;
   const bf16_t* k = (const bf16_t*)a.k + row0 * a.k_ld + (long)grp * N;
   const bf16_t* v = (const bf16_t*)a.v + row0 * a.v_ld + (long)h * P;
+  bf16_t* out = (bf16_t*)a.out + row0 * a.out_ld + (long)h * P;
   const bf16_t* dt = a.dt ? (const bf16_t*)a.dt + row0 * a.dt_ld + h : nullptr;
-  const float logd = a.dt ? 0.f : a.log_decay[h];
-  const float bias = a.dt ? a.dt_bias[h] : 0.f, na = a.dt ? a.neg_a[h] : 0.f;
+  const float logd = a.dt ? 0.f : a.log_decay[h] * SCAN_LOG2E;
+  const float bias = a.dt ? a.dt_bias[h] : 0.f, na = a.dt ? a.neg_a[h] * SCAN_LOG2E : 0.f;
   const float skip = a.skip ? a.skip[h] : 0.f;
 
-  // ---- state ----
-  f32x4_t S[2 * NK];
+  // ---- state: tile t, register r = channel 32 (t / 2) + 8 g + 4 (t % 2) + r ----
+  f32x4_t S[NV][2 * NK];
+  auto state_io = [&](float* p, bool store, bool zero) {
+    // opaque per call: the bounds masks of the load must not stay live (in
+    // scalar registers, spilled) until the store
+    int N = a.N, P = a.P;
+    asm volatile("" : "+s"(N), "+s"(P));
+#pragma unroll
+    for (int ct = 0; ct < NV; ++ct)
+#pragma unroll
+      for (int t = 0; t < 2 * NK; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int kk = 32 * (t >> 1) + 8 * g + 4 * (t & 1) + r, vc = vw + 16 * ct + c;
+          const bool ok = kk < N && vc < P;
+          if (store) {
+            if (ok) p[(long)kk * P + vc] = S[ct][t][r];
+          } else {
+            S[ct][t][r] = ok && !zero ? p[(long)kk * P + vc] : 0.f;
+          }
+        }
+  };
   {
-    const float* src = nullptr;
-    if constexpr (MODE == 0) {
-      if (!fresh) src = a.state + ((long)slot * a.H + h) * N * P;
-    } else if constexpr (MODE == 2) {
-      src = sg.ws + ((long)seg * a.H + h) * N * P;
-    }
-#pragma unroll
-    for (int t = 0; t < 2 * NK; ++t)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int kk = 16 * t + 4 * g + r;
-        S[t][r] = src && kk < N && vok ? src[(long)kk * P + vcol] : 0.f;
-      }
+    float* src = MODE == 2 ? sg.ws + ((long)seg * a.H + h) * N * P
+                           : a.state + ((long)slot * a.H + h) * N * P;
+    state_io(src, false, MODE == 1 || (MODE == 0 && fresh));
   }
 
-  // ---- staging: registers one chunk ahead ----
-  // q / k pieces: lane group of 4 covers 64 B of a row, 16 rows per wave
-  // instruction; v pieces the same over its 64 columns
-  u16x8 rq[NK], rk[NK], rv[2];
+  // ---- staging, one chunk ahead in registers.  q: 16-B pieces of rows.  k and
+  // v: items of 4 consecutive rows x 8 channels, so the transposed image is
+  // written 4 tokens (8 B) at a time ----
+  constexpr int KITEMS = 16 * NP, ITEMS = KITEMS + 2 * VT, NI = (ITEMS + 255) / 256;
+  u32x4_t rq[MODE == 1 ? 1 : NK], ri[NI][4];
   float rdt = 0.f;
-  const u16x8 zero8 = {{0, 0, 0, 0, 0, 0, 0, 0}};
-  const int prow = (tid >> 2), pch = tid & 3;            // 64 rows x 4 chunks per pass
-  auto fetch = [&](int t0) {
-    const bool ok = t0 + prow < n;
-    const long r = t0 + prow;
+  const u32x4_t zero4 = {0, 0, 0, 0};
+  // per-thread byte offsets from wave-uniform row bases (a chunk is far below 4 GB)
+  static_assert(256 % NP == 0, "a q pass is whole rows");
+  const int qr = tid / NP, qc = 8 * (tid % NP);
+  const uint32_t qoff = (uint32_t)((qr * a.q_ld + qc) * 2);
+  uint32_t ioff[NI];
+  int irow[NI];              // first of the item's 4 rows; beyond every chunk: no item
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int ch = 8 * (pch + 4 * i);
-      const bool in = ok && ch < N;
-      if constexpr (MODE != 1)
-        rq[i] = in ? *reinterpret_cast<const u16x8*>(q + r * a.q_ld + ch) : zero8;
-      rk[i] = in ? *reinterpret_cast<const u16x8*>(k + r * a.k_ld + ch) : zero8;
+  for (int i = 0; i < NI; ++i) {
+    const int it = tid + 256 * i;
+    const bool isk = it < KITEMS;                          // wave-uniform
+    const int x = isk ? it : it - KITEMS, np = isk ? NP : VT / 8;
+    const int ch = 8 * (x % np) + (isk ? 0 : v0);
+    irow[i] = it < ITEMS && ch < (isk ? N : P) ? 4 * (x / np) : 1 << 20;
+    ioff[i] = (uint32_t)((4 * (x / np) * (isk ? a.k_ld : a.v_ld) + ch) * 2);
+  }
+  auto at = [](const void* base, uint32_t off) {
+    return reinterpret_cast<const u32x4_t*>(reinterpret_cast<const char*>(base) + off);
+  };
+  auto fetch = [&](int t0) {
+    const int left = n - t0;
+    if constexpr (MODE != 1) {
+      const bf16_t* base = q + (long)t0 * a.q_ld;
+#pragma unroll
+      for (int i = 0; i < NK; ++i)
+        rq[i] = qr + (256 / NP) * i < left && qc < N
+                    ? *at(base + (long)(256 / NP) * i * a.q_ld, qoff) : zero4;
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int ch = v0 + 8 * (pch + 4 * i);
-      rv[i] = ok && ch < P ? *reinterpret_cast<const u16x8*>(v + r * a.v_ld + ch) : zero8;
+    for (int i = 0; i < NI; ++i) {
+      const bool isk = wave * 64 + 256 * i < KITEMS;
+      const long ld = isk ? a.k_ld : a.v_ld;
+      const bf16_t* base = (isk ? k : v) + t0 * ld;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        ri[i][r] = irow[i] + r < left ? *at(base + r * ld, ioff[i]) : zero4;
     }
     if (dt && tid < SC) rdt = t0 + tid < n ? bf2f(dt[(long)(t0 + tid) * a.dt_ld]) : 0.f;
   };
-  auto act8 = [&](u16x8& x) {
-    if (a.act) {
+  auto stage = [&](int m) {
+    if constexpr (MODE != 1) {
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const float f = bf2f(x.v[j]);
-        x.v[j] = f2bf(f / (1.f + __expf(-f)));
+      for (int i = 0; i < NK; ++i) {
+        const int it = tid + 256 * i;
+        if (a.act) silu_words(rq[i]);
+        *reinterpret_cast<u32x4_t*>(sQ + (it / NP) * LQ + qc) = rq[i];
       }
     }
-  };
-
-  float log_total = 0.f;
-  if (n > 0) fetch(0);
-  for (int t0 = 0; t0 < n; t0 += SC) {
-    const int m = min(SC, n - t0);
-    // ---- stage this chunk ----
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int ch = 8 * (pch + 4 * i);
-      act8(rk[i]);
-      if constexpr (MODE != 1) {
-        act8(rq[i]);
-        *reinterpret_cast<u16x8*>(sQ + prow * LQ + ch) = rq[i];
-        *reinterpret_cast<u16x8*>(sK + prow * LQ + ch) = rk[i];
+    for (int i = 0; i < NI; ++i) {
+      const int it = tid + 256 * i;
+      if (wave * 64 + 256 * i >= ITEMS) continue;
+      const bool isk = wave * 64 + 256 * i < KITEMS;
+      const int x = isk ? it : it - KITEMS, np = isk ? NP : VT / 8;
+      const int pc = x % np, qd = x / np;
+      bf16_t* const img = isk ? sKT : sVT;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        if (a.act) silu_words(ri[i][r]);
+        if constexpr (MODE != 1)
+          if (isk) *reinterpret_cast<u32x4_t*>(sK + (4 * qd + r) * LQ + 8 * pc) = ri[i][r];
       }
 #pragma unroll
-      for (int j = 0; j < 8; ++j) sKT[(ch + j) * SCP + prow] = rk[i].v[j];
-    }
-#pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int ch = 8 * (pch + 4 * i);
-      act8(rv[i]);
-#pragma unroll
-      for (int j = 0; j < 8; ++j) sVT[(ch + j) * SCP + prow] = rv[i].v[j];
+      for (int e = 0; e < 8; ++e) {
+        // tr_swz(8 pc + e) = swz(pc) ^ (e & 3): 4 addresses + immediates
+        const uint32_t sel = e & 1 ? 0x07060302u : 0x05040100u;
+        const u32x2_t w = {__builtin_amdgcn_perm(ri[i][1][e >> 1], ri[i][0][e >> 1], sel),
+                           __builtin_amdgcn_perm(ri[i][3][e >> 1], ri[i][2][e >> 1], sel)};
+        *reinterpret_cast<u32x2_t*>(img + 8 * pc * SC + 4 * (qd & 1) +
+                                    8 * (((qd >> 1) ^ tr_swz(8 * pc)) ^ (e & 3)) + e * SC) = w;
+      }
     }
     if (wave == 0) {
-      // log decays and their prefix sum; rows past the end neither decay nor add
+      // log2 decays and their prefix sum; rows past the end neither decay nor add
       float s = 1.f, la = logd;
       if (dt) { s = softplus_f(rdt + bias); la = na * s; }
       if (lane >= m) { s = 0.f; la = 0.f; }
@@ -366,20 +424,47 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
       }
       cum[lane] = x;
       sdt[lane] = s;
-      ecum[lane] = __expf(x);
+      ecum[lane] = fast_exp2(x);
+      wend[lane] = fast_exp2(__shfl(x, 63, 64) - x) * s;
     }
-    __syncthreads();
+  };
+
+  // k^T fragment addresses: row 32 tt + 8 (c / 4) + 4 b + c % 4, piece 4 ks + g:
+  // the swizzle leaves 4 lane offsets (index tt ^ 2 ks), the rest is immediate
+  const bf16_t* ktp[4];
+#pragma unroll
+  for (int z = 0; z < 4; ++z) {
+    const int row = 8 * (c >> 2) + (c & 3);
+    ktp[z] = sKT + row * SC + 8 * (g ^ tr_swz(row) ^ (2 * z));
+  }
+
+  float log_total = 0.f;
+  if (n > 0) fetch(0);
+  for (int t0 = 0; t0 < n; t0 += SC) {
+    const int m = min(SC, n - t0);
+    stage(m);
+    lds_barrier();
     if (t0 + SC < n) fetch(t0 + SC);
 
-    const float ctot = cum[SC - 1];
+    bf16x8_t vf[NV][2];        // v^T fragments of this wave's columns
+    auto load_v = [&]() {
+#pragma unroll
+      for (int ct = 0; ct < NV; ++ct) {
+        const int row = wave * 16 * NV + 16 * ct + c;
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks)
+          vf[ct][ks] = load_frag16B(sVT + row * SC + 8 * ((4 * ks + g) ^ tr_swz(row)));
+      }
+    };
+    if constexpr (MODE == 1) load_v();
     if constexpr (MODE != 1) {
-      // ---- scores of query rows 16 wave + c (transposed product: the query is
-      // the MFMA column) ----
+      // ---- scores of query rows 16 wave + c (the query is the MFMA column) ----
       f32x4_t sc[4];
 #pragma unroll
       for (int jt = 0; jt < 4; ++jt) sc[jt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < NK; ++ks) {
+        __builtin_amdgcn_sched_barrier(0);
         const bf16x8_t qf = load_frag16B(sQ + (wave * 16 + c) * LQ + 32 * ks + 8 * g);
 #pragma unroll
         for (int jt = 0; jt < 4; ++jt)
@@ -388,119 +473,150 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
       }
       const int qi = wave * 16 + c;
       const float ci = cum[qi];
-      bf16x4_t ph[4], pl[4];
-#pragma unroll
-      for (int jt = 0; jt < 4; ++jt)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int j = jt * 16 + 4 * g + r;
-          const float w = j <= qi ? sc[jt][r] * __expf(ci - cum[j]) * sdt[j] : 0.f;
-          short hi, lo;
-          split_bf16(w, hi, lo);
-          ph[jt][r] = hi;
-          pl[jt][r] = lo;
-        }
-      __syncthreads();                       // every wave is done with k's rows
+      u32x2_t ph[4], pl[4];
 #pragma unroll
       for (int jt = 0; jt < 4; ++jt) {
-        *reinterpret_cast<bf16x4_t*>(sP + qi * SCP + jt * 16 + 4 * g) = ph[jt];
-        *reinterpret_cast<bf16x4_t*>(sP + (SC + qi) * SCP + jt * 16 + 4 * g) = pl[jt];
-      }
-      __syncthreads();
-
-      // ---- outputs: 64 queries x this wave's 16 columns ----
-      f32x4_t o[4];
+        const f32x4_t cj = *reinterpret_cast<const f32x4_t*>(cum + jt * 16 + 4 * g);
+        const f32x4_t sj = *reinterpret_cast<const f32x4_t*>(sdt + jt * 16 + 4 * g);
+        float w[4];
+        // visible keys of this tile: all, up to the query's own, or none (opaque:
+        // the comparison masks are loop-invariant and would fill the scalar file)
+        int lim = jt < wave ? 64 : jt == wave ? c : -1;
+        asm volatile("" : "+v"(lim));
 #pragma unroll
-      for (int it = 0; it < 4; ++it) o[it] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        for (int r = 0; r < 4; ++r) {
+          w[r] = 4 * g + r <= lim ? sc[jt][r] * fast_exp2(ci - cj[r]) * sj[r] : 0.f;
+          // the skip term is a score of one's own v
+          if (jt == wave) w[r] += 4 * g + r == c ? skip : 0.f;
+        }
+        uint32_t h0, l0, h1, l1;
+        split2(w[0], w[1], h0, l0);
+        split2(w[2], w[3], h1, l1);
+        ph[jt] = u32x2_t{h0, h1};
+        pl[jt] = u32x2_t{l0, l1};
+      }
+      lds_barrier();                       // every wave is done with k's rows
+#pragma unroll
+      for (int jt = 0; jt < 4; ++jt) {
+        *reinterpret_cast<u32x2_t*>(sP + qi * SCP + jt * 16 + 4 * g) = ph[jt];
+        *reinterpret_cast<u32x2_t*>(sP + (SC + qi) * SCP + jt * 16 + 4 * g) = pl[jt];
+      }
+
+      // ---- outputs, transposed: state part 2^cum (S^T q) ----
+      f32x4_t o[NV][4];
+#pragma unroll
+      for (int ct = 0; ct < NV; ++ct)
+#pragma unroll
+        for (int it = 0; it < 4; ++it) o[ct][it] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < NK; ++ks) {
-        bf16x8_t sh, sl;
+        __builtin_amdgcn_sched_barrier(0);   // one k step's operands at a time
+        bf16x8_t sh[NV], sl[NV];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          short hi, lo;
-          split_bf16(S[2 * ks + (j >> 2)][j & 3], hi, lo);
-          sh[j] = hi;
-          sl[j] = lo;
+        for (int ct = 0; ct < NV; ++ct) {
+          u32x4_t hi, lo;
+#pragma unroll
+          for (int m2 = 0; m2 < 4; ++m2) {
+            uint32_t x, y;
+            const f32x4_t& t = S[ct][2 * ks + (m2 >> 1)];
+            split2(t[2 * (m2 & 1)], t[2 * (m2 & 1) + 1], x, y);
+            hi[m2] = x;
+            lo[m2] = y;
+          }
+          sh[ct] = __builtin_bit_cast(bf16x8_t, hi);
+          sl[ct] = __builtin_bit_cast(bf16x8_t, lo);
         }
 #pragma unroll
         for (int it = 0; it < 4; ++it) {
-          const bf16_t* qr = sQ + (it * 16 + c) * LQ + 32 * ks + 4 * g;
-          const bf16x8_t qf = frag_2x8(qr, qr + 16);
-          o[it] = mfma16(qf, sh, o[it]);
-          o[it] = mfma16(qf, sl, o[it]);
+          const bf16x8_t qf = load_frag16B(sQ + (it * 16 + c) * LQ + 32 * ks + 8 * g);
+#pragma unroll
+          for (int ct = 0; ct < NV; ++ct) {
+            o[ct][it] = mfma16(sh[ct], qf, o[ct][it]);
+            o[ct][it] = mfma16(sl[ct], qf, o[ct][it]);
+          }
         }
       }
-      const bf16x8_t vf0 = load_frag16B(sVT + (wave * 16 + c) * SCP + 8 * g);
-      const bf16x8_t vf1 = load_frag16B(sVT + (wave * 16 + c) * SCP + 32 + 8 * g);
+      load_v();
+      lds_barrier();                       // the scores of every query are in LDS
 #pragma unroll
       for (int it = 0; it < 4; ++it) {
+        __builtin_amdgcn_sched_barrier(0);
+        const int i = it * 16 + c;
+        const float ec = ecum[i];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) o[it][r] *= ecum[it * 16 + 4 * g + r];
-        const bf16_t* pr = sP + (it * 16 + c) * SCP + 8 * g;
-        o[it] = mfma16(load_frag16B(pr), vf0, o[it]);
-        o[it] = mfma16(load_frag16B(pr + SC * SCP), vf0, o[it]);
-        if (it >= 2) {
-          o[it] = mfma16(load_frag16B(pr + 32), vf1, o[it]);
-          o[it] = mfma16(load_frag16B(pr + SC * SCP + 32), vf1, o[it]);
+        for (int ct = 0; ct < NV; ++ct) o[ct][it] *= ec;
+#pragma unroll
+        for (int ks = 0; ks <= it / 2; ++ks) {
+          const bf16_t* pr = sP + i * SCP + 32 * ks + 8 * g;
+          const bf16x8_t pfh = load_frag16B(pr), pfl = load_frag16B(pr + SC * SCP);
+#pragma unroll
+          for (int ct = 0; ct < NV; ++ct) {
+            o[ct][it] = mfma16(vf[ct][ks], pfh, o[ct][it]);
+            o[ct][it] = mfma16(vf[ct][ks], pfl, o[ct][it]);
+          }
         }
-        const bf16x4_t xv =
-            *reinterpret_cast<const bf16x4_t*>(sVT + (wave * 16 + c) * SCP + it * 16 + 4 * g);
+        if (i < m) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int i = it * 16 + 4 * g + r;
-          const float y = o[it][r] + skip * bf2f((uint16_t)xv[r]);
-          if (i < m && vok)
-            ((bf16_t*)a.out)[(row0 + t0 + i) * a.out_ld + (long)h * P + vcol] = f2bf(y);
+          for (int ct = 0; ct < NV; ++ct) {
+            const int vc = vw + 16 * ct + 4 * g;           // P % 8 == 0: whole quads
+            if (vc < P) {
+              const f32x4_t& y = o[ct][it];
+              const u32x2_t yw = {pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+              *reinterpret_cast<u32x2_t*>(out + (long)(t0 + i) * a.out_ld + vc) = yw;
+            }
+          }
         }
       }
     }
-    // ---- state: S <- exp(ctot) S + k^T (w v),  w_j = exp(ctot - cum_j) s_j ----
-    const float et = __expf(ctot);
+    // ---- state: S <- 2^ctot S + k^T (w v) ----
+    const float ctot = cum[SC - 1], et = ecum[SC - 1];
     log_total += ctot;
-    bf16x8_t wh[2], wl[2];
+    bf16x8_t wh[NV][2], wl[NV][2];
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
-      const bf16x8_t vf = load_frag16B(sVT + (wave * 16 + c) * SCP + 32 * ks + 8 * g);
+      const f32x4_t w0 = *reinterpret_cast<const f32x4_t*>(wend + 32 * ks + 8 * g);
+      const f32x4_t w1 = *reinterpret_cast<const f32x4_t*>(wend + 32 * ks + 8 * g + 4);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int jj = 32 * ks + 8 * g + j;
-        short hi, lo;
-        split_bf16(bf2f((uint16_t)vf[j]) * __expf(ctot - cum[jj]) * sdt[jj], hi, lo);
-        wh[ks][j] = hi;
-        wl[ks][j] = lo;
+      for (int ct = 0; ct < NV; ++ct) {
+        const u32x4_t x = __builtin_bit_cast(u32x4_t, vf[ct][ks]);
+        u32x4_t hi, lo;
+#pragma unroll
+        for (int m2 = 0; m2 < 4; ++m2) {
+          const f32x4_t& w = m2 < 2 ? w0 : w1;
+          uint32_t xh, xl;
+          split2(__uint_as_float(x[m2] << 16) * w[2 * (m2 & 1)],
+                 __uint_as_float(x[m2] & 0xffff0000u) * w[2 * (m2 & 1) + 1], xh, xl);
+          hi[m2] = xh;
+          lo[m2] = xl;
+        }
+        wh[ct][ks] = __builtin_bit_cast(bf16x8_t, hi);
+        wl[ct][ks] = __builtin_bit_cast(bf16x8_t, lo);
       }
     }
 #pragma unroll
     for (int t = 0; t < 2 * NK; ++t) {
+      if (t % 2 == 0) __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) S[t][r] *= et;
+      for (int ct = 0; ct < NV; ++ct) S[ct][t] *= et;
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
-        const bf16x8_t kf = load_frag16B(sKT + (t * 16 + c) * SCP + 32 * ks + 8 * g);
-        S[t] = mfma16(kf, wh[ks], S[t]);
-        S[t] = mfma16(kf, wl[ks], S[t]);
+        const bf16x8_t kf =
+            load_frag16B(ktp[((t >> 1) ^ (2 * ks)) & 3] + (32 * (t >> 1) + 4 * (t & 1)) * SC);
+#pragma unroll
+        for (int ct = 0; ct < NV; ++ct) {
+          S[ct][t] = mfma16(kf, wh[ct][ks], S[ct][t]);
+          S[ct][t] = mfma16(kf, wl[ct][ks], S[ct][t]);
+        }
       }
     }
-    __syncthreads();                         // the next chunk overwrites the images
+    lds_barrier();                         // the next chunk overwrites the images
   }
 
-  float* dst = nullptr;
-  if constexpr (MODE == 0) dst = a.state + ((long)slot * a.H + h) * N * P;
   if constexpr (MODE == 1) {
-    dst = sg.ws + ((long)seg * a.H + h) * N * P;
+    state_io(sg.ws + ((long)seg * a.H + h) * N * P, true, false);
     if (tid == 0 && v0 == 0) sg.ws_log[(long)seg * a.H + h] = log_total;
-  }
-  if constexpr (MODE == 2) {
-    if (last) dst = a.state + ((long)slot * a.H + h) * N * P;
-  }
-  if (dst) {
-#pragma unroll
-    for (int t = 0; t < 2 * NK; ++t)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int kk = 16 * t + 4 * g + r;
-        if (kk < N && vok) dst[(long)kk * P + vcol] = S[t][r];
-      }
+  } else {
+    if (MODE == 0 || last) state_io(a.state + ((long)slot * a.H + h) * N * P, true, false);
   }
 }
 
@@ -523,7 +639,7 @@ __global__ void __launch_bounds__(256) scan_combine_kernel(ScanArgs a, SegArgs s
       float* p = sg.ws + ((long)f * a.H + h) * NP + i;
       const float own = f + 1 < f1 ? *p : 0.f;   // the last segment's own state is not needed
       *p = x;
-      x = __expf(sg.ws_log[(long)f * a.H + h]) * x + own;
+      x = fast_exp2(sg.ws_log[(long)f * a.H + h]) * x + own;
     }
   }
 }
@@ -536,22 +652,28 @@ bool scan_chunk_ok(const ScanArgs& a) {
          al(a.v, a.v_ld);
 }
 
-template <int NK, int MODE>
-static int launch_chunk(const ScanArgs& a, const SegArgs& sg, int nseg, hipStream_t stream) {
+template <int NK, int NV, int MODE>
+static int launch_chunk_nv(const ScanArgs& a, const SegArgs& sg, int nseg, hipStream_t stream) {
   constexpr int LQ = NK * 32 + 8;
-  constexpr int KB = SC * LQ * 2 > 2 * SC * SCP * 2 ? SC * LQ * 2 : 2 * SC * SCP * 2;
-  constexpr int smem = (MODE == 1 ? 0 : SC * LQ * 2 + KB) + NK * 32 * SCP * 2 + SVT * SCP * 2 +
-                       3 * SC * 4;
+  constexpr int KEL = SC * LQ > 2 * SC * SCP ? SC * LQ : 2 * SC * SCP;
+  constexpr int smem = ((MODE == 1 ? 0 : SC * LQ + KEL) + NK * 32 * SC + 64 * NV * SC) * 2 + 4 * SC * 4;
   static_assert(smem <= 160 * 1024, "chunk images fit the LDS");
   static bool attr = false;
   if (smem > 65536 && !attr) {
-    (void)hipFuncSetAttribute((const void*)scan_chunk_kernel<NK, MODE>,
+    (void)hipFuncSetAttribute((const void*)scan_chunk_kernel<NK, NV, MODE>,
                               hipFuncAttributeMaxDynamicSharedMemorySize, smem);
     attr = true;
   }
-  scan_chunk_kernel<NK, MODE><<<dim3(nseg, a.H, (a.P + SVT - 1) / SVT), dim3(256), smem, stream>>>(
-      a, sg);
+  scan_chunk_kernel<NK, NV, MODE>
+      <<<dim3(nseg, a.H, (a.P + 64 * NV - 1) / (64 * NV)), dim3(256), smem, stream>>>(a, sg);
   return (int)hipGetLastError();
+}
+
+template <int NK, int MODE>
+static int launch_chunk(const ScanArgs& a, const SegArgs& sg, int nseg, hipStream_t stream) {
+  if constexpr (NK <= 4)
+    if (a.P > 64) return launch_chunk_nv<NK, 2, MODE>(a, sg, nseg, stream);
+  return launch_chunk_nv<NK, 1, MODE>(a, sg, nseg, stream);
 }
 
 // segs / first: see SegArgs and scan_combine_kernel.  one_pass: one segment
@@ -566,7 +688,6 @@ int scan_chunked(const ScanArgs& a, const int* segs, int nseg, const int* first,
 #define LMX_CHUNK(MODE)                                                   \
   (nk <= 1 ? launch_chunk<1, MODE>(a, sg, nseg, stream)                   \
    : nk <= 2 ? launch_chunk<2, MODE>(a, sg, nseg, stream)                 \
-   : nk <= 3 ? launch_chunk<3, MODE>(a, sg, nseg, stream)                 \
    : nk <= 4 ? launch_chunk<4, MODE>(a, sg, nseg, stream)                 \
              : launch_chunk<8, MODE>(a, sg, nseg, stream))
   if (one_pass) return LMX_CHUNK(0);

@@ -22,7 +22,7 @@ from . import Partials, _chk, _ptr, _stream, native, ref
 
 CONV_TILE = 64        # tokens per convolution workgroup
 SCAN_CHUNK = 64       # SC in csrc/kernels/linscan.hip
-SCAN_VT = 64          # v columns per workgroup (SVT)
+SCAN_VT = 128         # v columns per workgroup (64 up to P = 64)
 SCAN_FILL = 512       # workgroups wanted before a sequence is cut into segments
 
 
