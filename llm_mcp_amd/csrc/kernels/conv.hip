@@ -40,7 +40,7 @@ struct ConvArgs {
   int C, taps, tile;
 };
 
-// Walk of one tile: emit(row, y) per token.  TAPS > 0: window in registers;
+// Walk of one tile: emit(row, y, last) per token.  TAPS > 0: window in registers;
 // TAPS == 0: any tap count, inputs re-read (cache hits).
 template <typename T, int V, int TAPS, typename Emit>
 __device__ __forceinline__ void conv_walk(const ConvArgs& a, int seq, int start, int c0, Emit emit) {
@@ -70,13 +70,16 @@ __device__ __forceinline__ void conv_walk(const ConvArgs& a, int seq, int start,
 #pragma unroll
   for (int e = 0; e < V; ++e) bias[e] = a.bias ? a.bias[c0 + e] : 0.f;
   if constexpr (TAPS > 0) {
-    float w[TAPS][V], win[TAPS][V];           // win[j]: input t - taps + 1 + j
+    float w[TAPS][V], win[TAPS][V], nxt[V];   // win[j]: input t - taps + 1 + j
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) ldv<V>(w[j], a.w + (long)j * a.C + c0);
 #pragma unroll
     for (int j = 0; j < TAPS - 1; ++j) input(start - (TAPS - 1) + j, win[j]);
+    input(start, nxt);
     for (int t = start; t < end; ++t) {
-      input(t, win[TAPS - 1]);
+#pragma unroll
+      for (int e = 0; e < V; ++e) win[TAPS - 1][e] = nxt[e];
+      if (t + 1 < end) input(t + 1, nxt);     // in flight under this token's work
       float y[V];
 #pragma unroll
       for (int e = 0; e < V; ++e) {
@@ -85,7 +88,7 @@ __device__ __forceinline__ void conv_walk(const ConvArgs& a, int seq, int start,
         for (int j = 0; j < TAPS; ++j) s += w[j][e] * win[j][e];
         y[e] = s;
       }
-      emit(row0 + t, y);
+      emit(row0 + t, y, t + 1 == end);
 #pragma unroll
       for (int j = 0; j + 1 < TAPS; ++j)
 #pragma unroll
@@ -103,7 +106,7 @@ __device__ __forceinline__ void conv_walk(const ConvArgs& a, int seq, int start,
 #pragma unroll
         for (int e = 0; e < V; ++e) y[e] += w[e] * x[e];
       }
-      emit(row0 + t, y);
+      emit(row0 + t, y, t + 1 == end);
     }
   }
   // state: inputs n - taps + 1 .. n - 1, written oldest first (entry s reads
@@ -124,7 +127,7 @@ __global__ void __launch_bounds__(256) short_conv_kernel(ConvArgs a, void* out, 
   const int start = a.tiles ? a.tiles[2 * blockIdx.x + 1] : 0;
   const int c0 = (blockIdx.y * 256 + threadIdx.x) * V;
   if (c0 >= a.C || a.slots[seq] < 0) return;
-  conv_walk<T, V, TAPS>(a, seq, start, c0, [&](int row, float (&y)[V]) {
+  conv_walk<T, V, TAPS>(a, seq, start, c0, [&](int row, float (&y)[V], bool) {
     if (act) {
 #pragma unroll
       for (int e = 0; e < V; ++e) y[e] *= sigmoid_t<T>(y[e]);
@@ -150,7 +153,11 @@ __global__ void __launch_bounds__(256) conv_qkv_cache_kernel(ConvArgs a, QkvOut 
   const int c0 = (blockIdx.y * 256 + threadIdx.x) * 8;
   if (c0 >= a.C || a.slots[seq] < 0) return;   // whole heads leave together
   const int head = c0 / o.D, d = c0 - head * o.D, lph = o.D >> 3;
-  conv_walk<T, 8, TAPS>(a, seq, start, c0, [&](int row, float (&y)[8]) {
+  // bf16 v: the last 4 tokens of each channel, newest in the top 16 bits; a
+  // key quad of the v page leaves as one 8-B store per channel
+  unsigned long long vq[8];
+  int vn = 0;                                  // tokens held since the walk began
+  conv_walk<T, 8, TAPS>(a, seq, start, c0, [&](int row, float (&y)[8], bool last) {
     if (head < o.Hq + o.Hkv) {
       float ss = 0.f;
 #pragma unroll
@@ -178,8 +185,25 @@ __global__ void __launch_bounds__(256) conv_qkv_cache_kernel(ConvArgs a, QkvOut 
     } else {
       const long kvh = head - o.Hq - o.Hkv;
       T* vp = (T*)o.vc + (blk * o.Hkv + kvh) * o.BS * o.D + vq_off(d, off, o.D);
+      if constexpr (sizeof(T) == 4) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) st1(vp + 4 * e, y[e]);
+        for (int e = 0; e < 8; ++e) vp[4 * e] = y[e];
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          vq[e] = (vn ? vq[e] >> 16 : 0ull) | (unsigned long long)f2bf(y[e]) << 48;
+        ++vn;
+        const int in_quad = (off & 3) + 1;     // tokens of this quad up to this one
+        if (in_quad == 4 && vn >= 4) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) *reinterpret_cast<unsigned long long*>(vp - 3 + 4 * e) = vq[e];
+        } else if (in_quad == 4 || last) {     // a quad this walk holds in part
+          const int k = min(in_quad, vn);
+          for (int i = 0; i < k; ++i)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) vp[4 * e - i] = (bf16_t)(vq[e] >> (48 - 16 * i));
+        }
+      }
     }
   });
 }

@@ -198,7 +198,7 @@ __global__ void __launch_bounds__(DTHREADS, 2) dgemm_kernel(
   static_assert(BK == 32 || BK == 64 || BK == 128, "BK");
   static_assert(BM % RPI == 0 && BN % RPW == 0, "stage rows");
   static_assert(EPI != 1 || (WN % 2 == 0 || WN == 1), "swiglu wave split");
-  static_assert(EPI != 3 || WTN % 32 == 0, "swiglu16: gate/up 16-column pairs inside a wave");
+  static_assert((EPI != 3 && EPI != 4) || WTN % 32 == 0, "swiglu16: gate/up 16-column pairs inside a wave");
   extern __shared__ __attribute__((aligned(16))) char smem[];
   bf16_t* const lds = reinterpret_cast<bf16_t*>(smem);
 
@@ -309,8 +309,8 @@ __global__ void __launch_bounds__(DTHREADS, 2) dgemm_kernel(
     }
     return;
   }
-  if constexpr (EPI == 3) {
-    // SwiGLU on 16-column pairs (ops.interleave_gate_up(w, 16): W rows
+  if constexpr (EPI == 3 || EPI == 4) {
+    // SwiGLU (4: ReLU-GLU) on 16-column pairs (ops.interleave_gate_up(w, 16): W rows
     // [16 gate | 16 up] per 16 channels): tiles 2j and 2j+1 of a wave are the
     // gate and up values of the same 16 channels in the same lane registers,
     // so the epilogue needs no LDS hand-off and any BN with WTN % 32 == 0 works
@@ -323,7 +323,8 @@ __global__ void __launch_bounds__(DTHREADS, 2) dgemm_kernel(
         bf16x4_t o;
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          o[r] = (short)f2bf(dg_silu(acc[i][2 * j][r]) * acc[i][2 * j + 1][r]);
+          o[r] = (short)f2bf((EPI == 3 ? dg_silu(acc[i][2 * j][r]) : fmaxf(acc[i][2 * j][r], 0.f)) *
+                             acc[i][2 * j + 1][r]);
         *reinterpret_cast<bf16x4_t*>(C + (long)m * ldc + ((n0 + wc * WTN) >> 1) + 16 * j +
                                      4 * fg) = o;
       }
@@ -570,7 +571,7 @@ int dgemm(void* C, const void* A, const void* W, float* slabs, unsigned* tickets
   const int nt = (cfg >> 5) & 1;      // bit 5: non-temporal weight stream
   const int sk = (cfg >> 6) & 1;      // bit 6: stream-K, `splits` = workgroups (0: 256)
   cfg &= 31;
-  if (cfg < 0 || cfg >= kNumDgCfgs || splits < 0 || epi < 0 || epi > 3) return -1;
+  if (cfg < 0 || cfg >= kNumDgCfgs || splits < 0 || epi < 0 || epi > 4) return -1;
   const DgCfg c = kDgCfgs[cfg];
   if (sk) {
     if (epi != 0 || N % c.bn != 0 || K % c.bk != 0) return -1;
@@ -593,6 +594,12 @@ int dgemm(void* C, const void* A, const void* W, float* slabs, unsigned* tickets
   if (epi == 3) {                                                                             \
     if constexpr ((BN / (8 / WM)) % 32 == 0)                                                  \
       return dg_launch<BM, BN, WM, NST, 3, ROT, NT, BK>(C_, A_, W_, slabs, tickets, M, N, K, \
+                                                        lda, ldw, ldc, splits, stream);       \
+    return -1;                                                                                \
+  }                                                                                           \
+  if (epi == 4) {                                                                             \
+    if constexpr ((BN / (8 / WM)) % 32 == 0)                                                  \
+      return dg_launch<BM, BN, WM, NST, 4, ROT, NT, BK>(C_, A_, W_, slabs, tickets, M, N, K, \
                                                         lda, ldw, ldc, splits, stream);       \
     return -1;                                                                                \
   }                                                                                           \

@@ -206,8 +206,8 @@ __device__ __forceinline__ void pg_store(RT& R, const PgOut& O, const PgThr& T,
       rs[i] = __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(
           O.rn, (T.wm * 128 + QM * 64 + 16 * i + T.fr) * 4, 0, 0));
   }
-  if constexpr (ACT == 3) {
-    // SwiGLU: 16-col tiles 0 (gate) and 1 (up) of the quadrant are one pair
+  if constexpr (ACT == 3 || ACT == 5) {
+    // SwiGLU (5: ReLU-GLU): 16-col tiles 0 (gate) and 1 (up) of the quadrant are one pair
     const int col = (O.n0 >> 1) + T.wn * 32 + QN * 16 + 4 * T.fg;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -219,7 +219,8 @@ __device__ __forceinline__ void pg_store(RT& R, const PgOut& O, const PgThr& T,
       const f32x4_t g = R.acc[QM][QN][i][0], u = R.acc[QM][QN][i][1];
       bf16x4_t o;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(g[r] / (1.f + __expf(-g[r])) * u[r]);
+      for (int r = 0; r < 4; ++r)
+        o[r] = (short)f2bf((ACT == 3 ? g[r] / (1.f + __expf(-g[r])) : fmaxf(g[r], 0.f)) * u[r]);
       __builtin_amdgcn_raw_buffer_store_b64(__builtin_bit_cast(u32x2_t, o), O.rc,
                                             (row * T.ldc + col) * 2, 0, 0);
     }
@@ -847,7 +848,7 @@ int pgemm(void* C, const void* A, const void* W, const void* bias, int M, int N,
   if (res && (act != 0 || bias != nullptr)) return -1;
   if (N % 256 != 0 || K % 64 != 0 || K < 192) return -1;
   if (lda % 8 || ldw % 8 || ldc % 4) return -1;
-  if (act < 0 || act > 4 || (act == 3 && bias != nullptr)) return -1;
+  if (act < 0 || act > 5 || ((act == 3 || act == 5) && bias != nullptr)) return -1;
   if (bias != nullptr && N > PG_MAX_BIAS) return -1;
   // byte offsets of one tile's rows are 32-bit
   if (256L * lda * 2 > 0x7fffffffL || 256L * ldw * 2 > 0x7fffffffL || 256L * ldc * 2 > 0x7fffffffL)
@@ -898,6 +899,7 @@ int pgemm(void* C, const void* A, const void* W, const void* bias, int M, int N,
     case 2: return pg_launch<2, 0>(C_, A_, W_, b_, M, N, K, ia, iw, ic, grid, stream);
     case 3: return pg_launch<3, 0>(C_, A_, W_, b_, M, N, K, ia, iw, ic, grid, stream);
     case 4: return pg_launch<4, 0>(C_, A_, W_, b_, M, N, K, ia, iw, ic, grid, stream);
+    case 5: return pg_launch<5, 0>(C_, A_, W_, b_, M, N, K, ia, iw, ic, grid, stream);
   }
   return -1;
 }

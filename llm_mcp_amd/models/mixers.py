@@ -222,19 +222,20 @@ class ReluGLU:
     """W_down (relu(W_gate h) * (W_up h))"""
 
     def __init__(self, m: dict, width: int):
-        self.ff, self.fp = m["ff"], _up(m["ff"], 8)
+        self.ff, self.fp = m["ff"], _up(m["ff"], 16)
         self.shapes = {"gate": (self.ff, width), "up": (self.ff, width),
                        "down": (width, self.ff)}
 
     def load(self, get, put):
-        self.w_gu = put(_fuse_rows([get("gate"), get("up")], [self.fp, self.fp]))
+        self.w_gu = put(ops.interleave_gate_up(
+            _fuse_rows([get("gate"), get("up")], [self.fp, self.fp]), 16))
         down = get("down")
         w = down.new_zeros((down.shape[0], self.fp))
         w[:, :self.ff] = down
         self.w_down = put(w)
 
     def forward(self, h, linear):
-        return linear(ops.relu_mul(linear(h, self.w_gu)), self.w_down, defer=True)
+        return linear(ops.linear_relu_glu(h, self.w_gu), self.w_down, defer=True)
 
 
 MIXERS = {"lightning": LightningMixer, "mamba2": Mamba2Mixer, "attention": ConvAttentionMixer}

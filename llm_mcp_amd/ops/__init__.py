@@ -501,16 +501,18 @@ def gelu_mul(x: torch.Tensor) -> torch.Tensor:
     return out
 
 
-def relu_mul(x: torch.Tensor) -> torch.Tensor:
-    """relu(gate) * up of a fused gate|up projection output (bf16 or fp32)."""
+def relu_mul(x: torch.Tensor, block: int = 0) -> torch.Tensor:
+    """relu(gate) * up of a fused gate|up projection output (bf16 or fp32);
+    ``block``: as in ``silu_mul``."""
     if not x.is_cuda:
-        return ref.relu_mul(x)
+        return ref.relu_mul(deinterleave_gate_up(x, block) if block else x)
     _chk(x.dtype in (torch.bfloat16, torch.float32) and x.is_contiguous()
          and x.shape[-1] % 16 == 0, "relu_mul shape")
     I = x.shape[-1] // 2
+    _chk(block % 8 == 0 and (block == 0 or I % block == 0), "relu_mul interleave block")
     rows = x.numel() // x.shape[-1]
     out = torch.empty(x.shape[:-1] + (I,), dtype=x.dtype, device=x.device)
-    native().glu(_ptr(out), _ptr(x), rows, I, 2, 0, int(x.dtype == torch.bfloat16), _stream())
+    native().glu(_ptr(out), _ptr(x), rows, I, 2, block, int(x.dtype == torch.bfloat16), _stream())
     return out
 
 
@@ -576,6 +578,7 @@ ACT_NONE, ACT_GELU, ACT_SILU = 0, 1, 2
 
 ACT_SWIGLU = 3
 ACT_GELU_ERF = 4   # exact (erf) GELU, BERT FFNs
+ACT_RELUGLU = 5    # the pair form of ACT_SWIGLU with ReLU on the gate
 
 
 def interleave_gate_up(w: torch.Tensor, block: int = 64) -> torch.Tensor:
@@ -864,6 +867,22 @@ def linear_swiglu(x: torch.Tensor, w: torch.Tensor, block: int,
     return _into(out, silu_mul(linear(x, w), block=block))
 
 
+def linear_relu_glu(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """relu(gate) * up of x @ w^T for gate|up weights interleaved per 16
+    channels (``interleave_gate_up(w, 16)``): the pair epilogue of the decode
+    GEMM where the table has one for this shape (measured with SwiGLU: the
+    epilogue's activation is not what it costs), of K13 for prefill-sized M,
+    else the product and the GLU kernel."""
+    if x.is_cuda and x.dtype == torch.bfloat16:
+        M, N, K = x.shape[0], w.shape[0], w.shape[1]
+        ch = dgemm_choice(M, N, K, epi=3)
+        if ch is not None and ch[0] >= 0 and swiglu16_ok(ch[0]):
+            return dgemm(x, w, ch[0], ch[1], epi=4)
+        if (large_gemm_backend(M, N, K, ACT_SWIGLU) == "k13" and pgemm_operands_ok(x, w)):
+            return pgemm(x, w, act=ACT_RELUGLU)
+    return relu_mul(linear(x, w), block=SWIGLU16)
+
+
 def swiglu_block(N: int, K: int) -> int:
     """Interleave block of the gate|up weights for the fused decode GEMM of
     this shape: 16 when the table has in-register-epilogue (epi 3) entries,
@@ -1119,20 +1138,22 @@ def dgemm(a: torch.Tensor, w: torch.Tensor, cfg: int, splits: int, epi: int = 0,
     per BN-column tile as [BN/2 gate | BN/2 up] rows (``interleave_gate_up``
     with ``block=BN/2``) and the result is silu(gate) * up (N/2 columns);
     epi=3: the same with ``w`` interleaved per 16 rows (block 16, any tile
-    whose wave tile width is a multiple of 32, ``swiglu16_ok``)."""
+    whose wave tile width is a multiple of 32, ``swiglu16_ok``); epi=4: epi 3
+    with ReLU on the gate."""
     M, K = a.shape
     N = w.shape[0]
     bm, bn = DGEMM_CONFIGS[cfg & DGEMM_CFG_MASK]
-    ncols = N // 2 if epi in (1, 3) else N
+    ncols = N // 2 if epi in (1, 3, 4) else N
     sk = bool(cfg & DGEMM_SK)
-    _chk(epi != 3 or swiglu16_ok(cfg), f"dgemm cfg {cfg} cannot run the epi-3 epilogue")
+    _chk(epi not in (3, 4) or swiglu16_ok(cfg), f"dgemm cfg {cfg} cannot run the epi-3 epilogue")
     _chk(not sk or epi == 0, "the stream-K form has the plain epilogue only")
     if not a.is_cuda:
         y = a.float() @ w.float().t()
-        if epi in (1, 3):
-            blk = SWIGLU16 if epi == 3 else bn // 2
+        if epi in (1, 3, 4):
+            blk = bn // 2 if epi == 1 else SWIGLU16
             y = y.view(M, N // (2 * blk), 2, blk)
-            y = (torch.nn.functional.silu(y[:, :, 0]) * y[:, :, 1]).reshape(M, ncols)
+            fn = torch.relu if epi == 4 else torch.nn.functional.silu
+            y = (fn(y[:, :, 0]) * y[:, :, 1]).reshape(M, ncols)
         y = y.to(a.dtype)
         if out is not None:
             out.copy_(y)
@@ -1531,8 +1552,8 @@ RESIDUAL_EPILOGUE = os.environ.get("LMX_RESIDUAL_EPILOGUE", "1") != "0"
 def pgemm_supported(N: int, K: int, act: int = 0, bias: bool = False) -> bool:
     """Shapes K13 takes: 256-column tiles, 64-deep K-steps, >= 3 of them;
     a bias row fits its LDS slot; the SwiGLU form takes no bias."""
-    return (N % 256 == 0 and K % 64 == 0 and K >= 192 and act in (0, 1, 2, 3, 4)
-            and not (bias and (N > PGEMM_MAX_BIAS or act == ACT_SWIGLU)))
+    return (N % 256 == 0 and K % 64 == 0 and K >= 192 and act in (0, 1, 2, 3, 4, 5)
+            and not (bias and (N > PGEMM_MAX_BIAS or act in (ACT_SWIGLU, ACT_RELUGLU))))
 
 
 def pgemm_operands_ok(a: torch.Tensor, w: torch.Tensor) -> bool:
@@ -1572,7 +1593,7 @@ def pgemm(a: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, ac
     packed = packed or is_packed_only(w)
     _chk(not packed or (bias is None and act in (ACT_NONE, ACT_SWIGLU) and a.is_cuda),
          "pgemm on packed W: plain / residual / SwiGLU products on CUDA")
-    ncols = N // 2 if act == ACT_SWIGLU else N
+    ncols = N // 2 if act in (ACT_SWIGLU, ACT_RELUGLU) else N
     if residual is not None:
         _chk(act == ACT_NONE and bias is None and out is None, "pgemm residual: plain product only")
         _chk(residual.shape == (M, N) and residual.dtype == a.dtype, "pgemm residual shape")
@@ -1593,9 +1614,10 @@ def pgemm(a: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, ac
                 out.copy_(y)
                 return out
             return y
-        if act == ACT_SWIGLU:
+        if act in (ACT_SWIGLU, ACT_RELUGLU):
             y = (a.float() @ w.float().t()).view(M, N // 32, 2, 16)
-            y = (torch.nn.functional.silu(y[:, :, 0]) * y[:, :, 1]).reshape(M, ncols).to(a.dtype)
+            fn = torch.nn.functional.silu if act == ACT_SWIGLU else torch.relu
+            y = (fn(y[:, :, 0]) * y[:, :, 1]).reshape(M, ncols).to(a.dtype)
         else:
             y = ref.gemm_nt(a, w, bias, act, None)
         if out is not None:

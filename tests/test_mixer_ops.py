@@ -129,6 +129,19 @@ def test_relu_glu(dev, dt):
     close(got, torch.relu(x[:, :24].double()) * x[:, 24:].double(), OUT_TOL[dt])
 
 
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("M,I,K", [(3, 48, 40), (64, 14336, 4096), (600, 256, 320)])
+def test_relu_glu_projection(dev, dt, M, I, K):
+    """Plain product + GLU kernel, the decode GEMM's pair epilogue (a measured
+    shape) and the prefill GEMM's."""
+    if dev == "cpu" and I > 1000:
+        pytest.skip("GPU GEMM shape")
+    x, w = rnd(M, K).to(dt), rnd(2 * I, K, seed=1, scale=K ** -0.5).to(dt)
+    got = ops.linear_relu_glu(x.to(dev), ops.interleave_gate_up(w, 16).to(dev))
+    y = x.to(dev).float() @ w.to(dev).float().t()
+    close(got, (torch.relu(y[:, :I]) * y[:, I:]).cpu(), 2e-2 if dt == torch.bfloat16 else 1e-4)
+
+
 # -------------------------------------------------------------- convolution --
 @pytest.mark.parametrize("dev,dt", DEV)
 @pytest.mark.parametrize("C,taps", [(64, 4), (16, 3), (40, 2), (24, 1), (24, 7), (13, 3)])
