@@ -36,6 +36,17 @@ NT_TOP = 4      # configurations re-timed with the non-temporal weight stream (c
 def shapes(model: str, tp: int = 1) -> dict:
     from ..models import config as mc
     c = mc.resolve(model)
+    if c.family == "zegopel":       # every distinct projection of its layers
+        from ..models.zegopel import ZegopelModel
+        out, seen = {}, set()
+        for L, (mix, ff) in zip(c.layers, ZegopelModel.layer_parts(c)):
+            for tag, part in ((L["type"], mix), ("mlp", ff)):
+                for k, (n, kk) in (part.proj.items() if part is not None else ()):
+                    if (n, kk) not in seen:
+                        seen.add((n, kk))
+                        out[f"{tag}.{k}"] = (n, kk, 1 if k == "gate_up" else 0)
+        out["lm_head"] = (c.vocab_size, c.hidden_size, 0)
+        return out
     d, hd = c.hidden_size, c.head_dim
     qkv = (c.num_heads // tp + 2 * max(1, c.num_kv_heads // tp)) * hd
     inter = c.intermediate_size // tp
@@ -178,7 +189,7 @@ def run(model: str, tp: int, ms: list[int], margin: float, only: str = "",
                                      "splits": 0, "bn": 0, "us": None,
                                      "lib_us": round(t_lib, 2), "shape": name})
             print(line, flush=True)
-            if name in DEFERRED and tp == 1:
+            if name.split(".")[-1] in DEFERRED and tp == 1:
                 best_entries.append(deferred(name, N, K, M, x, ws, ncopy, iters, cfgs, margin,
                                              rows))
         del ws, wil

@@ -372,7 +372,7 @@ struct SandwichArgs {
 };
 
 template <typename T, int V, int VPT>
-__global__ void __launch_bounds__(256) sandwich_norm_kernel(SandwichArgs a) {
+__global__ void __launch_bounds__(512) sandwich_norm_kernel(SandwichArgs a) {
   __shared__ float scratch[16];
   const long src = a.rows_idx ? a.rows_idx[blockIdx.x] : blockIdx.x;
   const int cols = a.cols, nchunk = cols / V;
@@ -455,14 +455,14 @@ int sandwich_norm(void* out, float* residual, const void* y, long y_ld, int slab
                        w_post, w_pre, rows_idx, cols, eps};
   const bool vec = cols % 8 == 0 && y_ld % 8 == 0;
   const int nchunk = vec ? cols / 8 : cols;
-  const int vpt = (nchunk + 255) / 256;
-  if (vpt > 8) return -2;
-  const int threads = nchunk >= 256 ? 256 : (nchunk + 63) / 64 * 64;
+  const int vpt = (nchunk + 511) / 512;
+  if (vpt > (vec ? 4 : 8)) return -2;
+  const int threads = nchunk >= 512 ? 512 : (nchunk + 63) / 64 * 64;
 #define LMX_SW(T, V, P) sandwich_norm_kernel<T, V, P><<<dim3(rows), dim3(threads), 0, stream>>>(a)
 #define LMX_SWT(T)                                                            \
   if (vec) {                                                                  \
     if (vpt == 1) LMX_SW(T, 8, 1); else if (vpt == 2) LMX_SW(T, 8, 2);        \
-    else if (vpt <= 4) LMX_SW(T, 8, 4); else LMX_SW(T, 8, 8);                 \
+    else LMX_SW(T, 8, 4);                                                     \
   } else {                                                                    \
     if (vpt == 1) LMX_SW(T, 1, 1); else LMX_SW(T, 1, 8);                      \
   }

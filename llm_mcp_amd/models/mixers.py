@@ -8,7 +8,7 @@ rows: ``forward(h, inp, cache, state)`` -> the mixer's output rows.
 
 Served layouts:
 * every mixer has ONE input projection (its projections fused by rows) and one
-  output projection; sections start at multiples of 8 rows (zero rows between)
+  output projection (``proj``: their served shapes); sections start at multiples of 8 rows (zero rows between)
   so row slices stay 16-byte aligned;
 * attention heads are padded to D = 64 / 128 / 256 / 512 channels with zero
   rows (and zero output columns), so unequal or odd query / value sizes run on
@@ -54,6 +54,7 @@ class LightningMixer:
         self.shapes = {"q": (H * N, width), "k": (H * N, width), "v": (H * P, width),
                        "g": (H * P, width), "o": (width, H * P), "norm": (H * P,)}
         self.qk, self.vg = _up(H * N, 8), _up(H * P, 8)
+        self.proj = {"in": (2 * (self.qk + self.vg), width), "o": self.shapes["o"]}
 
     def state_shapes(self, dtype):
         return [((self.H, self.N, self.P), torch.float32)]
@@ -94,7 +95,11 @@ class Mamba2Mixer:
         if H % G:
             raise ValueError("mamba2: heads must be a multiple of groups")
         self.inner, self.C = H * P, H * P + 2 * G * N
-        self.zp, self.cp, self.dp = _up(self.inner, 8), _up(self.C, 8), _up(H, 8)
+        self.zp, self.cp = _up(self.inner, 8), _up(self.C, 8)
+        # a wide projection is rounded up to whole 256-row GEMM tiles
+        rows = self.zp + self.cp + _up(H, 8)
+        self.dp = (_up(rows, 256) if rows >= 4096 else rows) - self.zp - self.cp
+        self.proj = {"in": (self.zp + self.cp + self.dp, width), "o": (width, self.inner)}
         self.shapes = {"in": (2 * self.inner + 2 * G * N + H, width),
                        "conv": (self.C, self.taps), "conv.b": (self.C,), "dt_bias": (H,),
                        "A_log": (H,), "D": (H,), "norm": (self.inner,),
@@ -165,6 +170,7 @@ class ConvAttentionMixer:
                        "o": (width, H * dv)}
         self.kv = (G, D)
         self.qkv = (H + 2 * G) * D
+        self.proj = {"in": (self.qkv + H * D, width), "o": (width, H * D)}
         # the MFMA attention kernels: head sizes 64 / 128, up to 16 query heads per kv head
         self.mfma_geometry = D in (64, 128) and H // G <= 16
         # queries per prefill workgroup (4 waves)
@@ -225,6 +231,7 @@ class ReluGLU:
         self.ff, self.fp = m["ff"], _up(m["ff"], 16)
         self.shapes = {"gate": (self.ff, width), "up": (self.ff, width),
                        "down": (width, self.ff)}
+        self.proj = {"gate_up": (2 * self.fp, width), "down": (width, self.fp)}
 
     def load(self, get, put):
         self.w_gu = put(ops.interleave_gate_up(

@@ -48,6 +48,7 @@ def tensor_shapes(cfg: ZegopelConfig) -> dict[str, tuple]:
 
 
 class ZegopelModel:
+    layer_parts = staticmethod(_layer_parts)
     prefix_cache_ok = False       # a cached page does not bring the state behind it
 
     def __init__(self, cfg: ZegopelConfig, device: torch.device | str = "cuda",

@@ -33,7 +33,7 @@ def main():
             if (e["N"], e["K"], e["epi"]) in have:
                 continue
             e["shape"] = f"{tag}.{e['shape']}"
-            e["note"] = "bench/dgemm_bench.py (cold weights), round 6 family sweep"
+            e["note"] = "bench/dgemm_bench.py (cold weights)"
             added.append(e)
         have |= {(e["N"], e["K"], e["epi"]) for e in added}
     doc["entries"] += added
