@@ -279,6 +279,8 @@ def cmd_serve(args):
     extra = ["--cpu"] if args.cpu else []
     if args.weights:       # real checkpoint for the chat model (each TP rank loads its shard)
         extra += ["--weights", args.weights]
+    if args.dtype != "bfloat16":
+        extra += ["--dtype", args.dtype]
     plan = [dict(w, replica=k) for w in plan for k in range(max(1, args.replicas_per_gpu))
             if k == 0 or w["tp"] == 1]
     for w in plan:
@@ -340,6 +342,8 @@ def main(argv=None):
             p.add_argument("--tp", type=int, default=int(os.environ.get("LMX_TP", "1")))
             p.add_argument("--weights", default=os.environ.get("LMX_WEIGHTS", ""),
                            help="safetensors dir of the chat model's real weights")
+            p.add_argument("--dtype", default="bfloat16", choices=("bfloat16", "float32"),
+                           help="float32: families that run in it (zegopel)")
             p.add_argument("--max-num-seqs", type=int,
                            default=int(os.environ.get("LMX_MAX_BATCH", "256")))
             p.add_argument("--registry", default=os.environ.get("LMX_MODEL_REGISTRY", ""),

@@ -86,8 +86,8 @@ __global__ void __launch_bounds__(256) scan_recurrent_kernel(ScanArgs a, int seq
     for (int e = 0; e < VEC; ++e) S[i][e] = 0.f;
     if (live && !fresh && kk < N && pc < P) {
       if constexpr (VEC == 4) {
-        const float4 t = *reinterpret_cast<const float4*>(st + (long)kk * P);
-        S[i][0] = t.x; S[i][1] = t.y; S[i][2] = t.z; S[i][3] = t.w;
+        const f32x4_t t = __builtin_nontemporal_load(reinterpret_cast<const f32x4_t*>(st + (long)kk * P));
+        S[i][0] = t[0]; S[i][1] = t[1]; S[i][2] = t[2]; S[i][3] = t[3];
       } else {
         S[i][0] = st[(long)kk * P];
       }
@@ -151,8 +151,8 @@ __global__ void __launch_bounds__(256) scan_recurrent_kernel(ScanArgs a, int seq
     const int kk = r + i * kr;
     if (live && kk < N && pc < P) {
       if constexpr (VEC == 4) {
-        *reinterpret_cast<float4*>(st + (long)kk * P) =
-            make_float4(S[i][0], S[i][1], S[i][2], S[i][3]);
+        const f32x4_t t = {S[i][0], S[i][1], S[i][2], S[i][3]};
+        __builtin_nontemporal_store(t, reinterpret_cast<f32x4_t*>(st + (long)kk * P));
       } else {
         st[(long)kk * P] = S[i][0];
       }

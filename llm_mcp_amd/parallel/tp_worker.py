@@ -196,7 +196,8 @@ def run_tp_worker(a) -> None:
     if tp.size != a.tp:
         raise SystemExit(f"--tp {a.tp} but the launcher started {tp.size} ranks")
     ecfg = EngineConfig(model=a.chat_model, max_num_seqs=a.max_num_seqs,
-                        max_model_len=a.max_model_len, kv_fraction=a.kv_fraction)
+                        max_model_len=a.max_model_len, kv_fraction=a.kv_fraction,
+                        dtype=getattr(a, "dtype", "bfloat16"))
     if a.max_batched_tokens:
         ecfg.max_batched_tokens = a.max_batched_tokens
     tag = f"{rocm_enum.host_id()}-{os.environ.get('MASTER_PORT', '0')}"

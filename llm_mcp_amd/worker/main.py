@@ -35,7 +35,10 @@ def build_parser():
     ap.add_argument("--max-model-len", type=int, default=8192)
     ap.add_argument("--kv-fraction", type=float, default=0.6)
     ap.add_argument("--lease-seconds", type=int, default=int(os.environ.get("WORKER_LEASE_SECONDS", "60")))
-    ap.add_argument("--weights", default="", help="safetensors dir of real weights (optional)")
+    ap.add_argument("--weights", default="", help="safetensors dir of real weights (optional; a "
+                    "--chat-model that is a checkpoint directory brings its own)")
+    ap.add_argument("--dtype", default="bfloat16", choices=("bfloat16", "float32"),
+                    help="float32: families that run in it (zegopel)")
     ap.add_argument("--embed-weights", default="",
                     help="safetensors dir of the embedding model (nomic-bert or BERT; optional)")
     ap.add_argument("--tp", type=int, default=1)
@@ -84,7 +87,8 @@ def main(argv=None):
             from ..models.weights import load_weights
             weights = load_weights(a.weights, cfg, dev)
         ecfg = EngineConfig(model=a.chat_model, max_num_seqs=a.max_num_seqs,
-                            max_model_len=a.max_model_len, kv_fraction=a.kv_fraction)
+                            max_model_len=a.max_model_len, kv_fraction=a.kv_fraction,
+                            dtype=a.dtype)
         if a.max_batched_tokens:
             ecfg.max_batched_tokens = a.max_batched_tokens
         elif (a.embed_model or a.replica) and not os.environ.get("LMX_MAX_BATCHED_TOKENS"):

@@ -3,13 +3,15 @@
 slots and pages that are used again, generation -- on the CPU references and on
 the GPU kernels, in bf16 and fp32."""
 import json
+import threading
+import time
 
 import numpy as np
 import pytest
 import torch
 
 import zegopel_oracle as oracle
-from llm_mcp_amd.engine.engine import EngineConfig, LLMEngine, SamplingParams
+from llm_mcp_amd.engine.engine import EngineConfig, GenRequest, LLMEngine, SamplingParams
 from llm_mcp_amd.models import config as mc
 from llm_mcp_amd.models.registry import model_class
 from llm_mcp_amd.models.weights import load_weights, save_zegopel
@@ -182,6 +184,42 @@ def test_generation_is_greedy_of_the_reference(device, dtype):
         assert float(short.max()) < 4 * TOL[dtype] * float(lg.std())
     if device == "cuda":
         assert e.stats["graph_steps"] > 0
+
+
+@pytest.mark.parametrize("device", ["cpu", pytest.param("cuda", marks=GPU)])
+def test_served_requests_come_and_go(device):
+    """The engine thread with requests submitted while others run (lookahead
+    stepping on the GPU): every stream equals the same request alone, whatever
+    slots and pages it got; a stop token ends one early."""
+    cfg = CASES["mixed"]
+    W = weights(cfg, 8)
+    e = engine(cfg, W, device, "float32", seqs=3, graphs=device == "cuda")
+    prompts = [tokens(cfg, n, seed=60 + n) for n in (4, 35, 1, 70, 20, 9, 50)]
+    sp = SamplingParams(temperature=0, max_tokens=20, ignore_eos=True)
+    alone = [e.generate([p], sp)[0] for p in prompts]
+    got, done = {}, threading.Event()
+
+    def sink(evs):
+        for v in evs:
+            got.setdefault(v.req.user, []).append(v.token)
+            if v.finish is not None and all(r.finished for r in reqs):
+                done.set()
+    reqs = []
+    e.event_sink = sink
+    stop = alone[3][7]
+    e.start()
+    try:
+        for i, p in enumerate(prompts):
+            params = sp if i != 3 else SamplingParams(temperature=0, max_tokens=20,
+                                                      stop_token_ids=[stop])
+            reqs.append(e.submit(GenRequest(p, params, user=i)))
+            time.sleep(0.01)
+        assert done.wait(60)
+    finally:
+        e.stop()
+    want = dict(enumerate(alone))
+    want[3] = alone[3][:alone[3].index(stop) + 1]
+    assert got == want
 
 
 @pytest.mark.parametrize("device,dtype", RUNS)
