@@ -130,7 +130,7 @@ def test_relu_glu(dev, dt):
 
 
 @pytest.mark.parametrize("dev,dt", DEV)
-@pytest.mark.parametrize("M,I,K", [(3, 48, 40), (64, 14336, 4096), (600, 256, 320)])
+@pytest.mark.parametrize("M,I,K", [(3, 48, 40), (64, 14336, 4096), (600, 256, 384)])
 def test_relu_glu_projection(dev, dt, M, I, K):
     """Plain product + GLU kernel, the decode GEMM's pair epilogue (a measured
     shape) and the prefill GEMM's."""
@@ -427,7 +427,7 @@ def test_temperature_steps_at_its_interval():
 
 
 @pytest.mark.parametrize("dev,dt", DEV)
-@pytest.mark.parametrize("every", [1.0, 8.0, 256.0])
+@pytest.mark.parametrize("every", [1.0, 8.0, 255.0])
 def test_query_temperature_of_the_kernel(dev, dt, every):
     """q rows leave the convolution kernel scaled by the temperature: positions
     around its steps, far out as well."""
@@ -442,9 +442,9 @@ def test_query_temperature_of_the_kernel(dev, dt, every):
     q = ops.conv_qkv_cache(u, torch.ones(1, C, device=dev), None, None,
                            torch.arange(T + 1, **i32), z + 1, torch.arange(T, **i32),
                            torch.tensor(pos, **i32), torch.arange(T, **i32) * 32, kc, vc, 2, 64,
-                           1e-5, (0.5, every))
+                           1e-5, (0.6, every))
     want = oracle.unit_rms(u.double().cpu()[:, :128].view(T, 2, 64), 1e-5) * \
-        oracle.query_temperature(torch.tensor(pos).double(), 0.5, every)[:, None, None]
+        oracle.query_temperature(torch.tensor(pos).double(), 0.6, every)[:, None, None]
     got = q.double().cpu().view(T, 2, 64)
     assert float(((got - want).abs() / want.abs().clamp_min(1e-2)).max()) < \
         (2e-6 if dt == torch.float32 else 5e-3)
