@@ -69,15 +69,15 @@ class LightningMixer:
         d = torch.tensor(self.decay, dtype=torch.float64)
         self.decays = (put(d, fp32=True), put(d.log().clamp_min(-1e30), fp32=True))
 
-    def forward(self, h, inp, cache, state, linear):
+    def forward(self, h, inp, cache, state):
         qk, vg = self.qk, self.vg
-        p = linear(h, self.w_in)
+        p = ops.linear(h, self.w_in)
         o = ops.linear_scan(p[:, :qk], p[:, qk:2 * qk], p[:, 2 * qk:2 * qk + vg], state[0],
                             inp.cu_q, inp.context_lens, inp.state_slots, decay=self.decays,
                             silu=True, num_decode=inp.num_decode,
                             segments=inp.aux.get(f"scan{self.scan_geometry}"))
         y = ops.gated_norm(o, p[:, 2 * qk + vg:], self.norm, 1, self.eps, gate_first=False)
-        return linear(y, self.w_o, defer=True)
+        return ops.linear(y, self.w_o, defer=True)
 
 
 class Mamba2Mixer:
@@ -127,9 +127,9 @@ class Mamba2Mixer:
         self.norm = put(get("norm"), fp32=True)
         self.w_o = put(get("o"))
 
-    def forward(self, h, inp, cache, state, linear):
+    def forward(self, h, inp, cache, state):
         i, gn = self.inner, self.G * self.N
-        p = linear(h, self.w_in)
+        p = ops.linear(h, self.w_in)
         z, u, dt = p[:, :i], p[:, self.zp:self.zp + self.cp], p[:, self.zp + self.cp:]
         c = ops.short_conv(u, self.conv, state[1] if self.taps > 1 else None, inp.cu_q,
                            inp.context_lens, inp.state_slots, bias=self.conv_b, silu=True,
@@ -140,7 +140,7 @@ class Mamba2Mixer:
                             num_decode=inp.num_decode,
                             segments=inp.aux.get(f"scan{self.scan_geometry}"))
         y = ops.gated_norm(y, z, self.norm, self.norm_groups, self.eps, gate_first=True)
-        return linear(y, self.w_o, defer=True)
+        return ops.linear(y, self.w_o, defer=True)
 
 
 class ConvAttentionMixer:
@@ -197,9 +197,9 @@ class ConvAttentionMixer:
                         .float().t(), fp32=True)
         self.w_o = put(self._heads(get("o").t().contiguous(), H, dv).t())
 
-    def forward(self, h, inp, cache, state, linear):
+    def forward(self, h, inp, cache, state):
         kc, vc = cache
-        p = linear(h, self.w_in)
+        p = ops.linear(h, self.w_in)
         gate = p[:, self.qkv:]
         q = ops.conv_qkv_cache(p[:, :self.qkv], self.conv, self.in_bias,
                                state[0] if self.taps > 1 else None, inp.cu_q, inp.context_lens,
@@ -209,7 +209,7 @@ class ConvAttentionMixer:
         if not self.mfma_geometry or q.dtype != torch.bfloat16:
             a = ops.attention_any(q, kc, vc, inp.block_tables, inp.cu_q, inp.context_lens,
                                   inp.positions, self.scale, self.Hq, gate=gate)
-            return linear(a, self.w_o, defer=True)
+            return ops.linear(a, self.w_o, defer=True)
         a = torch.empty((T, self.Hq * self.D), dtype=q.dtype, device=q.device)
         if nd:
             ops.paged_decode_attention(q[:nd], kc, vc, inp.block_tables, inp.context_lens,
@@ -221,7 +221,7 @@ class ConvAttentionMixer:
                                         inp.context_lens[nd:], inp.aux[f"attn{self.q_per_tile}"],
                                         self.scale, a, Hq=self.Hq, q_per_tile=self.q_per_tile,
                                         gate=gate, precise=True)
-        return linear(a, self.w_o, defer=True)
+        return ops.linear(a, self.w_o, defer=True)
 
 
 class ReluGLU:
@@ -241,8 +241,8 @@ class ReluGLU:
         w[:, :self.ff] = down
         self.w_down = put(w)
 
-    def forward(self, h, linear):
-        return linear(ops.linear_relu_glu(h, self.w_gu), self.w_down, defer=True)
+    def forward(self, h):
+        return ops.linear(ops.linear_relu_glu(h, self.w_gu), self.w_down, defer=True)
 
 
 MIXERS = {"lightning": LightningMixer, "mamba2": Mamba2Mixer, "attention": ConvAttentionMixer}

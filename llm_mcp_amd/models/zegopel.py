@@ -172,11 +172,11 @@ class ZegopelModel:
         all_rows = inp.sample_rows.numel() == T
         for i, ((mix, ff), n) in enumerate(zip(self.parts, self.norms)):
             state = [next(states) for _ in mix.state_shapes(dt)]
-            y = mix.forward(h, inp, next(kv) if mix.kv is not None else None, state, ops.linear)
+            y = mix.forward(h, inp, next(kv) if mix.kv is not None else None, state)
             last = i + 1 == len(self.parts)
             if ff is not None:
                 h = ops.sandwich_norm(x, eps, y=y, w_post=n[1], w_pre=n[2], dtype=dt)
-                y = ff.forward(h, ops.linear)
+                y = ff.forward(h)
             post = n[3] if ff is not None else n[1]
             if not last:
                 h = ops.sandwich_norm(x, eps, y=y, w_post=post, w_pre=self.norms[i + 1][0],
