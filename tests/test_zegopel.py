@@ -384,3 +384,15 @@ def test_trace_replay(tmp_path):
         got = np.fromfile(out / f"{step}.f32", "<f4").reshape(-1, cfg["vocab"])
         check(torch.from_numpy(got.copy()), want[places], "float32")
     assert e.sched.kv_usage == 0.0
+
+
+def test_feed_serves_other_families_too():
+    """Teacher-forced steps are the engine's, not one model's: portions of a
+    Llama sequence give the logits of the whole prompt."""
+    e = LLMEngine(EngineConfig(model="tiny-llama", max_num_seqs=2, max_batched_tokens=256,
+                               max_model_len=256, use_graphs=False), device="cpu")
+    toks = list(range(20, 90))
+    whole = e.feed([(1, toks, list(range(70)))], [1])
+    parts = torch.cat([e.feed([(2, toks[a:b], list(range(b - a)))])
+                       for a, b in ((0, 33), (33, 34), (34, 70))])
+    assert float((whole - parts).abs().max()) < 0.05 * float(whole.std())
