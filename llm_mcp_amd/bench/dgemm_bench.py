@@ -36,10 +36,10 @@ NT_TOP = 4      # configurations re-timed with the non-temporal weight stream (c
 def shapes(model: str, tp: int = 1) -> dict:
     from ..models import config as mc
     c = mc.resolve(model)
-    if c.family == "zegopel":       # every distinct projection of its layers
-        from ..models.zegopel import ZegopelModel
+    if isinstance(c, mc.LayerListConfig):       # every distinct projection of its layers
+        from ..models.registry import model_class
         out, seen = {}, set()
-        for L, (mix, ff) in zip(c.layers, ZegopelModel.layer_parts(c)):
+        for L, (mix, ff) in zip(c.layers, model_class(c).layer_parts(c)):
             for tag, part in ((L["type"], mix), ("mlp", ff)):
                 for k, (n, kk) in (part.proj.items() if part is not None else ()):
                     if (n, kk) not in seen:

@@ -35,12 +35,36 @@ int paged_prefill(const void*, long, const void*, const void*, const int*, int, 
 int attention_any(const void*, long, const void*, const void*, const int*, int, const int*, int,
                   const int*, int, void*, long, const void*, long, int, int, int, int, float, int,
                   hipStream_t);
-int sandwich_norm(void*, float*, const void*, long, int, long, const int*, const void*,
-                  const float*, const float*, const long*, int, int, float, int, hipStream_t);
+int sandwich_norm(void*, float*, const void*, long, int, long, const int*, const float*, int,
+                  const int*, const void*, float, const float*, const float*, const long*, int, int,
+                  float, int, hipStream_t);
+int gelu(void*, long, int, hipStream_t);
+int grouped(const void*, long, long, const void*, void*, long, long, int, int, int, int, const int*,
+            int, const int*, const int*, const float*, const void*, long, int, int, hipStream_t);
+int moe_route(const void*, long, const void*, int, int, int, int, int, int*, float*, int,
+              hipStream_t);
+int moe_plan(const int*, int, int, int, int, int, int*, int*, int*, int*, int*, hipStream_t);
+int rglru_chunks(const void*, const void*, long, const float*, const float*, const float*, void*,
+                 float*, const int*, const int*, const int*, int, int, const void*, int, const int*,
+                 int, const int*, float*, hipStream_t);
+int rglru_rows(const void*, const void*, long, const float*, const float*, const float*, void*,
+               float*, const int*, const int*, const int*, int, int, const void*, int, hipStream_t);
+int rglru_scan(const void*, const void*, long, const float*, const float*, const float*, void*,
+               float*, const int*, const int*, const int*, int, int, const float*, int, int,
+               hipStream_t);
+int rope_angles(const int*, const double*, int, int, float*, hipStream_t);
+int latent_prep(const void*, long, int, int, int, const float*, int, int, const float*,
+                const float*, int, const int*, void*, int, int, void*, float, int, hipStream_t);
+int latent_rotate(const void*, long, int, const float*, int, int, int, int, void*, long, int, int,
+                  hipStream_t);
+int latent_any(const void*, const void*, const int*, int, const int*, int, const int*, int, void*,
+               int, int, int, float, int, int, hipStream_t);
+int latent_rows(const void*, const void*, const int*, int, const int*, int, const int*, int, int,
+                void*, float*, float*, int, int, int, float, int, int, int, hipStream_t);
 int gated_norm(void*, long, const void*, long, const void*, long, const float*, int, int, int, int,
                float, int, hipStream_t);
-int short_conv(const void*, long, const float*, const float*, void*, const int*, int, int,
-               const int*, const int*, const int*, int, int, void*, long, int, int, hipStream_t);
+int short_conv(const void*, long, const float*, const float*, const float*, void*, const int*, int,
+               int, const int*, const int*, const int*, int, int, void*, long, int, int, hipStream_t);
 int conv_qkv_cache(const void*, long, const float*, const float*, void*, const int*, int, int, const int*,
                    const int*, const int*, int, void*, long, void*, void*, const int*, const int*,
                    int, int, int, int, int, float, float, float, int, hipStream_t);
@@ -183,14 +207,98 @@ PYBIND11_MODULE(_lmx_kernels, m) {
   });
   // ---- sandwich / gated norms (norm.hip) ----
   m.def("sandwich_norm", [](uptr out, uptr residual, uptr y, long y_ld, int slabs,
-                            long slab_stride, uptr ids, uptr table, uptr w_post, uptr w_pre,
-                            uptr rows_idx, int rows, int cols, float eps, int is_bf16,
+                            long slab_stride, uptr mix_pos, uptr mix_w, int mix_n, uptr ids,
+                            uptr table, float scale, uptr w_post, uptr w_pre, uptr rows_idx, int rows, int cols, float eps, int is_bf16,
                             uptr stream) {
     check(lmx::sandwich_norm(P<void>(out), P<float>(residual), P<void>(y), y_ld, slabs,
-                             slab_stride, P<int>(ids), P<void>(table), P<float>(w_post),
-                             P<float>(w_pre), P<long>(rows_idx), rows, cols, eps, is_bf16,
+                             slab_stride, P<int>(mix_pos), P<float>(mix_w), mix_n, P<int>(ids),
+                             P<void>(table), scale, P<float>(w_post), P<float>(w_pre), P<long>(rows_idx), rows, cols, eps, is_bf16,
                              S(stream)),
           "sandwich_norm");
+  });
+  m.def("gelu", [](uptr x, long n, int is_bf16, uptr stream) {
+    check(lmx::gelu(P<void>(x), n, is_bf16, S(stream)), "gelu");
+  });
+  m.def("grouped", [](uptr a, long lda, long a_gs, uptr w, uptr c, long ldc, long c_gs, int groups,
+                      int N, int K, int M, uptr tiles, int mtiles, uptr off, uptr src, uptr limit,
+                      uptr gate, long gate_ld, int bm, int is_bf16, uptr stream) {
+    check(lmx::grouped(P<void>(a), lda, a_gs, P<void>(w), P<void>(c), ldc, c_gs, groups, N, K, M,
+                       P<int>(tiles), mtiles, P<int>(off), P<int>(src), P<float>(limit),
+                       P<void>(gate), gate_ld, bm, is_bf16, S(stream)),
+          "grouped");
+  });
+  m.def("moe_route", [](uptr h, long h_ld, uptr w, int T, int d, int E, int top, int extra, uptr ids,
+                        uptr wts, int is_bf16, uptr stream) {
+    check(lmx::moe_route(P<void>(h), h_ld, P<void>(w), T, d, E, top, extra, P<int>(ids),
+                         P<float>(wts), is_bf16, S(stream)),
+          "moe_route");
+  });
+  m.def("moe_plan", [](uptr ids, int n, int J, int groups, int bm, int mtiles, uptr hist, uptr off,
+                       uptr src, uptr pos, uptr tiles, uptr stream) {
+    check(lmx::moe_plan(P<int>(ids), n, J, groups, bm, mtiles, P<int>(hist), P<int>(off),
+                        P<int>(src), P<int>(pos), P<int>(tiles), S(stream)),
+          "moe_plan");
+  });
+  m.def("rglru_chunks", [](uptr u, uptr y, long y_ld, uptr y_b, uptr g_b, uptr log_a, uptr out,
+                           uptr state, uptr cu_q, uptr ctx, uptr slots, int C, int bp, uptr w,
+                           int seq0, uptr segs, int nsegs, uptr first, uptr ws, uptr stream) {
+    check(lmx::rglru_chunks(P<void>(u), P<void>(y), y_ld, P<float>(y_b), P<float>(g_b),
+                            P<float>(log_a), P<void>(out), P<float>(state), P<int>(cu_q),
+                            P<int>(ctx), P<int>(slots), C, bp, P<void>(w), seq0, P<int>(segs), nsegs,
+                            P<int>(first), P<float>(ws), S(stream)),
+          "rglru_chunks");
+  });
+  m.def("rglru_rows", [](uptr u, uptr y, long y_ld, uptr y_b, uptr g_b, uptr log_a, uptr out,
+                         uptr state, uptr cu_q, uptr ctx, uptr slots, int C, int bp, uptr w,
+                         int rows, uptr stream) {
+    check(lmx::rglru_rows(P<void>(u), P<void>(y), y_ld, P<float>(y_b), P<float>(g_b),
+                          P<float>(log_a), P<void>(out), P<float>(state), P<int>(cu_q), P<int>(ctx),
+                          P<int>(slots), C, bp, P<void>(w), rows, S(stream)),
+          "rglru_rows");
+  });
+  m.def("rglru_scan", [](uptr u, uptr y, long y_ld, uptr y_b, uptr g_b, uptr log_a, uptr out,
+                         uptr state, uptr cu_q, uptr ctx, uptr slots, int C, int bp, uptr z, int nseq,
+                         int is_bf16, uptr stream) {
+    check(lmx::rglru_scan(P<void>(u), P<void>(y), y_ld, P<float>(y_b), P<float>(g_b),
+                          P<float>(log_a), P<void>(out), P<float>(state), P<int>(cu_q), P<int>(ctx),
+                          P<int>(slots), C, bp, P<float>(z), nseq, is_bf16, S(stream)),
+          "rglru_scan");
+  });
+  m.def("rope_angles", [](uptr positions, uptr freqs, int T, int n, uptr out, uptr stream) {
+    check(lmx::rope_angles(P<int>(positions), P<double>(freqs), T, n, P<float>(out), S(stream)),
+          "rope_angles");
+  });
+  m.def("latent_prep", [](uptr p, long p_ld, int T, int qr, int qp, uptr q_norm, int R, int Rp,
+                          uptr c_norm, uptr ang, int d, uptr slots, uptr pages, int BS, int D,
+                          uptr cq, float eps, int is_bf16, uptr stream) {
+    check(lmx::latent_prep(P<void>(p), p_ld, T, qr, qp, P<float>(q_norm), R, Rp, P<float>(c_norm),
+                           P<float>(ang), d, P<int>(slots), P<void>(pages), BS, D, P<void>(cq), eps,
+                           is_bf16, S(stream)),
+          "latent_prep");
+  });
+  m.def("latent_rotate", [](uptr q, long q_ld, int np, uptr ang, int d, int T, int H, int xp,
+                            uptr out, long o_ld, int Rp, int is_bf16, uptr stream) {
+    check(lmx::latent_rotate(P<void>(q), q_ld, np, P<float>(ang), d, T, H, xp, P<void>(out), o_ld,
+                             Rp, is_bf16, S(stream)),
+          "latent_rotate");
+  });
+  m.def("latent_any", [](uptr q, uptr pages, uptr bt, int bt_stride, uptr cu_q, int nseq,
+                         uptr positions, int rows, uptr out, int H, int Rp, int D, float scale,
+                         int window, int is_bf16, uptr stream) {
+    check(lmx::latent_any(P<void>(q), P<void>(pages), P<int>(bt), bt_stride, P<int>(cu_q), nseq,
+                          P<int>(positions), rows, P<void>(out), H, Rp, D, scale, window, is_bf16,
+                          S(stream)),
+          "latent_any");
+  });
+  m.def("latent_rows", [](uptr q, uptr pages, uptr bt, int bt_stride, uptr cu_q, int nseq,
+                          uptr positions, int rows, int num_decode, uptr out, uptr part_o,
+                          uptr part_ml, int H, int Rp, int D, float scale, int window,
+                          int part_keys, int max_parts, uptr stream) {
+    check(lmx::latent_rows(P<void>(q), P<void>(pages), P<int>(bt), bt_stride, P<int>(cu_q), nseq,
+                           P<int>(positions), rows, num_decode, P<void>(out), P<float>(part_o),
+                           P<float>(part_ml), H, Rp, D, scale, window, part_keys, max_parts,
+                           S(stream)),
+          "latent_rows");
   });
   m.def("gated_norm", [](uptr out, long out_ld, uptr x, long x_ld, uptr g, long g_ld, uptr w,
                          int rows, int cols, int groups, int gate_first, float eps, int is_bf16,
@@ -200,10 +308,10 @@ PYBIND11_MODULE(_lmx_kernels, m) {
           "gated_norm");
   });
   // ---- K16 short causal convolution (conv.hip) ----
-  m.def("short_conv", [](uptr u, long u_ld, uptr w, uptr bias, uptr state, uptr tiles, int ntiles,
-                         int tile, uptr cu_q, uptr ctx, uptr slots, int C, int taps, uptr out,
+  m.def("short_conv", [](uptr u, long u_ld, uptr w, uptr in_bias, uptr bias, uptr state, uptr tiles,
+                         int ntiles, int tile, uptr cu_q, uptr ctx, uptr slots, int C, int taps, uptr out,
                          long out_ld, int act, int is_bf16, uptr stream) {
-    check(lmx::short_conv(P<void>(u), u_ld, P<float>(w), P<float>(bias), P<void>(state),
+    check(lmx::short_conv(P<void>(u), u_ld, P<float>(w), P<float>(in_bias), P<float>(bias), P<void>(state),
                           P<int>(tiles), ntiles, tile, P<int>(cu_q), P<int>(ctx), P<int>(slots), C,
                           taps, P<void>(out), out_ld, act, is_bf16, S(stream)),
           "short_conv");

@@ -163,6 +163,33 @@ template <typename T> __device__ __forceinline__ float sigmoid_t(float x) {
   else return 1.f / (1.f + __expf(-x));
 }
 
+// 16 B per lane from global memory into LDS (lane-linear from the wave-uniform
+// `lds`), counted by vmcnt
+typedef __attribute__((address_space(3))) void lmx_lds_t;
+__device__ __forceinline__ void lds_dma16(const void* g, void* lds) {
+  __builtin_amdgcn_global_load_lds(g, (lmx_lds_t*)lds, 16, 0, 0);
+}
+
+// every wave's LDS-DMA and LDS accesses so far are done, then a barrier; no
+// memory access moves across
+__device__ __forceinline__ void dma_barrier() {
+  asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_sched_barrier(0);
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_sched_barrier(0);
+  asm volatile("" ::: "memory");
+}
+
+// a barrier after which LDS writes of every wave are visible; LDS-DMA and
+// global loads stay in flight
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_sched_barrier(0);
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_sched_barrier(0);
+  asm volatile("" ::: "memory");
+}
+
 // XCD-aware bijective remap of a linear workgroup id (cdna guide §5, T1):
 // consecutive logical tiles land on the same XCD so neighbouring tiles share L2.
 __device__ __forceinline__ int xcd_remap(int orig, int nwg) {

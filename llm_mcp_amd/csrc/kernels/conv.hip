@@ -221,12 +221,13 @@ static bool conv_ok(const ConvArgs& a, int nseq) {
     default: F(__VA_ARGS__, 0);                \
   }
 
-int short_conv(const void* u, long u_ld, const float* w, const float* bias, void* state,
+int short_conv(const void* u, long u_ld, const float* w, const float* in_bias, const float* bias,
+               void* state,
                const int* tiles, int ntiles, int tile, const int* cu_q, const int* ctx,
                const int* slots, int C, int taps, void* out, long out_ld, int act, int is_bf16,
                hipStream_t stream) {
   if (ntiles <= 0) return 0;
-  const ConvArgs a{u, u_ld, w, nullptr, bias, state, tiles, cu_q, ctx, slots, C, taps, tile};
+  const ConvArgs a{u, u_ld, w, in_bias, bias, state, tiles, cu_q, ctx, slots, C, taps, tile};
   if (!conv_ok(a, ntiles)) return -1;
   const bool vec = C % 8 == 0 && u_ld % 8 == 0 && out_ld % 8 == 0 &&
                    (((uintptr_t)u | (uintptr_t)out | (uintptr_t)state) & 15) == 0;

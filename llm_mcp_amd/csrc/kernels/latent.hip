@@ -1,0 +1,525 @@
+// K20: latent attention with a sliding window (models.mixers
+// LatentAttentionMixer).  A token's cache page row is [latent c (Rp) | rotated
+// key part (xp)], one row for all heads.
+//
+//   rope_angles    cos | sin of the step's positions (reduced in double)
+//   latent_prep    projection rows -> RMS-normed query latents; normed c and
+//                  the rotated key part into the pages
+//   latent_rotate  the rotated part of the queries that score latents
+//   latent_rows    attention on latents (MFMA): a workgroup serves one query
+//                  row, its heads are the MFMA columns
+//   latent_any     the same for fp32 and for other sizes (fp32 arithmetic)
+#include "common.h"
+
+namespace lmx {
+namespace {
+
+constexpr int BS = 32;   // tokens per page
+constexpr float LOG2E = 1.4426950408889634f;
+
+__global__ void __launch_bounds__(256) rope_angles_kernel(const int* __restrict__ positions,
+                                                          const double* __restrict__ freqs, int T,
+                                                          int n, float* __restrict__ out) {
+  const int e = blockIdx.x * 256 + threadIdx.x;
+  if (e >= T * n) return;
+  const int t = e / n, i = e - t * n;
+  // the angle modulo one turn in double, then single precision
+  const double turns = (double)positions[t] * freqs[i] * 0.15915494309189535;
+  const float a = (float)((turns - floor(turns)) * 6.283185307179586);
+  out[(long)t * 2 * n + i] = cosf(a);
+  out[(long)t * 2 * n + n + i] = sinf(a);
+}
+
+// grid rows, block 256: waves 0-2 the query latent, wave 3 the cache row.
+// Gains are zero in the padding, so padded columns come out zero.
+template <typename T>
+__global__ void __launch_bounds__(256) latent_prep_kernel(
+    const T* __restrict__ p, long p_ld, int qr, int qp, const float* __restrict__ q_norm, int R,
+    int Rp, const float* __restrict__ c_norm, const float* __restrict__ ang, int d,
+    const int* __restrict__ slots, T* __restrict__ pages, int D, T* __restrict__ cq, float eps) {
+  __shared__ float part[3];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const long row = blockIdx.x;
+  const T* src = p + row * p_ld;
+  if (wave == 3) {
+    const int slot = slots[row];
+    const T* cs = src + qp;
+    float ss = 0.f;
+    for (int c = lane * 8; c < Rp; c += 512) {
+      float v[8];
+      ldv<8>(v, cs + c);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
+    }
+    const float inv = rsqrtf(wave_sum(ss) / (float)R + eps);
+    if (slot >= 0) {
+      T* dst = pages + (long)slot * D;
+      for (int c = lane * 8; c < Rp; c += 512) {
+        float v[8], g[8];
+        ldv<8>(v, cs + c);
+        ldv<8>(g, c_norm + c);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] *= inv * g[e];
+        stv<8>(dst + c, v);
+      }
+      const float* an = ang + row * d;
+      const T* ks = cs + Rp;
+      const int half = d / 2;
+      for (int j = lane; j < D - Rp; j += 64) {
+        const int i = j < half ? j : j - half;
+        float o = 0.f;
+        if (j < d) {
+          const float a = ld1(ks + i), b = ld1(ks + half + i), cv = an[i], sv = an[half + i];
+          o = j < half ? a * cv - b * sv : b * cv + a * sv;
+        }
+        st1(dst + Rp + j, o);
+      }
+    }
+  } else {
+    float ss = 0.f;
+    for (int c = tid * 8; c < qp; c += 192 * 8) {
+      float v[8];
+      ldv<8>(v, src + c);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
+    }
+    ss = wave_sum(ss);
+    if (lane == 0) part[wave] = ss;
+  }
+  __syncthreads();
+  if (wave == 3) return;
+  const float inv = rsqrtf((part[0] + part[1] + part[2]) / (float)qr + eps);
+  for (int c = tid * 8; c < qp; c += 192 * 8) {
+    float v[8], g[8];
+    ldv<8>(v, src + c);
+    ldv<8>(g, q_norm + c);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] *= inv * g[e];
+    stv<8>(cq + row * qp + c, v);
+  }
+}
+
+// grid rows, block 256
+template <typename T>
+__global__ void __launch_bounds__(256) latent_rotate_kernel(const T* __restrict__ q, long q_ld,
+                                                            int np, const float* __restrict__ ang,
+                                                            int d, int H, int xp,
+                                                            T* __restrict__ out, long o_ld, int Rp) {
+  const long row = blockIdx.x;
+  const float* an = ang + row * d;
+  const int half = d / 2;
+  for (int e = threadIdx.x; e < H * xp; e += 256) {
+    const int h = e / xp, j = e - h * xp;
+    const T* x = q + row * q_ld + (long)h * (np + xp) + np;
+    const int i = j < half ? j : j - half;
+    float o = 0.f;
+    if (j < d) {
+      const float a = ld1(x + i), b = ld1(x + half + i), cv = an[i], sv = an[half + i];
+      o = j < half ? a * cv - b * sv : b * cv + a * sv;
+    }
+    st1(out + row * o_ld + (long)h * (Rp + xp) + Rp + j, o);
+  }
+}
+
+// the sequence of a row (cu_q ascending)
+__device__ __forceinline__ int row_seq(const int* __restrict__ cu_q, int S, int row) {
+  int lo = 0, hi = S - 1;
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (cu_q[mid] <= row) lo = mid; else hi = mid - 1;
+  }
+  return lo;
+}
+
+// One wave per (row, head): a lane scores one key of a 64-key block, then owns
+// every 64th latent channel of the weighted sum.  grid (rows, ceil(H / 4)),
+// block 256, dynamic LDS 4 D floats.
+template <typename T, int ND>
+__global__ void __launch_bounds__(256) latent_any_kernel(
+    const T* __restrict__ q, const T* __restrict__ pages, const int* __restrict__ bt, int bt_stride,
+    const int* __restrict__ cu_q, int S, const int* __restrict__ positions, T* __restrict__ out,
+    int H, int Rp, int D, float scale, int window) {
+  extern __shared__ float sq_all[];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const long row = blockIdx.x;
+  const int h = blockIdx.y * 4 + wave;
+  float* sq = sq_all + wave * D;
+  const bool on = h < H;
+  if (on)
+    for (int d = lane; d < D; d += 64) sq[d] = ld1(q + (row * H + h) * D + d);
+  __syncthreads();
+  if (!on) return;
+  const int* tab = bt + (long)row_seq(cu_q, S, (int)row) * bt_stride;
+  const int p = positions[row], j0 = max(0, p - window + 1);
+  float m = -INFINITY, l = 0.f, acc[ND];
+#pragma unroll
+  for (int i = 0; i < ND; ++i) acc[i] = 0.f;
+  for (int k0 = j0; k0 <= p; k0 += 64) {
+    const int key = k0 + lane;
+    float s = -INFINITY;
+    if (key <= p) {
+      const T* kp = pages + ((long)tab[key / BS] * BS + key % BS) * D;
+      float t = 0.f;
+      for (int d = 0; d < D; d += 8) {
+        float x[8];
+        ldv<8>(x, kp + d);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) t += x[e] * sq[d + e];
+      }
+      s = t * scale;
+    }
+    const float mn = fmaxf(m, wave_max(s));
+    const float al = expf(m - mn), w = expf(s - mn);   // exp(-inf) = 0
+    l = l * al + wave_sum(w);
+    m = mn;
+#pragma unroll
+    for (int i = 0; i < ND; ++i) acc[i] *= al;
+    const int cnt = min(64, p + 1 - k0);
+    for (int j = 0; j < cnt; ++j) {
+      const float wj = __shfl(w, j, 64);
+      const int kj = k0 + j;
+      const T* vp = pages + ((long)tab[kj / BS] * BS + kj % BS) * D;
+#pragma unroll
+      for (int i = 0; i < ND; ++i)
+        if (i * 64 < Rp) acc[i] += wj * ld1(vp + i * 64 + lane);
+    }
+  }
+  const float inv = 1.f / l;
+#pragma unroll
+  for (int i = 0; i < ND; ++i)
+    if (i * 64 < Rp) st1(out + (row * H + h) * Rp + i * 64 + lane, acc[i] * inv);
+}
+
+// ------------------------------------------------------ attention on latents ----
+// grid (parts, head groups, rows), block 256.  Columns = NG x 16 heads of one
+// row.  Keys come in tiles of 64 (two pages) into a double buffer by LDS-DMA;
+// wave w scores keys 16 w .. 16 w + 15 of the tile (S^T: keys x heads), the
+// waves agree on the columns' maxima, write the weights as MFMA operands (a
+// bf16 pair, so they keep fp32 precision to 2^-17) and each sums its quarter
+// of the latent's channels, V^T read from the same key rows with the
+// transposing LDS read.
+constexpr int TK = 64;
+
+typedef short s16x4_t __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) s16x4_t lds_s16x4_t;
+
+// each 16-lane group: lane i points at 4 elements of row i / 4, columns
+// 4 (i % 4)..; it receives the 4 rows' elements of column i
+__device__ __forceinline__ s16x4_t lds_read_tr(const bf16_t* p) {
+  return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_t*)p);
+}
+
+template <int R>
+__device__ __forceinline__ int lat_swz(int row) {
+  constexpr int D8 = (R + 64) / 64;                   // 8-chunk groups per row
+  return (D8 & 1) ? (row >> 1) & 7 : row & 7;
+}
+
+__device__ __forceinline__ float xmax(float x) {      // over lanes c, c + 16, c + 32, c + 48
+  x = fmaxf(x, __shfl_xor(x, 16, 64));
+  return fmaxf(x, __shfl_xor(x, 32, 64));
+}
+__device__ __forceinline__ float xsum(float x) {
+  x += __shfl_xor(x, 16, 64);
+  return x + __shfl_xor(x, 32, 64);
+}
+
+template <int R, int NG>
+__global__ void __launch_bounds__(256, 1) latent_rows_kernel(
+    const bf16_t* __restrict__ q, const bf16_t* __restrict__ pages, const int* __restrict__ bt,
+    int bt_stride, const int* __restrict__ cu_q, int S, const int* __restrict__ positions,
+    int num_decode, bf16_t* __restrict__ out, float* __restrict__ part_o,
+    float* __restrict__ part_ml, int H, float scale, int window, int part_keys, int max_parts) {
+  constexpr int D = R + 64, KS = D / 32, CH = D / 8;
+  constexpr int DT = R / 64;                          // 16-channel tiles per wave
+  extern __shared__ __attribute__((aligned(16))) char lt_smem[];
+  bf16_t* const kt = reinterpret_cast<bf16_t*>(lt_smem);              // [2][TK][D]
+  bf16_t* const pw = kt + 2 * TK * D;                                 // [hi, lo][2 k steps][NG][64 x 8]
+  float* const smax = reinterpret_cast<float*>(pw + 2 * 2 * NG * 512);  // [4][NG 16]
+  const int tid = threadIdx.x, lane = tid & 63, c = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const long row = blockIdx.z;
+  const int part = blockIdx.x, h0 = blockIdx.y * NG * 16;
+  const int pos = positions[row];
+  const int lo = max(0, pos - window + 1);
+  // the row's visible keys in parts of whole tiles
+  const int base = lo / TK * TK, span = pos + 1 - base;
+  int pk = max(part_keys, (span + max_parts - 1) / max_parts);
+  pk = (pk + TK - 1) / TK * TK;
+  const int nparts = (span + pk - 1) / pk;
+  if (part >= nparts) return;
+  const int b0 = base + part * pk, b1 = min(b0 + pk, pos + 1);
+  const int seq = row < num_decode ? (int)row : row_seq(cu_q, S, (int)row);
+  const int* tab = bt + (long)seq * bt_stride;
+  const int last_page = pos / BS;
+
+  auto stage = [&](int t0, int buf) {
+#pragma unroll
+    for (int i = 0; i < TK * CH / 256; ++i) {
+      const int e = i * 256 + tid, r = e / CH, ch = e % CH;
+      const int pg = min((t0 + r) / BS, last_page);
+      lds_dma16(pages + ((long)tab[pg] * BS + (r % BS)) * D + 8 * (ch ^ lat_swz<R>(r)),
+                kt + buf * TK * D + (i * 256 + wave * 64) * 8);
+    }
+  };
+  static_assert(TK * CH % 256 == 0, "a tile is whole DMA instructions");
+
+  bf16x8_t qf[NG][KS];
+#pragma unroll
+  for (int n = 0; n < NG; ++n) {
+    const int h = min(h0 + 16 * n + c, H - 1);
+#pragma unroll
+    for (int s = 0; s < KS; ++s) qf[n][s] = load_frag16B(q + (row * H + h) * D + 32 * s + 8 * g);
+  }
+  float m[NG], l[NG];
+  f32x4_t acc[NG][DT];
+#pragma unroll
+  for (int n = 0; n < NG; ++n) {
+    m[n] = -INFINITY;
+    l[n] = 0.f;
+#pragma unroll
+    for (int i = 0; i < DT; ++i) acc[n][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
+  const float sl = scale * LOG2E;
+  stage(b0, 0);
+  int buf = 0;
+  for (int t0 = b0; t0 < b1; t0 += TK, buf ^= 1) {
+    dma_barrier();                    // the tile landed; every wave is done with the other buffer
+    if (t0 + TK < b1) stage(t0 + TK, buf ^ 1);
+    const bf16_t* tile = kt + buf * TK * D;
+    f32x4_t s[NG];
+#pragma unroll
+    for (int n = 0; n < NG; ++n) s[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    {
+      const int r = 16 * wave + c;
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const bf16x8_t kf = load_frag16B(tile + r * D + 8 * ((4 * ks + g) ^ lat_swz<R>(r)));
+#pragma unroll
+        for (int n = 0; n < NG; ++n) s[n] = mfma16(kf, qf[n][ks], s[n]);
+      }
+    }
+    float x[NG][4];
+#pragma unroll
+    for (int n = 0; n < NG; ++n) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = t0 + 16 * wave + 4 * g + r;
+        x[n][r] = key >= lo && key < b1 ? s[n][r] * sl : -INFINITY;
+      }
+      const float mx = xmax(fmaxf(fmaxf(x[n][0], x[n][1]), fmaxf(x[n][2], x[n][3])));
+      if (g == 0) smax[wave * NG * 16 + 16 * n + c] = mx;
+    }
+    lds_barrier();
+#pragma unroll
+    for (int n = 0; n < NG; ++n) {
+      float mx = m[n];
+#pragma unroll
+      for (int w = 0; w < 4; ++w) mx = fmaxf(mx, smax[w * NG * 16 + 16 * n + c]);
+      const float mu = mx == -INFINITY ? 0.f : mx;
+      const float al = fast_exp2(m[n] - mu);
+      m[n] = mx;
+      float ps = 0.f;
+      bf16x4_t hi, lw;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float p = fast_exp2(x[n][r] - mu);
+        ps += p;
+        const uint16_t hb = f2bf(p);
+        hi[r] = (short)hb;
+        lw[r] = (short)f2bf(p - bf2f(hb));
+      }
+      l[n] = l[n] * al + ps;          // this lane's keys only; summed at the end
+      // k step wave / 2, lane group g: element 4 (wave & 1) + r
+      bf16_t* dst = pw + (((wave >> 1) * NG + n) * 64 + lane) * 8 + 4 * (wave & 1);
+      *reinterpret_cast<bf16x4_t*>(dst) = hi;
+      *reinterpret_cast<bf16x4_t*>(dst + 2 * NG * 512) = lw;
+#pragma unroll
+      for (int i = 0; i < DT; ++i) acc[n][i] *= al;
+    }
+    lds_barrier();
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+      bf16x8_t ph[NG], pl[NG];
+#pragma unroll
+      for (int n = 0; n < NG; ++n) {
+        const bf16_t* src = pw + ((ks * NG + n) * 64 + lane) * 8;
+        ph[n] = load_frag16B(src);
+        pl[n] = load_frag16B(src + 2 * NG * 512);
+      }
+      // V^T of keys 32 ks + 4 g + .. and 32 ks + 16 + 4 g + ..: row r, channel chunk
+      const int ra = 32 * ks + 4 * g + (c >> 2), rb = ra + 16;
+#pragma unroll
+      for (int i = 0; i < DT; ++i) {
+        const int d0 = (wave * DT + i) * 16 + 4 * (c & 3);
+        const s16x4_t va = lds_read_tr(tile + ra * D + 8 * ((d0 >> 3) ^ lat_swz<R>(ra)) + (d0 & 7));
+        const s16x4_t vb = lds_read_tr(tile + rb * D + 8 * ((d0 >> 3) ^ lat_swz<R>(rb)) + (d0 & 7));
+        const bf16x8_t vf = {va[0], va[1], va[2], va[3], vb[0], vb[1], vb[2], vb[3]};
+#pragma unroll
+        for (int n = 0; n < NG; ++n) {
+          acc[n][i] = mfma16(vf, ph[n], acc[n][i]);
+          acc[n][i] = mfma16(vf, pl[n], acc[n][i]);
+        }
+      }
+    }
+  }
+  // denominators over the waves
+#pragma unroll
+  for (int n = 0; n < NG; ++n) l[n] = xsum(l[n]);
+  lds_barrier();                      // smax is free
+  if (g == 0)
+#pragma unroll
+    for (int n = 0; n < NG; ++n) smax[wave * NG * 16 + 16 * n + c] = l[n];
+  lds_barrier();
+#pragma unroll
+  for (int n = 0; n < NG; ++n) {
+    const int h = h0 + 16 * n + c;
+    if (h >= H) continue;
+    float L = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) L += smax[w * NG * 16 + 16 * n + c];
+    if (nparts == 1) {
+      const float inv = 1.f / L;
+#pragma unroll
+      for (int i = 0; i < DT; ++i) {
+        bf16x4_t o;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[n][i][r] * inv);
+        *reinterpret_cast<bf16x4_t*>(out + (row * H + h) * R + (wave * DT + i) * 16 + 4 * g) = o;
+      }
+    } else {
+      const long idx = (row * H + h) * max_parts + part;
+#pragma unroll
+      for (int i = 0; i < DT; ++i)
+        *reinterpret_cast<f32x4_t*>(part_o + idx * R + (wave * DT + i) * 16 + 4 * g) = acc[n][i];
+      if (wave == 0 && g == 0) { part_ml[2 * idx] = m[n]; part_ml[2 * idx + 1] = L; }
+    }
+  }
+}
+
+// grid (H, rows), block 64: combine the parts of a row
+__global__ void __launch_bounds__(64) latent_reduce_kernel(
+    const float* __restrict__ part_o, const float* __restrict__ part_ml,
+    const int* __restrict__ positions, bf16_t* __restrict__ out, int H, int R, int window,
+    int part_keys, int max_parts) {
+  const long row = blockIdx.y, h = blockIdx.x;
+  const int pos = positions[row], base = max(0, pos - window + 1) / TK * TK, span = pos + 1 - base;
+  int pk = max(part_keys, (span + max_parts - 1) / max_parts);
+  pk = (pk + TK - 1) / TK * TK;
+  const int nparts = (span + pk - 1) / pk;
+  if (nparts == 1) return;
+  const long idx = (row * H + h) * max_parts;
+  float M = -INFINITY;
+  for (int p = 0; p < nparts; ++p) M = fmaxf(M, part_ml[2 * (idx + p)]);
+  for (int d = threadIdx.x * 4; d < R; d += 256) {
+    float L = 0.f;
+    f32x4_t o = {0.f, 0.f, 0.f, 0.f};
+    for (int p = 0; p < nparts; ++p) {
+      const float mp = part_ml[2 * (idx + p)], f = mp == -INFINITY ? 0.f : fast_exp2(mp - M);
+      L += f * part_ml[2 * (idx + p) + 1];
+      o += f * *reinterpret_cast<const f32x4_t*>(part_o + (idx + p) * R + d);
+    }
+    bf16x4_t r;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) r[e] = (short)f2bf(o[e] / L);
+    *reinterpret_cast<bf16x4_t*>(out + (row * H + h) * R + d) = r;
+  }
+}
+
+}  // namespace
+
+int rope_angles(const int* positions, const double* freqs, int T, int n, float* out,
+                hipStream_t stream) {
+  if (T <= 0 || n <= 0) return 0;
+  rope_angles_kernel<<<dim3((T * n + 255) / 256), dim3(256), 0, stream>>>(positions, freqs, T, n, out);
+  return (int)hipGetLastError();
+}
+
+int latent_prep(const void* p, long p_ld, int T, int qr, int qp, const float* q_norm, int R, int Rp,
+                const float* c_norm, const float* ang, int d, const int* slots, void* pages,
+                int block_size, int D, void* cq, float eps, int is_bf16, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (block_size != BS || qp % 8 || Rp % 8 || D % 8 || qr < 1 || qr > qp || R < 1 || R > Rp ||
+      d < 2 || d % 2 || d > D - Rp || p_ld % 8)
+    return -1;
+  if (is_bf16)
+    latent_prep_kernel<bf16_t><<<dim3(T), dim3(256), 0, stream>>>(
+        (const bf16_t*)p, p_ld, qr, qp, q_norm, R, Rp, c_norm, ang, d, slots, (bf16_t*)pages, D,
+        (bf16_t*)cq, eps);
+  else
+    latent_prep_kernel<float><<<dim3(T), dim3(256), 0, stream>>>(
+        (const float*)p, p_ld, qr, qp, q_norm, R, Rp, c_norm, ang, d, slots, (float*)pages, D,
+        (float*)cq, eps);
+  return (int)hipGetLastError();
+}
+
+int latent_rotate(const void* q, long q_ld, int np, const float* ang, int d, int T, int H, int xp,
+                  void* out, long o_ld, int Rp, int is_bf16, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (d < 2 || d % 2 || d > xp || H < 1) return -1;
+  if (is_bf16)
+    latent_rotate_kernel<bf16_t><<<dim3(T), dim3(256), 0, stream>>>(
+        (const bf16_t*)q, q_ld, np, ang, d, H, xp, (bf16_t*)out, o_ld, Rp);
+  else
+    latent_rotate_kernel<float><<<dim3(T), dim3(256), 0, stream>>>(
+        (const float*)q, q_ld, np, ang, d, H, xp, (float*)out, o_ld, Rp);
+  return (int)hipGetLastError();
+}
+
+int latent_any(const void* q, const void* pages, const int* bt, int bt_stride, const int* cu_q,
+               int S, const int* positions, int rows, void* out, int H, int Rp, int D, float scale,
+               int window, int is_bf16, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (S < 1 || H < 1 || Rp % 64 || D % 8 || Rp >= D || window < 1 || D > 4096) return -1;
+  const dim3 grid(rows, (H + 3) / 4);
+  const size_t smem = 4 * D * sizeof(float);
+#define LMX_LA(T, ND)                                                                          \
+  latent_any_kernel<T, ND><<<grid, dim3(256), smem, stream>>>(                                 \
+      (const T*)q, (const T*)pages, bt, bt_stride, cu_q, S, positions, (T*)out, H, Rp, D,      \
+      scale, window)
+#define LMX_LAN(T)                                                                             \
+  if (Rp <= 128) LMX_LA(T, 2); else if (Rp <= 256) LMX_LA(T, 4);                               \
+  else if (Rp <= 512) LMX_LA(T, 8); else if (Rp <= 1024) LMX_LA(T, 16); else return -2;
+  if (is_bf16) { LMX_LAN(bf16_t) } else { LMX_LAN(float) }
+#undef LMX_LAN
+#undef LMX_LA
+  return (int)hipGetLastError();
+}
+
+// rows before num_decode: row i is sequence i's first row.  part_o / part_ml:
+// [rows][H][max_parts][Rp] / [..][2] (max_parts > 1)
+int latent_rows(const void* q, const void* pages, const int* bt, int bt_stride, const int* cu_q,
+                int S, const int* positions, int rows, int num_decode, void* out, float* part_o,
+                float* part_ml, int H, int Rp, int D, float scale, int window, int part_keys,
+                int max_parts, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (S < 1 || H < 1 || window < 1 || D != Rp + 64 || part_keys < TK || max_parts < 1 ||
+      (max_parts > 1 && (!part_o || !part_ml)) || rows > 65535)
+    return -1;
+#define LMX_LR(R, NG)                                                                          \
+  {                                                                                            \
+    constexpr int smem = 2 * TK * (R + 64) * 2 + 2 * 2 * NG * 512 * 2 + 4 * NG * 16 * 4;       \
+    static bool attr = false;                                                                  \
+    if (smem > 65536 && !attr) {                                                               \
+      (void)hipFuncSetAttribute((const void*)latent_rows_kernel<R, NG>,                        \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, smem);             \
+      attr = true;                                                                             \
+    }                                                                                          \
+    latent_rows_kernel<R, NG>                                                                  \
+        <<<dim3(max_parts, (H + 16 * NG - 1) / (16 * NG), rows), dim3(256), smem, stream>>>(   \
+            (const bf16_t*)q, (const bf16_t*)pages, bt, bt_stride, cu_q, S, positions,         \
+            num_decode, (bf16_t*)out, part_o, part_ml, H, scale, window, part_keys, max_parts); \
+  }
+#define LMX_LRN(R) if (H <= 16) LMX_LR(R, 1) else LMX_LR(R, 2)
+  if (Rp == 64) { LMX_LRN(64) } else if (Rp == 128) { LMX_LRN(128) }
+  else if (Rp == 256) { LMX_LRN(256) } else if (Rp == 512) { LMX_LRN(512) }
+  else return -2;
+#undef LMX_LRN
+#undef LMX_LR
+  if (max_parts > 1)
+    latent_reduce_kernel<<<dim3(H, rows), dim3(64), 0, stream>>>(
+        part_o, part_ml, positions, (bf16_t*)out, H, Rp, window, part_keys, max_parts);
+  return (int)hipGetLastError();
+}
+
+}  // namespace lmx

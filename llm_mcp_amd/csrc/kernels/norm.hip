@@ -348,13 +348,14 @@ int layernorm(void* out, const void* x, const void* residual, const void* w, con
 // Sandwich norm: the norm after a sublayer, the residual add and the norm
 // before the next sublayer in one pass, over an fp32 residual stream.
 //
-//   r   = ids ? table[ids[row]] : residual[row]
+//   r   = ids ? scale * table[ids[row]] : residual[row]
 //   r  += norm(y[row]) * w_post              (y: the sublayer's output; optional)
-//   out = norm(r) * w_pre                    (optional)
+//   out = w_pre ? norm(r) * w_pre : r
 //
 // norm(x) = x / sqrt(mean(x^2) + eps); the gains are fp32 (a weight stored
-// around zero arrives as 1 + w).  y is T rows, or S fp32 split-K slabs
-// [S][rows][cols] summed here.  rows_idx (optional): out row i is source row
+// around zero arrives as 1 + w, a constant on what is added is part of w_post).
+// y is T rows, S fp32 split-K slabs [S][rows][cols] summed here, or a mixture
+// sum_j mix_w[row][j] y[mix_pos[row][j]] of T rows.  rows_idx (optional): out row i is source row
 // rows_idx[i] and the residual is left as it is (the final norm of the sampled
 // rows); otherwise the residual row is written when it changed.
 struct SandwichArgs {
@@ -363,8 +364,12 @@ struct SandwichArgs {
   const void* y;
   long y_ld, slab_stride;
   int slabs;                  // 0: y is T rows
+  const int* mix_pos;         // [rows][mix_n] or null
+  const float* mix_w;
+  int mix_n;
   const int* ids;
   const void* table;
+  float scale;
   const float *w_post, *w_pre;
   const long* rows_idx;
   int cols;
@@ -383,8 +388,13 @@ __global__ void __launch_bounds__(512) sandwich_norm_kernel(SandwichArgs a) {
   for (int i = 0; i < VPT; ++i) {
     const int c = threadIdx.x + i * blockDim.x;
     if (c >= nchunk) continue;
-    if (a.ids) ldv<V>(r[i], (const T*)a.table + (long)a.ids[src] * cols + c * V);
-    else ldv<V>(r[i], rr + c * V);
+    if (a.ids) {
+      ldv<V>(r[i], (const T*)a.table + (long)a.ids[src] * cols + c * V);
+#pragma unroll
+      for (int e = 0; e < V; ++e) r[i][e] *= a.scale;
+    } else {
+      ldv<V>(r[i], rr + c * V);
+    }
     if (a.y) {
       if (a.slabs) {
         const float* p = (const float*)a.y + src * cols + c * V;
@@ -394,6 +404,17 @@ __global__ void __launch_bounds__(512) sandwich_norm_kernel(SandwichArgs a) {
           ldv<V>(t, p + s * a.slab_stride);
 #pragma unroll
           for (int e = 0; e < V; ++e) y[i][e] += t[e];
+        }
+      } else if (a.mix_pos) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[i][e] = 0.f;
+#pragma unroll 4
+        for (int j = 0; j < a.mix_n; ++j) {
+          float t[V];
+          ldv<V>(t, (const T*)a.y + (long)a.mix_pos[src * a.mix_n + j] * a.y_ld + c * V);
+          const float w = a.mix_w[src * a.mix_n + j];
+#pragma unroll
+          for (int e = 0; e < V; ++e) y[i][e] += w * t[e];
         }
       } else {
         ldv<V>(y[i], (const T*)a.y + src * a.y_ld + c * V);
@@ -422,7 +443,14 @@ __global__ void __launch_bounds__(512) sandwich_norm_kernel(SandwichArgs a) {
       if (c < nchunk) stv<V>(rr + c * V, r[i]);
     }
   }
-  if (!a.w_pre) return;
+  if (!a.w_pre) {
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c < nchunk) stv<V>((T*)a.out + (long)blockIdx.x * cols + c * V, r[i]);
+    }
+    return;
+  }
   ss = 0.f;
 #pragma unroll
   for (int i = 0; i < VPT; ++i) {
@@ -446,13 +474,15 @@ __global__ void __launch_bounds__(512) sandwich_norm_kernel(SandwichArgs a) {
 }
 
 int sandwich_norm(void* out, float* residual, const void* y, long y_ld, int slabs, long slab_stride,
-                  const int* ids, const void* table, const float* w_post, const float* w_pre,
+                  const int* mix_pos, const float* mix_w, int mix_n, const int* ids,
+                  const void* table, float scale, const float* w_post, const float* w_pre,
                   const long* rows_idx, int rows, int cols, float eps, int is_bf16,
                   hipStream_t stream) {
   if (rows <= 0) return 0;
-  if (cols <= 0 || !residual || (y && !w_post) || (w_pre && !out)) return -1;
-  const SandwichArgs a{out, residual, y, y_ld, slab_stride, slabs, ids, table,
-                       w_post, w_pre, rows_idx, cols, eps};
+  if (cols <= 0 || !residual || !out || (y && !w_post) || (mix_pos && (!y || !mix_w || slabs)))
+    return -1;
+  const SandwichArgs a{out, residual, y, y_ld, slab_stride, slabs, mix_pos, mix_w, mix_n, ids,
+                       table, scale, w_post, w_pre, rows_idx, cols, eps};
   const bool vec = cols % 8 == 0 && y_ld % 8 == 0;
   const int nchunk = vec ? cols / 8 : cols;
   const int vpt = (nchunk + 511) / 512;

@@ -308,7 +308,7 @@ class LLMEngine:
         cap = 4 * (4 * T + ecfg.max_num_seqs * (self.max_blocks + 8) + 2 * T) + 16 * 64 + \
             8 * ecfg.max_num_seqs * 4 + 4 * ecfg.max_num_seqs * (PEN_WINDOW + 4) + \
             4 * ecfg.max_num_seqs + 16          # decode dispatch order
-        if self.states:      # state slots and the model's host plan
+        if self.model.needs_plan:      # state slots and the model's host plan
             cap += 4 * (3 * ecfg.max_num_seqs) + 64 * (T + 16 * ecfg.max_num_seqs)
         self.packer = _Packer(cap, self.device)
         self.event_sink = event_sink
@@ -410,10 +410,11 @@ class LLMEngine:
                      sum(t[0].numel() * t.element_size() for t in self.states) / 1e6)
 
     def _alloc_kv(self):
-        layers = self.model.kv_layers            # (kv heads, head size) per cache layer
+        layers = self.model.kv_layers            # (kv heads, key size, value size) per cache layer
         es = torch.empty((), dtype=self.model.dtype).element_size()
-        sizes = [Hkv * BLOCK_SIZE * D for Hkv, D in layers]     # elements per page of K (or V)
-        per_block = max(1, 2 * sum(sizes) * es)
+        # elements per page of keys and of values (0: the key rows hold both)
+        sizes = [(Hkv * BLOCK_SIZE * Dk, Hkv * BLOCK_SIZE * Dv) for Hkv, Dk, Dv in layers]
+        per_block = max(1, sum(k + v for k, v in sizes) * es)
         if self.ecfg.kv_cache_tokens is not None:
             kv_bytes = -(-self.ecfg.kv_cache_tokens // BLOCK_SIZE) * per_block
         elif self.ecfg.kv_cache_gb is not None:
@@ -439,13 +440,15 @@ class LLMEngine:
             self.num_blocks = int(t.item())
         # zero-filled: masked keys multiply P = 0 with V, which must be finite
         NB = self.num_blocks
-        self.kv = torch.zeros(2 * NB * sum(sizes), dtype=self.model.dtype, device=self.device)
+        self.kv = torch.zeros(NB * sum(k + v for k, v in sizes), dtype=self.model.dtype,
+                              device=self.device)
         self.k_caches, self.v_caches, off = [], [], 0
-        for (Hkv, D), n in zip(layers, sizes):
-            self.k_caches.append(self.kv[off:off + NB * n].view(NB, Hkv, BLOCK_SIZE, D))
-            off += NB * n
-            self.v_caches.append(self.kv[off:off + NB * n].view(NB, Hkv, BLOCK_SIZE // 4, D, 4))
-            off += NB * n
+        for (Hkv, Dk, Dv), (nk, nv) in zip(layers, sizes):
+            self.k_caches.append(self.kv[off:off + NB * nk].view(NB, Hkv, BLOCK_SIZE, Dk))
+            off += NB * nk
+            self.v_caches.append(self.kv[off:off + NB * nv].view(NB, Hkv, BLOCK_SIZE // 4, Dv, 4)
+                                 if nv else None)
+            off += NB * nv
         log.info("KV cache: %d blocks x %d tokens (%.1f GB)", NB, BLOCK_SIZE,
                  self.kv.numel() * es / 1e9)
 
@@ -1082,7 +1085,7 @@ class LLMEngine:
         if nd > 1:
             items.append(("order", ops.decode_order(plan["context_lens"][:nd])))
         host = None
-        if self.states:
+        if self.model.needs_plan:
             more, host = self.model.host_plan(plan)
             items += [("sslots", plan["state_slots"])] + more
         d = self.packer.pack(items + list(extra))
@@ -1090,7 +1093,7 @@ class LLMEngine:
         inp = StepInputs(d["ids"], d["pos"], d["slots"], nd, d["bt"], d["ctx"],
                          d["cu"], d["tiles"], d["rows"], T, S, decode_order=d.get("order"),
                          host={"cu_q": plan["cu_q"], "tiles": plan["prefill_tiles"], "rows": rows})
-        if self.states:
+        if self.model.needs_plan:
             inp.state_slots, inp.states = d["sslots"], self.states
             inp.aux = self.model.bind_plan(d, host)
         ws = self._decode_ws(nd) if nd else self.decode_ws
@@ -1132,7 +1135,7 @@ class LLMEngine:
             a = h[k]
             a[:n] = plan[_PLAN_KEY.get(k, k)]
             a[n:B] = fill
-        if self.states:
+        if self.model.needs_plan:
             h["sslots"][:n] = plan["state_slots"]
             h["sslots"][n:B] = -1
         src = plan.get("input_src")

@@ -144,24 +144,25 @@ class BertConfig:
 
 
 @dataclass
-class ZegopelConfig:
-    """Zegopel: a decoder whose layers each name their own token mixer
-    (``lightning`` linear attention, ``mamba2`` state-space, or ``attention``
-    with short convolutions) and feed-forward, with their own sizes.
-
-    ``layers`` holds one dict per layer, as in the checkpoint's config.json:
-    ``{"type": ..., "mixer": {sizes and constants}, "mlp": {"kind", "ff"} | None}``."""
-    name: str = "zegopel"
+class LayerListConfig:
+    """A decoder whose layers each name their own token mixer and feed-forward,
+    with their own sizes.  ``layers`` holds one dict per layer, as in the
+    checkpoint's config.json: ``{"type": ..., "mixer": {sizes and constants},
+    "mlp": {"kind", ...} | None, "weights_of": layer (optional)}``."""
+    name: str = ""
     vocab_size: int = 512
     hidden_size: int = 256
     layers: list = field(default_factory=list)
     rms_eps: float = 1e-5
-    # positions enter only through the query temperature: no table bounds them
+    # no table bounds the positions
     max_position: int = 1 << 20
     bos_token_id: int | None = None
     eos_token_ids: tuple = ()
-    family: str = "zegopel"
+    family: str = ""
     kind: str = "chat"
+    architecture: str = ""          # config.json's name of the family
+    embed_scale: float = 1.0        # the embedding's rows are multiplied by it
+    residual_mult: float = 1.0      # and so is what a sublayer adds
 
     @property
     def num_layers(self) -> int:
@@ -169,8 +170,8 @@ class ZegopelConfig:
 
     @property
     def params(self) -> int:
-        from .zegopel import tensor_shapes
-        return sum(math.prod(s) for s in tensor_shapes(self).values())
+        from .registry import model_class
+        return sum(math.prod(s) for s in model_class(self).tensor_shapes(self).values())
 
     @property
     def params_b(self) -> float:
@@ -182,6 +183,58 @@ class ZegopelConfig:
 
     def to_dict(self) -> dict:
         return asdict(self)
+
+    def to_json(self) -> dict:
+        """The checkpoint's config.json."""
+        js = {"architecture": self.architecture, "layers": self.layers,
+              "norm": {"eps": self.rms_eps}, "vocab": self.vocab_size, "width": self.hidden_size}
+        if self.eos_token_ids:
+            js["eos_token_id"] = list(self.eos_token_ids)
+        if self.bos_token_id is not None:
+            js["bos_token_id"] = self.bos_token_id
+        return js
+
+    @classmethod
+    def from_json(cls, js: dict, name: str):
+        from .registry import layer_list_class
+        layer_list_class(cls.family).check_layers(js["layers"])
+        eos = js.get("eos_token_id", ())
+        return cls(name=name, vocab_size=js["vocab"], hidden_size=js["width"],
+                   layers=js["layers"], rms_eps=js["norm"]["eps"],
+                   bos_token_id=js.get("bos_token_id"),
+                   eos_token_ids=tuple(eos) if isinstance(eos, (list, tuple)) else (eos,))
+
+
+@dataclass
+class ZegopelConfig(LayerListConfig):
+    """``lightning`` linear attention, ``mamba2`` state-space and ``attention``
+    with short convolutions."""
+    name: str = "zegopel"
+    family: str = "zegopel"
+    architecture: str = "Zegopel"
+
+
+@dataclass
+class PikesunConfig(LayerListConfig):
+    """``rglru`` gated linear recurrences and ``latent_attention``, dense and
+    ``moe`` feed-forwards."""
+    name: str = "pikesun"
+    family: str = "pikesun"
+    architecture: str = "Pikesun"
+
+    def to_json(self) -> dict:
+        return {**super().to_json(), "embedding": {"scale": self.embed_scale},
+                "residual_mult": self.residual_mult}
+
+    @classmethod
+    def from_json(cls, js: dict, name: str):
+        cfg = super().from_json(js, name)
+        cfg.embed_scale = float(js["embedding"]["scale"])
+        cfg.residual_mult = float(js["residual_mult"])
+        return cfg
+
+
+LAYER_LISTS = {c.architecture: c for c in (ZegopelConfig, PikesunConfig)}
 
 
 def zegopel_stack(pattern: str, ff: int, lightning: dict, mamba2: dict,
@@ -219,6 +272,45 @@ def _zegopel_8b() -> ZegopelConfig:
             dict(heads=64, vdim=128, state=128, groups=8, conv=4, norm_groups=8),
             dict(heads=32, kv_heads=8, dim=128, vdim=128, conv=4, scale=128 ** -0.5,
                  q_temp=dict(coef=0.1, every=8192))))
+
+
+def pikesun_stack(pattern: str, rglru: dict, latent: dict, dense: dict, moe: dict) -> list:
+    """Layer list from a pattern of R (rglru), A (latent attention): the first
+    layer's feed-forward is dense, the others' mixtures of experts."""
+    kinds = {"R": ("rglru", rglru), "A": ("latent_attention", latent)}
+    return [{"type": kinds[c][0], "mixer": dict(kinds[c][1]),
+             "mlp": dict(moe if i else dense)} for i, c in enumerate(pattern)]
+
+
+def _latent(heads: int, dim: int, rot: int, vdim: int, rank: int, q_rank: int, window: int,
+            base: float = 10000.0) -> dict:
+    return dict(heads=heads, dim=dim, rot_dim=rot, vdim=vdim, kv_rank=rank, q_rank=q_rank,
+                scale=(dim + rot) ** -0.5, mask=dict(size=window), rot=dict(base=base, dims=rot))
+
+
+def _moe(experts: int, top: int, ff: int, shared: int, limit: float = 7.0) -> dict:
+    return dict(kind="moe", router=dict(experts=experts, top=top),
+                expert=dict(ff=ff, limit=limit), shared=dict(ff=shared, limit=limit))
+
+
+def _pikesun_tiny() -> PikesunConfig:
+    layers = pikesun_stack("RARA", dict(width=192, blocks=3, conv=4),
+                           _latent(4, 48, 32, 40, 96, 64, 70), dict(kind="dense", ff=256),
+                           _moe(8, 2, 64, 96))
+    return PikesunConfig(name="tiny-pikesun", vocab_size=512, hidden_size=192, bos_token_id=506,
+                         eos_token_ids=(510,), layers=layers, embed_scale=192 ** 0.5,
+                         residual_mult=0.5)
+
+
+def _pikesun_8b() -> PikesunConfig:
+    """Llama-3-8B's width and size, all experts counted (random weights:
+    benchmarks)."""
+    layers = pikesun_stack("RRA" * 8, dict(width=4096, blocks=16, conv=4),
+                           _latent(32, 128, 64, 128, 512, 1536, 2048),
+                           dict(kind="dense", ff=14336), _moe(16, 4, 1024, 2048))
+    return PikesunConfig(name="pikesun-8b", vocab_size=128256, hidden_size=4096,
+                         bos_token_id=128000, eos_token_ids=(128001, 128009), layers=layers,
+                         embed_scale=64.0, residual_mult=0.5)
 
 
 _LLAMA32_ROPE = {"rope_type": "llama3", "factor": 32.0, "low_freq_factor": 1.0,
@@ -314,6 +406,8 @@ PRESETS: dict[str, object] = {
                                  embed_dim=256, max_position=256, pooling="mean"),
     "tiny-zegopel": _zegopel_tiny(),
     "zegopel-8b": _zegopel_8b(),
+    "tiny-pikesun": _pikesun_tiny(),
+    "pikesun-8b": _pikesun_8b(),
     "tiny-nomic": NomicBertConfig(name="tiny-nomic", vocab_size=512, hidden_size=256,
                                   intermediate_size=512, num_layers=2, num_heads=2, head_dim=128,
                                   embed_dim=256, max_position=2048),
@@ -354,7 +448,7 @@ def resolve(name: str):
         n = int(layers)
         if n < 1 or n > cfg.num_layers:
             raise KeyError(f"{name!r}: layer count must be 1..{cfg.num_layers}")
-        if isinstance(cfg, ZegopelConfig):
+        if isinstance(cfg, LayerListConfig):
             return dataclasses.replace(cfg, name=name, layers=cfg.layers[:n])
         cfg = dataclasses.replace(cfg, name=name, num_layers=n)
     return cfg
@@ -364,24 +458,12 @@ def is_checkpoint_dir(name: str) -> bool:
     return (Path(name) / "config.json").is_file()
 
 
-def _zegopel_from_json(cfg: dict, name: str) -> ZegopelConfig:
-    for i, L in enumerate(cfg["layers"]):
-        if L["type"] not in ("lightning", "mamba2", "attention"):
-            raise ValueError(f"layer {i}: unknown mixer {L['type']!r}")
-        if L.get("mlp") is not None and L["mlp"].get("kind") != "dense":
-            raise ValueError(f"layer {i}: unknown feed-forward {L['mlp'].get('kind')!r}")
-    eos = cfg.get("eos_token_id", ())
-    return ZegopelConfig(
-        name=name, vocab_size=cfg["vocab"], hidden_size=cfg["width"], layers=cfg["layers"],
-        rms_eps=cfg["norm"]["eps"], bos_token_id=cfg.get("bos_token_id"),
-        eos_token_ids=tuple(eos) if isinstance(eos, (list, tuple)) else (eos,))
-
-
 def from_hf_config(path: str | Path):
     """Build a config from a HF config.json (local file; no network)."""
     cfg = json.loads(Path(path).read_text())
-    if cfg.get("architecture") == "Zegopel":
-        return _zegopel_from_json(cfg, Path(path).resolve().parent.name)
+    family = LAYER_LISTS.get(cfg.get("architecture"))
+    if family is not None:
+        return family.from_json(cfg, Path(path).resolve().parent.name)
     arch = (cfg.get("architectures") or [""])[0]
     if "Llama" in arch or "Qwen2" in arch or "Qwen3" in arch or "Mistral" in arch:
         qwen = "Qwen2" in arch

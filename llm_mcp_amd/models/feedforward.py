@@ -1,0 +1,105 @@
+"""Feed-forwards of layer-list decoders (``models.layerlist``).
+
+Same protocol as the mixers: ``shapes`` (checkpoint tensors), ``proj`` (served
+projections), ``load`` and ``forward(h)`` -> the output rows, or something
+``ops.sandwich_norm`` sums itself (``ops.Partials``, ``ops.Mixture``).
+"""
+from __future__ import annotations
+
+import torch
+
+from .. import ops
+from .mixers import _fuse_rows, _up
+
+
+def _pad_cols(w: torch.Tensor, cols: int) -> torch.Tensor:
+    return w if w.shape[-1] == cols else torch.nn.functional.pad(w, (0, cols - w.shape[-1]))
+
+
+class ReluGLU:
+    """W_down (relu(W_gate h) * (W_up h))"""
+
+    def __init__(self, m: dict, width: int):
+        self.ff, self.fp = m["ff"], _up(m["ff"], 16)
+        self.shapes = {"gate": (self.ff, width), "up": (self.ff, width),
+                       "down": (width, self.ff)}
+        self.proj = {"gate_up": (2 * self.fp, width), "down": (width, self.fp)}
+
+    def load(self, get, put):
+        self.w_gu = put(ops.interleave_gate_up(
+            _fuse_rows([get("gate"), get("up")], [self.fp, self.fp]), 16))
+        self.w_down = put(_pad_cols(get("down"), self.fp))
+
+    def forward(self, h):
+        return ops.linear(ops.linear_relu_glu(h, self.w_gu), self.w_down, defer=True)
+
+
+class GeluMLP:
+    """W_down gelu(W_up h), the tanh form"""
+
+    def __init__(self, m: dict, width: int):
+        self.ff, self.fp = m["ff"], _up(m["ff"], 16)
+        self.shapes = {"up": (self.ff, width), "down": (width, self.ff)}
+        self.proj = {"up": (self.fp, width), "down": (width, self.fp)}
+
+    def load(self, get, put):
+        self.w_up = put(_fuse_rows([get("up")], [self.fp]))
+        self.w_down = put(_pad_cols(get("down"), self.fp))
+
+    def forward(self, h):
+        return ops.linear(ops.linear_gelu(h, self.w_up), self.w_down, defer=True)
+
+
+class MixtureOfExperts:
+    """``top`` of ``experts`` clamped GLUs per token, weighted by the softmax
+    over the chosen router logits, plus an optional shared one:
+
+        g = min(W_gate h, L), u = clamp(W_up h, -L, L), W_down (g sigmoid(1.702 g) (u + 1))
+
+    The shared expert runs as further experts of the routed ones' width that
+    every token uses with weight 1: one grouped product covers all of them."""
+
+    def __init__(self, m: dict, width: int):
+        self.width, self.kp = width, _up(width, 64)
+        self.E, self.top = m["router"]["experts"], m["router"]["top"]
+        if not 0 < self.top <= self.E:
+            raise ValueError("moe: top experts out of range")
+        ex, sh = m["expert"], m.get("shared")
+        self.ff = ex["ff"]
+        self.fp = _up(self.ff, 64)
+        self.sff = sh["ff"] if sh else 0
+        self.shared = -(-self.sff // self.fp)          # experts that hold the shared one
+        self.limits = [float(ex["limit"])] * self.E + [float(sh["limit"])] * self.shared \
+            if sh else [float(ex["limit"])] * self.E
+        self.shapes = {}
+        for e in range(self.E):
+            self.shapes.update({f"e{e}.gate": (self.ff, width), f"e{e}.up": (self.ff, width),
+                                f"e{e}.down": (width, self.ff)})
+        self.shapes["router"] = (self.E, width)
+        if sh:
+            self.shapes.update({"shared.gate": (self.sff, width), "shared.up": (self.sff, width),
+                                "shared.down": (width, self.sff)})
+        self.proj = {}
+
+    def load(self, get, put):
+        fp, kp = self.fp, self.kp
+
+        def expert(gate, up, down):
+            w1 = ops.interleave_gate_up(_fuse_rows([gate, up], [fp, fp]), 16)
+            return put(_pad_cols(w1, kp)), put(_pad_cols(down, fp))
+        each = [expert(*(get(f"e{e}.{n}") for n in ("gate", "up", "down"))) for e in range(self.E)]
+        if self.shared:
+            gate, up, down = (get(f"shared.{n}") for n in ("gate", "up", "down"))
+            for a in range(0, self.sff, fp):
+                each.append(expert(gate[a:a + fp], up[a:a + fp], down[:, a:a + fp]))
+        self.w1 = ops.pack_grouped(torch.stack([a for a, _ in each]))
+        self.w2 = ops.pack_grouped(torch.stack([b for _, b in each]))
+        self.limit = put(torch.tensor(self.limits), fp32=True)
+        self.router = put(get("router"))
+
+    def forward(self, h):
+        r = ops.moe_route(h, self.router, self.top, self.shared)
+        plan = ops.moe_plan(r, self.E + self.shared, self.w1.packed)
+        y = ops.grouped_linear(_pad_cols(h, self.kp), self.w1, plan, gather=True, glu=self.limit)
+        return ops.Mixture(ops.grouped_linear(y, self.w2, plan), plan.pos, r.weights)
+

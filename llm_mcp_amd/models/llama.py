@@ -253,23 +253,19 @@ class _Done:
 
 
 class LlamaModel:
-    # what the engine allocates and plans for a model (see ZegopelModel for one
+    # what the engine allocates and plans for a model (see LayerListModel for one
     # that uses all of it)
     prefix_cache_ok = True        # a cached prefix page is all a sequence needs of it
+    needs_plan = False            # no ``host_plan``, no state slots
 
     def state_shapes(self) -> list:
         """Per-slot state tensors: [(shape, dtype)]."""
         return []
 
-    def host_plan(self, plan: dict) -> tuple[list, dict]:
-        """Extra index arrays of an eager step [(name, int32 array)] and the
-        host values that go with them."""
-        return [], {}
-
     @property
     def kv_layers(self) -> list:
-        """(kv heads, head size) of each paged-cache layer."""
-        return [(self.Hkv, self.D)] * self.cfg.num_layers
+        """(kv heads, key size, value size) of each paged-cache layer."""
+        return [(self.Hkv, self.D, self.D)] * self.cfg.num_layers
 
     @property
     def q_per_tile(self) -> int:

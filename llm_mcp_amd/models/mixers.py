@@ -1,10 +1,13 @@
-"""Token mixers and feed-forward of layer-list decoders (``models.zegopel``).
+"""Token mixers of layer-list decoders (``models.layerlist``).
 
 A mixer is built for one layer from its ``mixer`` dict; it names its
 checkpoint tensors and shapes (``shapes``), fuses them into served weights
-(``load``), declares what it keeps per sequence -- ``kv`` (heads, head size) in
-the paged cache, ``state`` tensors in the state slots -- and runs on a step's
-rows: ``forward(h, inp, cache, state)`` -> the mixer's output rows.
+(``load``), declares what it keeps per sequence -- ``kv`` (heads, key size,
+value size) in the paged cache, ``state`` tensors in the state slots -- and runs
+on a step's rows: ``forward(h, inp, cache, state)`` -> the mixer's output rows.
+What it needs planned on the host for a step's multi-token sequences comes from
+``build_plan`` / ``bind_plan``, one plan for all layers of a ``plan_key``
+(``StepInputs.aux[plan_key]``).
 
 Served layouts:
 * every mixer has ONE input projection (its projections fused by rows) and one
@@ -22,6 +25,7 @@ import math
 import torch
 
 from .. import ops
+from ..ops import mixers as mixer_ops
 
 
 def _up(n: int, m: int) -> int:
@@ -38,12 +42,40 @@ def _fuse_rows(parts: list[torch.Tensor], pads: list[int]) -> torch.Tensor:
     return out
 
 
-class LightningMixer:
+class Mixer:
+    kv = None                     # (heads, key size, value size) of its cache pages
+    q_per_tile = 0
+    plan_key = None
+    rot = None                    # (base, dims) of its rotary positions
+
+    def state_shapes(self, dtype):
+        return []
+
+    def build_plan(self, qlens, ctx, seq0: int):
+        """(items to upload, host value) for the sequences from seq0 on."""
+        raise NotImplementedError
+
+    def bind_plan(self, dev: dict, host):
+        raise NotImplementedError
+
+
+class ScanMixer(Mixer):
+    """Plan of a segmented scan: ``plan_key`` = ("scan", heads, columns)."""
+
+    def build_plan(self, qlens, ctx, seq0):
+        _, H, P = self.plan_key
+        segs, first, one = mixer_ops.scan_segments(qlens, seq0, H, P)
+        return [(f"segs{H, P}", segs), (f"first{H, P}", first)], (len(segs), one)
+
+    def bind_plan(self, dev, host):
+        _, H, P = self.plan_key
+        return ops.ScanSegments(dev[f"segs{H, P}"], dev[f"first{H, P}"], *host)
+
+
+class LightningMixer(ScanMixer):
     """Linear attention with a constant decay per head: q, k, v = silu(W h),
     S <- decay S + k v^T, o = S^T q; heads concatenated, RMS-normed, times
     sigmoid(W_g h), projected."""
-    kv = None
-    q_per_tile = 0
 
     def __init__(self, m: dict, width: int, eps: float):
         self.H, self.N, self.P, self.eps = m["heads"], m["dim"], m["vdim"], eps
@@ -59,7 +91,7 @@ class LightningMixer:
     def state_shapes(self, dtype):
         return [((self.H, self.N, self.P), torch.float32)]
 
-    scan_geometry = property(lambda self: (self.H, self.P))
+    plan_key = property(lambda self: ("scan", self.H, self.P))
 
     def load(self, get, put):
         self.w_in = put(_fuse_rows([get("q"), get("k"), get("v"), get("g")],
@@ -75,18 +107,16 @@ class LightningMixer:
         o = ops.linear_scan(p[:, :qk], p[:, qk:2 * qk], p[:, 2 * qk:2 * qk + vg], state[0],
                             inp.cu_q, inp.context_lens, inp.state_slots, decay=self.decays,
                             silu=True, num_decode=inp.num_decode,
-                            segments=inp.aux.get(f"scan{self.scan_geometry}"))
+                            segments=inp.aux.get(self.plan_key))
         y = ops.gated_norm(o, p[:, 2 * qk + vg:], self.norm, 1, self.eps, gate_first=False)
         return ops.linear(y, self.w_o, defer=True)
 
 
-class Mamba2Mixer:
+class Mamba2Mixer(ScanMixer):
     """State-space mixer (scalar decay per head and token): z | x | B | C | dt
     from one projection, a short convolution with SiLU over x, B and C,
     S <- exp(-exp(A_log) s) S + s B x^T with s = softplus(dt + dt_bias),
     y = S^T C + D x; y silu(z) RMS-normed in parts, projected."""
-    kv = None
-    q_per_tile = 0
 
     def __init__(self, m: dict, width: int, eps: float):
         self.H, self.P, self.N, self.G = m["heads"], m["vdim"], m["state"], m["groups"]
@@ -111,7 +141,7 @@ class Mamba2Mixer:
             out.append(((self.taps - 1, self.cp), dtype))
         return out
 
-    scan_geometry = property(lambda self: (self.H, self.P))
+    plan_key = property(lambda self: ("scan", self.H, self.P))
 
     def load(self, get, put):
         w, i, c = get("in"), self.inner, self.C
@@ -138,16 +168,15 @@ class Mamba2Mixer:
                             inp.context_lens, inp.state_slots, heads_per_group=self.H // self.G,
                             dt=(dt, self.dt_bias, self.neg_a), skip=self.D,
                             num_decode=inp.num_decode,
-                            segments=inp.aux.get(f"scan{self.scan_geometry}"))
+                            segments=inp.aux.get(self.plan_key))
         y = ops.gated_norm(y, z, self.norm, self.norm_groups, self.eps, gate_first=True)
         return ops.linear(y, self.w_o, defer=True)
 
 
-class ConvAttentionMixer:
+class ConvAttentionMixer(Mixer):
     """Softmax attention without rotation: biased q, k, v through a short
     convolution, unit-RMS q and k, a position-dependent query temperature, an
     output gate sigmoid(W_g h)."""
-    scan_geometry = None
 
     def __init__(self, m: dict, width: int, eps: float):
         self.Hq, self.Hkv, self.dk, self.dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
@@ -168,7 +197,7 @@ class ConvAttentionMixer:
                        "q.conv": (H * dk, self.taps), "k.conv": (G * dk, self.taps),
                        "v.conv": (G * dv, self.taps), "g": (H * dv, width),
                        "o": (width, H * dv)}
-        self.kv = (G, D)
+        self.kv = (G, D, D)
         self.qkv = (H + 2 * G) * D
         self.proj = {"in": (self.qkv + H * D, width), "o": (width, H * D)}
         # the MFMA attention kernels: head sizes 64 / 128, up to 16 query heads per kv head
@@ -176,6 +205,15 @@ class ConvAttentionMixer:
         # queries per prefill workgroup (4 waves)
         self.q_per_tile = (4 * (4 if D == 64 else ops.PREFILL_GROUPS_PER_WAVE) * (16 // (H // G))
                            if self.mfma_geometry else 0)
+        if self.q_per_tile:
+            self.plan_key = ("attn", self.q_per_tile)
+
+    def build_plan(self, qlens, ctx, seq0):
+        q = self.q_per_tile
+        return [(f"attn{q}", mixer_ops.row_tiles(qlens, q).reshape(-1))], None
+
+    def bind_plan(self, dev, host):
+        return dev[f"attn{self.q_per_tile}"]
 
     def state_shapes(self, dtype):
         return [((self.taps - 1, self.qkv), dtype)] if self.taps > 1 else []
@@ -218,49 +256,192 @@ class ConvAttentionMixer:
                                        precise=True)
         if T > nd:
             ops.paged_prefill_attention(q, kc, vc, inp.block_tables[nd:], inp.cu_q[nd:],
-                                        inp.context_lens[nd:], inp.aux[f"attn{self.q_per_tile}"],
+                                        inp.context_lens[nd:], inp.aux[self.plan_key],
                                         self.scale, a, Hq=self.Hq, q_per_tile=self.q_per_tile,
                                         gate=gate, precise=True)
         return ops.linear(a, self.w_o, defer=True)
 
 
-class ReluGLU:
-    """W_down (relu(W_gate h) * (W_up h))"""
+class RGLRUMixer(ScanMixer):
+    """Gated linear recurrence between two branches: y = gelu(W_y h + b_y) and
+    u = conv(W_x h + b_x); gates r, i = sigmoid of block-diagonal maps of u;
+    log a = -8 r softplus(lam), S <- a S + sqrt(1 - a^2) i u; W_o (S y).
 
-    def __init__(self, m: dict, width: int):
-        self.ff, self.fp = m["ff"], _up(m["ff"], 16)
-        self.shapes = {"gate": (self.ff, width), "up": (self.ff, width),
-                       "down": (width, self.ff)}
-        self.proj = {"gate_up": (2 * self.fp, width), "down": (width, self.fp)}
+    Channels are served in blocks padded to powers of two from 32 (zero weights:
+    a padded channel stays zero)."""
+
+    def __init__(self, m: dict, width: int, eps: float):
+        self.W, self.n, self.taps = m["width"], m["blocks"], m["conv"]
+        if self.W % self.n:
+            raise ValueError("rglru: width must be a multiple of blocks")
+        W, n = self.W, self.n
+        self.bs = W // n
+        self.bp = 1 << max(5, (self.bs - 1).bit_length())
+        self.C = n * self.bp
+        self.shapes = {"y": (W, width), "y.b": (W,), "x": (W, width), "x.b": (W,),
+                       "conv": (W, self.taps), "conv.b": (W,), "ra": (n, self.bs, self.bs),
+                       "ra.b": (n, self.bs), "ri": (n, self.bs, self.bs), "ri.b": (n, self.bs),
+                       "lam": (W,), "o": (width, W)}
+        self.proj = {"in": (2 * self.C, width), "o": (width, self.C)}
+        self.plan_key = ("scan", -(-self.C // ops.RGLRU_TILE), 1)
+
+    def state_shapes(self, dtype):
+        out = [((self.C,), torch.float32)]
+        if self.taps > 1:
+            out.append(((self.taps - 1, self.C), dtype))
+        return out
+
+    def _blocks(self, t):
+        """[W, ...] channel rows -> [C, ...], each block padded with zeros."""
+        out = t.new_zeros((self.n, self.bp) + tuple(t.shape[1:]))
+        out[:, :self.bs] = t.reshape((self.n, self.bs) + tuple(t.shape[1:]))
+        return out.reshape((self.C,) + tuple(t.shape[1:]))
 
     def load(self, get, put):
-        self.w_gu = put(ops.interleave_gate_up(
-            _fuse_rows([get("gate"), get("up")], [self.fp, self.fp]), 16))
-        down = get("down")
-        w = down.new_zeros((down.shape[0], self.fp))
-        w[:, :self.ff] = down
-        self.w_down = put(w)
+        def vec(name):
+            return put(self._blocks(get(name).reshape(-1)), fp32=True)
+        self.w_in = put(torch.cat([self._blocks(get("y")), self._blocks(get("x"))]))
+        self.y_b, self.x_b, self.conv_b = vec("y.b"), vec("x.b"), vec("conv.b")
+        self.conv = put(self._blocks(get("conv")).float().t(), fp32=True)
+        gates = torch.stack([get("ra"), get("ri")], 1)              # [n, 2, out, in]
+        pad = self.bp - self.bs
+        gates = torch.nn.functional.pad(gates, (0, pad, 0, pad)).reshape(self.n, 2 * self.bp, -1)
+        self.gates = ops.pack_grouped(put(gates, fp32=self.bp > ops.RGLRU_MAX_BLOCK))
+        self.gate_b = put(torch.stack([self._blocks(get(k).reshape(-1).float())
+                                       for k in ("ra.b", "ri.b")]), fp32=True)
+        lam = get("lam").double()
+        self.log_a = put(self._blocks(-8.0 * torch.nn.functional.softplus(lam)), fp32=True)
+        self.w_o = put(self._blocks(get("o").t().contiguous()).t())
 
-    def forward(self, h):
-        return ops.linear(ops.linear_relu_glu(h, self.w_gu), self.w_down, defer=True)
+    def forward(self, h, inp, cache, state):
+        C = self.C
+        p = ops.linear(h, self.w_in)
+        u = ops.short_conv(p[:, C:], self.conv, state[1] if self.taps > 1 else None, inp.cu_q,
+                           inp.context_lens, inp.state_slots, bias=self.conv_b,
+                           in_bias=self.x_b, tiles=inp.aux.get("conv"))
+        y = ops.rglru(u, p[:, :C], self.y_b, self.gates, self.gate_b, self.log_a, state[0],
+                      inp.cu_q, inp.context_lens, inp.state_slots, num_decode=inp.num_decode,
+                      segments=inp.aux.get(self.plan_key))
+        return ops.linear(y, self.w_o, defer=True)
 
 
-MIXERS = {"lightning": LightningMixer, "mamba2": Mamba2Mixer, "attention": ConvAttentionMixer}
+class LatentAttentionMixer(Mixer):
+    """Latent attention with a sliding window and an output gate: queries
+    W_uq norm(W_dq h); keys and values W_uk c, W_uv c of a normed latent c,
+    beside one rotated key part shared by all heads.  A token's cache page row
+    is [c | rotated key].
+
+    Decode rows score latents: q W_uk against c, and W_uv the weighted sum of
+    latents.  Prompt rows expand the keys and values of the rows they see."""
+    Hkv = 1
+
+    def __init__(self, m: dict, width: int, eps: float):
+        self.Hq, self.dn, self.dr, self.dv = m["heads"], m["dim"], m["rot_dim"], m["vdim"]
+        self.R, self.qr, self.scale, self.eps = m["kv_rank"], m["q_rank"], float(m["scale"]), eps
+        self.window = int(m["mask"]["size"])
+        rot = m["rot"]
+        if rot["dims"] != self.dr or self.dr % 2 or self.window < 1:
+            raise ValueError("latent_attention: rot.dims = rot_dim, even; a window of at least 1")
+        H = self.Hq
+        self.rot = (float(rot["base"]), self.dr)
+        self.D = self.Rp = next((r for r in (64, 128, 256, 512) if r >= self.R), _up(self.R, 64))
+        self.xp = _up(self.dr, 64)
+        self.np, self.vp, self.qp = _up(self.dn, 64), _up(self.dv, 64), _up(self.qr, 64)
+        self.shapes = {"dq": (self.qr, width), "dq.norm": (self.qr,),
+                       "uq": (H * (self.dn + self.dr), self.qr),
+                       "dkv": (self.R + self.dr, width), "dkv.norm": (self.R,),
+                       "uk": (H * self.dn, self.R), "uv": (H * self.dv, self.R),
+                       "g": (H * self.dv, width), "o": (width, H * self.dv)}
+        self.kv = (1, self.Rp + self.xp, 0)
+        rows = self.qp + self.Rp + self.xp + H * self.vp
+        # a wide projection is rounded up to whole 256-row GEMM tiles
+        self.tail = (_up(rows, 256) if rows >= 4096 else rows) - rows
+        self.proj = {"in": (rows + self.tail, width), "uq": (H * (self.np + self.xp), self.qp),
+                     "o": (width, H * self.vp)}
+        self.expand = ops.latent_prefill_ok(self.np, self.xp, self.vp)
+        if self.expand:
+            self.plan_key = ("latent", self.window)
+
+    def build_plan(self, qlens, ctx, seq0):
+        w = self.window
+        rows, tiles, n = mixer_ops.latent_rows(qlens, ctx, w)
+        return [(f"lrows{w}", rows), (f"ltiles{w}", tiles)], n
+
+    def bind_plan(self, dev, host):
+        return ops.LatentRows(dev[f"lrows{self.window}"], dev[f"ltiles{self.window}"], host)
+
+    def _heads(self, t, d, p):
+        """[H * d, ...] rows -> [H, p, ...], padded with zeros."""
+        out = t.new_zeros((self.Hq, p) + tuple(t.shape[1:]))
+        out[:, :d] = t.reshape((self.Hq, d) + tuple(t.shape[1:]))
+        return out
+
+    def load(self, get, put):
+        H, dn, dr, dv, R = self.Hq, self.dn, self.dr, self.dv, self.R
+        dkv = get("dkv")
+        g = self._heads(get("g"), dv, self.vp).reshape(H * self.vp, -1)
+        self.w_in = put(_fuse_rows([get("dq"), dkv[:R], dkv[R:], g],
+                                   [self.qp, self.Rp, self.xp, H * self.vp + self.tail]))
+        pad = torch.nn.functional.pad
+        self.q_norm = put(pad(get("dq.norm"), (0, self.qp - self.qr)), fp32=True)
+        self.c_norm = put(pad(get("dkv.norm"), (0, self.Rp - R)), fp32=True)
+        uq = get("uq").reshape(H, dn + dr, self.qr)
+        q = uq.new_zeros((H, self.np + self.xp, self.qp))
+        q[:, :dn, :self.qr] = uq[:, :dn]
+        q[:, self.np:self.np + dr, :self.qr] = uq[:, dn:]
+        self.w_uq = put(q.reshape(-1, self.qp))
+        uk = pad(self._heads(get("uk"), dn, self.np), (0, self.Rp - R))      # [H, np, Rp]
+        uv = pad(self._heads(get("uv"), dv, self.vp), (0, self.Rp - R))      # [H, vp, Rp]
+        self.absorb = ops.pack_grouped(put(uk.transpose(1, 2).contiguous()))
+        self.unfold = ops.pack_grouped(put(uv))
+        self.w_kv = put(torch.cat([uk, uv], 1).reshape(-1, self.Rp)) if self.expand else None
+        self.w_o = put(self._heads(get("o").t().contiguous(), dv, self.vp)
+                       .reshape(H * self.vp, -1).t())
+
+    def forward(self, h, inp, cache, state):
+        H, T, nd = self.Hq, inp.num_tokens, inp.num_decode
+        pages, ang = cache[0], inp.aux["rot", self.rot]
+        p = ops.linear(h, self.w_in)
+        a0 = self.qp + self.Rp + self.xp
+        gate = p[:, a0:a0 + H * self.vp]
+        cq = ops.latent_prep(p, self.qr, self.qp, self.q_norm, self.R, self.c_norm, ang,
+                             inp.slots, pages, self.Rp, self.eps)
+        q = ops.linear(cq, self.w_uq)
+        out = torch.empty((T, H * self.vp), dtype=h.dtype, device=h.device)
+        rows = inp.aux.get(self.plan_key) if self.expand and q.dtype == torch.bfloat16 else None
+        n = nd if rows is not None else T              # rows on latents: the first n
+        if n:
+            ql = ops.latent_query(q[:n], self.absorb, ang, H, self.np, self.xp, self.Rp)
+            o = ops.latent_attention(ql, pages, inp.block_tables, inp.cu_q, inp.positions,
+                                     self.scale, self.window, H, self.Rp, ws=inp.decode_ws,
+                                     part_tokens=inp.part_tokens, num_decode=nd)
+            ops.grouped_heads(o, self.unfold, gate=gate[:n], out=out[:n])
+        if rows is not None:
+            ops.latent_prefill(q, pages, rows, self.w_kv, ang, inp.block_tables[nd:],
+                               inp.cu_q[nd:], inp.context_lens[nd:], self.scale, self.window, H,
+                               self.np, self.xp, self.vp, self.Rp, gate, out)
+        return ops.linear(out, self.w_o, defer=True)
 
 
-def init_std(name: str, shape: tuple, depth: int) -> tuple[float, float]:
+def init_std(name: str, shape: tuple, depth: int, zero_centred: bool = True) -> tuple[float, float]:
     """(mean, std) of a tensor's random initialisation (benchmarks, tests)."""
     leaf = name.rsplit(".", 1)[-1]
     if leaf in ("o", "down"):
         return 0.0, 0.02 / math.sqrt(2 * depth)
     if leaf == "conv":
         return 1.0 / shape[-1], 0.2
-    if name.endswith(".mix.norm") or leaf == "D":
+    if name.endswith(".mix.norm") or leaf == "D" or name.endswith(("dq.norm", "dkv.norm")):
         return 1.0, 0.1
     if leaf == "A_log":
         return 0.5, 0.5
     if leaf == "dt_bias":
         return -3.0, 1.0
+    if leaf == "lam":              # decays of 0.9 and slower
+        return -4.0, 1.0
+    if leaf in ("ra", "ri"):
+        return 0.0, shape[-1] ** -0.5
     if name == "embed":
         return 0.0, 1.0
+    if leaf.startswith("norm"):
+        return (0.0 if zero_centred else 1.0), 0.02
     return 0.0, 0.02

@@ -29,7 +29,7 @@ import os
 
 import torch
 
-from .config import LlamaConfig
+from .config import LayerListConfig, LlamaConfig
 
 
 def vocab_shard(vocab: int, size: int) -> int:
@@ -260,25 +260,20 @@ def load_tensors(path: str, shapes: dict[str, tuple]) -> dict:
 
 def load_weights(path: str, cfg, device, rank: int = 0, size: int = 1) -> dict:
     """This rank's weights of a chat model's checkpoint directory, by family."""
-    if cfg.family == "zegopel":
-        from .zegopel import tensor_shapes
+    if isinstance(cfg, LayerListConfig):
+        from .registry import model_class
         if size > 1:
-            raise ValueError("zegopel: no tensor-parallel form")
-        return load_tensors(path, tensor_shapes(cfg))
+            raise ValueError(f"{cfg.family}: no tensor-parallel form")
+        return load_tensors(path, model_class(cfg).tensor_shapes(cfg))
     return load_llama_weights(path, cfg, device, rank, size)
 
 
-def save_zegopel(weights: dict, cfg, path: str) -> None:
-    """Write named tensors and the configuration as a checkpoint directory."""
+def save_layer_list(weights: dict, cfg, path: str) -> None:
+    """Write a layer-list decoder's named tensors and configuration as a
+    checkpoint directory."""
     from safetensors.torch import save_file
     os.makedirs(path, exist_ok=True)
     save_file({k: v.detach().to("cpu").contiguous() for k, v in weights.items()},
               os.path.join(path, "model.safetensors"))
-    js = {"architecture": "Zegopel", "layers": cfg.layers, "norm": {"eps": cfg.rms_eps},
-          "vocab": cfg.vocab_size, "width": cfg.hidden_size}
-    if cfg.eos_token_ids:
-        js["eos_token_id"] = list(cfg.eos_token_ids)
-    if cfg.bos_token_id is not None:
-        js["bos_token_id"] = cfg.bos_token_id
     with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(js, f)
+        json.dump(cfg.to_json(), f)

@@ -883,6 +883,25 @@ def linear_relu_glu(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return relu_mul(linear(x, w), block=SWIGLU16)
 
 
+def gelu(x: torch.Tensor) -> torch.Tensor:
+    """gelu (tanh form) of a projection's rows (bf16 or fp32), in place."""
+    if not x.is_cuda:
+        return torch.nn.functional.gelu(x.float(), approximate="tanh").to(x.dtype)
+    _chk(x.dtype in (torch.bfloat16, torch.float32) and x.is_contiguous()
+         and x.numel() % 8 == 0, "gelu rows")
+    native().gelu(_ptr(x), x.numel(), int(x.dtype == torch.bfloat16), _stream())
+    return x
+
+
+def linear_gelu(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """gelu(x @ w^T), tanh form: K13's epilogue for prefill-sized M, else the
+    product and an elementwise pass."""
+    if (x.is_cuda and x.dtype == torch.bfloat16 and pgemm_operands_ok(x, w)
+            and large_gemm_backend(x.shape[0], w.shape[0], w.shape[1], ACT_GELU) == "k13"):
+        return pgemm(x, w, act=ACT_GELU)
+    return gelu(linear(x, w))
+
+
 def swiglu_block(N: int, K: int) -> int:
     """Interleave block of the gate|up weights for the fused decode GEMM of
     this shape: 16 when the table has in-register-epilogue (epi 3) entries,
@@ -1778,5 +1797,9 @@ def pgemm_sk(a: torch.Tensor, w: torch.Tensor, splits: int, act: int = 0, epi: i
     return out
 
 
-from .mixers import (ScanSegments, attention_any, conv_qkv_cache, gated_norm,  # noqa: E402,F401
-                     linear_scan, sandwich_norm, scan_segments, short_conv)
+from .grouped import (GroupedWeight, Mixture, MoePlan, Route, grouped_heads,  # noqa: E402,F401
+                      grouped_linear, moe_plan, moe_route, pack_grouped)
+from .mixers import (RGLRU_MAX_BLOCK, RGLRU_TILE, LatentRows, ScanSegments,  # noqa: E402,F401
+                     attention_any, conv_qkv_cache, gated_norm, latent_attention,
+                     latent_prefill_ok, latent_prep, latent_query, linear_scan, rglru,
+                     rope_angles, rope_freqs, sandwich_norm, scan_segments, short_conv)

@@ -13,12 +13,14 @@ slots are never cleared.
 """
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass
 
 import numpy as np
 import torch
 
 from . import Partials, _chk, _ptr, _stream, native, ref
+from .grouped import GroupedWeight, Mixture, grouped_heads
 
 CONV_TILE = 64        # tokens per convolution workgroup
 SCAN_CHUNK = 64       # SC in csrc/kernels/linscan.hip
@@ -47,26 +49,33 @@ def _meta(S: int, **ts) -> None:
 def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tensor | None = None,
                   w_pre: torch.Tensor | None = None, ids: torch.Tensor | None = None,
                   table: torch.Tensor | None = None, rows: torch.Tensor | None = None,
-                  dtype: torch.dtype = torch.bfloat16) -> torch.Tensor | None:
+                  dtype: torch.dtype = torch.bfloat16, scale: float = 1.0) -> torch.Tensor:
     """One pass over the fp32 residual stream between two sublayers:
 
-        r = table[ids] (if given) else residual
-        r += rms(y) * w_post         (y: sublayer output rows or ``Partials``)
+        r = scale table[ids] (if given) else residual
+        r += rms(y) * w_post         (y: sublayer output rows, ``Partials`` or ``Mixture``)
         residual = r                 (unless ``rows`` is given)
-        return rms(r) * w_pre        (``dtype`` rows; None without w_pre)
+        return rms(r) * w_pre        (``dtype`` rows; r itself without w_pre)
 
     ``rows`` (int64): only these rows are normed, the residual stays as it is.
     The gains are fp32 vectors."""
     T, d = residual.shape
     if not residual.is_cuda:
-        return ref.sandwich_norm(residual, eps, y, w_post, w_pre, ids, table, rows, dtype)
+        y = y.sum() if isinstance(y, Mixture) else y
+        return ref.sandwich_norm(residual, eps, y, w_post, w_pre, ids, table, rows, dtype, scale)
     _chk(residual.dtype == torch.float32 and residual.is_contiguous(), "residual: fp32 rows")
     _f32(w_post, d, "w_post"); _f32(w_pre, d, "w_pre")
     bf = int(dtype == torch.bfloat16)
-    yp, y_ld, slabs, sstride = 0, 0, 0, 0
+    yp, y_ld, slabs, sstride, mix = 0, 0, 0, 0, (0, 0, 0)
     if isinstance(y, Partials):
         _chk((y.M, y.N) == (T, d), "sandwich_norm partials shape")
         yp, y_ld, slabs, sstride = _ptr(y.slabs), d, y.S, y.M * y.N
+    elif isinstance(y, Mixture):
+        _chk(y.rows.shape[1] == d and y.rows.is_contiguous() and y.rows.dtype == dtype
+             and y.pos.shape == y.weights.shape and y.pos.shape[0] == T
+             and y.pos.dtype == torch.int32 and y.weights.dtype == torch.float32
+             and y.pos.is_contiguous() and y.weights.is_contiguous(), "sandwich_norm mixture")
+        yp, y_ld, mix = _ptr(y.rows), d, (_ptr(y.pos), _ptr(y.weights), y.pos.shape[1])
     elif y is not None:
         _chk(y.shape == (T, d) and y.stride(1) == 1 and y.dtype == dtype, "sandwich_norm y rows")
         yp, y_ld = _ptr(y), y.stride(0)
@@ -78,10 +87,10 @@ def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tens
     if rows is not None:
         _chk(rows.dtype == torch.int64 and rows.is_contiguous(), "rows: int64")
         n = rows.numel()
-    out = torch.empty((n, d), dtype=dtype, device=residual.device) if w_pre is not None else None
-    native().sandwich_norm(_ptr(out), _ptr(residual), yp, y_ld, slabs, sstride, _ptr(ids),
-                           _ptr(table), _ptr(w_post), _ptr(w_pre), _ptr(rows), n, d, float(eps),
-                           bf, _stream())
+    out = torch.empty((n, d), dtype=dtype, device=residual.device)
+    native().sandwich_norm(_ptr(out), _ptr(residual), yp, y_ld, slabs, sstride, *mix, _ptr(ids),
+                           _ptr(table), float(scale), _ptr(w_post), _ptr(w_pre), _ptr(rows), n, d,
+                           float(eps), bf, _stream())
     return out
 
 
@@ -138,20 +147,22 @@ def _conv_meta(u, w, state, tiles, cu_q, ctx, slots):
 
 def short_conv(u: torch.Tensor, w: torch.Tensor, state: torch.Tensor | None, cu_q, ctx, slots,
                bias: torch.Tensor | None = None, silu: bool = False,
-               tiles: torch.Tensor | None = None) -> torch.Tensor:
+               tiles: torch.Tensor | None = None,
+               in_bias: torch.Tensor | None = None) -> torch.Tensor:
     """Causal convolution over time of each channel (w fp32 [taps, C], last
     tap = the current token), optionally SiLU; ``state`` [slots, taps - 1, C]
-    carries the last inputs.  ``tiles`` (``conv_tiles``): needed when a
-    sequence has more than one row."""
+    carries the last inputs.  ``in_bias``: the projection's own bias (fp32 [C],
+    added to u).  ``tiles`` (``conv_tiles``): needed when a sequence has more
+    than one row."""
     taps, C = w.shape
     out = torch.empty((u.shape[0], C), dtype=u.dtype, device=u.device)
     if not u.is_cuda:
-        ref.short_conv(u, w, bias, state, cu_q, ctx, slots, out, silu)
+        ref.short_conv(u, w, bias, state, cu_q, ctx, slots, out, silu, in_bias)
         return out
     bf = _rows_dtype(u, "u")
     taps, C, n = _conv_meta(u, w, state, tiles, cu_q, ctx, slots)
-    _f32(bias, C, "conv bias")
-    native().short_conv(_ptr(u), u.stride(0), _ptr(w), _ptr(bias), _ptr(state), _ptr(tiles), n,
+    _f32(bias, C, "conv bias"); _f32(in_bias, C, "projection bias")
+    native().short_conv(_ptr(u), u.stride(0), _ptr(w), _ptr(in_bias), _ptr(bias), _ptr(state), _ptr(tiles), n,
                         CONV_TILE, _ptr(cu_q), _ptr(ctx), _ptr(slots), C, taps, _ptr(out),
                         out.stride(0), int(silu), bf, _stream())
     return out
@@ -313,3 +324,179 @@ def attention_any(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, ctx, po
                            gate.stride(0) if gate is not None else 0, Hq, Hkv, D, BS,
                            float(scale), bf, _stream())
     return out
+
+
+# -------------------------------------------------- gated linear recurrence --
+RGLRU_TILE = 64            # channels per workgroup (csrc/kernels/rglru.hip)
+RGLRU_MAX_BLOCK = 512      # gate blocks the MFMA kernels hold in registers
+
+
+def rglru(u: torch.Tensor, y: torch.Tensor, y_bias: torch.Tensor, gates: GroupedWeight,
+          gate_bias: torch.Tensor, log_a: torch.Tensor, state: torch.Tensor, cu_q, ctx, slots,
+          num_decode: int = 0, segments: ScanSegments | None = None) -> torch.Tensor:
+    """Per channel, over each sequence's rows and from / to ``state`` (fp32
+    [slots, C]):
+
+        r, i = sigmoid(block-diagonal gates of u + gate_bias)      [2, C]
+        a = exp(log_a r);  S <- a S + sqrt(1 - a^2) i u
+        out = S gelu_tanh(y + y_bias)
+
+    gates: [blocks, 2 * C/blocks, C/blocks], the r rows before the i rows of a
+    block.  Sequences before ``num_decode`` (one row each) take the row kernel,
+    the others the chunked one (``segments``); fp32 rows and blocks above
+    ``RGLRU_MAX_BLOCK`` a plain scan of fp32 gates."""
+    T, C = u.shape
+    n, bp, S = gates.groups, gates.K, ctx.numel()
+    _chk(n * bp == C and gates.N == 2 * bp, "rglru gate blocks")
+    out = torch.empty((T, C), dtype=u.dtype, device=u.device)
+    if not u.is_cuda:
+        ref.rglru(u, y, y_bias, gates.data, gate_bias, log_a, out, state, cu_q, ctx, slots)
+        return out
+    bf = _rows_dtype(u, "u")
+    _chk(u.is_contiguous() and y.dtype == u.dtype and y.shape == (T, C) and y.stride(1) == 1,
+         "rglru rows")
+    _chk(state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] == C,
+         "rglru state")
+    _f32(y_bias, C, "y bias"); _f32(gate_bias, 2 * C, "gate bias"); _f32(log_a, C, "log_a")
+    _meta(S, cu_q=cu_q, ctx=ctx, slots=slots)
+    args = (_ptr(u), _ptr(y), y.stride(0), _ptr(y_bias), _ptr(gate_bias), _ptr(log_a), _ptr(out),
+            _ptr(state), _ptr(cu_q), _ptr(ctx), _ptr(slots), C, bp)
+    if not gates.packed:
+        z = grouped_heads(u.float(), gates)
+        native().rglru_scan(*args, _ptr(z), S, bf, _stream())
+        return out
+    if num_decode:
+        native().rglru_rows(*args, _ptr(gates.data), num_decode, _stream())
+    if S > num_decode:
+        g = segments
+        _chk(g is not None and g.segs.dtype == torch.int32 and g.segs.numel() >= 4 * g.n
+             and g.first.dtype == torch.int32 and g.first.numel() == S - num_decode + 1,
+             "rglru segments")
+        ws = None if g.one_pass else torch.empty((3, g.n, C), dtype=torch.float32, device=u.device)
+        native().rglru_chunks(*args, _ptr(gates.data), num_decode, _ptr(g.segs), g.n,
+                              _ptr(g.first), _ptr(ws), _stream())
+    return out
+
+
+# --------------------------------------------------------- latent attention --
+def rope_freqs(base: float, dims: int, device="cpu") -> torch.Tensor:
+    """base^(-2i / dims), i < dims / 2 (double)."""
+    i = torch.arange(dims // 2, dtype=torch.float64, device=device)
+    return torch.exp(-2.0 * math.log(base) / dims * i)
+
+
+def rope_angles(positions: torch.Tensor, freqs: torch.Tensor) -> torch.Tensor:
+    """fp32 [T, dims]: cos | sin of position * frequency (reduced in double, so
+    no table bounds the positions)."""
+    if not positions.is_cuda:
+        return ref.rope_angles(positions, freqs)
+    T, n = positions.numel(), freqs.numel()
+    _chk(positions.dtype == torch.int32 and freqs.dtype == torch.float64, "rope_angles")
+    out = torch.empty((T, 2 * n), dtype=torch.float32, device=positions.device)
+    native().rope_angles(_ptr(positions), _ptr(freqs), T, n, _ptr(out), _stream())
+    return out
+
+
+def latent_prep(p: torch.Tensor, qr: int, qp: int, q_norm: torch.Tensor, R: int,
+                c_norm: torch.Tensor, angles: torch.Tensor, slots: torch.Tensor,
+                pages: torch.Tensor, Rp: int, eps: float) -> torch.Tensor:
+    """Projection rows [query latent (qr of qp) | latent c (R of Rp) | rotated
+    key part | ..]: returns the RMS-normed query latents [T, qp]; the normed c
+    and the key part turned by ``angles`` go to the pages' rows at ``slots``
+    (-1: none).  Gains fp32 [qp], [Rp], zero in the padding."""
+    T, d = angles.shape
+    _, _, BS, D = pages.shape
+    if not p.is_cuda:
+        return ref.latent_prep(p, qr, qp, q_norm, R, c_norm, angles, slots, pages, Rp, eps)
+    bf = _rows_dtype(p, "p")
+    _f32(q_norm, qp, "q_norm"); _f32(c_norm, Rp, "c_norm"); _f32(angles, T * d, "angles")
+    _meta(T, slots=slots)
+    _chk(p.shape[0] == T and p.shape[1] >= qp + D and p.stride(1) == 1 and p.stride(0) % 8 == 0
+         and p.data_ptr() % 16 == 0 and qp % 8 == 0 and Rp % 8 == 0 and d <= D - Rp
+         and pages.dtype == p.dtype and pages.is_contiguous(), "latent_prep rows")
+    cq = torch.empty((T, qp), dtype=p.dtype, device=p.device)
+    native().latent_prep(_ptr(p), p.stride(0), T, qr, qp, _ptr(q_norm), R, Rp, _ptr(c_norm),
+                         _ptr(angles), d, _ptr(slots), _ptr(pages), BS, D, _ptr(cq), float(eps),
+                         bf, _stream())
+    return cq
+
+
+def latent_query(q: torch.Tensor, absorb: GroupedWeight, angles: torch.Tensor, H: int, np_: int,
+                 xp: int, Rp: int) -> torch.Tensor:
+    """Query rows of H x [np_ unrotated | xp to rotate] -> H x [W_uk^T q (Rp) |
+    rotated part (xp)]: queries that score latent rows."""
+    T, d = q.shape[0], angles.shape[1]
+    if not q.is_cuda:
+        return ref.latent_query(q, absorb.data, angles, H, np_, xp, Rp)
+    bf = _rows_dtype(q, "q")
+    _chk(q.stride(1) == 1 and q.shape[1] == H * (np_ + xp) and absorb.N == Rp
+         and absorb.K == np_ and absorb.groups == H and d <= xp and angles.shape[0] >= T,
+         "latent_query rows")
+    out = torch.empty((T, H * (Rp + xp)), dtype=q.dtype, device=q.device)
+    grouped_heads(q, absorb, out=out, in_stride=np_ + xp, out_stride=Rp + xp)
+    native().latent_rotate(_ptr(q), q.stride(0), np_, _ptr(angles), d, T, H, xp, _ptr(out),
+                           out.stride(0), Rp, bf, _stream())
+    return out
+
+
+def latent_attention(q: torch.Tensor, pages: torch.Tensor, block_tables, cu_q, positions,
+                     scale: float, window: int, H: int, Rp: int, ws=None, part_tokens: int = 512,
+                     num_decode: int = 0) -> torch.Tensor:
+    """Attention of query rows (``latent_query``) over latent pages: row t of a
+    sequence sees the ``window`` last positions up to its own; returns the
+    weighted sums of latents [T, H * Rp].  Rows before ``num_decode`` are the
+    first row of sequence t."""
+    T = q.shape[0]
+    _, one, BS, D = pages.shape
+    S = cu_q.numel() - 1
+    if not q.is_cuda:
+        return ref.latent_attention(q, pages, block_tables, cu_q, positions, scale, window, H, Rp)
+    bf = _rows_dtype(q, "q")
+    _chk(one == 1 and BS == 32 and q.shape[1] == H * D and q.is_contiguous()
+         and pages.dtype == q.dtype and 0 < Rp < D and window > 0, "latent_attention")
+    _meta(S, cu_q=cu_q)
+    _meta(T, positions=positions)
+    _chk(block_tables.dtype == torch.int32 and block_tables.shape[0] >= S
+         and block_tables.stride(1) == 1, "block tables")
+    out = torch.empty((T, H * Rp), dtype=q.dtype, device=q.device)
+    args = (_ptr(q), _ptr(pages), _ptr(block_tables), block_tables.stride(0), _ptr(cu_q), S,
+            _ptr(positions), T)
+    tail = (_ptr(out), H, Rp, D, float(scale), window)
+    if not bf or D != Rp + 64 or Rp not in LATENT_RANKS:
+        native().latent_any(*args, *tail, bf, _stream())
+        return out
+    # decode steps split a row's keys over workgroups until the chip is filled
+    parts = ws.max_parts if ws is not None and T <= num_decode else 1
+    if parts > 1:
+        _chk(ws.part_o.numel() >= T * H * parts * Rp and ws.part_ml.numel() >= T * H * parts * 2,
+             "latent_attention workspace")
+    native().latent_rows(*args, num_decode, _ptr(out), _ptr(ws.part_o) if ws else 0,
+                         _ptr(ws.part_ml) if ws else 0, *tail[1:], 128, parts, _stream())
+    return out
+
+
+LATENT_RANKS = (64, 128, 256, 512)   # latent widths of the MFMA kernel
+LATENT_QT = 128            # query rows per prefill workgroup (latent.hip)
+
+
+def latent_prefill_ok(np_: int, xp: int, vp: int) -> bool:
+    """Head sizes of the expanded prefill kernel."""
+    return False
+
+
+@dataclass
+class LatentRows:
+    """Key rows a step's multi-token sequences see, gathered back to back."""
+    seqs: torch.Tensor      # int32 [sequences + 1, 2]: first gathered row, first position
+    tiles: torch.Tensor     # int32 [n, 2]: sequence, first query row
+    n: int                  # gathered rows
+
+
+def latent_rows(qlens, ctx, window: int) -> tuple[np.ndarray, np.ndarray, int]:
+    """Host plan of ``LatentRows``: a sequence with ``qlens`` new rows up to
+    position ctx - 1 sees positions from ctx - qlens - window + 1."""
+    ctx, qlens = np.asarray(ctx, np.int64), np.asarray(qlens, np.int64)
+    k0 = np.maximum(ctx - qlens - (window - 1), 0)
+    first = np.concatenate([[0], np.cumsum(ctx - k0)])
+    seqs = np.stack([first, np.append(k0, 0)], 1).astype(np.int32)
+    return seqs, row_tiles(qlens, LATENT_QT), int(first[-1])

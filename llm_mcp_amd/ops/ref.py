@@ -404,15 +404,15 @@ def _unit(x, eps):
 
 
 def sandwich_norm(residual, eps, y=None, w_post=None, w_pre=None, ids=None, table=None,
-                  rows=None, dtype=torch.bfloat16):
-    r = table[ids.long()].float() if ids is not None else residual
+                  rows=None, dtype=torch.bfloat16, scale=1.0):
+    r = table[ids.long()].float() * scale if ids is not None else residual
     if rows is not None:
         r, y = r[rows], None if y is None else y[rows]
     if y is not None:
         r = r + _unit(y.float(), eps) * w_post
     if rows is None:
         residual.copy_(r)
-    return None if w_pre is None else (_unit(r, eps) * w_pre).to(dtype)
+    return (r if w_pre is None else _unit(r, eps) * w_pre).to(dtype)
 
 
 def gated_norm(x, gate, w, groups, eps, gate_first):
@@ -447,8 +447,8 @@ def _conv_rows(u, w, bias, in_bias, state, cu_q, ctx, slots):
     return y if bias is None else y + bias
 
 
-def short_conv(u, w, bias, state, cu_q, ctx, slots, out, silu):
-    y = _conv_rows(u, w, bias, None, state, cu_q, ctx, slots)
+def short_conv(u, w, bias, state, cu_q, ctx, slots, out, silu, in_bias=None):
+    y = _conv_rows(u, w, bias, in_bias, state, cu_q, ctx, slots)
     out.copy_(torch.nn.functional.silu(y) if silu else y)
 
 
@@ -491,3 +491,112 @@ def linear_scan(q, k, v, out, state, cu_q, ctx, slots, hpg, decay, dt, skip, sil
                 o = o + skip[:, None] * vs[t]
             out[a + t, :H * P] = o.reshape(-1).to(out.dtype)
         state[slot] = S
+
+
+def rglru(u, y, y_bias, gates, gate_bias, log_a, out, state, cu_q, ctx, slots):
+    """See ops.rglru; one token after the other, fp32.  gates [n, 2 bp, bp]."""
+    T, C = u.shape
+    n, _, bp = gates.shape
+    x = u.float()
+    z = torch.einsum("tnk,nzok->tzno", x.view(T, n, bp),
+                     gates.float().view(n, 2, bp, bp)).reshape(T, 2, C)
+    r, i = torch.sigmoid(z + gate_bias).unbind(1)
+    la = log_a * r
+    b = torch.sqrt(-torch.expm1(2.0 * la)) * i * x
+    a = torch.exp(la)
+    g = torch.nn.functional.gelu(y.float() + y_bias, approximate="tanh")
+    for s in range(len(ctx)):
+        t0, t1, slot = int(cu_q[s]), int(cu_q[s + 1]), int(slots[s])
+        if slot < 0:
+            continue
+        S = torch.zeros(C) if int(ctx[s]) == t1 - t0 else state[slot].clone()
+        for t in range(t0, t1):
+            S = a[t] * S + b[t]
+            out[t] = (S * g[t]).to(out.dtype)
+        state[slot] = S
+
+
+# ------------------------------------------------------- latent attention ---
+def rope_angles(positions, freqs):
+    a = positions.double()[:, None] * freqs
+    return torch.cat([a.cos(), a.sin()], 1).float()
+
+
+def rotate(x, ang):
+    """x [T, ..., d] (halves paired) by the angles of ``rope_angles`` [T, d]."""
+    h = x.shape[-1] // 2
+    cs = ang.reshape((x.shape[0],) + (1,) * (x.dim() - 2) + (2 * h,))
+    c, s = cs[..., :h], cs[..., h:]
+    a, b = x[..., :h].float(), x[..., h:].float()
+    return torch.cat([a * c - b * s, b * c + a * s], -1)
+
+
+def latent_prep(p, qr, qp, q_norm, R, c_norm, ang, slots, pages, Rp, eps):
+    T, d = ang.shape
+    cq = torch.zeros((T, qp), dtype=p.dtype)
+    cq[:, :qr] = (_unit(p[:, :qr].float(), eps) * q_norm[:qr]).to(p.dtype)
+    row = torch.zeros((T, pages.shape[3]))
+    row[:, :R] = _unit(p[:, qp:qp + R].float(), eps) * c_norm[:R]
+    row[:, Rp:Rp + d] = rotate(p[:, qp + Rp:qp + Rp + d], ang)
+    BS = pages.shape[2]
+    for t in range(T):
+        s = int(slots[t])
+        if s >= 0:
+            pages[s // BS, 0, s % BS] = row[t].to(pages.dtype)
+    return cq
+
+
+def latent_query(q, absorb, ang, H, np_, xp, Rp):
+    T, d = q.shape[0], ang.shape[1]
+    q3 = q.view(T, H, np_ + xp)
+    out = torch.zeros((T, H, Rp + xp), dtype=q.dtype)
+    out[..., :Rp] = torch.einsum("thk,hrk->thr", q3[..., :np_].float(), absorb.float()).to(q.dtype)
+    out[..., Rp:Rp + d] = rotate(q3[..., np_:np_ + d], ang[:T]).to(q.dtype)
+    return out.view(T, -1)
+
+
+def latent_attention(ql, pages, block_tables, cu_q, positions, scale, window, H, Rp):
+    T = ql.shape[0]
+    BS = pages.shape[2]
+    q = ql.view(T, H, -1).float()
+    out = torch.zeros((T, H, Rp), dtype=ql.dtype)
+    cu = [int(x) for x in cu_q]
+    for s in range(len(cu) - 1):
+        for t in range(cu[s], min(cu[s + 1], T)):
+            p = int(positions[t])
+            j = torch.arange(max(0, p - window + 1), p + 1)
+            k = pages[block_tables[s, j // BS].long(), 0, j % BS].float()
+            w = torch.softmax((q[t] @ k.T) * scale, -1)
+            out[t] = (w @ k[:, :Rp]).to(out.dtype)
+    return out.view(T, -1)
+
+
+# ----------------------------------------------------- grouped products -----
+def clamped_glu(g, u, limit):
+    g = torch.clamp(g, max=limit)
+    u = torch.clamp(u, -limit, limit)
+    return g * torch.sigmoid(1.702 * g) * (u + 1.0)
+
+
+def moe_route(h, w, top, extra):
+    z = h.float() @ w.float().t()
+    v, e = torch.sort(z, dim=-1, descending=True, stable=True)
+    T, E = z.shape
+    ids = torch.cat([e[:, :top], torch.arange(E, E + extra).expand(T, extra)], 1)
+    wts = torch.cat([torch.softmax(v[:, :top], -1), torch.ones(T, extra)], 1)
+    return ids.to(torch.int32), wts
+
+
+def grouped_rows(x, w, src, off, gather, limit):
+    """Rows off[e]..off[e+1] of the expert order times w[e]^T."""
+    K = w.shape[2]
+    out = torch.zeros((src.numel(), w.shape[1] // (2 if limit is not None else 1)), dtype=x.dtype)
+    for e in range(w.shape[0]):
+        a, b = int(off[e]), int(off[e + 1])
+        rows = x[src[a:b].long()] if gather else x[a:b]
+        y = rows[:, :K].float() @ w[e].float().t()
+        if limit is not None:
+            y = y.view(b - a, w.shape[1] // 32, 2, 16)
+            y = clamped_glu(y[:, :, 0], y[:, :, 1], float(limit[e])).reshape(b - a, out.shape[1])
+        out[a:b] = y.to(x.dtype)
+    return out

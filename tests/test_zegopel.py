@@ -14,7 +14,7 @@ import zegopel_oracle as oracle
 from llm_mcp_amd.engine.engine import EngineConfig, GenRequest, LLMEngine, SamplingParams
 from llm_mcp_amd.models import config as mc
 from llm_mcp_amd.models.registry import model_class
-from llm_mcp_amd.models.weights import load_weights, save_zegopel
+from llm_mcp_amd.models.weights import load_weights, save_layer_list
 from llm_mcp_amd.models.zegopel import ZegopelModel, tensor_shapes
 from zegopel_cases import CASES, config, layer, shapes, tokens, weights
 from zegopel_cases import ATTN, LIGHT, MAMBA, MLP
@@ -28,7 +28,7 @@ TOL = {"float32": 2e-5, "bfloat16": 0.04}
 
 
 def product_config(cfg, name="case"):
-    return mc._zegopel_from_json(cfg, name)
+    return mc.ZegopelConfig.from_json(cfg, name)
 
 
 def engine(cfg, W, device, dtype, tokens=512, seqs=4, graphs=False, **kw):
@@ -286,7 +286,7 @@ def test_checkpoint_directory_round_trip(tmp_path):
     W = weights(cfg)
     pc = product_config(cfg)
     assert {k: tuple(v) for k, v in tensor_shapes(pc).items()} == shapes(cfg)
-    save_zegopel(W, pc, str(tmp_path))
+    save_layer_list(W, pc, str(tmp_path))
     back = mc.resolve(str(tmp_path))
     assert back.family == "zegopel" and model_class(back) is ZegopelModel
     assert (back.layers, back.vocab_size, back.hidden_size, back.rms_eps) == \
@@ -295,7 +295,7 @@ def test_checkpoint_directory_round_trip(tmp_path):
     assert all(torch.equal(W[k], W2[k]) for k in W)
     assert back.params == sum(t.numel() for t in W.values())
     bad = dict(W, head=W["head"][:-1])
-    save_zegopel(bad, pc, str(tmp_path))
+    save_layer_list(bad, pc, str(tmp_path))
     with pytest.raises(ValueError, match="head"):
         load_weights(str(tmp_path), back, "cpu")
 
@@ -361,7 +361,7 @@ def test_trace_replay(tmp_path):
     from llm_mcp_amd.engine import trace
     cfg = CASES["mixed"]
     W = weights(cfg)
-    save_zegopel(W, product_config(cfg), str(tmp_path / "m"))
+    save_layer_list(W, product_config(cfg), str(tmp_path / "m"))
     e = trace.build_engine(str(tmp_path / "m"), "float32", 130, 4, "cpu")
     assert e.num_blocks == 5 and len(e.states[0]) == 4
     toks = tokens(cfg, 40)
