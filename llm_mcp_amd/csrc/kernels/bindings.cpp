@@ -59,6 +59,10 @@ int latent_rotate(const void*, long, int, const float*, int, int, int, int, void
                   hipStream_t);
 int latent_any(const void*, const void*, const int*, int, const int*, int, const int*, int, void*,
                int, int, int, float, int, int, hipStream_t);
+int latent_gather(const void*, const int*, int, const int*, int, int, int, void*, hipStream_t);
+int latent_prefill(const void*, long, const void*, const void*, const float*, const int*,
+                   const int*, int, const int*, const int*, const void*, long, void*, long, int, int,
+                   int, int, int, int, float, int, hipStream_t);
 int latent_rows(const void*, const void*, const int*, int, const int*, int, const int*, int, int,
                 void*, float*, float*, int, int, int, float, int, int, int, hipStream_t);
 int gated_norm(void*, long, const void*, long, const void*, long, const float*, int, int, int, int,
@@ -289,6 +293,22 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                           P<int>(positions), rows, P<void>(out), H, Rp, D, scale, window, is_bf16,
                           S(stream)),
           "latent_any");
+  });
+  m.def("latent_gather", [](uptr pages, uptr bt, int bt_stride, uptr seqs, int nseq, int n, int D,
+                            uptr out, uptr stream) {
+    check(lmx::latent_gather(P<void>(pages), P<int>(bt), bt_stride, P<int>(seqs), nseq, n, D,
+                             P<void>(out), S(stream)),
+          "latent_gather");
+  });
+  m.def("latent_prefill", [](uptr q, long q_ld, uptr kv, uptr lat, uptr ang, uptr seqs, uptr tiles,
+                             int ntiles, uptr cu_q, uptr ctx, uptr gate, long gate_ld, uptr out,
+                             long out_ld, int H, int NP, int VP, int D, int Rp, int d, float scale,
+                             int window, uptr stream) {
+    check(lmx::latent_prefill(P<void>(q), q_ld, P<void>(kv), P<void>(lat), P<float>(ang),
+                              P<int>(seqs), P<int>(tiles), ntiles, P<int>(cu_q), P<int>(ctx),
+                              P<void>(gate), gate_ld, P<void>(out), out_ld, H, NP, VP, D, Rp, d,
+                              scale, window, S(stream)),
+          "latent_prefill");
   });
   m.def("latent_rows", [](uptr q, uptr pages, uptr bt, int bt_stride, uptr cu_q, int nseq,
                           uptr positions, int rows, int num_decode, uptr out, uptr part_o,

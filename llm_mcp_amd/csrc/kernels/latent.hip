@@ -9,6 +9,8 @@
 //   latent_rows    attention on latents (MFMA): a workgroup serves one query
 //                  row, its heads are the MFMA columns
 //   latent_any     the same for fp32 and for other sizes (fp32 arithmetic)
+//   latent_gather  the cached rows a step's prompt rows see, back to back
+//   latent_prefill prompt rows on keys and values expanded from those rows
 #include "common.h"
 
 namespace lmx {
@@ -426,6 +428,264 @@ __global__ void __launch_bounds__(64) latent_reduce_kernel(
   }
 }
 
+// ------------------------------------------------------------- prompt rows ----
+// seqs[s] = (first gathered row, first position) of sequence s, S + 1 entries
+__device__ __forceinline__ int gathered_seq(const int* __restrict__ seqs, int S, int row) {
+  int lo = 0, hi = S - 1;
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (seqs[2 * mid] <= row) lo = mid; else hi = mid - 1;
+  }
+  return lo;
+}
+
+// grid ceil(n / 4), block 256: one wave per row
+__global__ void __launch_bounds__(256) latent_gather_kernel(const bf16_t* __restrict__ pages,
+                                                            const int* __restrict__ bt,
+                                                            int bt_stride,
+                                                            const int* __restrict__ seqs, int S,
+                                                            int n, int D, bf16_t* __restrict__ out) {
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (row >= n) return;
+  const int s = gathered_seq(seqs, S, row), pos = row - seqs[2 * s] + seqs[2 * s + 1];
+  const bf16_t* src = pages + ((long)bt[(long)s * bt_stride + pos / BS] * BS + pos % BS) * D;
+  for (int c = lane * 8; c < D; c += 512)
+    *reinterpret_cast<u16x8*>(out + (long)row * D + c) = *reinterpret_cast<const u16x8*>(src + c);
+}
+
+// 8 elements j0.. of a rotated part x [d of 64] by the angles an [d] (cos | sin)
+__device__ __forceinline__ bf16x8_t rotated_frag(const bf16_t* __restrict__ x,
+                                                 const float* __restrict__ an, int d, int j0) {
+  const int half = d / 2;
+  bf16x8_t o = {0, 0, 0, 0, 0, 0, 0, 0};
+  if (j0 >= d) return o;
+  if (half % 8 == 0) {
+    const bool up = j0 >= half;
+    const int i0 = up ? j0 - half : j0;
+    const bf16x8_t lo = load_frag16B(x + i0), hi = load_frag16B(x + half + i0);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float a = bf2f((uint16_t)lo[e]), b = bf2f((uint16_t)hi[e]);
+      const float cv = an[i0 + e], sv = an[half + i0 + e];
+      o[e] = (short)f2bf(up ? b * cv + a * sv : a * cv - b * sv);
+    }
+    return o;
+  }
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const int j = j0 + e, i = j < half ? j : j - half;
+    if (j < d) {
+      const float a = bf2f(x[i]), b = bf2f(x[half + i]), cv = an[i], sv = an[half + i];
+      o[e] = (short)f2bf(j < half ? a * cv - b * sv : b * cv + a * sv);
+    }
+  }
+  return o;
+}
+
+template <int CH>
+__device__ __forceinline__ int pre_swz(int row) {
+  return CH % 16 == 0 ? row & 15 : (row >> 1) & 7;
+}
+
+// One head of one 128-query tile per workgroup; a wave owns NG groups of 16
+// queries (MFMA columns).  Keys W_uk c | rotated part and values W_uv c come in
+// 64-key tiles by LDS-DMA, double-buffered; S^T leaves the weights where the
+// PV product reads them (permuted keys, as in attention.hip), V^T comes from
+// the value rows with the transposing LDS read.  Weights enter PV as a bf16
+// pair.  grid tiles x heads, block 256.
+struct LatentPre {
+  const bf16_t* q;        // rows [H][NP + 64], not rotated
+  const bf16_t* kv;       // gathered rows [H][NP + VP]
+  const bf16_t* lat;      // gathered rows [D], rotated key part from Rp
+  const float* ang;       // [rows][d]
+  const int *seqs, *tiles, *cu_q, *ctx;
+  const bf16_t* gate;     // rows [H][VP]
+  bf16_t* out;            // rows [H][VP]
+  long q_ld, gate_ld, out_ld;
+  int ntiles, H, D, Rp, d, window;
+  float scale;
+};
+
+template <int NP, int VP>
+__global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatentPre p) {
+  constexpr int NG = 2, KD = NP + 64, KS = KD / 32, KC = KD / 8, VC = VP / 8, VT = VP / 16;
+  constexpr int KN = TK * KC / 256, VN = TK * VC / 256;   // DMA instructions per tile
+  extern __shared__ __attribute__((aligned(16))) char lp_smem[];
+  bf16_t* const sk = reinterpret_cast<bf16_t*>(lp_smem);            // [2][TK][KD]
+  bf16_t* const sv = sk + 2 * TK * KD;                              // [2][TK][VP]
+  const int tid = threadIdx.x, lane = tid & 63, c = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  // a head's tiles are consecutive on one XCD: they share its keys in L2; the
+  // list is walked backwards (long key walks first)
+  const int lin = xcd_remap(blockIdx.x, gridDim.x);
+  const int h = lin / p.ntiles, tile = p.ntiles - 1 - lin % p.ntiles;
+  const int s = p.tiles[2 * tile], q0 = p.tiles[2 * tile + 1];
+  const int qbeg = p.cu_q[s], qlen = p.cu_q[s + 1] - qbeg, p0 = p.ctx[s] - qlen;
+  const int k0 = p.seqs[2 * s + 1];                       // first gathered position
+  const long krow = (long)p.seqs[2 * s] - k0;             // gathered row of position 0
+  const int wq1 = min(q0 + 128, qlen);                    // one past the tile's last query
+  const int kmax = p0 + wq1 - 1;
+  const int t_lo = k0 + (max(p0 + q0 - p.window + 1, k0) - k0) / TK * TK;
+
+  const bf16_t* src[KN + VN];
+  int srow[KN + VN];
+  long sld[KN + VN];
+  const long kvld = (long)p.H * (NP + VP);
+#pragma unroll
+  for (int i = 0; i < KN; ++i) {
+    const int e = i * 256 + tid, r = e / KC, ch = (e % KC) ^ pre_swz<KC>(r);
+    srow[i] = r;
+    const bool kr = ch >= NP / 8;
+    src[i] = kr ? p.lat + p.Rp + 8 * (ch - NP / 8) : p.kv + (long)h * (NP + VP) + 8 * ch;
+    sld[i] = kr ? p.D : kvld;
+  }
+#pragma unroll
+  for (int i = 0; i < VN; ++i) {
+    const int e = i * 256 + tid, r = e / VC, ch = (e % VC) ^ pre_swz<VC>(r);
+    srow[KN + i] = r;
+    src[KN + i] = p.kv + (long)h * (NP + VP) + NP + 8 * ch;
+    sld[KN + i] = kvld;
+  }
+  auto stage = [&](int t0, int buf) {
+#pragma unroll
+    for (int i = 0; i < KN + VN; ++i) {
+      bf16_t* dst = i < KN ? sk + buf * TK * KD + (i * 256 + wave * 64) * 8
+                           : sv + buf * TK * VP + ((i - KN) * 256 + wave * 64) * 8;
+      lds_dma16(src[i] + (krow + min(t0 + srow[i], kmax)) * sld[i], dst);
+    }
+  };
+  stage(t_lo, 0);
+
+  int pos[NG];
+  bf16x8_t qf[NG][KS];
+#pragma unroll
+  for (int n = 0; n < NG; ++n) {
+    const int qi = q0 + (wave * NG + n) * 16 + c;
+    pos[n] = p0 + qi;
+    const long row = qbeg + min(qi, qlen - 1);
+    const bf16_t* qr = p.q + row * p.q_ld + (long)h * KD;
+#pragma unroll
+    for (int ks = 0; ks < NP / 32; ++ks) qf[n][ks] = load_frag16B(qr + 32 * ks + 8 * g);
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks)
+      qf[n][NP / 32 + ks] = rotated_frag(qr + NP, p.ang + row * p.d, p.d, 32 * ks + 8 * g);
+  }
+  const int w0 = q0 + wave * NG * 16;                     // the wave's first query
+  const bool idle = w0 >= qlen;
+  const int whi = p0 + min(w0 + NG * 16, qlen) - 1;       // its last query's position
+  const int wlo = p0 + w0 - p.window + 1;                 // first key any of them sees
+  float m[NG], l[NG];
+  f32x4_t acc[NG][VT];
+#pragma unroll
+  for (int n = 0; n < NG; ++n) {
+    m[n] = -INFINITY;
+    l[n] = 0.f;
+#pragma unroll
+    for (int i = 0; i < VT; ++i) acc[n][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
+  const float sl = p.scale * LOG2E;
+  int buf = 0;
+  for (int t0 = t_lo; t0 <= kmax; t0 += TK, buf ^= 1) {
+    dma_barrier();                    // the tile landed; every wave is done with the other buffer
+    if (t0 + TK <= kmax) stage(t0 + TK, buf ^ 1);
+    if (idle || t0 > whi || t0 + TK <= wlo) continue;
+    const bf16_t* kt = sk + buf * TK * KD;
+    const bf16_t* vt = sv + buf * TK * VP;
+    f32x4_t sc[NG][4];
+#pragma unroll
+    for (int kb = 0; kb < 4; ++kb) {
+      const int r = 16 * kb + c;
+#pragma unroll
+      for (int n = 0; n < NG; ++n) sc[n][kb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const bf16x8_t kf = load_frag16B(kt + r * KD + 8 * ((4 * ks + g) ^ pre_swz<KC>(r)));
+#pragma unroll
+        for (int n = 0; n < NG; ++n) sc[n][kb] = mfma16(kf, qf[n][ks], sc[n][kb]);
+      }
+    }
+    // every key of the tile visible to every query of the wave: no mask
+    const bool mask = t0 + TK - 1 > p0 + w0 || t0 < whi - p.window + 1;
+    bf16x8_t ph[NG][2], pl[NG][2];
+    float al[NG];
+    bool grew = false;
+#pragma unroll
+    for (int n = 0; n < NG; ++n) {
+      float mx = -INFINITY;
+      if (mask) {
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int key = t0 + 16 * kb + 4 * g + r;
+            if (key > pos[n] || key <= pos[n] - p.window) sc[n][kb][r] = -INFINITY;
+          }
+      }
+#pragma unroll
+      for (int kb = 0; kb < 4; ++kb)
+        mx = fmaxf(mx, fmaxf(fmaxf(sc[n][kb][0], sc[n][kb][1]), fmaxf(sc[n][kb][2], sc[n][kb][3])));
+      mx = xmax(mx) * sl;
+      const float mn = fmaxf(m[n], mx);
+      const float mu = mn == -INFINITY ? 0.f : mn;
+      al[n] = fast_exp2(m[n] - mu);
+      grew |= mn > m[n];
+      m[n] = mn;
+      float ps = 0.f;
+#pragma unroll
+      for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float w = fast_exp2(sc[n][kb][r] * sl - mu);
+          ps += w;
+          const uint16_t hb = f2bf(w);
+          ph[n][kb >> 1][4 * (kb & 1) + r] = (short)hb;
+          pl[n][kb >> 1][4 * (kb & 1) + r] = (short)f2bf(w - bf2f(hb));
+        }
+      l[n] = l[n] * al[n] + ps;       // this lane's keys only; summed at the end
+    }
+    if (__ballot(grew)) {
+#pragma unroll
+      for (int n = 0; n < NG; ++n)
+#pragma unroll
+        for (int i = 0; i < VT; ++i) acc[n][i] *= al[n];
+    }
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+      const int ra = 32 * ks + 4 * g + (c >> 2), rb = ra + 16;
+#pragma unroll
+      for (int i = 0; i < VT; ++i) {
+        const int d0 = 16 * i + 4 * (c & 3);
+        const s16x4_t va = lds_read_tr(vt + ra * VP + 8 * ((d0 >> 3) ^ pre_swz<VC>(ra)) + (d0 & 7));
+        const s16x4_t vb = lds_read_tr(vt + rb * VP + 8 * ((d0 >> 3) ^ pre_swz<VC>(rb)) + (d0 & 7));
+        const bf16x8_t vf = {va[0], va[1], va[2], va[3], vb[0], vb[1], vb[2], vb[3]};
+#pragma unroll
+        for (int n = 0; n < NG; ++n) {
+          acc[n][i] = mfma16(vf, ph[n][ks], acc[n][i]);
+          acc[n][i] = mfma16(vf, pl[n][ks], acc[n][i]);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int n = 0; n < NG; ++n) {
+    const float L = xsum(l[n]);
+    const int qi = q0 + (wave * NG + n) * 16 + c;
+    if (qi >= qlen) continue;
+    const float inv = 1.f / L;
+    const long row = qbeg + qi;
+#pragma unroll
+    for (int i = 0; i < VT; ++i) {
+      const long col = (long)h * VP + 16 * i + 4 * g;
+      const bf16x4_t gt = *reinterpret_cast<const bf16x4_t*>(p.gate + row * p.gate_ld + col);
+      bf16x4_t o;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        o[r] = (short)f2bf(acc[n][i][r] * inv / (1.f + __expf(-bf2f((uint16_t)gt[r]))));
+      *reinterpret_cast<bf16x4_t*>(p.out + row * p.out_ld + col) = o;
+    }
+  }
+}
+
 }  // namespace
 
 int rope_angles(const int* positions, const double* freqs, int T, int n, float* out,
@@ -519,6 +779,46 @@ int latent_rows(const void* q, const void* pages, const int* bt, int bt_stride, 
   if (max_parts > 1)
     latent_reduce_kernel<<<dim3(H, rows), dim3(64), 0, stream>>>(
         part_o, part_ml, positions, (bf16_t*)out, H, Rp, window, part_keys, max_parts);
+  return (int)hipGetLastError();
+}
+
+int latent_gather(const void* pages, const int* bt, int bt_stride, const int* seqs, int S, int n,
+                  int D, void* out, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (S < 1 || D % 8) return -1;
+  latent_gather_kernel<<<dim3((n + 3) / 4), dim3(256), 0, stream>>>(
+      (const bf16_t*)pages, bt, bt_stride, seqs, S, n, D, (bf16_t*)out);
+  return (int)hipGetLastError();
+}
+
+int latent_prefill(const void* q, long q_ld, const void* kv, const void* lat, const float* ang,
+                   const int* seqs, const int* tiles, int ntiles, const int* cu_q, const int* ctx,
+                   const void* gate, long gate_ld, void* out, long out_ld, int H, int NP, int VP,
+                   int D, int Rp, int d, float scale, int window, hipStream_t stream) {
+  if (ntiles <= 0) return 0;
+  if (H < 1 || D != Rp + 64 || D % 8 || d < 2 || d % 2 || d > 64 || window < 1 || q_ld % 8 ||
+      gate_ld % 4 || out_ld % 4)
+    return -1;
+  const LatentPre p{(const bf16_t*)q, (const bf16_t*)kv, (const bf16_t*)lat, ang, seqs, tiles, cu_q,
+                    ctx, (const bf16_t*)gate, (bf16_t*)out, q_ld, gate_ld, out_ld, ntiles, H, D, Rp,
+                    d, window, scale};
+#define LMX_LP(NPV, VPV)                                                                       \
+  {                                                                                            \
+    constexpr int smem = 2 * TK * (NPV + 64 + VPV) * 2;                                        \
+    static bool attr = false;                                                                  \
+    if (smem > 65536 && !attr) {                                                               \
+      (void)hipFuncSetAttribute((const void*)latent_prefill_kernel<NPV, VPV>,                  \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, smem);             \
+      attr = true;                                                                             \
+    }                                                                                          \
+    latent_prefill_kernel<NPV, VPV><<<dim3(ntiles * H), dim3(256), smem, stream>>>(p);         \
+  }
+  if (NP == 64 && VP == 64) LMX_LP(64, 64)
+  else if (NP == 64 && VP == 128) LMX_LP(64, 128)
+  else if (NP == 128 && VP == 64) LMX_LP(128, 64)
+  else if (NP == 128 && VP == 128) LMX_LP(128, 128)
+  else return -2;
+#undef LMX_LP
   return (int)hipGetLastError();
 }
 

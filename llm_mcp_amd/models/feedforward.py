@@ -60,7 +60,7 @@ class MixtureOfExperts:
     every token uses with weight 1: one grouped product covers all of them."""
 
     def __init__(self, m: dict, width: int):
-        self.width, self.kp = width, _up(width, 64)
+        self.width, self.kp, self.np = width, _up(width, 64), _up(width, 16)
         self.E, self.top = m["router"]["experts"], m["router"]["top"]
         if not 0 < self.top <= self.E:
             raise ValueError("moe: top experts out of range")
@@ -86,7 +86,7 @@ class MixtureOfExperts:
 
         def expert(gate, up, down):
             w1 = ops.interleave_gate_up(_fuse_rows([gate, up], [fp, fp]), 16)
-            return put(_pad_cols(w1, kp)), put(_pad_cols(down, fp))
+            return put(_pad_cols(w1, kp)), put(_pad_cols(_fuse_rows([down], [self.np]), fp))
         each = [expert(*(get(f"e{e}.{n}") for n in ("gate", "up", "down"))) for e in range(self.E)]
         if self.shared:
             gate, up, down = (get(f"shared.{n}") for n in ("gate", "up", "down"))

@@ -359,7 +359,7 @@ class LatentAttentionMixer(Mixer):
         self.proj = {"in": (rows + self.tail, width), "uq": (H * (self.np + self.xp), self.qp),
                      "o": (width, H * self.vp)}
         self.expand = ops.latent_prefill_ok(self.np, self.xp, self.vp)
-        if self.expand:
+        if self.expand:            # prompt rows of bf16 engines
             self.plan_key = ("latent", self.window)
 
     def build_plan(self, qlens, ctx, seq0):
@@ -408,7 +408,8 @@ class LatentAttentionMixer(Mixer):
                              inp.slots, pages, self.Rp, self.eps)
         q = ops.linear(cq, self.w_uq)
         out = torch.empty((T, H * self.vp), dtype=h.dtype, device=h.device)
-        rows = inp.aux.get(self.plan_key) if self.expand and q.dtype == torch.bfloat16 else None
+        fast = self.expand and q.is_cuda and q.dtype == torch.bfloat16
+        rows = inp.aux.get(self.plan_key) if fast else None
         n = nd if rows is not None else T              # rows on latents: the first n
         if n:
             ql = ops.latent_query(q[:n], self.absorb, ang, H, self.np, self.xp, self.Rp)
@@ -419,7 +420,7 @@ class LatentAttentionMixer(Mixer):
         if rows is not None:
             ops.latent_prefill(q, pages, rows, self.w_kv, ang, inp.block_tables[nd:],
                                inp.cu_q[nd:], inp.context_lens[nd:], self.scale, self.window, H,
-                               self.np, self.xp, self.vp, self.Rp, gate, out)
+                               self.np, self.vp, self.Rp, gate, out)
         return ops.linear(out, self.w_o, defer=True)
 
 

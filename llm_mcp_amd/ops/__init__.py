@@ -1801,5 +1801,5 @@ from .grouped import (GroupedWeight, Mixture, MoePlan, Route, grouped_heads,  # 
                       grouped_linear, moe_plan, moe_route, pack_grouped)
 from .mixers import (RGLRU_MAX_BLOCK, RGLRU_TILE, LatentRows, ScanSegments,  # noqa: E402,F401
                      attention_any, conv_qkv_cache, gated_norm, latent_attention,
-                     latent_prefill_ok, latent_prep, latent_query, linear_scan, rglru,
+                     latent_prefill, latent_prefill_ok, latent_prep, latent_query, linear_scan, rglru,
                      rope_angles, rope_freqs, sandwich_norm, scan_segments, short_conv)

@@ -13,6 +13,7 @@ slots are never cleared.
 """
 from __future__ import annotations
 
+import importlib
 import math
 from dataclasses import dataclass
 
@@ -61,7 +62,7 @@ def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tens
     The gains are fp32 vectors."""
     T, d = residual.shape
     if not residual.is_cuda:
-        y = y.sum() if isinstance(y, Mixture) else y
+        y = y.sum()[:, :d] if isinstance(y, Mixture) else y
         return ref.sandwich_norm(residual, eps, y, w_post, w_pre, ids, table, rows, dtype, scale)
     _chk(residual.dtype == torch.float32 and residual.is_contiguous(), "residual: fp32 rows")
     _f32(w_post, d, "w_post"); _f32(w_pre, d, "w_pre")
@@ -71,11 +72,11 @@ def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tens
         _chk((y.M, y.N) == (T, d), "sandwich_norm partials shape")
         yp, y_ld, slabs, sstride = _ptr(y.slabs), d, y.S, y.M * y.N
     elif isinstance(y, Mixture):
-        _chk(y.rows.shape[1] == d and y.rows.is_contiguous() and y.rows.dtype == dtype
+        _chk(y.rows.shape[1] >= d and y.rows.stride(1) == 1 and y.rows.dtype == dtype
              and y.pos.shape == y.weights.shape and y.pos.shape[0] == T
              and y.pos.dtype == torch.int32 and y.weights.dtype == torch.float32
              and y.pos.is_contiguous() and y.weights.is_contiguous(), "sandwich_norm mixture")
-        yp, y_ld, mix = _ptr(y.rows), d, (_ptr(y.pos), _ptr(y.weights), y.pos.shape[1])
+        yp, y_ld, mix = _ptr(y.rows), y.rows.stride(0), (_ptr(y.pos), _ptr(y.weights), y.pos.shape[1])
     elif y is not None:
         _chk(y.shape == (T, d) and y.stride(1) == 1 and y.dtype == dtype, "sandwich_norm y rows")
         yp, y_ld = _ptr(y), y.stride(0)
@@ -480,8 +481,8 @@ LATENT_QT = 128            # query rows per prefill workgroup (latent.hip)
 
 
 def latent_prefill_ok(np_: int, xp: int, vp: int) -> bool:
-    """Head sizes of the expanded prefill kernel."""
-    return False
+    """Head sizes of the expanded prefill kernel (bf16)."""
+    return np_ in (64, 128) and xp == 64 and vp in (64, 128)
 
 
 @dataclass
@@ -500,3 +501,36 @@ def latent_rows(qlens, ctx, window: int) -> tuple[np.ndarray, np.ndarray, int]:
     first = np.concatenate([[0], np.cumsum(ctx - k0)])
     seqs = np.stack([first, np.append(k0, 0)], 1).astype(np.int32)
     return seqs, row_tiles(qlens, LATENT_QT), int(first[-1])
+
+
+def latent_prefill(q: torch.Tensor, pages: torch.Tensor, rows: LatentRows, w_kv: torch.Tensor,
+                   angles: torch.Tensor, block_tables, cu_q, ctx, scale: float, window: int, H: int,
+                   np_: int, vp: int, Rp: int, gate: torch.Tensor, out: torch.Tensor) -> None:
+    """Prompt rows (bf16, GPU) of the sequences of ``block_tables`` / ``cu_q`` /
+    ``ctx``: the cached rows they see are gathered, expanded by ``w_kv`` (H x
+    [np_ key | vp value] rows of latents) and attended to; ``q`` as projected
+    (H x [np_ | 64 to rotate]).  Output rows times sigmoid(gate), H x vp."""
+    linear = importlib.import_module(__package__).linear
+    S, D = ctx.numel(), pages.shape[3]
+    d = angles.shape[1]
+    for t, w in ((q, H * (np_ + 64)), (gate, H * vp), (out, H * vp)):
+        _chk(t.dtype == torch.bfloat16 and t.shape[1] >= w and t.stride(1) == 1
+             and t.data_ptr() % 16 == 0, "latent_prefill rows")
+    _chk(q.shape[0] == gate.shape[0] == out.shape[0] == angles.shape[0]
+         and angles.dtype == torch.float32, "latent_prefill rows")
+    _chk(pages.dtype == torch.bfloat16 and pages.shape[1:3] == (1, 32) and D == Rp + 64 and d <= 64
+         and tuple(w_kv.shape) == (H * (np_ + vp), Rp), "latent_prefill sizes")
+    _meta(S, cu_q=cu_q, ctx=ctx)
+    _chk(rows.seqs.dtype == rows.tiles.dtype == torch.int32 and rows.seqs.numel() == 2 * (S + 1)
+         and rows.seqs.is_contiguous() and rows.tiles.is_contiguous(), "latent_prefill plan")
+    _chk(block_tables.dtype == torch.int32 and block_tables.shape[0] == S
+         and block_tables.stride(1) == 1, "block tables")
+    k = native()
+    lat = torch.empty((rows.n, D), dtype=q.dtype, device=q.device)
+    k.latent_gather(_ptr(pages), _ptr(block_tables), block_tables.stride(0), _ptr(rows.seqs), S,
+                    rows.n, D, _ptr(lat), _stream())
+    kv = linear(lat[:, :Rp], w_kv)
+    k.latent_prefill(_ptr(q), q.stride(0), _ptr(kv), _ptr(lat), _ptr(angles), _ptr(rows.seqs),
+                     _ptr(rows.tiles), rows.tiles.shape[0], _ptr(cu_q), _ptr(ctx), _ptr(gate),
+                     gate.stride(0), _ptr(out), out.stride(0), H, np_, vp, D, Rp, d, float(scale),
+                     window, _stream())

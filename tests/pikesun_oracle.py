@@ -135,7 +135,9 @@ def moe_ff(h, W, p, m):
         for j in range(e.shape[1]):
             y[t] += wt[t, j] * clamped_glu(h[t:t + 1], W, f"{p}e{int(e[t, j])}.",
                                            m["expert"]["limit"])[0]
-    return y + clamped_glu(h, W, p + "shared.", m["shared"]["limit"])
+    if m.get("shared"):
+        y = y + clamped_glu(h, W, p + "shared.", m["shared"]["limit"])
+    return y
 
 
 MIXERS = {"rglru": rglru_mixer, "latent_attention": latent_attention_mixer}

@@ -1,0 +1,476 @@
+"""The ops of gated linear recurrences, latent attention and mixtures of
+experts one by one against the plain equations of ``pikesun_oracle``, on the CPU
+references and the GPU kernels."""
+import math
+
+import pytest
+import torch
+
+import pikesun_oracle as oracle
+from llm_mcp_amd import ops
+from llm_mcp_amd.ops import mixers
+from test_mixer_ops import DEV, OUT_TOL, Batch, close, rnd
+
+GPU = pytest.mark.gpu
+F64 = torch.float64
+
+
+@pytest.fixture(autouse=True, scope="module")
+def _one_thread():
+    n = torch.get_num_threads()
+    torch.set_num_threads(1)
+    yield
+    torch.set_num_threads(n)
+
+
+# ------------------------------------------------------------ residual pass --
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("d", [64, 100, 4096])
+def test_post_norm_over_a_mixture(dev, dt, d):
+    """x += w rms(sum_j weight_j row_j), the plain copy, and picked rows through
+    a norm; the embedding's scale."""
+    T, n, J, eps = 6, 11, 3, 1e-4
+    x, rows = rnd(T, d), rnd(n, d, seed=1).to(dt)
+    g = torch.Generator().manual_seed(2)
+    pos = torch.randint(0, n, (T, J), generator=g).to(torch.int32)
+    wt = torch.rand(T, J, generator=g)
+    post, pre = 1 + 0.3 * rnd(d, seed=3), 1 + 0.3 * rnd(d, seed=4)
+    mix = ops.Mixture(rows.to(dev), pos.to(dev), wt.to(dev))
+    y = torch.stack([sum(wt[t, j].double() * rows[pos[t, j].long()].double() for j in range(J))
+                     for t in range(T)])
+    want = x.double() + oracle.rms_norm(y, post.double(), eps)
+    res = x.clone().to(dev)
+    h = ops.sandwich_norm(res, eps, y=mix, w_post=post.to(dev), dtype=dt)
+    close(res, want, 4e-6, "residual")
+    close(h, want, OUT_TOL[dt], "copy")
+    assert h.dtype == dt
+    pick = torch.tensor([4, 0, 5], device=dev)
+    res = x.clone().to(dev)
+    h = ops.sandwich_norm(res, eps, y=mix, w_post=post.to(dev), w_pre=pre.to(dev), rows=pick,
+                          dtype=dt)
+    close(h, oracle.rms_norm(want, pre.double(), eps)[[4, 0, 5]], OUT_TOL[dt], "picked")
+    assert torch.equal(res.cpu(), x)
+    table = rnd(9, d, seed=5).to(dt)
+    ids = torch.tensor([3, 8, 0, 3, 1, 7], dtype=torch.int32)
+    res = torch.empty(T, d, device=dev)
+    h = ops.sandwich_norm(res, eps, ids=ids.to(dev), table=table.to(dev), scale=5.5, dtype=dt)
+    close(res, table[ids.long()].double() * 5.5, 1e-6, "embedding")
+    close(h, table[ids.long()].double() * 5.5, OUT_TOL[dt], "embedding copy")
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+def test_gelu(dev, dt):
+    x = rnd(7, 48, scale=3.0).to(dt)
+    close(ops.gelu(x.clone().to(dev)), oracle.gelu_tanh(x.double()), OUT_TOL[dt])
+    w = rnd(32, 48, seed=1, scale=0.2).to(dt)
+    close(ops.linear_gelu(x.to(dev), w.to(dev)), oracle.gelu_tanh(x.double() @ w.double().T),
+          2 * OUT_TOL[dt])
+
+
+# ------------------------------------------------------------- convolution --
+@pytest.mark.parametrize("dev,dt", DEV)
+def test_convolution_with_both_biases(dev, dt):
+    """The projection's bias enters before the taps: zeros, not biases, before
+    the first token."""
+    C, taps, n = 40, 4, 70
+    u, w = rnd(n, C).to(dt), rnd(taps, C, seed=1)
+    ib, b = rnd(C, seed=2), rnd(C, seed=3)
+    want = oracle.causal_conv(u.double() + ib.double(), w.T.double(), b.double())
+    st = torch.full((3, taps - 1, C), 9.0, dtype=dt, device=dev)
+    got, at = [], 0
+    for k in (2, 1, 40, 27):
+        bt = Batch(dev, [k], [at], [1])
+        got.append(ops.short_conv(u[at:at + k].to(dev), w.to(dev), st, bt.cu, bt.ctx, bt.slots,
+                                  bias=b.to(dev), in_bias=ib.to(dev), tiles=bt.tiles))
+        at += k
+    close(torch.cat(got), want, OUT_TOL[dt])
+
+
+# ------------------------------------------------- gated linear recurrence --
+class Recurrence:
+    def __init__(self, n, bp, seed=0):
+        self.n, self.bp, self.C = n, bp, n * bp
+        self.ra, self.ri = (rnd(n, bp, bp, seed=seed + k, scale=2 / math.sqrt(bp))
+                            .to(torch.bfloat16) for k in (1, 2))
+        self.gb = rnd(2, self.C, seed=seed + 3, scale=0.5)
+        self.lam = rnd(self.C, seed=seed + 4, scale=1.5) - 3.0
+        self.yb = rnd(self.C, seed=seed + 5, scale=0.5)
+
+    def want(self, u, y):
+        u, y = u.double(), y.double()
+        r = oracle.block_gate(u, self.ra.double(), self.gb[0].double().view(self.n, -1))
+        i = oracle.block_gate(u, self.ri.double(), self.gb[1].double().view(self.n, -1))
+        S = oracle.gated_linear_recurrence(u, r, i, self.lam.double())
+        return S * oracle.gelu_tanh(y + self.yb.double()), S
+
+    def run(self, u, y, state, b, dev, dt, segs="plan"):
+        big = self.bp > ops.RGLRU_MAX_BLOCK
+        gates = torch.stack([self.ra, self.ri], 1).reshape(self.n, 2 * self.bp, self.bp)
+        w = ops.pack_grouped(gates.to(dev, torch.float32 if big else dt))
+        log_a = (-8.0 * oracle.softplus(self.lam.double())).float()
+        pad = torch.zeros(len(y), 8).to(dt)
+        y2 = torch.cat([y, pad], 1).to(dev)[:, :self.C]       # rows of a wider projection
+        if segs == "plan":
+            segs = b.segments(-(-self.C // ops.RGLRU_TILE), 1) if b.nd < len(b.q) else None
+        return ops.rglru(u.to(dev), y2, self.yb.to(dev), w, self.gb.to(dev), log_a.to(dev), state,
+                         b.cu, b.ctx, b.slots, num_decode=b.nd, segments=segs)
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("n,bp", [(2, 32), (3, 32), (2, 64), (1, 128), (2, 256), (1, 512), (1, 544)])
+def test_recurrence_in_a_mixed_batch(n, bp, dev, dt):
+    """Decode rows first (one of them a sequence's first token), then unequal
+    portions; slots hold rubbish that a fresh sequence must not see."""
+    R = Recurrence(n, bp)
+    starts = [10, 0, 5, 0, 66]                       # tokens before this step
+    full = [(rnd(s + q, R.C, seed=20 + k).to(dt), rnd(s + q, R.C, seed=40 + k).to(dt))
+            for k, (s, q) in enumerate(zip(starts, [1, 1, 70, 130, 2]))]
+    qs = [1, 1, 70, 130, 2]
+    state = torch.full((8, R.C), 7.0, device=dev)
+    slots = [3, 0, 6, 1, 4]
+    for k in range(5):                                  # earlier tokens of each sequence
+        if starts[k]:
+            b = Batch(dev, [starts[k]], [0], [slots[k]])
+            R.run(full[k][0][:starts[k]], full[k][1][:starts[k]], state, b, dev, dt)
+    b = Batch(dev, qs, starts, slots)
+    u = torch.cat([full[k][0][starts[k]:] for k in range(5)])
+    y = torch.cat([full[k][1][starts[k]:] for k in range(5)])
+    got = R.run(u, y, state, b, dev, dt)
+    for k in range(5):
+        want, S = R.want(*full[k])
+        close(got[b.rows(k)], want[starts[k]:], OUT_TOL[dt], f"sequence {k}")
+        close(state[slots[k]], S[-1], 1e-5 if dt == torch.float32 else 2e-4, f"state {k}")
+    assert torch.equal(state[[2, 5, 7]].cpu(), torch.full((3, R.C), 7.0))
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+def test_recurrence_in_segments(dev, dt):
+    """One long sequence cut into many segments, from a state that matters, and
+    a second one beside it; padding slots are skipped."""
+    R = Recurrence(1, 64, seed=7)
+    R.lam = R.lam - 3.0                               # long memory: segments must chain
+    n, m = 1100, 300
+    u, y = rnd(n, 64, seed=1).to(dt), rnd(n, 64, seed=2).to(dt)
+    u2, y2 = rnd(m, 64, seed=3).to(dt), rnd(m, 64, seed=4).to(dt)
+    state = torch.full((3, 64), 5.0, device=dev)
+    R.run(u[:90], y[:90], state, Batch(dev, [90], [0], [2]), dev, dt)
+    b = Batch(dev, [n - 90, m, 40], [90, 0, 0], [2, 0, -1])
+    g = b.segments(1, 1)
+    assert g.n >= 6 and not g.one_pass
+    got = R.run(torch.cat([u[90:], u2, u2[:40]]), torch.cat([y[90:], y2, y2[:40]]), state, b, dev,
+                dt, g)
+    want, S = R.want(u, y)
+    close(got[:n - 90], want[90:], OUT_TOL[dt])
+    close(state[2], S[-1], 2e-4)
+    want, S = R.want(u2, y2)
+    close(got[b.rows(1)], want, OUT_TOL[dt])
+    close(state[0], S[-1], 2e-4)
+    assert float((state[1] - 5.0).abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+def test_slow_decays_keep_their_input(dev, dt):
+    """a within 1e-5 of 1: sqrt(1 - a^2) must not be lost."""
+    R = Recurrence(2, 32, seed=3)
+    R.lam = torch.full((64,), -12.0) + 0.5 * rnd(64)
+    u, y = rnd(200, 64, seed=1).to(dt), rnd(200, 64, seed=2).to(dt)
+    state = torch.zeros(1, 64, device=dev)
+    got = R.run(u, y, state, Batch(dev, [200], [0], [0]), dev, dt)
+    want, S = R.want(u, y)
+    close(got, want, OUT_TOL[dt])
+    close(state[0], S[-1], 2e-4)
+
+
+# -------------------------------------------------------- latent attention --
+@pytest.mark.parametrize("dev", ["cpu", pytest.param("cuda", marks=GPU)])
+def test_rotary_angles_far_out(dev):
+    base, d = 20000.0, 24
+    pos = torch.tensor([0, 1, 31, 4095, 100_003, 3_000_017], dtype=torch.int32)
+    ang = ops.rope_angles(pos.to(dev), ops.rope_freqs(base, d, device=dev)).cpu()
+    for t, p in enumerate(pos.tolist()):
+        for i in range(d // 2):
+            a = p * base ** (-2.0 * i / d)
+            assert abs(float(ang[t, i]) - math.cos(a)) < 2e-6
+            assert abs(float(ang[t, d // 2 + i]) - math.sin(a)) < 2e-6
+
+
+class Latent:
+    """One layer's sizes; cached rows are made up directly."""
+
+    def __init__(self, H, dn, dr, dv, R, window, scale, seed=0):
+        self.H, self.dn, self.dr, self.dv, self.R = H, dn, dr, dv, R
+        self.window, self.scale = window, scale
+        up = mixers_up
+        self.Rp = next((r for r in (64, 128, 256, 512) if r >= R), up(R, 64))
+        self.xp, self.np, self.vp = up(dr, 64), up(dn, 64), up(dv, 64)
+        self.uk = rnd(H, dn, R, seed=seed + 1, scale=R ** -0.5).to(torch.bfloat16)
+        self.uv = rnd(H, dv, R, seed=seed + 2, scale=R ** -0.5).to(torch.bfloat16)
+
+    def pad(self, t, n, dim=-1):
+        shape = list(t.shape)
+        shape[dim] = n - shape[dim]
+        return torch.cat([t, t.new_zeros(shape)], dim)
+
+    def served(self, dev, dt):
+        uk = self.pad(self.pad(self.uk, self.Rp), self.np, 1).to(dev, dt)
+        uv = self.pad(self.pad(self.uv, self.Rp), self.vp, 1).to(dev, dt)
+        return (ops.pack_grouped(uk.transpose(1, 2).contiguous()), ops.pack_grouped(uv),
+                torch.cat([uk, uv], 1).reshape(-1, self.Rp).contiguous())
+
+    def want(self, q, c, kr, pos0, gate):
+        """q [n, H, dn + dr] not rotated, at positions pos0..; c, kr of all positions."""
+        n, H = q.shape[0], self.H
+        T = c.shape[0]
+        uk, uv = self.uk.double(), self.uv.double()
+        k = torch.cat([torch.einsum("tr,hdr->thd", c.double(), uk),
+                       kr.double()[:, None].expand(T, H, self.dr)], -1)
+        v = torch.einsum("tr,hdr->thd", c.double(), uv)
+        pos = torch.arange(pos0, pos0 + n)
+        qd = q.double()
+        qr = oracle.rotate_half(qd[..., self.dn:], pos, 777.0)
+        full = torch.zeros(T, H, self.dn + self.dr, dtype=F64)
+        full[pos0:pos0 + n] = torch.cat([qd[..., :self.dn], qr], -1)
+        o = oracle.window_attention(full, k, v, self.scale, self.window)[pos0:pos0 + n]
+        return o * oracle.sigmoid(gate.double())
+
+
+def mixers_up(n, m):
+    return -(-n // m) * m
+
+
+def pages_of(L, seqs, tables, NB, dev, dt):
+    """Pages with each sequence's [c | rotated key part] rows at its table."""
+    pg = torch.full((NB, 1, 32, L.Rp + L.xp), 3.0)       # stale rows of other owners
+    for (c, kr), tab in zip(seqs, tables):
+        for j in range(c.shape[0]):
+            row = torch.zeros(L.Rp + L.xp)
+            row[:L.R], row[L.Rp:L.Rp + L.dr] = c[j].float(), kr[j].float()
+            pg[tab[j // 32], 0, j % 32] = row
+    return pg.to(dev, dt)
+
+
+GEOS = {"small": (3, 20, 12, 24, 40, 37, 0.5), "wide": (20, 100, 64, 72, 200, 90, 0.3),
+        "fast": (32, 128, 64, 128, 512, 300, 0.25), "one": (1, 8, 2, 8, 16, 1, 1.0),
+        "rank256": (16, 64, 32, 128, 256, 64, 0.4), "beyond": (2, 136, 66, 140, 520, 50, 0.3)}
+
+
+def latent_case(name, dev, dt, qlens, ctxs, far=None):
+    """Decode rows and prompt rows of a step; ``far`` = (sequence, query row in
+    it, distance): that key is made to stand out for that query."""
+    L = Latent(*GEOS[name])
+    g = torch.Generator().manual_seed(5)
+    perm = torch.randperm(64, generator=g).tolist()
+    seqs, tables = [], []
+    for k, n in enumerate(ctxs):
+        seqs.append((rnd(n, L.R, seed=100 + k).to(dt).float(), rnd(n, L.dr, seed=200 + k).to(dt).float()))
+        tables.append([perm.pop() for _ in range(-(-n // 32))])
+    T, H = sum(qlens), L.H
+    q = rnd(T, H, L.dn + L.dr, seed=300).to(dt)
+    gate = rnd(T, H, L.dv, seed=301).to(dt)
+    cu = [0]
+    for n in qlens:
+        cu.append(cu[-1] + n)
+    if far:
+        s, r, dist = far
+        key = ctxs[s] - qlens[s] + r - dist
+        if key >= 0:
+            qn = torch.einsum("hd,hdr->r", q[cu[s] + r, :, :L.dn].float(), L.uk.float())
+            seqs[s][0][key] = (6.0 * qn / qn.pow(2).mean().sqrt()).to(dt).float()
+    pages = pages_of(L, seqs, tables, 64, dev, dt)
+    W = max(len(t) for t in tables)
+    bt = torch.tensor([t + [0] * (W - len(t)) for t in tables], dtype=torch.int32, device=dev)
+    pos = torch.cat([torch.arange(c - n, c) for n, c in zip(qlens, ctxs)]).to(torch.int32)
+    ang = ops.rope_angles(pos.to(dev), ops.rope_freqs(777.0, L.dr, device=dev))
+    qs = torch.zeros(T, H, L.np + L.xp)
+    qs[..., :L.dn], qs[..., L.np:L.np + L.dr] = q[..., :L.dn].float(), q[..., L.dn:].float()
+    qs = qs.reshape(T, -1).to(dev, dt)
+    gs = L.pad(gate, L.vp).reshape(T, -1).to(dev)
+    i32 = dict(dtype=torch.int32, device=dev)
+    meta = dict(bt=bt, cu=torch.tensor(cu, **i32), ctx=torch.tensor(ctxs, **i32), pos=pos.to(dev))
+    want = torch.cat([L.want(q[a:b], *seqs[k], ctxs[k] - qlens[k], gate[a:b])
+                      for k, (a, b) in enumerate(zip(cu, cu[1:]))])
+    return L, qs, gs, ang, pages, meta, want.reshape(T, H, L.dv)
+
+
+def on_latents(L, qs, gs, ang, pages, meta, dev, dt, nd, ws=None):
+    absorb, unfold, _ = L.served(dev, dt)
+    ql = ops.latent_query(qs, absorb, ang, L.H, L.np, L.xp, L.Rp)
+    o = ops.latent_attention(ql, pages, meta["bt"], meta["cu"], meta["pos"], L.scale, L.window, L.H,
+                             L.Rp, ws=ws, num_decode=nd)
+    y = ops.grouped_heads(o, unfold, gate=gs)
+    return y.view(len(qs), L.H, L.vp)[..., :L.dv]
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("name", sorted(GEOS))
+def test_latent_rows(name, dev, dt):
+    """Decode rows and prompt rows on latents, through shuffled pages."""
+    ctxs = [1, 33, 128, 64, 75]
+    qlens = [1, 1, 1, 20, 3]
+    L, qs, gs, ang, pages, meta, want = latent_case(name, dev, dt, qlens, ctxs)
+    got = on_latents(L, qs, gs, ang, pages, meta, dev, dt, 3)
+    close(got, want, 2e-5 if dt == torch.float32 else 2e-2)
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("parts", [1, 3, 8])
+def test_latent_decode_in_parts(parts, dev, dt):
+    """Long windows split over workgroups, unequal contexts in one batch."""
+    ctxs = [700, 5, 290, 64, 331, 32]
+    L, qs, gs, ang, pages, meta, want = latent_case("fast", dev, dt, [1] * 6, ctxs)
+    ws = ops.DecodeWorkspace(6, L.H, L.Rp, parts, dev)
+    got = on_latents(L, qs, gs, ang, pages, meta, dev, dt, 6, ws)
+    close(got, want, 2e-5 if dt == torch.float32 else 2e-2)
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("dist", [0, 36, 37, 31, 32])
+def test_a_key_that_stands_out_at_the_window_edge(dist, dev, dt):
+    """Distance 36 is the last inside a window of 37, 37 the first outside."""
+    L, qs, gs, ang, pages, meta, want = latent_case("small", dev, dt, [1, 9], [97, 64], (0, 0, dist))
+    got = on_latents(L, qs, gs, ang, pages, meta, dev, dt, 1)
+    close(got, want, 2e-5 if dt == torch.float32 else 2e-2)
+    near = [latent_case("small", "cpu", torch.float32, [1, 9], [97, 64], (0, 0, d))[-1]
+            for d in (36, 37)]
+    assert float((near[0] - near[1]).abs()[0].max()) > 0.2      # it would show
+
+
+@GPU
+@pytest.mark.parametrize("name", ["small", "wide", "fast", "one", "rank256"])
+@pytest.mark.parametrize("far", [None, (1, 63, 36), (1, 63, 37), (2, 4, 299), (2, 4, 300)])
+def test_latent_prefill(name, far):
+    """Prompt rows on expanded keys: whole prompts, portions from the middle of
+    a page, two-token portions."""
+    dt = torch.bfloat16
+    ctxs, qlens = [150, 200, 340, 40], [150, 131, 7, 2]
+    L, qs, gs, ang, pages, meta, want = latent_case(name, "cuda", dt, qlens, ctxs, far)
+    rows, tiles, n = mixers.latent_rows(qlens, ctxs, L.window)
+    plan = ops.LatentRows(torch.tensor(rows, device="cuda").contiguous(),
+                          torch.tensor(tiles, device="cuda").contiguous(), n)
+    out = torch.empty((len(qs), L.H * L.vp), dtype=dt, device="cuda")
+    ops.latent_prefill(qs, pages, plan, L.served("cuda", dt)[2], ang, meta["bt"], meta["cu"],
+                       meta["ctx"], L.scale, L.window, L.H, L.np, L.vp, L.Rp, gs, out)
+    got = out.view(len(qs), L.H, L.vp)
+    close(got[..., :L.dv], want, 2e-2)
+    assert float(got[..., L.dv:].abs().max() if L.vp > L.dv else 0.0) == 0.0
+
+
+def test_gathered_rows_are_the_visible_ones():
+    seqs, tiles, n = mixers.latent_rows([5, 130, 1], [5, 400, 64], 33)
+    assert seqs.tolist() == [[0, 0], [5, 238], [167, 31], [200, 0]] and n == 200
+    assert tiles.tolist() == [[0, 0], [1, 0], [1, 128], [2, 0]]
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+def test_latent_prep(dev, dt):
+    """Norms over the true sizes, zero padding, the rotated part, page rows at
+    their slots and nowhere else."""
+    T, qr, qp, R, Rp, d, xp, eps = 5, 56, 64, 40, 64, 12, 64, 1e-3
+    p = torch.zeros(T, qp + Rp + xp + 24)
+    p[:, :qr], p[:, qp:qp + R], p[:, qp + Rp:qp + Rp + d] = rnd(T, qr), rnd(T, R, seed=1), \
+        rnd(T, d, seed=2)
+    p = p.to(dt)
+    qn, cn = torch.zeros(qp), torch.zeros(Rp)
+    qn[:qr], cn[:R] = 1 + 0.3 * rnd(qr, seed=3), 1 + 0.3 * rnd(R, seed=4)
+    pos = torch.tensor([0, 7, 31, 32, 1000], dtype=torch.int32)
+    ang = ops.rope_angles(pos.to(dev), ops.rope_freqs(100.0, d, device=dev))
+    slots = torch.tensor([33, -1, 0, 95, 64], dtype=torch.int32, device=dev)
+    pages = torch.full((3, 1, 32, Rp + xp), 2.0, dtype=dt, device=dev)
+    cq = ops.latent_prep(p.to(dev), qr, qp, qn.to(dev), R, cn.to(dev), ang, slots, pages, Rp, eps)
+    pd = p.double()
+    close(cq[:, :qr], oracle.rms_norm(pd[:, :qr], qn[:qr].double(), eps), OUT_TOL[dt])
+    assert float(cq[:, qr:].abs().max()) == 0.0
+    flat = pages.view(96, -1)
+    for t, s in enumerate(slots.tolist()):
+        if s < 0:
+            continue
+        row = flat[s]
+        close(row[:R], oracle.rms_norm(pd[t, qp:qp + R], cn[:R].double(), eps), OUT_TOL[dt])
+        close(row[Rp:Rp + d], oracle.rotate_half(pd[t:t + 1, qp + Rp:qp + Rp + d], pos[t:t + 1],
+                                                 100.0)[0], OUT_TOL[dt])
+        assert float(row[R:Rp].abs().max()) == 0.0 and float(row[Rp + d:].abs().max()) == 0.0
+    rest = [s for s in range(96) if s not in slots.tolist()]
+    assert float((flat[rest] - 2.0).abs().max()) == 0.0
+
+
+# ------------------------------------------------------- mixture of experts --
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("E,top,d", [(3, 3, 24), (16, 4, 320), (40, 1, 64), (100, 9, 72), (200, 2, 50)])
+def test_routing(E, top, d, dev, dt):
+    T, extra = 37, 2
+    h, w = rnd(T, d).to(dt), rnd(E, d, seed=1).to(dt)
+    r = ops.moe_route(h.to(dev), w.to(dev), top, extra)
+    e, wt = oracle.route(h.double(), w.double(), top)
+    assert torch.equal(r.ids[:, :top].cpu().long(), e)
+    assert r.ids[:, top:].tolist() == [[E, E + 1]] * T
+    close(r.weights[:, :top], wt, 1e-5)
+    assert float((r.weights[:, top:] - 1).abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("dev", ["cpu", pytest.param("cuda", marks=GPU)])
+def test_equal_logits_take_the_lowest_expert(dev):
+    h = torch.ones(2, 8)
+    w = torch.tensor([0.5, 1.0, 1.0, 0.2, 1.0])[:, None].expand(5, 8).contiguous()
+    r = ops.moe_route(h.to(dev), w.to(dev), 2)
+    assert r.ids.tolist() == [[1, 2]] * 2
+
+
+@pytest.mark.parametrize("dev", ["cpu", pytest.param("cuda", marks=GPU)])
+@pytest.mark.parametrize("T,J,G", [(1, 3, 8), (50, 4, 7), (300, 6, 40), (5000, 4, 18)])
+def test_sorting_uses_by_expert(T, J, G, dev):
+    g = torch.Generator().manual_seed(T)
+    ids = torch.stack([torch.randperm(G - 1, generator=g)[:J] for _ in range(T)]).to(torch.int32)
+    plan = ops.moe_plan(ops.Route(ids.to(dev), None), G)     # the last expert stays empty
+    src, pos, off = plan.src.cpu().long(), plan.pos.cpu().long(), plan.off.cpu().long()
+    assert sorted(pos.reshape(-1).tolist()) == list(range(T * J))
+    assert torch.equal(src[pos], torch.arange(T)[:, None].expand(T, J))
+    where = torch.bucketize(pos, off[1:], right=True)        # the expert whose range holds it
+    assert torch.equal(where, ids.long())
+    if dev == "cuda":
+        got = sorted((e, r) for e, r in plan.tiles.cpu().tolist() if e >= 0)
+        assert got == [(e, r) for e in range(G) for r in range(int(off[e]), int(off[e + 1]), plan.bm)]
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("T,width,ff", [(5, 64, 64), (90, 192, 128), (700, 128, 192)])
+def test_experts(T, width, ff, dev, dt):
+    """Both grouped products over a route, tiles of every size (few and many
+    rows per expert), against each expert applied to each row."""
+    E, top = 5, 2
+    h = rnd(T, width).to(dt)
+    W = {}
+    for e in range(E):
+        for n, s in (("gate", (ff, width)), ("up", (ff, width)), ("down", (width, ff))):
+            W[f"e{e}.{n}"] = rnd(*s, seed=10 * e + len(n), scale=1.5 / math.sqrt(s[1])).to(dt)
+    W["router"] = rnd(E, width, seed=99).to(dt)
+    sf = ff + 24
+    for n, s in (("gate", (sf, width)), ("up", (sf, width)), ("down", (width, sf))):
+        W[f"shared.{n}"] = rnd(*s, seed=77 + len(n), scale=1.5 / math.sqrt(s[1])).to(dt)
+    m = dict(kind="moe", router=dict(experts=E, top=top), expert=dict(ff=ff, limit=1.1),
+             shared=dict(ff=sf, limit=0.6))
+    from llm_mcp_amd.models.feedforward import MixtureOfExperts
+    ff_ = MixtureOfExperts(m, width)
+    assert {k: tuple(v.shape) for k, v in W.items()} == ff_.shapes
+
+    def put(t, fp32=False):
+        return t.to(dev, torch.float32 if fp32 else dt).contiguous()
+    ff_.load(W.__getitem__, put)
+    got = ff_.forward(h.to(dev)).sum()
+    want = oracle.moe_ff(h.double(), {k: v.double() for k, v in W.items()}, "", m)
+    e = (got.double().cpu()[:, :width] - want).abs().amax(-1) / want.abs().max()
+    # a near tie of the router may fall the other way only if the logits do
+    assert float(e.max()) < (2e-5 if dt == torch.float32 else 2e-2), float(e.max())
+
+
+@pytest.mark.parametrize("dev,dt", DEV)
+@pytest.mark.parametrize("M", [1, 17, 100, 300])
+def test_per_head_products(M, dev, dt):
+    H, K, N = 3, 64, 192
+    x = rnd(M, H * (K + 64)).to(dt)
+    w = rnd(H, N, K, seed=1, scale=K ** -0.5).to(dt)
+    gate = rnd(M, H * N + 16, seed=2).to(dt)
+    y = ops.grouped_heads(x.to(dev), ops.pack_grouped(w.to(dev)), gate=gate.to(dev)[:, :H * N],
+                          in_stride=K + 64)
+    want = torch.einsum("mhk,hnk->mhn", x.double().view(M, H, -1)[..., :K], w.double()) \
+        .reshape(M, -1) * oracle.sigmoid(gate.double()[:, :H * N])
+    close(y, want, OUT_TOL[dt])
