@@ -41,6 +41,8 @@ int sandwich_norm(void*, float*, const void*, long, int, long, const int*, const
 int gelu(void*, long, int, hipStream_t);
 int grouped(const void*, long, long, const void*, void*, long, long, int, int, int, int, const int*,
             int, const int*, const int*, const float*, const void*, long, int, int, hipStream_t);
+int pgemm_grouped(void*, const void*, const void*, int, int, int, long, long, int, const int*, int,
+                  const int*, const int*, const float*, hipStream_t);
 int moe_route(const void*, long, const void*, int, int, int, int, int, int*, float*, int,
               hipStream_t);
 int moe_plan(const int*, int, int, int, int, int, int*, int*, int*, int*, int*, hipStream_t);
@@ -230,6 +232,14 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                        P<int>(tiles), mtiles, P<int>(off), P<int>(src), P<float>(limit),
                        P<void>(gate), gate_ld, bm, is_bf16, S(stream)),
           "grouped");
+  });
+  m.def("pgemm_grouped", [](uptr c, uptr a, uptr w, int M, int N, int K, long lda, long ldc,
+                            int a_rows, uptr tiles, int mtiles, uptr off, uptr src, uptr limit,
+                            uptr stream) {
+    check(lmx::pgemm_grouped(P<void>(c), P<void>(a), P<void>(w), M, N, K, lda, ldc, a_rows,
+                             P<int>(tiles), mtiles, P<int>(off), P<int>(src), P<float>(limit),
+                             S(stream)),
+          "pgemm_grouped");
   });
   m.def("moe_route", [](uptr h, long h_ld, uptr w, int T, int d, int E, int top, int extra, uptr ids,
                         uptr wts, int is_bf16, uptr stream) {

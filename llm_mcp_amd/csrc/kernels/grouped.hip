@@ -17,7 +17,7 @@
 // operands are swapped (D = W . A^T): a lane's 4 accumulators are 4
 // consecutive output columns of one row.
 //
-//   grouped_small   BM x 64 tiles, BM = 16 / 64: decode batches, bound by the
+//   grouped_small   BM x 64 tiles, BM = 16 / 32 / 64: decode batches, bound by the
 //                   weight stream; A in LDS, one 16-column tile per wave
 //   grouped_large   128 x 128 tiles of 64-deep K steps, double-buffered
 //                   LDS-DMA, 4 waves of 64 x 64
@@ -321,7 +321,7 @@ __global__ void __launch_bounds__(256) grouped_f32_kernel(GroupArgs p) {
 
 }  // namespace
 
-// bm: rows per tile (32 fp32; 16 / 64 / 128 bf16); mtiles: row tiles (experts:
+// bm: rows per tile (32 fp32; 16 / 32 / 64 / 128 bf16); mtiles: row tiles (experts:
 // the tile list's length)
 int grouped(const void* a, long lda, long a_gs, const void* w, void* c, long ldc, long c_gs,
             int groups, int N, int K, int M, const int* tiles, int mtiles, const int* off,
@@ -341,6 +341,8 @@ int grouped(const void* a, long lda, long a_gs, const void* w, void* c, long ldc
     return -3;
   if (bm == 16)
     grouped_small_kernel<16><<<dim3((N + 63) / 64, mtiles, gz), dim3(256), 0, stream>>>(p);
+  else if (bm == 32)
+    grouped_small_kernel<32><<<dim3((N + 63) / 64, mtiles, gz), dim3(256), 0, stream>>>(p);
   else if (bm == 64)
     grouped_small_kernel<64><<<dim3((N + 63) / 64, mtiles, gz), dim3(256), 0, stream>>>(p);
   else if (bm == LBM)

@@ -255,12 +255,14 @@ __global__ void __launch_bounds__(256, 1) latent_rows_kernel(
   const int* tab = bt + (long)seq * bt_stride;
   const int last_page = pos / BS;
 
+  // page ids by scalar loads: a vector load would wait behind the DMAs before it
   auto stage = [&](int t0, int buf) {
+    const int pg = t0 / BS;
+    const long pa = (long)tab[pg] * BS * D, pb = (long)tab[min(pg + 1, last_page)] * BS * D;
 #pragma unroll
     for (int i = 0; i < TK * CH / 256; ++i) {
       const int e = i * 256 + tid, r = e / CH, ch = e % CH;
-      const int pg = min((t0 + r) / BS, last_page);
-      lds_dma16(pages + ((long)tab[pg] * BS + (r % BS)) * D + 8 * (ch ^ lat_swz<R>(r)),
+      lds_dma16(pages + (r < BS ? pa : pb) + (r % BS) * D + 8 * (ch ^ lat_swz<R>(r)),
                 kt + buf * TK * D + (i * 256 + wave * 64) * 8);
     }
   };

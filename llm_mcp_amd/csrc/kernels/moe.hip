@@ -4,7 +4,7 @@
 //              index first among equals) and the softmax over just those; then
 //              `extra` further experts every row uses with weight 1.
 //              bf16 rows, up to 128 experts: 16 rows per workgroup on MFMA, the K
-//              range split over the 4 waves; otherwise one row per workgroup on the VALU.
+//              range split over the waves; otherwise one row per workgroup on the VALU.
 //   moe_plan   the uses (row, expert) sorted by expert: expert row ranges, the
 //              row of every sorted use and the sorted place of every use, and
 //              the row tiles of the grouped products (grouped.hip).
@@ -55,44 +55,60 @@ __device__ __forceinline__ void moe_select(const float* z, int E, int top, int e
   }
 }
 
-// grid ceil(T / 16), block 256
-template <int NT>
-__global__ void __launch_bounds__(256) moe_route_mfma_kernel(const bf16_t* __restrict__ h, long h_ld,
-                                                             const bf16_t* __restrict__ w, int T,
-                                                             int d, int E, int top, int extra,
-                                                             int* __restrict__ ids,
-                                                             float* __restrict__ wts) {
-  __shared__ float part[4][16][NT * 16 + 1];
+// grid ceil(T / 16), block 64 NW: NW waves split the K range
+template <int NT, int NW>
+__global__ void __launch_bounds__(64 * NW) moe_route_mfma_kernel(
+    const bf16_t* __restrict__ h, long h_ld, const bf16_t* __restrict__ w, int T, int d, int E,
+    int top, int extra, int* __restrict__ ids, float* __restrict__ wts) {
+  __shared__ float part[NW][16][NT * 16 + 1];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, q = lane >> 4;
   const int t0 = blockIdx.x * 16;
-  const bf16_t* hr = h + (long)min(t0 + c, T - 1) * h_ld;
+  const bf16_t* hr = h + (long)min(t0 + c, T - 1) * h_ld + 8 * q;
+  const bf16_t* wr[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) wr[i] = w + (long)min(16 * i + c, E - 1) * d + 8 * q;
   f32x4_t acc[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   const bf16x8_t zero = {0, 0, 0, 0, 0, 0, 0, 0};
-#pragma unroll 4
-  for (int k0 = wave * 32; k0 < d; k0 += 128) {
-    const int k = k0 + 8 * q;
-    const bool in = k < d;                     // d is a multiple of 8
-    const bf16x8_t x = in ? load_frag16B(hr + k) : zero;
+  const int kc = ((d + 31) / 32 + NW - 1) / NW * 32;      // whole K32 steps per wave
+  const int k1 = min((wave + 1) * kc, d);
+  int k0 = wave * kc;
+  constexpr int U = NT <= 2 ? 8 : 4;
+  for (; k0 + 32 * U <= k1; k0 += 32 * U) {
+    bf16x8_t x[U], wv[U][NT];
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int e = min(16 * i + c, E - 1);
-      const bf16x8_t wv = in ? load_frag16B(w + (long)e * d + k) : zero;
-      acc[i] = mfma16(wv, x, acc[i]);          // D: row = expert, column = token
+    for (int s = 0; s < U; ++s) {
+      x[s] = load_frag16B(hr + k0 + 32 * s);
+#pragma unroll
+      for (int i = 0; i < NT; ++i) wv[s][i] = load_frag16B(wr[i] + k0 + 32 * s);
     }
+#pragma unroll
+    for (int s = 0; s < U; ++s)
+#pragma unroll
+      for (int i = 0; i < NT; ++i) acc[i] = mfma16(wv[s][i], x[s], acc[i]);  // row = expert, column = token
+  }
+  for (; k0 < k1; k0 += 32) {
+    const bool in = k0 + 8 * q < d;                      // d is a multiple of 8
+    const bf16x8_t x = in ? load_frag16B(hr + k0) : zero;
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+      acc[i] = mfma16(in ? load_frag16B(wr[i] + k0) : zero, x, acc[i]);
   }
 #pragma unroll
   for (int i = 0; i < NT; ++i)
 #pragma unroll
     for (int r = 0; r < 4; ++r) part[wave][c][16 * i + 4 * q + r] = acc[i][r];
   __syncthreads();
-  for (int e = threadIdx.x; e < 16 * NT * 16; e += 256) {
+  for (int e = threadIdx.x; e < 16 * NT * 16; e += 64 * NW) {
     const int t = e / (NT * 16), n = e % (NT * 16);
-    part[0][t][n] += part[1][t][n] + part[2][t][n] + part[3][t][n];
+    float s = part[0][t][n];
+#pragma unroll
+    for (int v = 1; v < NW; ++v) s += part[v][t][n];
+    part[0][t][n] = s;
   }
   __syncthreads();
-  for (int t = wave; t < 16; t += 4)
+  for (int t = wave; t < 16; t += NW)
     if (t0 + t < T)
       moe_select(part[0][t], E, top, extra, ids + (long)(t0 + t) * (top + extra),
                  wts + (long)(t0 + t) * (top + extra));
@@ -124,7 +140,8 @@ constexpr int SMALL = 8192;      // uses one workgroup sorts alone
 struct PlanArgs {
   const int* ids;
   int n, J, groups, bm, mtiles, blocks;
-  int *hist, *off, *src, *pos, *tiles;
+  int *hist, *off, *src, *pos;
+  int* tiles;              // [mtiles][2], then the number of used ones
 };
 
 // expert ranges and tiles from the counts cnt[groups] (LDS); beg[] gets the
@@ -143,6 +160,7 @@ __device__ __forceinline__ void plan_ranges(const PlanArgs& p, const int* cnt, i
   }
   __syncthreads();
   for (int g = threadIdx.x; g <= p.groups; g += blockDim.x) p.off[g] = beg[g];
+  if (threadIdx.x == 0) p.tiles[2 * p.mtiles] = tbeg[p.groups];
   for (int t = threadIdx.x; t < p.mtiles; t += blockDim.x) {
     int g = -1, r = 0;
     if (t < tbeg[p.groups]) {
@@ -226,11 +244,11 @@ int moe_route(const void* h, long h_ld, const void* w, int T, int d, int E, int 
     return -1;
   if (is_bf16 && E <= 128 && d % 8 == 0 && h_ld % 8 == 0 && !(((uintptr_t)h | (uintptr_t)w) & 15)) {
     const int nt = (E + 15) / 16;
-#define LMX_RT(NT)                                                                           \
-  moe_route_mfma_kernel<NT><<<dim3((T + 15) / 16), dim3(256), 0, stream>>>(                  \
+#define LMX_RT(NT, NW)                                                                       \
+  moe_route_mfma_kernel<NT, NW><<<dim3((T + 15) / 16), dim3(64 * NW), 0, stream>>>(          \
       (const bf16_t*)h, h_ld, (const bf16_t*)w, T, d, E, top, extra, ids, wts)
-    if (nt == 1) LMX_RT(1); else if (nt == 2) LMX_RT(2); else if (nt <= 4) LMX_RT(4);
-    else LMX_RT(8);
+    if (nt == 1) LMX_RT(1, 16); else if (nt == 2) LMX_RT(2, 16); else if (nt <= 4) LMX_RT(4, 8);
+    else LMX_RT(8, 4);
 #undef LMX_RT
   } else if (is_bf16) {
     moe_route_any_kernel<bf16_t><<<dim3(T), dim3(256), 0, stream>>>(

@@ -47,6 +47,12 @@
 // 1 KB per wave-instruction and the fragment reads are linear (lane x 16 B,
 // conflict-free without the XOR swizzle).
 //
+// WP 2 (grouped rows, pgemm_grouped): the rows of A are sorted into groups, each
+// with its own W in the packed layout of grouped.hip ([N / 16][K / 32] runs of
+// 1 KB); a device-built list names each 256-row tile's group and first row, and
+// src (optional) the A row of a sorted row, gathered by the DMA's per-lane
+// addresses.  ACT 6 is the clamped GLU of such products.
+//
 // Requirements (checked by the launcher): N % 256 == 0, K % 64 == 0, K >= 192,
 // lda / ldw / ldc multiples of 8 elements, 16-B aligned operands; bias (if
 // any) N <= 8192.
@@ -102,6 +108,7 @@ struct PgLoad {
   __amdgpu_buffer_rsrc_t ra;     // A rows [m0, M) of the cursor's tile
   __amdgpu_buffer_rsrc_t rw;     // W rows [n0, N)
   int kbyte;                     // k * 128
+  int av[2][2];                  // WP 2: A source offsets of the cursor's tile (PgThr::a_voff)
   int k, tile;                   // K-step in the tile, tile index of this workgroup
   bool done;                     // past the last step: re-issue the last one (free halves)
 };
@@ -111,6 +118,16 @@ struct PgOut {
   __amdgpu_buffer_rsrc_t rc;     // C rows [m0, M)
   __amdgpu_buffer_rsrc_t rn;     // NRM 1: row scales [m0, M); NRM 2: ssq partials of rows [m0, M)
   int n0;
+  float lim;                     // ACT 6: the group's clamp
+};
+
+// grouped rows (WP 2)
+struct PgGroups {
+  const int* tiles;              // [mtiles][2] group, first row; then the number of used tiles
+  const int* off;                // [groups + 1] first rows
+  const int* src;                // A row of a sorted row, or null
+  const float* limit;            // ACT 6
+  int mtiles;
 };
 
 // thread constants
@@ -143,7 +160,11 @@ __device__ __forceinline__ void pg_issue(char* smem, int stage, const PgLoad& L,
   for (int i = 0; i < 2; ++i) {
     if constexpr (H == HA0 || H == HA1) {
       __builtin_amdgcn_raw_ptr_buffer_load_lds(L.ra, (lds_void_t*)(dst + i * 8192), 16,
-                                               T.a_voff[H][i], L.kbyte, 0, 0);
+                                               WP == 2 ? L.av[H][i] : T.a_voff[H][i], L.kbyte, 0, 0);
+    } else if constexpr (WP == 2) {
+      // K-step s of a 16-column tile starts at s * 2 KB
+      __builtin_amdgcn_raw_ptr_buffer_load_lds(L.rw, (lds_void_t*)(dst + i * 8192), 16,
+                                               T.wp_voff[H - HW0][i], L.kbyte * 16, 0, 0);
     } else if constexpr (WP) {
       // K-step s of a packed tile starts at s * 4 KB of every wave block
       __builtin_amdgcn_raw_ptr_buffer_load_lds(L.rw, (lds_void_t*)(dst + i * 8192), 16,
@@ -206,8 +227,8 @@ __device__ __forceinline__ void pg_store(RT& R, const PgOut& O, const PgThr& T,
       rs[i] = __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(
           O.rn, (T.wm * 128 + QM * 64 + 16 * i + T.fr) * 4, 0, 0));
   }
-  if constexpr (ACT == 3 || ACT == 5) {
-    // SwiGLU (5: ReLU-GLU): 16-col tiles 0 (gate) and 1 (up) of the quadrant are one pair
+  if constexpr (ACT == 3 || ACT == 5 || ACT == 6) {
+    // SwiGLU (5: ReLU-GLU, 6: clamped GLU): 16-col tiles 0 (gate) and 1 (up) of the quadrant are one pair
     const int col = (O.n0 >> 1) + T.wn * 32 + QN * 16 + 4 * T.fg;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -218,6 +239,13 @@ __device__ __forceinline__ void pg_store(RT& R, const PgOut& O, const PgThr& T,
       }
       const f32x4_t g = R.acc[QM][QN][i][0], u = R.acc[QM][QN][i][1];
       bf16x4_t o;
+      if constexpr (ACT == 6) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float gc = fminf(g[r], O.lim), uc = fminf(fmaxf(u[r], -O.lim), O.lim);
+          o[r] = (short)f2bf(gc / (1.f + __expf(-1.702f * gc)) * (uc + 1.f));
+        }
+      } else
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         o[r] = (short)f2bf((ACT == 3 ? g[r] / (1.f + __expf(-g[r])) : fmaxf(g[r], 0.f)) * u[r]);
@@ -396,11 +424,11 @@ __device__ __forceinline__ void pp_phase(PpRegs& R, char* smem, int stage, const
     pg_read_a<HA0>(R.a, smem, stage, T);
     pg_read_w<0, WP>(R.w0, smem, stage, T);
     pg_read_w<1, WP>(R.w1, smem, stage, T);
-    pg_issue<HA1>(smem, stage ^ 1, L1, T);
+    pg_issue<HA1, WP>(smem, stage ^ 1, L1, T);
     if constexpr (SCHED == 1) pg_issue<HW1, WP>(smem, stage ^ 1, L1, T);
   } else {
     pg_read_a<HA1>(R.a, smem, stage, T);
-    pg_issue<HA0>(smem, stage, L2, T);
+    pg_issue<HA0, WP>(smem, stage, L2, T);
     pg_issue<HW0, WP>(smem, stage, L2, T);
     if constexpr (SCHED == 0) pg_issue<HW1, WP>(smem, stage, L2, T);
   }
@@ -427,13 +455,14 @@ template <int ACT, int BIAS, int SCHED, int WP = 0, int NRM = 0>
 __global__ void __launch_bounds__(PG_THREADS, 1) pgemm_pp2_kernel(
     bf16_t* __restrict__ C, const bf16_t* __restrict__ A, const bf16_t* __restrict__ W,
     const bf16_t* __restrict__ bias, int M, int N, int K, int lda, int ldw, int ldc,
-    float* __restrict__ nrm) {
+    float* __restrict__ nrm, PgGroups grp) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  const int tiles_m = (M + 255) / 256, tiles_n = N / 256, ntiles = tiles_m * tiles_n;
+  const int tiles_m = WP == 2 ? grp.tiles[2 * grp.mtiles] : (M + 255) / 256, tiles_n = N / 256, ntiles = tiles_m * tiles_n;
   const int G = gridDim.x;
   const int r = xcd_remap(blockIdx.x, G);
   const int my_tiles = (ntiles - r + G - 1) / G;
   const int nk = K / 64;
+  if (WP == 2 && my_tiles <= 0) return;      // fewer used tiles than workgroups
 
   PgThr T;
   const int lane = threadIdx.x & 63;
@@ -469,7 +498,8 @@ __global__ void __launch_bounds__(PG_THREADS, 1) pgemm_pp2_kernel(
 #pragma unroll
         for (int i = 0; i < 2; ++i) {
           const int r = 8 * i + T.wave, wn = r >> 2, kk = (r >> 1) & 1, j = r & 1;
-          T.wp_voff[h][i] = (2 * wn + h) * kb * 2048 + kk * 2048 + j * 1024 + lane * 16;
+          T.wp_voff[h][i] = WP == 2 ? ((2 * wn + h) * 2 + j) * kb * 1024 + kk * 1024 + lane * 16
+                                    : (2 * wn + h) * kb * 2048 + kk * 2048 + j * 1024 + lane * 16;
         }
       T.rwp_off = T.wn * 4096 + lane * 16;
     }
@@ -485,6 +515,22 @@ __global__ void __launch_bounds__(PG_THREADS, 1) pgemm_pp2_kernel(
   auto set_tile = [&](PgLoad& L, int t) {
     int tm, tn;
     pg_tile_coords(t * G + r, tiles_m, tiles_n, tm, tn);
+    if constexpr (WP == 2) {
+      const int g = grp.tiles[2 * tm], m0 = grp.tiles[2 * tm + 1], m1 = grp.off[g + 1];
+      const int sc = (lane & 7) ^ ((4 * T.wave + (lane >> 4)) & 7);
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+          const int row = min(m0 + 128 * i + 64 * h + 8 * T.wave + (lane >> 3), m1 - 1);
+          L.av[h][i] = (grp.src ? grp.src[row] : row - m0) * lda * 2 + sc * 16;
+        }
+      L.ra = __builtin_amdgcn_make_buffer_rsrc((void*)(A + (grp.src ? 0L : (long)m0 * lda)),
+                                               (short)0, 0x7fffffff, 0x00020000);
+      L.rw = __builtin_amdgcn_make_buffer_rsrc((void*)(W + ((long)g * N + tn * 256) * K), (short)0,
+                                               (int)(256L * K * 2), 0x00020000);
+      return;
+    }
     const int m0 = tm * 256, n0 = tn * 256;
     const long abytes = (long)(M - m0) * lda * 2;
     L.ra = __builtin_amdgcn_make_buffer_rsrc((void*)(A + (long)m0 * lda), (short)0,
@@ -496,8 +542,14 @@ __global__ void __launch_bounds__(PG_THREADS, 1) pgemm_pp2_kernel(
   auto set_out = [&](PgOut& O, int t) {
     int tm, tn;
     pg_tile_coords(t * G + r, tiles_m, tiles_n, tm, tn);
-    const int m0 = tm * 256;
-    const long cbytes = (long)(M - m0) * ldc * 2;
+    int m0 = tm * 256, m1 = M;
+    if constexpr (WP == 2) {
+      const int g = grp.tiles[2 * tm];
+      m0 = grp.tiles[2 * tm + 1];
+      m1 = grp.off[g + 1];
+      if constexpr (ACT == 6) O.lim = grp.limit[g];
+    }
+    const long cbytes = (long)(m1 - m0) * ldc * 2;
     O.rc = __builtin_amdgcn_make_buffer_rsrc((void*)(C + (long)m0 * ldc), (short)0,
                                              (int)(cbytes < 0x7fffffffL ? cbytes : 0x7fffffffL),
                                              0x00020000);
@@ -536,24 +588,24 @@ __global__ void __launch_bounds__(PG_THREADS, 1) pgemm_pp2_kernel(
 
   // ---- prologue: the DMA of the phases before K-step 0, in loop order
   if constexpr (SCHED == 0) {
-    pg_issue<HA0>(smem, 0, L2, T);
+    pg_issue<HA0, WP>(smem, 0, L2, T);
     pg_issue<HW0, WP>(smem, 0, L2, T);
     pg_issue<HW1, WP>(smem, 0, L2, T);
-    pg_issue<HA1>(smem, 0, L2, T);
+    pg_issue<HA1, WP>(smem, 0, L2, T);
     advance(L2);
-    pg_issue<HA0>(smem, 1, L2, T);
+    pg_issue<HA0, WP>(smem, 1, L2, T);
     pg_issue<HW0, WP>(smem, 1, L2, T);
     pg_issue<HW1, WP>(smem, 1, L2, T);
     L1 = L2;
     advance(L2);
     pg_vmwait<8>();                 // A0, W0, W1 of K-step 0
   } else {
-    pg_issue<HA0>(smem, 0, L2, T);
+    pg_issue<HA0, WP>(smem, 0, L2, T);
     pg_issue<HW0, WP>(smem, 0, L2, T);
-    pg_issue<HA1>(smem, 0, L2, T);
+    pg_issue<HA1, WP>(smem, 0, L2, T);
     pg_issue<HW1, WP>(smem, 0, L2, T);
     advance(L2);
-    pg_issue<HA0>(smem, 1, L2, T);
+    pg_issue<HA0, WP>(smem, 1, L2, T);
     pg_issue<HW0, WP>(smem, 1, L2, T);
     L1 = L2;
     advance(L2);
@@ -816,7 +868,7 @@ static int g_pg_cus = 0;
 template <int ACT, int BIAS, int WP = 0, int NRM = 0>
 static int pg_launch(bf16_t* C, const bf16_t* A, const bf16_t* W, const bf16_t* bias, int M,
                      int N, int K, int lda, int ldw, int ldc, int grid, hipStream_t stream,
-                     float* nrm = nullptr) {
+                     float* nrm = nullptr, PgGroups grp = PgGroups{}) {
   constexpr size_t smem = PG_RING_B + (BIAS == 1 ? PG_MAX_BIAS * 2 : 0);
   static_assert(smem <= 160 * 1024, "LDS");
   static bool attr = false;
@@ -827,8 +879,41 @@ static int pg_launch(bf16_t* C, const bf16_t* A, const bf16_t* W, const bf16_t* 
     attr = true;
   }
   pgemm_pp2_kernel<ACT, BIAS, 0, WP, NRM><<<dim3(grid), dim3(PG_THREADS), smem, stream>>>(
-      C, A, W, bias, M, N, K, lda, ldw, ldc, nrm);
+      C, A, W, bias, M, N, K, lda, ldw, ldc, nrm, grp);
   return (int)hipGetLastError();
+}
+
+static int pg_cus() {
+  if (g_pg_cus == 0) {
+    int dev = 0;
+    hipDeviceProp_t p;
+    if (hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&p, dev) == hipSuccess)
+      g_pg_cus = p.multiProcessorCount;
+  }
+  return g_pg_cus;
+}
+
+// Grouped rows on the persistent 256 x 256 tile: M sorted rows (A rows src[..] or
+// the rows themselves, a_rows of them), W [groups] in grouped.hip's packed
+// layout, C rows [M][N] or, with limit, the clamped GLU [M][N / 2].
+int pgemm_grouped(void* C, const void* A, const void* W, int M, int N, int K, long lda, long ldc,
+                  int a_rows, const int* tiles, int mtiles, const int* off, const int* src,
+                  const float* limit, hipStream_t stream) {
+  if (M <= 0 || mtiles <= 0) return 0;
+  if (N % 256 != 0 || K % 64 != 0 || K < 192 || lda % 8 || ldc % 4 || !tiles || !off) return -1;
+  // byte offsets are 32-bit: a tile's rows, or with src the whole of A
+  if (256L * lda * 2 > 0x7fffffffL || 256L * K * 2 > 0x7fffffffL || 256L * ldc * 2 > 0x7fffffffL ||
+      (src && (long)a_rows * lda * 2 > 0x7fffffffL))
+    return -1;
+  if (pg_cus() == 0) return -2;
+  const long all = (long)mtiles * (N / 256);
+  const int grid = (int)(all < g_pg_cus ? all : g_pg_cus);
+  const PgGroups grp{tiles, off, src, limit, mtiles};
+  auto C_ = (bf16_t*)C;
+  auto A_ = (const bf16_t*)A;
+  auto W_ = (const bf16_t*)W;
+  if (limit) return pg_launch<6, 0, 2>(C_, A_, W_, nullptr, M, N, K, (int)lda, K, (int)ldc, grid, stream, nullptr, grp);
+  return pg_launch<0, 0, 2>(C_, A_, W_, nullptr, M, N, K, (int)lda, K, (int)ldc, grid, stream, nullptr, grp);
 }
 
 // res 1: C is read as well -- C = bf16(C + bf16(A . W^T)) (the residual
@@ -853,13 +938,7 @@ int pgemm(void* C, const void* A, const void* W, const void* bias, int M, int N,
   // byte offsets of one tile's rows are 32-bit
   if (256L * lda * 2 > 0x7fffffffL || 256L * ldw * 2 > 0x7fffffffL || 256L * ldc * 2 > 0x7fffffffL)
     return -1;
-  if (g_pg_cus == 0) {
-    int dev = 0;
-    if (hipGetDevice(&dev) != hipSuccess) return -2;
-    hipDeviceProp_t p;
-    if (hipGetDeviceProperties(&p, dev) != hipSuccess) return -2;
-    g_pg_cus = p.multiProcessorCount;
-  }
+  if (pg_cus() == 0) return -2;
   const long tiles = (long)((M + 255) / 256) * (N / 256);
   if (grid <= 0) grid = g_pg_cus;
   if (grid > tiles) grid = (int)tiles;

@@ -99,7 +99,8 @@ class MixtureOfExperts:
 
     def forward(self, h):
         r = ops.moe_route(h, self.router, self.top, self.shared)
-        plan = ops.moe_plan(r, self.E + self.shared, self.w1.packed)
+        plan = ops.moe_plan(r, self.E + self.shared, self.w1.packed,
+                            ops.wide_tiles(self.w1) and ops.wide_tiles(self.w2))
         y = ops.grouped_linear(_pad_cols(h, self.kp), self.w1, plan, gather=True, glu=self.limit)
         return ops.Mixture(ops.grouped_linear(y, self.w2, plan), plan.pos, r.weights)
 

@@ -1798,7 +1798,7 @@ def pgemm_sk(a: torch.Tensor, w: torch.Tensor, splits: int, act: int = 0, epi: i
 
 
 from .grouped import (GroupedWeight, Mixture, MoePlan, Route, grouped_heads,  # noqa: E402,F401
-                      grouped_linear, moe_plan, moe_route, pack_grouped)
+                      grouped_linear, moe_plan, moe_route, pack_grouped, wide_tiles)
 from .mixers import (RGLRU_MAX_BLOCK, RGLRU_TILE, LatentRows, ScanSegments,  # noqa: E402,F401
                      attention_any, conv_qkv_cache, gated_norm, latent_attention,
                      latent_prefill, latent_prefill_ok, latent_prep, latent_query, linear_scan, rglru,

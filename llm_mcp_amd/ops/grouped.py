@@ -77,21 +77,27 @@ class MoePlan:
     src: torch.Tensor        # int32 [n]: row of each sorted use
     pos: torch.Tensor        # int32 [T, J]: sorted place of each use
     off: torch.Tensor        # int32 [groups + 1]
-    tiles: torch.Tensor | None   # int32 [mtiles, 2]: group (-1: none), first sorted row
-    bm: int
+    tiles: torch.Tensor | None   # int32 [mtiles, 2]: group (-1: none), first sorted row; one
+    bm: int                      # more entry: the number of used ones
 
 
-def _tile_rows(n: int, groups: int, bf16: bool) -> int:
-    """Rows per tile of the grouped kernels for n rows over ``groups``."""
+def _tile_rows(n: int, groups: int, bf16: bool, wide: bool) -> int:
+    """Rows per tile of the grouped kernels for n rows over ``groups``; 256: the
+    persistent tile of K13, for products of whole 256-column tiles (``wide``)."""
     if not bf16:
         return 32
     mean = n / groups
-    return 16 if mean <= 24 else 64 if mean < 96 else 128
+    return 16 if mean <= 6 else 32 if mean <= 24 else 64 if mean < 96 else 256 if wide and mean >= 192 else 128
 
 
-def moe_plan(r: Route, groups: int, bf16: bool = True) -> MoePlan:
+def wide_tiles(w: GroupedWeight) -> bool:
+    """K13's grouped form takes this weight."""
+    return w.packed and w.N % 256 == 0 and w.K % 64 == 0 and w.K >= 192
+
+
+def moe_plan(r: Route, groups: int, bf16: bool = True, wide: bool = False) -> MoePlan:
     """Sort a route's uses by expert and list the row tiles (``bf16``: of the
-    packed kernels)."""
+    packed kernels; ``wide``: every product of the plan is ``wide_tiles``)."""
     T, J = r.ids.shape
     n = T * J
     ids = r.ids
@@ -103,11 +109,11 @@ def moe_plan(r: Route, groups: int, bf16: bool = True) -> MoePlan:
         off = torch.cat([torch.zeros(1, dtype=torch.int64), cnt.cumsum(0)]).to(torch.int32)
         return MoePlan((order // J).to(torch.int32), pos.view(T, J), off, None, 0)
     _chk(0 < groups <= MOE_MAX_EXPERTS and ids.is_contiguous(), "moe_plan")
-    bm = _tile_rows(n, groups, bf16)
+    bm = _tile_rows(n, groups, bf16, wide)
     mt = min(n, -(-n // bm) + groups)
     i32 = dict(dtype=torch.int32, device=ids.device)
     src, pos = torch.empty(n, **i32), torch.empty((T, J), **i32)
-    off, tiles = torch.empty(groups + 1, **i32), torch.empty((mt, 2), **i32)
+    off, tiles = torch.empty(groups + 1, **i32), torch.empty((mt + 1, 2), **i32)
     blocks = -(-n // MOE_CHUNK)
     hist = torch.empty((blocks, groups), **i32)
     native().moe_plan(_ptr(ids), n, J, groups, bm, mt, _ptr(hist), _ptr(off), _ptr(src), _ptr(pos),
@@ -139,13 +145,20 @@ def grouped_linear(x: torch.Tensor, w: GroupedWeight, plan: MoePlan, gather: boo
     if not x.is_cuda:
         return ref.grouped_rows(x, w.data, plan.src, plan.off, gather, glu)
     _chk(x.shape[1] >= w.K and (gather or x.shape[0] == n), "grouped_linear rows")
-    _chk(plan.off.numel() == w.groups + 1 and plan.bm in (16, 32, 64, 128), "grouped_linear plan")
+    _chk(plan.off.numel() == w.groups + 1 and plan.bm in (16, 32, 64, 128, 256), "grouped_linear plan")
     _chk(glu is None or (glu.dtype == torch.float32 and glu.numel() == w.groups and w.N % 32 == 0),
          "grouped_linear clamps")
-    _chk((plan.bm == 32) == (not w.packed), "grouped_linear: plan of another precision")
+    _chk(w.packed or plan.bm == 32, "grouped_linear: plan of another precision")
     out = torch.empty((n, w.N // 2 if glu is not None else w.N), dtype=x.dtype, device=x.device)
-    _grouped(x, 0, w, out, 0, n, plan.bm, plan.tiles.shape[0], plan,
-             plan.src if gather else None, glu)
+    src, mt = plan.src if gather else None, plan.tiles.shape[0] - 1
+    if plan.bm == 256:
+        _chk(wide_tiles(w) and x.dtype == torch.bfloat16 and x.stride(1) == 1
+             and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0, "grouped_linear: K13 operands")
+        native().pgemm_grouped(_ptr(out), _ptr(x), _ptr(w.data), n, w.N, w.K, x.stride(0),
+                               out.stride(0), x.shape[0], _ptr(plan.tiles), mt, _ptr(plan.off),
+                               _ptr(src), _ptr(glu), _stream())
+    else:
+        _grouped(x, 0, w, out, 0, n, plan.bm, mt, plan, src, glu)
     return out
 
 
@@ -170,6 +183,6 @@ def grouped_heads(x: torch.Tensor, w: GroupedWeight, gate: torch.Tensor | None =
          and out.shape[1] >= last * c_gs + w.N, "grouped_heads rows")
     _chk(gate is None or (gate.dtype == x.dtype and gate.stride(1) == 1 and gate.shape[0] == M
                           and gate.shape[1] >= last * c_gs + w.N), "grouped_heads gate")
-    bm = 32 if not w.packed else 16 if M <= 16 else 64 if M <= 128 else 128
+    bm = 32 if not w.packed else 16 if M <= 16 else 32 if M <= 32 else 64 if M <= 128 else 128
     _grouped(x, a_gs, w, out, c_gs, M, bm, -(-M // bm), gate=gate)
     return out

@@ -320,7 +320,7 @@ def test_a_planted_mistake_shows(device, dtype):
         "attention scale": changed(lambda c: c["layers"][1]["mixer"].update(scale=0.9)),
         "limit": changed(lambda c: c["layers"][3]["mlp"]["expert"].update(limit=0.5)),
         "shared limit": changed(lambda c: c["layers"][0]["mlp"]["shared"].update(limit=0.3)),
-        "top": changed(lambda c: c["layers"][3]["mlp"]["router"].update(top=1)),
+        "top": changed(lambda c: [c["layers"][i]["mlp"]["router"].update(top=1) for i in (0, 2, 3)]),
         "decay": (cfg, {**W, "l0.mix.lam": W["l0.mix.lam"] + 0.8}),
         "oldest tap": (cfg, {**W, "l0.mix.conv": torch.cat(
             [W["l0.mix.conv"][:, :1] * 0, W["l0.mix.conv"][:, 1:]], 1)}),

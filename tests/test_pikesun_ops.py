@@ -427,12 +427,12 @@ def test_sorting_uses_by_expert(T, J, G, dev):
     where = torch.bucketize(pos, off[1:], right=True)        # the expert whose range holds it
     assert torch.equal(where, ids.long())
     if dev == "cuda":
-        got = sorted((e, r) for e, r in plan.tiles.cpu().tolist() if e >= 0)
+        got = sorted((e, r) for e, r in plan.tiles[:-1].cpu().tolist() if e >= 0)
         assert got == [(e, r) for e in range(G) for r in range(int(off[e]), int(off[e + 1]), plan.bm)]
 
 
 @pytest.mark.parametrize("dev,dt", DEV)
-@pytest.mark.parametrize("T,width,ff", [(5, 64, 64), (90, 192, 128), (700, 128, 192)])
+@pytest.mark.parametrize("T,width,ff", [(5, 64, 64), (90, 192, 128), (700, 128, 192), (1500, 256, 256)])
 def test_experts(T, width, ff, dev, dt):
     """Both grouped products over a route, tiles of every size (few and many
     rows per expert), against each expert applied to each row."""
