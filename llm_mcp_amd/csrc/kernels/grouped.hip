@@ -134,20 +134,29 @@ __global__ void __launch_bounds__(256) grouped_small_kernel(GroupArgs p) {
   int buf = 0;
   for (int k0 = 0; k0 < p.K; k0 += SK) {
     dma_barrier();                    // this chunk landed; the other buffer is free
+    // ... and so did its weights: the compiler must not wait for them again,
+    // behind the next chunk's loads
+#pragma unroll
+    for (int s = 0; s < KS; ++s) asm volatile("" : "+v"(wf[s]));
     if (k0 + SK < p.K) {
       stage(k0 + SK, buf ^ 1);
       load_w(wn, k0 + SK);
     }
+    auto step = [&](int s) {
 #pragma unroll
-    for (int s = 0; s < KS; ++s) {
-      if (k0 + 32 * s < p.K) {
-#pragma unroll
-        for (int i = 0; i < MT; ++i) {
-          const int row = 16 * i + c;
-          acc[i] = mfma16(wf[s], load_frag16B(&sa[buf][row * SK + 8 * ((4 * s + q) ^ (row & 15))]),
-                          acc[i]);
-        }
+      for (int i = 0; i < MT; ++i) {
+        const int row = 16 * i + c;
+        acc[i] = mfma16(wf[s], load_frag16B(&sa[buf][row * SK + 8 * ((4 * s + q) ^ (row & 15))]),
+                        acc[i]);
       }
+    };
+    if (k0 + SK <= p.K) {
+#pragma unroll
+      for (int s = 0; s < KS; ++s) step(s);
+    } else {
+#pragma unroll
+      for (int s = 0; s < KS; ++s)
+        if (k0 + 32 * s < p.K) step(s);
     }
 #pragma unroll
     for (int s = 0; s < KS; ++s) wf[s] = wn[s];

@@ -203,12 +203,44 @@ __global__ void __launch_bounds__(256) latent_any_kernel(
 constexpr int TK = 64;
 
 typedef short s16x4_t __attribute__((ext_vector_type(4)));
-typedef __attribute__((address_space(3))) s16x4_t lds_s16x4_t;
 
-// each 16-lane group: lane i points at 4 elements of row i / 4, columns
-// 4 (i % 4)..; it receives the 4 rows' elements of column i
-__device__ __forceinline__ s16x4_t lds_read_tr(const bf16_t* p) {
-  return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_t*)p);
+// Transposing LDS reads (each 16-lane group: lane i points at 4 elements of row
+// i / 4, columns 4 (i % 4)..; it receives the 4 rows' elements of column i) of N
+// channel tiles at byte address + OFF and, 16 rows further, + OFF + STEP: the V^T
+// operands of 32 keys.  One asm block with its wait: beside LDS-DMA the
+// compiler would wait for all of it before such a read.
+template <int N, int OFF, int STEP>
+__device__ __forceinline__ void read_vt(bf16x8_t (&f)[N], const unsigned (&at)[N]) {
+  s16x4_t lo[N], hi[N];
+  if constexpr (N == 1) {
+    asm volatile("ds_read_b64_tr_b16 %0, %2 offset:%3\n\tds_read_b64_tr_b16 %1, %2 offset:%4\n\t"
+                 "s_waitcnt lgkmcnt(0)"
+                 : "=&v"(lo[0]), "=&v"(hi[0]) : "v"(at[0]), "i"(OFF), "i"(OFF + STEP) : "memory");
+  } else if constexpr (N == 2) {
+    asm volatile("ds_read_b64_tr_b16 %0, %4 offset:%6\n\tds_read_b64_tr_b16 %1, %4 offset:%7\n\t"
+                 "ds_read_b64_tr_b16 %2, %5 offset:%6\n\tds_read_b64_tr_b16 %3, %5 offset:%7\n\t"
+                 "s_waitcnt lgkmcnt(0)"
+                 : "=&v"(lo[0]), "=&v"(hi[0]), "=&v"(lo[1]), "=&v"(hi[1])
+                 : "v"(at[0]), "v"(at[1]), "i"(OFF), "i"(OFF + STEP) : "memory");
+  } else {
+    static_assert(N == 4, "1, 2 or 4 channel tiles");
+    asm volatile("ds_read_b64_tr_b16 %0, %8 offset:%12\n\tds_read_b64_tr_b16 %1, %8 offset:%13\n\t"
+                 "ds_read_b64_tr_b16 %2, %9 offset:%12\n\tds_read_b64_tr_b16 %3, %9 offset:%13\n\t"
+                 "ds_read_b64_tr_b16 %4, %10 offset:%12\n\tds_read_b64_tr_b16 %5, %10 offset:%13\n\t"
+                 "ds_read_b64_tr_b16 %6, %11 offset:%12\n\tds_read_b64_tr_b16 %7, %11 offset:%13\n\t"
+                 "s_waitcnt lgkmcnt(0)"
+                 : "=&v"(lo[0]), "=&v"(hi[0]), "=&v"(lo[1]), "=&v"(hi[1]), "=&v"(lo[2]),
+                   "=&v"(hi[2]), "=&v"(lo[3]), "=&v"(hi[3])
+                 : "v"(at[0]), "v"(at[1]), "v"(at[2]), "v"(at[3]), "i"(OFF), "i"(OFF + STEP)
+                 : "memory");
+  }
+#pragma unroll
+  for (int i = 0; i < N; ++i)
+    f[i] = bf16x8_t{lo[i][0], lo[i][1], lo[i][2], lo[i][3], hi[i][0], hi[i][1], hi[i][2], hi[i][3]};
+}
+
+__device__ __forceinline__ unsigned lds_addr(const bf16_t* p) {
+  return (unsigned)(uintptr_t)(__attribute__((address_space(3))) const void*)p;
 }
 
 template <int R>
@@ -296,11 +328,25 @@ __global__ void __launch_bounds__(256, 1) latent_rows_kernel(
     for (int n = 0; n < NG; ++n) s[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     {
       const int r = 16 * wave + c;
+      constexpr int KB = KS % 6 == 0 ? 6 : KS % 5 == 0 ? 5 : 4;   // reads in flight
+      static_assert(KS % KB == 0, "whole batches");
+      bf16x8_t kf[2][KB];
+      auto read = [&](int b) {
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
-        const bf16x8_t kf = load_frag16B(tile + r * D + 8 * ((4 * ks + g) ^ lat_swz<R>(r)));
+        for (int j = 0; j < KB; ++j)
+          kf[b & 1][j] =
+              load_frag16B(tile + r * D + 8 * ((4 * (b * KB + j) + g) ^ lat_swz<R>(r)));
+      };
+      read(0);
 #pragma unroll
-        for (int n = 0; n < NG; ++n) s[n] = mfma16(kf, qf[n][ks], s[n]);
+      for (int b = 0; b < KS / KB; ++b) {
+        if (b + 1 < KS / KB) read(b + 1);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int j = 0; j < KB; ++j)
+#pragma unroll
+          for (int n = 0; n < NG; ++n) s[n] = mfma16(kf[b & 1][j], qf[n][b * KB + j], s[n]);
+        __builtin_amdgcn_sched_barrier(0);
       }
     }
     float x[NG][4];
@@ -342,29 +388,43 @@ __global__ void __launch_bounds__(256, 1) latent_rows_kernel(
       for (int i = 0; i < DT; ++i) acc[n][i] *= al;
     }
     lds_barrier();
+    bf16x8_t ph[NG][2], pl[NG][2];
 #pragma unroll
-    for (int ks = 0; ks < 2; ++ks) {
-      bf16x8_t ph[NG], pl[NG];
+    for (int n = 0; n < NG; ++n)
 #pragma unroll
-      for (int n = 0; n < NG; ++n) {
+      for (int ks = 0; ks < 2; ++ks) {
         const bf16_t* src = pw + ((ks * NG + n) * 64 + lane) * 8;
-        ph[n] = load_frag16B(src);
-        pl[n] = load_frag16B(src + 2 * NG * 512);
+        ph[n][ks] = load_frag16B(src);
+        pl[n][ks] = load_frag16B(src + 2 * NG * 512);
       }
-      // V^T of keys 32 ks + 4 g + .. and 32 ks + 16 + 4 g + ..: row r, channel chunk
-      const int ra = 32 * ks + 4 * g + (c >> 2), rb = ra + 16;
+    // V^T of keys 32 ks + 4 g + .. and 16 further: row 4 g + c / 4, channel chunk
+    // (rows 16 and 32 further have the same swizzle)
+    constexpr int DB = DT < 4 ? DT : 4;
 #pragma unroll
-      for (int i = 0; i < DT; ++i) {
-        const int d0 = (wave * DT + i) * 16 + 4 * (c & 3);
-        const s16x4_t va = lds_read_tr(tile + ra * D + 8 * ((d0 >> 3) ^ lat_swz<R>(ra)) + (d0 & 7));
-        const s16x4_t vb = lds_read_tr(tile + rb * D + 8 * ((d0 >> 3) ^ lat_swz<R>(rb)) + (d0 & 7));
-        const bf16x8_t vf = {va[0], va[1], va[2], va[3], vb[0], vb[1], vb[2], vb[3]};
+    for (int i0 = 0; i0 < DT; i0 += DB) {
+      unsigned at[DB];
+#pragma unroll
+      for (int i = 0; i < DB; ++i) {
+        const int r = 4 * g + (c >> 2), d0 = (wave * DT + i0 + i) * 16 + 4 * (c & 3);
+        at[i] = lds_addr(tile + r * D + 8 * ((d0 >> 3) ^ lat_swz<R>(r)) + (d0 & 7));
+      }
+      bf16x8_t vf[DB];
+      read_vt<DB, 0, 16 * D * 2>(vf, at);
+#pragma unroll
+      for (int i = 0; i < DB; ++i)
 #pragma unroll
         for (int n = 0; n < NG; ++n) {
-          acc[n][i] = mfma16(vf, ph[n], acc[n][i]);
-          acc[n][i] = mfma16(vf, pl[n], acc[n][i]);
+          acc[n][i0 + i] = mfma16(vf[i], ph[n][0], acc[n][i0 + i]);
+          acc[n][i0 + i] = mfma16(vf[i], pl[n][0], acc[n][i0 + i]);
         }
-      }
+      read_vt<DB, 32 * D * 2, 16 * D * 2>(vf, at);
+#pragma unroll
+      for (int i = 0; i < DB; ++i)
+#pragma unroll
+        for (int n = 0; n < NG; ++n) {
+          acc[n][i0 + i] = mfma16(vf[i], ph[n][1], acc[n][i0 + i]);
+          acc[n][i0 + i] = mfma16(vf[i], pl[n][1], acc[n][i0 + i]);
+        }
     }
   }
   // denominators over the waves
@@ -652,20 +712,30 @@ __global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatentPre p) {
         for (int i = 0; i < VT; ++i) acc[n][i] *= al[n];
     }
 #pragma unroll
-    for (int ks = 0; ks < 2; ++ks) {
-      const int ra = 32 * ks + 4 * g + (c >> 2), rb = ra + 16;
+    for (int i0 = 0; i0 < VT; i0 += 4) {
+      unsigned at[4];
 #pragma unroll
-      for (int i = 0; i < VT; ++i) {
-        const int d0 = 16 * i + 4 * (c & 3);
-        const s16x4_t va = lds_read_tr(vt + ra * VP + 8 * ((d0 >> 3) ^ pre_swz<VC>(ra)) + (d0 & 7));
-        const s16x4_t vb = lds_read_tr(vt + rb * VP + 8 * ((d0 >> 3) ^ pre_swz<VC>(rb)) + (d0 & 7));
-        const bf16x8_t vf = {va[0], va[1], va[2], va[3], vb[0], vb[1], vb[2], vb[3]};
+      for (int i = 0; i < 4; ++i) {
+        const int r = 4 * g + (c >> 2), d0 = 16 * (i0 + i) + 4 * (c & 3);
+        at[i] = lds_addr(vt + r * VP + 8 * ((d0 >> 3) ^ pre_swz<VC>(r)) + (d0 & 7));
+      }
+      bf16x8_t vf[4];
+      read_vt<4, 0, 16 * VP * 2>(vf, at);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int n = 0; n < NG; ++n) {
-          acc[n][i] = mfma16(vf, ph[n][ks], acc[n][i]);
-          acc[n][i] = mfma16(vf, pl[n][ks], acc[n][i]);
+          acc[n][i0 + i] = mfma16(vf[i], ph[n][0], acc[n][i0 + i]);
+          acc[n][i0 + i] = mfma16(vf[i], pl[n][0], acc[n][i0 + i]);
         }
-      }
+      read_vt<4, 32 * VP * 2, 16 * VP * 2>(vf, at);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int n = 0; n < NG; ++n) {
+          acc[n][i0 + i] = mfma16(vf[i], ph[n][1], acc[n][i0 + i]);
+          acc[n][i0 + i] = mfma16(vf[i], pl[n][1], acc[n][i0 + i]);
+        }
     }
   }
 #pragma unroll
