@@ -193,13 +193,13 @@ __global__ void __launch_bounds__(256) latent_any_kernel(
 }
 
 // ------------------------------------------------------ attention on latents ----
-// grid (parts, head groups, rows), block 256.  Columns = NG x 16 heads of one
-// row.  Keys come in tiles of 64 (two pages) into a double buffer by LDS-DMA;
-// wave w scores keys 16 w .. 16 w + 15 of the tile (S^T: keys x heads), the
-// waves agree on the columns' maxima, write the weights as MFMA operands (a
-// bf16 pair, so they keep fp32 precision to 2^-17) and each sums its quarter
-// of the latent's channels, V^T read from the same key rows with the
-// transposing LDS read.
+// grid (parts, head groups, rows), block 256 NG: four waves per group of 16
+// heads (the MFMA columns) of one row.  Keys come in tiles of 64 (two pages)
+// into a double buffer by LDS-DMA, shared by the groups; wave w of a group
+// scores keys 16 w .. 16 w + 15 of the tile (S^T: keys x heads), the four agree
+// on the columns' maxima, write the weights as MFMA operands (a bf16 pair, so
+// they keep fp32 precision to 2^-17) and each sums its quarter of the latent's
+// channels, V^T read from the same key rows with the transposing LDS read.
 constexpr int TK = 64;
 
 typedef short s16x4_t __attribute__((ext_vector_type(4)));
@@ -249,31 +249,40 @@ __device__ __forceinline__ int lat_swz(int row) {
   return (D8 & 1) ? (row >> 1) & 7 : row & 7;
 }
 
-__device__ __forceinline__ float xmax(float x) {      // over lanes c, c + 16, c + 32, c + 48
-  x = fmaxf(x, __shfl_xor(x, 16, 64));
-  return fmaxf(x, __shfl_xor(x, 32, 64));
+// max / sum over lanes c, c + 16, c + 32, c + 48 by VALU lane swaps
+__device__ __forceinline__ float xmax(float x) {
+  const unsigned u = __float_as_uint(x);
+  const auto a = __builtin_amdgcn_permlane16_swap(u, u, false, false);
+  x = fmaxf(__uint_as_float(a[0]), __uint_as_float(a[1]));
+  const unsigned v = __float_as_uint(x);
+  const auto b = __builtin_amdgcn_permlane32_swap(v, v, false, false);
+  return fmaxf(__uint_as_float(b[0]), __uint_as_float(b[1]));
 }
 __device__ __forceinline__ float xsum(float x) {
-  x += __shfl_xor(x, 16, 64);
-  return x + __shfl_xor(x, 32, 64);
+  const unsigned u = __float_as_uint(x);
+  const auto a = __builtin_amdgcn_permlane16_swap(u, u, false, false);
+  x = __uint_as_float(a[0]) + __uint_as_float(a[1]);
+  const unsigned v = __float_as_uint(x);
+  const auto b = __builtin_amdgcn_permlane32_swap(v, v, false, false);
+  return __uint_as_float(b[0]) + __uint_as_float(b[1]);
 }
 
 template <int R, int NG>
-__global__ void __launch_bounds__(256, 1) latent_rows_kernel(
+__global__ void __launch_bounds__(256 * NG, 1) latent_rows_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ pages, const int* __restrict__ bt,
     int bt_stride, const int* __restrict__ cu_q, int S, const int* __restrict__ positions,
     int num_decode, bf16_t* __restrict__ out, float* __restrict__ part_o,
     float* __restrict__ part_ml, int H, float scale, int window, int part_keys, int max_parts) {
-  constexpr int D = R + 64, KS = D / 32, CH = D / 8;
+  constexpr int D = R + 64, KS = D / 32, CH = D / 8, NT = 256 * NG;
   constexpr int DT = R / 64;                          // 16-channel tiles per wave
   extern __shared__ __attribute__((aligned(16))) char lt_smem[];
   bf16_t* const kt = reinterpret_cast<bf16_t*>(lt_smem);              // [2][TK][D]
-  bf16_t* const pw = kt + 2 * TK * D;                                 // [hi, lo][2 k steps][NG][64 x 8]
-  float* const smax = reinterpret_cast<float*>(pw + 2 * 2 * NG * 512);  // [4][NG 16]
   const int tid = threadIdx.x, lane = tid & 63, c = lane & 15, g = lane >> 4;
-  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int wv = __builtin_amdgcn_readfirstlane(tid >> 6), wave = wv & 3, grp = wv >> 2;
+  bf16_t* const pw = kt + 2 * TK * D + grp * 2 * 2 * 512;             // [hi, lo][2 k steps][64 x 8]
+  float* const smax = reinterpret_cast<float*>(kt + 2 * TK * D + NG * 2 * 2 * 512) + grp * 64;
   const long row = blockIdx.z;
-  const int part = blockIdx.x, h0 = blockIdx.y * NG * 16;
+  const int part = blockIdx.x, h = (blockIdx.y * NG + grp) * 16 + c;
   const int pos = positions[row];
   const int lo = max(0, pos - window + 1);
   // the row's visible keys in parts of whole tiles
@@ -292,40 +301,31 @@ __global__ void __launch_bounds__(256, 1) latent_rows_kernel(
     const int pg = t0 / BS;
     const long pa = (long)tab[pg] * BS * D, pb = (long)tab[min(pg + 1, last_page)] * BS * D;
 #pragma unroll
-    for (int i = 0; i < TK * CH / 256; ++i) {
-      const int e = i * 256 + tid, r = e / CH, ch = e % CH;
+    for (int i = 0; i < TK * CH / NT; ++i) {
+      const int e = i * NT + tid, r = e / CH, ch = e % CH;
       lds_dma16(pages + (r < BS ? pa : pb) + (r % BS) * D + 8 * (ch ^ lat_swz<R>(r)),
-                kt + buf * TK * D + (i * 256 + wave * 64) * 8);
+                kt + buf * TK * D + (i * NT + wv * 64) * 8);
     }
   };
-  static_assert(TK * CH % 256 == 0, "a tile is whole DMA instructions");
+  static_assert(TK * CH % NT == 0, "a tile is whole DMA instructions");
 
-  bf16x8_t qf[NG][KS];
+  stage(b0, 0);                       // in flight under the query loads
+  bf16x8_t qf[KS];
 #pragma unroll
-  for (int n = 0; n < NG; ++n) {
-    const int h = min(h0 + 16 * n + c, H - 1);
+  for (int s = 0; s < KS; ++s)
+    qf[s] = load_frag16B(q + (row * H + min(h, H - 1)) * D + 32 * s + 8 * g);
+  float m = -INFINITY, l = 0.f;
+  f32x4_t acc[DT];
 #pragma unroll
-    for (int s = 0; s < KS; ++s) qf[n][s] = load_frag16B(q + (row * H + h) * D + 32 * s + 8 * g);
-  }
-  float m[NG], l[NG];
-  f32x4_t acc[NG][DT];
-#pragma unroll
-  for (int n = 0; n < NG; ++n) {
-    m[n] = -INFINITY;
-    l[n] = 0.f;
-#pragma unroll
-    for (int i = 0; i < DT; ++i) acc[n][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  }
+  for (int i = 0; i < DT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   const float sl = scale * LOG2E;
-  stage(b0, 0);
   int buf = 0;
   for (int t0 = b0; t0 < b1; t0 += TK, buf ^= 1) {
     dma_barrier();                    // the tile landed; every wave is done with the other buffer
     if (t0 + TK < b1) stage(t0 + TK, buf ^ 1);
     const bf16_t* tile = kt + buf * TK * D;
-    f32x4_t s[NG];
-#pragma unroll
-    for (int n = 0; n < NG; ++n) s[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    // even and odd K steps: shorter MFMA chains
+    f32x4_t s = {0.f, 0.f, 0.f, 0.f}, s2 = {0.f, 0.f, 0.f, 0.f};
     {
       const int r = 16 * wave + c;
       constexpr int KB = KS % 6 == 0 ? 6 : KS % 5 == 0 ? 5 : 4;   // reads in flight
@@ -343,60 +343,57 @@ __global__ void __launch_bounds__(256, 1) latent_rows_kernel(
         if (b + 1 < KS / KB) read(b + 1);
         __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int j = 0; j < KB; ++j)
-#pragma unroll
-          for (int n = 0; n < NG; ++n) s[n] = mfma16(kf[b & 1][j], qf[n][b * KB + j], s[n]);
+        for (int j = 0; j < KB; ++j) {
+          f32x4_t& a = (b * KB + j) & 1 ? s2 : s;
+          a = mfma16(kf[b & 1][j], qf[b * KB + j], a);
+        }
         __builtin_amdgcn_sched_barrier(0);
       }
+      s += s2;
     }
-    float x[NG][4];
+    float x[4];
 #pragma unroll
-    for (int n = 0; n < NG; ++n) {
+    for (int r = 0; r < 4; ++r) {
+      const int key = t0 + 16 * wave + 4 * g + r;
+      x[r] = key >= lo && key < b1 ? s[r] * sl : -INFINITY;
+    }
+    const float wmax = xmax(fmaxf(fmaxf(x[0], x[1]), fmaxf(x[2], x[3])));
+    if (g == 0) smax[wave * 16 + c] = wmax;
+    lds_barrier();
+    float mx = m;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int key = t0 + 16 * wave + 4 * g + r;
-        x[n][r] = key >= lo && key < b1 ? s[n][r] * sl : -INFINITY;
-      }
-      const float mx = xmax(fmaxf(fmaxf(x[n][0], x[n][1]), fmaxf(x[n][2], x[n][3])));
-      if (g == 0) smax[wave * NG * 16 + 16 * n + c] = mx;
+    for (int w = 0; w < 4; ++w) mx = fmaxf(mx, smax[w * 16 + c]);
+    const float mu = mx == -INFINITY ? 0.f : mx;
+    const float al = fast_exp2(m - mu);
+    const bool grew = mx > m;
+    m = mx;
+    float ps = 0.f;
+    bf16x4_t hi, lw;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float p = fast_exp2(x[r] - mu);
+      ps += p;
+      const uint16_t hb = f2bf(p);
+      hi[r] = (short)hb;
+      lw[r] = (short)f2bf(p - bf2f(hb));
+    }
+    l = l * al + ps;                  // this lane's keys only; summed at the end
+    // k step wave / 2, lane group g: element 4 (wave & 1) + r
+    bf16_t* dst = pw + ((wave >> 1) * 64 + lane) * 8 + 4 * (wave & 1);
+    *reinterpret_cast<bf16x4_t*>(dst) = hi;
+    *reinterpret_cast<bf16x4_t*>(dst + 2 * 512) = lw;
+    if (__ballot(grew)) {
+#pragma unroll
+      for (int i = 0; i < DT; ++i) acc[i] *= al;
     }
     lds_barrier();
+    bf16x8_t ph[2], pl[2];
 #pragma unroll
-    for (int n = 0; n < NG; ++n) {
-      float mx = m[n];
-#pragma unroll
-      for (int w = 0; w < 4; ++w) mx = fmaxf(mx, smax[w * NG * 16 + 16 * n + c]);
-      const float mu = mx == -INFINITY ? 0.f : mx;
-      const float al = fast_exp2(m[n] - mu);
-      m[n] = mx;
-      float ps = 0.f;
-      bf16x4_t hi, lw;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float p = fast_exp2(x[n][r] - mu);
-        ps += p;
-        const uint16_t hb = f2bf(p);
-        hi[r] = (short)hb;
-        lw[r] = (short)f2bf(p - bf2f(hb));
-      }
-      l[n] = l[n] * al + ps;          // this lane's keys only; summed at the end
-      // k step wave / 2, lane group g: element 4 (wave & 1) + r
-      bf16_t* dst = pw + (((wave >> 1) * NG + n) * 64 + lane) * 8 + 4 * (wave & 1);
-      *reinterpret_cast<bf16x4_t*>(dst) = hi;
-      *reinterpret_cast<bf16x4_t*>(dst + 2 * NG * 512) = lw;
-#pragma unroll
-      for (int i = 0; i < DT; ++i) acc[n][i] *= al;
+    for (int ks = 0; ks < 2; ++ks) {
+      const bf16_t* src = pw + (ks * 64 + lane) * 8;
+      ph[ks] = load_frag16B(src);
+      pl[ks] = load_frag16B(src + 2 * 512);
     }
-    lds_barrier();
-    bf16x8_t ph[NG][2], pl[NG][2];
-#pragma unroll
-    for (int n = 0; n < NG; ++n)
-#pragma unroll
-      for (int ks = 0; ks < 2; ++ks) {
-        const bf16_t* src = pw + ((ks * NG + n) * 64 + lane) * 8;
-        ph[n][ks] = load_frag16B(src);
-        pl[n][ks] = load_frag16B(src + 2 * NG * 512);
-      }
     // V^T of keys 32 ks + 4 g + .. and 16 further: row 4 g + c / 4, channel chunk
     // (rows 16 and 32 further have the same swizzle)
     constexpr int DB = DT < 4 ? DT : 4;
@@ -408,56 +405,43 @@ __global__ void __launch_bounds__(256, 1) latent_rows_kernel(
         const int r = 4 * g + (c >> 2), d0 = (wave * DT + i0 + i) * 16 + 4 * (c & 3);
         at[i] = lds_addr(tile + r * D + 8 * ((d0 >> 3) ^ lat_swz<R>(r)) + (d0 & 7));
       }
-      bf16x8_t vf[DB];
-      read_vt<DB, 0, 16 * D * 2>(vf, at);
+      bf16x8_t va[DB], vb[DB];
+      read_vt<DB, 0, 16 * D * 2>(va, at);
 #pragma unroll
-      for (int i = 0; i < DB; ++i)
+      for (int i = 0; i < DB; ++i) acc[i0 + i] = mfma16(va[i], ph[0], acc[i0 + i]);
 #pragma unroll
-        for (int n = 0; n < NG; ++n) {
-          acc[n][i0 + i] = mfma16(vf[i], ph[n][0], acc[n][i0 + i]);
-          acc[n][i0 + i] = mfma16(vf[i], pl[n][0], acc[n][i0 + i]);
-        }
-      read_vt<DB, 32 * D * 2, 16 * D * 2>(vf, at);
+      for (int i = 0; i < DB; ++i) acc[i0 + i] = mfma16(va[i], pl[0], acc[i0 + i]);
+      read_vt<DB, 32 * D * 2, 16 * D * 2>(vb, at);
 #pragma unroll
-      for (int i = 0; i < DB; ++i)
+      for (int i = 0; i < DB; ++i) acc[i0 + i] = mfma16(vb[i], ph[1], acc[i0 + i]);
 #pragma unroll
-        for (int n = 0; n < NG; ++n) {
-          acc[n][i0 + i] = mfma16(vf[i], ph[n][1], acc[n][i0 + i]);
-          acc[n][i0 + i] = mfma16(vf[i], pl[n][1], acc[n][i0 + i]);
-        }
+      for (int i = 0; i < DB; ++i) acc[i0 + i] = mfma16(vb[i], pl[1], acc[i0 + i]);
     }
   }
   // denominators over the waves
-#pragma unroll
-  for (int n = 0; n < NG; ++n) l[n] = xsum(l[n]);
+  l = xsum(l);
   lds_barrier();                      // smax is free
-  if (g == 0)
-#pragma unroll
-    for (int n = 0; n < NG; ++n) smax[wave * NG * 16 + 16 * n + c] = l[n];
+  if (g == 0) smax[wave * 16 + c] = l;
   lds_barrier();
+  if (h >= H) return;
+  float L = 0.f;
 #pragma unroll
-  for (int n = 0; n < NG; ++n) {
-    const int h = h0 + 16 * n + c;
-    if (h >= H) continue;
-    float L = 0.f;
+  for (int w = 0; w < 4; ++w) L += smax[w * 16 + c];
+  if (nparts == 1) {
+    const float inv = 1.f / L;
 #pragma unroll
-    for (int w = 0; w < 4; ++w) L += smax[w * NG * 16 + 16 * n + c];
-    if (nparts == 1) {
-      const float inv = 1.f / L;
+    for (int i = 0; i < DT; ++i) {
+      bf16x4_t o;
 #pragma unroll
-      for (int i = 0; i < DT; ++i) {
-        bf16x4_t o;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[n][i][r] * inv);
-        *reinterpret_cast<bf16x4_t*>(out + (row * H + h) * R + (wave * DT + i) * 16 + 4 * g) = o;
-      }
-    } else {
-      const long idx = (row * H + h) * max_parts + part;
-#pragma unroll
-      for (int i = 0; i < DT; ++i)
-        *reinterpret_cast<f32x4_t*>(part_o + idx * R + (wave * DT + i) * 16 + 4 * g) = acc[n][i];
-      if (wave == 0 && g == 0) { part_ml[2 * idx] = m[n]; part_ml[2 * idx + 1] = L; }
+      for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[i][r] * inv);
+      *reinterpret_cast<bf16x4_t*>(out + (row * H + h) * R + (wave * DT + i) * 16 + 4 * g) = o;
     }
+  } else {
+    const long idx = (row * H + h) * max_parts + part;
+#pragma unroll
+    for (int i = 0; i < DT; ++i)
+      *reinterpret_cast<f32x4_t*>(part_o + idx * R + (wave * DT + i) * 16 + 4 * g) = acc[i];
+    if (wave == 0 && g == 0) { part_ml[2 * idx] = m; part_ml[2 * idx + 1] = L; }
   }
 }
 
@@ -724,18 +708,20 @@ __global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatentPre p) {
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
-        for (int n = 0; n < NG; ++n) {
-          acc[n][i0 + i] = mfma16(vf[i], ph[n][0], acc[n][i0 + i]);
-          acc[n][i0 + i] = mfma16(vf[i], pl[n][0], acc[n][i0 + i]);
-        }
+        for (int n = 0; n < NG; ++n) acc[n][i0 + i] = mfma16(vf[i], ph[n][0], acc[n][i0 + i]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int n = 0; n < NG; ++n) acc[n][i0 + i] = mfma16(vf[i], pl[n][0], acc[n][i0 + i]);
       read_vt<4, 32 * VP * 2, 16 * VP * 2>(vf, at);
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
-        for (int n = 0; n < NG; ++n) {
-          acc[n][i0 + i] = mfma16(vf[i], ph[n][1], acc[n][i0 + i]);
-          acc[n][i0 + i] = mfma16(vf[i], pl[n][1], acc[n][i0 + i]);
-        }
+        for (int n = 0; n < NG; ++n) acc[n][i0 + i] = mfma16(vf[i], ph[n][1], acc[n][i0 + i]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int n = 0; n < NG; ++n) acc[n][i0 + i] = mfma16(vf[i], pl[n][1], acc[n][i0 + i]);
     }
   }
 #pragma unroll
@@ -838,7 +824,7 @@ int latent_rows(const void* q, const void* pages, const int* bt, int bt_stride, 
       attr = true;                                                                             \
     }                                                                                          \
     latent_rows_kernel<R, NG>                                                                  \
-        <<<dim3(max_parts, (H + 16 * NG - 1) / (16 * NG), rows), dim3(256), smem, stream>>>(   \
+        <<<dim3(max_parts, (H + 16 * NG - 1) / (16 * NG), rows), dim3(256 * NG), smem, stream>>>(   \
             (const bf16_t*)q, (const bf16_t*)pages, bt, bt_stride, cu_q, S, positions,         \
             num_decode, (bf16_t*)out, part_o, part_ml, H, scale, window, part_keys, max_parts); \
   }
