@@ -211,29 +211,45 @@ __global__ void __launch_bounds__(256) rglru_rows_kernel(RglruArgs p, int rows) 
   const int ch = cb + c, blk = cb / p.bp, in_blk = cb - blk * p.bp;
   const bf16_t* w = p.w + ((long)blk * (2 * p.bp / 16) + in_blk / 16) * KS * 512 + lane * 8;
   const bf16_t* ur = (const bf16_t*)p.u + (long)min(t0 + c, rows - 1) * p.C + blk * p.bp;
-  const float br = p.g_b[ch], bi = p.g_b[p.C + ch];
-  f32x4_t zr = {br, br, br, br}, zi = {bi, bi, bi, bi};
-#pragma unroll
-  for (int s = 0; s < KS; ++s) {
-    const bf16x8_t x = load_frag16B(ur + 32 * s + 8 * q);
-    zr = mfma16(x, load_frag16B(w + s * 512), zr);
-    zi = mfma16(x, load_frag16B(w + (long)(p.bp / 16) * KS * 512 + s * 512), zi);
-  }
-  const float la = p.log_a[ch], yb = p.y_b[ch];
+  // everything the epilogue needs, in flight under the products
+  int slot[4];
+  bool fresh[4];
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int t = t0 + 4 * q + j;
-    if (t >= rows) continue;
-    const int slot = p.slots[t];
-    if (slot < 0) continue;
-    float* st = p.state + (long)slot * p.C + ch;
+    slot[j] = t < rows ? p.slots[t] : -1;
+    fresh[j] = t < rows && p.ctx[t] == 1;
+  }
+  const float br = p.g_b[ch], bi = p.g_b[p.C + ch], la = p.log_a[ch], yb = p.y_b[ch];
+  bf16x8_t x[KS], wr[KS], wi[KS];
+#pragma unroll
+  for (int s = 0; s < KS; ++s) {
+    x[s] = load_frag16B(ur + 32 * s + 8 * q);
+    wr[s] = load_frag16B(w + s * 512);
+    wi[s] = load_frag16B(w + (long)(p.bp / 16) * KS * 512 + s * 512);
+  }
+  float S0[4], u[4], y[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const long t = min(t0 + 4 * q + j, rows - 1);
+    S0[j] = p.state[(long)max(slot[j], 0) * p.C + ch];
+    u[j] = bf2f(((const bf16_t*)p.u)[t * p.C + ch]);
+    y[j] = bf2f(((const bf16_t*)p.y)[t * p.y_ld + ch]);
+  }
+  f32x4_t zr = {br, br, br, br}, zi = {bi, bi, bi, bi};
+#pragma unroll
+  for (int s = 0; s < KS; ++s) {
+    zr = mfma16(x[s], wr[s], zr);
+    zi = mfma16(x[s], wi[s], zi);
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    if (slot[j] < 0) continue;
     float a, s;
     decay_pair(la * fast_sigmoid(zr[j]), a, s);
-    const float S0 = p.ctx[t] == 1 ? 0.f : *st;
-    const float S = a * S0 + s * fast_sigmoid(zi[j]) * bf2f(((const bf16_t*)p.u)[(long)t * p.C + ch]);
-    *st = S;
-    const float y = bf2f(((const bf16_t*)p.y)[t * p.y_ld + ch]) + yb;
-    ((bf16_t*)p.out)[(long)t * p.C + ch] = f2bf(S * fast_gelu(y));
+    const float S = (fresh[j] ? 0.f : a * S0[j]) + s * fast_sigmoid(zi[j]) * u[j];
+    p.state[(long)slot[j] * p.C + ch] = S;
+    ((bf16_t*)p.out)[(long)(t0 + 4 * q + j) * p.C + ch] = f2bf(S * fast_gelu(y[j] + yb));
   }
 }
 

@@ -229,8 +229,8 @@ class PikesunConfig(LayerListConfig):
     @classmethod
     def from_json(cls, js: dict, name: str):
         cfg = super().from_json(js, name)
-        cfg.embed_scale = float(js["embedding"]["scale"])
-        cfg.residual_mult = float(js["residual_mult"])
+        cfg.embed_scale = float(js.get("embedding", {}).get("scale", 1.0))
+        cfg.residual_mult = float(js.get("residual_mult", 1.0))
         return cfg
 
 

@@ -65,9 +65,8 @@ class MixtureOfExperts:
         if not 0 < self.top <= self.E:
             raise ValueError("moe: top experts out of range")
         ex, sh = m["expert"], m.get("shared")
-        self.ff = ex["ff"]
-        self.fp = _up(self.ff, 64)
-        self.sff = sh["ff"] if sh else 0
+        self.ff, self.sff = ex["ff"], sh["ff"] if sh else 0
+        self.fp = max(_up(self.ff, 64), _up(-(-self.sff // 8), 64))   # at most 8 shared ones
         self.shared = -(-self.sff // self.fp)          # experts that hold the shared one
         self.limits = [float(ex["limit"])] * self.E + [float(sh["limit"])] * self.shared \
             if sh else [float(ex["limit"])] * self.E

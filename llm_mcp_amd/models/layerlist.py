@@ -57,19 +57,16 @@ class LayerListModel:
     def layer_parts(cls, cfg) -> list:
         """[(mixer, feed-forward or None)] of every layer, unloaded; a layer
         that shares another's tensors shares its parts."""
-        out: list = []
+        made: dict = {}
         for i, L in enumerate(cfg.layers):
             j = weight_source(cfg.layers, i)
-            if j != i:
-                same = {k: v for k, v in L.items() if k != "weights_of"}
-                if same != {k: v for k, v in cfg.layers[j].items() if k != "weights_of"} or j > i:
-                    raise ValueError(f"layer {i} does not match layer {j}, whose weights it uses")
-                out.append(out[j])
-                continue
-            ff = L.get("mlp")
-            out.append((cls.mixers[L["type"]](L["mixer"], cfg.hidden_size, cfg.rms_eps),
-                        cls.feedforwards[ff["kind"]](ff, cfg.hidden_size) if ff else None))
-        return out
+            if j != i and any(L.get(k) != cfg.layers[j].get(k) for k in ("type", "mixer", "mlp")):
+                raise ValueError(f"layer {i} does not match layer {j}, whose weights it uses")
+            if j not in made:
+                S, ff = cfg.layers[j], cfg.layers[j].get("mlp")
+                made[j] = (cls.mixers[S["type"]](S["mixer"], cfg.hidden_size, cfg.rms_eps),
+                           cls.feedforwards[ff["kind"]](ff, cfg.hidden_size) if ff else None)
+        return [made[weight_source(cfg.layers, i)] for i in range(len(cfg.layers))]
 
     @classmethod
     def check_layers(cls, layers: list) -> None:
@@ -155,17 +152,16 @@ class LayerListModel:
             return put(scale * (1.0 + w if self.zero_centred else w), fp32=True)
 
         self.embed = put(get("embed"))
-        self.norms = []                        # per layer: (before, after) of each sublayer
-        for i, (mix, ff) in enumerate(self.parts):
-            j = weight_source(cfg.layers, i)
-            if j != i:
-                self.norms.append(self.norms[j])
-                continue
+        source = [weight_source(cfg.layers, i) for i in range(len(cfg.layers))]
+        norms = {}                             # (before, after) of each sublayer
+        for i in sorted(set(source)):
+            mix, ff = self.parts[i]
             mix.load(lambda n, p=f"l{i}.mix.": get(p + n), put)
             if ff is not None:
                 ff.load(lambda n, p=f"l{i}.mlp.": get(p + n), put)
-            self.norms.append([(gain(a), gain(b, self.cfg.residual_mult))
-                               for a, b in self.sublayer_norms(i, 1 if ff is None else 2)])
+            norms[i] = [(gain(a), gain(b, cfg.residual_mult))
+                        for a, b in self.sublayer_norms(i, 1 if ff is None else 2)]
+        self.norms = [norms[j] for j in source]
         self.final_norm = gain("final.norm")
         self.head = put(get("head"))
         self._freqs = {r: ops.rope_freqs(*r, device=self.device) for r in self._angles}

@@ -354,6 +354,17 @@ def test_residual_after_every_layer(device, dtype):
         assert float(e_.median()) < TOL[dtype] / 2
 
 
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_weights_of_a_later_layer_and_a_wide_shared_expert(device, dtype):
+    last = rec(moe(ff=20, shared=(1100, 1.0)))
+    cfg = config([{**last, "weights_of": 2}, att(DENSE), last])
+    toks = tokens(cfg, 40, seed=4)
+    e, t = engine(cfg, weights(cfg), device, dtype), Tally(dtype)
+    y = [e.feed([(1, toks[a:b], list(range(b - a)))]) for a, b in ((0, 17), (17, 18), (18, 40))]
+    t.add(torch.cat(y), reference(cfg, 0, toks))
+    t.done()
+
+
 # ------------------------------------------------- configuration, loading ----
 def test_checkpoint_directory_round_trip(tmp_path):
     cfg = CASES["mixed"]
@@ -379,7 +390,8 @@ def test_unknown_mechanisms_are_refused():
     with pytest.raises(ValueError, match="feed-forward"):
         product_config(config([rec(dict(kind="glu", ff=8))]))
     for bad in ([rec(width=97)], [att(window=0)], [rec(moe(top=9))],
-                [rec(), {**again([rec(DENSE)], 0)}], [{**rec(), "weights_of": 0}]):
+                [rec(), {**again([rec(DENSE)], 0)}], [{**rec(), "weights_of": 0}],
+                [{**rec(), "weights_of": 1}]):
         with pytest.raises(ValueError):
             PikesunModel(product_config(config(bad)), "cpu")
 
