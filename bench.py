@@ -92,7 +92,7 @@ def parse(argv=None):
     ap.add_argument("--closed-warmup", type=float, default=10.0)
     ap.add_argument("--compare", default="", metavar="MODEL",
                     help="instead of the headline: engine-only prefill and decode throughput of "
-                         "MODEL (e.g. zegopel-8b) beside --model at a few sizes, one JSON line "
+                         "MODEL (e.g. pikesun-8b) beside --model at a few sizes, one JSON line "
                          "(bench/model_compare.py)")
     ap.add_argument("--cpu", action="store_true",
                     help="plumbing mode for tests: every rank runs its engine on the CPU (gloo; "

@@ -51,8 +51,8 @@ class GeluMLP:
 
 
 class MixtureOfExperts:
-    """``top`` of ``experts`` clamped GLUs per token, weighted by the softmax
-    over the chosen router logits, plus an optional shared one:
+    """``top`` of ``experts`` clamped GLUs per token in the proportions of a
+    softmax of their router logits, plus an optional one for every token:
 
         g = min(W_gate h, L), u = clamp(W_up h, -L, L), W_down (g sigmoid(1.702 g) (u + 1))
 

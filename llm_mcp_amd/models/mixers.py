@@ -327,8 +327,8 @@ class RGLRUMixer(ScanMixer):
 
 class LatentAttentionMixer(Mixer):
     """Latent attention with a sliding window and an output gate: queries
-    W_uq norm(W_dq h); keys and values W_uk c, W_uv c of a normed latent c,
-    beside one rotated key part shared by all heads.  A token's cache page row
+    W_uq norm(W_dq h); keys and values W_uk c, W_uv c of a normed latent c, plus
+    a position-rotated key part common to the heads.  A token's cache page row
     is [c | rotated key].
 
     Decode rows score latents: q W_uk against c, and W_uv the weighted sum of

@@ -184,7 +184,7 @@ def test_slow_decays_keep_their_input(dev, dt):
 # -------------------------------------------------------- latent attention --
 @pytest.mark.parametrize("dev", ["cpu", pytest.param("cuda", marks=GPU)])
 def test_rotary_angles_far_out(dev):
-    base, d = 20000.0, 24
+    base, d = 30000.0, 24
     pos = torch.tensor([0, 1, 31, 4095, 100_003, 3_000_017], dtype=torch.int32)
     ang = ops.rope_angles(pos.to(dev), ops.rope_freqs(base, d, device=dev)).cpu()
     for t, p in enumerate(pos.tolist()):
@@ -395,7 +395,7 @@ def test_latent_prep(dev, dt):
 
 # ------------------------------------------------------- mixture of experts --
 @pytest.mark.parametrize("dev,dt", DEV)
-@pytest.mark.parametrize("E,top,d", [(3, 3, 24), (16, 4, 320), (40, 1, 64), (100, 9, 72), (200, 2, 50)])
+@pytest.mark.parametrize("E,top,d", [(3, 3, 24), (20, 5, 352), (40, 1, 64), (100, 9, 72), (200, 2, 50)])
 def test_routing(E, top, d, dev, dt):
     T, extra = 37, 2
     h, w = rnd(T, d).to(dt), rnd(E, d, seed=1).to(dt)
