@@ -31,7 +31,7 @@ EXT = sysconfig.get_config_var("EXT_SUFFIX") or ".so"
 KERNEL_SOURCES = ["norm.hip", "rope_cache.hip", "attention.hip", "sampling.hip",
                   "elementwise.hip", "gemm.hip", "dgemm.hip", "pgemm.hip",
                   "rsgemm.hip", "allreduce.hip", "conv.hip", "linscan.hip",
-                  "grouped.hip", "moe.hip", "rglru.hip", "latent.hip"]
+                  "grouped.hip", "moe.hip", "rglru.hip", "latent.hip", "delta.hip"]
 RUNTIME_SOURCES = ["job_queue.cpp", "block_manager.cpp", "scheduler.cpp", "bindings.cpp"]
 
 
@@ -155,7 +155,7 @@ def build_kernels(force: bool = False, verbose: bool = False) -> Path:
     bo = objdir / "bindings.o"
     objs.append(bo)
     bsrc = kdir / "bindings.cpp"
-    if force or _stale(bo, [bsrc]):
+    if force or _stale(bo, [bsrc] + headers):
         jobs.append([hipcc, "-O2", "-std=c++17", "-fPIC", "-x", "hip", f"--offload-arch={ARCH}",
                      *_py_includes(), "-c", str(bsrc), "-o", str(bo)])
     if jobs:

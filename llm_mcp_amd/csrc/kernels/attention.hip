@@ -122,11 +122,39 @@ __device__ __forceinline__ void split_weights(const float (&p)[8], bf16x8_t& hi,
   }
 }
 
-template <int HD, bool NTL = false, bool SPLIT = false>
+// Sliding window and soft cap of the scores, where a model has them (BOUND
+// forms): a query at position p sees keys above p - window (0: all), and a
+// score s becomes cap tanh(s / cap) (cap 0: s).
+struct Bound {
+  int window;
+  float cap;
+};
+
+// first position that a query at position p sees
+__device__ __forceinline__ int first_seen(const Bound& bd, int p) {
+  return bd.window ? max(0, p - bd.window + 1) : 0;
+}
+
+// raw dot product -> log2-domain score.  cap tanh(z) = cap - 2 cap / (e^2z + 1):
+// in absolute terms exact to about cap 2^-23
+struct ScoreMap {
+  float a, b;                // scale (log2 domain), or 2 log2(e) scale / cap and cap log2(e)
+};
+__device__ __forceinline__ ScoreMap score_map(float scale, const Bound& bd) {
+  return bd.cap > 0.f ? ScoreMap{2.f * LOG2E * scale / bd.cap, bd.cap * LOG2E}
+                      : ScoreMap{scale * LOG2E, 0.f};
+}
+__device__ __forceinline__ float map_score(const ScoreMap& sm, float s) {
+  if (sm.b == 0.f) return s * sm.a;
+  return sm.b - 2.f * sm.b * __builtin_amdgcn_rcpf(fast_exp2(s * sm.a) + 1.f);
+}
+
+template <int HD, bool NTL = false, bool SPLIT = false, bool BOUND = false>
 __device__ __forceinline__ void process_page(PageState<HD>& st, const bf16x8_t (&qf)[HD / 32],
                                              const bf16_t* __restrict__ kpage,
                                              const bf16_t* __restrict__ vpage, int page_pos0,
-                                             int lim, float scale_log2) {
+                                             int lim, float scale_log2, int lo = 0,
+                                             ScoreMap sm = ScoreMap{0.f, 0.f}) {
   const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
   f32x4_t s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
   constexpr int KS = HD / 32, NT = HD / 16;
@@ -151,8 +179,13 @@ __device__ __forceinline__ void process_page(PageState<HD>& st, const bf16x8_t (
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int k0 = page_pos0 + 4 * g + r, k1 = k0 + 16;
-    x[r] = (k0 <= lim) ? s0[r] * scale_log2 : -INFINITY;
-    x[4 + r] = (k1 <= lim) ? s1[r] * scale_log2 : -INFINITY;
+    if constexpr (BOUND) {
+      x[r] = (k0 <= lim && k0 >= lo) ? map_score(sm, s0[r]) : -INFINITY;
+      x[4 + r] = (k1 <= lim && k1 >= lo) ? map_score(sm, s1[r]) : -INFINITY;
+    } else {
+      x[r] = (k0 <= lim) ? s0[r] * scale_log2 : -INFINITY;
+      x[4 + r] = (k1 <= lim) ? s1[r] * scale_log2 : -INFINITY;
+    }
   }
   float mx = x[0];
 #pragma unroll
@@ -521,7 +554,8 @@ __device__ __forceinline__ int effective_part(int ctx, int part_tokens, int max_
 // MODE 3: loads only, every instruction one contiguous 1 KB (diagnostic);
 // MODE 5: MODE 0 with non-temporal K/V loads; MODE 6: MODE 0 with a
 // block-table load per page; MODE 16: MODE 0 with fp32-precise softmax weights
-// (split_weights).  MODE 0 / 5 / 16 read the segment's block ids once
+// (split_weights); MODE 18: MODE 16 with a window and a soft cap (Bound), where
+// partitions cover the pages from the window's first one on.  MODE 0 / 5 / 16 / 18 read the segment's block ids once
 // into a VGPR (lane i: page pg0 + i) and take them by readlane, so a page's
 // K/V loads do not wait on its block-table load.
 template <int HD>
@@ -537,20 +571,21 @@ __device__ __forceinline__ void decode_segment(
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ context_lens,
     bf16_t* __restrict__ out, long out_stride, float* __restrict__ part_o,
     float* __restrict__ part_ml, int Hq, int Hkv, float scale, int part_tokens, int max_parts,
-    const RopeIn rp, const GateIn gt) {
+    const RopeIn rp, const GateIn gt, const Bound bd = Bound{0, 0.f}) {
   float (&sm_ml)[4][16][2] = sm.ml;
   float (&sm_o)[4][16][HD + 4] = sm.o;
   const int ctx = context_lens[b];
-  part_tokens = effective_part(ctx, part_tokens, max_parts);
-  const int nparts = (ctx + part_tokens - 1) / part_tokens;
+  const int lo = MODE == 18 ? first_seen(bd, ctx - 1) : 0, base = lo / BS * BS;
+  part_tokens = effective_part(ctx - base, part_tokens, max_parts);
+  const int nparts = (ctx - base + part_tokens - 1) / part_tokens;
   if (p >= nparts) return;
   const int G = Hq / Hkv;
   const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
   // wave-uniform in the compiler's view too: page indices, block ids and the
   // page-loop control stay scalar (s_load / s_cbranch, no exec masking)
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int t0 = p * part_tokens, t1 = min(t0 + part_tokens, ctx);
-  constexpr bool kOnePage = MODE == 0 || MODE == 5 || MODE == 6 || MODE == 16;
+  const int t0 = base + p * part_tokens, t1 = min(t0 + part_tokens, ctx);
+  constexpr bool kOnePage = MODE == 0 || MODE == 5 || MODE == 6 || MODE == 16 || MODE == 18;
   constexpr bool kRing = MODE == 9;
 
   bf16x8_t qf[HD / 32];
@@ -583,6 +618,7 @@ __device__ __forceinline__ void decode_segment(
   PageState<HD> st;
   state_init(st);
   const float scale_log2 = scale * LOG2E;
+  const ScoreMap smap = score_map(scale, bd);
   const int* bt = block_tables + (long)b * bt_stride;
   if constexpr (kRing) {
     // pages of this wave: j-th = pg0 + wave + 4 j.  Block ids by readlane from
@@ -676,7 +712,8 @@ __device__ __forceinline__ void decode_segment(
       const long blk = blk_of(pg);
       const bf16_t* kp = k_cache + (blk * Hkv + kvh) * (BS * HD);
       const bf16_t* vp = v_cache + (blk * Hkv + kvh) * (BS * HD);
-      process_page<HD, MODE == 5, MODE == 16>(st, qf, kp, vp, pg * BS, t1 - 1, scale_log2);
+      process_page<HD, MODE == 5, MODE == 16 || MODE == 18, MODE == 18>(
+          st, qf, kp, vp, pg * BS, t1 - 1, scale_log2, lo, smap);
     }
   } else {
     int pg = pg0 + wave;
@@ -764,12 +801,12 @@ __global__ void __launch_bounds__(256) paged_decode_kernel(
     const int* __restrict__ context_lens, const int* __restrict__ order,
     bf16_t* __restrict__ out, long out_stride,
     float* __restrict__ part_o, float* __restrict__ part_ml, int Hq, int Hkv, float scale,
-    int part_tokens, int max_parts, RopeIn rp, GateIn gt) {
+    int part_tokens, int max_parts, RopeIn rp, GateIn gt, Bound bd) {
   __shared__ DecodeSmem<HD> sm;
   decode_segment<HD, MODE>(sm, blockIdx.x, blockIdx.y, order ? order[blockIdx.z] : blockIdx.z, q,
                            q_stride, k_cache, v_cache, block_tables, bt_stride, context_lens,
                            out, out_stride, part_o, part_ml, Hq, Hkv, scale, part_tokens,
-                           max_parts, rp, gt);
+                           max_parts, rp, gt, bd);
 }
 
 // Persistent form (one partition per sequence): a fixed grid of about the
@@ -783,14 +820,14 @@ __global__ void __launch_bounds__(256, OCC) paged_decode_persist_kernel(
     const bf16_t* __restrict__ v_cache, const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ context_lens, const int* __restrict__ order,
     bf16_t* __restrict__ out, long out_stride, int B, int Hq, int Hkv, float scale,
-    int part_tokens, RopeIn rp, GateIn gt) {
+    int part_tokens, RopeIn rp, GateIn gt, Bound bd) {
   __shared__ DecodeSmem<HD> sm;
   const int nseg = B * Hkv;
   for (int seg = blockIdx.x; seg < nseg; seg += gridDim.x) {
     const int r = seg / Hkv, kvh = seg - r * Hkv;
     decode_segment<HD, MODE>(sm, 0, kvh, order ? order[r] : r, q, q_stride, k_cache, v_cache,
                           block_tables, bt_stride, context_lens, out, out_stride, nullptr,
-                          nullptr, Hq, Hkv, scale, part_tokens, 1, rp, gt);
+                          nullptr, Hq, Hkv, scale, part_tokens, 1, rp, gt, bd);
     __syncthreads();            // the segment's LDS combine is read before the next reuses it
   }
 }
@@ -800,9 +837,10 @@ template <int HD>
 __global__ void __launch_bounds__(128) paged_decode_reduce_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     const int* __restrict__ context_lens, bf16_t* __restrict__ out, long out_stride, int Hq,
-    int part_tokens, int max_parts, GateIn gt) {
+    int part_tokens, int max_parts, GateIn gt, Bound bd) {
   const int head = blockIdx.x, b = blockIdx.y, d = threadIdx.x;
-  const int ctx = context_lens[b];
+  // the length the partitions cut (decode_segment)
+  const int ctx = context_lens[b] - first_seen(bd, context_lens[b] - 1) / BS * BS;
   part_tokens = effective_part(ctx, part_tokens, max_parts);
   const int nparts = (ctx + part_tokens - 1) / part_tokens;
   if (nparts <= 1) return;
@@ -846,9 +884,13 @@ int paged_decode(const void* q, long q_stride, const void* k_cache, const void* 
                  long out_stride, float* part_o, float* part_ml, int B, int Hq, int Hkv, int D,
                  int block_size, float scale, int part_tokens, int max_parts,
                  const int* rope_positions, const float* cos_sin, const int* slots,
-                 const void* gate, long gate_stride, int split_p, hipStream_t stream) {
+                 const void* gate, long gate_stride, int split_p, int window, float cap,
+                 hipStream_t stream) {
   if (B <= 0) return 0;
   if (split_p && cos_sin) return -6;     // the split form has no rotary variant
+  if (window < 0 || cap < 0.f || (!split_p && (window || cap > 0.f))) return -7;
+  const Bound bd{window, cap};
+  const bool bound = window || cap > 0.f;
   const GateIn gt{(const bf16_t*)gate, gate_stride};
   if (cos_sin && (!rope_positions || !slots)) return -5;
   const RopeIn rp{rope_positions, cos_sin, slots};
@@ -860,19 +902,19 @@ int paged_decode(const void* q, long q_stride, const void* k_cache, const void* 
   paged_decode_kernel<HDV, MODE><<<dim3(max_parts, Hkv, B), dim3(256), 0, stream>>>(          \
       (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, \
       bt_stride, context_lens, order, (bf16_t*)out, out_stride, part_o, part_ml, Hq, Hkv,     \
-      scale, part_tokens, max_parts, rp, gt);
+      scale, part_tokens, max_parts, rp, gt, bd);
 #define LMX_DEC_P(HDV, MODE)                                                                  \
   paged_decode_persist_kernel<HDV, MODE><<<dim3(std::min(B * Hkv, decode_resident_wgs())), dim3(256), \
                                       0, stream>>>(                                           \
       (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, \
       bt_stride, context_lens, order, (bf16_t*)out, out_stride, B, Hq, Hkv, scale, part_tokens, \
-      rp, gt);
+      rp, gt, bd);
 #define LMX_DEC_R(HDV, OCC)                                                                   \
   paged_decode_persist_kernel<HDV, 9, OCC>                                                    \
       <<<dim3(std::min(B * Hkv, decode_resident_wgs(OCC))), dim3(256), 0, stream>>>(          \
       (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, \
       bt_stride, context_lens, order, (bf16_t*)out, out_stride, B, Hq, Hkv, scale, part_tokens, \
-      rp, gt);
+      rp, gt, bd);
   // mode 0 with no more segments than CUs (a TP rank's single kv head, e.g.
   // 256 rows x 1 kv head): one workgroup per segment, the grid form -- the
   // persistent form walks one segment per workgroup there anyway and measured
@@ -881,7 +923,9 @@ int paged_decode(const void* q, long q_stride, const void* k_cache, const void* 
                    : (g_decode_mode == 0 && max_parts == 1 && B * Hkv <= decode_resident_wgs(1))
                        ? 4 : g_decode_mode;
 #define LMX_DEC(HDV)                                                                          \
-  if (mode == 16) { LMX_DEC_P(HDV, 16) }                                                      \
+  if (mode == 16 && bound) { LMX_DEC_P(HDV, 18) }                                             \
+  else if (mode == 17 && bound) { LMX_DEC_K(HDV, 18) }                                        \
+  else if (mode == 16) { LMX_DEC_P(HDV, 16) }                                                 \
   else if (mode == 17) { LMX_DEC_K(HDV, 16) }                                                 \
   else if (mode == 9 && max_parts == 1) { LMX_DEC_R(HDV, 2) }                                      \
   else if (mode == 10 && max_parts == 1) { LMX_DEC_R(HDV, 3) }                       \
@@ -897,7 +941,7 @@ int paged_decode(const void* q, long q_stride, const void* k_cache, const void* 
   else { LMX_DEC_K(HDV, 0) }                                                                  \
   if (max_parts > 1)                                                                          \
     paged_decode_reduce_kernel<HDV><<<dim3(Hq, B), dim3(HDV), 0, stream>>>(                   \
-        part_o, part_ml, context_lens, (bf16_t*)out, out_stride, Hq, part_tokens, max_parts, gt);
+        part_o, part_ml, context_lens, (bf16_t*)out, out_stride, Hq, part_tokens, max_parts, gt, bd);
   if (D == 128) { LMX_DEC(128) } else { LMX_DEC(64) }
 #undef LMX_DEC
 #undef LMX_DEC_K
@@ -998,14 +1042,17 @@ __device__ __forceinline__ void pf_vmwait() {
 // that tile latency, not by the MFMAs.
 // SPLIT: the softmax weights enter the PV product as a bf16 pair (high part +
 // remainder), i.e. with fp32 precision to within 2^-17.
-template <int HD, int NST, int PW = 4, bool SPLIT = false, int PF_NG = pf_groups<HD>()>
+// BOUND: sliding window and soft cap; the tiles start at the one that holds the
+// first key of the workgroup's first query.
+template <int HD, int NST, int PW = 4, bool SPLIT = false, bool BOUND = false,
+          int PF_NG = pf_groups<HD>()>
 __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
     const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ context_lens,
     const int* __restrict__ tiles, bf16_t* __restrict__ out, long out_stride, int Hq, int Hkv,
     float scale, int causal, float rescale_thr, int xcd, const int* __restrict__ rope_pos,
-    const float* __restrict__ rope_cs, GateIn gt) {
+    const float* __restrict__ rope_cs, GateIn gt, Bound bd) {
   extern __shared__ __attribute__((aligned(16))) char pf_smem[];
   constexpr int PAGE = BS * HD;
   // buffer b: K pages at b*4*PAGE + {0, PAGE}, V pages at b*4*PAGE + 2*PAGE + {0, PAGE}
@@ -1034,7 +1081,8 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
   const int ctx = context_lens[seq];
   const int wg_q1 = min(q_start + PW * PF_NG * QG, qlen);  // one past the WG's last query
   const int wg_lim = causal ? (ctx - qlen + wg_q1 - 1) : (ctx - 1);
-  const int ntiles = wg_lim / PF_TK + 1;
+  const int tile0 = BOUND ? first_seen(bd, ctx - qlen + q_start) / PF_TK : 0;
+  const int ntiles = wg_lim / PF_TK + 1 - tile0;
   const int last_page = (ctx - 1) / BS;
   const int* bt = block_tables + (long)seq * bt_stride;
 
@@ -1052,7 +1100,7 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
   auto stage = [&](int t, int buf) {
 #pragma unroll
     for (int pp = 0; pp < 2; ++pp) {
-      const int pg = min(2 * t + pp, last_page);
+      const int pg = min(2 * (t + tile0) + pp, last_page);
       const long blk = bt[pg];
       const bf16_t* kp = k_cache + (blk * Hkv + kvh) * PAGE;
       const bf16_t* vp = v_cache + (blk * Hkv + kvh) * PAGE;
@@ -1127,6 +1175,15 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
   wave_lo = min(wave_lo, __shfl_xor(wave_lo, 2, 64));
   wave_lo = min(wave_lo, __shfl_xor(wave_lo, 4, 64));
   wave_lo = min(wave_lo, __shfl_xor(wave_lo, 8, 64));
+  // largest one: tiles from its first visible key on need no lower mask
+  int wave_hi = -1;
+  if constexpr (BOUND) {
+#pragma unroll
+    for (int n = 0; n < PF_NG; ++n) wave_hi = max(wave_hi, lim[n]);
+#pragma unroll
+    for (int o = 1; o < 16; o <<= 1) wave_hi = max(wave_hi, __shfl_xor(wave_hi, o, 64));
+  }
+  const ScoreMap smap = score_map(scale, bd);
   const bool wave_idle = q_start + wave * PF_NG * QG >= qlen;   // wave-uniform
 
   float m[PF_NG], l[PF_NG];
@@ -1154,7 +1211,7 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
     if (wave_idle) continue;
     const bf16_t* kt = lds + buf * 4 * PAGE;
     const bf16_t* vt = kt + 2 * PAGE;
-    const int key0 = t * PF_TK;
+    const int key0 = (t + tile0) * PF_TK;
     // One 64-key tile, software-pipelined over the wave's column groups so the
     // softmax VALU of group n-1 issues between the S MFMAs of group n, and the
     // softmax of the last group between the PV MFMAs of group 0 (the MFMA and
@@ -1194,14 +1251,21 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
 #pragma unroll
         for (int kb = 0; kb < 4; ++kb)
 #pragma unroll
-          for (int h = 0; h < 2; ++h) x[2 * kb + h] = f32x2_t{s[n][kb][2 * h], s[n][kb][2 * h + 1]};
+          for (int h = 0; h < 2; ++h) {
+            if constexpr (BOUND)
+              x[2 * kb + h] = f32x2_t{map_score(smap, s[n][kb][2 * h]), map_score(smap, s[n][kb][2 * h + 1])};
+            else
+              x[2 * kb + h] = f32x2_t{s[n][kb][2 * h], s[n][kb][2 * h + 1]};
+          }
         if constexpr (MASK) {
 #pragma unroll
           for (int kb = 0; kb < 4; ++kb)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int key = key0 + kb * 16 + 4 * g + r;
-              x[2 * kb + (r >> 1)][r & 1] = key <= lim[n] ? x[2 * kb + (r >> 1)][r & 1] : -INFINITY;
+              const bool seen = key <= lim[n] &&
+                                (!BOUND || !bd.window || key > lim[n] - bd.window);
+              x[2 * kb + (r >> 1)][r & 1] = seen ? x[2 * kb + (r >> 1)][r & 1] : -INFINITY;
             }
         }
         // 16 values: a max3 tree (8 instructions, depth 3)
@@ -1210,7 +1274,8 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
         const float t4 = max3f(x[6].x, x[6].y, x[7].x);
         float mx = max3f(max3f(t0, t1, t2), max3f(t3, t4, x[7].y), -INFINITY);
         mx = col4_max(mx);
-        const float mx2 = mx * scale_log2;               // -inf stays -inf (scale > 0)
+        // -inf stays -inf (scale > 0); BOUND scores are in log2 units already
+        const float mx2 = BOUND ? mx : mx * scale_log2;
         // lazy rescale (guide T13): the running max m (log2 units) is raised
         // only when a tile's max exceeds it by more than rescale_thr; until then
         // p = 2^(x - m) <= 2^thr.  The wave rescales together (exact alpha per
@@ -1227,7 +1292,7 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
         f32x2_t rs2 = {0.f, 0.f};
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          f32x2_t y = x[j] * sc2 + nm2;
+          f32x2_t y = BOUND ? x[j] + nm2 : x[j] * sc2 + nm2;
           y.x = fast_exp2(y.x);
           y.y = fast_exp2(y.y);
           x[j] = y;
@@ -1301,7 +1366,8 @@ __global__ void __launch_bounds__(64 * PW, 8 / PW) paged_prefill_kernel(
 #pragma unroll
       for (int n = 1; n < PF_NG; ++n) pv(n);
     };
-    const bool need_mask = key0 + PF_TK - 1 > wave_lo;
+    const bool need_mask = key0 + PF_TK - 1 > wave_lo ||
+                           (BOUND && bd.window && key0 <= wave_hi - bd.window);
     if (need_mask) tile_body(std::true_type{}); else tile_body(std::false_type{});
   }
   // Epilogue: O^T through LDS, so every output row leaves as whole 16-B pieces
@@ -1373,7 +1439,11 @@ int paged_prefill(const void* q, long q_stride, const void* k_cache, const void*
                   const int* context_lens, const int* tiles, int num_tiles, void* out,
                   long out_stride, int Hq, int Hkv, int D, int block_size, float scale,
                   int causal, int q_per_tile, const int* rope_pos, const float* rope_cs,
-                  const void* gate, long gate_stride, int split_p, hipStream_t stream) {
+                  const void* gate, long gate_stride, int split_p, int window, float cap,
+                  hipStream_t stream) {
+  const Bound bd{window, cap};
+  const bool bound = window || cap > 0.f;
+  if (window < 0 || cap < 0.f || (bound && (!split_p || !causal))) return -6;
   const GateIn gt{(const bf16_t*)gate, gate_stride};
   if ((rope_pos == nullptr) != (rope_cs == nullptr)) return -4;
   if (num_tiles <= 0) return 0;
@@ -1382,20 +1452,20 @@ int paged_prefill(const void* q, long q_stride, const void* k_cache, const void*
   const int per_wave = (D == 128 ? pf_groups<128>() : pf_groups<64>()) * (16 / (Hq / Hkv));
   const int pw = q_per_tile / per_wave;
   if (q_per_tile % per_wave != 0 || (pw != 4 && pw != 8) || (pw == 8 && D != 128)) return -3;
-#define LMX_PRE(HDV, NSTV, PWV, SPL)                                                          \
+#define LMX_PRE(HDV, NSTV, PWV, ...)                                                          \
   {                                                                                           \
     constexpr int smem = NSTV * 4 * BS * HDV * 2;                                             \
     static bool attr = false;                                                                 \
     if (smem > 65536 && !attr) {                                                              \
-      (void)hipFuncSetAttribute((const void*)paged_prefill_kernel<HDV, NSTV, PWV, SPL>,       \
+      (void)hipFuncSetAttribute((const void*)paged_prefill_kernel<HDV, NSTV, PWV, __VA_ARGS__>, \
                                 hipFuncAttributeMaxDynamicSharedMemorySize, smem);            \
       attr = true;                                                                            \
     }                                                                                         \
-    paged_prefill_kernel<HDV, NSTV, PWV, SPL><<<dim3(num_tiles, Hkv), dim3(64 * PWV), smem,   \
+    paged_prefill_kernel<HDV, NSTV, PWV, __VA_ARGS__><<<dim3(num_tiles, Hkv), dim3(64 * PWV), smem,   \
                                                 stream>>>(                                         \
         (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,           \
         block_tables, bt_stride, cu_q, context_lens, tiles, (bf16_t*)out, out_stride, Hq, Hkv, \
-        scale, causal, g_prefill_rescale_thr, g_prefill_xcd, rope_pos, rope_cs, gt);              \
+        scale, causal, g_prefill_rescale_thr, g_prefill_xcd, rope_pos, rope_cs, gt, bd);          \
   }
   // 2 slots by default: 3 measured equal at D = 64 and 1.55x slower at D = 128
   // with 4-wave workgroups (96 KB of LDS leaves one workgroup per CU) --
@@ -1403,7 +1473,9 @@ int paged_prefill(const void* q, long q_stride, const void* k_cache, const void*
   const int nst = g_prefill_stages ? g_prefill_stages : 2;
   if (split_p) {
     if (pw != 4) return -5;
-    if (D == 128) LMX_PRE(128, 2, 4, true) else LMX_PRE(64, 2, 4, true)
+    if (bound) {
+      if (D == 128) LMX_PRE(128, 2, 4, true, true) else LMX_PRE(64, 2, 4, true, true)
+    } else if (D == 128) LMX_PRE(128, 2, 4, true) else LMX_PRE(64, 2, 4, true)
   } else if (D == 128) {
     if (pw == 8) {
       if (nst == 3) LMX_PRE(128, 3, 8, false) else LMX_PRE(128, 2, 8, false)
@@ -1428,7 +1500,7 @@ __global__ void __launch_bounds__(256) attention_any_kernel(
     const T* __restrict__ q, long q_stride, const T* __restrict__ kc, const T* __restrict__ vc,
     const int* __restrict__ bt, int bt_stride, const int* __restrict__ cu_q, int S,
     const int* __restrict__ positions, T* __restrict__ out, long out_stride,
-    const T* __restrict__ gate, long gate_stride, int Hq, int Hkv, float scale) {
+    const T* __restrict__ gate, long gate_stride, int Hq, int Hkv, float scale, Bound bd) {
   constexpr int D = ND * 64;
   __shared__ float sq[4][D];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -1444,12 +1516,12 @@ __global__ void __launch_bounds__(256) attention_any_kernel(
     if (cu_q[mid] <= row) lo = mid; else hi = mid - 1;
   }
   const int* tab = bt + (long)lo * bt_stride;
-  const int n = positions[row] + 1;
+  const int n = positions[row] + 1, first = first_seen(bd, n - 1);
   const long kvh = h / (Hq / Hkv);
   float m = -INFINITY, l = 0.f, acc[ND];
 #pragma unroll
   for (int i = 0; i < ND; ++i) acc[i] = 0.f;
-  for (int k0 = 0; k0 < n; k0 += 64) {
+  for (int k0 = first; k0 < n; k0 += 64) {
     const int key = k0 + lane;
     float s = -INFINITY;
     if (key < n) {
@@ -1462,6 +1534,7 @@ __global__ void __launch_bounds__(256) attention_any_kernel(
         for (int e = 0; e < 8; ++e) t += x[e] * sq[wave][d + e];
       }
       s = t * scale;
+      if (bd.cap > 0.f) s = bd.cap * tanhf(s / bd.cap);
     }
     const float mn = fmaxf(m, wave_max(s));
     const float al = expf(m - mn), p = expf(s - mn);   // exp(-inf) = 0
@@ -1491,14 +1564,16 @@ __global__ void __launch_bounds__(256) attention_any_kernel(
 int attention_any(const void* q, long q_stride, const void* kc, const void* vc, const int* bt,
                   int bt_stride, const int* cu_q, int S, const int* positions, int rows, void* out,
                   long out_stride, const void* gate, long gate_stride, int Hq, int Hkv, int D,
-                  int block_size, float scale, int is_bf16, hipStream_t stream) {
+                  int block_size, float scale, int window, float cap, int is_bf16,
+                  hipStream_t stream) {
   if (rows <= 0) return 0;
-  if (block_size != BS || S < 1 || Hq % Hkv != 0) return -1;
+  if (block_size != BS || S < 1 || Hq % Hkv != 0 || window < 0 || cap < 0.f) return -1;
+  const Bound bd{window, cap};
   const dim3 grid(rows, (Hq + 3) / 4);
 #define LMX_ANY(T, ND)                                                                           \
   attention_any_kernel<T, ND><<<grid, dim3(256), 0, stream>>>(                                   \
       (const T*)q, q_stride, (const T*)kc, (const T*)vc, bt, bt_stride, cu_q, S, positions,      \
-      (T*)out, out_stride, (const T*)gate, gate_stride, Hq, Hkv, scale)
+      (T*)out, out_stride, (const T*)gate, gate_stride, Hq, Hkv, scale, bd)
 #define LMX_ANY_D(T)                                                                             \
   if (D == 64) LMX_ANY(T, 1); else if (D == 128) LMX_ANY(T, 2); else if (D == 256) LMX_ANY(T, 4); \
   else if (D == 512) LMX_ANY(T, 8); else return -2;

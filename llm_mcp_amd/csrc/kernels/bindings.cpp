@@ -12,6 +12,8 @@
 #include <stdexcept>
 #include <string>
 
+#include "delta.h"
+
 namespace lmx {
 int rmsnorm(void*, void*, const void*, const void*, int, int, long, long, float, hipStream_t);
 int layernorm(void*, const void*, const void*, const void*, const void*, int, int, float,
@@ -28,23 +30,36 @@ void set_prefill_xcd(int);
 int paged_decode(const void*, long, const void*, const void*, const int*, int, const int*,
                  const int*, void*,
                  long, float*, float*, int, int, int, int, int, float, int, int, const int*,
-                 const float*, const int*, const void*, long, int, hipStream_t);
+                 const float*, const int*, const void*, long, int, int, float, hipStream_t);
 int paged_prefill(const void*, long, const void*, const void*, const int*, int, const int*,
                   const int*, const int*, int, void*, long, int, int, int, int, float, int, int,
-                  const int*, const float*, const void*, long, int, hipStream_t);
+                  const int*, const float*, const void*, long, int, int, float, hipStream_t);
 int attention_any(const void*, long, const void*, const void*, const int*, int, const int*, int,
                   const int*, int, void*, long, const void*, long, int, int, int, int, float, int,
-                  hipStream_t);
+                  float, int, hipStream_t);
 int sandwich_norm(void*, float*, const void*, long, int, long, const int*, const float*, int,
                   const int*, const void*, float, const float*, const float*, const long*, int, int,
                   float, int, hipStream_t);
+int sum_norm(void*, float*, const void*, long, int, long, const int*, const float*, int,
+             const void*, long, int, long, const float*, const float*, float, const float*,
+             const float*, const float*, const long*, int, int, float, int, hipStream_t);
+int soft_cap(void*, long, float, float, int, hipStream_t);
+int rotate_rows(void*, long, void*, long, const float*, int, int, int, int, int, float,
+                hipStream_t);
+int norm_rope_cache(const void*, long, const float*, const float*, const float*, int, const int*,
+                    const int*, int, void*, void*, void*, int, int, int, int, int, float, int,
+                    hipStream_t);
+int delta_recurrent(const DeltaArgs&, int, int, hipStream_t);
+int delta_chunks(const DeltaArgs&, int, int, const int*, int, const int*, void*, float*,
+                 hipStream_t);
 int gelu(void*, long, int, hipStream_t);
 int grouped(const void*, long, long, const void*, void*, long, long, int, int, int, int, const int*,
-            int, const int*, const int*, const float*, const void*, long, int, int, hipStream_t);
+            int, const int*, const int*, const float*, float, float, const void*, long, int, int,
+            hipStream_t);
 int pgemm_grouped(void*, const void*, const void*, int, int, int, long, long, int, const int*, int,
-                  const int*, const int*, const float*, hipStream_t);
-int moe_route(const void*, long, const void*, int, int, int, int, int, int*, float*, int,
-              hipStream_t);
+                  const int*, const int*, const float*, float, float, hipStream_t);
+int moe_route(const void*, long, const void*, int, int, int, int, int, int, const float*, int, int,
+              int*, float*, int, hipStream_t);
 int moe_plan(const int*, int, int, int, int, int, int*, int*, int*, int*, int*, hipStream_t);
 int rglru_chunks(const void*, const void*, long, const float*, const float*, const float*, void*,
                  float*, const int*, const int*, const int*, int, int, const void*, int, const int*,
@@ -54,7 +69,7 @@ int rglru_rows(const void*, const void*, long, const float*, const float*, const
 int rglru_scan(const void*, const void*, long, const float*, const float*, const float*, void*,
                float*, const int*, const int*, const int*, int, int, const float*, int, int,
                hipStream_t);
-int rope_angles(const int*, const double*, int, int, float*, hipStream_t);
+int rope_angles(const int*, const double*, int, int, float, float*, hipStream_t);
 int latent_prep(const void*, long, int, int, int, const float*, int, int, const float*,
                 const float*, int, const int*, void*, int, int, void*, float, int, hipStream_t);
 int latent_rotate(const void*, long, int, const float*, int, int, int, int, void*, long, int, int,
@@ -76,8 +91,9 @@ int conv_qkv_cache(const void*, long, const float*, const float*, void*, const i
                    int, int, int, int, int, float, float, float, int, hipStream_t);
 int linear_scan(const void*, long, const void*, long, const void*, long, const void*, long,
                 const float*, const float*, const float*, const float*, const float*, void*, long,
-                float*, const int*, const int*, const int*, int, int, int, int, int, int, int, int,
-                const int*, int, const int*, int, float*, float*, hipStream_t);
+                float*, const int*, const int*, const int*, int, int, int, int, int, int,
+                const float*, int, float, int, int, const int*, int, const int*, int, float*,
+                float*, hipStream_t);
 int sample(const void*, int, long, int, int, const float*, const int*, const float*,
            const uint64_t*, const int*, int*, float*, int, hipStream_t);
 int glu(void*, const void*, long, int, int, int, int, hipStream_t);
@@ -172,12 +188,13 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                            uptr ctx, uptr order, uptr out, long out_stride, uptr part_o,
                            uptr part_ml, int B, int Hq, int Hkv, int D, int BS, float scale,
                            int part_tokens, int max_parts, uptr positions, uptr cos_sin,
-                           uptr slots, uptr gate, long gate_stride, int split_p, uptr stream) {
+                           uptr slots, uptr gate, long gate_stride, int split_p, int window,
+                           float cap, uptr stream) {
     check(lmx::paged_decode(P<void>(q), q_stride, P<void>(kc), P<void>(vc), P<int>(bt), bt_stride,
                             P<int>(ctx), P<int>(order), P<void>(out), out_stride, P<float>(part_o),
                             P<float>(part_ml), B, Hq, Hkv, D, BS, scale, part_tokens, max_parts,
                             P<int>(positions), P<float>(cos_sin), P<int>(slots), P<void>(gate),
-                            gate_stride, split_p, S(stream)),
+                            gate_stride, split_p, window, cap, S(stream)),
           "paged_decode");
   });
   m.def("set_slab_norm_threads", [](int t) { lmx::set_slab_norm_threads(t); },
@@ -194,21 +211,24 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                             uptr cu_q, uptr ctx, uptr tiles, int num_tiles, uptr out,
                             long out_stride, int Hq, int Hkv, int D, int BS, float scale,
                             int causal, int q_per_tile, uptr rope_pos, uptr rope_cs, uptr gate,
-                            long gate_stride, int split_p, uptr stream) {
+                            long gate_stride, int split_p, int window, float cap,
+                            uptr stream) {
     check(lmx::paged_prefill(P<void>(q), q_stride, P<void>(kc), P<void>(vc), P<int>(bt),
                              bt_stride, P<int>(cu_q), P<int>(ctx), P<int>(tiles), num_tiles,
                              P<void>(out), out_stride, Hq, Hkv, D, BS, scale, causal, q_per_tile,
                              P<int>(rope_pos), P<float>(rope_cs), P<void>(gate), gate_stride,
-                             split_p, S(stream)),
+                             split_p, window, cap, S(stream)),
           "paged_prefill");
   });
   m.def("attention_any", [](uptr q, long q_stride, uptr kc, uptr vc, uptr bt, int bt_stride,
                             uptr cu_q, int nseq, uptr positions, int rows, uptr out,
                             long out_stride, uptr gate, long gate_stride, int Hq, int Hkv, int D,
-                            int BS, float scale, int is_bf16, uptr stream) {
+                            int BS, float scale, int window, float cap, int is_bf16,
+                            uptr stream) {
     check(lmx::attention_any(P<void>(q), q_stride, P<void>(kc), P<void>(vc), P<int>(bt), bt_stride,
                              P<int>(cu_q), nseq, P<int>(positions), rows, P<void>(out), out_stride,
-                             P<void>(gate), gate_stride, Hq, Hkv, D, BS, scale, is_bf16, S(stream)),
+                             P<void>(gate), gate_stride, Hq, Hkv, D, BS, scale, window, cap,
+                             is_bf16, S(stream)),
           "attention_any");
   });
   // ---- sandwich / gated norms (norm.hip) ----
@@ -222,29 +242,85 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                              S(stream)),
           "sandwich_norm");
   });
+  m.def("sum_norm", [](uptr out, uptr residual, uptr ya, long a_ld, int a_slabs, long a_stride,
+                       uptr mix_pos, uptr mix_w, int mix_n, uptr yb, long b_ld, int b_slabs,
+                       long b_stride, uptr wa, uptr wb, float alpha, uptr scale, uptr w_post,
+                       uptr w_pre, uptr rows_idx, int rows, int cols, float eps, int is_bf16,
+                       uptr stream) {
+    check(lmx::sum_norm(P<void>(out), P<float>(residual), P<void>(ya), a_ld, a_slabs, a_stride,
+                        P<int>(mix_pos), P<float>(mix_w), mix_n, P<void>(yb), b_ld, b_slabs,
+                        b_stride, P<float>(wa), P<float>(wb), alpha, P<float>(scale),
+                        P<float>(w_post), P<float>(w_pre), P<long>(rows_idx), rows, cols, eps,
+                        is_bf16, S(stream)),
+          "sum_norm");
+  });
+  m.def("soft_cap", [](uptr x, long n, float scale, float cap, int is_bf16, uptr stream) {
+    check(lmx::soft_cap(P<void>(x), n, scale, cap, is_bf16, S(stream)), "soft_cap");
+  });
+  m.def("rotate_rows", [](uptr q, long q_ld, uptr k, long k_ld, uptr ang, int n, int r0, int r1,
+                          int groups, int N, float k_scale, uptr stream) {
+    check(lmx::rotate_rows(P<void>(q), q_ld, P<void>(k), k_ld, P<float>(ang), n, r0, r1, groups, N,
+                           k_scale, S(stream)),
+          "rotate_rows");
+  });
+  m.def("norm_rope_cache", [](uptr p, long p_ld, uptr q_norm, uptr k_norm, uptr ang, int n,
+                              uptr slots, uptr quads, int groups, uptr q, uptr kc, uptr vc, int Hq,
+                              int Hkv, int D, int dk, int BS, float eps, int is_bf16, uptr stream) {
+    check(lmx::norm_rope_cache(P<void>(p), p_ld, P<float>(q_norm), P<float>(k_norm), P<float>(ang),
+                               n, P<int>(slots), P<int>(quads), groups, P<void>(q), P<void>(kc),
+                               P<void>(vc), Hq, Hkv, D, dk, BS, eps, is_bf16, S(stream)),
+          "norm_rope_cache");
+  });
+  // ---- K21 gated delta rule (delta.hip) ----
+  m.def("delta_recurrent", [](uptr q, long q_ld, uptr k, long k_ld, uptr v, long v_ld, uptr b,
+                              long b_ld, uptr a, long a_ld, uptr dt_bias, uptr neg_a, uptr out,
+                              long out_ld, uptr state, uptr cu_q, uptr ctx, uptr slots, int H,
+                              int G, int N, int Pd, int nseq, int is_bf16, uptr stream) {
+    const lmx::DeltaArgs d{P<void>(q), P<void>(k), P<void>(v), P<void>(b), P<void>(a), q_ld, k_ld,
+                           v_ld, b_ld, a_ld, P<float>(dt_bias), P<float>(neg_a), P<void>(out),
+                           out_ld, P<float>(state), P<int>(cu_q), P<int>(ctx), P<int>(slots), H, G,
+                           N, Pd};
+    check(lmx::delta_recurrent(d, nseq, is_bf16, S(stream)), "delta_recurrent");
+  });
+  m.def("delta_chunks", [](uptr q, long q_ld, uptr k, long k_ld, uptr v, long v_ld, uptr b,
+                           long b_ld, uptr a, long a_ld, uptr dt_bias, uptr neg_a, uptr out,
+                           long out_ld, uptr state, uptr cu_q, uptr ctx, uptr slots, int H, int G,
+                           int N, int Pd, int seq0, int nseq, uptr chunks, int nchunks, uptr first,
+                           uptr mats, uptr vecs, uptr stream) {
+    const lmx::DeltaArgs d{P<void>(q), P<void>(k), P<void>(v), P<void>(b), P<void>(a), q_ld, k_ld,
+                           v_ld, b_ld, a_ld, P<float>(dt_bias), P<float>(neg_a), P<void>(out),
+                           out_ld, P<float>(state), P<int>(cu_q), P<int>(ctx), P<int>(slots), H, G,
+                           N, Pd};
+    check(lmx::delta_chunks(d, seq0, nseq, P<int>(chunks), nchunks, P<int>(first), P<void>(mats),
+                            P<float>(vecs), S(stream)),
+          "delta_chunks");
+  });
   m.def("gelu", [](uptr x, long n, int is_bf16, uptr stream) {
     check(lmx::gelu(P<void>(x), n, is_bf16, S(stream)), "gelu");
   });
   m.def("grouped", [](uptr a, long lda, long a_gs, uptr w, uptr c, long ldc, long c_gs, int groups,
                       int N, int K, int M, uptr tiles, int mtiles, uptr off, uptr src, uptr limit,
-                      uptr gate, long gate_ld, int bm, int is_bf16, uptr stream) {
+                      float slope, float shift, uptr gate, long gate_ld, int bm, int is_bf16,
+                      uptr stream) {
     check(lmx::grouped(P<void>(a), lda, a_gs, P<void>(w), P<void>(c), ldc, c_gs, groups, N, K, M,
-                       P<int>(tiles), mtiles, P<int>(off), P<int>(src), P<float>(limit),
-                       P<void>(gate), gate_ld, bm, is_bf16, S(stream)),
+                       P<int>(tiles), mtiles, P<int>(off), P<int>(src), P<float>(limit), slope,
+                       shift, P<void>(gate), gate_ld, bm, is_bf16, S(stream)),
           "grouped");
   });
   m.def("pgemm_grouped", [](uptr c, uptr a, uptr w, int M, int N, int K, long lda, long ldc,
                             int a_rows, uptr tiles, int mtiles, uptr off, uptr src, uptr limit,
-                            uptr stream) {
+                            float slope, float shift, uptr stream) {
     check(lmx::pgemm_grouped(P<void>(c), P<void>(a), P<void>(w), M, N, K, lda, ldc, a_rows,
                              P<int>(tiles), mtiles, P<int>(off), P<int>(src), P<float>(limit),
-                             S(stream)),
+                             slope, shift, S(stream)),
           "pgemm_grouped");
   });
-  m.def("moe_route", [](uptr h, long h_ld, uptr w, int T, int d, int E, int top, int extra, uptr ids,
-                        uptr wts, int is_bf16, uptr stream) {
-    check(lmx::moe_route(P<void>(h), h_ld, P<void>(w), T, d, E, top, extra, P<int>(ids),
-                         P<float>(wts), is_bf16, S(stream)),
+  m.def("moe_route", [](uptr h, long h_ld, uptr w, int T, int d, int E, int rows, int top,
+                        int extra, uptr correction, int groups, int keep, uptr ids, uptr wts,
+                        int is_bf16, uptr stream) {
+    check(lmx::moe_route(P<void>(h), h_ld, P<void>(w), T, d, E, rows, top, extra,
+                         P<float>(correction), groups, keep, P<int>(ids), P<float>(wts), is_bf16,
+                         S(stream)),
           "moe_route");
   });
   m.def("moe_plan", [](uptr ids, int n, int J, int groups, int bm, int mtiles, uptr hist, uptr off,
@@ -278,8 +354,10 @@ PYBIND11_MODULE(_lmx_kernels, m) {
                           P<int>(slots), C, bp, P<float>(z), nseq, is_bf16, S(stream)),
           "rglru_scan");
   });
-  m.def("rope_angles", [](uptr positions, uptr freqs, int T, int n, uptr out, uptr stream) {
-    check(lmx::rope_angles(P<int>(positions), P<double>(freqs), T, n, P<float>(out), S(stream)),
+  m.def("rope_angles", [](uptr positions, uptr freqs, int T, int n, float scale, uptr out,
+                          uptr stream) {
+    check(lmx::rope_angles(P<int>(positions), P<double>(freqs), T, n, scale, P<float>(out),
+                           S(stream)),
           "rope_angles");
   });
   m.def("latent_prep", [](uptr p, long p_ld, int T, int qr, int qp, uptr q_norm, int R, int Rp,
@@ -362,14 +440,15 @@ PYBIND11_MODULE(_lmx_kernels, m) {
   m.def("linear_scan", [](uptr q, long q_ld, uptr k, long k_ld, uptr v, long v_ld, uptr dt,
                           long dt_ld, uptr dt_bias, uptr neg_a, uptr decay, uptr log_decay,
                           uptr skip, uptr out, long out_ld, uptr state, uptr cu_q, uptr ctx,
-                          uptr slots, int H, int N, int Pd, int hpg, int act, int is_bf16, int seq0,
+                          uptr slots, int H, int N, int Pd, int hpg, int act, int is_bf16,
+                          uptr ang, int nrot, float k_scale, int seq0,
                           int nseq, uptr segs, int nseg, uptr first, int one_pass, uptr ws,
                           uptr ws_log, uptr stream) {
     check(lmx::linear_scan(P<void>(q), q_ld, P<void>(k), k_ld, P<void>(v), v_ld, P<void>(dt),
                            dt_ld, P<float>(dt_bias), P<float>(neg_a), P<float>(decay),
                            P<float>(log_decay), P<float>(skip), P<void>(out), out_ld,
                            P<float>(state), P<int>(cu_q), P<int>(ctx), P<int>(slots), H, N, Pd, hpg,
-                           act, is_bf16, seq0, nseq, P<int>(segs), nseg, P<int>(first), one_pass,
+                           act, is_bf16, P<float>(ang), nrot, k_scale, seq0, nseq, P<int>(segs), nseg, P<int>(first), one_pass,
                            P<float>(ws), P<float>(ws_log), S(stream)),
           "linear_scan");
   });

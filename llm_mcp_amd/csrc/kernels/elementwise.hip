@@ -303,4 +303,32 @@ int bias_act(void* x, const void* bias, long rows, int n, int act, hipStream_t s
   return (int)hipGetLastError();
 }
 
+// x <- cap tanh(scale x / cap) in place (cap 0: scale x); the logits of models
+// that cap them.  8 elements per thread.
+template <typename T>
+__global__ void __launch_bounds__(256) soft_cap_kernel(T* __restrict__ x, long n, float scale,
+                                                       float cap) {
+  const long i = ((long)blockIdx.x * 256 + threadIdx.x) * 8;
+  const float in = cap > 0.f ? scale / cap : scale;
+  auto f = [&](float v) { return cap > 0.f ? cap * tanhf(v * in) : v * in; };
+  if (i + 8 <= n) {
+    float v[8];
+    ldv<8>(v, x + i);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = f(v[e]);
+    stv<8>(x + i, v);
+  } else {
+    for (long j = i; j < n; ++j) st1(x + j, f(ld1(x + j)));
+  }
+}
+
+int soft_cap(void* x, long n, float scale, float cap, int is_bf16, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (((uintptr_t)x & 15) || cap < 0.f) return -1;
+  const dim3 grid((unsigned)((n + 2047) / 2048));
+  if (is_bf16) soft_cap_kernel<bf16_t><<<grid, dim3(256), 0, stream>>>((bf16_t*)x, n, scale, cap);
+  else soft_cap_kernel<float><<<grid, dim3(256), 0, stream>>>((float*)x, n, scale, cap);
+  return (int)hipGetLastError();
+}
+
 }  // namespace lmx

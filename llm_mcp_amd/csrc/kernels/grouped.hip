@@ -7,7 +7,8 @@
 //   experts  rows sorted by group (moe_plan): a tile list names each tile's
 //            group and first row, src (optional) the A row of a sorted row
 // Epilogues: none; a clamped GLU over 16-column gate / up pairs
-//   g = min(gate, L), u = clamp(up, -L, L), g sigmoid(1.702 g) (u + 1);
+//   g = min(gate, L), u = clamp(up, -L, L), g sigmoid(slope g) (u + shift)
+//   (SiLU-GLU: no clamp, slope 1, shift 0);
 // or a multiplication with sigmoid(gate rows).
 //
 // bf16 weights come packed in MFMA fragment order,
@@ -38,6 +39,7 @@ struct GroupArgs {
   const int* off;         // experts: [groups + 1] first rows
   const int* src;         // experts: A row of a sorted row; null: the row itself
   const float* limit;     // GLU clamp per group; null: no GLU
+  float slope, shift;
   const void* gate;       // sigmoid gate rows (heads); null: none
   long gate_ld;
 };
@@ -59,10 +61,10 @@ __device__ __forceinline__ bool group_tile(const GroupArgs& p, int mt, int gz, i
 }
 
 template <typename T>
-__device__ __forceinline__ float clamped_glu(float g, float u, float lim) {
+__device__ __forceinline__ float clamped_glu(const GroupArgs& p, float g, float u, float lim) {
   g = fminf(g, lim);
   u = fminf(fmaxf(u, -lim), lim);
-  return g * sigmoid_t<T>(1.702f * g) * (u + 1.f);
+  return g * sigmoid_t<T>(p.slope * g) * (u + p.shift);
 }
 
 // 4 consecutive columns n.. of row `row`
@@ -79,10 +81,10 @@ __device__ __forceinline__ void group_store(const GroupArgs& p, int g, long row,
   *reinterpret_cast<bf16x4_t*>((bf16_t*)p.c + row * p.ldc + (long)g * p.c_gs + n) = o;
 }
 
-__device__ __forceinline__ f32x4_t glu4(f32x4_t g, f32x4_t u, float lim) {
+__device__ __forceinline__ f32x4_t glu4(const GroupArgs& p, f32x4_t g, f32x4_t u, float lim) {
   f32x4_t o;
 #pragma unroll
-  for (int r = 0; r < 4; ++r) o[r] = clamped_glu<bf16_t>(g[r], u[r], lim);
+  for (int r = 0; r < 4; ++r) o[r] = clamped_glu<bf16_t>(p, g[r], u[r], lim);
   return o;
 }
 
@@ -175,7 +177,7 @@ __global__ void __launch_bounds__(256) grouped_small_kernel(GroupArgs p) {
 #pragma unroll
     for (int i = 0; i < MT; ++i) {
       const int row = r0 + 16 * i + c;
-      const f32x4_t o = glu4(acc[i], ex[((wave >> 1) * MT + i) * 64 + lane], lim);
+      const f32x4_t o = glu4(p, acc[i], ex[((wave >> 1) * MT + i) * 64 + lane], lim);
       if (row < r1) group_store(p, g, row, nt / 2 * 16 + 4 * q, o);
     }
     return;
@@ -267,7 +269,7 @@ __global__ void __launch_bounds__(256, 2) grouped_large_kernel(GroupArgs p, int 
 #pragma unroll
       for (int j = 0; j < 4; j += 2) {
         const int t = ntl * 8 + wn * 4 + j;
-        if (t < n16) group_store(p, g, row, t / 2 * 16 + 4 * q, glu4(acc[i][j], acc[i][j + 1], lim));
+        if (t < n16) group_store(p, g, row, t / 2 * 16 + 4 * q, glu4(p, acc[i][j], acc[i][j + 1], lim));
       }
     } else {
 #pragma unroll
@@ -314,7 +316,7 @@ __global__ void __launch_bounds__(256) grouped_f32_kernel(GroupArgs p) {
     if (row >= r1) continue;
     float* cr = (float*)p.c + row * p.ldc + (long)g * p.c_gs;
     if (p.limit) {                     // columns n0.. are 16 gate, 16 up
-      if (n0 + 16 + tx < p.N) cr[n0 / 2 + tx] = clamped_glu<float>(acc[i][0], acc[i][1], p.limit[g]);
+      if (n0 + 16 + tx < p.N) cr[n0 / 2 + tx] = clamped_glu<float>(p, acc[i][0], acc[i][1], p.limit[g]);
       continue;
     }
 #pragma unroll
@@ -334,11 +336,12 @@ __global__ void __launch_bounds__(256) grouped_f32_kernel(GroupArgs p) {
 // the tile list's length)
 int grouped(const void* a, long lda, long a_gs, const void* w, void* c, long ldc, long c_gs,
             int groups, int N, int K, int M, const int* tiles, int mtiles, const int* off,
-            const int* src, const float* limit, const void* gate, long gate_ld, int bm,
-            int is_bf16, hipStream_t stream) {
+            const int* src, const float* limit, float slope, float shift, const void* gate,
+            long gate_ld, int bm, int is_bf16, hipStream_t stream) {
   if (M <= 0 || mtiles <= 0) return 0;
   if (groups < 1 || N < 1 || K < 1 || (tiles && (!off || gate)) || (limit && N % 32)) return -1;
-  const GroupArgs p{a, lda, a_gs, w, c, ldc, c_gs, N, K, M, tiles, off, src, limit, gate, gate_ld};
+  const GroupArgs p{a, lda, a_gs, w, c, ldc, c_gs, N, K, M, tiles, off, src, limit, slope, shift,
+                    gate, gate_ld};
   const int gz = tiles ? 1 : groups;
   if (!is_bf16) {
     if (bm != 32) return -2;

@@ -2,7 +2,7 @@
 // LatentAttentionMixer).  A token's cache page row is [latent c (Rp) | rotated
 // key part (xp)], one row for all heads.
 //
-//   rope_angles    cos | sin of the step's positions (reduced in double)
+//   rope_angles    cos | sin of the step's positions (reduced in double), scaled
 //   latent_prep    projection rows -> RMS-normed query latents; normed c and
 //                  the rotated key part into the pages
 //   latent_rotate  the rotated part of the queries that score latents
@@ -21,15 +21,16 @@ constexpr float LOG2E = 1.4426950408889634f;
 
 __global__ void __launch_bounds__(256) rope_angles_kernel(const int* __restrict__ positions,
                                                           const double* __restrict__ freqs, int T,
-                                                          int n, float* __restrict__ out) {
+                                                          int n, float scale,
+                                                          float* __restrict__ out) {
   const int e = blockIdx.x * 256 + threadIdx.x;
   if (e >= T * n) return;
   const int t = e / n, i = e - t * n;
   // the angle modulo one turn in double, then single precision
   const double turns = (double)positions[t] * freqs[i] * 0.15915494309189535;
   const float a = (float)((turns - floor(turns)) * 6.283185307179586);
-  out[(long)t * 2 * n + i] = cosf(a);
-  out[(long)t * 2 * n + n + i] = sinf(a);
+  out[(long)t * 2 * n + i] = scale * cosf(a);
+  out[(long)t * 2 * n + n + i] = scale * sinf(a);
 }
 
 // grid rows, block 256: waves 0-2 the query latent, wave 3 the cache row.
@@ -746,10 +747,11 @@ __global__ void __launch_bounds__(256, 2) latent_prefill_kernel(LatentPre p) {
 
 }  // namespace
 
-int rope_angles(const int* positions, const double* freqs, int T, int n, float* out,
+int rope_angles(const int* positions, const double* freqs, int T, int n, float scale, float* out,
                 hipStream_t stream) {
   if (T <= 0 || n <= 0) return 0;
-  rope_angles_kernel<<<dim3((T * n + 255) / 256), dim3(256), 0, stream>>>(positions, freqs, T, n, out);
+  rope_angles_kernel<<<dim3((T * n + 255) / 256), dim3(256), 0, stream>>>(positions, freqs, T, n, scale,
+                                                                     out);
   return (int)hipGetLastError();
 }
 

@@ -8,7 +8,10 @@
 //   * linear attention with a constant decay per head (a_t = decay[h], s_t = 1,
 //     SiLU applied to q, k and v as they are loaded), and
 //   * the state-space form: s_t = softplus(dt_t + dt_bias), a_t = exp(-exp(A_log)
-//     s_t), D the skip weight.
+//     s_t), D the skip weight;
+//   * retention: linear attention whose q and k are rotated by their position
+//     (neighbouring channels a pair) and k scaled: the recurrent form turns them
+//     as it loads them, the chunked one runs on rows turned in place before.
 // The state of a sequence lives in its slot of state[slots][H][N][P] between
 // steps; a row range that starts at position 0 starts from the zero state
 // whatever the slot holds, so slots are reused uncleared.
@@ -27,7 +30,7 @@
 // them, pass 2 runs every segment from its true start state.
 #include <algorithm>
 
-#include "common.h"
+#include "scan.h"
 
 namespace lmx {
 
@@ -38,8 +41,6 @@ template <> __device__ __forceinline__ float silu_as<float>(float x) { return x 
 template <> __device__ __forceinline__ float silu_as<bf16_t>(float x) {
   return bf2f(f2bf(x / (1.f + __expf(-x))));
 }
-
-__device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
 struct ScanArgs {
   const void *q, *k, *v;     // T rows, first head's channels
@@ -54,6 +55,9 @@ struct ScanArgs {
   float* state;              // [slots][H][N][P]
   const int *cu_q, *ctx, *slots;
   int H, N, P, hpg, act;     // act: SiLU on q, k, v
+  const float* ang;          // [rows][nrot] cos | sin (recurrent form), or null
+  int nrot;
+  float k_scale;
 };
 
 // ------------------------------------------------------------- recurrent ----
@@ -103,7 +107,13 @@ __global__ void __launch_bounds__(256) scan_recurrent_kernel(ScanArgs a, int seq
     for (int i = threadIdx.x; i < N; i += 256) {
       const float qv = ld1(q + t * a.q_ld + i), kv = ld1(k + t * a.k_ld + i);
       sq[i] = a.act ? silu_as<T>(qv) : qv;
-      sk[i] = a.act ? silu_as<T>(kv) : kv;
+      sk[i] = (a.act ? silu_as<T>(kv) : kv) * a.k_scale;
+      if (i < a.nrot) {
+        const float* an = a.ang + (long)(row0 + t) * a.nrot + (i >> 1);
+        const float cs = an[0], sn = i & 1 ? an[a.nrot >> 1] : -an[a.nrot >> 1];
+        sq[i] = qv * cs + ld1(q + t * a.q_ld + (i ^ 1)) * sn;
+        sk[i] = (kv * cs + ld1(k + t * a.k_ld + (i ^ 1)) * sn) * a.k_scale;
+      }
     }
     for (int i = threadIdx.x; i < pt; i += 256) {
       const float vv = p0 + i < P ? ld1(v + t * a.v_ld + p0 + i) : 0.f;
@@ -160,20 +170,6 @@ __global__ void __launch_bounds__(256) scan_recurrent_kernel(ScanArgs a, int seq
   }
 }
 
-// columns per workgroup: the largest power of two up to `want_pt` whose rows
-// per thread fit the register tile (16 x 4 or 8 x 1 values)
-static bool recurrent_shape(int N, int P, int want_pt, int* vec, int* pt, int* rpt) {
-  *vec = P % 4 == 0 ? 4 : 1;
-  int t = 16;
-  while (t < P && t < want_pt) t *= 2;
-  for (;; t /= 2) {
-    const int ncol = t / *vec;
-    if (ncol < 1 || t < 4) return false;
-    const int kr = 256 / ncol, r = (N + kr - 1) / kr;
-    if (r <= (*vec == 4 ? 16 : 8)) { *pt = t; *rpt = r; return true; }
-  }
-}
-
 int scan_recurrent(const ScanArgs& a, int is_bf16, int seq0, int nseq, hipStream_t stream) {
   if (nseq <= 0) return 0;
   if (a.N <= 0 || a.P <= 0 || a.H <= 0 || a.hpg <= 0 || (a.dt == nullptr) == (a.decay == nullptr))
@@ -208,22 +204,11 @@ int scan_recurrent(const ScanArgs& a, int is_bf16, int seq0, int nseq, hipStream
 // --------------------------------------------------------------- chunked ----
 constexpr int SC = 64;     // tokens per chunk
 constexpr int SCP = 72;    // padded row of the score images (16-B aligned)
-constexpr float SCAN_LOG2E = 1.4426950408889634f;
-
 struct SegArgs {
   const int* segs;         // [nseg][4]: sequence, first row, last row (in the sequence), last-of-sequence
   float* ws;               // [nseg][H][N][P] segment states (modes 1, 2)
   float* ws_log;           // [nseg][H] log2 of the segment's total decay (mode 1)
 };
-
-typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
-typedef uint32_t u32x2_t __attribute__((ext_vector_type(2)));
-
-// (a, b) as packed bf16 pairs: hi + lo = the values to within 2^-17
-__device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
-  hi = pack_bf16x2(a, b);
-  lo = pack_bf16x2(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
-}
 
 __device__ __forceinline__ float silu_fast(float x) {
   return x * __builtin_amdgcn_rcpf(1.f + fast_exp2(-x * SCAN_LOG2E));
@@ -234,22 +219,6 @@ __device__ __forceinline__ void silu_words(u32x4_t& w) {
   for (int m = 0; m < 4; ++m)
     w[m] = pack_bf16x2(silu_fast(__uint_as_float(w[m] << 16)),
                        silu_fast(__uint_as_float(w[m] & 0xffff0000u)));
-}
-
-// Transposed LDS image [rows][64 tokens]: 16-B pieces (8 tokens) of a row are
-// XOR-permuted by the row so that both the 8-B transposing stores (16 row
-// groups x 4 token quads per wave) and the 16-B fragment reads (16 rows x 4
-// pieces) spread evenly over the banks.
-__device__ __forceinline__ int tr_swz(int row) {
-  return ((row & 3) | ((row >> 1) & 4)) ^ ((row >> 4) & 7);
-}
-
-// Barrier over LDS only: __syncthreads would also wait for every global load
-// in flight, i.e. for the next chunk's rows.
-__device__ __forceinline__ void lds_barrier() {
-  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-  __builtin_amdgcn_s_barrier();
-  asm volatile("" ::: "memory");
 }
 
 // NK: N / 32 rounded up; NV: 16-column tiles per wave (a workgroup covers 64
@@ -702,15 +671,74 @@ int scan_chunked(const ScanArgs& a, const int* segs, int nseg, const int* first,
 #undef LMX_CHUNK
 }
 
+// Rows r0..r1 - 1 of q and k (bf16, `groups` heads of N channels), in place: the
+// first n channels of a head turned by the row's angles, k times k_scale.  A
+// thread owns 8 channels of up to RH heads.  grid (ceil(rows N / 8 / 256),
+// ceil(groups / RH), 2: q, k)
+constexpr int RH = 8;
+__global__ void __launch_bounds__(256) rotate_rows_kernel(bf16_t* q, long q_ld, bf16_t* k, long k_ld,
+                                                          const float* __restrict__ ang, int n,
+                                                          int r0, int rows, int groups, int N,
+                                                          float k_scale) {
+  const int np = N / 8;
+  const long e0 = (long)blockIdx.x * 256 + threadIdx.x;
+  if (e0 >= (long)rows * np) return;
+  const long row = r0 + e0 / np;
+  const int c0 = 8 * (int)(e0 % np);
+  const bool isk = blockIdx.z != 0;
+  const float sc = isk ? k_scale : 1.f;
+  if (c0 >= n && sc == 1.f) return;
+  bf16_t* base = (isk ? k + row * k_ld : q + row * q_ld) + c0;
+  const int h0 = blockIdx.y * RH, h1 = min(h0 + RH, groups);
+  float x[RH][8];
+#pragma unroll
+  for (int i = 0; i < RH; ++i)
+    if (h0 + i < h1) ldv<8>(x[i], base + (long)(h0 + i) * N);
+  float cs[4], sn[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const bool on = c0 + 2 * e < n;
+    const float* a = ang + row * n + (c0 >> 1) + e;
+    cs[e] = on ? a[0] * sc : sc;
+    sn[e] = on ? a[n >> 1] * sc : 0.f;
+  }
+#pragma unroll
+  for (int i = 0; i < RH; ++i) {
+    if (h0 + i >= h1) continue;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float u = x[i][2 * e], v = x[i][2 * e + 1];
+      x[i][2 * e] = u * cs[e] - v * sn[e];
+      x[i][2 * e + 1] = v * cs[e] + u * sn[e];
+    }
+    stv<8>(base + (long)(h0 + i) * N, x[i]);
+  }
+}
+
+int rotate_rows(void* q, long q_ld, void* k, long k_ld, const float* ang, int n, int r0, int r1,
+                int groups, int N, float k_scale, hipStream_t stream) {
+  if (r1 <= r0) return 0;
+  if (groups < 1 || N < 8 || N % 8 || n < 0 || n % 2 || n > N || (n && !ang) || q_ld % 8 ||
+      k_ld % 8 || (((uintptr_t)q | (uintptr_t)k) & 15))
+    return -1;
+  const long pieces = (long)(r1 - r0) * (N / 8);
+  rotate_rows_kernel<<<dim3((unsigned)((pieces + 255) / 256), (groups + RH - 1) / RH, 2), dim3(256), 0,
+                       stream>>>((bf16_t*)q, q_ld, (bf16_t*)k, k_ld, ang, n, r0, r1 - r0, groups, N,
+                                 k_scale);
+  return (int)hipGetLastError();
+}
+
 int linear_scan(const void* q, long q_ld, const void* k, long k_ld, const void* v, long v_ld,
                 const void* dt, long dt_ld, const float* dt_bias, const float* neg_a,
                 const float* decay, const float* log_decay, const float* skip, void* out,
                 long out_ld, float* state, const int* cu_q, const int* ctx, const int* slots, int H,
-                int N, int P, int hpg, int act, int is_bf16, int seq0, int nseq, const int* segs,
+                int N, int P, int hpg, int act, int is_bf16, const float* ang, int nrot,
+                float k_scale, int seq0, int nseq, const int* segs,
                 int nseg, const int* first, int one_pass, float* ws, float* ws_log,
                 hipStream_t stream) {
   ScanArgs a{q, k, v, q_ld, k_ld, v_ld, dt, dt_ld, dt_bias, neg_a, decay, log_decay, skip,
-             out, out_ld, state, cu_q, ctx, slots, H, N, P, hpg, act};
+             out, out_ld, state, cu_q, ctx, slots, H, N, P, hpg, act, ang, nrot, k_scale};
+  if (nrot < 0 || nrot % 2 || nrot > N || (nrot && (!ang || act))) return -5;
   if (nseg > 0) {
     if (!is_bf16) return -4;
     return scan_chunked(a, segs, nseg, first, seq0, nseq, one_pass, ws, ws_log, stream);

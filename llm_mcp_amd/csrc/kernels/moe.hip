@@ -2,7 +2,10 @@
 //
 //   moe_route  router logits in fp32, the top experts of every row (lowest
 //              index first among equals) and the softmax over just those; then
-//              `extra` further experts every row uses with weight 1.
+//              `extra` further experts every row uses with weight 1.  Or by
+//              scores s = sigmoid(logit): the top s + correction among the best
+//              groups of neighbouring experts, in the proportions of their s;
+//              the extra ones then weigh sigmoid of one more logit.
 //              bf16 rows, up to 128 experts: 16 rows per workgroup on MFMA, the K
 //              range split over the waves; otherwise one row per workgroup on the VALU.
 //   moe_plan   the uses (row, expert) sorted by expert: expert row ranges, the
@@ -15,13 +18,55 @@ namespace {
 
 constexpr int MAXE = 256, MAXTOP = 32;
 
+struct RouteBy {
+  const float* correction;   // [E]: sigmoid scores; null: softmax over the top logits
+  int groups, keep;
+  int rows;                  // router rows: E, or E + 1 with the extra experts' logit
+};
+
 // One wave ranks one row's logits z[E] (LDS) and writes its uses.
-__device__ __forceinline__ void moe_select(const float* z, int E, int top, int extra, int* ids,
-                                           float* wts) {
+__device__ __forceinline__ void moe_select(float* z, int E, int top, int extra, const RouteBy& by,
+                                           int* ids, float* wts) {
   const int lane = threadIdx.x & 63;
   float v[MAXE / 64];
+  float more = 1.f;          // weight of the extra experts
+  if (by.correction) {
+    // z becomes the scores, v the choice scores of the kept groups
+    if (by.rows > E) more = 1.f / (1.f + expf(-z[E]));
 #pragma unroll
-  for (int i = 0; i < MAXE / 64; ++i) v[i] = i * 64 + lane < E ? z[i * 64 + lane] : -INFINITY;
+    for (int i = 0; i < MAXE / 64; ++i) {
+      const int e = i * 64 + lane;
+      v[i] = -INFINITY;
+      if (e < E) {
+        const float s = 1.f / (1.f + expf(-z[e]));
+        z[e] = s;
+        v[i] = s + by.correction[e];
+      }
+    }
+    __builtin_amdgcn_wave_barrier();
+    const int size = E / by.groups;
+    float a = -INFINITY, b = -INFINITY;       // the two largest of lane's group
+    if (lane < by.groups)
+      for (int e = lane * size; e < (lane + 1) * size; ++e) {
+        const float c = z[e] + by.correction[e];
+        if (c > a) { b = a; a = c; } else if (c > b) { b = c; }
+      }
+    const float score = lane < by.groups ? a + (size > 1 ? b : 0.f) : -INFINITY;
+    int rank = 0;
+    for (int g = 0; g < by.groups; ++g) {
+      const float o = __shfl(score, g, 64);
+      rank += o > score || (o == score && g < lane);
+    }
+    const unsigned long long kept = __ballot(lane < by.groups && rank < by.keep);
+#pragma unroll
+    for (int i = 0; i < MAXE / 64; ++i) {
+      const int e = i * 64 + lane;
+      if (e < E && !(kept >> (e / size) & 1)) v[i] = -INFINITY;
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < MAXE / 64; ++i) v[i] = i * 64 + lane < E ? z[i * 64 + lane] : -INFINITY;
+  }
   float first = 0.f, mine = 0.f, sum = 0.f;
   int id = 0;
   for (int j = 0; j < top; ++j) {
@@ -42,16 +87,16 @@ __device__ __forceinline__ void moe_select(const float* z, int E, int top, int e
     for (int i = 0; i < MAXE / 64; ++i)
       if (i * 64 + lane == at) v[i] = -INFINITY;
     if (j == 0) first = best;
-    const float w = expf(best - first);
+    const float w = by.correction ? z[at] : expf(best - first);
     sum += w;
     if (lane == j) { mine = w; id = at; }
   }
   if (lane < top) {
     ids[lane] = id;
-    wts[lane] = mine / sum;
+    wts[lane] = mine / (by.correction ? sum + 1e-20f : sum);
   } else if (lane < top + extra) {
     ids[lane] = E + lane - top;
-    wts[lane] = 1.f;
+    wts[lane] = more;
   }
 }
 
@@ -59,14 +104,14 @@ __device__ __forceinline__ void moe_select(const float* z, int E, int top, int e
 template <int NT, int NW>
 __global__ void __launch_bounds__(64 * NW) moe_route_mfma_kernel(
     const bf16_t* __restrict__ h, long h_ld, const bf16_t* __restrict__ w, int T, int d, int E,
-    int top, int extra, int* __restrict__ ids, float* __restrict__ wts) {
+    int top, int extra, RouteBy by, int* __restrict__ ids, float* __restrict__ wts) {
   __shared__ float part[NW][16][NT * 16 + 1];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, q = lane >> 4;
   const int t0 = blockIdx.x * 16;
   const bf16_t* hr = h + (long)min(t0 + c, T - 1) * h_ld + 8 * q;
   const bf16_t* wr[NT];
 #pragma unroll
-  for (int i = 0; i < NT; ++i) wr[i] = w + (long)min(16 * i + c, E - 1) * d + 8 * q;
+  for (int i = 0; i < NT; ++i) wr[i] = w + (long)min(16 * i + c, by.rows - 1) * d + 8 * q;
   f32x4_t acc[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -110,7 +155,7 @@ __global__ void __launch_bounds__(64 * NW) moe_route_mfma_kernel(
   __syncthreads();
   for (int t = wave; t < 16; t += NW)
     if (t0 + t < T)
-      moe_select(part[0][t], E, top, extra, ids + (long)(t0 + t) * (top + extra),
+      moe_select(part[0][t], E, top, extra, by, ids + (long)(t0 + t) * (top + extra),
                  wts + (long)(t0 + t) * (top + extra));
 }
 
@@ -118,20 +163,21 @@ __global__ void __launch_bounds__(64 * NW) moe_route_mfma_kernel(
 template <typename T_>
 __global__ void __launch_bounds__(256) moe_route_any_kernel(const T_* __restrict__ h, long h_ld,
                                                             const T_* __restrict__ w, int d, int E,
-                                                            int top, int extra,
+                                                            int top, int extra, RouteBy by,
                                                             int* __restrict__ ids,
                                                             float* __restrict__ wts) {
   __shared__ float z[MAXE];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const long t = blockIdx.x;
-  for (int e = wave; e < E; e += 4) {
+  for (int e = wave; e < by.rows; e += 4) {
     float s = 0.f;
     for (int k = lane; k < d; k += 64) s += ld1(h + t * h_ld + k) * ld1(w + (long)e * d + k);
     s = wave_sum(s);
     if (lane == 0) z[e] = s;
   }
   __syncthreads();
-  if (wave == 0) moe_select(z, E, top, extra, ids + t * (top + extra), wts + t * (top + extra));
+  if (wave == 0)
+    moe_select(z, E, top, extra, by, ids + t * (top + extra), wts + t * (top + extra));
 }
 
 constexpr int CHUNK = 1024;      // uses per block of the sort (ops MOE_CHUNK)
@@ -237,25 +283,31 @@ __global__ void __launch_bounds__(256) moe_scatter_kernel(PlanArgs p) {
 
 }  // namespace
 
-int moe_route(const void* h, long h_ld, const void* w, int T, int d, int E, int top, int extra,
-              int* ids, float* wts, int is_bf16, hipStream_t stream) {
+int moe_route(const void* h, long h_ld, const void* w, int T, int d, int E, int rows, int top,
+              int extra, const float* correction, int groups, int keep, int* ids, float* wts,
+              int is_bf16, hipStream_t stream) {
   if (T <= 0) return 0;
+  if (rows < E || rows > E + 1 || rows > MAXE || (rows > E && !correction) ||
+      (correction && (groups < 1 || groups > 64 || E % groups || keep < 1 || keep > groups ||
+                      keep * (E / groups) < top)))
+    return -1;
+  const RouteBy by{correction, groups, keep, rows};
   if (E < 1 || E > MAXE || top < 1 || top > E || extra < 0 || top + extra > MAXTOP || d < 1)
     return -1;
-  if (is_bf16 && E <= 128 && d % 8 == 0 && h_ld % 8 == 0 && !(((uintptr_t)h | (uintptr_t)w) & 15)) {
-    const int nt = (E + 15) / 16;
+  if (is_bf16 && rows <= 128 && d % 8 == 0 && h_ld % 8 == 0 && !(((uintptr_t)h | (uintptr_t)w) & 15)) {
+    const int nt = (rows + 15) / 16;
 #define LMX_RT(NT, NW)                                                                       \
   moe_route_mfma_kernel<NT, NW><<<dim3((T + 15) / 16), dim3(64 * NW), 0, stream>>>(          \
-      (const bf16_t*)h, h_ld, (const bf16_t*)w, T, d, E, top, extra, ids, wts)
+      (const bf16_t*)h, h_ld, (const bf16_t*)w, T, d, E, top, extra, by, ids, wts)
     if (nt == 1) LMX_RT(1, 16); else if (nt == 2) LMX_RT(2, 16); else if (nt <= 4) LMX_RT(4, 8);
     else LMX_RT(8, 4);
 #undef LMX_RT
   } else if (is_bf16) {
     moe_route_any_kernel<bf16_t><<<dim3(T), dim3(256), 0, stream>>>(
-        (const bf16_t*)h, h_ld, (const bf16_t*)w, d, E, top, extra, ids, wts);
+        (const bf16_t*)h, h_ld, (const bf16_t*)w, d, E, top, extra, by, ids, wts);
   } else {
     moe_route_any_kernel<float><<<dim3(T), dim3(256), 0, stream>>>(
-        (const float*)h, h_ld, (const float*)w, d, E, top, extra, ids, wts);
+        (const float*)h, h_ld, (const float*)w, d, E, top, extra, by, ids, wts);
   }
   return (int)hipGetLastError();
 }

@@ -502,16 +502,178 @@ int sandwich_norm(void* out, float* residual, const void* y, long y_ld, int slab
   return (int)hipGetLastError();
 }
 
+// Norm of the sum: a decoder whose residual stream (fp32) is the layer norm of
+// what is added up.
+//
+//   r   = ln(alpha residual[row] + scale y[row]) * w_post    (residual[row] without y)
+//   out = w_pre ? ln(r) * w_pre : r
+//
+// ln(x) = (x - mean) / sqrt(mean((x - mean)^2) + eps).  y is T rows, split-K
+// slabs, a mixture of expert rows (all as in the sandwich norm), or two such
+// branches, each divided by its root mean square, with a gain each.  rows_idx:
+// as in the sandwich norm.
+struct SubRows {
+  const void* y;
+  long ld, slab_stride;
+  int slabs;                  // 0: T rows
+};
+
+template <typename T, int V>
+__device__ __forceinline__ void load_sub(float (&f)[V], const SubRows& s, long row, int cols, int c0) {
+  if (s.slabs) {
+    const float* p = (const float*)s.y + row * cols + c0;
+    ldv<V>(f, p);
+    for (int i = 1; i < s.slabs; ++i) {
+      float t[V];
+      ldv<V>(t, p + i * s.slab_stride);
+#pragma unroll
+      for (int e = 0; e < V; ++e) f[e] += t[e];
+    }
+  } else {
+    ldv<V>(f, (const T*)s.y + row * s.ld + c0);
+  }
+}
+
+struct SumNormArgs {
+  void* out;
+  float* residual;
+  SubRows a, b;               // b.y: the second branch, or null
+  const int* mix_pos;         // [rows][mix_n] or null: a is expert rows
+  const float* mix_w;
+  int mix_n;
+  const float *wa, *wb;       // gains of the branches
+  float alpha;
+  const float *scale, *w_post, *w_pre;
+  const long* rows_idx;
+  int cols;
+  float eps;
+};
+
+template <typename T, int V, int VPT>
+__global__ void __launch_bounds__(512) sum_norm_kernel(SumNormArgs a) {
+  __shared__ float scratch[16];
+  const long src = a.rows_idx ? a.rows_idx[blockIdx.x] : blockIdx.x;
+  const int cols = a.cols, nchunk = cols / V;
+  float* rr = a.residual + src * cols;
+  float r[VPT][V];
+  auto chunks = [&](auto&& body) {
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c < nchunk) body(i, c * V);
+    }
+  };
+  auto ln = [&](const float* __restrict__ gain) {
+    float s = 0.f, q = 0.f;
+    chunks([&](int i, int) {
+#pragma unroll
+      for (int e = 0; e < V; ++e) s += r[i][e];
+    });
+    const float mean = block_sum(s, scratch) / (float)cols;
+    chunks([&](int i, int) {
+#pragma unroll
+      for (int e = 0; e < V; ++e) { r[i][e] -= mean; q += r[i][e] * r[i][e]; }
+    });
+    const float inv = rsqrtf(block_sum(q, scratch) / (float)cols + a.eps);
+    chunks([&](int i, int c0) {
+      float w[V];
+      ldv<V>(w, gain + c0);
+#pragma unroll
+      for (int e = 0; e < V; ++e) r[i][e] *= inv * w[e];
+    });
+  };
+  chunks([&](int i, int c0) { ldv<V>(r[i], rr + c0); });
+  if (a.a.y) {
+    float y[VPT][V];
+    if (a.mix_pos) {
+      chunks([&](int i, int c0) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[i][e] = 0.f;
+#pragma unroll 4
+        for (int j = 0; j < a.mix_n; ++j) {
+          float t[V];
+          ldv<V>(t, (const T*)a.a.y + (long)a.mix_pos[src * a.mix_n + j] * a.a.ld + c0);
+          const float w = a.mix_w[src * a.mix_n + j];
+#pragma unroll
+          for (int e = 0; e < V; ++e) y[i][e] += w * t[e];
+        }
+      });
+    } else {
+      chunks([&](int i, int c0) { load_sub<T, V>(y[i], a.a, src, cols, c0); });
+      if (a.b.y) {
+        float z[VPT][V], sa = 0.f, sb = 0.f;
+        chunks([&](int i, int c0) {
+          load_sub<T, V>(z[i], a.b, src, cols, c0);
+#pragma unroll
+          for (int e = 0; e < V; ++e) { sa += y[i][e] * y[i][e]; sb += z[i][e] * z[i][e]; }
+        });
+        const float ia = rsqrtf(block_sum(sa, scratch) / (float)cols + a.eps);
+        const float ib = rsqrtf(block_sum(sb, scratch) / (float)cols + a.eps);
+        chunks([&](int i, int c0) {
+          float wa[V], wb[V];
+          ldv<V>(wa, a.wa + c0);
+          ldv<V>(wb, a.wb + c0);
+#pragma unroll
+          for (int e = 0; e < V; ++e) y[i][e] = y[i][e] * ia * wa[e] + z[i][e] * ib * wb[e];
+        });
+      }
+    }
+    chunks([&](int i, int c0) {
+      float s[V];
+      ldv<V>(s, a.scale + c0);
+#pragma unroll
+      for (int e = 0; e < V; ++e) r[i][e] = a.alpha * r[i][e] + s[e] * y[i][e];
+    });
+    ln(a.w_post);
+    if (!a.rows_idx) chunks([&](int i, int c0) { stv<V>(rr + c0, r[i]); });
+  }
+  if (a.w_pre) ln(a.w_pre);
+  chunks([&](int i, int c0) { stv<V>((T*)a.out + (long)blockIdx.x * cols + c0, r[i]); });
+}
+
+int sum_norm(void* out, float* residual, const void* ya, long a_ld, int a_slabs, long a_stride,
+             const int* mix_pos, const float* mix_w, int mix_n, const void* yb, long b_ld,
+             int b_slabs, long b_stride, const float* wa, const float* wb, float alpha,
+             const float* scale, const float* w_post, const float* w_pre, const long* rows_idx,
+             int rows, int cols, float eps, int is_bf16, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (cols <= 0 || !residual || !out || (ya && (!w_post || !scale)) || (!ya && !w_pre) ||
+      (mix_pos && (!ya || !mix_w || a_slabs || yb)) || (yb && (!ya || !wa || !wb)))
+    return -1;
+  const SumNormArgs a{out, residual, {ya, a_ld, a_stride, a_slabs}, {yb, b_ld, b_stride, b_slabs},
+                      mix_pos, mix_w, mix_n, wa, wb, alpha, scale, w_post, w_pre, rows_idx, cols, eps};
+  const bool vec = cols % 8 == 0 && a_ld % 8 == 0 && b_ld % 8 == 0 &&
+                   (((uintptr_t)ya | (uintptr_t)yb) & 15) == 0;
+  const int nchunk = vec ? cols / 8 : cols;
+  const int vpt = (nchunk + 511) / 512;
+  if (vpt > (vec ? 4 : 8)) return -2;
+  const int threads = nchunk >= 512 ? 512 : (nchunk + 63) / 64 * 64;
+#define LMX_SN(T, V, P) sum_norm_kernel<T, V, P><<<dim3(rows), dim3(threads), 0, stream>>>(a)
+#define LMX_SNT(T)                                                            \
+  if (vec) {                                                                  \
+    if (vpt == 1) LMX_SN(T, 8, 1); else if (vpt == 2) LMX_SN(T, 8, 2);        \
+    else LMX_SN(T, 8, 4);                                                     \
+  } else {                                                                    \
+    if (vpt == 1) LMX_SN(T, 1, 1); else LMX_SN(T, 1, 8);                      \
+  }
+  if (is_bf16) { LMX_SNT(bf16_t) } else { LMX_SNT(float) }
+#undef LMX_SNT
+#undef LMX_SN
+  return (int)hipGetLastError();
+}
+
 // Gated RMS norm of a mixer's output, in `groups` equal parts of a row, each
 // divided by its own root mean square:
-//   gate_first 0: out = norm(x) * w * sigmoid(g)      (linear attention)
-//   gate_first 1: out = norm(x * silu(g)) * w         (state-space mixer)
-// grid (rows, groups), one workgroup per part.
+//   mode 0: out = norm(x) * w * sigmoid(g)      (linear attention)
+//   mode 1: out = norm(x * silu(g)) * w         (state-space mixer)
+//   mode 2: out = norm(x) * w * silu(g)         (retention, delta rule)
+// grid (rows, groups), one workgroup per part; parts of up to 512 columns with
+// a power of two of 8-column pieces: one lane group per part, grid (row blocks).
 template <typename T, int V, int VPT>
 __global__ void __launch_bounds__(256) gated_norm_kernel(T* out, long out_ld, const T* x, long x_ld,
                                                          const T* g, long g_ld,
                                                          const float* __restrict__ w, int part,
-                                                         int gate_first, float eps) {
+                                                         int mode, float eps) {
   __shared__ float scratch[16];
   const long row = blockIdx.x, off = (long)blockIdx.y * part;
   const T* xr = x + row * x_ld + off;
@@ -528,8 +690,8 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(T* out, long out_ld, co
 #pragma unroll
     for (int e = 0; e < V; ++e) {
       const float s = sigmoid_t<T>(gt[i][e]);
-      if (gate_first) v[i][e] *= gt[i][e] * s;
-      gt[i][e] = gate_first ? 1.f : s;
+      if (mode == 1) v[i][e] *= gt[i][e] * s;
+      gt[i][e] = mode == 0 ? s : mode == 1 ? 1.f : gt[i][e] * s;
       ss += v[i][e] * v[i][e];
     }
   }
@@ -547,21 +709,62 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(T* out, long out_ld, co
   }
 }
 
+// lanes = part / 8 (a power of two up to 64): a part is one aligned lane group
+template <typename T>
+__global__ void __launch_bounds__(256) gated_norm_lanes_kernel(
+    T* out, long out_ld, const T* x, long x_ld, const T* g, long g_ld,
+    const float* __restrict__ w, long pieces, int per_row, int lanes, int mode, float eps) {
+  const long e0 = (long)blockIdx.x * 256 + threadIdx.x;
+  const bool on = e0 < pieces;
+  const long it = on ? e0 : pieces - 1;         // every lane takes part in the exchange
+  const long row = it / per_row;
+  const int c0 = 8 * (int)(it - row * per_row);
+  float v[8], gt[8], wv[8], ss = 0.f;
+  ldv<8>(v, x + row * x_ld + c0);
+  ldv<8>(gt, g + row * g_ld + c0);
+  ldv<8>(wv, w + c0);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float s = sigmoid_t<T>(gt[e]);
+    if (mode == 1) v[e] *= gt[e] * s;
+    wv[e] *= mode == 0 ? s : mode == 1 ? 1.f : gt[e] * s;
+    ss += v[e] * v[e];
+  }
+  for (int o = lanes >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+  const float inv = rsqrtf(ss / (float)(8 * lanes) + eps);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) wv[e] *= v[e] * inv;
+  if (on) stv<8>(out + row * out_ld + c0, wv);
+}
+
 int gated_norm(void* out, long out_ld, const void* x, long x_ld, const void* g, long g_ld,
-               const float* w, int rows, int cols, int groups, int gate_first, float eps,
+               const float* w, int rows, int cols, int groups, int mode, float eps,
                int is_bf16, hipStream_t stream) {
   if (rows <= 0) return 0;
-  if (groups < 1 || cols % groups != 0) return -1;
+  if (groups < 1 || cols % groups != 0 || mode < 0 || mode > 2) return -1;
   const int part = cols / groups;
   const bool vec = part % 8 == 0 && out_ld % 8 == 0 && x_ld % 8 == 0 && g_ld % 8 == 0 &&
                    (((uintptr_t)x | (uintptr_t)g | (uintptr_t)out) & 15) == 0;
   const int nchunk = vec ? part / 8 : part, vpt = (nchunk + 255) / 256;
   if (vpt > (vec ? 8 : 16)) return -2;
+  if (vec && nchunk <= 64 && (nchunk & (nchunk - 1)) == 0) {
+    const long pieces = (long)rows * (cols / 8);
+    const dim3 gl((unsigned)((pieces + 255) / 256));
+    if (is_bf16)
+      gated_norm_lanes_kernel<bf16_t><<<gl, dim3(256), 0, stream>>>(
+          (bf16_t*)out, out_ld, (const bf16_t*)x, x_ld, (const bf16_t*)g, g_ld, w, pieces, cols / 8,
+          nchunk, mode, eps);
+    else
+      gated_norm_lanes_kernel<float><<<gl, dim3(256), 0, stream>>>(
+          (float*)out, out_ld, (const float*)x, x_ld, (const float*)g, g_ld, w, pieces, cols / 8,
+          nchunk, mode, eps);
+    return (int)hipGetLastError();
+  }
   const int threads = nchunk >= 256 ? 256 : (nchunk + 63) / 64 * 64;
   const dim3 grid(rows, groups);
 #define LMX_GN(T, V, P)                                                                         \
   gated_norm_kernel<T, V, P><<<grid, dim3(threads), 0, stream>>>(                               \
-      (T*)out, out_ld, (const T*)x, x_ld, (const T*)g, g_ld, w, part, gate_first, eps)
+      (T*)out, out_ld, (const T*)x, x_ld, (const T*)g, g_ld, w, part, mode, eps)
 #define LMX_GNT(T)                                                                              \
   if (vec) {                                                                                    \
     if (vpt == 1) LMX_GN(T, 8, 1); else if (vpt == 2) LMX_GN(T, 8, 2); else LMX_GN(T, 8, 8);    \

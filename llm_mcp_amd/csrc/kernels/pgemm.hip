@@ -118,7 +118,7 @@ struct PgOut {
   __amdgpu_buffer_rsrc_t rc;     // C rows [m0, M)
   __amdgpu_buffer_rsrc_t rn;     // NRM 1: row scales [m0, M); NRM 2: ssq partials of rows [m0, M)
   int n0;
-  float lim;                     // ACT 6: the group's clamp
+  float lim, slope, shift;       // ACT 6: the group's clamp, the GLU's constants
 };
 
 // grouped rows (WP 2)
@@ -126,7 +126,8 @@ struct PgGroups {
   const int* tiles;              // [mtiles][2] group, first row; then the number of used tiles
   const int* off;                // [groups + 1] first rows
   const int* src;                // A row of a sorted row, or null
-  const float* limit;            // ACT 6
+  const float* limit;            // ACT 6: clamp per group
+  float slope, shift;            // ACT 6: g sigmoid(slope g) (u + shift)
   int mtiles;
 };
 
@@ -243,7 +244,7 @@ __device__ __forceinline__ void pg_store(RT& R, const PgOut& O, const PgThr& T,
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const float gc = fminf(g[r], O.lim), uc = fminf(fmaxf(u[r], -O.lim), O.lim);
-          o[r] = (short)f2bf(gc / (1.f + __expf(-1.702f * gc)) * (uc + 1.f));
+          o[r] = (short)f2bf(gc / (1.f + __expf(-O.slope * gc)) * (uc + O.shift));
         }
       } else
 #pragma unroll
@@ -547,7 +548,7 @@ __global__ void __launch_bounds__(PG_THREADS, 1) pgemm_pp2_kernel(
       const int g = grp.tiles[2 * tm];
       m0 = grp.tiles[2 * tm + 1];
       m1 = grp.off[g + 1];
-      if constexpr (ACT == 6) O.lim = grp.limit[g];
+      if constexpr (ACT == 6) { O.lim = grp.limit[g]; O.slope = grp.slope; O.shift = grp.shift; }
     }
     const long cbytes = (long)(m1 - m0) * ldc * 2;
     O.rc = __builtin_amdgcn_make_buffer_rsrc((void*)(C + (long)m0 * ldc), (short)0,
@@ -898,7 +899,7 @@ static int pg_cus() {
 // layout, C rows [M][N] or, with limit, the clamped GLU [M][N / 2].
 int pgemm_grouped(void* C, const void* A, const void* W, int M, int N, int K, long lda, long ldc,
                   int a_rows, const int* tiles, int mtiles, const int* off, const int* src,
-                  const float* limit, hipStream_t stream) {
+                  const float* limit, float slope, float shift, hipStream_t stream) {
   if (M <= 0 || mtiles <= 0) return 0;
   if (N % 256 != 0 || K % 64 != 0 || K < 192 || lda % 8 || ldc % 4 || !tiles || !off) return -1;
   // byte offsets are 32-bit: a tile's rows, or with src the whole of A
@@ -908,7 +909,7 @@ int pgemm_grouped(void* C, const void* A, const void* W, int M, int N, int K, lo
   if (pg_cus() == 0) return -2;
   const long all = (long)mtiles * (N / 256);
   const int grid = (int)(all < g_pg_cus ? all : g_pg_cus);
-  const PgGroups grp{tiles, off, src, limit, mtiles};
+  const PgGroups grp{tiles, off, src, limit, slope, shift, mtiles};
   auto C_ = (bf16_t*)C;
   auto A_ = (const bf16_t*)A;
   auto W_ = (const bf16_t*)W;

@@ -327,6 +327,110 @@ int rope_cache(void* qkv, long qkv_stride, const int* positions, const float* co
   return (int)hipGetLastError();
 }
 
+// Attention heads padded to D channels (true size dk): q and k RMS-normed over
+// the head (gains fp32 [D], zero in the padding), the first n channels turned by
+// the row's angles (ang [T][n]: cos | sin, neighbouring channels a pair), k and v
+// into their cache pages, q to rows.  A thread owns 8 channels of one head in up
+// to 4 rows that share a key quad (quads: row starts, then the end; null: one
+// row each), so values leave as whole quads.  D / 8 lanes reduce a head's norm.
+// grid (row groups, ceil(heads D / 2048)), block 256
+template <typename T>
+__global__ void __launch_bounds__(256) norm_rope_cache_kernel(
+    const T* __restrict__ p, long p_ld, const float* __restrict__ q_norm,
+    const float* __restrict__ k_norm, const float* __restrict__ ang, int n,
+    const int* __restrict__ slots, const int* __restrict__ quads, T* __restrict__ q,
+    T* __restrict__ kc, T* __restrict__ vc, int Hq, int Hkv, int D, int dk, int BS, float eps) {
+  const int c0 = (blockIdx.y * 256 + threadIdx.x) * 8;
+  const int head = c0 / D, d = c0 - head * D;
+  if (head >= Hq + 2 * Hkv) return;            // whole heads leave together
+  const int r0 = quads ? quads[blockIdx.x] : blockIdx.x;
+  const int cnt = quads ? min(4, quads[blockIdx.x + 1] - r0) : 1;
+  float x[4][8];
+  int slot[4];
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    slot[t] = -1;
+    if (t < cnt) {
+      ldv<8>(x[t], p + (long)(r0 + t) * p_ld + c0);
+      slot[t] = slots[r0 + t];
+    }
+  }
+  if (head >= Hq + Hkv) {
+    const long kvh = head - Hq - Hkv;
+    bool quad = cnt == 4 && slot[0] >= 0 && slot[0] % 4 == 0;
+#pragma unroll
+    for (int t = 1; t < 4; ++t) quad = quad && slot[t] == slot[0] + t;
+    if (quad) {
+      T* vp = vc + ((long)(slot[0] / BS) * Hkv + kvh) * BS * D + vq_off(d, slot[0] % BS, D);
+#pragma unroll
+      for (int e = 0; e < 8; e += 2) {
+        const float w[8] = {x[0][e], x[1][e], x[2][e], x[3][e],
+                            x[0][e + 1], x[1][e + 1], x[2][e + 1], x[3][e + 1]};
+        stv<8>(vp + 4 * e, w);
+      }
+      return;
+    }
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      if (t >= cnt || slot[t] < 0) continue;
+      T* vp = vc + ((long)(slot[t] / BS) * Hkv + kvh) * BS * D + vq_off(d, slot[t] % BS, D);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) st1(vp + 4 * e, x[t][e]);
+    }
+    return;
+  }
+  float w[8];
+  ldv<8>(w, (head < Hq ? q_norm : k_norm) + d);
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    if (t >= cnt) continue;
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += x[t][e] * x[t][e];
+    for (int o = D >> 4; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float inv = rsqrtf(ss / (float)dk + eps);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[t][e] *= inv * w[e];
+    if (d < n) {
+      const float* a = ang + (long)(r0 + t) * n;
+#pragma unroll
+      for (int e = 0; e < 8; e += 2) {
+        if (d + e >= n) continue;
+        const float c = a[(d + e) >> 1], s = a[(n + d + e) >> 1];
+        const float u = x[t][e], v = x[t][e + 1];
+        x[t][e] = u * c - v * s;
+        x[t][e + 1] = v * c + u * s;
+      }
+    }
+    if (head < Hq) {
+      stv<8>(q + (long)(r0 + t) * Hq * D + c0, x[t]);
+    } else if (slot[t] >= 0) {
+      stv<8>(kc + (((long)(slot[t] / BS) * Hkv + head - Hq) * BS + slot[t] % BS) * D + d, x[t]);
+    }
+  }
+}
+
+int norm_rope_cache(const void* p, long p_ld, const float* q_norm, const float* k_norm,
+                    const float* ang, int n, const int* slots, const int* quads, int groups,
+                    void* q, void* kc, void* vc, int Hq, int Hkv, int D, int dk, int BS, float eps,
+                    int is_bf16, hipStream_t stream) {
+  if (groups <= 0) return 0;
+  // a head's D / 8 lanes reduce inside one wave: D a power of two, 8..512
+  if (D < 8 || D > 512 || (D & (D - 1)) || dk < 1 || dk > D || n < 0 || n % 2 || n > dk ||
+      (n && !ang) || BS % 4 || p_ld % 8 || (((uintptr_t)p | (uintptr_t)q) & 15))
+    return -1;
+  const dim3 grid(groups, ((Hq + 2 * Hkv) * D / 8 + 255) / 256);
+  if (is_bf16)
+    norm_rope_cache_kernel<bf16_t><<<grid, dim3(256), 0, stream>>>(
+        (const bf16_t*)p, p_ld, q_norm, k_norm, ang, n, slots, quads, (bf16_t*)q, (bf16_t*)kc,
+        (bf16_t*)vc, Hq, Hkv, D, dk, BS, eps);
+  else
+    norm_rope_cache_kernel<float><<<grid, dim3(256), 0, stream>>>(
+        (const float*)p, p_ld, q_norm, k_norm, ang, n, slots, quads, (float*)q, (float*)kc,
+        (float*)vc, Hq, Hkv, D, dk, BS, eps);
+  return (int)hipGetLastError();
+}
+
 // Plain cache write (no rotation), used by the paged-cache tests and by
 // models without rotary embeddings.
 __global__ void kv_write_kernel(const bf16_t* __restrict__ k, const bf16_t* __restrict__ v,

@@ -234,7 +234,34 @@ class PikesunConfig(LayerListConfig):
         return cfg
 
 
-LAYER_LISTS = {c.architecture: c for c in (ZegopelConfig, PikesunConfig)}
+@dataclass
+class RefolixConfig(LayerListConfig):
+    """``retention`` and ``parallel`` (windowed attention beside a gated delta
+    rule) mixers, ``moe`` feed-forwards, the norm after the sum."""
+    name: str = "refolix"
+    family: str = "refolix"
+    architecture: str = "Refolix"
+    postln_alpha: float = 1.0       # the residual's weight in the sum that is normed
+    logit_scale: float = 1.0
+    logit_softcap: float | None = None
+
+    def to_json(self) -> dict:
+        return {**super().to_json(), "embedding": {"scale": self.embed_scale},
+                "postln_alpha": self.postln_alpha, "logit_scale": self.logit_scale,
+                "logit_softcap": self.logit_softcap}
+
+    @classmethod
+    def from_json(cls, js: dict, name: str):
+        cfg = super().from_json(js, name)
+        cfg.embed_scale = float(js.get("embedding", {}).get("scale", 1.0))
+        cfg.postln_alpha = float(js.get("postln_alpha", 1.0))
+        cfg.logit_scale = float(js.get("logit_scale", 1.0))
+        cap = js.get("logit_softcap")
+        cfg.logit_softcap = float(cap) if cap is not None else None
+        return cfg
+
+
+LAYER_LISTS = {c.architecture: c for c in (ZegopelConfig, PikesunConfig, RefolixConfig)}
 
 
 def zegopel_stack(pattern: str, ff: int, lightning: dict, mamba2: dict,
@@ -311,6 +338,54 @@ def _pikesun_8b() -> PikesunConfig:
     return PikesunConfig(name="pikesun-8b", vocab_size=128256, hidden_size=4096,
                          bos_token_id=128000, eos_token_ids=(128001, 128009), layers=layers,
                          embed_scale=64.0, residual_mult=0.5)
+
+
+def refolix_stack(pattern: str, retention: dict, parallel: dict, moe: dict) -> list:
+    """Layer list from a pattern of R (retention), P (parallel)."""
+    kinds = {"R": ("retention", retention), "P": ("parallel", parallel)}
+    return [{"type": kinds[c][0], "mixer": dict(kinds[c][1]), "mlp": dict(moe)} for c in pattern]
+
+
+def _grouped_moe(experts: int, top: int, ff: int, shared: int, groups: int, keep: int) -> dict:
+    return dict(kind="moe", router=dict(experts=experts, top=top,
+                                        groups=dict(count=groups, keep=keep)),
+                expert=dict(ff=ff), shared=dict(ff=shared))
+
+
+def _refolix_tiny() -> RefolixConfig:
+    left = dict(heads=4, kv_heads=2, dim=64, vdim=48, scale=0.125, softcap=30.0,
+                mask=dict(size=70), rot=dict(base=10000.0, dims=32, scaling=dict(
+                    factor=4.0, original=256, fast=32.0, slow=1.0)))
+    layers = refolix_stack(
+        "RPR", dict(heads=3, dim=32, vdim=56, decay=_retention_decays(3),
+                    rot=dict(base=10000.0, dims=32)),
+        dict(left=left, right=dict(heads=4, kv_heads=2, dim=48, vdim=40, conv=4)),
+        _grouped_moe(8, 2, 64, 96, 4, 2))
+    return RefolixConfig(name="tiny-refolix", vocab_size=512, hidden_size=192, bos_token_id=506,
+                         eos_token_ids=(510,), layers=layers, embed_scale=192 ** 0.5,
+                         postln_alpha=2.0, logit_scale=0.5, logit_softcap=30.0)
+
+
+def _retention_decays(heads: int) -> list:
+    """Per-head decays 1 - 2^(-5 - 7 h / heads): from fast to slow."""
+    return [1.0 - 2.0 ** (-5.0 - 7.0 * h / heads) for h in range(heads)]
+
+
+def _refolix_8b() -> RefolixConfig:
+    """Llama-3-8B's width and size, all experts counted (random weights:
+    benchmarks)."""
+    left = dict(heads=32, kv_heads=8, dim=128, vdim=128, scale=128 ** -0.5, softcap=50.0,
+                mask=dict(size=2048), rot=dict(base=500000.0, dims=64, scaling=dict(
+                    factor=4.0, original=8192, fast=32.0, slow=1.0)))
+    layers = refolix_stack(
+        "RRP" * 7, dict(heads=32, dim=128, vdim=128, decay=_retention_decays(32),
+                        rot=dict(base=10000.0, dims=128)),
+        dict(left=left, right=dict(heads=32, kv_heads=16, dim=128, vdim=128, conv=4)),
+        _grouped_moe(16, 4, 1024, 2048, 4, 2))
+    return RefolixConfig(name="refolix-8b", vocab_size=128256, hidden_size=4096,
+                         bos_token_id=128000, eos_token_ids=(128001, 128009), layers=layers,
+                         embed_scale=64.0, postln_alpha=3.0, logit_scale=0.25,
+                         logit_softcap=30.0)
 
 
 _LLAMA32_ROPE = {"rope_type": "llama3", "factor": 32.0, "low_freq_factor": 1.0,
@@ -408,6 +483,8 @@ PRESETS: dict[str, object] = {
     "zegopel-8b": _zegopel_8b(),
     "tiny-pikesun": _pikesun_tiny(),
     "pikesun-8b": _pikesun_8b(),
+    "tiny-refolix": _refolix_tiny(),
+    "refolix-8b": _refolix_8b(),
     "tiny-nomic": NomicBertConfig(name="tiny-nomic", vocab_size=512, hidden_size=256,
                                   intermediate_size=512, num_layers=2, num_heads=2, head_dim=128,
                                   embed_dim=256, max_position=2048),

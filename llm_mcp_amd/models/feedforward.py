@@ -58,6 +58,11 @@ class MixtureOfExperts:
 
     The shared expert runs as further experts of the routed ones' width that
     every token uses with weight 1: one grouped product covers all of them."""
+    glu = (1.702, 1.0)                     # slope of the gate's sigmoid, added to up
+
+    @staticmethod
+    def _limit(m: dict) -> float:
+        return float(m["limit"])
 
     def __init__(self, m: dict, width: int):
         self.width, self.kp, self.np = width, _up(width, 64), _up(width, 16)
@@ -68,8 +73,7 @@ class MixtureOfExperts:
         self.ff, self.sff = ex["ff"], sh["ff"] if sh else 0
         self.fp = max(_up(self.ff, 64), _up(-(-self.sff // 8), 64))   # at most 8 shared ones
         self.shared = -(-self.sff // self.fp)          # experts that hold the shared one
-        self.limits = [float(ex["limit"])] * self.E + [float(sh["limit"])] * self.shared \
-            if sh else [float(ex["limit"])] * self.E
+        self.limits = [self._limit(ex)] * self.E + ([self._limit(sh)] * self.shared if sh else [])
         self.shapes = {}
         for e in range(self.E):
             self.shapes.update({f"e{e}.gate": (self.ff, width), f"e{e}.up": (self.ff, width),
@@ -96,10 +100,47 @@ class MixtureOfExperts:
         self.limit = put(torch.tensor(self.limits), fp32=True)
         self.router = put(get("router"))
 
+    def _route(self, h):
+        return ops.moe_route(h, self.router, self.top, self.shared)
+
     def forward(self, h):
-        r = ops.moe_route(h, self.router, self.top, self.shared)
+        r = self._route(h)
         plan = ops.moe_plan(r, self.E + self.shared, self.w1.packed,
                             ops.wide_tiles(self.w1) and ops.wide_tiles(self.w2))
-        y = ops.grouped_linear(_pad_cols(h, self.kp), self.w1, plan, gather=True, glu=self.limit)
+        y = ops.grouped_linear(_pad_cols(h, self.kp), self.w1, plan, gather=True, glu=self.limit,
+                               act=self.glu)
         return ops.Mixture(ops.grouped_linear(y, self.w2, plan), plan.pos, r.weights)
+
+
+class GroupRoutedMoE(MixtureOfExperts):
+    """SiLU GLUs, routed by sigmoid scores s of the logits: the ``top`` largest
+    s + correction among the experts of the best groups (ranked by the sum of
+    their two largest), in the proportions of their s; the shared expert is
+    weighted by the sigmoid of one more logit."""
+    glu = (1.0, 0.0)
+
+    @staticmethod
+    def _limit(m: dict) -> float:
+        return float("inf")
+
+    def __init__(self, m: dict, width: int):
+        super().__init__(m, width)
+        g = m["router"].get("groups") or {"count": 1, "keep": 1}
+        self.groups, self.keep = g["count"], g["keep"]
+        if (self.groups < 1 or self.E % self.groups or not 0 < self.keep <= self.groups
+                or self.keep * (self.E // self.groups) < self.top):
+            raise ValueError("moe: groups do not fit the experts")
+        self.shapes["correction"] = (self.E,)
+        if self.shared:
+            self.shapes["shared.sg"] = (1, width)
+
+    def load(self, get, put):
+        super().load(get, put)
+        self.correction = put(get("correction"), fp32=True)
+        if self.shared:                    # the shared expert's logit: one more row
+            self.router = put(torch.cat([get("router"), get("shared.sg")]))
+
+    def _route(self, h):
+        return ops.moe_route(h, self.router, self.top, self.shared,
+                             ops.GroupScores(self.correction, self.groups, self.keep))
 

@@ -1,5 +1,5 @@
 """Decoders whose configuration lists their layers one by one (Zegopel,
-Pikesun), in the in-process serving engine.
+Pikesun, Refolix), in the in-process serving engine.
 
 A layer is a token mixer (``models.mixers``) and, where it has one, a
 feed-forward (``models.feedforward``), each between an optional norm before and
@@ -9,7 +9,8 @@ a norm after it around an fp32 residual stream:
 
 The norm after a sublayer, the residual add and the norm before the next
 sublayer (or the plain copy of the stream where there is none) are one kernel
-(``ops.sandwich_norm``), so a step is
+(``ops.sandwich_norm``; a family that norms the sum itself has its own form,
+``_join``), so a step is
 
   embedding + first norm -> per sublayer: input projection -> mixer kernels
   -> output projection -> sandwich norm -> ... -> LM head on the sampled rows
@@ -51,6 +52,7 @@ class LayerListModel:
     feedforwards: dict = {}       # mlp "kind" -> feed-forward class
     zero_centred = False          # stored gains act as 1 + w
     tail = "b"                    # suffix of the norm after a sublayer ("": no norm before it)
+    layer_scale = ""              # name of the per-channel scale of a sublayer's output, if any
 
     # ------------------------------------------------------------ layout ----
     @classmethod
@@ -94,6 +96,9 @@ class LayerListModel:
                 continue
             for names in cls.sublayer_norms(i, 1 if ff is None else 2):
                 out.update({n: (d,) for n in names if n})
+            if cls.layer_scale:
+                out.update({f"l{i}.{cls.layer_scale}{k}": (d,)
+                            for k in range(1, 2 if ff is None else 3)})
             out.update({f"l{i}.mix.{k}": s for k, s in mix.shapes.items()})
             if ff is not None:
                 out.update({f"l{i}.mlp.{k}": s for k, s in ff.shapes.items()})
@@ -119,10 +124,11 @@ class LayerListModel:
         self.D = max((m.D for m in kv), default=64)
         self.q_per_tile = next((m.q_per_tile for m in kv if m.q_per_tile), 16)
         self._plans = {}                       # key -> the part that builds that plan
-        for m, _ in self.parts:
+        mixing = [p for m, _ in self.parts for p in m.members()]
+        for m in mixing:
             if m.plan_key is not None:
                 self._plans.setdefault(m.plan_key, m)
-        self._angles = sorted({m.rot for m, _ in self.parts if m.rot is not None})
+        self._angles = sorted({m.rot for m in mixing if m.rot is not None})
         self._load(weights, seed)
 
     # ----------------------------------------------------------- weights ----
@@ -161,6 +167,9 @@ class LayerListModel:
                 ff.load(lambda n, p=f"l{i}.mlp.": get(p + n), put)
             norms[i] = [(gain(a), gain(b, cfg.residual_mult))
                         for a, b in self.sublayer_norms(i, 1 if ff is None else 2)]
+            if self.layer_scale:       # after: (norm, scale)
+                norms[i] = [(a, (b, put(get(f"l{i}.{self.layer_scale}{k + 1}"), fp32=True)))
+                            for k, (a, b) in enumerate(norms[i])]
         self.norms = [norms[j] for j in source]
         self.final_norm = gain("final.norm")
         self.head = put(get("head"))
@@ -169,8 +178,9 @@ class LayerListModel:
     def weight_bytes(self, copies: bool = False) -> int:
         """Bytes of the served weights (padding included)."""
         ts = [self.embed, self.head, self.final_norm]
-        ts += [t for ns in self.norms for pair in ns for t in pair if t is not None]
-        for o in (o for pair in self.parts for o in pair if o is not None):
+        ts += [t for ns in self.norms for pair in ns for p in pair
+               for t in (p if isinstance(p, tuple) else (p,)) if t is not None]
+        for o in (o for m, ff in self.parts for o in (m, *m.members(), ff) if o is not None):
             vals = [v.data if isinstance(v, ops.GroupedWeight) else v for v in vars(o).values()]
             ts += [t for t in vals if isinstance(t, torch.Tensor)]
         return sum({t.data_ptr(): t.numel() * t.element_size() for t in ts}.values())
@@ -209,6 +219,15 @@ class LayerListModel:
         return aux
 
     # ----------------------------------------------------------- forward ----
+    def _join(self, x, y, post, pre, rows=None):
+        """Take a sublayer's output y into the residual x (``post``: what
+        belongs to the norm after it) and return the rows the next one reads."""
+        return ops.sandwich_norm(x, self.cfg.rms_eps, y=y, w_post=post, w_pre=pre, rows=rows,
+                                 dtype=self.dtype)
+
+    def _logits(self, h):
+        return ops.linear(h, self.head)
+
     def forward(self, inp: StepInputs, k_caches: list, v_caches: list, decode_ws=None,
                 part_tokens: int = 512, layers_out: list | None = None) -> torch.Tensor:
         """Logits [len(sample_rows), vocab].  ``layers_out``: receives a copy of
@@ -217,7 +236,8 @@ class LayerListModel:
         inp.decode_ws, inp.part_tokens = decode_ws, part_tokens
         inp.aux = dict(inp.aux or {})
         for r in self._angles:
-            inp.aux["rot", r] = ops.rope_angles(inp.positions, self._freqs[r])
+            inp.aux["rot", r] = ops.rope_angles(inp.positions, self._freqs[r],
+                                                ops.rope_magnitude(*r))
         T = inp.num_tokens
         x = torch.empty((T, self.cfg.hidden_size), dtype=torch.float32, device=self.device)
         h = ops.sandwich_norm(x, eps, w_pre=self.norms[0][0][0], ids=inp.input_ids,
@@ -230,20 +250,18 @@ class LayerListModel:
             y = mix.forward(h, inp, next(kv) if mix.kv is not None else None, state)
             last = i + 1 == len(self.parts)
             if ff is not None:
-                h = ops.sandwich_norm(x, eps, y=y, w_post=n[0][1], w_pre=n[1][0], dtype=dt)
+                h = self._join(x, y, n[0][1], n[1][0])
                 y = ff.forward(h)
             post = n[-1][1]
             if not last:
-                h = ops.sandwich_norm(x, eps, y=y, w_post=post, w_pre=self.norms[i + 1][0][0],
-                                      dtype=dt)
+                h = self._join(x, y, post, self.norms[i + 1][0][0])
             elif layers_out is None:
                 # the final norm on the sampled rows only
-                h = ops.sandwich_norm(x, eps, y=y, w_post=post, w_pre=self.final_norm,
-                                      rows=None if all_rows else inp.sample_rows, dtype=dt)
+                h = self._join(x, y, post, self.final_norm,
+                               None if all_rows else inp.sample_rows)
             else:
-                ops.sandwich_norm(x, eps, y=y, w_post=post, dtype=dt)
-                h = ops.sandwich_norm(x, eps, w_pre=self.final_norm, rows=inp.sample_rows,
-                                      dtype=dt)
+                self._join(x, y, post, None)
+                h = self._join(x, None, None, self.final_norm, inp.sample_rows)
             if layers_out is not None:
                 layers_out.append(x.clone())
-        return ops.linear(h, self.head)
+        return self._logits(h)

@@ -42,11 +42,25 @@ def _fuse_rows(parts: list[torch.Tensor], pads: list[int]) -> torch.Tensor:
     return out
 
 
+def _head_size(d: int) -> int:
+    """Channels a head of d is padded to in the cache."""
+    D = 64
+    while D < d:
+        D *= 2
+    if D > 512:
+        raise ValueError("attention: head sizes up to 512")
+    return D
+
+
 class Mixer:
     kv = None                     # (heads, key size, value size) of its cache pages
     q_per_tile = 0
     plan_key = None
-    rot = None                    # (base, dims) of its rotary positions
+    rot = None                    # its rotary positions: ``ops.rope_freqs`` arguments
+
+    def members(self):
+        """The mixers it is made of: those that plan and rotate."""
+        return [self]
 
     def state_shapes(self, dtype):
         return []
@@ -185,12 +199,7 @@ class ConvAttentionMixer(Mixer):
         self.temp = (float(t["coef"]), float(t["every"]))
         if self.Hq % self.Hkv:
             raise ValueError("attention: heads must be a multiple of kv_heads")
-        D = 64
-        while D < max(self.dk, self.dv):
-            D *= 2
-        if D > 512:
-            raise ValueError("attention: head sizes up to 512")
-        self.D = D
+        D = self.D = _head_size(max(self.dk, self.dv))
         H, G, dk, dv = self.Hq, self.Hkv, self.dk, self.dv
         self.shapes = {"q": (H * dk, width), "k": (G * dk, width), "v": (G * dv, width),
                        "q.b": (H * dk,), "k.b": (G * dk,), "v.b": (G * dv,),
@@ -424,6 +433,277 @@ class LatentAttentionMixer(Mixer):
         return ops.linear(out, self.w_o, defer=True)
 
 
+def rotary(rot: dict | None, dim: int) -> tuple | None:
+    """``Mixer.rot`` of a configuration's rotation of the first ``dims`` of
+    ``dim`` channels, with its length scaling."""
+    if not rot or not rot["dims"]:
+        return None
+    if rot["dims"] % 2 or not 0 < rot["dims"] <= dim:
+        raise ValueError("rotation: an even number of a head's channels")
+    s = rot.get("scaling")
+    return (float(rot["base"]), int(rot["dims"])) + (
+        (float(s["factor"]), float(s["original"]), float(s["fast"]), float(s["slow"]))
+        if s else ())
+
+
+class RetentionMixer(ScanMixer):
+    """Linear attention with a constant decay per head on rotated queries and
+    keys: S <- decay S + k v^T, o = S^T q with k scaled by dim^-1/2; each head
+    divided by its root mean square, times silu(W_g h), projected.
+
+    The rotated channels of q and k are served with the pairs (i, i + dims/2)
+    next to each other: scores do not depend on the order of the channels."""
+
+    def __init__(self, m: dict, width: int, eps: float):
+        self.H, self.N, self.P, self.eps = m["heads"], m["dim"], m["vdim"], eps
+        self.decay = [float(x) for x in m["decay"]]
+        if len(self.decay) != self.H:
+            raise ValueError("retention: one decay per head")
+        H, N, P = self.H, self.N, self.P
+        self.rot = rotary(m.get("rot"), N)
+        self.shapes = {"q": (H * N, width), "k": (H * N, width), "v": (H * P, width),
+                       "g": (H * P, width), "o": (width, H * P)}
+        self.qk, self.vg = _up(H * N, 8), _up(H * P, 8)
+        self.proj = {"in": (2 * (self.qk + self.vg), width), "o": self.shapes["o"]}
+
+    def state_shapes(self, dtype):
+        return [((self.H, self.N, self.P), torch.float32)]
+
+    plan_key = property(lambda self: ("scan", self.H, self.P))
+
+    def _paired(self, w):
+        """[H * N, ...] rows with each head's rotated pairs next to each other."""
+        if self.rot is None:
+            return w
+        d = self.rot[1]
+        i = torch.arange(self.N)
+        i[:d] = torch.stack([i[:d // 2], i[d // 2:d]], 1).reshape(-1)
+        return w.reshape(self.H, self.N, -1)[:, i.to(w.device)].reshape(self.H * self.N, -1)
+
+    def load(self, get, put):
+        self.w_in = put(_fuse_rows([self._paired(get("q")), self._paired(get("k")), get("v"),
+                                    get("g")], [self.qk, self.qk, self.vg, self.vg]))
+        self.w_o = put(get("o"))
+        self.norm = put(torch.ones(self.H * self.P), fp32=True)
+        d = torch.tensor(self.decay, dtype=torch.float64)
+        self.decays = (put(d, fp32=True), put(d.log().clamp_min(-1e30), fp32=True))
+
+    def forward(self, h, inp, cache, state):
+        qk, vg = self.qk, self.vg
+        p = ops.linear(h, self.w_in)
+        ang = inp.aux["rot", self.rot] if self.rot else None
+        o = ops.linear_scan(p[:, :qk], p[:, qk:2 * qk], p[:, 2 * qk:2 * qk + vg], state[0],
+                            inp.cu_q, inp.context_lens, inp.state_slots, decay=self.decays,
+                            num_decode=inp.num_decode, segments=inp.aux.get(self.plan_key),
+                            angles=ang, k_scale=self.N ** -0.5)
+        y = ops.gated_norm(o, p[:, 2 * qk + vg:], self.norm, self.H, self.eps, gate_first=False,
+                           silu=True)
+        return ops.linear(y, self.w_o, defer=True)
+
+
+class SoftcapAttentionMixer(Mixer):
+    """Softmax attention in a sliding window: q and k RMS-normed per head, their
+    first channels rotated (neighbours paired), scores softly capped."""
+
+    def __init__(self, m: dict, width: int, eps: float):
+        self.Hq, self.Hkv, self.dk, self.dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        self.scale, self.eps = float(m["scale"]), eps
+        self.cap = float(m.get("softcap") or 0.0)
+        mask = m.get("mask")
+        self.window = int(mask["size"]) if mask else 0
+        if mask and self.window < 1:
+            raise ValueError("attention: a window of at least 1")
+        if self.Hq % self.Hkv:
+            raise ValueError("attention: heads must be a multiple of kv_heads")
+        self.rot = rotary(m.get("rot"), self.dk)
+        H, G, dk, dv = self.Hq, self.Hkv, self.dk, self.dv
+        self.D = _head_size(max(dk, dv))
+        self.shapes = {"q": (H * dk, width), "k": (G * dk, width), "v": (G * dv, width),
+                       "q.norm": (dk,), "k.norm": (dk,), "o": (width, H * dv)}
+        self.kv = (G, self.D, self.D)
+        self.rows = (H + 2 * G) * self.D
+        self.proj = {"in": (self.rows, width), "o": (width, H * self.D)}
+        # the MFMA attention kernels: head sizes 64 / 128, up to 16 query heads per kv head
+        self.mfma_geometry = self.D in (64, 128) and H // G <= 16
+        # queries per prefill workgroup (4 waves)
+        self.q_per_tile = (4 * (4 if self.D == 64 else ops.PREFILL_GROUPS_PER_WAVE)
+                           * (16 // (H // G)) if self.mfma_geometry else 0)
+        self.plan_key = ("rope_attn", self.q_per_tile)
+
+    def build_plan(self, qlens, ctx, seq0):
+        q = self.q_per_tile
+        items = [("quads", mixer_ops.row_quads(qlens, ctx, seq0))]
+        if q:
+            items.append((f"attn{q}", mixer_ops.row_tiles(qlens, q).reshape(-1)))
+        return items, None
+
+    def bind_plan(self, dev, host):
+        return dev["quads"], dev.get(f"attn{self.q_per_tile}")
+
+    def _heads(self, t, n, d):
+        """[n * d, ...] rows -> [n * D, ...], each head padded with zeros."""
+        out = t.new_zeros((n, self.D) + tuple(t.shape[1:]))
+        out[:, :d] = t.reshape((n, d) + tuple(t.shape[1:]))
+        return out.reshape((n * self.D,) + tuple(t.shape[1:]))
+
+    def in_rows(self, get):
+        return torch.cat([self._heads(get("q"), self.Hq, self.dk),
+                          self._heads(get("k"), self.Hkv, self.dk),
+                          self._heads(get("v"), self.Hkv, self.dv)])
+
+    def load(self, get, put, own_projection=True):
+        if own_projection:
+            self.w_in = put(self.in_rows(get))
+        self.q_norm = put(self._heads(get("q.norm"), 1, self.dk), fp32=True)
+        self.k_norm = put(self._heads(get("k.norm"), 1, self.dk), fp32=True)
+        self.w_o = put(self._heads(get("o").t().contiguous(), self.Hq, self.dv).t())
+
+    def forward(self, h, inp, cache, state):
+        return self.mix(ops.linear(h, self.w_in), inp, cache, state)
+
+    def mix(self, p, inp, cache, state):
+        """Output rows of projection rows p = [q | k | v | ..]."""
+        kc, vc = cache
+        quads, tiles = inp.aux.get(self.plan_key, (None, None))
+        ang = inp.aux["rot", self.rot] if self.rot else None
+        q = ops.norm_rope_cache(p, self.q_norm, self.k_norm, ang, inp.slots, kc, vc, self.Hq,
+                                self.dk, self.eps, quads)
+        T, nd = inp.num_tokens, inp.num_decode
+        if not self.mfma_geometry or q.dtype != torch.bfloat16:
+            a = ops.attention_any(q, kc, vc, inp.block_tables, inp.cu_q, inp.context_lens,
+                                  inp.positions, self.scale, self.Hq, window=self.window,
+                                  cap=self.cap)
+            return ops.linear(a, self.w_o, defer=True)
+        a = torch.empty((T, self.Hq * self.D), dtype=q.dtype, device=q.device)
+        if nd:
+            ops.paged_decode_attention(q[:nd], kc, vc, inp.block_tables, inp.context_lens,
+                                       self.scale, a[:nd], inp.decode_ws, inp.part_tokens,
+                                       Hq=self.Hq, order=inp.decode_order, precise=True,
+                                       window=self.window, cap=self.cap)
+        if T > nd:
+            ops.paged_prefill_attention(q, kc, vc, inp.block_tables[nd:], inp.cu_q[nd:],
+                                        inp.context_lens[nd:], tiles, self.scale, a, Hq=self.Hq,
+                                        q_per_tile=self.q_per_tile, precise=True,
+                                        window=self.window, cap=self.cap)
+        return ops.linear(a, self.w_o, defer=True)
+
+
+class GatedDeltaMixer(Mixer):
+    """Gated delta rule: q, k, v through a short convolution with SiLU, q and k
+    unit vectors per head (shared by heads / kv_heads value heads);
+
+        S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+
+    with beta = sigmoid(W_b h) and ln g = -exp(A_log) softplus(W_a h + dt_bias)
+    per head; each head of o divided by its root mean square, times a gain and
+    silu(W_g h), projected."""
+
+    def __init__(self, m: dict, width: int, eps: float):
+        self.H, self.G, self.N, self.P = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        self.taps, self.eps = m["conv"], eps
+        H, G, N, P = self.H, self.G, self.N, self.P
+        if H % G:
+            raise ValueError("delta rule: heads must be a multiple of kv_heads")
+        self.shapes = {"q": (G * N, width), "k": (G * N, width), "v": (H * P, width),
+                       "q.conv": (G * N, self.taps), "k.conv": (G * N, self.taps),
+                       "v.conv": (H * P, self.taps), "b": (H, width), "A_log": (H,),
+                       "norm": (P,), "a": (H, width), "dt_bias": (H,), "g": (H * P, width),
+                       "o": (width, H * P)}
+        self.qk, self.vp, self.hp = _up(G * N, 8), _up(H * P, 8), _up(H, 8)
+        self.C = 2 * self.qk + self.vp             # convolved channels
+        self.rows = self.C + self.vp + 2 * self.hp
+        self.proj = {"in": (self.rows, width), "o": (width, H * P)}
+
+    plan_key = ("delta",)
+
+    def build_plan(self, qlens, ctx, seq0):
+        chunks, first = mixer_ops.delta_chunks(qlens, seq0)
+        return [("dchunks", chunks), ("dfirst", first)], len(chunks)
+
+    def bind_plan(self, dev, host):
+        return ops.DeltaChunks(dev["dchunks"], dev["dfirst"], host)
+
+    def state_shapes(self, dtype):
+        out = [((self.H, self.N, self.P), torch.float32)]
+        if self.taps > 1:
+            out.append(((self.taps - 1, self.C), dtype))
+        return out
+
+    def in_rows(self, get):
+        return _fuse_rows([get(n) for n in ("q", "k", "v", "g", "b", "a")],
+                          [self.qk, self.qk, self.vp, self.vp, self.hp, self.hp])
+
+    def load(self, get, put, own_projection=True):
+        if own_projection:
+            self.w_in = put(self.in_rows(get))
+        self.conv = put(_fuse_rows([get(n + ".conv").float() for n in "qkv"],
+                                   [self.qk, self.qk, self.vp]).t(), fp32=True)
+        self.neg_a = put(-torch.exp(get("A_log").float()), fp32=True)
+        self.dt_bias = put(get("dt_bias"), fp32=True)
+        self.norm = put(get("norm").float().repeat(self.H), fp32=True)
+        self.w_o = put(get("o"))
+
+    def forward(self, h, inp, cache, state):
+        return self.mix(ops.linear(h, self.w_in), inp, cache, state)
+
+    def mix(self, p, inp, cache, state):
+        """Output rows of projection rows p = [q | k | v | g | b | a | ..]."""
+        C, qk, vp, hp = self.C, self.qk, self.vp, self.hp
+        u = ops.short_conv(p[:, :C], self.conv, state[1] if self.taps > 1 else None, inp.cu_q,
+                           inp.context_lens, inp.state_slots, silu=True,
+                           tiles=inp.aux.get("conv"))
+        b, a = p[:, C + vp:C + vp + hp], p[:, C + vp + hp:C + vp + 2 * hp]
+        o = ops.delta_rule(u[:, :qk], u[:, qk:2 * qk], u[:, 2 * qk:], b, a, self.dt_bias,
+                           self.neg_a, state[0], inp.cu_q, inp.context_lens, inp.state_slots,
+                           self.G, num_decode=inp.num_decode, chunks=inp.aux.get(self.plan_key))
+        y = ops.gated_norm(o, p[:, C:C + vp], self.norm, self.H, self.eps, gate_first=False,
+                           silu=True)
+        return ops.linear(y, self.w_o, defer=True)
+
+
+class ParallelMixer(Mixer):
+    """Windowed attention and a gated delta rule side by side on the same rows:
+    half the sum of their outputs, each RMS-normed over the width.  One input
+    projection serves both."""
+
+    def __init__(self, m: dict, width: int, eps: float):
+        self.left = SoftcapAttentionMixer(m["left"], width, eps)
+        self.right = GatedDeltaMixer(m["right"], width, eps)
+        self.shapes = {}
+        for name, part in (("left", self.left), ("right", self.right)):
+            self.shapes.update({f"{name}.{k}": s for k, s in part.shapes.items()})
+            self.shapes[name + ".out"] = (width,)
+        self.kv, self.q_per_tile = self.left.kv, self.left.q_per_tile
+        self.Hq, self.Hkv, self.D = self.left.Hq, self.left.Hkv, self.left.D
+        rows = self.left.rows + self.right.rows
+        # a wide projection is rounded up to whole 256-row GEMM tiles
+        self.tail = (_up(rows, 256) if rows >= 4096 else rows) - rows
+        self.proj = {"in": (rows + self.tail, width), "left.o": self.left.proj["o"],
+                     "right.o": self.right.proj["o"]}
+
+    def members(self):
+        return [self.left, self.right]
+
+    def state_shapes(self, dtype):
+        return self.right.state_shapes(dtype)
+
+    def load(self, get, put):
+        left, right = (lambda n, s=s: get(f"{s}.{n}") for s in ("left", "right"))
+        parts = [self.left.in_rows(left), self.right.in_rows(right)]
+        self.w_in = put(_fuse_rows(parts, [self.left.rows, self.right.rows + self.tail]))
+        self.left.load(left, put, own_projection=False)
+        self.right.load(right, put, own_projection=False)
+        self.out_left, self.out_right = (put(0.5 * get(s + ".out").float(), fp32=True)
+                                         for s in ("left", "right"))
+
+    def forward(self, h, inp, cache, state):
+        p = ops.linear(h, self.w_in)
+        n = self.left.rows
+        return ops.NormedPair(self.left.mix(p[:, :n], inp, cache, state),
+                              self.right.mix(p[:, n:], inp, cache, state),
+                              self.out_left, self.out_right)
+
+
 def init_std(name: str, shape: tuple, depth: int, zero_centred: bool = True) -> tuple[float, float]:
     """(mean, std) of a tensor's random initialisation (benchmarks, tests)."""
     leaf = name.rsplit(".", 1)[-1]
@@ -431,7 +711,8 @@ def init_std(name: str, shape: tuple, depth: int, zero_centred: bool = True) -> 
         return 0.0, 0.02 / math.sqrt(2 * depth)
     if leaf == "conv":
         return 1.0 / shape[-1], 0.2
-    if name.endswith(".mix.norm") or leaf == "D" or name.endswith(("dq.norm", "dkv.norm")):
+    if name.endswith((".mix.norm", "dq.norm", "dkv.norm", ".q.norm", ".k.norm", ".right.norm",
+                      ".out")) or leaf in ("D", "ls1", "ls2"):
         return 1.0, 0.1
     if leaf == "A_log":
         return 0.5, 0.5

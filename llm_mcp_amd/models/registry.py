@@ -21,6 +21,9 @@ def layer_list_class(family: str):
     if family == "pikesun":
         from .pikesun import PikesunModel
         return PikesunModel
+    if family == "refolix":
+        from .refolix import RefolixModel
+        return RefolixModel
     raise ValueError(f"{family}: not a layer-list family")
 
 

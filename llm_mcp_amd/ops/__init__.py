@@ -231,8 +231,8 @@ def paged_decode_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cont
                            scale: float, out: torch.Tensor, ws: DecodeWorkspace | None = None,
                            part_tokens: int = 512, Hq: int | None = None,
                            order: torch.Tensor | None = None, rope: tuple | None = None,
-                           gate: torch.Tensor | None = None, precise: bool = False
-                           ) -> torch.Tensor:
+                           gate: torch.Tensor | None = None, precise: bool = False,
+                           window: int = 0, cap: float = 0.0) -> torch.Tensor:
     """q: [B, Hq*D] rows (row stride = q.stride(0)); out: [B, Hq*D].
     ``order`` (int32 [B], optional): a permutation of the rows, longest
     context first -- the workgroup dispatch order (``decode_order``).
@@ -242,7 +242,9 @@ def paged_decode_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cont
     ``slots`` itself (K2 + K5 fused into K4: ``rope_and_cache`` is skipped for
     these rows; no q/k-norm models).  ``gate`` ([B, Hq*D] rows): the output is
     multiplied by sigmoid(gate).  ``precise``: softmax weights enter the PV
-    product with fp32 precision (a bf16 pair) instead of one bf16."""
+    product with fp32 precision (a bf16 pair) instead of one bf16.  ``window``
+    (0: all): only that many last positions are seen; ``cap`` (0: none): scores
+    become cap tanh(score / cap); both with ``precise``."""
     B = q.shape[0]
     NB, Hkv, BS, D = k_cache.shape
     Hq = Hq or (q.shape[1] // D)
@@ -252,13 +254,14 @@ def paged_decode_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cont
         rope = None
     if not q.is_cuda:
         o = ref.paged_decode(q[:, : Hq * D].reshape(B, Hq, D), k_cache, v_cache, block_tables,
-                             context_lens, scale)
+                             context_lens, scale, window, cap)
         out.copy_(ref.gate_rows(o.reshape(B, Hq * D), gate))
         return out
     _bf16(q, "q")
     _chk(gate is None or (gate.stride(1) == 1 and gate.dtype == torch.bfloat16
                           and gate.shape[0] >= B and gate.shape[1] >= Hq * D), "gate rows")
     _chk(not (precise and rope is not None), "precise weights: no fused-rotary form")
+    _chk(precise or not (window or cap), "window / cap: with precise weights")
     _chk(D in (64, 128) and BS == 32, "paged decode kernel needs D in (64,128), BS=32")
     _chk(Hq % Hkv == 0 and Hq // Hkv <= 16, "GQA group must be <= 16")
     _chk(block_tables.dtype == torch.int32 and context_lens.dtype == torch.int32, "int32 meta")
@@ -281,7 +284,7 @@ def paged_decode_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cont
                           _ptr(ws.part_o) if ws else 0, _ptr(ws.part_ml) if ws else 0, B, Hq, Hkv,
                           D, BS, float(scale), part_tokens, max_parts, _ptr(pos), _ptr(cs),
                           _ptr(slots), _ptr(gate), gate.stride(0) if gate is not None else 0,
-                          int(precise), _stream())
+                          int(precise), window, float(cap), _stream())
     return out
 
 
@@ -298,15 +301,15 @@ def paged_prefill_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_
                             context_lens, tiles, scale: float, out: torch.Tensor,
                             causal: bool = True, Hq: int | None = None,
                             q_per_tile: int | None = None, rope=None,
-                            gate: torch.Tensor | None = None,
-                            precise: bool = False) -> torch.Tensor:
+                            gate: torch.Tensor | None = None, precise: bool = False,
+                            window: int = 0, cap: float = 0.0) -> torch.Tensor:
     """Varlen prefill. q/out: [T, Hq*D] rows; tiles: int32 [(seq, q_start)]
     built with ``q_per_tile`` queries per tile (default
     ``prefill_q_per_tile(Hq, Hkv, D)``; the kernel's workgroup width follows
     from it).  ``rope`` = (positions int32 [rows], cos_sin fp32 [P, D]): q is
     unrotated and the kernel applies the rotary embedding (the rope/cache
-    kernel ran with ``skip_q``).  ``gate`` / ``precise``: as in
-    ``paged_decode_attention``."""
+    kernel ran with ``skip_q``).  ``gate`` / ``precise`` / ``window`` / ``cap``:
+    as in ``paged_decode_attention``."""
     NB, Hkv, BS, D = k_cache.shape
     T = q.shape[0]
     Hq = Hq or (q.shape[1] // D)
@@ -316,7 +319,7 @@ def paged_prefill_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_
         q = qr
     if not q.is_cuda:
         o = ref.paged_prefill(q[:, : Hq * D].reshape(T, Hq, D), k_cache, v_cache, block_tables,
-                              cu_q, context_lens, scale, causal)
+                              cu_q, context_lens, scale, causal, window, cap)
         a, b = int(cu_q[0]), int(cu_q[len(context_lens)])
         out[a:b].copy_(ref.gate_rows(o.reshape(T, Hq * D), gate)[a:b])
         return out
@@ -326,6 +329,7 @@ def paged_prefill_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_
                           and gate.data_ptr() % 16 == 0), "gate rows")
     _chk(D in (64, 128) and BS == 32, "paged prefill kernel needs D in (64,128), BS=32")
     _chk(Hq % Hkv == 0 and Hq // Hkv <= 16, "GQA group must be <= 16")
+    _chk((precise and causal) or not (window or cap), "window / cap: causal, with precise weights")
     _chk(tiles.dtype == torch.int32 and cu_q.dtype == torch.int32, "int32 meta")
     num_tiles = tiles.numel() // 2
     native().paged_prefill(_ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache),
@@ -335,7 +339,8 @@ def paged_prefill_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_
                            q_per_tile or prefill_q_per_tile(Hq, Hkv, D),
                            _ptr(rope[0]) if rope is not None else 0,
                            _ptr(rope[1]) if rope is not None else 0, _ptr(gate),
-                           gate.stride(0) if gate is not None else 0, int(precise), _stream())
+                           gate.stride(0) if gate is not None else 0, int(precise), window,
+                           float(cap), _stream())
     return out
 
 
@@ -1797,9 +1802,10 @@ def pgemm_sk(a: torch.Tensor, w: torch.Tensor, splits: int, act: int = 0, epi: i
     return out
 
 
-from .grouped import (GroupedWeight, Mixture, MoePlan, Route, grouped_heads,  # noqa: E402,F401
-                      grouped_linear, moe_plan, moe_route, pack_grouped, wide_tiles)
-from .mixers import (RGLRU_MAX_BLOCK, RGLRU_TILE, LatentRows, ScanSegments,  # noqa: E402,F401
-                     attention_any, conv_qkv_cache, gated_norm, latent_attention,
-                     latent_prefill, latent_prefill_ok, latent_prep, latent_query, linear_scan, rglru,
-                     rope_angles, rope_freqs, sandwich_norm, scan_segments, short_conv)
+from .grouped import (GroupedWeight, GroupScores, Mixture, MoePlan, Route,  # noqa: E402,F401
+                      grouped_heads, grouped_linear, moe_plan, moe_route, pack_grouped, wide_tiles)
+from .mixers import (RGLRU_MAX_BLOCK, RGLRU_TILE, DeltaChunks, LatentRows,  # noqa: E402,F401
+                     NormedPair, ScanSegments, attention_any, conv_qkv_cache, delta_rule,
+                     gated_norm, latent_attention, latent_prefill, latent_prefill_ok, latent_prep,
+                     latent_query, linear_scan, norm_rope_cache, rglru, rope_angles, rope_freqs,
+                     rope_magnitude, sandwich_norm, scan_segments, short_conv, soft_cap, sum_norm)

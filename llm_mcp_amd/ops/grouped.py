@@ -11,6 +11,7 @@ from . import _chk, _ptr, _stream, native, ref
 
 MOE_MAX_EXPERTS = 256      # experts a router kernel ranks
 MOE_MAX_TOP = 32
+MOE_MAX_GROUPS = 64
 
 
 @dataclass
@@ -52,22 +53,48 @@ class Route:
     weights: torch.Tensor    # fp32 [T, J]
 
 
-def moe_route(h: torch.Tensor, w: torch.Tensor, top: int, extra: int = 0) -> Route:
+@dataclass
+class GroupScores:
+    """Routing by sigmoid scores s: experts are chosen by s + ``correction``
+    (fp32 [E]) within the ``keep`` best of ``groups`` groups of neighbours."""
+    correction: torch.Tensor
+    groups: int = 1
+    keep: int = 1
+
+
+def moe_route(h: torch.Tensor, w: torch.Tensor, top: int, extra: int = 0,
+              scores: GroupScores | None = None) -> Route:
     """The ``top`` largest of the fp32 logits w h per row (lowest index first
     among equals) with the softmax over just those; then experts E, E + 1, ..
-    (``extra`` of them) with weight 1."""
-    E, d = w.shape
+    (``extra`` of them) with weight 1.
+
+    With ``scores``: the ``top`` largest s + correction, s = sigmoid(w h), among
+    the groups with the largest sums of two such scores, in the proportions of
+    their s; a row of w behind the E experts' is the logit whose sigmoid weighs
+    the extra ones."""
+    rows, d = w.shape
+    E = rows if scores is None else scores.correction.numel()
     T = h.shape[0]
-    _chk(0 < top <= E, "moe_route: top")
+    _chk(0 < top <= E and rows - E in (0, 1), "moe_route: top, router rows")
+    if scores is not None:
+        _chk(E % scores.groups == 0 and scores.groups <= MOE_MAX_GROUPS
+             and 0 < scores.keep <= scores.groups and scores.keep * (E // scores.groups) >= top,
+             "moe_route: groups")
     if not h.is_cuda:
-        return Route(*ref.moe_route(h, w, top, extra))
-    _chk(E <= MOE_MAX_EXPERTS and top + extra <= MOE_MAX_TOP, "moe_route: sizes")
+        return Route(*(ref.moe_route(h, w, top, extra) if scores is None else
+                       ref.moe_route_groups(h, w, top, extra, scores)))
+    _chk(rows <= MOE_MAX_EXPERTS and top + extra <= MOE_MAX_TOP, "moe_route: sizes")
+    corr, groups, keep = None, 1, 1
+    if scores is not None:
+        corr, groups, keep = scores.correction, scores.groups, scores.keep
+        _chk(corr.dtype == torch.float32 and corr.is_contiguous() and corr.is_cuda,
+             "moe_route: fp32 correction")
     _chk(h.dtype == w.dtype and h.dtype in (torch.bfloat16, torch.float32)
          and h.shape[1] == d and h.stride(1) == 1 and w.is_contiguous(), "moe_route operands")
     ids = torch.empty((T, top + extra), dtype=torch.int32, device=h.device)
     wts = torch.empty((T, top + extra), dtype=torch.float32, device=h.device)
-    native().moe_route(_ptr(h), h.stride(0), _ptr(w), T, d, E, top, extra, _ptr(ids), _ptr(wts),
-                       int(h.dtype == torch.bfloat16), _stream())
+    native().moe_route(_ptr(h), h.stride(0), _ptr(w), T, d, E, rows, top, extra, _ptr(corr), groups,
+                       keep, _ptr(ids), _ptr(wts), int(h.dtype == torch.bfloat16), _stream())
     return Route(ids, wts)
 
 
@@ -125,25 +152,26 @@ MOE_CHUNK = 1024           # uses per block of the sort (moe.hip)
 
 
 def _grouped(a, a_gs, w: GroupedWeight, c, c_gs, M, bm, mtiles, plan=None, src=None, limit=None,
-             gate=None):
+             gate=None, act=(1.702, 1.0)):
     bf = int(w.packed)
     _chk(a.dtype == w.data.dtype == c.dtype and a.stride(1) == 1 and c.stride(1) == 1
          and (w.packed or a.dtype == torch.float32), "grouped operands")
     native().grouped(_ptr(a), a.stride(0), a_gs, _ptr(w.data), _ptr(c), c.stride(0), c_gs,
                      w.groups, w.N, w.K, M, _ptr(plan.tiles) if plan else 0, mtiles,
-                     _ptr(plan.off) if plan else 0, _ptr(src), _ptr(limit), _ptr(gate),
+                     _ptr(plan.off) if plan else 0, _ptr(src), _ptr(limit), *act, _ptr(gate),
                      gate.stride(0) if gate is not None else 0, bm, bf, _stream())
 
 
 def grouped_linear(x: torch.Tensor, w: GroupedWeight, plan: MoePlan, gather: bool = False,
-                   glu: torch.Tensor | None = None) -> torch.Tensor:
+                   glu: torch.Tensor | None = None,
+                   act: tuple[float, float] = (1.702, 1.0)) -> torch.Tensor:
     """Rows in expert order [n, N]: x[src] (``gather``) or x's own rows times
-    their expert's w^T.  ``glu`` (fp32 [groups], the clamps): w's rows are gate
-    / up interleaved per 16, the result is g sigmoid(1.702 g) (u + 1) of the
-    clamped pair, [n, N / 2]."""
+    their expert's w^T.  ``glu`` (fp32 [groups], the clamps; inf: none): w's
+    rows are gate / up interleaved per 16, the result is g sigmoid(act[0] g)
+    (u + act[1]) of the clamped pair, [n, N / 2]."""
     n = plan.src.numel()
     if not x.is_cuda:
-        return ref.grouped_rows(x, w.data, plan.src, plan.off, gather, glu)
+        return ref.grouped_rows(x, w.data, plan.src, plan.off, gather, glu, act)
     _chk(x.shape[1] >= w.K and (gather or x.shape[0] == n), "grouped_linear rows")
     _chk(plan.off.numel() == w.groups + 1 and plan.bm in (16, 32, 64, 128, 256), "grouped_linear plan")
     _chk(glu is None or (glu.dtype == torch.float32 and glu.numel() == w.groups and w.N % 32 == 0),
@@ -156,9 +184,9 @@ def grouped_linear(x: torch.Tensor, w: GroupedWeight, plan: MoePlan, gather: boo
              and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0, "grouped_linear: K13 operands")
         native().pgemm_grouped(_ptr(out), _ptr(x), _ptr(w.data), n, w.N, w.K, x.stride(0),
                                out.stride(0), x.shape[0], _ptr(plan.tiles), mt, _ptr(plan.off),
-                               _ptr(src), _ptr(glu), _stream())
+                               _ptr(src), _ptr(glu), *act, _stream())
     else:
-        _grouped(x, 0, w, out, 0, n, plan.bm, mt, plan, src, glu)
+        _grouped(x, 0, w, out, 0, n, plan.bm, mt, plan, src, glu, act=act)
     return out
 
 

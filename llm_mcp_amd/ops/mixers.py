@@ -95,21 +95,107 @@ def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tens
     return out
 
 
+class NormedPair:
+    """Sublayer output rows rms(a) * wa + rms(b) * wb of two branches (rows or
+    ``Partials``), left to the consuming kernel."""
+    __slots__ = ("a", "b", "wa", "wb")
+
+    def __init__(self, a, b, wa: torch.Tensor, wb: torch.Tensor):
+        self.a, self.b, self.wa, self.wb = a, b, wa, wb
+
+    def sum(self, eps: float) -> torch.Tensor:
+        a, b = (x.float() * torch.rsqrt(x.float().pow(2).mean(-1, keepdim=True) + eps)
+                for x in (self.a, self.b))
+        return a * self.wa + b * self.wb
+
+
+def _sublayer_rows(y, T: int, d: int, dtype, name: str) -> tuple:
+    """(rows, row stride, slabs, slab stride) of rows or ``Partials``."""
+    if isinstance(y, Partials):
+        _chk((y.M, y.N) == (T, d), f"{name} partials shape")
+        return _ptr(y.slabs), d, y.S, y.M * y.N
+    _chk(y.shape == (T, d) and y.stride(1) == 1 and y.dtype == dtype, f"{name} rows")
+    return _ptr(y), y.stride(0), 0, 0
+
+
+def sum_norm(residual: torch.Tensor, eps: float, y, alpha: float, scale: torch.Tensor | None,
+             w_post: torch.Tensor | None, w_pre: torch.Tensor | None = None,
+             rows: torch.Tensor | None = None,
+             dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
+    """The fp32 residual stream of a decoder that layer-norms the sum:
+
+        r = ln(alpha residual + scale y) * w_post    (residual without y)
+        residual = r                                  (unless ``rows`` is given)
+        return ln(r) * w_pre                          (``dtype`` rows; r itself without w_pre)
+
+    ln(x) = (x - mean) / sqrt(variance + eps).  y: sublayer output rows,
+    ``Partials``, ``Mixture`` or ``NormedPair``; ``rows`` (int64) and the fp32
+    vectors as in ``sandwich_norm``."""
+    T, d = residual.shape
+    if not residual.is_cuda:
+        if isinstance(y, Mixture):
+            y = y.sum()[:, :d]
+        elif isinstance(y, NormedPair):
+            y = y.sum(eps)
+        return ref.sum_norm(residual, eps, y, alpha, scale, w_post, w_pre, rows, dtype)
+    _chk(residual.dtype == torch.float32 and residual.is_contiguous(), "residual: fp32 rows")
+    _f32(scale, d, "scale"); _f32(w_post, d, "w_post"); _f32(w_pre, d, "w_pre")
+    _chk((y is None) == (w_post is None) == (scale is None) and (y is not None or w_pre is not None),
+         "sum_norm: y, its scale and its norm go together")
+    a, b, mix, gains = (0, 0, 0, 0), (0, 0, 0, 0), (0, 0, 0), (0, 0)
+    if isinstance(y, Mixture):
+        _chk(y.rows.shape[1] >= d and y.rows.stride(1) == 1 and y.rows.dtype == dtype
+             and y.pos.shape == y.weights.shape and y.pos.shape[0] == T
+             and y.pos.dtype == torch.int32 and y.weights.dtype == torch.float32
+             and y.pos.is_contiguous() and y.weights.is_contiguous(), "sum_norm mixture")
+        a, mix = (_ptr(y.rows), y.rows.stride(0), 0, 0), (_ptr(y.pos), _ptr(y.weights), y.pos.shape[1])
+    elif isinstance(y, NormedPair):
+        _f32(y.wa, d, "pair gain"); _f32(y.wb, d, "pair gain")
+        a, b = (_sublayer_rows(x, T, d, dtype, "sum_norm pair") for x in (y.a, y.b))
+        gains = (_ptr(y.wa), _ptr(y.wb))
+    elif y is not None:
+        a = _sublayer_rows(y, T, d, dtype, "sum_norm y")
+    n = T
+    if rows is not None:
+        _chk(rows.dtype == torch.int64 and rows.is_contiguous(), "rows: int64")
+        n = rows.numel()
+    out = torch.empty((n, d), dtype=dtype, device=residual.device)
+    native().sum_norm(_ptr(out), _ptr(residual), *a, *mix, *b, *gains, float(alpha), _ptr(scale),
+                      _ptr(w_post), _ptr(w_pre), _ptr(rows), n, d, float(eps),
+                      int(dtype == torch.bfloat16), _stream())
+    return out
+
+
+def soft_cap(x: torch.Tensor, scale: float, cap: float | None) -> torch.Tensor:
+    """x <- cap tanh(scale x / cap) in place (cap None: scale x)."""
+    if scale == 1.0 and cap is None:
+        return x
+    if not x.is_cuda:
+        y = x.float() * scale
+        return x.copy_(y if cap is None else cap * torch.tanh(y / cap))
+    bf = _rows_dtype(x, "x")
+    _chk(x.is_contiguous(), "soft_cap: contiguous rows")
+    native().soft_cap(_ptr(x), x.numel(), float(scale), float(cap or 0.0), bf, _stream())
+    return x
+
+
 def gated_norm(x: torch.Tensor, gate: torch.Tensor, w: torch.Tensor, groups: int, eps: float,
-               gate_first: bool) -> torch.Tensor:
+               gate_first: bool, silu: bool = False) -> torch.Tensor:
     """RMS norm of x in ``groups`` equal parts of a row, gain w (fp32), gated:
-    rms(x) * w * sigmoid(gate), or with ``gate_first`` rms(x * silu(gate)) * w."""
+    rms(x) * w * sigmoid(gate) (``silu``: silu(gate)), or with ``gate_first``
+    rms(x * silu(gate)) * w."""
     T, C = x.shape
     _chk(C % groups == 0, "gated_norm groups")
     if not x.is_cuda:
-        return ref.gated_norm(x, gate, w, groups, eps, gate_first)
+        return ref.gated_norm(x, gate, w, groups, eps, gate_first, silu)
     bf = _rows_dtype(x, "x")
     _f32(w, C, "w")
     _chk(gate.dtype == x.dtype and gate.shape[0] == T and gate.shape[1] >= C
          and gate.stride(1) == 1 and x.stride(1) == 1, "gated_norm rows")
     out = torch.empty((T, C), dtype=x.dtype, device=x.device)
     native().gated_norm(_ptr(out), out.stride(0), _ptr(x), x.stride(0), _ptr(gate),
-                        gate.stride(0), _ptr(w), T, C, groups, int(gate_first), float(eps), bf,
+                        gate.stride(0), _ptr(w), T, C, groups,
+                        1 if gate_first else 2 if silu else 0, float(eps), bf,
                         _stream())
     return out
 
@@ -239,7 +325,8 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
                 decay: tuple[torch.Tensor, torch.Tensor] | None = None,
                 dt: tuple[torch.Tensor, torch.Tensor, torch.Tensor] | None = None,
                 skip: torch.Tensor | None = None, silu: bool = False, num_decode: int = 0,
-                segments: ScanSegments | None = None) -> torch.Tensor:
+                segments: ScanSegments | None = None, angles: torch.Tensor | None = None,
+                k_scale: float = 1.0) -> torch.Tensor:
     """Per head S <- a S + s k v^T, o = S^T q + skip v over each sequence's rows,
     from and to ``state`` (fp32 [slots, H, N, P]).
 
@@ -249,7 +336,11 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
     bias fp32 [H], neg_a fp32 [H]): s = softplus(dt + bias), a = exp(neg_a s).
     Sequences before ``num_decode`` (one row each) take the recurrent kernel;
     the others the chunked MFMA kernel when ``segments`` is given and the shape
-    allows it, the recurrent one otherwise.  Returns rows [T, H * P]."""
+    allows it, the recurrent one otherwise.  Returns rows [T, H * P].
+
+    ``angles`` (``rope_angles`` [T, n]): the first n channels of q and k are
+    turned by them, neighbours paired, and k is multiplied by ``k_scale``; the
+    rows of q and k that the chunked kernel reads are rotated in place."""
     _, H, N, P = state.shape
     T, S = q.shape[0], ctx.numel()
     _chk((decay is None) != (dt is None), "linear_scan: decay or dt")
@@ -257,7 +348,7 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
     out = torch.empty((T, H * P), dtype=q.dtype, device=q.device)
     if not q.is_cuda:
         ref.linear_scan(q, k, v, out, state, cu_q, ctx, slots, heads_per_group, decay, dt, skip,
-                        silu, range(S))
+                        silu, range(S), angles, k_scale)
         return out
     bf = _rows_dtype(q, "q")
     gn = H // heads_per_group * N
@@ -275,13 +366,20 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
     else:
         _f32(decay[0], H, "decay"); _f32(decay[1], H, "log decay")
         scal = (0, 0, 0, 0, _ptr(decay[0]), _ptr(decay[1]))
+    nrot = 0
+    if angles is not None:
+        nrot = angles.shape[1]
+        _f32(angles, T * nrot, "angles")
+        _chk(nrot % 2 == 0 and nrot <= N and not silu, "linear_scan: rotated channels")
+    turned = angles is not None or k_scale != 1.0
     args = (_ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), *scal, _ptr(skip),
             _ptr(out), out.stride(0), _ptr(state), _ptr(cu_q), _ptr(ctx), _ptr(slots), H, N, P,
             heads_per_group, int(silu), bf)
     chunked = segments is not None and S > num_decode and _chunk_ok(N, P, q, k, v)
     n_rec = num_decode if chunked else S
     if n_rec:
-        native().linear_scan(*args, 0, n_rec, 0, 0, 0, 0, 0, 0, _stream())
+        native().linear_scan(*args, _ptr(angles), nrot, float(k_scale), 0, n_rec, 0, 0, 0, 0, 0, 0,
+                             _stream())
     if chunked:
         g = segments
         _chk(g.segs.dtype == torch.int32 and g.segs.numel() >= 4 * g.n
@@ -291,23 +389,147 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
         if not g.one_pass:
             ws = torch.empty((g.n, H, N, P), dtype=torch.float32, device=q.device)
             wl = torch.empty((g.n, H), dtype=torch.float32, device=q.device)
-        native().linear_scan(*args, num_decode, S - num_decode, _ptr(g.segs), g.n, _ptr(g.first),
-                             int(g.one_pass), _ptr(ws), _ptr(wl), _stream())
+        if turned:                # decode rows come first, one each
+            native().rotate_rows(_ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(angles), nrot,
+                                 num_decode, T, gn // N, N, float(k_scale), _stream())
+        native().linear_scan(*args, 0, 0, 1.0, num_decode, S - num_decode, _ptr(g.segs), g.n,
+                             _ptr(g.first), int(g.one_pass), _ptr(ws), _ptr(wl), _stream())
     return out
 
 
+# ---------------------------------------------------------- gated delta rule --
+DELTA_CHUNK = 64           # DC in csrc/kernels/delta.hip
+
+
+@dataclass
+class DeltaChunks:
+    """Chunks of a step's multi-token sequences for the chunked delta rule."""
+    chunks: torch.Tensor    # int32 [n, 2]: sequence, first row in it
+    first: torch.Tensor     # int32 [sequences + 1]: each sequence's first chunk
+    n: int
+
+
+def delta_chunks(qlens, seq0: int) -> tuple[np.ndarray, np.ndarray]:
+    """Host plan of ``DeltaChunks`` for sequences seq0, seq0 + 1, ..."""
+    t = row_tiles(qlens, DELTA_CHUNK)
+    t[:, 0] += seq0
+    n = -(-np.asarray(qlens, np.int64) // DELTA_CHUNK)
+    return t, np.concatenate([[0], np.cumsum(n)]).astype(np.int32)
+
+
+def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b: torch.Tensor, a: torch.Tensor,
+               dt_bias: torch.Tensor, neg_a: torch.Tensor, state: torch.Tensor, cu_q, ctx, slots,
+               G: int, num_decode: int = 0, chunks: DeltaChunks | None = None) -> torch.Tensor:
+    """Gated delta rule over each sequence's rows, from and to ``state`` (fp32
+    [slots, H, N, P]): with q, k (rows of G x N channels, shared by H / G heads)
+    divided by their norms sqrt(sum + 1e-6), q also by sqrt(N), v of H x P,
+    beta = sigmoid(b), g = exp(neg_a softplus(a + dt_bias)) per head,
+
+        S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+
+    Sequences before ``num_decode`` (one row each) take the recurrent kernel;
+    the others the chunked MFMA kernels when ``chunks`` is given and the shape
+    allows it, the recurrent one otherwise.  Returns rows [T, H * P]."""
+    _, H, N, P = state.shape
+    T, S = q.shape[0], ctx.numel()
+    _chk(H % G == 0, "delta_rule: heads per group")
+    out = torch.empty((T, H * P), dtype=q.dtype, device=q.device)
+    if not q.is_cuda:
+        ref.delta_rule(q, k, v, b, a, dt_bias, neg_a, out, state, cu_q, ctx, slots, G)
+        return out
+    bf = _rows_dtype(q, "q")
+    for t, c, name in ((q, G * N, "q"), (k, G * N, "k"), (v, H * P, "v"), (b, H, "b"), (a, H, "a")):
+        _chk(t.dtype == q.dtype and t.shape[0] == T and t.shape[1] >= c and t.stride(1) == 1,
+             f"delta_rule {name} rows")
+    _chk(state.dtype == torch.float32 and state.is_contiguous(), "delta_rule state: fp32")
+    _meta(S, cu_q=cu_q, ctx=ctx, slots=slots)
+    _f32(dt_bias, H, "dt bias"); _f32(neg_a, H, "neg_a")
+    args = (_ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(b), b.stride(0),
+            _ptr(a), a.stride(0), _ptr(dt_bias), _ptr(neg_a), _ptr(out), out.stride(0), _ptr(state),
+            _ptr(cu_q), _ptr(ctx), _ptr(slots), H, G, N, P)
+    chunked = chunks is not None and S > num_decode and _chunk_ok(N, P, q, k, v)
+    n_rec = num_decode if chunked else S
+    if n_rec:
+        native().delta_recurrent(*args, n_rec, bf, _stream())
+    if chunked:
+        g = chunks
+        _chk(g.chunks.dtype == torch.int32 and g.chunks.numel() >= 2 * g.n
+             and g.first.dtype == torch.int32 and g.first.numel() == S - num_decode + 1,
+             "delta_rule chunks")
+        mats = torch.empty((g.n, H, DELTA_MATS), dtype=torch.bfloat16, device=q.device)
+        vecs = torch.empty((g.n, H, DELTA_VECS), dtype=torch.float32, device=q.device)
+        native().delta_chunks(*args, num_decode, S - num_decode, _ptr(g.chunks), g.n,
+                              _ptr(g.first), _ptr(mats), _ptr(vecs), _stream())
+    return out
+
+
+DELTA_MATS = 4 * 6 * 512   # per chunk and head: two triangular matrices as bf16 pairs
+DELTA_VECS = 5 * 64        # per chunk and head: per-token factors (delta.hip)
+
+
 # ---------------------------------------------------------------- attention --
+def row_quads(qlens, ctx, seq0: int) -> np.ndarray:
+    """int32 [n + 1]: row starts of groups of up to 4 rows that share a key quad
+    of the cache (positions 4i .. 4i + 3), then the end; the rows of the seq0
+    single-row sequences in front are groups of their own."""
+    qlens, ctx = np.asarray(qlens, np.int64), np.asarray(ctx, np.int64)
+    p0 = ctx - qlens
+    n = (ctx - 1) // 4 - p0 // 4 + 1
+    i = np.arange(int(n.sum())) - np.repeat(np.cumsum(n) - n, n)
+    row0 = seq0 + np.cumsum(qlens) - qlens
+    start = np.maximum((np.repeat(p0 // 4, n) + i) * 4, np.repeat(p0, n))
+    rows = np.repeat(row0 - p0, n) + start
+    return np.concatenate([np.arange(seq0), rows, [seq0 + qlens.sum()]]).astype(np.int32)
+
+
+def norm_rope_cache(p: torch.Tensor, q_norm: torch.Tensor, k_norm: torch.Tensor,
+                    angles: torch.Tensor | None, slots, k_cache, v_cache, Hq: int, dk: int,
+                    eps: float, quads: torch.Tensor | None = None) -> torch.Tensor:
+    """The projection rows' q | k | v heads (each padded to D channels): q and k
+    RMS-normed over the ``dk`` true channels (gains fp32 [D], zero in the
+    padding), their first channels turned by ``angles`` (neighbours paired); k
+    and v go to the paged cache at ``slots`` (-1: none).  ``quads``
+    (``row_quads``): rows whose values are written together (None: every row
+    alone).  Returns q rows [T, Hq * D]."""
+    _, Hkv, BS, D = k_cache.shape
+    T = p.shape[0]
+    if not p.is_cuda:
+        return ref.norm_rope_cache(p, q_norm, k_norm, angles, slots, k_cache, v_cache, Hq, dk, eps)
+    bf = _rows_dtype(p, "p")
+    C = (Hq + 2 * Hkv) * D
+    _f32(q_norm, D, "q_norm"); _f32(k_norm, D, "k_norm")
+    n = 0
+    if angles is not None:
+        n = angles.shape[1]
+        _f32(angles, T * n, "angles")
+    _meta(T, slots=slots)
+    _chk(p.shape[1] >= C and p.stride(1) == 1 and p.stride(0) % 8 == 0 and p.data_ptr() % 16 == 0
+         and n <= dk <= D and k_cache.dtype == v_cache.dtype == p.dtype
+         and k_cache.is_contiguous() and v_cache.is_contiguous(), "norm_rope_cache rows")
+    _chk(quads is None or (quads.dtype == torch.int32 and quads.is_contiguous()
+                           and quads.numel() >= 2), "row quads")
+    q = torch.empty((T, Hq * D), dtype=p.dtype, device=p.device)
+    groups = T if quads is None else quads.numel() - 1
+    native().norm_rope_cache(_ptr(p), p.stride(0), _ptr(q_norm), _ptr(k_norm), _ptr(angles), n,
+                             _ptr(slots), _ptr(quads), groups, _ptr(q), _ptr(k_cache),
+                             _ptr(v_cache), Hq, Hkv, D, dk, BS, float(eps), bf, _stream())
+    return q
+
+
 def attention_any(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, ctx, positions,
-                  scale: float, Hq: int, gate: torch.Tensor | None = None) -> torch.Tensor:
+                  scale: float, Hq: int, gate: torch.Tensor | None = None, window: int = 0,
+                  cap: float = 0.0) -> torch.Tensor:
     """Causal paged attention of every row (decode and prompt rows alike), fp32
     arithmetic, for what the MFMA kernels do not cover: fp32 caches, head sizes
     256 / 512, more than 16 query heads per kv head.  Output times
-    sigmoid(gate) when given."""
+    sigmoid(gate) when given.  ``window`` (0: all): a row sees that many last
+    positions; ``cap`` (0: none): scores become cap tanh(score / cap)."""
     _, Hkv, BS, D = k_cache.shape
     T, S = q.shape[0], ctx.numel()
     out = torch.empty((T, Hq * D), dtype=q.dtype, device=q.device)
     if not q.is_cuda:
-        o = ref.paged_prefill(q.reshape(T, Hq, D), k_cache, v_cache, block_tables, cu_q, ctx, scale)
+        o = ref.paged_prefill(q.reshape(T, Hq, D), k_cache, v_cache, block_tables, cu_q, ctx, scale,
+                              True, window, cap)
         out.copy_(ref.gate_rows(o.reshape(T, Hq * D), gate))
         return out
     bf = _rows_dtype(q, "q")
@@ -323,7 +545,7 @@ def attention_any(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, ctx, po
                            _ptr(block_tables), block_tables.stride(0), _ptr(cu_q), S,
                            _ptr(positions), T, _ptr(out), out.stride(0), _ptr(gate),
                            gate.stride(0) if gate is not None else 0, Hq, Hkv, D, BS,
-                           float(scale), bf, _stream())
+                           float(scale), window, float(cap), bf, _stream())
     return out
 
 
@@ -380,21 +602,39 @@ def rglru(u: torch.Tensor, y: torch.Tensor, y_bias: torch.Tensor, gates: Grouped
 
 
 # --------------------------------------------------------- latent attention --
-def rope_freqs(base: float, dims: int, device="cpu") -> torch.Tensor:
-    """base^(-2i / dims), i < dims / 2 (double)."""
+def rope_freqs(base: float, dims: int, factor: float = 1.0, original: float = 0.0,
+               fast: float = 0.0, slow: float = 0.0, device="cpu") -> torch.Tensor:
+    """base^(-2i / dims), i < dims / 2 (double).  ``original`` > 0: a context of
+    that length stretched by ``factor`` -- components that turn ``fast`` times
+    and more within it stay, those that turn ``slow`` times and less are divided
+    by the factor, a ramp between them."""
     i = torch.arange(dims // 2, dtype=torch.float64, device=device)
-    return torch.exp(-2.0 * math.log(base) / dims * i)
+    f = torch.exp(-2.0 * math.log(base) / dims * i)
+    if not original:
+        return f
+
+    def turning(times):        # the component that turns that often
+        return dims * math.log(original / (2 * math.pi * times)) / (2 * math.log(base))
+    lo = max(math.floor(turning(fast)), 0)
+    hi = min(math.ceil(turning(slow)), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+    return f / factor * ramp + f * (1 - ramp)
 
 
-def rope_angles(positions: torch.Tensor, freqs: torch.Tensor) -> torch.Tensor:
-    """fp32 [T, dims]: cos | sin of position * frequency (reduced in double, so
-    no table bounds the positions)."""
+def rope_magnitude(base: float, dims: int, factor: float = 1.0, original: float = 0.0, *_) -> float:
+    """What cos and sin of a rotation (``rope_freqs`` arguments) are multiplied by."""
+    return 0.1 * math.log(factor) + 1.0 if original else 1.0
+
+
+def rope_angles(positions: torch.Tensor, freqs: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+    """fp32 [T, dims]: cos | sin of position * frequency, times ``scale``
+    (reduced in double, so no table bounds the positions)."""
     if not positions.is_cuda:
-        return ref.rope_angles(positions, freqs)
+        return ref.rope_angles(positions, freqs, scale)
     T, n = positions.numel(), freqs.numel()
     _chk(positions.dtype == torch.int32 and freqs.dtype == torch.float64, "rope_angles")
     out = torch.empty((T, 2 * n), dtype=torch.float32, device=positions.device)
-    native().rope_angles(_ptr(positions), _ptr(freqs), T, n, _ptr(out), _stream())
+    native().rope_angles(_ptr(positions), _ptr(freqs), T, n, float(scale), _ptr(out), _stream())
     return out
 
 

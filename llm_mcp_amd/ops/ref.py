@@ -109,33 +109,38 @@ def gather_kv(k_cache, v_cache, block_table, n):
     return k, v
 
 
-def attention_dense(q, k, v, scale, causal_offset: int | None):
-    """q [Tq, Hq, D], k/v [Tk, Hkv, D]; query i sees keys <= causal_offset + i."""
+def attention_dense(q, k, v, scale, causal_offset: int | None, window: int = 0, cap: float = 0.0):
+    """q [Tq, Hq, D], k/v [Tk, Hkv, D]; query i sees keys <= causal_offset + i
+    (the last ``window`` of them), scores softly capped."""
     Hq, Hkv = q.shape[1], k.shape[1]
     G = Hq // Hkv
     kf = k.float().repeat_interleave(G, dim=1)
     vf = v.float().repeat_interleave(G, dim=1)
     s = torch.einsum("qhd,khd->hqk", q.float(), kf) * scale
+    if cap:
+        s = cap * torch.tanh(s / cap)
     if causal_offset is not None:
         Tq, Tk = q.shape[0], k.shape[0]
         qi = torch.arange(Tq, device=q.device)[:, None] + causal_offset
         ki = torch.arange(Tk, device=q.device)[None, :]
-        s = s.masked_fill((ki > qi)[None], float("-inf"))
+        hidden = (ki > qi) | (ki <= qi - window) if window else ki > qi
+        s = s.masked_fill(hidden[None], float("-inf"))
     p = torch.softmax(s, dim=-1)
     return torch.einsum("hqk,khd->qhd", p, vf)
 
 
-def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale):
+def paged_decode(q, k_cache, v_cache, block_tables, context_lens, scale, window=0, cap=0.0):
     """q [B, Hq, D] -> [B, Hq, D] (one query per sequence at position ctx-1)."""
     out = torch.empty_like(q)
     for b in range(q.shape[0]):
         n = int(context_lens[b])
         k, v = gather_kv(k_cache, v_cache, block_tables[b], n)
-        out[b] = attention_dense(q[b:b + 1], k, v, scale, None)[0].to(q.dtype)
+        out[b] = attention_dense(q[b:b + 1], k, v, scale, n - 1, window, cap)[0].to(q.dtype)
     return out
 
 
-def paged_prefill(q, k_cache, v_cache, block_tables, cu_q, context_lens, scale, causal=True):
+def paged_prefill(q, k_cache, v_cache, block_tables, cu_q, context_lens, scale, causal=True,
+                  window=0, cap=0.0):
     """q [T, Hq, D] for a varlen batch; keys come from the paged cache."""
     out = torch.empty_like(q)
     for s in range(len(context_lens)):
@@ -143,7 +148,7 @@ def paged_prefill(q, k_cache, v_cache, block_tables, cu_q, context_lens, scale, 
         n = int(context_lens[s])
         k, v = gather_kv(k_cache, v_cache, block_tables[s], n)
         off = (n - (b - a)) if causal else None
-        out[a:b] = attention_dense(q[a:b], k, v, scale, off).to(q.dtype)
+        out[a:b] = attention_dense(q[a:b], k, v, scale, off, window, cap).to(q.dtype)
     return out
 
 
@@ -415,14 +420,27 @@ def sandwich_norm(residual, eps, y=None, w_post=None, w_pre=None, ids=None, tabl
     return (r if w_pre is None else _unit(r, eps) * w_pre).to(dtype)
 
 
-def gated_norm(x, gate, w, groups, eps, gate_first):
+def sum_norm(residual, eps, y, alpha, scale, w_post, w_pre=None, rows=None, dtype=torch.bfloat16):
+    def norm(z, w):
+        z = z - z.mean(-1, keepdim=True)
+        return _unit(z, eps) * w
+    r = residual if rows is None else residual[rows]
+    if y is not None:
+        y = y if rows is None else y[rows]
+        r = norm(alpha * r + scale * y.float(), w_post)
+    if rows is None:
+        residual.copy_(r)
+    return (r if w_pre is None else norm(r, w_pre)).to(dtype)
+
+
+def gated_norm(x, gate, w, groups, eps, gate_first, silu=False):
     T, C = x.shape
     v, g = x.float(), gate[:, :C].float()
     if gate_first:
         v = v * torch.nn.functional.silu(g)
     v = _unit(v.reshape(T, groups, C // groups), eps).reshape(T, C) * w
     if not gate_first:
-        v = v * torch.sigmoid(g)
+        v = v * (torch.nn.functional.silu(g) if silu else torch.sigmoid(g))
     return v.to(x.dtype)
 
 
@@ -463,10 +481,64 @@ def conv_qkv_cache(u, w, in_bias, state, cu_q, ctx, state_slots, q_out, k_cache,
     write_cache((y * inv)[:, Hq:Hq + Hkv], y[:, Hq + Hkv:Hq + 2 * Hkv], slots, k_cache, v_cache)
 
 
-def linear_scan(q, k, v, out, state, cu_q, ctx, slots, hpg, decay, dt, skip, silu, seqs):
+def norm_rope_cache(p, q_norm, k_norm, ang, slots, k_cache, v_cache, Hq, dk, eps):
+    _, Hkv, _, D = k_cache.shape
+    T = p.shape[0]
+    x = p[:, :(Hq + 2 * Hkv) * D].float().view(T, -1, D)
+    qk = x[:, :Hq + Hkv]
+    qk = qk * torch.rsqrt(qk.pow(2).sum(-1, keepdim=True) / dk + eps)
+    qk = rotate_pairs(torch.cat([qk[:, :Hq] * q_norm, qk[:, Hq:] * k_norm], 1), ang)
+    write_cache(qk[:, Hq:], x[:, Hq + Hkv:], slots, k_cache, v_cache)
+    return qk[:, :Hq].reshape(T, Hq * D).to(p.dtype)
+
+
+def rotate_pairs(x, ang):
+    """x [T, H, d] fp32: components (2i, 2i + 1) turned by the angles [T, n] of
+    ``rope_angles``, the first n of d (None: none)."""
+    if ang is None:
+        return x
+    n = ang.shape[1]
+    c, s = ang[:, None, :n // 2], ang[:, None, n // 2:]
+    u, v = x[..., 0:n:2], x[..., 1:n:2]
+    y = torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2)
+    return torch.cat([y, x[..., n:]], -1)
+
+
+def delta_rule(q, k, v, b, a, dt_bias, neg_a, out, state, cu_q, ctx, slots, G):
+    """See ops.delta_rule; one token after the other, fp32."""
+    _, H, N, P = state.shape
+    T = q.shape[0]
+
+    def heads(x):
+        x = x[:, :G * N].float().view(T, G, N)
+        x = x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) + 1e-6)
+        return x.repeat_interleave(H // G, 1)
+    qs, ks, vs = heads(q) * N ** -0.5, heads(k), v[:, :H * P].float().view(T, H, P)
+    beta = torch.sigmoid(b[:, :H].float())
+    g = torch.exp(neg_a * torch.nn.functional.softplus(a[:, :H].float() + dt_bias))
+    for s in range(len(ctx)):
+        t0, t1, slot = int(cu_q[s]), int(cu_q[s + 1]), int(slots[s])
+        if slot < 0:
+            continue
+        S = torch.zeros(H, N, P) if int(ctx[s]) == t1 - t0 else state[slot].clone()
+        for t in range(t0, t1):
+            S = g[t][:, None, None] * S
+            u = beta[t][:, None] * (vs[t] - torch.einsum("hnp,hn->hp", S, ks[t]))
+            S = S + ks[t][:, :, None] * u[:, None, :]
+            out[t, :H * P] = torch.einsum("hnp,hn->hp", S, qs[t]).reshape(-1).to(out.dtype)
+        state[slot] = S
+
+
+def linear_scan(q, k, v, out, state, cu_q, ctx, slots, hpg, decay, dt, skip, silu, seqs,
+                angles=None, k_scale=1.0):
     """See ops.linear_scan; one token after the other, fp32."""
     _, H, N, P = state.shape
     G = H // hpg
+    if angles is not None or k_scale != 1.0:
+        T = q.shape[0]
+        q = rotate_pairs(q[:, :G * N].float().view(T, G, N), angles).to(q.dtype).view(T, -1)
+        k = (rotate_pairs(k[:, :G * N].float().view(T, G, N), angles) * k_scale).to(k.dtype) \
+            .view(T, -1)
     act = (lambda x: torch.nn.functional.silu(x.float()).to(q.dtype).float()) if silu \
         else (lambda x: x.float())
     for s in seqs:
@@ -517,9 +589,9 @@ def rglru(u, y, y_bias, gates, gate_bias, log_a, out, state, cu_q, ctx, slots):
 
 
 # ------------------------------------------------------- latent attention ---
-def rope_angles(positions, freqs):
+def rope_angles(positions, freqs, scale=1.0):
     a = positions.double()[:, None] * freqs
-    return torch.cat([a.cos(), a.sin()], 1).float()
+    return (torch.cat([a.cos(), a.sin()], 1) * scale).float()
 
 
 def rotate(x, ang):
@@ -572,10 +644,27 @@ def latent_attention(ql, pages, block_tables, cu_q, positions, scale, window, H,
 
 
 # ----------------------------------------------------- grouped products -----
-def clamped_glu(g, u, limit):
+def clamped_glu(g, u, limit, act=(1.702, 1.0)):
     g = torch.clamp(g, max=limit)
     u = torch.clamp(u, -limit, limit)
-    return g * torch.sigmoid(1.702 * g) * (u + 1.0)
+    return g * torch.sigmoid(act[0] * g) * (u + act[1])
+
+
+def moe_route_groups(h, w, top, extra, scores):
+    E, n = scores.correction.numel(), scores.groups
+    z = torch.sigmoid(h.float() @ w.float().t())
+    s, T = z[:, :E], h.shape[0]
+    c = s + scores.correction
+    rank = c.view(T, n, E // n).topk(min(2, E // n), -1).values.sum(-1)
+    g = torch.sort(rank, dim=-1, descending=True, stable=True).indices[:, :scores.keep]
+    kept = torch.zeros(T, n, dtype=torch.bool).scatter_(1, g, True)
+    c = c.masked_fill(~kept.repeat_interleave(E // n, 1), float("-inf"))
+    ids = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :top]
+    wts = s.gather(1, ids)
+    wts = wts / (wts.sum(-1, keepdim=True) + 1e-20)
+    ids = torch.cat([ids, torch.arange(E, E + extra).expand(T, extra)], 1)
+    shared = z[:, E:].expand(T, extra) if z.shape[1] > E else torch.ones(T, extra)
+    return ids.to(torch.int32), torch.cat([wts, shared], 1)
 
 
 def moe_route(h, w, top, extra):
@@ -587,7 +676,7 @@ def moe_route(h, w, top, extra):
     return ids.to(torch.int32), wts
 
 
-def grouped_rows(x, w, src, off, gather, limit):
+def grouped_rows(x, w, src, off, gather, limit, act=(1.702, 1.0)):
     """Rows off[e]..off[e+1] of the expert order times w[e]^T."""
     K = w.shape[2]
     out = torch.zeros((src.numel(), w.shape[1] // (2 if limit is not None else 1)), dtype=x.dtype)
@@ -597,6 +686,6 @@ def grouped_rows(x, w, src, off, gather, limit):
         y = rows[:, :K].float() @ w[e].float().t()
         if limit is not None:
             y = y.view(b - a, w.shape[1] // 32, 2, 16)
-            y = clamped_glu(y[:, :, 0], y[:, :, 1], float(limit[e])).reshape(b - a, out.shape[1])
+            y = clamped_glu(y[:, :, 0], y[:, :, 1], float(limit[e]), act).reshape(b - a, out.shape[1])
         out[a:b] = y.to(x.dtype)
     return out
