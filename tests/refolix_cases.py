@@ -112,10 +112,11 @@ def shapes(cfg):
     return out
 
 
-def weights(cfg, seed=0):
+def weights(cfg, seed=0, calm=False):
     """bf16 weights under which every mechanism moves the logits: gains away
     from 1, corrections that outweigh scores, decays that neither vanish nor
-    hold."""
+    hold.  ``calm``: routers whose choices stay clear of ties (a choice that
+    falls the other way in bf16 moves every later token)."""
     g = torch.Generator().manual_seed(seed)
     out = {}
     for name, s in shapes(cfg).items():
@@ -127,6 +128,8 @@ def weights(cfg, seed=0):
             t = 1.0 + 0.3 * t
         elif leaf == "correction":
             t = 0.4 * t - 0.3
+        elif leaf == "router" and calm:
+            t = 0.03 * t / math.sqrt(s[-1])
         elif leaf == "A_log":
             t = 0.5 * t
         elif leaf == "dt_bias":
