@@ -214,7 +214,7 @@ __device__ __forceinline__ f32x4_t mfma_f32(float a, float b, f32x4_t c) {
 }
 
 // grid (chunks, H), block 256.  The score images are overlaid by the fp32
-// matrices A, T, B.
+// matrices A and T; B passes through T's place first.
 template <int NK>
 __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs a, const int* __restrict__ chunks,
                                                          bf16_t* __restrict__ mats,
@@ -226,7 +226,6 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs a, const int*
   bf16_t* const sQ = sK + DC * LQ;
   float* const mA = reinterpret_cast<float*>(prep_sm);
   float* const mT = mA + DC * DTL;
-  float* const mB = mT + DC * DTL;
   const int chunk = blockIdx.x, h = blockIdx.y;
   const int seq = chunks[2 * chunk], b0 = chunks[2 * chunk + 1];
   const long row0 = a.cu_q[seq] + b0;
@@ -308,11 +307,36 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs a, const int*
       const int t = wave * 16 + 4 * g + r, j = jt * 16 + c;
       const float dec = j <= t ? fast_exp2(cum[t] - cum[j]) * rk[j] : 0.f;
       mA[t * DTL + j] = j < t ? beta[t] * rk[t] * dec * kk[jt][r] : 0.f;
-      mB[t * DTL + j] = j <= t ? rq[t] * dec * qk[jt][r] : 0.f;
-      if (jt > wave) mT[t * DTL + j] = 0.f;
+      mT[t * DTL + j] = j <= t ? rq[t] * dec * qk[jt][r] : 0.f;
     }
+  bf16_t* const out = mats + ((long)chunk * a.H + h) * DMATS;
+  auto emit = [&](int tri, int which) {
+    const int it = tri < 2 ? tri : tri < 4 ? 2 : 3, ks = tri < 2 ? 0 : tri & 1;
+    const float* src = mT + (16 * it + c) * DTL + 32 * ks + 4 * g;
+    const f32x4_t x0 = *reinterpret_cast<const f32x4_t*>(src);
+    const f32x4_t x1 = *reinterpret_cast<const f32x4_t*>(src + 16);
+    u32x4_t hi, lo;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const f32x4_t& x = e < 2 ? x0 : x1;
+      uint32_t p, r;
+      split2(x[2 * (e & 1)], x[2 * (e & 1) + 1], p, r);
+      hi[e] = p;
+      lo[e] = r;
+    }
+    *reinterpret_cast<u32x4_t*>(out + ((2 * which) * DTILES + tri) * 512 + lane * 8) = hi;
+    *reinterpret_cast<u32x4_t*>(out + ((2 * which + 1) * DTILES + tri) * 512 + lane * 8) = lo;
+  };
+  __syncthreads();
+  emit(wave, 1);
+  if (wave < 2) emit(4 + wave, 1);
   __syncthreads();
   {
+#pragma unroll
+    for (int jt = 1; jt < 4; ++jt)
+      if (jt > wave)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) mT[(wave * 16 + 4 * g + r) * DTL + jt * 16 + c] = 0.f;
     // diagonal block of T, one column per lane (the four lane groups agree)
     const float* A = mA + wave * 16 * DTL + wave * 16;
     float x[16];
@@ -347,26 +371,8 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs a, const int*
     }
     __syncthreads();
   }
-  bf16_t* const out = mats + ((long)chunk * a.H + h) * DMATS;
-#pragma unroll
-  for (int i = 0; i < 3; ++i) {
-    const int f = wave + 4 * i, tri = f % DTILES, isb = f / DTILES;
-    const int it = tri < 2 ? tri : tri < 4 ? 2 : 3, ks = tri < 2 ? 0 : tri & 1;
-    const float* src = (isb ? mB : mT) + (16 * it + c) * DTL + 32 * ks + 4 * g;
-    const f32x4_t x0 = *reinterpret_cast<const f32x4_t*>(src);
-    const f32x4_t x1 = *reinterpret_cast<const f32x4_t*>(src + 16);
-    u32x4_t hi, lo;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const f32x4_t& x = e < 2 ? x0 : x1;
-      uint32_t p, r;
-      split2(x[2 * (e & 1)], x[2 * (e & 1) + 1], p, r);
-      hi[e] = p;
-      lo[e] = r;
-    }
-    *reinterpret_cast<u32x4_t*>(out + ((2 * isb) * DTILES + tri) * 512 + lane * 8) = hi;
-    *reinterpret_cast<u32x4_t*>(out + ((2 * isb + 1) * DTILES + tri) * 512 + lane * 8) = lo;
-  }
+  emit(wave, 0);
+  if (wave < 2) emit(4 + wave, 0);
   if (tid < DC) {
     float* w = vecs + ((long)chunk * a.H + h) * DVECS;
     const float e = fast_exp2(cum[tid]);
@@ -460,34 +466,47 @@ __global__ void __launch_bounds__(64 * W, W == 8 ? 2 : 1) delta_chunk_kernel(
   u32x4_t rq[QI], ri[NI][4], rm[MI];
   float rw[2];
   const u32x4_t zero4 = {0, 0, 0, 0};
-  auto fetch = [&](int t0) {
-    const int left = n - t0;
+  // per-thread byte offsets from wave-uniform bases (a chunk is far below 4 GB);
+  // row numbers beyond every chunk where there is nothing to load
+  static_assert(NT % NP == 0, "a q pass is whole rows");
+  constexpr int QR = NT / NP;
+  const int qc = 8 * (tid % NP), qrow = qc < N ? tid / NP : 1 << 20;
+  const uint32_t qoff = (uint32_t)((tid / NP * a.q_ld + qc) * 2);
+  uint32_t ioff[NI];
+  int irow[NI];
 #pragma unroll
-    for (int i = 0; i < QI; ++i) {
-      const int it = tid + NT * i, row = it / NP, ch = 8 * (it % NP);
-      rq[i] = row < left && row < DC && ch < N
-                  ? *reinterpret_cast<const u32x4_t*>(q + (long)(t0 + row) * a.q_ld + ch) : zero4;
-    }
+  for (int i = 0; i < NI; ++i) {
+    const int it = tid + NT * i;
+    const bool isk = wave * 64 + NT * i < KITEMS;          // wave-uniform
+    const int x = isk ? it : it - KITEMS, np = isk ? NP : VT / 8;
+    const int ch = 8 * (x % np) + (isk ? 0 : v0), r0 = 4 * (x / np);
+    irow[i] = it < ITEMS && ch < (isk ? N : P) ? r0 : 1 << 20;
+    ioff[i] = (uint32_t)((r0 * (isk ? a.k_ld : a.v_ld) + ch) * 2);
+  }
+  auto at = [](const void* base, uint32_t off) {
+    return reinterpret_cast<const u32x4_t*>(reinterpret_cast<const char*>(base) + off);
+  };
+  auto fetch = [&](int t0) {
+    const int left = min(n - t0, DC);
+#pragma unroll
+    for (int i = 0; i < QI; ++i)
+      rq[i] = qrow + QR * i < left ? *at(q + (long)(t0 + QR * i) * a.q_ld, qoff) : zero4;
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      const int it = tid + NT * i;
-      const bool isk = wave * 64 + NT * i < KITEMS;        // wave-uniform
-      const int x = isk ? it : it - KITEMS, np = isk ? NP : VT / 8;
-      const int ch = 8 * (x % np) + (isk ? 0 : v0), r0 = 4 * (x / np);
-      const bool on = it < ITEMS && ch < (isk ? N : P);
+      const bool isk = wave * 64 + NT * i < KITEMS;
       const long ld = isk ? a.k_ld : a.v_ld;
-      const bf16_t* base = (isk ? k : v) + (long)(t0 + r0) * ld + ch;
+      const bf16_t* base = (isk ? k : v) + t0 * ld;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        ri[i][r] = on && r0 + r < left ? *reinterpret_cast<const u32x4_t*>(base + r * ld) : zero4;
+        ri[i][r] = irow[i] + r < left ? *at(base + r * ld, ioff[i]) : zero4;
     }
-    const long at = (long)(t0 / DC) * a.H;
+    const bf16_t* mb = mats + (long)(t0 / DC) * a.H * DMATS;
+    const float* vb = vecs + (long)(t0 / DC) * a.H * DVECS;
 #pragma unroll
-    for (int i = 0; i < MI; ++i)
-      rm[i] = *reinterpret_cast<const u32x4_t*>(mats + at * DMATS + (tid + NT * i) * 8);
+    for (int i = 0; i < MI; ++i) rm[i] = *at(mb + NT * i * 8, tid * 16u);
 #pragma unroll
     for (int i = 0; i < 2; ++i)
-      rw[i] = tid + NT * i < DVECS ? vecs[at * DVECS + tid + NT * i] : 0.f;
+      rw[i] = tid + NT * i < DVECS ? vb[tid + NT * i] : 0.f;
   };
   auto stage = [&]() {
 #pragma unroll
@@ -525,9 +544,6 @@ __global__ void __launch_bounds__(64 * W, W == 8 ? 2 : 1) delta_chunk_kernel(
     for (int i = 0; i < 2; ++i)
       if (tid + NT * i < DVECS) sW[tid + NT * i] = rw[i];
   };
-  auto mat = [&](int which, int it, int ks) {
-    return load_frag16B(sM + (which * DTILES + tri_tile(it, ks)) * 512 + lane * 8);
-  };
   const f32x4_t z4 = {0.f, 0.f, 0.f, 0.f};
 
   if (n > 0) fetch(0);
@@ -547,18 +563,23 @@ __global__ void __launch_bounds__(64 * W, W == 8 ? 2 : 1) delta_chunk_kernel(
       bf16x8_t sh[NV], sl[NV];
 #pragma unroll
       for (int ct = 0; ct < NV; ++ct) split_tiles(S[ct][2 * ks], S[ct][2 * ks + 1], sh[ct], sl[ct]);
+      bf16x8_t kf[4], qf[4];
 #pragma unroll
       for (int it = 0; it < 4; ++it) {
-        const bf16x8_t kf = load_frag16B(sK + (it * 16 + c) * LQ + 32 * ks + 8 * g);
-        const bf16x8_t qf = load_frag16B(sQ + (it * 16 + c) * LQ + 32 * ks + 8 * g);
-#pragma unroll
-        for (int ct = 0; ct < NV; ++ct) {
-          x[ct][it] = mfma16(kf, sh[ct], x[ct][it]);
-          x[ct][it] = mfma16(kf, sl[ct], x[ct][it]);
-          o[ct][it] = mfma16(sh[ct], qf, o[ct][it]);
-          o[ct][it] = mfma16(sl[ct], qf, o[ct][it]);
-        }
+        kf[it] = load_frag16B(sK + (it * 16 + c) * LQ + 32 * ks + 8 * g);
+        qf[it] = load_frag16B(sQ + (it * 16 + c) * LQ + 32 * ks + 8 * g);
       }
+      // accumulators in turn: products of one do not follow each other
+#pragma unroll
+      for (int half = 0; half < 2; ++half)
+#pragma unroll
+        for (int ct = 0; ct < NV; ++ct)
+#pragma unroll
+          for (int it = 0; it < 4; ++it) {
+            const bf16x8_t sf = half ? sl[ct] : sh[ct];
+            x[ct][it] = mfma16(kf[it], sf, x[ct][it]);
+            o[ct][it] = mfma16(sf, qf[it], o[ct][it]);
+          }
     }
     __builtin_amdgcn_sched_barrier(0);
     // ---- beta (v - c K S), then U = T of it ----
@@ -581,20 +602,29 @@ __global__ void __launch_bounds__(64 * W, W == 8 ? 2 : 1) delta_chunk_kernel(
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) split_tiles(x[ct][2 * ks], x[ct][2 * ks + 1], rh[ct][ks], rl[ct][ks]);
     }
+    bf16x8_t mh[4], ml[4];
+    auto load_mat = [&](int which, int ks) {
 #pragma unroll
-    for (int it = 0; it < 4; ++it) {
-#pragma unroll
-      for (int ct = 0; ct < NV; ++ct) x[ct][it] = z4;
-#pragma unroll
-      for (int ks = 0; ks <= it / 2; ++ks) {
-        const bf16x8_t th = mat(0, it, ks), tl = mat(1, it, ks);
-#pragma unroll
-        for (int ct = 0; ct < NV; ++ct) {
-          x[ct][it] = mfma16(th, rh[ct][ks], x[ct][it]);
-          x[ct][it] = mfma16(th, rl[ct][ks], x[ct][it]);
-          x[ct][it] = mfma16(tl, rh[ct][ks], x[ct][it]);
-        }
+      for (int it = 2 * ks; it < 4; ++it) {
+        const int f = tri_tile(it, ks);
+        mh[it] = load_frag16B(sM + (which * DTILES + f) * 512 + lane * 8);
+        ml[it] = load_frag16B(sM + ((which + 1) * DTILES + f) * 512 + lane * 8);
       }
+    };
+#pragma unroll
+    for (int ct = 0; ct < NV; ++ct)
+#pragma unroll
+      for (int it = 0; it < 4; ++it) x[ct][it] = z4;
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+      load_mat(0, ks);
+#pragma unroll
+      for (int e = 0; e < 3; ++e)
+#pragma unroll
+        for (int ct = 0; ct < NV; ++ct)
+#pragma unroll
+          for (int it = 2 * ks; it < 4; ++it)
+            x[ct][it] = mfma16(e == 2 ? ml[it] : mh[it], e == 1 ? rl[ct][ks] : rh[ct][ks], x[ct][it]);
     }
     __builtin_amdgcn_sched_barrier(0);
     // ---- outputs (transposed) and c_end / c U ----
@@ -604,20 +634,24 @@ __global__ void __launch_bounds__(64 * W, W == 8 ? 2 : 1) delta_chunk_kernel(
       for (int ks = 0; ks < 2; ++ks) split_tiles(x[ct][2 * ks], x[ct][2 * ks + 1], rh[ct][ks], rl[ct][ks]);
 #pragma unroll
     for (int it = 0; it < 4; ++it) {
-      const int i = it * 16 + c;
-      const float cq = sW[i];
+      const float cq = sW[it * 16 + c];
 #pragma unroll
       for (int ct = 0; ct < NV; ++ct) o[ct][it] *= cq;
+    }
 #pragma unroll
-      for (int ks = 0; ks <= it / 2; ++ks) {
-        const bf16x8_t bh = mat(2, it, ks), bl = mat(3, it, ks);
+    for (int ks = 0; ks < 2; ++ks) {
+      load_mat(2, ks);
 #pragma unroll
-        for (int ct = 0; ct < NV; ++ct) {
-          o[ct][it] = mfma16(rh[ct][ks], bh, o[ct][it]);
-          o[ct][it] = mfma16(rl[ct][ks], bh, o[ct][it]);
-          o[ct][it] = mfma16(rh[ct][ks], bl, o[ct][it]);
-        }
-      }
+      for (int e = 0; e < 3; ++e)
+#pragma unroll
+        for (int ct = 0; ct < NV; ++ct)
+#pragma unroll
+          for (int it = 2 * ks; it < 4; ++it)
+            o[ct][it] = mfma16(e == 1 ? rl[ct][ks] : rh[ct][ks], e == 2 ? ml[it] : mh[it], o[ct][it]);
+    }
+#pragma unroll
+    for (int it = 0; it < 4; ++it) {
+      const int i = it * 16 + c;
       if (t0 + i < n) {
 #pragma unroll
         for (int ct = 0; ct < NV; ++ct) {
@@ -642,19 +676,28 @@ __global__ void __launch_bounds__(64 * W, W == 8 ? 2 : 1) delta_chunk_kernel(
     }
     const float et = sW[4 * DC];
 #pragma unroll
-    for (int t = 0; t < 2 * NK; ++t) {
+    for (int tb = 0; tb < 2 * NK; tb += 4 < 2 * NK ? 4 : 2 * NK) {
+      constexpr int TB = 4 < 2 * NK ? 4 : 2 * NK;
+      __builtin_amdgcn_sched_barrier(0);
+      bf16x8_t kf[TB][2];
 #pragma unroll
-      for (int ct = 0; ct < NV; ++ct) S[ct][t] *= et;
+      for (int t = 0; t < TB; ++t)
 #pragma unroll
-      for (int ks = 0; ks < 2; ++ks) {
-        const int row = 32 * (t >> 1) + 8 * (c >> 2) + 4 * (t & 1) + (c & 3);
-        const bf16x8_t kf = load_frag16B(sKT + row * DC + 8 * ((4 * ks + g) ^ tr_swz(row)));
-#pragma unroll
-        for (int ct = 0; ct < NV; ++ct) {
-          S[ct][t] = mfma16(kf, rh[ct][ks], S[ct][t]);
-          S[ct][t] = mfma16(kf, rl[ct][ks], S[ct][t]);
+        for (int ks = 0; ks < 2; ++ks) {
+          const int row = 32 * ((tb + t) >> 1) + 8 * (c >> 2) + 4 * (t & 1) + (c & 3);
+          kf[t][ks] = load_frag16B(sKT + row * DC + 8 * ((4 * ks + g) ^ tr_swz(row)));
         }
-      }
+#pragma unroll
+      for (int ct = 0; ct < NV; ++ct)
+#pragma unroll
+        for (int t = 0; t < TB; ++t) S[ct][tb + t] *= et;
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int ct = 0; ct < NV; ++ct)
+#pragma unroll
+          for (int t = 0; t < TB; ++t)
+            S[ct][tb + t] = mfma16(kf[t][e >> 1], e & 1 ? rl[ct][e >> 1] : rh[ct][e >> 1], S[ct][tb + t]);
     }
     lds_barrier();                             // the next chunk overwrites the images
   }
@@ -664,7 +707,7 @@ __global__ void __launch_bounds__(64 * W, W == 8 ? 2 : 1) delta_chunk_kernel(
 template <int NK>
 static int launch_prep(const DeltaArgs& a, const int* chunks, int nchunks, bf16_t* mats, float* vecs,
                        hipStream_t stream) {
-  constexpr int smem = std::max(2 * DC * (32 * NK + 8) * 2, 3 * DC * DTL * 4);
+  constexpr int smem = std::max(2 * DC * (32 * NK + 8) * 2, 2 * DC * DTL * 4);
   static_assert(smem <= 128 * 1024, "images fit the LDS");
   static bool attr = false;
   if (smem > 65536 && !attr) {
@@ -698,7 +741,9 @@ static int delta_pair(const DeltaArgs& a, int seq0, int nseq, const int* chunks,
                       const int* first, bf16_t* mats, float* vecs, hipStream_t stream) {
   const int rc = launch_prep<NK>(a, chunks, nchunks, mats, vecs, stream);
   if (rc) return rc;
-  if (a.P > 64) return launch_delta<NK, 1, 8>(a, seq0, nseq, first, mats, vecs, stream);
+  // 128 columns per workgroup once they fill the chip, 64 (shorter steps) below
+  if ((long)nseq * a.H * ((a.P + 127) / 128) >= 192 && a.P > 64)
+    return launch_delta<NK, 1, 8>(a, seq0, nseq, first, mats, vecs, stream);
   return launch_delta<NK, 1, 4>(a, seq0, nseq, first, mats, vecs, stream);
 }
 
