@@ -343,7 +343,7 @@ def main(argv=None):
             p.add_argument("--weights", default=os.environ.get("LMX_WEIGHTS", ""),
                            help="safetensors dir of the chat model's real weights")
             p.add_argument("--dtype", default="bfloat16", choices=("bfloat16", "float32"),
-                           help="float32: families that run in it (zegopel, pikesun, refolix)")
+                           help="float32: families that run in it (zegopel, pikesun, refolix, zovozen)")
             p.add_argument("--max-num-seqs", type=int,
                            default=int(os.environ.get("LMX_MAX_BATCH", "256")))
             p.add_argument("--registry", default=os.environ.get("LMX_MODEL_REGISTRY", ""),

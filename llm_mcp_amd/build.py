@@ -31,7 +31,7 @@ EXT = sysconfig.get_config_var("EXT_SUFFIX") or ".so"
 KERNEL_SOURCES = ["norm.hip", "rope_cache.hip", "attention.hip", "sampling.hip",
                   "elementwise.hip", "gemm.hip", "dgemm.hip", "pgemm.hip",
                   "rsgemm.hip", "allreduce.hip", "conv.hip", "linscan.hip",
-                  "grouped.hip", "moe.hip", "rglru.hip", "latent.hip", "delta.hip"]
+                  "grouped.hip", "moe.hip", "rglru.hip", "latent.hip", "delta.hip", "talk.hip"]
 RUNTIME_SOURCES = ["job_queue.cpp", "block_manager.cpp", "scheduler.cpp", "bindings.cpp"]
 
 

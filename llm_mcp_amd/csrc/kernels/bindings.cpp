@@ -38,7 +38,7 @@ int attention_any(const void*, long, const void*, const void*, const int*, int, 
                   const int*, int, void*, long, const void*, long, int, int, int, int, float, int,
                   float, int, hipStream_t);
 int sandwich_norm(void*, float*, const void*, long, int, long, const int*, const float*, int,
-                  const int*, const void*, float, const float*, const float*, const long*, int, int,
+                  const float*, const float*, const int*, const void*, float, const float*, const float*, const long*, int, int,
                   float, int, hipStream_t);
 int sum_norm(void*, float*, const void*, long, int, long, const int*, const float*, int,
              const void*, long, int, long, const float*, const float*, float, const float*,
@@ -59,7 +59,24 @@ int grouped(const void*, long, long, const void*, void*, long, long, int, int, i
 int pgemm_grouped(void*, const void*, const void*, int, int, int, long, long, int, const int*, int,
                   const int*, const int*, const float*, float, float, hipStream_t);
 int moe_route(const void*, long, const void*, int, int, int, int, int, int, const float*, int, int,
-              int*, float*, int, hipStream_t);
+              int, int, int*, float*, float*, int, hipStream_t);
+int bias_relu2(void*, const float*, long, int, int, hipStream_t);
+int qkv_norm_rope_cache(const void*, long, const float*, const float*, const float*, const float*, int,
+                        const int*, const int*, int, void*, void*, void*, int, int, int, int, int, int,
+                        float, int, hipStream_t);
+int talk_prefill(const void*, const void*, const void*, const void*, const float*, float, int, int, int,
+                 int, const int*, int, const int*, const int*, const int*, int, const void*, long,
+                 void*, long, hipStream_t);
+int talk_decode(const void*, const void*, const void*, const void*, const float*, float, int, int, int,
+                int, const int*, int, const int*, int, const void*, long, void*, long, float*, float*,
+                int, int, hipStream_t);
+int talk_any(const void*, const void*, const void*, const int*, int, const int*, int, const int*, int,
+             const void*, const float*, void*, long, const void*, long, float, int, int, int, int, int,
+             hipStream_t);
+int memory_scan(const void*, long, const void*, long, const void*, long, const void*, const void*, long,
+                const float*, float, void*, long, float*, float*, float*, const int*, const int*,
+                const int*, int, int, int, int, int, int, const int*, int, const int*, int, float*,
+                float*, hipStream_t);
 int moe_plan(const int*, int, int, int, int, int, int*, int*, int*, int*, int*, hipStream_t);
 int rglru_chunks(const void*, const void*, long, const float*, const float*, const float*, void*,
                  float*, const int*, const int*, const int*, int, int, const void*, int, const int*,
@@ -233,12 +250,12 @@ PYBIND11_MODULE(_lmx_kernels, m) {
   });
   // ---- sandwich / gated norms (norm.hip) ----
   m.def("sandwich_norm", [](uptr out, uptr residual, uptr y, long y_ld, int slabs,
-                            long slab_stride, uptr mix_pos, uptr mix_w, int mix_n, uptr ids,
-                            uptr table, float scale, uptr w_post, uptr w_pre, uptr rows_idx, int rows, int cols, float eps, int is_bf16,
+                            long slab_stride, uptr mix_pos, uptr mix_w, int mix_n, uptr own,
+                            uptr bias, uptr ids, uptr table, float scale, uptr w_post, uptr w_pre, uptr rows_idx, int rows, int cols, float eps, int is_bf16,
                             uptr stream) {
     check(lmx::sandwich_norm(P<void>(out), P<float>(residual), P<void>(y), y_ld, slabs,
-                             slab_stride, P<int>(mix_pos), P<float>(mix_w), mix_n, P<int>(ids),
-                             P<void>(table), scale, P<float>(w_post), P<float>(w_pre), P<long>(rows_idx), rows, cols, eps, is_bf16,
+                             slab_stride, P<int>(mix_pos), P<float>(mix_w), mix_n, P<float>(own),
+                             P<float>(bias), P<int>(ids), P<void>(table), scale, P<float>(w_post), P<float>(w_pre), P<long>(rows_idx), rows, cols, eps, is_bf16,
                              S(stream)),
           "sandwich_norm");
   });
@@ -316,12 +333,69 @@ PYBIND11_MODULE(_lmx_kernels, m) {
           "pgemm_grouped");
   });
   m.def("moe_route", [](uptr h, long h_ld, uptr w, int T, int d, int E, int rows, int top,
-                        int extra, uptr correction, int groups, int keep, uptr ids, uptr wts,
-                        int is_bf16, uptr stream) {
+                        int extra, uptr correction, int groups, int keep, int softmax, int identity,
+                        uptr ids, uptr wts, uptr own, int is_bf16, uptr stream) {
     check(lmx::moe_route(P<void>(h), h_ld, P<void>(w), T, d, E, rows, top, extra,
-                         P<float>(correction), groups, keep, P<int>(ids), P<float>(wts), is_bf16,
-                         S(stream)),
+                         P<float>(correction), groups, keep, softmax, identity, P<int>(ids),
+                         P<float>(wts), P<float>(own), is_bf16, S(stream)),
           "moe_route");
+  });
+  m.def("bias_relu2", [](uptr x, uptr bias, long rows, int cols, int is_bf16, uptr stream) {
+    check(lmx::bias_relu2(P<void>(x), P<float>(bias), rows, cols, is_bf16, S(stream)), "bias_relu2");
+  });
+  // ---- K22 talking heads (talk.hip) ----
+  m.def("qkv_norm_rope_cache", [](uptr p, long p_ld, uptr bias, uptr q_norm, uptr k_norm, uptr ang,
+                                  int n, uptr slots, uptr quads, int groups, uptr q, uptr kc, uptr vc,
+                                  int Hq, int Hkv, int D, int dk, int dv, int BS, float eps,
+                                  int is_bf16, uptr stream) {
+    check(lmx::qkv_norm_rope_cache(P<void>(p), p_ld, P<float>(bias), P<float>(q_norm),
+                                   P<float>(k_norm), P<float>(ang), n, P<int>(slots), P<int>(quads),
+                                   groups, P<void>(q), P<void>(kc), P<void>(vc), Hq, Hkv, D, dk, dv,
+                                   BS, eps, is_bf16, S(stream)),
+          "qkv_norm_rope_cache");
+  });
+  m.def("talk_prefill", [](uptr q, uptr kc, uptr vc, uptr mix, uptr sink, float out_scale, int Hq,
+                           int Hkv, int D, int chunk, uptr bt, int bt_stride, uptr cu_q, uptr ctx,
+                           uptr tiles, int n, uptr gate, long gate_ld, uptr out, long out_ld,
+                           uptr stream) {
+    check(lmx::talk_prefill(P<void>(q), P<void>(kc), P<void>(vc), P<void>(mix), P<float>(sink),
+                            out_scale, Hq, Hkv, D, chunk, P<int>(bt), bt_stride, P<int>(cu_q),
+                            P<int>(ctx), P<int>(tiles), n, P<void>(gate), gate_ld, P<void>(out),
+                            out_ld, S(stream)),
+          "talk_prefill");
+  });
+  m.def("talk_decode", [](uptr q, uptr kc, uptr vc, uptr mix, uptr sink, float out_scale, int Hq,
+                          int Hkv, int D, int chunk, uptr bt, int bt_stride, uptr ctx, int rows,
+                          uptr gate, long gate_ld, uptr out, long out_ld, uptr part_o, uptr part_ml,
+                          int part_tokens, int max_parts, uptr stream) {
+    check(lmx::talk_decode(P<void>(q), P<void>(kc), P<void>(vc), P<void>(mix), P<float>(sink),
+                           out_scale, Hq, Hkv, D, chunk, P<int>(bt), bt_stride, P<int>(ctx), rows,
+                           P<void>(gate), gate_ld, P<void>(out), out_ld, P<float>(part_o),
+                           P<float>(part_ml), part_tokens, max_parts, S(stream)),
+          "talk_decode");
+  });
+  m.def("talk_any", [](uptr q, uptr kc, uptr vc, uptr bt, int bt_stride, uptr cu_q, int nseq,
+                       uptr positions, int rows, uptr mix, uptr sink, uptr out, long out_ld, uptr gate,
+                       long gate_ld, float out_scale, int Hq, int Hkv, int D, int chunk, int is_bf16,
+                       uptr stream) {
+    check(lmx::talk_any(P<void>(q), P<void>(kc), P<void>(vc), P<int>(bt), bt_stride, P<int>(cu_q),
+                        nseq, P<int>(positions), rows, P<void>(mix), P<float>(sink), P<void>(out),
+                        out_ld, P<void>(gate), gate_ld, out_scale, Hq, Hkv, D, chunk, is_bf16,
+                        S(stream)),
+          "talk_any");
+  });
+  // ---- K15 matrix memory (linscan.hip) ----
+  m.def("memory_scan", [](uptr q, long q_ld, uptr k, long k_ld, uptr v, long v_ld, uptr ig, uptr fg,
+                          long gate_ld, uptr gate_bias, float cap, uptr out, long out_ld, uptr state,
+                          uptr sn, uptr sm, uptr cu_q, uptr ctx, uptr slots, int H, int N, int Pd,
+                          int is_bf16, int seq0, int nseq, uptr segs, int nseg, uptr first,
+                          int one_pass, uptr ws, uptr ws_n, uptr stream) {
+    check(lmx::memory_scan(P<void>(q), q_ld, P<void>(k), k_ld, P<void>(v), v_ld, P<void>(ig),
+                           P<void>(fg), gate_ld, P<float>(gate_bias), cap, P<void>(out), out_ld,
+                           P<float>(state), P<float>(sn), P<float>(sm), P<int>(cu_q), P<int>(ctx),
+                           P<int>(slots), H, N, Pd, is_bf16, seq0, nseq, P<int>(segs), nseg,
+                           P<int>(first), one_pass, P<float>(ws), P<float>(ws_n), S(stream)),
+          "memory_scan");
   });
   m.def("moe_plan", [](uptr ids, int n, int J, int groups, int bm, int mtiles, uptr hist, uptr off,
                        uptr src, uptr pos, uptr tiles, uptr stream) {

@@ -84,6 +84,36 @@ int gelu(void* x, long n, int is_bf16, hipStream_t stream) {
   return (int)hipGetLastError();
 }
 
+// x = relu(x + bias)^2 in place, 8 elements per thread
+template <typename T>
+__global__ void __launch_bounds__(256) bias_relu2_kernel(T* __restrict__ x,
+                                                         const float* __restrict__ bias, long n8,
+                                                         int per_row) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= n8) return;
+  float v[8], b[8];
+  ldv<8>(v, x + 8 * i);
+  ldv<8>(b, bias + 8 * (i % per_row));
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const float z = fmaxf(v[j] + b[j], 0.f);
+    v[j] = z * z;
+  }
+  stv<8>(x + 8 * i, v);
+}
+
+int bias_relu2(void* x, const float* bias, long rows, int cols, int is_bf16, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  const long n8 = rows * (cols / 8);
+  if (cols <= 0 || cols % 8 != 0 || (n8 + 255) / 256 > 0x7fffffffL) return -1;
+  const dim3 grid((unsigned)((n8 + 255) / 256));
+  if (is_bf16)
+    bias_relu2_kernel<bf16_t><<<grid, dim3(256), 0, stream>>>((bf16_t*)x, bias, n8, cols / 8);
+  else
+    bias_relu2_kernel<float><<<grid, dim3(256), 0, stream>>>((float*)x, bias, n8, cols / 8);
+  return (int)hipGetLastError();
+}
+
 __global__ void __launch_bounds__(256) embed_gather_kernel(bf16_t* __restrict__ out,
                                                            const bf16_t* __restrict__ table,
                                                            const int* __restrict__ ids, int d,

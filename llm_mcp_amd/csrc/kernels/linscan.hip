@@ -11,7 +11,14 @@
 //     s_t), D the skip weight;
 //   * retention: linear attention whose q and k are rotated by their position
 //     (neighbouring channels a pair) and k scaled: the recurrent form turns them
-//     as it loads them, the chunked one runs on rows turned in place before.
+//     as it loads them, the chunked one runs on rows turned in place before;
+//   * matrix memory (MEM): exponential input gates i and forget gates f (both as
+//     logarithms) under a running maximum m that starts at 0,
+//         m_t = max(f_t + m_{t-1}, i_t),  a_t = e^(f_t + m_{t-1} - m_t),
+//         s_t = e^(i_t - m_t),  n_t = a_t n_{t-1} + s_t k_t,
+//         o_t = S_t^T q_t / (max(|n_t q_t|, e^-m_t) + 1e-6);
+//     with F the prefix sum of f, m_t - F_t is a running maximum of i_j - F_j, so
+//     a chunk's weights e^(F_t - m_t - (F_j - i_j)) come from two vectors.
 // The state of a sequence lives in its slot of state[slots][H][N][P] between
 // steps; a row range that starts at position 0 starts from the zero state
 // whatever the slot holds, so slots are reused uncleared.
@@ -58,7 +65,23 @@ struct ScanArgs {
   const float* ang;          // [rows][nrot] cos | sin (recurrent form), or null
   int nrot;
   float k_scale;
+  // matrix memory
+  const void *ig, *fg;       // T rows [.., H]: gate projections
+  long gate_ld;
+  const float* gate_bias;    // [2][H]
+  float cap, q_scale;
+  float *sn, *sm;            // [slots][H][N], [slots][H]
 };
+
+// logarithms of the gates: cap tanh((x + b) / cap), and ln sigmoid of such a value
+template <typename T>
+__device__ __forceinline__ void memory_gates(const ScanArgs& a, long row, int h, float& i, float& f) {
+  const float x = ld1((const T*)a.ig + row * a.gate_ld + h) + a.gate_bias[h];
+  const float y = ld1((const T*)a.fg + row * a.gate_ld + h) + a.gate_bias[a.H + h];
+  i = a.cap * tanhf(x / a.cap);
+  const float z = a.cap * tanhf(y / a.cap);
+  f = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+}
 
 // ------------------------------------------------------------- recurrent ----
 // grid (sequences, H, P tiles of `pt` columns), block 256 = (pt / VEC) column
@@ -201,6 +224,152 @@ int scan_recurrent(const ScanArgs& a, int is_bf16, int seq0, int nseq, hipStream
   return (int)hipGetLastError();
 }
 
+// Matrix memory, token after token: one workgroup of BT threads per (sequence,
+// head), since its columns share n and m; the columns in tiles of `pt`, each
+// walking the tokens from the same n and m.  grid (sequences, H), layout of a tile
+// as above.
+template <typename T, int VEC, int RPT, int BT>
+__global__ void __launch_bounds__(BT) memory_recurrent_kernel(ScanArgs a, int seq0, int pt) {
+  extern __shared__ float scan_sm[];
+  __shared__ float scratch[16];
+  const int seq = seq0 + blockIdx.x, h = blockIdx.y;
+  const int slot = a.slots[seq];
+  if (slot < 0) return;                       // padding row of a captured step
+  const int N = a.N, P = a.P, tid = threadIdx.x;
+  const int ncol = pt / VEC, kr = BT / ncol;
+  const int c = tid % ncol, r = tid / ncol;
+  const bool live = r < kr;
+  float* sq = scan_sm;                        // [N]
+  float* sk = sq + N;                         // [N]
+  float* sn = sk + N;                         // [N]
+  float* sv = sn + N;                         // [pt]
+  float* red = sv + pt;                       // [kr][pt]
+  const int row0 = a.cu_q[seq], n = a.cu_q[seq + 1] - row0;
+  const bool fresh = a.ctx[seq] == n;
+  const long head = (long)slot * a.H + h;
+  const float m0 = fresh ? 0.f : a.sm[head];
+  const T* q = (const T*)a.q + (long)row0 * a.q_ld + (long)h * N;
+  const T* k = (const T*)a.k + (long)row0 * a.k_ld + (long)h * N;
+  const T* v = (const T*)a.v + (long)row0 * a.v_ld + (long)h * P;
+  T* out = (T*)a.out + (long)row0 * a.out_ld + (long)h * P;
+  float m = m0;
+  for (int p0 = 0; p0 < P; p0 += pt) {
+    const int pc = p0 + c * VEC;
+    float* st = a.state + head * N * P + pc;
+    float S[RPT][VEC];
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+      const int kk = r + i * kr;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) S[i][e] = 0.f;
+      if (live && !fresh && kk < N && pc < P) {
+        if constexpr (VEC == 4) {
+          const f32x4_t t = __builtin_nontemporal_load(reinterpret_cast<const f32x4_t*>(st + (long)kk * P));
+          S[i][0] = t[0]; S[i][1] = t[1]; S[i][2] = t[2]; S[i][3] = t[3];
+        } else {
+          S[i][0] = st[(long)kk * P];
+        }
+      }
+    }
+    // a thread's entries of n stay its own until the last tile stores them
+    for (int i = tid; i < N; i += BT) sn[i] = fresh ? 0.f : a.sn[head * N + i];
+    m = m0;
+    for (int t = 0; t < n; ++t) {
+      float ig, f;
+      memory_gates<T>(a, row0 + t, h, ig, f);
+      const float mn = fmaxf(f + m, ig), keep = expf(f + m - mn), add = expf(ig - mn);
+      m = mn;
+      float dot = 0.f;
+      for (int i = tid; i < N; i += BT) {
+        const float qv = ld1(q + t * a.q_ld + i) * a.q_scale, kv = ld1(k + t * a.k_ld + i);
+        const float x = keep * sn[i] + add * kv;
+        sq[i] = qv;
+        sk[i] = kv;
+        sn[i] = x;
+        dot += x * qv;
+      }
+      for (int i = tid; i < pt; i += BT) sv[i] = p0 + i < P ? ld1(v + t * a.v_ld + p0 + i) : 0.f;
+      dot = block_sum(dot, scratch);          // (and a barrier)
+      if (live) {
+        float vs[VEC], o[VEC];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) { vs[e] = sv[c * VEC + e] * add; o[e] = 0.f; }
+#pragma unroll
+        for (int i = 0; i < RPT; ++i) {
+          const int kk = r + i * kr;
+          if (kk < N) {
+            const float kv = sk[kk], qv = sq[kk];
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) {
+              S[i][e] = keep * S[i][e] + kv * vs[e];
+              o[e] += qv * S[i][e];
+            }
+          }
+        }
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) red[r * pt + c * VEC + e] = o[e];
+      }
+      __syncthreads();
+      const float inv = 1.f / (fmaxf(fabsf(dot), expf(-m)) + 1e-6f);
+      for (int i = tid; i < pt; i += BT) {
+        if (p0 + i < P) {
+          float o = 0.f;
+          for (int j = 0; j < kr; ++j) o += red[j * pt + i];
+          st1(out + t * a.out_ld + p0 + i, o * inv);
+        }
+      }
+      __syncthreads();
+    }
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+      const int kk = r + i * kr;
+      if (live && kk < N && pc < P) {
+        if constexpr (VEC == 4) {
+          const f32x4_t t = {S[i][0], S[i][1], S[i][2], S[i][3]};
+          __builtin_nontemporal_store(t, reinterpret_cast<f32x4_t*>(st + (long)kk * P));
+        } else {
+          st[(long)kk * P] = S[i][0];
+        }
+      }
+    }
+  }
+  for (int i = tid; i < N; i += BT) a.sn[head * N + i] = sn[i];
+  if (tid == 0) a.sm[head] = m;               // read by every thread before the barriers above
+}
+
+int memory_recurrent(const ScanArgs& a, int is_bf16, int seq0, int nseq, hipStream_t stream) {
+  if (nseq <= 0) return 0;
+  // 256 threads once the batch alone fills the chip, 1024 (shallower tiles) below
+  const int bt = (long)nseq * a.H >= 1024 ? 256 : 1024;
+  const int vec = a.P % 4 == 0 ? 4 : 1;
+  int pt = 16;
+  while (pt < a.P && pt < 512) pt *= 2;
+  for (;; pt /= 2) {
+    const int kr = bt / (pt / vec);
+    if (pt < 4) return -2;
+    if (kr >= 1 && (a.N + kr - 1) / kr <= 16) break;
+  }
+  const int kr = bt / (pt / vec), rpt = (a.N + kr - 1) / kr;
+  const size_t smem = (size_t)(3 * a.N + pt + kr * pt) * sizeof(float);
+  if (smem > 65536) return -3;
+  const dim3 grid(nseq, a.H);
+#define LMX_MR(TT, V, R, B) \
+  memory_recurrent_kernel<TT, V, R, B><<<grid, dim3(B), smem, stream>>>(a, seq0, pt)
+#define LMX_MRR(TT, V, B)                                                          \
+  if (rpt <= 2) LMX_MR(TT, V, 2, B); else if (rpt <= 4) LMX_MR(TT, V, 4, B);        \
+  else if (rpt <= 8) LMX_MR(TT, V, 8, B); else LMX_MR(TT, V, 16, B);
+#define LMX_MRB(TT, V) if (bt == 256) { LMX_MRR(TT, V, 256) } else { LMX_MRR(TT, V, 1024) }
+  if (is_bf16) {
+    if (vec == 4) { LMX_MRB(bf16_t, 4) } else { LMX_MRB(bf16_t, 1) }
+  } else {
+    if (vec == 4) { LMX_MRB(float, 4) } else { LMX_MRB(float, 1) }
+  }
+#undef LMX_MRB
+#undef LMX_MRR
+#undef LMX_MR
+  return (int)hipGetLastError();
+}
+
 // --------------------------------------------------------------- chunked ----
 constexpr int SC = 64;     // tokens per chunk
 constexpr int SCP = 72;    // padded row of the score images (16-B aligned)
@@ -208,6 +377,8 @@ struct SegArgs {
   const int* segs;         // [nseg][4]: sequence, first row, last row (in the sequence), last-of-sequence
   float* ws;               // [nseg][H][N][P] segment states (modes 1, 2)
   float* ws_log;           // [nseg][H] log2 of the segment's total decay (mode 1)
+  // MEM: [nseg][H][N + 3]: n, own m, total forget logarithm, start m (all log2)
+  float* ws_n;
 };
 
 __device__ __forceinline__ float silu_fast(float x) {
@@ -237,7 +408,13 @@ __device__ __forceinline__ void silu_words(u32x4_t& w) {
 // that is the operand layout of the products with q, so the state is split
 // into bf16 pairs in place, with no exchange.  Outputs are computed transposed
 // (MFMA row = v column): a lane ends up with 4 consecutive columns of a row.
-template <int NK, int NV, int MODE>
+//
+// MEM: matrix memory.  cum holds F_t - m_t and sdt F_j - i_j (log2), ecum the factor
+// e^(F_t + m_0 - m_t) of the chunk's start state; n is a vector in LDS that the
+// first waves advance, n q is taken from the query fragments and the row sums of
+// the scores.  The workgroup of the first columns writes n and m back, so where
+// there are several the sequence must not run in mode 0.
+template <int NK, int NV, int MODE, bool MEM = false>
 __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanArgs a, SegArgs sg) {
   extern __shared__ __attribute__((aligned(16))) char chunk_sm[];
   constexpr int DK = NK * 32, LQ = DK + 8, VT = 64 * NV, NP = 4 * NK;
@@ -251,6 +428,9 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
   float* const sdt = cum + SC;
   float* const ecum = sdt + SC;
   float* const wend = ecum + SC;
+  float* const sinv = wend + SC;           // MEM: 1 / divisor of a row
+  float* const emt = sinv + SC;            // MEM: e^-m_t
+  float* const nvec = emt + SC;            // MEM: n
 
   const int seg = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VT;
   const int seq = sg.segs[4 * seg], b = sg.segs[4 * seg + 1], e = sg.segs[4 * seg + 2];
@@ -270,7 +450,7 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
   const bf16_t* v = (const bf16_t*)a.v + row0 * a.v_ld + (long)h * P;
   bf16_t* out = (bf16_t*)a.out + row0 * a.out_ld + (long)h * P;
   const bf16_t* dt = a.dt ? (const bf16_t*)a.dt + row0 * a.dt_ld + h : nullptr;
-  const float logd = a.dt ? 0.f : a.log_decay[h] * SCAN_LOG2E;
+  const float logd = MEM || a.dt ? 0.f : a.log_decay[h] * SCAN_LOG2E;
   const float bias = a.dt ? a.dt_bias[h] : 0.f, na = a.dt ? a.neg_a[h] * SCAN_LOG2E : 0.f;
   const float skip = a.skip ? a.skip[h] : 0.f;
 
@@ -301,13 +481,30 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
                            : a.state + ((long)slot * a.H + h) * N * P;
     state_io(src, false, MODE == 1 || (MODE == 0 && fresh));
   }
+  // MEM: the segment's n and (wave 0) running maximum, log2
+  float* const wsn = MEM && MODE != 0 ? sg.ws_n + ((long)seg * a.H + h) * (N + 3) : nullptr;
+  float* const slot_n = MEM ? a.sn + ((long)slot * a.H + h) * N : nullptr;
+  float mrun = 0.f;
+  if constexpr (MEM) {
+    for (int i = tid; i < DK; i += 256) {
+      float x = 0.f;
+      if (i < N && MODE == 2) x = wsn[i];
+      if (i < N && MODE == 0 && !fresh) x = slot_n[i];
+      nvec[i] = x;
+    }
+    if (MODE == 1) mrun = -INFINITY;
+    if (MODE == 2) mrun = wsn[N + 2];
+    if (MODE == 0 && !fresh) mrun = a.sm[(long)slot * a.H + h] * SCAN_LOG2E;
+  }
+
+  float log_total = 0.f;
 
   // ---- staging, one chunk ahead in registers.  q: 16-B pieces of rows.  k and
   // v: items of 4 consecutive rows x 8 channels, so the transposed image is
   // written 4 tokens (8 B) at a time ----
   constexpr int KITEMS = 16 * NP, ITEMS = KITEMS + 2 * VT, NI = (ITEMS + 255) / 256;
   u32x4_t rq[MODE == 1 ? 1 : NK], ri[NI][4];
-  float rdt = 0.f;
+  float rdt = 0.f, rfg = 0.f;              // MEM: logarithms of the gates, log2
   const u32x4_t zero4 = {0, 0, 0, 0};
   // per-thread byte offsets from wave-uniform row bases (a chunk is far below 4 GB)
   static_assert(256 % NP == 0, "a q pass is whole rows");
@@ -345,7 +542,15 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
       for (int r = 0; r < 4; ++r)
         ri[i][r] = irow[i] + r < left ? *at(base + r * ld, ioff[i]) : zero4;
     }
-    if (dt && tid < SC) rdt = t0 + tid < n ? bf2f(dt[(long)(t0 + tid) * a.dt_ld]) : 0.f;
+    if constexpr (MEM) {
+      if (tid < SC && t0 + tid < n) {
+        memory_gates<bf16_t>(a, row0 + t0 + tid, h, rdt, rfg);
+        rdt *= SCAN_LOG2E;
+        rfg *= SCAN_LOG2E;
+      }
+    } else {
+      if (dt && tid < SC) rdt = t0 + tid < n ? bf2f(dt[(long)(t0 + tid) * a.dt_ld]) : 0.f;
+    }
   };
   auto stage = [&](int m) {
     if constexpr (MODE != 1) {
@@ -380,7 +585,29 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
                                     8 * (((qd >> 1) ^ tr_swz(8 * pc)) ^ (e & 3)) + e * SC) = w;
       }
     }
-    if (wave == 0) {
+    if (MEM && wave == 0) {
+      float f = lane < m ? rfg : 0.f, b = 0.f;     // rows past the end neither decay nor add
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const float y = __shfl_up(f, o, 64);
+        if (lane >= o) f += y;
+      }
+      b = lane < m ? f - rdt : INFINITY;
+      float mx = fmaxf(mrun, -b);
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const float y = __shfl_up(mx, o, 64);
+        if (lane >= o) mx = fmaxf(mx, y);
+      }
+      const float mt = f + mx, fend = __shfl(f, 63, 64), mend = __shfl(mt, 63, 64);
+      cum[lane] = f - mt;
+      sdt[lane] = b;
+      ecum[lane] = fast_exp2(f + mrun - mt);
+      wend[lane] = fast_exp2(fend - mend - b);
+      emt[lane] = fast_exp2(-mt);
+      mrun = mend;
+      log_total += fend;
+    } else if (!MEM && wave == 0) {
       // log2 decays and their prefix sum; rows past the end neither decay nor add
       float s = 1.f, la = logd;
       if (dt) { s = softplus_f(rdt + bias); la = na * s; }
@@ -407,7 +634,6 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
     ktp[z] = sKT + row * SC + 8 * (g ^ tr_swz(row) ^ (2 * z));
   }
 
-  float log_total = 0.f;
   if (n > 0) fetch(0);
   for (int t0 = 0; t0 < n; t0 += SC) {
     const int m = min(SC, n - t0);
@@ -431,10 +657,17 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
       f32x4_t sc[4];
 #pragma unroll
       for (int jt = 0; jt < 4; ++jt) sc[jt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      float nq = 0.f;                      // MEM: n q, this lane's channels
 #pragma unroll
       for (int ks = 0; ks < NK; ++ks) {
         __builtin_amdgcn_sched_barrier(0);
         const bf16x8_t qf = load_frag16B(sQ + (wave * 16 + c) * LQ + 32 * ks + 8 * g);
+        if constexpr (MEM) {
+          float nv[8];
+          ldv<8>(nv, nvec + 32 * ks + 8 * g);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) nq += nv[e] * bf2f((uint16_t)qf[e]);
+        }
 #pragma unroll
         for (int jt = 0; jt < 4; ++jt)
           if (jt <= wave)
@@ -442,6 +675,7 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
       }
       const int qi = wave * 16 + c;
       const float ci = cum[qi];
+      float rows = 0.f;                    // MEM: row sum of the scores, this lane's keys
       u32x2_t ph[4], pl[4];
 #pragma unroll
       for (int jt = 0; jt < 4; ++jt) {
@@ -454,15 +688,26 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
         asm volatile("" : "+v"(lim));
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          w[r] = 4 * g + r <= lim ? sc[jt][r] * fast_exp2(ci - cj[r]) * sj[r] : 0.f;
-          // the skip term is a score of one's own v
-          if (jt == wave) w[r] += 4 * g + r == c ? skip : 0.f;
+          if constexpr (MEM) {
+            w[r] = 4 * g + r <= lim ? sc[jt][r] * fast_exp2(ci - sj[r]) : 0.f;
+            rows += w[r];
+          } else {
+            w[r] = 4 * g + r <= lim ? sc[jt][r] * fast_exp2(ci - cj[r]) * sj[r] : 0.f;
+            // the skip term is a score of one's own v
+            if (jt == wave) w[r] += 4 * g + r == c ? skip : 0.f;
+          }
         }
         uint32_t h0, l0, h1, l1;
         split2(w[0], w[1], h0, l0);
         split2(w[2], w[3], h1, l1);
         ph[jt] = u32x2_t{h0, h1};
         pl[jt] = u32x2_t{l0, l1};
+      }
+      if constexpr (MEM) {
+        float x = rows + ecum[qi] * nq;
+        x += __shfl_xor(x, 16, 64);
+        x += __shfl_xor(x, 32, 64);
+        if (g == 0) sinv[qi] = a.q_scale / (fmaxf(fabsf(x * a.q_scale), emt[qi]) + 1e-6f);
       }
       lds_barrier();                       // every wave is done with k's rows
 #pragma unroll
@@ -525,11 +770,13 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
           }
         }
         if (i < m) {
+          const float inv = MEM ? sinv[i] : 1.f;
 #pragma unroll
           for (int ct = 0; ct < NV; ++ct) {
             const int vc = vw + 16 * ct + 4 * g;           // P % 8 == 0: whole quads
             if (vc < P) {
-              const f32x4_t& y = o[ct][it];
+              f32x4_t y = o[ct][it];
+              if constexpr (MEM) y *= inv;
               const u32x2_t yw = {pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
               *reinterpret_cast<u32x2_t*>(out + (long)(t0 + i) * a.out_ld + vc) = yw;
             }
@@ -539,7 +786,21 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
     }
     // ---- state: S <- 2^ctot S + k^T (w v) ----
     const float ctot = cum[SC - 1], et = ecum[SC - 1];
-    log_total += ctot;
+    if constexpr (!MEM) log_total += ctot;
+    if constexpr (MEM) {                   // n <- 2^.. n + k^T wend, a channel per thread
+      for (int ch = tid; ch < DK; ch += 256) {
+        float x = et * nvec[ch];
+#pragma unroll
+        for (int pc = 0; pc < 8; ++pc) {
+          float kv[8], wv[8];
+          ldv<8>(kv, sKT + ch * SC + 8 * (pc ^ tr_swz(ch)));
+          ldv<8>(wv, wend + 8 * pc);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x += kv[e] * wv[e];
+        }
+        nvec[ch] = x;
+      }
+    }
     bf16x8_t wh[NV][2], wl[NV][2];
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
@@ -583,9 +844,20 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
 
   if constexpr (MODE == 1) {
     state_io(sg.ws + ((long)seg * a.H + h) * N * P, true, false);
-    if (tid == 0 && v0 == 0) sg.ws_log[(long)seg * a.H + h] = log_total;
+    if (!MEM && tid == 0 && v0 == 0) sg.ws_log[(long)seg * a.H + h] = log_total;
   } else {
     if (MODE == 0 || last) state_io(a.state + ((long)slot * a.H + h) * N * P, true, false);
+  }
+  if constexpr (MEM) {
+    if (v0 == 0) {
+      float* const dst = MODE == 1 ? wsn : slot_n;
+      if (MODE != 2 || last)
+        for (int i = tid; i < N; i += 256) dst[i] = nvec[i];
+      if (tid == 0) {
+        if (MODE == 1) { wsn[N] = mrun; wsn[N + 1] = log_total; }
+        else if (MODE == 0 || last) a.sm[(long)slot * a.H + h] = mrun / SCAN_LOG2E;
+      }
+    }
   }
 }
 
@@ -613,6 +885,31 @@ __global__ void __launch_bounds__(256) scan_combine_kernel(ScanArgs a, SegArgs s
   }
 }
 
+// The same for matrix memories: segments chain under their running maxima.  grid
+// (sequences, H, ceil((N P + N) / 1024)).
+__global__ void __launch_bounds__(256) memory_combine_kernel(ScanArgs a, SegArgs sg, int seq0,
+                                                             const int* __restrict__ first) {
+  const int s = blockIdx.x, h = blockIdx.y, seq = seq0 + s, N = a.N;
+  const long NP = (long)N * a.P, head = (long)a.slots[seq] * a.H + h;
+  const bool fresh = a.ctx[seq] == a.cu_q[seq + 1] - a.cu_q[seq];
+  const int f0 = first[s], f1 = first[s + 1];
+  const float m0 = fresh ? 0.f : a.sm[head] * SCAN_LOG2E;
+  for (int e = 0; e < 4; ++e) {
+    const long i = (long)blockIdx.z * 1024 + e * 256 + threadIdx.x;
+    if (i >= NP + N) return;
+    float x = fresh ? 0.f : i < NP ? a.state[head * NP + i] : a.sn[head * N + i - NP], m = m0;
+    for (int f = f0; f < f1; ++f) {
+      float* const w = sg.ws_n + ((long)f * a.H + h) * (N + 3);
+      float* const p = i < NP ? sg.ws + ((long)f * a.H + h) * NP + i : w + i - NP;
+      if (i == 0) w[N + 2] = m;
+      const float own = *p, mn = fmaxf(w[N + 1] + m, w[N]);
+      *p = x;
+      x = fast_exp2(w[N + 1] + m - mn) * x + fast_exp2(w[N] - mn) * own;
+      m = mn;
+    }
+  }
+}
+
 bool scan_chunk_ok(const ScanArgs& a) {
   auto al = [](const void* p, long ld) {
     return ((uintptr_t)p & 15) == 0 && ld % 8 == 0;
@@ -621,28 +918,28 @@ bool scan_chunk_ok(const ScanArgs& a) {
          al(a.v, a.v_ld);
 }
 
-template <int NK, int NV, int MODE>
+template <int NK, int NV, int MODE, bool MEM>
 static int launch_chunk_nv(const ScanArgs& a, const SegArgs& sg, int nseg, hipStream_t stream) {
   constexpr int LQ = NK * 32 + 8;
   constexpr int KEL = SC * LQ > 2 * SC * SCP ? SC * LQ : 2 * SC * SCP;
-  constexpr int smem = ((MODE == 1 ? 0 : SC * LQ + KEL) + NK * 32 * SC + 64 * NV * SC) * 2 + 4 * SC * 4;
+  constexpr int smem = ((MODE == 1 ? 0 : SC * LQ + KEL) + NK * 32 * SC + 64 * NV * SC) * 2 + 4 * SC * 4 + (MEM ? (2 * SC + NK * 32) * 4 : 0);
   static_assert(smem <= 160 * 1024, "chunk images fit the LDS");
   static bool attr = false;
   if (smem > 65536 && !attr) {
-    (void)hipFuncSetAttribute((const void*)scan_chunk_kernel<NK, NV, MODE>,
+    (void)hipFuncSetAttribute((const void*)scan_chunk_kernel<NK, NV, MODE, MEM>,
                               hipFuncAttributeMaxDynamicSharedMemorySize, smem);
     attr = true;
   }
-  scan_chunk_kernel<NK, NV, MODE>
+  scan_chunk_kernel<NK, NV, MODE, MEM>
       <<<dim3(nseg, a.H, (a.P + 64 * NV - 1) / (64 * NV)), dim3(256), smem, stream>>>(a, sg);
   return (int)hipGetLastError();
 }
 
-template <int NK, int MODE>
+template <int NK, int MODE, bool MEM = false>
 static int launch_chunk(const ScanArgs& a, const SegArgs& sg, int nseg, hipStream_t stream) {
   if constexpr (NK <= 4)
-    if (a.P > 64) return launch_chunk_nv<NK, 2, MODE>(a, sg, nseg, stream);
-  return launch_chunk_nv<NK, 1, MODE>(a, sg, nseg, stream);
+    if (a.P > 64) return launch_chunk_nv<NK, 2, MODE, MEM>(a, sg, nseg, stream);
+  return launch_chunk_nv<NK, 1, MODE, MEM>(a, sg, nseg, stream);
 }
 
 // segs / first: see SegArgs and scan_combine_kernel.  one_pass: one segment
@@ -652,7 +949,7 @@ int scan_chunked(const ScanArgs& a, const int* segs, int nseg, const int* first,
   if (nseg <= 0) return 0;
   if (!scan_chunk_ok(a) || (a.dt == nullptr) == (a.log_decay == nullptr)) return -1;
   if (!one_pass && (!ws || !ws_log || !first)) return -2;
-  const SegArgs sg{segs, ws, ws_log};
+  const SegArgs sg{segs, ws, ws_log, nullptr};
   const int nk = (a.N + 31) / 32;
 #define LMX_CHUNK(MODE)                                                   \
   (nk <= 1 ? launch_chunk<1, MODE>(a, sg, nseg, stream)                   \
@@ -664,6 +961,32 @@ int scan_chunked(const ScanArgs& a, const int* segs, int nseg, const int* first,
   if (rc) return rc;
   const long NP = (long)a.N * a.P;
   scan_combine_kernel<<<dim3(nseq, a.H, (unsigned)((NP + 1023) / 1024)), dim3(256), 0, stream>>>(
+      a, sg, seq0, first);
+  rc = (int)hipGetLastError();
+  if (rc) return rc;
+  return LMX_CHUNK(2);
+#undef LMX_CHUNK
+}
+
+int memory_chunked(const ScanArgs& a, const int* segs, int nseg, const int* first, int seq0,
+                   int nseq, int one_pass, float* ws, float* ws_n, hipStream_t stream) {
+  if (nseg <= 0) return 0;
+  if (!scan_chunk_ok(a)) return -1;
+  // several workgroups of one head may not read and write its n and m in one pass
+  if (one_pass && a.P > (a.N <= 128 ? 128 : 64)) return -6;
+  if (!one_pass && (!ws || !ws_n || !first)) return -2;
+  const SegArgs sg{segs, ws, nullptr, ws_n};
+  const int nk = (a.N + 31) / 32;
+#define LMX_CHUNK(MODE)                                                         \
+  (nk <= 1 ? launch_chunk<1, MODE, true>(a, sg, nseg, stream)                   \
+   : nk <= 2 ? launch_chunk<2, MODE, true>(a, sg, nseg, stream)                 \
+   : nk <= 4 ? launch_chunk<4, MODE, true>(a, sg, nseg, stream)                 \
+             : launch_chunk<8, MODE, true>(a, sg, nseg, stream))
+  if (one_pass) return LMX_CHUNK(0);
+  int rc = LMX_CHUNK(1);
+  if (rc) return rc;
+  const long n = (long)a.N * a.P + a.N;
+  memory_combine_kernel<<<dim3(nseq, a.H, (unsigned)((n + 1023) / 1024)), dim3(256), 0, stream>>>(
       a, sg, seq0, first);
   rc = (int)hipGetLastError();
   if (rc) return rc;
@@ -737,13 +1060,31 @@ int linear_scan(const void* q, long q_ld, const void* k, long k_ld, const void* 
                 int nseg, const int* first, int one_pass, float* ws, float* ws_log,
                 hipStream_t stream) {
   ScanArgs a{q, k, v, q_ld, k_ld, v_ld, dt, dt_ld, dt_bias, neg_a, decay, log_decay, skip,
-             out, out_ld, state, cu_q, ctx, slots, H, N, P, hpg, act, ang, nrot, k_scale};
+             out, out_ld, state, cu_q, ctx, slots, H, N, P, hpg, act, ang, nrot, k_scale,
+             nullptr, nullptr, 0, nullptr, 1.f, 1.f, nullptr, nullptr};
   if (nrot < 0 || nrot % 2 || nrot > N || (nrot && (!ang || act))) return -5;
   if (nseg > 0) {
     if (!is_bf16) return -4;
     return scan_chunked(a, segs, nseg, first, seq0, nseq, one_pass, ws, ws_log, stream);
   }
   return scan_recurrent(a, is_bf16, seq0, nseq, stream);
+}
+
+int memory_scan(const void* q, long q_ld, const void* k, long k_ld, const void* v, long v_ld,
+                const void* ig, const void* fg, long gate_ld, const float* gate_bias, float cap,
+                void* out, long out_ld, float* state, float* sn, float* sm, const int* cu_q,
+                const int* ctx, const int* slots, int H, int N, int P, int is_bf16, int seq0,
+                int nseq, const int* segs, int nseg, const int* first, int one_pass, float* ws,
+                float* ws_n, hipStream_t stream) {
+  if (N <= 0 || P <= 0 || H <= 0 || !ig || !fg || !gate_bias || cap <= 0.f || !sn || !sm) return -1;
+  const ScanArgs a{q, k, v, q_ld, k_ld, v_ld, nullptr, 0, nullptr, nullptr, nullptr, nullptr,
+                   nullptr, out, out_ld, state, cu_q, ctx, slots, H, N, P, 1, 0, nullptr, 0, 1.f,
+                   ig, fg, gate_ld, gate_bias, cap, 1.f / sqrtf((float)N), sn, sm};
+  if (nseg > 0) {
+    if (!is_bf16) return -4;
+    return memory_chunked(a, segs, nseg, first, seq0, nseq, one_pass, ws, ws_n, stream);
+  }
+  return memory_recurrent(a, is_bf16, seq0, nseq, stream);
 }
 
 }  // namespace lmx

@@ -4,8 +4,11 @@
 //              index first among equals) and the softmax over just those; then
 //              `extra` further experts every row uses with weight 1.  Or by
 //              scores s = sigmoid(logit): the top s + correction among the best
-//              groups of neighbouring experts, in the proportions of their s;
-//              the extra ones then weigh sigmoid of one more logit.
+//              groups of neighbouring experts, in the proportions of their s; the
+//              extra ones then weigh sigmoid of one more logit.  Or by s = softmax
+//              over all logits, groups ranked by their largest score, weighted by s
+//              itself.  The last `identity` experts return their input: they are no
+//              uses (id -1), their weights are summed per row.
 //              bf16 rows, up to 128 experts: 16 rows per workgroup on MFMA, the K
 //              range split over the waves; otherwise one row per workgroup on the VALU.
 //   moe_plan   the uses (row, expert) sorted by expert: expert row ranges, the
@@ -19,26 +22,35 @@ namespace {
 constexpr int MAXE = 256, MAXTOP = 32;
 
 struct RouteBy {
-  const float* correction;   // [E]: sigmoid scores; null: softmax over the top logits
+  const float* correction;   // [E]: scores of all experts; null: softmax over the top logits
   int groups, keep;
   int rows;                  // router rows: E, or E + 1 with the extra experts' logit
+  int softmax;               // the scores are a softmax, else sigmoids
+  int identity;              // of the E
 };
 
 // One wave ranks one row's logits z[E] (LDS) and writes its uses.
 __device__ __forceinline__ void moe_select(float* z, int E, int top, int extra, const RouteBy& by,
-                                           int* ids, float* wts) {
+                                           int* ids, float* wts, float* own) {
   const int lane = threadIdx.x & 63;
   float v[MAXE / 64];
   float more = 1.f;          // weight of the extra experts
   if (by.correction) {
     // z becomes the scores, v the choice scores of the kept groups
     if (by.rows > E) more = 1.f / (1.f + expf(-z[E]));
+    float zmax = -INFINITY, zsum = 0.f;
+    if (by.softmax) {
+      for (int e = lane; e < E; e += 64) zmax = fmaxf(zmax, z[e]);
+      zmax = wave_max(zmax);
+      for (int e = lane; e < E; e += 64) zsum += expf(z[e] - zmax);
+      zsum = wave_sum(zsum);
+    }
 #pragma unroll
     for (int i = 0; i < MAXE / 64; ++i) {
       const int e = i * 64 + lane;
       v[i] = -INFINITY;
       if (e < E) {
-        const float s = 1.f / (1.f + expf(-z[e]));
+        const float s = by.softmax ? expf(z[e] - zmax) / zsum : 1.f / (1.f + expf(-z[e]));
         z[e] = s;
         v[i] = s + by.correction[e];
       }
@@ -51,7 +63,7 @@ __device__ __forceinline__ void moe_select(float* z, int E, int top, int extra, 
         const float c = z[e] + by.correction[e];
         if (c > a) { b = a; a = c; } else if (c > b) { b = c; }
       }
-    const float score = lane < by.groups ? a + (size > 1 ? b : 0.f) : -INFINITY;
+    const float score = lane < by.groups ? a + (size > 1 && !by.softmax ? b : 0.f) : -INFINITY;
     int rank = 0;
     for (int g = 0; g < by.groups; ++g) {
       const float o = __shfl(score, g, 64);
@@ -91,11 +103,17 @@ __device__ __forceinline__ void moe_select(float* z, int E, int top, int extra, 
     sum += w;
     if (lane == j) { mine = w; id = at; }
   }
+  const int real = E - by.identity;
+  const bool same = lane < top && id >= real;        // an identity expert
+  if (own) {
+    const float w = wave_sum(same ? mine : 0.f);
+    if (lane == 0) *own = w;
+  }
   if (lane < top) {
-    ids[lane] = id;
-    wts[lane] = mine / (by.correction ? sum + 1e-20f : sum);
+    ids[lane] = same ? -1 : id;
+    wts[lane] = same ? 0.f : by.softmax ? mine : mine / (by.correction ? sum + 1e-20f : sum);
   } else if (lane < top + extra) {
-    ids[lane] = E + lane - top;
+    ids[lane] = real + lane - top;
     wts[lane] = more;
   }
 }
@@ -104,7 +122,8 @@ __device__ __forceinline__ void moe_select(float* z, int E, int top, int extra, 
 template <int NT, int NW>
 __global__ void __launch_bounds__(64 * NW) moe_route_mfma_kernel(
     const bf16_t* __restrict__ h, long h_ld, const bf16_t* __restrict__ w, int T, int d, int E,
-    int top, int extra, RouteBy by, int* __restrict__ ids, float* __restrict__ wts) {
+    int top, int extra, RouteBy by, int* __restrict__ ids, float* __restrict__ wts,
+    float* __restrict__ own) {
   __shared__ float part[NW][16][NT * 16 + 1];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, q = lane >> 4;
   const int t0 = blockIdx.x * 16;
@@ -156,7 +175,7 @@ __global__ void __launch_bounds__(64 * NW) moe_route_mfma_kernel(
   for (int t = wave; t < 16; t += NW)
     if (t0 + t < T)
       moe_select(part[0][t], E, top, extra, by, ids + (long)(t0 + t) * (top + extra),
-                 wts + (long)(t0 + t) * (top + extra));
+                 wts + (long)(t0 + t) * (top + extra), own ? own + t0 + t : nullptr);
 }
 
 // grid T, block 256
@@ -165,7 +184,8 @@ __global__ void __launch_bounds__(256) moe_route_any_kernel(const T_* __restrict
                                                             const T_* __restrict__ w, int d, int E,
                                                             int top, int extra, RouteBy by,
                                                             int* __restrict__ ids,
-                                                            float* __restrict__ wts) {
+                                                            float* __restrict__ wts,
+                                                            float* __restrict__ own) {
   __shared__ float z[MAXE];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const long t = blockIdx.x;
@@ -177,7 +197,8 @@ __global__ void __launch_bounds__(256) moe_route_any_kernel(const T_* __restrict
   }
   __syncthreads();
   if (wave == 0)
-    moe_select(z, E, top, extra, by, ids + t * (top + extra), wts + t * (top + extra));
+    moe_select(z, E, top, extra, by, ids + t * (top + extra), wts + t * (top + extra),
+               own ? own + t : nullptr);
 }
 
 constexpr int CHUNK = 1024;      // uses per block of the sort (ops MOE_CHUNK)
@@ -224,8 +245,9 @@ __device__ __forceinline__ void plan_ranges(const PlanArgs& p, const int* cnt, i
 }
 
 __device__ __forceinline__ void place_use(const PlanArgs& p, int i, int* next) {
-  const int at = atomicAdd(&next[p.ids[i]], 1);
-  p.src[at] = i / p.J;
+  const int g = p.ids[i];
+  const int at = g < 0 ? -1 : atomicAdd(&next[g], 1);
+  if (at >= 0) p.src[at] = i / p.J;
   p.pos[i] = at;
 }
 
@@ -233,7 +255,8 @@ __global__ void __launch_bounds__(1024) moe_plan_small_kernel(PlanArgs p) {
   __shared__ int cnt[MAXE], beg[MAXE + 1], tbeg[MAXE + 1];
   for (int g = threadIdx.x; g < p.groups; g += blockDim.x) cnt[g] = 0;
   __syncthreads();
-  for (int i = threadIdx.x; i < p.n; i += blockDim.x) atomicAdd(&cnt[p.ids[i]], 1);
+  for (int i = threadIdx.x; i < p.n; i += blockDim.x)
+    if (p.ids[i] >= 0) atomicAdd(&cnt[p.ids[i]], 1);
   __syncthreads();
   plan_ranges(p, cnt, beg, tbeg);
   __syncthreads();
@@ -245,7 +268,8 @@ __global__ void __launch_bounds__(256) moe_hist_kernel(PlanArgs p) {
   for (int g = threadIdx.x; g < p.groups; g += 256) cnt[g] = 0;
   __syncthreads();
   const int i1 = min(p.n, (int)(blockIdx.x + 1) * CHUNK);
-  for (int i = blockIdx.x * CHUNK + threadIdx.x; i < i1; i += 256) atomicAdd(&cnt[p.ids[i]], 1);
+  for (int i = blockIdx.x * CHUNK + threadIdx.x; i < i1; i += 256)
+    if (p.ids[i] >= 0) atomicAdd(&cnt[p.ids[i]], 1);
   __syncthreads();
   for (int g = threadIdx.x; g < p.groups; g += 256) p.hist[blockIdx.x * p.groups + g] = cnt[g];
 }
@@ -284,35 +308,37 @@ __global__ void __launch_bounds__(256) moe_scatter_kernel(PlanArgs p) {
 }  // namespace
 
 int moe_route(const void* h, long h_ld, const void* w, int T, int d, int E, int rows, int top,
-              int extra, const float* correction, int groups, int keep, int* ids, float* wts,
-              int is_bf16, hipStream_t stream) {
+              int extra, const float* correction, int groups, int keep, int softmax, int identity,
+              int* ids, float* wts, float* own, int is_bf16, hipStream_t stream) {
   if (T <= 0) return 0;
   if (rows < E || rows > E + 1 || rows > MAXE || (rows > E && !correction) ||
       (correction && (groups < 1 || groups > 64 || E % groups || keep < 1 || keep > groups ||
                       keep * (E / groups) < top)))
     return -1;
-  const RouteBy by{correction, groups, keep, rows};
+  if ((softmax || identity) && (!correction || rows > E)) return -1;
+  if (identity < 0 || identity >= E || (identity > 0) != (own != nullptr)) return -1;
+  const RouteBy by{correction, groups, keep, rows, softmax, identity};
   if (E < 1 || E > MAXE || top < 1 || top > E || extra < 0 || top + extra > MAXTOP || d < 1)
     return -1;
   if (is_bf16 && rows <= 128 && d % 8 == 0 && h_ld % 8 == 0 && !(((uintptr_t)h | (uintptr_t)w) & 15)) {
     const int nt = (rows + 15) / 16;
 #define LMX_RT(NT, NW)                                                                       \
   moe_route_mfma_kernel<NT, NW><<<dim3((T + 15) / 16), dim3(64 * NW), 0, stream>>>(          \
-      (const bf16_t*)h, h_ld, (const bf16_t*)w, T, d, E, top, extra, by, ids, wts)
+      (const bf16_t*)h, h_ld, (const bf16_t*)w, T, d, E, top, extra, by, ids, wts, own)
     if (nt == 1) LMX_RT(1, 16); else if (nt == 2) LMX_RT(2, 16); else if (nt <= 4) LMX_RT(4, 8);
     else LMX_RT(8, 4);
 #undef LMX_RT
   } else if (is_bf16) {
     moe_route_any_kernel<bf16_t><<<dim3(T), dim3(256), 0, stream>>>(
-        (const bf16_t*)h, h_ld, (const bf16_t*)w, d, E, top, extra, by, ids, wts);
+        (const bf16_t*)h, h_ld, (const bf16_t*)w, d, E, top, extra, by, ids, wts, own);
   } else {
     moe_route_any_kernel<float><<<dim3(T), dim3(256), 0, stream>>>(
-        (const float*)h, h_ld, (const float*)w, d, E, top, extra, by, ids, wts);
+        (const float*)h, h_ld, (const float*)w, d, E, top, extra, by, ids, wts, own);
   }
   return (int)hipGetLastError();
 }
 
-// every id is in 0..groups - 1 (moe_route's)
+// every id is in -1..groups - 1 (moe_route's; -1: no use)
 int moe_plan(const int* ids, int n, int J, int groups, int bm, int mtiles, int* hist, int* off,
              int* src, int* pos, int* tiles, hipStream_t stream) {
   if (n <= 0) return 0;

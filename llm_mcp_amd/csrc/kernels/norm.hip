@@ -349,13 +349,15 @@ int layernorm(void* out, const void* x, const void* residual, const void* w, con
 // before the next sublayer in one pass, over an fp32 residual stream.
 //
 //   r   = ids ? scale * table[ids[row]] : residual[row]
-//   r  += norm(y[row]) * w_post              (y: the sublayer's output; optional)
+//   r  += norm(y[row] + bias + own[row] r) * w_post
+//                           (y: the sublayer's output, bias, own: all optional)
 //   out = w_pre ? norm(r) * w_pre : r
 //
 // norm(x) = x / sqrt(mean(x^2) + eps); the gains are fp32 (a weight stored
 // around zero arrives as 1 + w, a constant on what is added is part of w_post).
 // y is T rows, S fp32 split-K slabs [S][rows][cols] summed here, or a mixture
-// sum_j mix_w[row][j] y[mix_pos[row][j]] of T rows.  rows_idx (optional): out row i is source row
+// sum_j mix_w[row][j] y[mix_pos[row][j]] of T rows (pos -1: no such row).
+// rows_idx (optional): out row i is source row
 // rows_idx[i] and the residual is left as it is (the final norm of the sampled
 // rows); otherwise the residual row is written when it changed.
 struct SandwichArgs {
@@ -367,6 +369,8 @@ struct SandwichArgs {
   const int* mix_pos;         // [rows][mix_n] or null
   const float* mix_w;
   int mix_n;
+  const float* own;           // [rows] or null: weight of the stream's own row
+  const float* bias;          // [cols] or null
   const int* ids;
   const void* table;
   float scale;
@@ -411,13 +415,26 @@ __global__ void __launch_bounds__(512) sandwich_norm_kernel(SandwichArgs a) {
 #pragma unroll 4
         for (int j = 0; j < a.mix_n; ++j) {
           float t[V];
-          ldv<V>(t, (const T*)a.y + (long)a.mix_pos[src * a.mix_n + j] * a.y_ld + c * V);
+          const int at = a.mix_pos[src * a.mix_n + j];
+          if (at < 0) continue;
+          ldv<V>(t, (const T*)a.y + (long)at * a.y_ld + c * V);
           const float w = a.mix_w[src * a.mix_n + j];
 #pragma unroll
           for (int e = 0; e < V; ++e) y[i][e] += w * t[e];
         }
       } else {
         ldv<V>(y[i], (const T*)a.y + src * a.y_ld + c * V);
+      }
+      if (a.own) {
+        const float w = a.own[src];
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[i][e] += w * r[i][e];
+      }
+      if (a.bias) {
+        float t[V];
+        ldv<V>(t, a.bias + c * V);
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[i][e] += t[e];
       }
 #pragma unroll
       for (int e = 0; e < V; ++e) ss += y[i][e] * y[i][e];
@@ -474,15 +491,17 @@ __global__ void __launch_bounds__(512) sandwich_norm_kernel(SandwichArgs a) {
 }
 
 int sandwich_norm(void* out, float* residual, const void* y, long y_ld, int slabs, long slab_stride,
-                  const int* mix_pos, const float* mix_w, int mix_n, const int* ids,
+                  const int* mix_pos, const float* mix_w, int mix_n, const float* own,
+                  const float* bias, const int* ids,
                   const void* table, float scale, const float* w_post, const float* w_pre,
                   const long* rows_idx, int rows, int cols, float eps, int is_bf16,
                   hipStream_t stream) {
   if (rows <= 0) return 0;
-  if (cols <= 0 || !residual || !out || (y && !w_post) || (mix_pos && (!y || !mix_w || slabs)))
+  if (cols <= 0 || !residual || !out || (y && !w_post) || (mix_pos && (!y || !mix_w || slabs)) ||
+      ((own || bias) && !y))
     return -1;
-  const SandwichArgs a{out, residual, y, y_ld, slab_stride, slabs, mix_pos, mix_w, mix_n, ids,
-                       table, scale, w_post, w_pre, rows_idx, cols, eps};
+  const SandwichArgs a{out, residual, y, y_ld, slab_stride, slabs, mix_pos, mix_w, mix_n, own,
+                       bias, ids, table, scale, w_post, w_pre, rows_idx, cols, eps};
   const bool vec = cols % 8 == 0 && y_ld % 8 == 0;
   const int nchunk = vec ? cols / 8 : cols;
   const int vpt = (nchunk + 511) / 512;

@@ -68,7 +68,7 @@ constexpr int PG_THREADS = 512;
 constexpr int PG_HALF_B = 128 * 64 * 2;       // one half-tile image: 128 rows x 64 bf16
 constexpr int PG_STAGE_B = 4 * PG_HALF_B;     // A0 A1 W0 W1
 constexpr int PG_RING_B = 2 * PG_STAGE_B;     // 128 KB
-constexpr int PG_MAX_BIAS = 8192;
+constexpr int PG_MAX_BIAS = 14336;
 constexpr int PG_GROUP_M = 8;                 // M-tiles per tile group (L2 reuse)
 constexpr int HA0 = 0, HA1 = 1, HW0 = 2, HW1 = 3;
 
@@ -98,6 +98,9 @@ __device__ __forceinline__ float pg_act(float v) {
     return v / (1.f + __expf(-v));
   } else if constexpr (ACT == 4) {
     return 0.5f * v * (1.f + erff(v * 0.70710678118f));
+  } else if constexpr (ACT == 7) {
+    v = fmaxf(v, 0.f);
+    return v * v;
   } else {
     return v;
   }
@@ -934,7 +937,9 @@ int pgemm(void* C, const void* A, const void* W, const void* bias, int M, int N,
   if (res && (act != 0 || bias != nullptr)) return -1;
   if (N % 256 != 0 || K % 64 != 0 || K < 192) return -1;
   if (lda % 8 || ldw % 8 || ldc % 4) return -1;
-  if (act < 0 || act > 5 || ((act == 3 || act == 5) && bias != nullptr)) return -1;
+  if (act < 0 || act > 7 || act == 6 || ((act == 3 || act == 5) && bias != nullptr) ||
+      (act == 7 && bias == nullptr))
+    return -1;
   if (bias != nullptr && N > PG_MAX_BIAS) return -1;
   // byte offsets of one tile's rows are 32-bit
   if (256L * lda * 2 > 0x7fffffffL || 256L * ldw * 2 > 0x7fffffffL || 256L * ldc * 2 > 0x7fffffffL)
@@ -954,6 +959,7 @@ int pgemm(void* C, const void* A, const void* W, const void* bias, int M, int N,
       case 1: return pg_launch<1, 1>(C_, A_, W_, b_, M, N, K, ia, iw, ic, grid, stream);
       case 2: return pg_launch<2, 1>(C_, A_, W_, b_, M, N, K, ia, iw, ic, grid, stream);
       case 4: return pg_launch<4, 1>(C_, A_, W_, b_, M, N, K, ia, iw, ic, grid, stream);
+      case 7: return pg_launch<7, 1>(C_, A_, W_, b_, M, N, K, ia, iw, ic, grid, stream);
     }
     return -1;
   }

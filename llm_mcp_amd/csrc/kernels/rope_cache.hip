@@ -431,6 +431,157 @@ int norm_rope_cache(const void* p, long p_ld, const float* q_norm, const float* 
   return (int)hipGetLastError();
 }
 
+// As above for q and k RMS-normed over the whole projection (all heads' true
+// channels at once, gains fp32 [heads D]), after the projections' biases (fp32,
+// all heads); v heads divided by their own root mean square over dv channels.
+// One workgroup per row group; a thread owns IT pieces of 8 channels in its rows.
+template <typename T, int IT>
+__global__ void __launch_bounds__(1024) qkv_norm_rope_cache_kernel(
+    const T* __restrict__ p, long p_ld, const float* __restrict__ bias,
+    const float* __restrict__ q_norm, const float* __restrict__ k_norm,
+    const float* __restrict__ ang, int n, const int* __restrict__ slots,
+    const int* __restrict__ quads, T* __restrict__ q, T* __restrict__ kc, T* __restrict__ vc, int Hq,
+    int Hkv, int D, int dk, int dv, int BS, float eps) {
+  __shared__ float part[16][8];                // per wave: sums of squares of q and k, 4 rows
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+  const int pieces = (Hq + 2 * Hkv) * D / 8;
+  const int r0 = quads ? quads[blockIdx.x] : blockIdx.x;
+  const int cnt = quads ? min(4, quads[blockIdx.x + 1] - r0) : 1;
+  float x[IT][4][8], sq[4] = {0.f, 0.f, 0.f, 0.f}, sk[4] = {0.f, 0.f, 0.f, 0.f};
+  int slot[4];
+#pragma unroll
+  for (int t = 0; t < 4; ++t) slot[t] = t < cnt ? slots[r0 + t] : -1;
+#pragma unroll
+  for (int i = 0; i < IT; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c >= pieces) continue;
+    const int head = 8 * c / D;
+    float b[8];
+    ldv<8>(b, bias + 8 * c);
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      if (t >= cnt) continue;
+      ldv<8>(x[i][t], p + (long)(r0 + t) * p_ld + 8 * c);
+      float ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        x[i][t][e] += b[e];
+        ss += x[i][t][e] * x[i][t][e];
+      }
+      if (head < Hq) sq[t] += ss; else if (head < Hq + Hkv) sk[t] += ss;
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    if (t >= cnt) continue;
+    const float a = wave_sum(sq[t]), b = wave_sum(sk[t]);
+    if (lane == 0) { part[wave][t] = a; part[wave][4 + t] = b; }
+  }
+  __syncthreads();
+  float iq[4], ik[4];
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    if (t >= cnt) continue;
+    float a = 0.f, b = 0.f;
+    for (int w = 0; w < nw; ++w) { a += part[w][t]; b += part[w][4 + t]; }
+    iq[t] = rsqrtf(a / ((float)Hq * dk) + eps);
+    ik[t] = rsqrtf(b / ((float)Hkv * dk) + eps);
+  }
+  bool quad = cnt == 4 && slot[0] >= 0 && slot[0] % 4 == 0;
+#pragma unroll
+  for (int t = 1; t < 4; ++t) quad = quad && slot[t] == slot[0] + t;
+#pragma unroll
+  for (int i = 0; i < IT; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c >= pieces) continue;                 // whole heads leave together
+    const int head = 8 * c / D, d = 8 * c - head * D;
+    if (head >= Hq + Hkv) {
+      const long kvh = head - Hq - Hkv;
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        if (t >= cnt) continue;
+        float ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += x[i][t][e] * x[i][t][e];
+        for (int o = D >> 4; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+        const float inv = rsqrtf(ss / (float)dv + eps);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[i][t][e] *= inv;
+      }
+      if (quad) {
+        T* vp = vc + ((long)(slot[0] / BS) * Hkv + kvh) * BS * D + vq_off(d, slot[0] % BS, D);
+#pragma unroll
+        for (int e = 0; e < 8; e += 2) {
+          const float w[8] = {x[i][0][e], x[i][1][e], x[i][2][e], x[i][3][e],
+                              x[i][0][e + 1], x[i][1][e + 1], x[i][2][e + 1], x[i][3][e + 1]};
+          stv<8>(vp + 4 * e, w);
+        }
+        continue;
+      }
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        if (t >= cnt || slot[t] < 0) continue;
+        T* vp = vc + ((long)(slot[t] / BS) * Hkv + kvh) * BS * D + vq_off(d, slot[t] % BS, D);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) st1(vp + 4 * e, x[i][t][e]);
+      }
+      continue;
+    }
+    const bool isq = head < Hq;
+    float w[8];
+    ldv<8>(w, isq ? q_norm + 8 * c : k_norm + 8 * c - Hq * D);
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      if (t >= cnt) continue;
+      const float inv = isq ? iq[t] : ik[t];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[i][t][e] *= inv * w[e];
+      if (d < n) {
+        const float* a = ang + (long)(r0 + t) * n;
+#pragma unroll
+        for (int e = 0; e < 8; e += 2) {
+          if (d + e >= n) continue;
+          const float cs = a[(d + e) >> 1], sn = a[(n + d + e) >> 1];
+          const float u = x[i][t][e], v = x[i][t][e + 1];
+          x[i][t][e] = u * cs - v * sn;
+          x[i][t][e + 1] = v * cs + u * sn;
+        }
+      }
+      if (isq) {
+        stv<8>(q + (long)(r0 + t) * Hq * D + 8 * c, x[i][t]);
+      } else if (slot[t] >= 0) {
+        stv<8>(kc + (((long)(slot[t] / BS) * Hkv + head - Hq) * BS + slot[t] % BS) * D + d,
+               x[i][t]);
+      }
+    }
+  }
+}
+
+int qkv_norm_rope_cache(const void* p, long p_ld, const float* bias, const float* q_norm,
+                        const float* k_norm, const float* ang, int n, const int* slots,
+                        const int* quads, int groups, void* q, void* kc, void* vc, int Hq, int Hkv,
+                        int D, int dk, int dv, int BS, float eps, int is_bf16, hipStream_t stream) {
+  if (groups <= 0) return 0;
+  // a head's D / 8 lanes reduce inside one wave: D a power of two, 64..512
+  if (D < 64 || D > 512 || (D & (D - 1)) || dk < 1 || dk > D || dv < 1 || dv > D || n < 0 || n % 2 ||
+      n > dk || (n && !ang) || BS % 4 || p_ld % 8 || (((uintptr_t)p | (uintptr_t)q) & 15) || Hq < 1 ||
+      Hkv < 1)
+    return -1;
+  const int pieces = (Hq + 2 * Hkv) * D / 8;
+  const int threads = pieces >= 1024 ? 1024 : (pieces + 63) / 64 * 64;
+  const int it = (pieces + threads - 1) / threads;
+  if (it > 4) return -2;
+#define LMX_QN(T, I)                                                                            \
+  qkv_norm_rope_cache_kernel<T, I><<<dim3(groups), dim3(threads), 0, stream>>>(                 \
+      (const T*)p, p_ld, bias, q_norm, k_norm, ang, n, slots, quads, (T*)q, (T*)kc, (T*)vc, Hq, \
+      Hkv, D, dk, dv, BS, eps)
+#define LMX_QNT(T) if (it == 1) LMX_QN(T, 1); else if (it == 2) LMX_QN(T, 2); else LMX_QN(T, 4);
+  if (is_bf16) { LMX_QNT(bf16_t) } else { LMX_QNT(float) }
+#undef LMX_QNT
+#undef LMX_QN
+  return (int)hipGetLastError();
+}
+
 // Plain cache write (no rotation), used by the paged-cache tests and by
 // models without rotary embeddings.
 __global__ void kv_write_kernel(const bf16_t* __restrict__ k, const bf16_t* __restrict__ v,

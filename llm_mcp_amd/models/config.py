@@ -261,7 +261,18 @@ class RefolixConfig(LayerListConfig):
         return cfg
 
 
-LAYER_LISTS = {c.architecture: c for c in (ZegopelConfig, PikesunConfig, RefolixConfig)}
+@dataclass
+class ZovozenConfig(LayerListConfig):
+    """``parallel`` mixers (attention with talking heads in chunks beside a
+    matrix memory), ``dense`` and ``moe`` feed-forwards, the head tied to the
+    embedding."""
+    name: str = "zovozen"
+    family: str = "zovozen"
+    architecture: str = "Zovozen"
+
+
+LAYER_LISTS = {c.architecture: c for c in (ZegopelConfig, PikesunConfig, RefolixConfig,
+                                           ZovozenConfig)}
 
 
 def zegopel_stack(pattern: str, ff: int, lightning: dict, mamba2: dict,
@@ -388,6 +399,44 @@ def _refolix_8b() -> RefolixConfig:
                          logit_softcap=30.0)
 
 
+def zovozen_stack(pattern: str, parallel: dict, dense: dict, moe: dict) -> list:
+    """Layer list from a pattern of D (dense), M (mixture of experts): every
+    layer has both mixers."""
+    return [{"type": "parallel", "mixer": dict(parallel),
+             "mlp": dict(dense if c == "D" else moe)} for c in pattern]
+
+
+def _identity_moe(experts: int, identity: int, top: int, ff: int, shared: int, groups: int,
+                  keep: int) -> dict:
+    return dict(kind="moe", router=dict(experts=experts, identity=identity, top=top,
+                                        groups=dict(count=groups, keep=keep)),
+                expert=dict(ff=ff), shared=dict(ff=shared))
+
+
+def _zovozen_tiny() -> ZovozenConfig:
+    left = dict(heads=6, kv_heads=3, dim=40, vdim=64, scale=40 ** -0.5, mask=dict(size=72),
+                rot=dict(base=10000.0, dims=24, scaling=dict(factor=4.0)))
+    layers = zovozen_stack(
+        "DMM", dict(left=left, right=dict(heads=3, dim=32, vdim=40, gate_cap=15.0),
+                    left_scale=0.8, right_scale=1.1), dict(kind="dense", ff=320),
+        _identity_moe(9, 3, 3, 64, 96, 3, 2))
+    return ZovozenConfig(name="tiny-zovozen", vocab_size=512, hidden_size=192, bos_token_id=506,
+                         eos_token_ids=(510,), layers=layers)
+
+
+def _zovozen_8b() -> ZovozenConfig:
+    """Llama-3-8B's width and size, all experts counted (random weights:
+    benchmarks)."""
+    left = dict(heads=32, kv_heads=8, dim=128, vdim=128, scale=128 ** -0.5, mask=dict(size=2048),
+                rot=dict(base=500000.0, dims=64, scaling=dict(factor=4.0)))
+    layers = zovozen_stack(
+        "DMM" * 7, dict(left=left, right=dict(heads=32, dim=128, vdim=128, gate_cap=15.0),
+                        left_scale=0.8, right_scale=0.6), dict(kind="dense", ff=14336),
+        _identity_moe(14, 2, 4, 1024, 2048, 4, 2))
+    return ZovozenConfig(name="zovozen-8b", vocab_size=128256, hidden_size=4096,
+                         bos_token_id=128000, eos_token_ids=(128001, 128009), layers=layers)
+
+
 _LLAMA32_ROPE = {"rope_type": "llama3", "factor": 32.0, "low_freq_factor": 1.0,
                  "high_freq_factor": 4.0, "original_max_position_embeddings": 8192}
 
@@ -485,6 +534,8 @@ PRESETS: dict[str, object] = {
     "pikesun-8b": _pikesun_8b(),
     "tiny-refolix": _refolix_tiny(),
     "refolix-8b": _refolix_8b(),
+    "tiny-zovozen": _zovozen_tiny(),
+    "zovozen-8b": _zovozen_8b(),
     "tiny-nomic": NomicBertConfig(name="tiny-nomic", vocab_size=512, hidden_size=256,
                                   intermediate_size=512, num_layers=2, num_heads=2, head_dim=128,
                                   embed_dim=256, max_position=2048),

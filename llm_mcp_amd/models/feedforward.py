@@ -59,6 +59,7 @@ class MixtureOfExperts:
     The shared expert runs as further experts of the routed ones' width that
     every token uses with weight 1: one grouped product covers all of them."""
     glu = (1.702, 1.0)                     # slope of the gate's sigmoid, added to up
+    identity = 0                           # routed experts that return their input
 
     @staticmethod
     def _limit(m: dict) -> float:
@@ -67,7 +68,8 @@ class MixtureOfExperts:
     def __init__(self, m: dict, width: int):
         self.width, self.kp, self.np = width, _up(width, 64), _up(width, 16)
         self.E, self.top = m["router"]["experts"], m["router"]["top"]
-        if not 0 < self.top <= self.E:
+        self.routed = self.E + self.identity
+        if not (self.E > 0 and self.identity >= 0 and 0 < self.top <= self.routed):
             raise ValueError("moe: top experts out of range")
         ex, sh = m["expert"], m.get("shared")
         self.ff, self.sff = ex["ff"], sh["ff"] if sh else 0
@@ -78,7 +80,7 @@ class MixtureOfExperts:
         for e in range(self.E):
             self.shapes.update({f"e{e}.gate": (self.ff, width), f"e{e}.up": (self.ff, width),
                                 f"e{e}.down": (width, self.ff)})
-        self.shapes["router"] = (self.E, width)
+        self.shapes["router"] = (self.routed, width)
         if sh:
             self.shapes.update({"shared.gate": (self.sff, width), "shared.up": (self.sff, width),
                                 "shared.down": (width, self.sff)})
@@ -109,7 +111,7 @@ class MixtureOfExperts:
                             ops.wide_tiles(self.w1) and ops.wide_tiles(self.w2))
         y = ops.grouped_linear(_pad_cols(h, self.kp), self.w1, plan, gather=True, glu=self.limit,
                                act=self.glu)
-        return ops.Mixture(ops.grouped_linear(y, self.w2, plan), plan.pos, r.weights)
+        return ops.Mixture(ops.grouped_linear(y, self.w2, plan), plan.pos, r.weights, r.own)
 
 
 class GroupRoutedMoE(MixtureOfExperts):
@@ -118,6 +120,7 @@ class GroupRoutedMoE(MixtureOfExperts):
     their two largest), in the proportions of their s; the shared expert is
     weighted by the sigmoid of one more logit."""
     glu = (1.0, 0.0)
+    shared_gate = True
 
     @staticmethod
     def _limit(m: dict) -> float:
@@ -127,20 +130,60 @@ class GroupRoutedMoE(MixtureOfExperts):
         super().__init__(m, width)
         g = m["router"].get("groups") or {"count": 1, "keep": 1}
         self.groups, self.keep = g["count"], g["keep"]
-        if (self.groups < 1 or self.E % self.groups or not 0 < self.keep <= self.groups
-                or self.keep * (self.E // self.groups) < self.top):
+        n = self.routed
+        if (self.groups < 1 or n % self.groups or not 0 < self.keep <= self.groups
+                or self.keep * (n // self.groups) < self.top):
             raise ValueError("moe: groups do not fit the experts")
-        self.shapes["correction"] = (self.E,)
-        if self.shared:
+        self.shapes["correction"] = (n,)
+        if self.shared and self.shared_gate:
             self.shapes["shared.sg"] = (1, width)
 
     def load(self, get, put):
         super().load(get, put)
         self.correction = put(get("correction"), fp32=True)
-        if self.shared:                    # the shared expert's logit: one more row
+        if self.shared and self.shared_gate:     # the shared expert's logit: one more row
             self.router = put(torch.cat([get("router"), get("shared.sg")]))
 
     def _route(self, h):
         return ops.moe_route(h, self.router, self.top, self.shared,
                              ops.GroupScores(self.correction, self.groups, self.keep))
 
+
+class SoftmaxGroupMoE(GroupRoutedMoE):
+    """SiLU GLUs, routed by a softmax over the logits of the experts and of
+    ``identity`` experts behind them, whose output is their input: the ``top``
+    largest s + correction among the experts of the best groups (ranked by the
+    largest), with their s as they are; the shared expert has weight 1.  For
+    sublayers that read the stream itself."""
+    shared_gate = False
+
+    def __init__(self, m: dict, width: int):
+        r = m["router"]
+        self.identity = int(r.get("identity") or 0)
+        super().__init__(m, width)
+
+    def _route(self, h):
+        return ops.moe_route(h, self.router, self.top, self.shared,
+                             ops.GroupScores(self.correction, self.groups, self.keep, True,
+                                             self.identity))
+
+
+class ReluSquaredMLP:
+    """W_down relu(W_up h + b)^2 + b'"""
+
+    def __init__(self, m: dict, width: int):
+        self.ff, self.fp = m["ff"], _up(m["ff"], 16)
+        self.shapes = {"up": (self.ff, width), "up.b": (self.ff,), "down": (width, self.ff),
+                       "down.b": (width,)}
+        self.proj = {"up": (self.fp, width), "down": (width, self.fp)}
+
+    def load(self, get, put):
+        self.w_up = put(_fuse_rows([get("up")], [self.fp]))
+        self.w_down = put(_pad_cols(get("down"), self.fp))
+        b = _pad_cols(get("up.b"), self.fp)
+        self.up_bias, self.up_bias_row = put(b, fp32=True), put(b)
+        self.down_bias = put(get("down.b"), fp32=True)
+
+    def forward(self, h):
+        y = ops.linear_relu2(h, self.w_up, self.up_bias, self.up_bias_row)
+        return ops.Biased(ops.linear(y, self.w_down, defer=True), self.down_bias)

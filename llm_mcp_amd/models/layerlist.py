@@ -1,5 +1,5 @@
 """Decoders whose configuration lists their layers one by one (Zegopel,
-Pikesun, Refolix), in the in-process serving engine.
+Pikesun, Refolix, Zovozen), in the in-process serving engine.
 
 A layer is a token mixer (``models.mixers``) and, where it has one, a
 feed-forward (``models.feedforward``), each between an optional norm before and
@@ -52,6 +52,7 @@ class LayerListModel:
     feedforwards: dict = {}       # mlp "kind" -> feed-forward class
     zero_centred = False          # stored gains act as 1 + w
     tail = "b"                    # suffix of the norm after a sublayer ("": no norm before it)
+    tied_head = False             # the logits use the embedding table
     layer_scale = ""              # name of the per-channel scale of a sublayer's output, if any
 
     # ------------------------------------------------------------ layout ----
@@ -102,7 +103,9 @@ class LayerListModel:
             out.update({f"l{i}.mix.{k}": s for k, s in mix.shapes.items()})
             if ff is not None:
                 out.update({f"l{i}.mlp.{k}": s for k, s in ff.shapes.items()})
-        out.update({"final.norm": (d,), "head": (cfg.vocab_size, d)})
+        out["final.norm"] = (d,)
+        if not cls.tied_head:
+            out["head"] = (cfg.vocab_size, d)
         return out
 
     def __init__(self, cfg, device: torch.device | str = "cuda", dtype=torch.bfloat16,
@@ -172,7 +175,7 @@ class LayerListModel:
                             for k, (a, b) in enumerate(norms[i])]
         self.norms = [norms[j] for j in source]
         self.final_norm = gain("final.norm")
-        self.head = put(get("head"))
+        self.head = self.embed if self.tied_head else put(get("head"))
         self._freqs = {r: ops.rope_freqs(*r, device=self.device) for r in self._angles}
 
     def weight_bytes(self, copies: bool = False) -> int:
@@ -181,7 +184,8 @@ class LayerListModel:
         ts += [t for ns in self.norms for pair in ns for p in pair
                for t in (p if isinstance(p, tuple) else (p,)) if t is not None]
         for o in (o for m, ff in self.parts for o in (m, *m.members(), ff) if o is not None):
-            vals = [v.data if isinstance(v, ops.GroupedWeight) else v for v in vars(o).values()]
+            vals = [v.data if isinstance(v, ops.GroupedWeight) else
+                    v.mix if isinstance(v, ops.Talk) else v for v in vars(o).values()]
             ts += [t for t in vals if isinstance(t, torch.Tensor)]
         return sum({t.data_ptr(): t.numel() * t.element_size() for t in ts}.values())
 

@@ -441,9 +441,21 @@ def rotary(rot: dict | None, dim: int) -> tuple | None:
     if rot["dims"] % 2 or not 0 < rot["dims"] <= dim:
         raise ValueError("rotation: an even number of a head's channels")
     s = rot.get("scaling")
-    return (float(rot["base"]), int(rot["dims"])) + (
-        (float(s["factor"]), float(s["original"]), float(s["fast"]), float(s["slow"]))
-        if s else ())
+    if s and "original" not in s:               # every frequency divided
+        s = (float(s["factor"]),)
+    elif s:
+        s = (float(s["factor"]), float(s["original"]), float(s["fast"]), float(s["slow"]))
+    return (float(rot["base"]), int(rot["dims"])) + (s or ())
+
+
+def _pairs_together(heads: int, dim: int, rot: tuple | None) -> torch.Tensor:
+    """Order of [heads * dim] channels that puts each head's rotated pairs (i, i
+    + dims/2) next to each other."""
+    i = torch.arange(dim)
+    if rot is not None:
+        d = rot[1]
+        i[:d] = torch.stack([i[:d // 2], i[d // 2:d]], 1).reshape(-1)
+    return (torch.arange(heads)[:, None] * dim + i).reshape(-1)
 
 
 class RetentionMixer(ScanMixer):
@@ -473,12 +485,7 @@ class RetentionMixer(ScanMixer):
 
     def _paired(self, w):
         """[H * N, ...] rows with each head's rotated pairs next to each other."""
-        if self.rot is None:
-            return w
-        d = self.rot[1]
-        i = torch.arange(self.N)
-        i[:d] = torch.stack([i[:d // 2], i[d // 2:d]], 1).reshape(-1)
-        return w.reshape(self.H, self.N, -1)[:, i.to(w.device)].reshape(self.H * self.N, -1)
+        return w[_pairs_together(self.H, self.N, self.rot).to(w.device)]
 
     def load(self, get, put):
         self.w_in = put(_fuse_rows([self._paired(get("q")), self._paired(get("k")), get("v"),
@@ -661,25 +668,22 @@ class GatedDeltaMixer(Mixer):
         return ops.linear(y, self.w_o, defer=True)
 
 
-class ParallelMixer(Mixer):
-    """Windowed attention and a gated delta rule side by side on the same rows:
-    half the sum of their outputs, each RMS-normed over the width.  One input
-    projection serves both."""
+class Branches(Mixer):
+    """Attention (``left_class``) and a recurrence (``right_class``) side by
+    side on the same rows.  One input projection serves both."""
+    left_class = right_class = None
 
     def __init__(self, m: dict, width: int, eps: float):
-        self.left = SoftcapAttentionMixer(m["left"], width, eps)
-        self.right = GatedDeltaMixer(m["right"], width, eps)
-        self.shapes = {}
-        for name, part in (("left", self.left), ("right", self.right)):
-            self.shapes.update({f"{name}.{k}": s for k, s in part.shapes.items()})
-            self.shapes[name + ".out"] = (width,)
+        self.left = self.left_class(m["left"], width, eps)
+        self.right = self.right_class(m["right"], width, eps)
+        self.shapes = {f"{name}.{k}": s for name, part in (("left", self.left), ("right", self.right))
+                       for k, s in part.shapes.items()}
         self.kv, self.q_per_tile = self.left.kv, self.left.q_per_tile
         self.Hq, self.Hkv, self.D = self.left.Hq, self.left.Hkv, self.left.D
         rows = self.left.rows + self.right.rows
         # a wide projection is rounded up to whole 256-row GEMM tiles
         self.tail = (_up(rows, 256) if rows >= 4096 else rows) - rows
-        self.proj = {"in": (rows + self.tail, width), "left.o": self.left.proj["o"],
-                     "right.o": self.right.proj["o"]}
+        self.proj = {"in": (rows + self.tail, width)}
 
     def members(self):
         return [self.left, self.right]
@@ -693,6 +697,20 @@ class ParallelMixer(Mixer):
         self.w_in = put(_fuse_rows(parts, [self.left.rows, self.right.rows + self.tail]))
         self.left.load(left, put, own_projection=False)
         self.right.load(right, put, own_projection=False)
+
+
+class ParallelMixer(Branches):
+    """Windowed attention beside a gated delta rule: half the sum of their
+    outputs, each RMS-normed over the width."""
+    left_class, right_class = SoftcapAttentionMixer, GatedDeltaMixer
+
+    def __init__(self, m: dict, width: int, eps: float):
+        super().__init__(m, width, eps)
+        self.shapes.update({"left.out": (width,), "right.out": (width,)})
+        self.proj.update({"left.o": self.left.proj["o"], "right.o": self.right.proj["o"]})
+
+    def load(self, get, put):
+        super().load(get, put)
         self.out_left, self.out_right = (put(0.5 * get(s + ".out").float(), fp32=True)
                                          for s in ("left", "right"))
 
@@ -702,6 +720,183 @@ class ParallelMixer(Mixer):
         return ops.NormedPair(self.left.mix(p[:, :n], inp, cache, state),
                               self.right.mix(p[:, n:], inp, cache, state),
                               self.out_left, self.out_right)
+
+
+class TalkingAttentionMixer(Mixer):
+    """Softmax attention whose heads' scores are mixed: q and k (biased)
+    RMS-normed over the whole projection and partly rotated (pairs i, i +
+    dims/2), v divided by its root mean square per head; scores times a number
+    per head, mixed over the heads; a row sees its own chunk of positions; a
+    sink per head in the softmax; output gate sigmoid(W_g h).
+
+    q is served with the score's scale and the heads' numbers in its gain, and
+    with each head's rotated pairs next to each other, as k is."""
+    Hkv = 1                       # all heads of a row run in one workgroup
+
+    def __init__(self, m: dict, width: int, eps: float):
+        self.Hq, self.G, self.dk, self.dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        self.scale, self.eps = float(m["scale"]), eps
+        mask = m.get("mask")
+        self.chunk = int(mask["size"]) if mask else 0
+        if mask and self.chunk < 1:
+            raise ValueError("attention: a chunk of at least 1")
+        if self.Hq % self.G:
+            raise ValueError("attention: heads must be a multiple of kv_heads")
+        self.rot = rotary(m.get("rot"), self.dk)
+        H, G, dk, dv = self.Hq, self.G, self.dk, self.dv
+        D = self.D = _head_size(max(dk, dv))
+        self.shapes = {"q": (H * dk, width), "k": (G * dk, width), "v": (G * dv, width),
+                       "q.b": (H * dk,), "k.b": (G * dk,), "v.b": (G * dv,),
+                       "q.norm": (H * dk,), "k.norm": (G * dk,), "talk": (H, H), "temp": (H,),
+                       "sink": (H,), "g": (H * dv, width), "o": (width, H * dv), "o.b": (width,)}
+        self.kv = (G, D, D)
+        self.qkv = (H + 2 * G) * D
+        self.rows = self.qkv + H * D
+        self.proj = {"in": (self.rows, width), "o": (width, H * D)}
+        self.q_per_tile = ops.TALK_QT
+        self.plan_key = ("talk",)
+
+    def build_plan(self, qlens, ctx, seq0):
+        return [("quads", mixer_ops.row_quads(qlens, ctx, seq0)),
+                ("talk", mixer_ops.row_tiles(qlens, ops.TALK_QT).reshape(-1))], None
+
+    def bind_plan(self, dev, host):
+        return dev["quads"], dev["talk"]
+
+    def _heads(self, t, n, d, pairs=False):
+        """[n * d, ...] rows -> [n * D, ...], each head padded with zeros."""
+        if pairs:
+            t = t[_pairs_together(n, d, self.rot).to(t.device)]
+        out = t.new_zeros((n, self.D) + tuple(t.shape[1:]))
+        out[:, :d] = t.reshape((n, d) + tuple(t.shape[1:]))
+        return out.reshape((n * self.D,) + tuple(t.shape[1:]))
+
+    def _qkv(self, get, suffix=""):
+        return [self._heads(get("q" + suffix), self.Hq, self.dk, True),
+                self._heads(get("k" + suffix), self.G, self.dk, True),
+                self._heads(get("v" + suffix), self.G, self.dv)]
+
+    def in_rows(self, get):
+        return torch.cat(self._qkv(get) + [self._heads(get("g"), self.Hq, self.dv)])
+
+    def out_rows(self, get):
+        """The output projection, [width, H * D]."""
+        return self._heads(get("o").t().contiguous(), self.Hq, self.dv).t()
+
+    def load(self, get, put, own_projection=True):
+        if own_projection:
+            self.w_in, self.w_o = put(self.in_rows(get)), put(self.out_rows(get))
+            self.out_bias = put(get("o.b"), fp32=True)
+        self.in_bias = put(torch.cat(self._qkv(get, ".b")), fp32=True)
+        w = get("q.norm").float().view(self.Hq, self.dk) * get("temp").float()[:, None] * self.scale
+        self.q_norm = put(self._heads(w.reshape(-1), self.Hq, self.dk, True), fp32=True)
+        self.k_norm = put(self._heads(get("k.norm"), self.G, self.dk, True), fp32=True)
+        self.talk = ops.Talk(put(get("talk")), put(get("sink"), fp32=True))
+
+    def forward(self, h, inp, cache, state):
+        p = ops.linear(h, self.w_in)
+        a = torch.empty((p.shape[0], self.Hq * self.D), dtype=p.dtype, device=p.device)
+        self.attend(p, inp, cache, a)
+        return ops.Biased(ops.linear(a, self.w_o, defer=True), self.out_bias)
+
+    def attend(self, p, inp, cache, out, scale=1.0):
+        """The gated heads of projection rows p = [q | k | v | g | ..], times
+        ``scale``, into ``out`` [T, H * D]."""
+        kc, vc = cache
+        quads, tiles = inp.aux.get(self.plan_key, (None, None))
+        ang = inp.aux["rot", self.rot] if self.rot else None
+        q = ops.qkv_norm_rope_cache(p, self.in_bias, self.q_norm, self.k_norm, ang, inp.slots, kc,
+                                    vc, self.Hq, self.dk, self.dv, self.eps, quads)
+        ops.talking_attention(q, kc, vc, inp.block_tables, inp.cu_q, inp.context_lens,
+                              inp.positions, self.talk, self.Hq, p[:, self.qkv:self.rows], out,
+                              self.chunk, scale, inp.num_decode, tiles, inp.decode_ws)
+
+
+class MatrixMemoryMixer(ScanMixer):
+    """Matrix memory with exponential gates (``ops.memory_scan``): q, k, v and
+    gates projected; each head's output divided by its root mean square, times
+    a gain and sigmoid(W_g h), projected."""
+
+    def __init__(self, m: dict, width: int, eps: float):
+        self.H, self.N, self.P = m["heads"], m["dim"], m["vdim"]
+        self.cap, self.eps = float(m["gate_cap"]), eps
+        if not self.cap > 0:
+            raise ValueError("matrix memory: a positive gate_cap")
+        H, N, P = self.H, self.N, self.P
+        self.shapes = {"q": (H * N, width), "k": (H * N, width), "v": (H * P, width),
+                       "g": (H * P, width), "o": (width, H * P), "norm": (H * P,),
+                       "i": (H, width), "i.b": (H,), "f": (H, width), "f.b": (H,)}
+        self.qk, self.vg, self.hp = _up(H * N, 8), _up(H * P, 8), _up(H, 8)
+        self.rows = 2 * (self.qk + self.vg + self.hp)
+        self.proj = {"in": (self.rows, width), "o": (width, H * P)}
+
+    def state_shapes(self, dtype):
+        H, N, P = self.H, self.N, self.P
+        return [((H, N, P), torch.float32), ((H, N), torch.float32), ((H,), torch.float32)]
+
+    plan_key = property(lambda self: ("scan", self.H, self.P))
+
+    def in_rows(self, get):
+        return _fuse_rows([get(n) for n in ("q", "k", "v", "g", "i", "f")],
+                          [self.qk, self.qk, self.vg, self.vg, self.hp, self.hp])
+
+    def out_rows(self, get):
+        return get("o")
+
+    def load(self, get, put, own_projection=True):
+        if own_projection:
+            self.w_in, self.w_o = put(self.in_rows(get)), put(self.out_rows(get))
+        self.gate_bias = put(torch.stack([get("i.b").float(), get("f.b").float()]), fp32=True)
+        self.norm = put(get("norm"), fp32=True)
+
+    def forward(self, h, inp, cache, state):
+        p = ops.linear(h, self.w_in)
+        return ops.linear(self.recall(p, inp, state), self.w_o, defer=True)
+
+    def recall(self, p, inp, state, out=None):
+        """The gated heads of projection rows p = [q | k | v | g | i | f | ..]."""
+        qk, vg, hp = self.qk, self.vg, self.hp
+        a = 2 * (qk + vg)
+        y = ops.memory_scan(p[:, :qk], p[:, qk:2 * qk], p[:, 2 * qk:2 * qk + vg], p[:, a:a + hp],
+                            p[:, a + hp:a + 2 * hp], self.gate_bias, self.cap, state, inp.cu_q,
+                            inp.context_lens, inp.state_slots, num_decode=inp.num_decode,
+                            segments=inp.aux.get(self.plan_key))
+        return ops.gated_norm(y, p[:, 2 * qk + vg:a], self.norm, self.H, self.eps,
+                              gate_first=False, out=out)
+
+
+class TalkingMemoryMixer(Branches):
+    """Attention with talking heads beside a matrix memory, left_scale left +
+    right_scale right.  The scales act on the branches' rows in fp32 and one
+    product projects both."""
+    left_class, right_class = TalkingAttentionMixer, MatrixMemoryMixer
+
+    def __init__(self, m: dict, width: int, eps: float):
+        super().__init__(m, width, eps)
+        self.scales = float(m["left_scale"]), float(m["right_scale"])
+        self.split = self.left.Hq * self.left.D
+        self.cols = self.split + _up(self.right.H * self.right.P, 8)
+        self.proj["o"] = (width, self.cols)
+
+    def load(self, get, put):
+        super().load(get, put)
+        left, right = (lambda n, s=s: get(f"{s}.{n}") for s in ("left", "right"))
+        w = get("left.o").new_zeros(self.proj["o"])
+        w[:, :self.split] = self.left.out_rows(left)
+        w[:, self.split:self.split + self.right.H * self.right.P] = self.right.out_rows(right)
+        self.w_o = put(w)
+        self.out_bias = put(self.scales[0] * left("o.b").float(), fp32=True)
+        self.right.norm.mul_(self.scales[1])
+
+    def forward(self, h, inp, cache, state):
+        p = ops.linear(h, self.w_in)
+        T, n, c = p.shape[0], self.split, self.right.H * self.right.P
+        y = torch.empty((T, self.cols), dtype=p.dtype, device=p.device)
+        if self.cols > n + c:
+            y[:, n + c:].zero_()
+        self.left.attend(p[:, :self.left.rows], inp, cache, y[:, :n], self.scales[0])
+        self.right.recall(p[:, self.left.rows:], inp, state, out=y[:, n:n + c])
+        return ops.Biased(ops.linear(y, self.w_o, defer=True), self.out_bias)
 
 
 def init_std(name: str, shape: tuple, depth: int, zero_centred: bool = True) -> tuple[float, float]:
@@ -722,6 +917,12 @@ def init_std(name: str, shape: tuple, depth: int, zero_centred: bool = True) -> 
         return -4.0, 1.0
     if leaf in ("ra", "ri"):
         return 0.0, shape[-1] ** -0.5
+    if leaf == "temp":
+        return 1.0, 0.1
+    if leaf == "talk":
+        return 1.0 / shape[-1], 0.3
+    if name.endswith("right.f.b"):     # slow forgetting
+        return 4.0, 1.0
     if name == "embed":
         return 0.0, 1.0
     if leaf.startswith("norm"):

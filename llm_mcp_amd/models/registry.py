@@ -24,6 +24,9 @@ def layer_list_class(family: str):
     if family == "refolix":
         from .refolix import RefolixModel
         return RefolixModel
+    if family == "zovozen":
+        from .zovozen import ZovozenModel
+        return ZovozenModel
     raise ValueError(f"{family}: not a layer-list family")
 
 

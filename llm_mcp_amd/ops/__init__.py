@@ -584,6 +584,7 @@ ACT_NONE, ACT_GELU, ACT_SILU = 0, 1, 2
 ACT_SWIGLU = 3
 ACT_GELU_ERF = 4   # exact (erf) GELU, BERT FFNs
 ACT_RELUGLU = 5    # the pair form of ACT_SWIGLU with ReLU on the gate
+ACT_RELU2 = 7      # relu(z)^2, with a bias (6 is the grouped products' clamped GLU)
 
 
 def interleave_gate_up(w: torch.Tensor, block: int = 64) -> torch.Tensor:
@@ -905,6 +906,31 @@ def linear_gelu(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
             and large_gemm_backend(x.shape[0], w.shape[0], w.shape[1], ACT_GELU) == "k13"):
         return pgemm(x, w, act=ACT_GELU)
     return gelu(linear(x, w))
+
+
+def bias_relu2(x: torch.Tensor, bias: torch.Tensor) -> torch.Tensor:
+    """relu(x + bias)^2 of a projection's rows (bf16 or fp32; bias fp32 [N]), in
+    place."""
+    if not x.is_cuda:
+        return ref.bias_relu2(x, bias)
+    _chk(x.dtype in (torch.bfloat16, torch.float32) and x.is_contiguous() and x.dim() == 2
+         and x.shape[1] % 8 == 0 and bias.dtype == torch.float32 and bias.is_contiguous()
+         and bias.numel() == x.shape[1], "bias_relu2 rows")
+    native().bias_relu2(_ptr(x), _ptr(bias), x.shape[0], x.shape[1],
+                        int(x.dtype == torch.bfloat16), _stream())
+    return x
+
+
+def linear_relu2(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor,
+                 bias_bf16: torch.Tensor | None = None) -> torch.Tensor:
+    """relu(x @ w^T + bias)^2 (bias fp32 [N]): K13's epilogue for prefill-sized
+    M where the bias is given in bf16 as well, else the product and an
+    elementwise pass."""
+    if (x.is_cuda and x.dtype == torch.bfloat16 and bias_bf16 is not None
+            and pgemm_operands_ok(x, w) and pgemm_bias_ok(bias_bf16, w.shape[0])
+            and large_gemm_backend(x.shape[0], w.shape[0], w.shape[1], ACT_RELU2, True) == "k13"):
+        return pgemm(x, w, bias=bias_bf16, act=ACT_RELU2)
+    return bias_relu2(linear(x, w), bias)
 
 
 def swiglu_block(N: int, K: int) -> int:
@@ -1568,7 +1594,7 @@ def rsgemm(a: torch.Tensor, w: torch.Tensor, cfg: int, splits: int, epi: int = 0
 # ---------------------------------------------------------------------------
 # K13: large-M GEMM (csrc/kernels/pgemm.hip): prefill chunks, encoder batches
 # ---------------------------------------------------------------------------
-PGEMM_MAX_BIAS = 8192
+PGEMM_MAX_BIAS = 14336
 PGEMM_CALLS = [0]          # host-side launch count (tests: the K13 path really ran)
 RESIDUAL_EPILOGUE = os.environ.get("LMX_RESIDUAL_EPILOGUE", "1") != "0"
 
@@ -1576,8 +1602,9 @@ RESIDUAL_EPILOGUE = os.environ.get("LMX_RESIDUAL_EPILOGUE", "1") != "0"
 def pgemm_supported(N: int, K: int, act: int = 0, bias: bool = False) -> bool:
     """Shapes K13 takes: 256-column tiles, 64-deep K-steps, >= 3 of them;
     a bias row fits its LDS slot; the SwiGLU form takes no bias."""
-    return (N % 256 == 0 and K % 64 == 0 and K >= 192 and act in (0, 1, 2, 3, 4, 5)
-            and not (bias and (N > PGEMM_MAX_BIAS or act in (ACT_SWIGLU, ACT_RELUGLU))))
+    return (N % 256 == 0 and K % 64 == 0 and K >= 192 and act in (0, 1, 2, 3, 4, 5, 7)
+            and not (bias and (N > PGEMM_MAX_BIAS or act in (ACT_SWIGLU, ACT_RELUGLU)))
+            and (bias or act != ACT_RELU2))
 
 
 def pgemm_operands_ok(a: torch.Tensor, w: torch.Tensor) -> bool:
@@ -1804,8 +1831,10 @@ def pgemm_sk(a: torch.Tensor, w: torch.Tensor, splits: int, act: int = 0, epi: i
 
 from .grouped import (GroupedWeight, GroupScores, Mixture, MoePlan, Route,  # noqa: E402,F401
                       grouped_heads, grouped_linear, moe_plan, moe_route, pack_grouped, wide_tiles)
-from .mixers import (RGLRU_MAX_BLOCK, RGLRU_TILE, DeltaChunks, LatentRows,  # noqa: E402,F401
-                     NormedPair, ScanSegments, attention_any, conv_qkv_cache, delta_rule,
-                     gated_norm, latent_attention, latent_prefill, latent_prefill_ok, latent_prep,
-                     latent_query, linear_scan, norm_rope_cache, rglru, rope_angles, rope_freqs,
-                     rope_magnitude, sandwich_norm, scan_segments, short_conv, soft_cap, sum_norm)
+from .mixers import (RGLRU_MAX_BLOCK, RGLRU_TILE, TALK_QT, Biased, DeltaChunks,  # noqa: E402,F401
+                     LatentRows, NormedPair, ScanSegments, Talk, attention_any, conv_qkv_cache,
+                     delta_rule, gated_norm, latent_attention, latent_prefill, latent_prefill_ok,
+                     latent_prep, latent_query, linear_scan, memory_scan, norm_rope_cache,
+                     qkv_norm_rope_cache, rglru, rope_angles, rope_freqs, rope_magnitude,
+                     sandwich_norm, scan_segments, short_conv, soft_cap, sum_norm, talk_kernel_ok,
+                     talking_attention)

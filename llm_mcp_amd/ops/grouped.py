@@ -37,29 +37,43 @@ def pack_grouped(w: torch.Tensor) -> GroupedWeight:
 
 class Mixture:
     """Sublayer output rows as weighted sums of expert rows, left to the
-    consuming kernel: row t = sum_j weights[t, j] rows[pos[t, j]]."""
-    __slots__ = ("rows", "pos", "weights")
+    consuming kernel: row t = sum_j weights[t, j] rows[pos[t, j]] (pos -1: no
+    such row), plus ``own``[t] (fp32 [T], optional) times the stream's own row,
+    which such a sublayer reads as it is."""
+    __slots__ = ("rows", "pos", "weights", "own")
 
-    def __init__(self, rows: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor):
-        self.rows, self.pos, self.weights = rows, pos, weights
+    def __init__(self, rows: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor,
+                 own: torch.Tensor | None = None):
+        self.rows, self.pos, self.weights, self.own = rows, pos, weights, own
 
     def sum(self) -> torch.Tensor:
-        return (self.rows[self.pos.long()].float() * self.weights[..., None]).sum(1)
+        x = self.rows[self.pos.clamp_min(0).long()].float()
+        return (x * (self.weights * (self.pos >= 0))[..., None]).sum(1)
 
 
 @dataclass
 class Route:
-    ids: torch.Tensor        # int32 [T, J] expert of each use
+    ids: torch.Tensor        # int32 [T, J] expert of each use (-1: an identity expert)
     weights: torch.Tensor    # fp32 [T, J]
+    own: torch.Tensor | None = None   # fp32 [T]: weight of a row's identity experts
 
 
 @dataclass
 class GroupScores:
-    """Routing by sigmoid scores s: experts are chosen by s + ``correction``
-    (fp32 [E]) within the ``keep`` best of ``groups`` groups of neighbours."""
+    """Routing by scores s of the logits: experts are chosen by s +
+    ``correction`` (fp32 [E]) within the ``keep`` best of ``groups`` groups of
+    neighbours.
+
+    ``softmax``: s is the softmax over all E logits, a group ranks by its
+    largest corrected score and the weights are the s as they are; otherwise s =
+    sigmoid, a group ranks by the sum of its two largest, the weights are in
+    proportion to s.  ``identity``: that many of the last experts return their
+    input."""
     correction: torch.Tensor
     groups: int = 1
     keep: int = 1
+    softmax: bool = False
+    identity: int = 0
 
 
 def moe_route(h: torch.Tensor, w: torch.Tensor, top: int, extra: int = 0,
@@ -71,7 +85,8 @@ def moe_route(h: torch.Tensor, w: torch.Tensor, top: int, extra: int = 0,
     With ``scores``: the ``top`` largest s + correction, s = sigmoid(w h), among
     the groups with the largest sums of two such scores, in the proportions of
     their s; a row of w behind the E experts' is the logit whose sigmoid weighs
-    the extra ones."""
+    the extra ones.  ``GroupScores`` has the other forms; the identity experts a
+    row chose are in ``Route.own``, not among the uses."""
     rows, d = w.shape
     E = rows if scores is None else scores.correction.numel()
     T = h.shape[0]
@@ -80,13 +95,18 @@ def moe_route(h: torch.Tensor, w: torch.Tensor, top: int, extra: int = 0,
         _chk(E % scores.groups == 0 and scores.groups <= MOE_MAX_GROUPS
              and 0 < scores.keep <= scores.groups and scores.keep * (E // scores.groups) >= top,
              "moe_route: groups")
+        _chk(0 <= scores.identity < E and not (scores.softmax and rows > E),
+             "moe_route: identity experts, router rows")
     if not h.is_cuda:
         return Route(*(ref.moe_route(h, w, top, extra) if scores is None else
                        ref.moe_route_groups(h, w, top, extra, scores)))
     _chk(rows <= MOE_MAX_EXPERTS and top + extra <= MOE_MAX_TOP, "moe_route: sizes")
-    corr, groups, keep = None, 1, 1
+    corr, groups, keep, soft, ident, own = None, 1, 1, 0, 0, None
     if scores is not None:
         corr, groups, keep = scores.correction, scores.groups, scores.keep
+        soft, ident = int(scores.softmax), scores.identity
+        if ident:
+            own = torch.empty(T, dtype=torch.float32, device=h.device)
         _chk(corr.dtype == torch.float32 and corr.is_contiguous() and corr.is_cuda,
              "moe_route: fp32 correction")
     _chk(h.dtype == w.dtype and h.dtype in (torch.bfloat16, torch.float32)
@@ -94,15 +114,16 @@ def moe_route(h: torch.Tensor, w: torch.Tensor, top: int, extra: int = 0,
     ids = torch.empty((T, top + extra), dtype=torch.int32, device=h.device)
     wts = torch.empty((T, top + extra), dtype=torch.float32, device=h.device)
     native().moe_route(_ptr(h), h.stride(0), _ptr(w), T, d, E, rows, top, extra, _ptr(corr), groups,
-                       keep, _ptr(ids), _ptr(wts), int(h.dtype == torch.bfloat16), _stream())
-    return Route(ids, wts)
+                       keep, soft, ident, _ptr(ids), _ptr(wts), _ptr(own),
+                       int(h.dtype == torch.bfloat16), _stream())
+    return Route(ids, wts, own)
 
 
 @dataclass
 class MoePlan:
-    """Uses (row, expert) sorted by expert."""
+    """Uses (row, expert) sorted by expert; those with id -1 are left out."""
     src: torch.Tensor        # int32 [n]: row of each sorted use
-    pos: torch.Tensor        # int32 [T, J]: sorted place of each use
+    pos: torch.Tensor        # int32 [T, J]: sorted place of each use (-1: left out)
     off: torch.Tensor        # int32 [groups + 1]
     tiles: torch.Tensor | None   # int32 [mtiles, 2]: group (-1: none), first sorted row; one
     bm: int                      # more entry: the number of used ones
@@ -129,10 +150,12 @@ def moe_plan(r: Route, groups: int, bf16: bool = True, wide: bool = False) -> Mo
     n = T * J
     ids = r.ids
     if not ids.is_cuda:
-        order = torch.argsort(ids.reshape(-1).long(), stable=True)
+        flat = ids.reshape(-1).long()
+        order = torch.argsort(torch.where(flat < 0, groups, flat), stable=True)
         pos = torch.empty(n, dtype=torch.int32)
         pos[order] = torch.arange(n, dtype=torch.int32)
-        cnt = torch.bincount(ids.reshape(-1).long(), minlength=groups)
+        pos[flat < 0] = -1
+        cnt = torch.bincount(flat[flat >= 0], minlength=groups)
         off = torch.cat([torch.zeros(1, dtype=torch.int64), cnt.cumsum(0)]).to(torch.int32)
         return MoePlan((order // J).to(torch.int32), pos.view(T, J), off, None, 0)
     _chk(0 < groups <= MOE_MAX_EXPERTS and ids.is_contiguous(), "moe_plan")

@@ -54,16 +54,23 @@ def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tens
     """One pass over the fp32 residual stream between two sublayers:
 
         r = scale table[ids] (if given) else residual
-        r += rms(y) * w_post         (y: sublayer output rows, ``Partials`` or ``Mixture``)
+        r += rms(y) * w_post         (y: sublayer output rows, ``Partials``, ``Mixture`` or
+                                      one of them ``Biased``)
         residual = r                 (unless ``rows`` is given)
         return rms(r) * w_pre        (``dtype`` rows; r itself without w_pre)
 
     ``rows`` (int64): only these rows are normed, the residual stays as it is.
     The gains are fp32 vectors."""
     T, d = residual.shape
+    bias = own = None
+    if isinstance(y, Biased):
+        y, bias = y.rows, y.bias
+    if isinstance(y, Mixture):
+        own = y.own
     if not residual.is_cuda:
         y = y.sum()[:, :d] if isinstance(y, Mixture) else y
-        return ref.sandwich_norm(residual, eps, y, w_post, w_pre, ids, table, rows, dtype, scale)
+        return ref.sandwich_norm(residual, eps, y, w_post, w_pre, ids, table, rows, dtype, scale,
+                                 bias, own)
     _chk(residual.dtype == torch.float32 and residual.is_contiguous(), "residual: fp32 rows")
     _f32(w_post, d, "w_post"); _f32(w_pre, d, "w_pre")
     bf = int(dtype == torch.bfloat16)
@@ -81,6 +88,7 @@ def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tens
         _chk(y.shape == (T, d) and y.stride(1) == 1 and y.dtype == dtype, "sandwich_norm y rows")
         yp, y_ld = _ptr(y), y.stride(0)
     _chk((y is None) == (w_post is None), "w_post goes with y")
+    _f32(bias, d, "sublayer bias"); _f32(own, T, "the stream's own weights")
     if ids is not None:
         _chk(ids.dtype == torch.int32 and ids.numel() >= T and table.dtype == dtype
              and table.is_contiguous() and table.shape[1] == d, "embedding rows")
@@ -89,10 +97,20 @@ def sandwich_norm(residual: torch.Tensor, eps: float, y=None, w_post: torch.Tens
         _chk(rows.dtype == torch.int64 and rows.is_contiguous(), "rows: int64")
         n = rows.numel()
     out = torch.empty((n, d), dtype=dtype, device=residual.device)
-    native().sandwich_norm(_ptr(out), _ptr(residual), yp, y_ld, slabs, sstride, *mix, _ptr(ids),
+    native().sandwich_norm(_ptr(out), _ptr(residual), yp, y_ld, slabs, sstride, *mix, _ptr(own),
+                           _ptr(bias), _ptr(ids),
                            _ptr(table), float(scale), _ptr(w_post), _ptr(w_pre), _ptr(rows), n, d,
                            float(eps), bf, _stream())
     return out
+
+
+class Biased:
+    """Sublayer output rows + bias (fp32 [d]), left to the consuming kernel;
+    rows: what ``sandwich_norm`` takes."""
+    __slots__ = ("rows", "bias")
+
+    def __init__(self, rows, bias: torch.Tensor):
+        self.rows, self.bias = rows, bias
 
 
 class NormedPair:
@@ -132,6 +150,8 @@ def sum_norm(residual: torch.Tensor, eps: float, y, alpha: float, scale: torch.T
     ``Partials``, ``Mixture`` or ``NormedPair``; ``rows`` (int64) and the fp32
     vectors as in ``sandwich_norm``."""
     T, d = residual.shape
+    _chk(not isinstance(y, Biased) and getattr(y, "own", None) is None,
+         "sum_norm: no bias, no weight of the stream's own rows")
     if not residual.is_cuda:
         if isinstance(y, Mixture):
             y = y.sum()[:, :d]
@@ -180,19 +200,24 @@ def soft_cap(x: torch.Tensor, scale: float, cap: float | None) -> torch.Tensor:
 
 
 def gated_norm(x: torch.Tensor, gate: torch.Tensor, w: torch.Tensor, groups: int, eps: float,
-               gate_first: bool, silu: bool = False) -> torch.Tensor:
+               gate_first: bool, silu: bool = False,
+               out: torch.Tensor | None = None) -> torch.Tensor:
     """RMS norm of x in ``groups`` equal parts of a row, gain w (fp32), gated:
     rms(x) * w * sigmoid(gate) (``silu``: silu(gate)), or with ``gate_first``
-    rms(x * silu(gate)) * w."""
+    rms(x * silu(gate)) * w.  ``out``: rows to write (any row stride)."""
     T, C = x.shape
     _chk(C % groups == 0, "gated_norm groups")
+    _chk(out is None or (out.shape == (T, C) and out.dtype == x.dtype and out.stride(1) == 1),
+         "gated_norm output rows")
     if not x.is_cuda:
-        return ref.gated_norm(x, gate, w, groups, eps, gate_first, silu)
+        y = ref.gated_norm(x, gate, w, groups, eps, gate_first, silu)
+        return y if out is None else out.copy_(y)
     bf = _rows_dtype(x, "x")
     _f32(w, C, "w")
     _chk(gate.dtype == x.dtype and gate.shape[0] == T and gate.shape[1] >= C
          and gate.stride(1) == 1 and x.stride(1) == 1, "gated_norm rows")
-    out = torch.empty((T, C), dtype=x.dtype, device=x.device)
+    if out is None:
+        out = torch.empty((T, C), dtype=x.dtype, device=x.device)
     native().gated_norm(_ptr(out), out.stride(0), _ptr(x), x.stride(0), _ptr(gate),
                         gate.stride(0), _ptr(w), T, C, groups,
                         1 if gate_first else 2 if silu else 0, float(eps), bf,
@@ -516,6 +541,182 @@ def norm_rope_cache(p: torch.Tensor, q_norm: torch.Tensor, k_norm: torch.Tensor,
     return q
 
 
+# ------------------------------------------------- attention of mixed heads --
+@dataclass
+class Talk:
+    """What talking heads add to attention: the heads' scores mixed, score_h <-
+    sum_g mix[h, g] score_g (scores are already scaled in the queries), and a
+    sink per head, exp(sink_h) more in the softmax's denominator."""
+    mix: torch.Tensor           # [H, H], the model's dtype
+    sink: torch.Tensor          # fp32 [H]
+
+
+TALK_QT = 16                    # query rows per prefill workgroup (talk.hip)
+TALK_MAX_HEADS = 32             # heads of the MFMA kernels (head sizes 64, 128)
+TALK_PART = 128                 # least keys of a decode partition
+
+
+def talk_kernel_ok(Hq: int, Hkv: int, D: int) -> bool:
+    """Geometries of the MFMA kernels (bf16)."""
+    return D in (64, 128) and Hq <= TALK_MAX_HEADS and Hq % Hkv == 0 and Hq // Hkv <= 16
+
+
+def talking_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, ctx, positions,
+                      talk: Talk, Hq: int, gate: torch.Tensor, out: torch.Tensor,
+                      chunk: int = 0, out_scale: float = 1.0, num_decode: int = 0, tiles=None,
+                      ws=None) -> torch.Tensor:
+    """Causal paged attention of every row with mixed heads (``Talk``), decode
+    and prompt rows alike: query rows [T, Hq * D] that carry their scale.
+    ``chunk`` (0: none): a row sees the positions up to its own of its chunk of
+    that many, counted from position 0.  Output rows times out_scale
+    sigmoid(gate) into ``out`` (any row stride).
+
+    Rows before ``num_decode`` are single rows of their sequences; ``tiles``
+    (``row_tiles`` of TALK_QT rows) covers the others.  bf16 rows of
+    ``talk_kernel_ok`` geometries run on MFMA."""
+    _, Hkv, BS, D = k_cache.shape
+    T, S, nd = q.shape[0], ctx.numel(), num_decode
+    _chk(out.shape == (T, Hq * D) and out.dtype == q.dtype and out.stride(1) == 1
+         and gate.dtype == q.dtype and gate.shape[0] == T and gate.shape[1] >= Hq * D
+         and gate.stride(1) == 1 and chunk >= 0, "talking_attention rows")
+    if not q.is_cuda:
+        o = ref.talking_attention(q.reshape(T, Hq, D), k_cache, v_cache, block_tables, cu_q, ctx,
+                                  1.0, talk.mix, talk.sink, chunk).reshape(T, Hq * D).float()
+        return out.copy_(o * torch.sigmoid(gate[:, :Hq * D].float()) * out_scale)
+    bf = _rows_dtype(q, "q")
+    _chk(q.shape[1] == Hq * D and q.is_contiguous() and k_cache.dtype == v_cache.dtype == q.dtype
+         and BS == 32 and D in (64, 128, 256, 512), "talking_attention")
+    _chk(talk.mix.shape == (Hq, Hq) and talk.mix.dtype == q.dtype and talk.mix.is_contiguous(),
+         "talking_attention: head mix")
+    _f32(talk.sink, Hq, "sink")
+    _meta(S, cu_q=cu_q, ctx=ctx)
+    _meta(T, positions=positions)
+    _chk(block_tables.dtype == torch.int32 and block_tables.shape[0] >= S
+         and block_tables.stride(1) == 1, "block tables")
+    k = native()
+    if not bf or not talk_kernel_ok(Hq, Hkv, D):
+        k.talk_any(_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
+                   block_tables.stride(0), _ptr(cu_q), S, _ptr(positions), T, _ptr(talk.mix),
+                   _ptr(talk.sink), _ptr(out), out.stride(0), _ptr(gate), gate.stride(0),
+                   float(out_scale), Hq, Hkv, D, chunk, bf, _stream())
+        return out
+    _chk(out.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0 and gate.stride(0) % 8 == 0
+         and gate.data_ptr() % 16 == 0, "talking_attention: aligned rows")
+    args = (_ptr(k_cache), _ptr(v_cache), _ptr(talk.mix), _ptr(talk.sink), float(out_scale), Hq,
+            Hkv, D, chunk)
+    if nd:
+        parts = ws.max_parts if ws is not None else 1
+        _chk(parts == 1 or (ws.part_o.numel() >= nd * Hq * parts * D
+                            and ws.part_ml.numel() >= nd * Hq * parts * 2),
+             "talking_attention workspace")
+        k.talk_decode(_ptr(q), *args, _ptr(block_tables), block_tables.stride(0), _ptr(ctx), nd,
+                      _ptr(gate), gate.stride(0), _ptr(out), out.stride(0),
+                      _ptr(ws.part_o) if ws else 0, _ptr(ws.part_ml) if ws else 0, TALK_PART,
+                      parts, _stream())
+    if T > nd:
+        _chk(tiles is not None and tiles.dtype == torch.int32 and tiles.is_contiguous(),
+             "talking_attention tiles")
+        k.talk_prefill(_ptr(q), *args, _ptr(block_tables[nd:]), block_tables.stride(0),
+                       _ptr(cu_q[nd:]), _ptr(ctx[nd:]), _ptr(tiles), tiles.numel() // 2,
+                       _ptr(gate), gate.stride(0), _ptr(out), out.stride(0), _stream())
+    return out
+
+
+def qkv_norm_rope_cache(p: torch.Tensor, bias: torch.Tensor, q_norm: torch.Tensor,
+                        k_norm: torch.Tensor, angles: torch.Tensor | None, slots, k_cache, v_cache,
+                        Hq: int, dk: int, dv: int, eps: float,
+                        quads: torch.Tensor | None = None) -> torch.Tensor:
+    """The projection rows' q | k | v heads (each padded to D channels) plus
+    ``bias`` (fp32, all heads): q, and k, RMS-normed over the ``dk`` true
+    channels of all their heads at once (gains fp32 [heads * D], zero in the
+    padding), each head's first channels turned by ``angles`` (neighbours
+    paired); v heads divided by their root mean square over ``dv``.  k and v go
+    to the paged cache at ``slots`` (-1: none).  ``quads`` as in
+    ``norm_rope_cache``.  Returns q rows [T, Hq * D]."""
+    _, Hkv, BS, D = k_cache.shape
+    T, C = p.shape[0], (Hq + 2 * Hkv) * D
+    if not p.is_cuda:
+        return ref.qkv_norm_rope_cache(p, bias, q_norm, k_norm, angles, slots, k_cache, v_cache,
+                                       Hq, dk, dv, eps)
+    bf = _rows_dtype(p, "p")
+    _f32(bias, C, "bias"); _f32(q_norm, Hq * D, "q_norm"); _f32(k_norm, Hkv * D, "k_norm")
+    n = 0
+    if angles is not None:
+        n = angles.shape[1]
+        _f32(angles, T * n, "angles")
+    _meta(T, slots=slots)
+    _chk(p.shape[1] >= C and p.stride(1) == 1 and p.stride(0) % 8 == 0 and p.data_ptr() % 16 == 0
+         and n <= dk <= D and 0 < dv <= D and k_cache.dtype == v_cache.dtype == p.dtype
+         and k_cache.is_contiguous() and v_cache.is_contiguous(), "qkv_norm_rope_cache rows")
+    _chk(quads is None or (quads.dtype == torch.int32 and quads.is_contiguous()
+                           and quads.numel() >= 2), "row quads")
+    q = torch.empty((T, Hq * D), dtype=p.dtype, device=p.device)
+    groups = T if quads is None else quads.numel() - 1
+    native().qkv_norm_rope_cache(_ptr(p), p.stride(0), _ptr(bias), _ptr(q_norm), _ptr(k_norm),
+                                 _ptr(angles), n, _ptr(slots), _ptr(quads), groups, _ptr(q),
+                                 _ptr(k_cache), _ptr(v_cache), Hq, Hkv, D, dk, dv, BS, float(eps),
+                                 bf, _stream())
+    return q
+
+
+# ------------------------------------------------------------ matrix memory --
+def memory_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, ig: torch.Tensor,
+                fg: torch.Tensor, bias: torch.Tensor, cap: float, state, cu_q, ctx, slots,
+                num_decode: int = 0, segments: ScanSegments | None = None) -> torch.Tensor:
+    """Matrix memory with exponential gates over each sequence's rows, from and
+    to ``state`` = (S fp32 [slots, H, N, P], n fp32 [slots, H, N], m fp32
+    [slots, H]), from S = n = m = 0.  Per head, with i = cap tanh((ig + bias[0])
+    / cap), f = ln sigmoid(cap tanh((fg + bias[1]) / cap)) and q scaled by
+    N^-1/2,
+
+        m' = max(f + m, i);  S <- e^(f + m - m') S + e^(i - m') k v^T, n alike;
+        o = S^T q / (max(|n q|, e^-m') + 1e-6)
+
+    q, k: rows of H x N channels, v of H x P, ig and fg of H; bias fp32 [2, H].
+    Sequences before ``num_decode`` (one row each) take the recurrent kernel;
+    the others the chunked MFMA kernel when ``segments`` is given and the shape
+    allows it, the recurrent one otherwise.  Returns rows [T, H * P]."""
+    S_, n_, m_ = state
+    _, H, N, P = S_.shape
+    T, S = q.shape[0], ctx.numel()
+    out = torch.empty((T, H * P), dtype=q.dtype, device=q.device)
+    if not q.is_cuda:
+        ref.memory_scan(q, k, v, ig, fg, bias, cap, out, state, cu_q, ctx, slots)
+        return out
+    bf = _rows_dtype(q, "q")
+    for t, c, name in ((q, H * N, "q"), (k, H * N, "k"), (v, H * P, "v"), (ig, H, "ig"), (fg, H, "fg")):
+        _chk(t.dtype == q.dtype and t.shape[0] == T and t.shape[1] >= c and t.stride(1) == 1,
+             f"memory_scan {name} rows")
+    for t, shape, name in ((S_, (H, N, P), "S"), (n_, (H, N), "n"), (m_, (H,), "m")):
+        _chk(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape[1:]) == shape
+             and t.shape[0] == S_.shape[0], f"memory_scan state {name}")
+    _chk(ig.stride(0) == fg.stride(0) and cap > 0, "memory_scan gates")
+    _f32(bias, 2 * H, "gate bias")
+    _meta(S, cu_q=cu_q, ctx=ctx, slots=slots)
+    args = (_ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(ig), _ptr(fg),
+            ig.stride(0), _ptr(bias), float(cap), _ptr(out), out.stride(0), _ptr(S_), _ptr(n_),
+            _ptr(m_), _ptr(cu_q), _ptr(ctx), _ptr(slots), H, N, P, bf)
+    chunked = segments is not None and S > num_decode and _chunk_ok(N, P, q, k, v)
+    n_rec = num_decode if chunked else S
+    if n_rec:
+        native().memory_scan(*args, 0, n_rec, 0, 0, 0, 0, 0, 0, _stream())
+    if chunked:
+        g = segments
+        _chk(g.segs.dtype == torch.int32 and g.segs.numel() >= 4 * g.n
+             and g.first.dtype == torch.int32 and g.first.numel() == S - num_decode + 1,
+             "scan segments")
+        ws = wn = None
+        # a head of several column tiles chains its segments even where each is a
+        # whole sequence: the tiles share n and m
+        one_pass = g.one_pass and P <= (SCAN_VT if N <= 128 else SCAN_VT // 2)
+        if not one_pass:
+            ws = torch.empty((g.n, H, N, P), dtype=torch.float32, device=q.device)
+            wn = torch.empty((g.n, H, N + 3), dtype=torch.float32, device=q.device)
+        native().memory_scan(*args, num_decode, S - num_decode, _ptr(g.segs), g.n, _ptr(g.first),
+                             int(one_pass), _ptr(ws), _ptr(wn), _stream())
+    return out
+
+
 def attention_any(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, ctx, positions,
                   scale: float, Hq: int, gate: torch.Tensor | None = None, window: int = 0,
                   cap: float = 0.0) -> torch.Tensor:
@@ -604,14 +805,14 @@ def rglru(u: torch.Tensor, y: torch.Tensor, y_bias: torch.Tensor, gates: Grouped
 # --------------------------------------------------------- latent attention --
 def rope_freqs(base: float, dims: int, factor: float = 1.0, original: float = 0.0,
                fast: float = 0.0, slow: float = 0.0, device="cpu") -> torch.Tensor:
-    """base^(-2i / dims), i < dims / 2 (double).  ``original`` > 0: a context of
+    """base^(-2i / dims) / factor, i < dims / 2 (double).  ``original`` > 0: a context of
     that length stretched by ``factor`` -- components that turn ``fast`` times
     and more within it stay, those that turn ``slow`` times and less are divided
     by the factor, a ramp between them."""
     i = torch.arange(dims // 2, dtype=torch.float64, device=device)
     f = torch.exp(-2.0 * math.log(base) / dims * i)
     if not original:
-        return f
+        return f / factor
 
     def turning(times):        # the component that turns that often
         return dims * math.log(original / (2 * math.pi * times)) / (2 * math.log(base))

@@ -186,6 +186,8 @@ def gemm_nt(a, w, bias=None, act=0, residual=None):
         y = torch.nn.functional.silu(y)
     elif act == 4:
         y = torch.nn.functional.gelu(y)
+    elif act == 7:
+        y = torch.relu(y) ** 2
     if residual is not None:
         y = y + residual.float()
     return y.to(a.dtype)
@@ -409,12 +411,18 @@ def _unit(x, eps):
 
 
 def sandwich_norm(residual, eps, y=None, w_post=None, w_pre=None, ids=None, table=None,
-                  rows=None, dtype=torch.bfloat16, scale=1.0):
+                  rows=None, dtype=torch.bfloat16, scale=1.0, bias=None, own=None):
     r = table[ids.long()].float() * scale if ids is not None else residual
+    if y is not None:
+        y = y.float()
+        if bias is not None:
+            y = y + bias
+        if own is not None:
+            y = y + own[:, None] * residual
     if rows is not None:
         r, y = r[rows], None if y is None else y[rows]
     if y is not None:
-        r = r + _unit(y.float(), eps) * w_post
+        r = r + _unit(y, eps) * w_post
     if rows is None:
         residual.copy_(r)
     return (r if w_pre is None else _unit(r, eps) * w_pre).to(dtype)
@@ -652,19 +660,29 @@ def clamped_glu(g, u, limit, act=(1.702, 1.0)):
 
 def moe_route_groups(h, w, top, extra, scores):
     E, n = scores.correction.numel(), scores.groups
-    z = torch.sigmoid(h.float() @ w.float().t())
+    z = h.float() @ w.float().t()
+    z = torch.softmax(z, -1) if scores.softmax else torch.sigmoid(z)
     s, T = z[:, :E], h.shape[0]
     c = s + scores.correction
-    rank = c.view(T, n, E // n).topk(min(2, E // n), -1).values.sum(-1)
+    best = 1 if scores.softmax else min(2, E // n)
+    rank = c.view(T, n, E // n).topk(best, -1).values.sum(-1)
     g = torch.sort(rank, dim=-1, descending=True, stable=True).indices[:, :scores.keep]
     kept = torch.zeros(T, n, dtype=torch.bool).scatter_(1, g, True)
     c = c.masked_fill(~kept.repeat_interleave(E // n, 1), float("-inf"))
     ids = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :top]
     wts = s.gather(1, ids)
-    wts = wts / (wts.sum(-1, keepdim=True) + 1e-20)
+    if not scores.softmax:
+        wts = wts / (wts.sum(-1, keepdim=True) + 1e-20)
+    own = None
+    if scores.identity:
+        E -= scores.identity
+        own = (wts * (ids >= E)).sum(-1)
+        wts = wts * (ids < E)
+        ids = torch.where(ids < E, ids, -1)
     ids = torch.cat([ids, torch.arange(E, E + extra).expand(T, extra)], 1)
-    shared = z[:, E:].expand(T, extra) if z.shape[1] > E else torch.ones(T, extra)
-    return ids.to(torch.int32), torch.cat([wts, shared], 1)
+    shared = z[:, E:].expand(T, extra) if z.shape[1] > scores.correction.numel() \
+        else torch.ones(T, extra)
+    return ids.to(torch.int32), torch.cat([wts, shared], 1), own
 
 
 def moe_route(h, w, top, extra):
@@ -689,3 +707,78 @@ def grouped_rows(x, w, src, off, gather, limit, act=(1.702, 1.0)):
             y = clamped_glu(y[:, :, 0], y[:, :, 1], float(limit[e]), act).reshape(b - a, out.shape[1])
         out[a:b] = y.to(x.dtype)
     return out
+
+
+# ------------------------------- talking heads, matrix memory, projections --
+def qkv_norm_rope_cache(p, bias, q_norm, k_norm, ang, slots, k_cache, v_cache, Hq, dk, dv, eps):
+    """See ops.qkv_norm_rope_cache."""
+    _, Hkv, _, D = k_cache.shape
+    T = p.shape[0]
+    x = (p[:, :(Hq + 2 * Hkv) * D].float() + bias).view(T, -1, D)
+
+    def whole(y, w):
+        inv = torch.rsqrt(y.pow(2).sum((1, 2)) / (y.shape[1] * dk) + eps)
+        return rotate_pairs(y * inv[:, None, None] * w.view(1, -1, D), ang)
+    v = x[:, Hq + Hkv:]
+    v = v * torch.rsqrt(v.pow(2).sum(-1, keepdim=True) / dv + eps)
+    write_cache(whole(x[:, Hq:Hq + Hkv], k_norm), v, slots, k_cache, v_cache)
+    return whole(x[:, :Hq], q_norm).reshape(T, Hq * D).to(p.dtype)
+
+
+def talking_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, scale, talk, sink, chunk):
+    """q [T, Hq, D], every row of the sequences; see ops.talking_attention."""
+    T, H, D = q.shape
+    out = torch.zeros_like(q)
+    for s in range(len(ctx)):
+        a, b, n = int(cu_q[s]), int(cu_q[s + 1]), int(ctx[s])
+        k, v = gather_kv(k_cache, v_cache, block_tables[s], n)
+        per = H // k.shape[1]
+        k, v = (x.float().repeat_interleave(per, 1) for x in (k, v))
+        raw = torch.einsum("thd,nhd->htn", q[a:b].float(), k) * scale
+        if talk is not None:
+            raw = torch.einsum("hg,gtn->htn", talk.float(), raw)
+        p = torch.arange(n - (b - a), n)[:, None]
+        j = torch.arange(n)[None]
+        seen = j <= p
+        if chunk:
+            seen = seen & (j >= p // chunk * chunk)
+        x = raw.masked_fill(~seen, float("-inf"))
+        if sink is not None:
+            x = torch.cat([x, sink.float()[:, None, None].expand(H, b - a, 1)], -1)
+        w = torch.softmax(x, -1)[..., :n]
+        out[a:b] = torch.einsum("htn,nhd->thd", w, v).to(q.dtype)
+    return out
+
+
+def memory_scan(q, k, v, ig, fg, bias, cap, out, state, cu_q, ctx, slots):
+    """See ops.memory_scan; one token after the other, fp32."""
+    S_, n_, m_ = state
+    _, H, N, P = S_.shape
+    T = q.shape[0]
+    qs, ks = (x[:, :H * N].float().view(T, H, N) for x in (q, k))
+    qs, vs = qs * N ** -0.5, v[:, :H * P].float().view(T, H, P)
+    i, f = (cap * torch.tanh((x[:, :H].float() + b) / cap) for x, b in zip((ig, fg), bias))
+    f = torch.nn.functional.logsigmoid(f)
+    for s in range(len(ctx)):
+        a, b, slot = int(cu_q[s]), int(cu_q[s + 1]), int(slots[s])
+        if slot < 0:
+            continue
+        if int(ctx[s]) == b - a:
+            S, n, m = torch.zeros(H, N, P), torch.zeros(H, N), torch.zeros(H)
+        else:
+            S, n, m = S_[slot].clone(), n_[slot].clone(), m_[slot].clone()
+        for t in range(a, b):
+            new = torch.maximum(f[t] + m, i[t])
+            keep, add = torch.exp(f[t] + m - new), torch.exp(i[t] - new)
+            S = keep[:, None, None] * S + (add[:, None] * ks[t])[:, :, None] * vs[t][:, None, :]
+            n = keep[:, None] * n + add[:, None] * ks[t]
+            m = new
+            den = torch.maximum((n * qs[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
+            o = torch.einsum("hnp,hn->hp", S, qs[t]) / den[:, None]
+            out[t, :H * P] = o.reshape(-1).to(out.dtype)
+        S_[slot], n_[slot], m_[slot] = S, n, m
+
+
+def bias_relu2(x, bias):
+    y = torch.relu(x.float() + bias)
+    return (y * y).to(x.dtype)

@@ -38,7 +38,7 @@ def build_parser():
     ap.add_argument("--weights", default="", help="safetensors dir of real weights (optional; a "
                     "--chat-model that is a checkpoint directory brings its own)")
     ap.add_argument("--dtype", default="bfloat16", choices=("bfloat16", "float32"),
-                    help="float32: families that run in it (zegopel, pikesun, refolix)")
+                    help="float32: families that run in it (zegopel, pikesun, refolix, zovozen)")
     ap.add_argument("--embed-weights", default="",
                     help="safetensors dir of the embedding model (nomic-bert or BERT; optional)")
     ap.add_argument("--tp", type=int, default=1)
