@@ -73,13 +73,11 @@ struct ScanArgs {
   float *sn, *sm;            // [slots][H][N], [slots][H]
 };
 
-// logarithms of the gates: cap tanh((x + b) / cap), and ln sigmoid of such a value
-template <typename T>
-__device__ __forceinline__ void memory_gates(const ScanArgs& a, long row, int h, float& i, float& f) {
-  const float x = ld1((const T*)a.ig + row * a.gate_ld + h) + a.gate_bias[h];
-  const float y = ld1((const T*)a.fg + row * a.gate_ld + h) + a.gate_bias[a.H + h];
-  i = a.cap * tanhf(x / a.cap);
-  const float z = a.cap * tanhf(y / a.cap);
+// logarithms of the gates from their projections (biased): cap tanh(x / cap), and
+// ln sigmoid of such a value
+__device__ __forceinline__ void memory_gates(float cap, float& i, float& f) {
+  i = cap * tanhf(i / cap);
+  const float z = cap * tanhf(f / cap);
   f = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
 }
 
@@ -275,8 +273,10 @@ __global__ void __launch_bounds__(BT) memory_recurrent_kernel(ScanArgs a, int se
     for (int i = tid; i < N; i += BT) sn[i] = fresh ? 0.f : a.sn[head * N + i];
     m = m0;
     for (int t = 0; t < n; ++t) {
-      float ig, f;
-      memory_gates<T>(a, row0 + t, h, ig, f);
+      const long at = (row0 + t) * a.gate_ld + h;
+      float ig = ld1((const T*)a.ig + at) + a.gate_bias[h];
+      float f = ld1((const T*)a.fg + at) + a.gate_bias[a.H + h];
+      memory_gates(a.cap, ig, f);
       const float mn = fmaxf(f + m, ig), keep = expf(f + m - mn), add = expf(ig - mn);
       m = mn;
       float dot = 0.f;
@@ -504,7 +504,7 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
   // written 4 tokens (8 B) at a time ----
   constexpr int KITEMS = 16 * NP, ITEMS = KITEMS + 2 * VT, NI = (ITEMS + 255) / 256;
   u32x4_t rq[MODE == 1 ? 1 : NK], ri[NI][4];
-  float rdt = 0.f, rfg = 0.f;              // MEM: logarithms of the gates, log2
+  float rdt = 0.f, rfg = 0.f;              // MEM: both gates' projections
   const u32x4_t zero4 = {0, 0, 0, 0};
   // per-thread byte offsets from wave-uniform row bases (a chunk is far below 4 GB)
   static_assert(256 % NP == 0, "a q pass is whole rows");
@@ -544,9 +544,9 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
     }
     if constexpr (MEM) {
       if (tid < SC && t0 + tid < n) {
-        memory_gates<bf16_t>(a, row0 + t0 + tid, h, rdt, rfg);
-        rdt *= SCAN_LOG2E;
-        rfg *= SCAN_LOG2E;
+        const long at = (row0 + t0 + tid) * a.gate_ld + h;
+        rdt = bf2f(((const bf16_t*)a.ig)[at]);
+        rfg = bf2f(((const bf16_t*)a.fg)[at]);
       }
     } else {
       if (dt && tid < SC) rdt = t0 + tid < n ? bf2f(dt[(long)(t0 + tid) * a.dt_ld]) : 0.f;
@@ -586,13 +586,16 @@ __global__ void __launch_bounds__(256, NK <= 4 ? 2 : 1) scan_chunk_kernel(ScanAr
       }
     }
     if (MEM && wave == 0) {
-      float f = lane < m ? rfg : 0.f, b = 0.f;     // rows past the end neither decay nor add
+      __builtin_amdgcn_sched_barrier(0);
+      float ig = rdt + a.gate_bias[h], f = rfg + a.gate_bias[a.H + h];
+      memory_gates(a.cap, ig, f);
+      f = lane < m ? f * SCAN_LOG2E : 0.f;       // rows past the end neither decay nor add
 #pragma unroll
       for (int o = 1; o < 64; o <<= 1) {
         const float y = __shfl_up(f, o, 64);
         if (lane >= o) f += y;
       }
-      b = lane < m ? f - rdt : INFINITY;
+      const float b = lane < m ? f - ig * SCAN_LOG2E : INFINITY;
       float mx = fmaxf(mrun, -b);
 #pragma unroll
       for (int o = 1; o < 64; o <<= 1) {

@@ -8,10 +8,10 @@
 // bf16 rows on MFMA, fp32 everywhere else: raw scores enter the mixing product,
 // and softmax weights the product with V, as a bf16 pair (high part + remainder,
 // 2^-17); the mix is bf16 as stored.
-//   talk_prefill  16 query rows x all heads per workgroup, a 32-key page at a
+//   talk_prefill  8 query rows x all heads per workgroup, a 32-key page at a
 //                 time: wave w scores its heads (columns = queries), the raw
-//                 scores go through LDS to the wave that mixes and softmaxes two
-//                 queries' heads (columns = heads), the weights go back through
+//                 scores go through LDS to the wave that mixes and softmaxes one
+//                 query's heads (columns = heads), the weights go back through
 //                 LDS to the heads' waves for the product with V.
 //   talk_decode   one row per workgroup, wave w = key heads w, w + W, ..: raw
 //                 scores of a page through LDS, then every wave mixes its own
@@ -67,33 +67,53 @@ __device__ __forceinline__ void split1(float x, uint16_t& hi, uint16_t& lo) {
   lo = f2bf(x - bf2f(hi));
 }
 
+// two values to packed bf16, one instruction
+__device__ __forceinline__ uint32_t cvt_pk(float a, float b) {
+  uint32_t r;
+  asm("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r) : "v"(a), "v"(b));
+  return r;
+}
+__device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
+  hi = cvt_pk(a, b);
+  lo = cvt_pk(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
+}
+
 // four outputs of a row's head times the gate
 __device__ __forceinline__ void store_gated(const TalkArgs& a, long row, long col, const f32x4_t& o) {
   const bf16x4_t gv = *reinterpret_cast<const bf16x4_t*>((const bf16_t*)a.gate + row * a.gate_ld + col);
   bf16x4_t w;
 #pragma unroll
   for (int r = 0; r < 4; ++r)
-    w[r] = (short)f2bf(o[r] * a.out_scale / (1.f + __expf(-bf2f((uint16_t)gv[r]))));
+    w[r] = (short)f2bf(o[r] * a.out_scale *
+                       __builtin_amdgcn_rcpf(1.f + fast_exp2(-LOG2E * bf2f((uint16_t)gv[r]))));
   *reinterpret_cast<bf16x4_t*>((bf16_t*)a.out + row * a.out_ld + col) = w;
 }
 
 // --------------------------------------------------------------- prefill ----
-constexpr int TQ = 16;       // query rows per workgroup
+constexpr int TQ = 8;        // query rows per workgroup
 constexpr int TW = 8;        // waves
 
-// HPW: heads per wave (Hq <= 8 HPW).  grid (tiles), block 512.
-template <int HD, int HPW>
+// HPW: heads per wave (Hq <= 8 HPW), from h0 = HPW wave on.  A column group is 8
+// queries (c % 8) x two heads (c / 8): group i holds head h0 + 2 (c / 8) + i of 4,
+// h0 + c / 8 of 2, h0 of 1 (its other half idle).  Between two barriers a wave
+// scores the next page, mixes this one and weighs the one before, through two
+// images each.  SHARED: a wave's heads have one key head, whose pages are loaded
+// ahead: K once a page's scores are made, V once its product is.  grid (tiles),
+// block 512.
+template <int HD, int HPW, bool SHARED>
 __global__ void __launch_bounds__(64 * TW, 2) talk_prefill_kernel(
     TalkArgs a, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
     const int* __restrict__ tiles) {
   extern __shared__ __attribute__((aligned(16))) char talk_sm[];
-  constexpr int KS = HD / 32, NT = HD / 16, HT = HPW > 1 ? HPW / 2 : 1;
-  char* const sS = talk_sm;                              // raw scores: group = query, row = key
-  char* const sP = talk_sm + TQ * PAIR_GROUP;            // weights: group = query, row = head
-  float* const sAl = reinterpret_cast<float*>(sP + TQ * PAIR_GROUP);    // [32 heads][16]
-  const int tile = gridDim.x - 1 - blockIdx.x;           // long walks first
+  constexpr int KS = HD / 32, NT = HD / 16, HT = HPW > 1 ? HPW / 2 : 1, NG = HPW == 4 ? 2 : 1;
+  constexpr int IMG = TQ * PAIR_GROUP;
+  char* const sS = talk_sm;                              // 2 x raw scores: group = query, row = key
+  char* const sP = talk_sm + 2 * IMG;                    // 2 x weights: group = query, row = head
+  float* const sAl = reinterpret_cast<float*>(sP + 2 * IMG);    // 2 x [32 heads][8]
+  // neighbouring tiles, which walk the same pages, on one XCD; long walks first
+  const int tile = gridDim.x - 1 - xcd_remap(blockIdx.x, gridDim.x);
   const int seq = tiles[2 * tile], q0 = tiles[2 * tile + 1];
-  const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
+  const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4, cq = c & 7, cs = c >> 3;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int qbeg = cu_q[seq], qlen = cu_q[seq + 1] - qbeg, ctx = ctx_lens[seq];
   const int p0 = ctx - qlen + q0, p1 = ctx - qlen + min(q0 + TQ, qlen) - 1;   // positions
@@ -102,195 +122,236 @@ __global__ void __launch_bounds__(64 * TW, 2) talk_prefill_kernel(
   const int Hq = a.Hq, Hkv = a.Hkv, G = Hq / Hkv, h0 = wave * HPW;
   const bf16_t* kc = (const bf16_t*)a.kc;
   const bf16_t* vc = (const bf16_t*)a.vc;
+  auto head = [&](int i, int s) { return h0 + (HPW == 4 ? 2 * s + i : HPW == 2 ? s : 0); };
+  auto mine = [&](int i) { return head(i, cs) < Hq && (HPW > 1 || cs == 0); };   // this lane's column
 
-  for (int i = threadIdx.x; i < TQ * PAIR_GROUP / 16; i += 64 * TW)   // heads that do not exist
-    reinterpret_cast<f32x4_t*>(sS)[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  if constexpr (HPW < 4) {                               // heads that do not exist
+    for (int i = threadIdx.x; i < 2 * IMG / 16; i += 64 * TW)
+      reinterpret_cast<f32x4_t*>(sS)[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
 
-  // this wave's heads: queries as columns
-  bf16x8_t qf[HPW][KS];
+  bf16x8_t qf[NG][KS];
 #pragma unroll
-  for (int i = 0; i < HPW; ++i) {
-    const bool on = h0 + i < Hq && q0 + c < qlen;
-    const bf16_t* qr = (const bf16_t*)a.q + ((long)(qbeg + (on ? q0 + c : 0)) * Hq + (on ? h0 + i : 0)) * HD;
+  for (int i = 0; i < NG; ++i) {
+    const bool on = mine(i) && q0 + cq < qlen;
+    const bf16_t* qr = (const bf16_t*)a.q +
+                       ((long)(qbeg + (on ? q0 + cq : 0)) * Hq + (on ? head(i, cs) : 0)) * HD;
 #pragma unroll
     for (int s = 0; s < KS; ++s)
       qf[i][s] = on ? load_frag16B(qr + 32 * s + 8 * g) : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
   }
-  // mixing: queries 2 wave, 2 wave + 1, heads as columns
+  // mixing: query `wave`, heads as columns
   bf16x8_t mf[HT];
-  float m[2][HT], l[2][HT];
-  int lim[2], lo[2];
+  float m[HT], l[HT];
 #pragma unroll
   for (int t = 0; t < HT; ++t) {
     const int h = 16 * t + c;
     mf[t] = mix_frag((const bf16_t*)a.mix, Hq, h, h < Hq, g);
-#pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      m[u][t] = h < Hq ? a.sink[h] * LOG2E : 0.f;        // the sink opens the sum
-      l[u][t] = 1.f;
-    }
+    m[t] = h < Hq ? a.sink[h] * LOG2E : 0.f;             // the sink opens the sum
+    l[t] = 1.f;
   }
+  const int lim = q0 + wave < qlen ? ctx - qlen + q0 + wave : -1;
+  const int lo = chunk_first(a.chunk, max(lim, 0));
+  f32x4_t acc[NG][NT];
 #pragma unroll
-  for (int u = 0; u < 2; ++u) {
-    const int qi = q0 + 2 * wave + u;
-    lim[u] = qi < qlen ? ctx - qlen + qi : -1;
-    lo[u] = chunk_first(a.chunk, max(lim[u], 0));
-  }
-  f32x4_t acc[HPW][NT];
-#pragma unroll
-  for (int i = 0; i < HPW; ++i)
+  for (int i = 0; i < NG; ++i)
 #pragma unroll
     for (int n = 0; n < NT; ++n) acc[i][n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  lds_barrier();
 
-  for (int pg = pg0; pg <= pg1; ++pg) {
-    const long blk = bt[pg];
-    // ---- raw scores of the wave's heads: rows = keys, columns = queries ----
-    if (h0 < Hq) {
-      f32x4_t s[HPW][2];
-      bf16x8_t ka[KS], kb[KS];
-      int have = -1;
+  bf16x8_t ka[KS], kb[KS], vf[NT];
+  const int kvw = min(h0, Hq - 1) / G;                   // SHARED: the wave's key head
+  auto load_k = [&](long blk, int kv) {
+    const bf16_t* kp = kc + (blk * Hkv + kv) * (BS * HD);
 #pragma unroll
-      for (int i = 0; i < HPW; ++i) {
-        s[i][0] = s[i][1] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-        if (h0 + i < Hq) {
-          const int kv = (h0 + i) / G;
-          if (kv != have) {
-            const bf16_t* kp = kc + (blk * Hkv + kv) * (BS * HD);
+    for (int t = 0; t < KS; ++t) {
+      ka[t] = load_frag16B(kp + c * HD + 32 * t + 8 * g);
+      kb[t] = load_frag16B(kp + (16 + c) * HD + 32 * t + 8 * g);
+    }
+  };
+  auto load_v = [&](long blk, int kv) {
+    const bf16_t* vp = vc + (blk * Hkv + kv) * (BS * HD);
 #pragma unroll
-            for (int t = 0; t < KS; ++t) {
-              ka[t] = load_frag16B(kp + c * HD + 32 * t + 8 * g);
-              kb[t] = load_frag16B(kp + (16 + c) * HD + 32 * t + 8 * g);
-            }
-            have = kv;
-          }
+    for (int n = 0; n < NT; ++n)
+      vf[n] = load_frag_2x8B(vp + vq_off(16 * n + c, 8 * g, HD), vp + vq_off(16 * n + c, 8 * g + 4, HD));
+  };
+  // raw scores of the wave's heads: rows = keys, columns = (head, query)
+  auto score = [&](int pg, char* img, int ahead) {       // ahead: block of the page to load
+    f32x4_t s[NG][2];
+#pragma unroll
+    for (int i = 0; i < NG; ++i) {
+      s[i][0] = s[i][1] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if constexpr (SHARED) {
+#pragma unroll
+        for (int t = 0; t < KS; ++t) {
+          s[i][0] = mfma16(ka[t], qf[i][t], s[i][0]);
+          s[i][1] = mfma16(kb[t], qf[i][t], s[i][1]);
+        }
+      } else {
+        const long blk = bt[pg];
+#pragma unroll
+        for (int half = 0; half < 2; ++half) {
+          load_k(blk, min(head(i, half), Hq - 1) / G);
+          f32x4_t x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int t = 0; t < KS; ++t) {
-            s[i][0] = mfma16(ka[t], qf[i][t], s[i][0]);
-            s[i][1] = mfma16(kb[t], qf[i][t], s[i][1]);
+            x = mfma16(ka[t], qf[i][t], x);
+            y = mfma16(kb[t], qf[i][t], y);
+          }
+          s[i][0] = cs == half ? x : s[i][0];
+          s[i][1] = cs == half ? y : s[i][1];
+        }
+      }
+    }
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = 16 * b + 4 * g + r, h = head(0, cs);
+        char* ph = img + pair_off(cq, key, h >> 3) + 2 * (h & 7);
+        char* pl = img + pair_off(cq, key, 4 + (h >> 3)) + 2 * (h & 7);
+        if constexpr (NG == 2) {
+          uint32_t hi, lw;
+          split2(s[0][b][r], s[NG - 1][b][r], hi, lw);
+          *reinterpret_cast<uint32_t*>(ph) = hi;
+          *reinterpret_cast<uint32_t*>(pl) = lw;
+        } else {
+          uint16_t hi, lw;
+          split1(s[0][b][r], hi, lw);
+          if (HPW > 1 || cs == 0) {
+            *reinterpret_cast<uint16_t*>(ph) = hi;
+            *reinterpret_cast<uint16_t*>(pl) = lw;
           }
         }
       }
+    if (SHARED) load_k(ahead, kvw);
+  };
+  // a query: mix (rows = keys, columns = heads), softmax
+  auto mix = [&](int pg, const char* img, char* pimg, float* al_img) {
+    f32x4_t x[HT][2];
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      const bf16x8_t sh = *reinterpret_cast<const bf16x8_t*>(img + pair_off(wave, 16 * b + c, g));
+      const bf16x8_t sl = *reinterpret_cast<const bf16x8_t*>(img + pair_off(wave, 16 * b + c, 4 + g));
+#pragma unroll
+      for (int t = 0; t < HT; ++t) {
+        x[t][b] = mfma16(sh, mf[t], f32x4_t{0.f, 0.f, 0.f, 0.f});
+        x[t][b] = mfma16(sl, mf[t], x[t][b]);
+      }
+    }
+    // a page of which every key is seen needs no mask
+    if (pg * BS + BS - 1 > lim || pg * BS < lo) {
 #pragma unroll
       for (int b = 0; b < 2; ++b)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          uint16_t hi[HPW], lw[HPW];
+          const int key = pg * BS + 16 * b + 4 * g + r;
 #pragma unroll
-          for (int i = 0; i < HPW; ++i) split1(s[i][b][r], hi[i], lw[i]);
-          const int key = 16 * b + 4 * g + r, piece = 2 * h0 / 16, sub = 2 * h0 % 16;
-          char* ph = sS + pair_off(c, key, piece) + sub;
-          char* pl = sS + pair_off(c, key, 4 + piece) + sub;
-          if constexpr (HPW == 4) {
-            *reinterpret_cast<uint2*>(ph) = make_uint2(hi[0] | hi[1] << 16, hi[2] | hi[3] << 16);
-            *reinterpret_cast<uint2*>(pl) = make_uint2(lw[0] | lw[1] << 16, lw[2] | lw[3] << 16);
-          } else if constexpr (HPW == 2) {
-            *reinterpret_cast<uint32_t*>(ph) = hi[0] | hi[1] << 16;
-            *reinterpret_cast<uint32_t*>(pl) = lw[0] | lw[1] << 16;
-          } else {
-            *reinterpret_cast<uint16_t*>(ph) = hi[0];
-            *reinterpret_cast<uint16_t*>(pl) = lw[0];
-          }
+          for (int t = 0; t < HT; ++t)
+            if (key > lim || key < lo) x[t][b][r] = -INFINITY;
         }
     }
-    lds_barrier();
-    // ---- two queries: mix (rows = keys, columns = heads), softmax ----
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int qi = 2 * wave + u;
-      f32x4_t x[HT][2];
+    for (int t = 0; t < HT; ++t) {
+      const f32x4_t &u = x[t][0], &v = x[t][1];
+      const float mx = max3f(max3f(u[0], u[1], u[2]), max3f(u[3], v[0], v[1]), max2f(v[2], v[3]));
+      const float mn = max2f(m[t], col4_max(mx) * LOG2E);
+      const float al = fast_exp2(m[t] - mn);
+      m[t] = mn;
+      float sum = 0.f;
 #pragma unroll
       for (int b = 0; b < 2; ++b) {
-        const bf16x8_t sh = *reinterpret_cast<const bf16x8_t*>(sS + pair_off(qi, 16 * b + c, g));
-        const bf16x8_t sl = *reinterpret_cast<const bf16x8_t*>(sS + pair_off(qi, 16 * b + c, 4 + g));
+        float w[4];
 #pragma unroll
-        for (int t = 0; t < HT; ++t) {
-          x[t][b] = mfma16(sh, mf[t], f32x4_t{0.f, 0.f, 0.f, 0.f});
-          x[t][b] = mfma16(sl, mf[t], x[t][b]);
+        for (int r = 0; r < 4; ++r) {
+          w[r] = fast_exp2(x[t][b][r] * LOG2E - mn);
+          sum += w[r];
         }
+        uint32_t h01, l01, h23, l23;
+        split2(w[0], w[1], h01, l01);
+        split2(w[2], w[3], h23, l23);
+        const int h = 16 * t + c, piece = 2 * b + (g >> 1), sub = 8 * (g & 1);
+        *reinterpret_cast<uint2*>(pimg + pair_off(wave, h, piece) + sub) = make_uint2(h01, h23);
+        *reinterpret_cast<uint2*>(pimg + pair_off(wave, h, 4 + piece) + sub) = make_uint2(l01, l23);
       }
+      l[t] = l[t] * al + col4_sum(sum);
+      if (g == 0) al_img[(16 * t + c) * TQ + wave] = al;
+    }
+  };
+  // weights times V: rows = channels, columns = (head, query)
+  auto weigh = [&](int pg, const char* pimg, const float* al_img, int ahead) {
 #pragma unroll
-      for (int t = 0; t < HT; ++t) {
-        float mx = -INFINITY;
+    for (int i = 0; i < NG; ++i) {
+      const int h = head(i, cs);                       // beyond Hq: a row of the image all the same
+      const bf16x8_t ph = *reinterpret_cast<const bf16x8_t*>(pimg + pair_off(cq, h, g));
+      const bf16x8_t pl = *reinterpret_cast<const bf16x8_t*>(pimg + pair_off(cq, h, 4 + g));
+      const float al = al_img[h * TQ + cq];
 #pragma unroll
-        for (int b = 0; b < 2; ++b)
+      for (int n = 0; n < NT; ++n) acc[i][n] *= al;
+      if constexpr (SHARED) {
 #pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const int key = pg * BS + 16 * b + 4 * g + r;
-            x[t][b][r] = key <= lim[u] && key >= lo[u] ? x[t][b][r] * LOG2E : -INFINITY;
-            mx = fmaxf(mx, x[t][b][r]);
-          }
-        const float mn = fmaxf(m[u][t], col4_max(mx));
-        const float al = fast_exp2(m[u][t] - mn);
-        m[u][t] = mn;
-        float sum = 0.f;
-#pragma unroll
-        for (int b = 0; b < 2; ++b) {
-          uint16_t hi[4], lw[4];
-#pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const float p = fast_exp2(x[t][b][r] - mn);
-            sum += p;
-            split1(p, hi[r], lw[r]);
-          }
-          const int h = 16 * t + c, piece = 2 * b + (g >> 1), sub = 8 * (g & 1);
-          *reinterpret_cast<uint2*>(sP + pair_off(qi, h, piece) + sub) =
-              make_uint2(hi[0] | hi[1] << 16, hi[2] | hi[3] << 16);
-          *reinterpret_cast<uint2*>(sP + pair_off(qi, h, 4 + piece) + sub) =
-              make_uint2(lw[0] | lw[1] << 16, lw[2] | lw[3] << 16);
+        for (int n = 0; n < NT; ++n) {
+          acc[i][n] = mfma16(vf[n], ph, acc[i][n]);
+          acc[i][n] = mfma16(vf[n], pl, acc[i][n]);
         }
-        l[u][t] = l[u][t] * al + col4_sum(sum);
-        if (g == 0) sAl[(16 * t + c) * 16 + qi] = al;
+      } else {
+        const bf16x8_t zero = {0, 0, 0, 0, 0, 0, 0, 0};
+        const long blk = bt[pg];
+#pragma unroll
+        for (int half = 0; half < 2; ++half) {
+          load_v(blk, min(head(i, half), Hq - 1) / G);
+#pragma unroll
+          for (int n = 0; n < NT; ++n) {
+            acc[i][n] = mfma16(vf[n], cs == half ? ph : zero, acc[i][n]);
+            acc[i][n] = mfma16(vf[n], cs == half ? pl : zero, acc[i][n]);
+          }
+        }
       }
     }
+    if (SHARED) load_v(ahead, kvw);
+  };
+  // block ids: lane i holds page base + i
+  int base = pg0, ids = bt[min(pg0 + lane, pg1)];
+  asm volatile("" : "+v"(ids));                          // landed before the loop's loads are counted
+  auto page = [&](int pg) { return __builtin_amdgcn_readlane(ids, min(pg, pg1) - base); };
+  if (SHARED) load_k(page(pg0), kvw);
+  lds_barrier();                                         // the zeros are in place
+  score(pg0, sS, page(pg0 + 1));
+  lds_barrier();
+  score(min(pg0 + 1, pg1), sS + IMG, page(pg0 + 2));
+  // in the order of the loop's loads, K before V: the waits are counted
+  __builtin_amdgcn_sched_barrier(0);
+  if (SHARED) load_v(page(pg0), kvw);
+  mix(pg0, sS, sP, sAl);
+  lds_barrier();
+  int cur = 1;                                           // image of this page
+  for (int pg = pg0 + 1; pg <= pg1; ++pg, cur ^= 1) {
+    if (pg - base >= 32) {
+      base = pg;
+      ids = bt[min(pg + lane, pg1)];
+      asm volatile("" : "+v"(ids));
+    }
+    score(min(pg + 1, pg1), sS + (cur ^ 1) * IMG, page(pg + 2));
+    mix(pg, sS + cur * IMG, sP + cur * IMG, sAl + cur * 32 * TQ);
+    weigh(pg - 1, sP + (cur ^ 1) * IMG, sAl + (cur ^ 1) * 32 * TQ, page(pg));
     lds_barrier();
-    // ---- weights times V: rows = channels, columns = queries ----
-    if (h0 < Hq) {
-      bf16x8_t ph[HPW], pl[HPW];
-#pragma unroll
-      for (int i = 0; i < HPW; ++i) {
-        const int h = h0 + i;
-        ph[i] = *reinterpret_cast<const bf16x8_t*>(sP + pair_off(c, h, g));
-        pl[i] = *reinterpret_cast<const bf16x8_t*>(sP + pair_off(c, h, 4 + g));
-        const float al = sAl[h * 16 + c];
-#pragma unroll
-        for (int n = 0; n < NT; ++n) acc[i][n] *= al;
-      }
-      const bool shared = h0 / G == (min(h0 + HPW, Hq) - 1) / G;      // one key head
-#pragma unroll
-      for (int n = 0; n < NT; ++n) {
-        const int d = 16 * n + c;
-        bf16x8_t vf;
-#pragma unroll
-        for (int i = 0; i < HPW; ++i) {
-          if (h0 + i >= Hq) continue;
-          if (i == 0 || !shared) {
-            const bf16_t* vp = vc + (blk * Hkv + (h0 + i) / G) * (BS * HD);
-            vf = load_frag_2x8B(vp + vq_off(d, 8 * g, HD), vp + vq_off(d, 8 * g + 4, HD));
-          }
-          acc[i][n] = mfma16(vf, ph[i], acc[i][n]);
-          acc[i][n] = mfma16(vf, pl[i], acc[i][n]);
-        }
-      }
-    }
   }
+  weigh(pg1, sP + (cur ^ 1) * IMG, sAl + (cur ^ 1) * 32 * TQ, page(pg1));
   // the weights' sums go to the heads' waves
   lds_barrier();
 #pragma unroll
-  for (int u = 0; u < 2; ++u)
-#pragma unroll
-    for (int t = 0; t < HT; ++t)
-      if (g == 0) sAl[(16 * t + c) * 16 + 2 * wave + u] = 1.f / l[u][t];
+  for (int t = 0; t < HT; ++t)
+    if (g == 0) sAl[(16 * t + c) * TQ + wave] = 1.f / l[t];
   lds_barrier();
-  if (q0 + c < qlen) {
-    const long row = qbeg + q0 + c;
+  if (q0 + cq < qlen) {
+    const long row = qbeg + q0 + cq;
 #pragma unroll
-    for (int i = 0; i < HPW; ++i) {
-      if (h0 + i >= Hq) continue;
-      const float inv = sAl[(h0 + i) * 16 + c];
+    for (int i = 0; i < NG; ++i) {
+      if (!mine(i)) continue;
+      const int h = head(i, cs);
+      const float inv = sAl[h * TQ + cq];
 #pragma unroll
       for (int n = 0; n < NT; ++n)
-        store_gated(a, row, (long)(h0 + i) * HD + 16 * n + 4 * g, acc[i][n] * inv);
+        store_gated(a, row, (long)h * HD + 16 * n + 4 * g, acc[i][n] * inv);
     }
   }
 }
@@ -337,21 +398,16 @@ __global__ void __launch_bounds__(512) talk_decode_kernel(TalkArgs a, const int*
 #pragma unroll
     for (int n = 0; n < NT; ++n) acc[i][n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   }
-  bf16x8_t ka[KPW][KS], kb[KPW][KS];
-  auto load_k = [&](int pg) {
-    const long blk = bt[pg];
+  bf16x8_t ka[KS], kb[KS];             // one key head per wave: a page ahead
+  auto load_k = [&](long blk, int kv) {
+    const bf16_t* kp = kc + (blk * Hkv + min(kv, Hkv - 1)) * (BS * HD);
 #pragma unroll
-    for (int i = 0; i < KPW; ++i) {
-      const int kv = min(wave + i * W, Hkv - 1);
-      const bf16_t* kp = kc + (blk * Hkv + kv) * (BS * HD);
-#pragma unroll
-      for (int t = 0; t < KS; ++t) {
-        ka[i][t] = load_frag16B(kp + c * HD + 32 * t + 8 * g);
-        kb[i][t] = load_frag16B(kp + (16 + c) * HD + 32 * t + 8 * g);
-      }
+    for (int t = 0; t < KS; ++t) {
+      ka[t] = load_frag16B(kp + c * HD + 32 * t + 8 * g);
+      kb[t] = load_frag16B(kp + (16 + c) * HD + 32 * t + 8 * g);
     }
   };
-  load_k(pg0);
+  if (KPW == 1) load_k(bt[pg0], wave);
   lds_barrier();
   for (int pg = pg0; pg < pg1; ++pg) {
     char* const img = sS[(pg - pg0) & 1];
@@ -366,12 +422,14 @@ __global__ void __launch_bounds__(512) talk_decode_kernel(TalkArgs a, const int*
     // raw scores: rows = the key head's query heads, columns = keys
 #pragma unroll
     for (int i = 0; i < KPW; ++i) {
+      if (KPW > 1) __builtin_amdgcn_sched_barrier(0);    // one key head's operands at a time
       const int kv = wave + i * W;
       f32x4_t s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+      if (KPW > 1) load_k(blk, kv);
 #pragma unroll
       for (int t = 0; t < KS; ++t) {
-        s[0] = mfma16(qf[i][t], ka[i][t], s[0]);
-        s[1] = mfma16(qf[i][t], kb[i][t], s[1]);
+        s[0] = mfma16(qf[i][t], ka[t], s[0]);
+        s[1] = mfma16(qf[i][t], kb[t], s[1]);
       }
       if (kv < Hkv) {
 #pragma unroll
@@ -387,7 +445,7 @@ __global__ void __launch_bounds__(512) talk_decode_kernel(TalkArgs a, const int*
           }
       }
     }
-    if (pg + 1 < pg1) load_k(pg + 1);
+    if (KPW == 1 && pg + 1 < pg1) load_k(bt[pg + 1], wave);
     lds_barrier();
     bf16x8_t sh[2], sl[2];
 #pragma unroll
@@ -397,6 +455,7 @@ __global__ void __launch_bounds__(512) talk_decode_kernel(TalkArgs a, const int*
     }
 #pragma unroll
     for (int i = 0; i < KPW; ++i) {
+      if (KPW > 1) __builtin_amdgcn_sched_barrier(0);
       const int kv = min(wave + i * W, Hkv - 1);
       float x[8], mx = -INFINITY;
 #pragma unroll
@@ -562,19 +621,27 @@ bool talk_mfma_ok(const TalkArgs& a, int D) {
          a.out_ld % 8 == 0 && !(((uintptr_t)a.q | (uintptr_t)a.gate | (uintptr_t)a.out) & 15);
 }
 
-template <int HD, int HPW>
-int launch_prefill(const TalkArgs& a, const int* cu_q, const int* ctx, const int* tiles, int n,
-                   hipStream_t stream) {
-  constexpr int smem = 2 * TQ * PAIR_GROUP + 32 * 16 * 4;
+template <int HD, int HPW, bool SHARED>
+int launch_prefill_as(const TalkArgs& a, const int* cu_q, const int* ctx, const int* tiles, int n,
+                      hipStream_t stream) {
+  constexpr int smem = 4 * TQ * PAIR_GROUP + 2 * 32 * TQ * 4;
   static bool attr = false;
   if (!attr) {
-    const hipError_t e = hipFuncSetAttribute((const void*)talk_prefill_kernel<HD, HPW>,
+    const hipError_t e = hipFuncSetAttribute((const void*)talk_prefill_kernel<HD, HPW, SHARED>,
                                              hipFuncAttributeMaxDynamicSharedMemorySize, smem);
     if (e != hipSuccess) return (int)e;
     attr = true;
   }
-  talk_prefill_kernel<HD, HPW><<<dim3(n), dim3(64 * TW), smem, stream>>>(a, cu_q, ctx, tiles);
+  talk_prefill_kernel<HD, HPW, SHARED><<<dim3(n), dim3(64 * TW), smem, stream>>>(a, cu_q, ctx, tiles);
   return (int)hipGetLastError();
+}
+
+template <int HD, int HPW>
+int launch_prefill(const TalkArgs& a, const int* cu_q, const int* ctx, const int* tiles, int n,
+                   hipStream_t stream) {
+  if constexpr (HPW > 1)
+    if (a.Hq / a.Hkv % HPW) return launch_prefill_as<HD, HPW, false>(a, cu_q, ctx, tiles, n, stream);
+  return launch_prefill_as<HD, HPW, true>(a, cu_q, ctx, tiles, n, stream);
 }
 
 }  // namespace

@@ -551,7 +551,7 @@ class Talk:
     sink: torch.Tensor          # fp32 [H]
 
 
-TALK_QT = 16                    # query rows per prefill workgroup (talk.hip)
+TALK_QT = 8                     # query rows per prefill workgroup (talk.hip)
 TALK_MAX_HEADS = 32             # heads of the MFMA kernels (head sizes 64, 128)
 TALK_PART = 128                 # least keys of a decode partition
 
