@@ -110,8 +110,7 @@ __global__ void __launch_bounds__(64 * TW, 2) talk_prefill_kernel(
   char* const sS = talk_sm;                              // 2 x raw scores: group = query, row = key
   char* const sP = talk_sm + 2 * IMG;                    // 2 x weights: group = query, row = head
   float* const sAl = reinterpret_cast<float*>(sP + 2 * IMG);    // 2 x [32 heads][8]
-  // neighbouring tiles, which walk the same pages, on one XCD; long walks first
-  const int tile = gridDim.x - 1 - xcd_remap(blockIdx.x, gridDim.x);
+  const int tile = blockIdx.x;
   const int seq = tiles[2 * tile], q0 = tiles[2 * tile + 1];
   const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4, cq = c & 7, cs = c >> 3;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);

@@ -212,7 +212,7 @@ class LayerListModel:
         host = {}
         for key, m in self._plans.items():
             more, host[key] = m.build_plan(qlens, ctx, nd)
-            items += more
+            items += [x for x in more if x[0] not in {name for name, _ in items}]
         return items, host
 
     def bind_plan(self, dev: dict, host: dict) -> dict:

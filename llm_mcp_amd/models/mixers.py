@@ -754,14 +754,14 @@ class TalkingAttentionMixer(Mixer):
         self.rows = self.qkv + H * D
         self.proj = {"in": (self.rows, width), "o": (width, H * D)}
         self.q_per_tile = ops.TALK_QT
-        self.plan_key = ("talk",)
+        self.plan_key = ("talk", self.chunk)
 
     def build_plan(self, qlens, ctx, seq0):
         return [("quads", mixer_ops.row_quads(qlens, ctx, seq0)),
-                ("talk", mixer_ops.row_tiles(qlens, ops.TALK_QT).reshape(-1))], None
+                (f"talk{self.chunk}", mixer_ops.talk_tiles(qlens, ctx, self.chunk).reshape(-1))], None
 
     def bind_plan(self, dev, host):
-        return dev["quads"], dev["talk"]
+        return dev["quads"], dev[f"talk{self.chunk}"]
 
     def _heads(self, t, n, d, pairs=False):
         """[n * d, ...] rows -> [n * D, ...], each head padded with zeros."""

@@ -556,6 +556,26 @@ TALK_MAX_HEADS = 32             # heads of the MFMA kernels (head sizes 64, 128)
 TALK_PART = 128                 # least keys of a decode partition
 
 
+def talk_tiles(qlens, ctx, chunk: int) -> np.ndarray:
+    """``row_tiles`` of TALK_QT rows in dispatch order: blocks of 8 neighbours,
+    which walk the same pages, keep to one XCD (workgroup b runs on XCD b % 8),
+    the longest walks first."""
+    t = row_tiles(qlens, TALK_QT)
+    n = np.asarray(qlens, np.int64)[t[:, 0]]
+    p0 = np.asarray(ctx, np.int64)[t[:, 0]] - n + t[:, 1]
+    p1 = p0 + np.minimum(TALK_QT, n - t[:, 1]) - 1
+    first = p0 // chunk * chunk if chunk else np.zeros_like(p0)
+    walk = p1 // 32 - first // 32 + 1
+    blocks = -(-len(t) // 64) * 8
+    at = np.full(blocks * 8, -1)
+    at[:len(t)] = np.arange(len(t))
+    cost = np.zeros(blocks * 8, np.int64)
+    cost[:len(t)] = walk
+    order = np.argsort(-cost.reshape(blocks, 8).max(1), kind="stable")
+    at = at.reshape(blocks, 8)[order].reshape(-1, 8, 8).transpose(0, 2, 1).reshape(-1)
+    return t[at[at >= 0]]
+
+
 def talk_kernel_ok(Hq: int, Hkv: int, D: int) -> bool:
     """Geometries of the MFMA kernels (bf16)."""
     return D in (64, 128) and Hq <= TALK_MAX_HEADS and Hq % Hkv == 0 and Hq // Hkv <= 16
@@ -572,7 +592,7 @@ def talking_attention(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, ctx
     sigmoid(gate) into ``out`` (any row stride).
 
     Rows before ``num_decode`` are single rows of their sequences; ``tiles``
-    (``row_tiles`` of TALK_QT rows) covers the others.  bf16 rows of
+    (``talk_tiles``) covers the others.  bf16 rows of
     ``talk_kernel_ok`` geometries run on MFMA."""
     _, Hkv, BS, D = k_cache.shape
     T, S, nd = q.shape[0], ctx.numel(), num_decode
