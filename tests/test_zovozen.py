@@ -1,0 +1,555 @@
+"""Zovozen in the serving engine against the plain reference of
+``zovozen_oracle``: whole prompts, token-by-token decoding, portions, batches,
+slots and pages that are used again, chunks' edges, generation -- on the CPU
+references and on the GPU kernels, in bf16 and fp32."""
+import json
+
+import numpy as np
+import pytest
+import torch
+
+import zovozen_oracle as oracle
+from llm_mcp_amd.engine.engine import EngineConfig, LLMEngine, SamplingParams
+from llm_mcp_amd.models import config as mc
+from llm_mcp_amd.models.zovozen import ZovozenModel, tensor_shapes
+from llm_mcp_amd.models.registry import model_class
+from llm_mcp_amd.models.weights import load_weights, save_layer_list
+from zovozen_cases import (CASES, attention, config, dense, memory, moe, par, shapes, tokens,
+                           weights)
+
+GPU = pytest.mark.gpu
+RUNS = [pytest.param("cpu", "float32", id="cpu-fp32"),
+        pytest.param("cuda", "float32", id="gpu-fp32", marks=GPU),
+        pytest.param("cuda", "bfloat16", id="gpu-bf16", marks=GPU)]
+# rms error over the vocabulary, relative to the logits' own rms
+TOL = {"float32": 5e-5, "bfloat16": 0.08}
+# what a mistake must move (the upper quarter of the positions)
+SHOWS = {"float32": 0.02, "bfloat16": 0.04}
+# positions that may be over: a dot product with the memory's n that nearly cancels
+# divides by a difference of roundings; in bf16 also a near tie of a router that falls
+# the other way, which the tokens behind it see.  None may be far over in fp32.
+STRAY = {"float32": 0.02, "bfloat16": 0.05}
+FAR = {"float32": 1e-3, "bfloat16": float("inf")}
+
+
+def product_config(cfg, name="case"):
+    return mc.ZovozenConfig.from_json(json.loads(json.dumps(cfg)), name)
+
+
+def engine(cfg, W, device, dtype, tokens=512, seqs=4, graphs=False, **kw):
+    ecfg = dict(max_num_seqs=seqs, max_batched_tokens=512, mixed_prefill_tokens=0,
+                max_model_len=512, kv_cache_tokens=tokens, use_graphs=graphs, dtype=dtype)
+    ecfg.update(kw)
+    return LLMEngine(EngineConfig(**ecfg), device=device, model_cfg=product_config(cfg), weights=W)
+
+
+@pytest.fixture(autouse=True, scope="module")
+def _one_thread():
+    """Tiny tensors: intra-op threads only cost."""
+    n = torch.get_num_threads()
+    torch.set_num_threads(1)
+    yield
+    torch.set_num_threads(n)
+
+
+_MADE = {}
+
+
+def weights_for(cfg, dtype, seed=0):
+    key = (json.dumps(cfg), dtype == "bfloat16", seed)
+    if key not in _MADE:
+        _MADE[key] = weights(cfg, seed, calm=key[1])
+    return _MADE[key]
+
+
+def reference(cfg, W, toks):
+    key = (id(W), tuple(toks))            # W of ``weights_for``: kept
+    if key not in _MADE:
+        _MADE[key] = oracle.forward(cfg, W, toks)
+    return _MADE[key]
+
+
+def errors(got, want):
+    got, want = got.double(), want.double()
+    d = got - want
+    d = d - d.mean(-1, keepdim=True)
+    return d.pow(2).mean(-1).sqrt() / want.std()
+
+
+class Tally:
+    """Errors of a test's positions, judged together."""
+
+    def __init__(self, dtype):
+        self.dtype, self.errs, self.where = dtype, [], []
+
+    def add(self, got, want, what=""):
+        e = errors(got, want)
+        self.errs += e.tolist()
+        self.where += [f"{what}+{k}" for k in range(len(e))]
+
+    def done(self):
+        bad = [(w, round(e, 6)) for w, e in zip(self.where, self.errs) if not e < TOL[self.dtype]]
+        n = len(self.errs)
+        assert n and len(bad) <= max(1, STRAY[self.dtype] * n) and max(self.errs) < FAR[self.dtype], \
+            f"{len(bad)} of {n}: {bad[:6]}"
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+@pytest.mark.parametrize("case", sorted(CASES))
+def test_whole_prompt_and_decode(case, device, dtype):
+    """Every position of one prompt in one step, then the same tokens with the
+    tail one by one: the state and cache the prompt left must be the ones a
+    longer prompt would have used."""
+    cfg = CASES[case]
+    W = weights_for(cfg, dtype)
+    n, tail = 90, 12
+    toks = tokens(cfg, n)
+    want = reference(cfg, W, toks)
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    t.add(e.feed([(1, toks, list(range(n)))], [1]), want, "whole")
+    t.add(e.feed([(2, toks[:n - tail], list(range(n - tail)))]), want[:n - tail], "prompt")
+    for i in range(n - tail, n):
+        t.add(e.feed([(2, toks[i:i + 1], [0])], [2] if i == n - 1 else []), want[i:i + 1], f"at {i}")
+    t.done()
+    assert e.sched.kv_usage == 0.0
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+@pytest.mark.parametrize("case", ["mixed", "odd"])
+def test_token_by_token_from_the_start(case, device, dtype):
+    cfg = CASES[case]
+    W = weights_for(cfg, dtype)
+    toks = tokens(cfg, 50, seed=3)
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    t.add(torch.cat([e.feed([(7, [x], [0])]) for x in toks]), reference(cfg, W, toks))
+    t.done()
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+@pytest.mark.parametrize("case", ["mixed", "odd", "fast"])
+def test_portions(case, device, dtype):
+    """Portions cut inside pages, chunks and scan chunks, down to two tokens and one."""
+    cfg = CASES[case]
+    W = weights_for(cfg, dtype)
+    n = 150
+    toks = tokens(cfg, n, seed=5)
+    want = reference(cfg, W, toks)
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    for k, cuts in enumerate([[2] * 20, [31, 1, 2, 33, 64, 3, 16], [65, 2, 2], [1, 149]]):
+        at = 0
+        for c in cuts:
+            y = e.feed([(k + 1, toks[at:at + c], list(range(c)))])
+            t.add(y, want[at:at + c], f"cuts {k} at {at}")
+            at += c
+        e.feed([], [k + 1])
+    t.done()
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+@pytest.mark.parametrize("case", ["mixed", "beyond"])
+def test_unequal_requests_share_steps_pages_and_slots(case, device, dtype):
+    """Up to four live requests of unequal lengths in shared steps, portions
+    beside decoded tokens, some left out of a step; requests end and their
+    pages and slots go to the next ones (seven requests, a pool of four)."""
+    cfg = CASES[case]
+    W = weights_for(cfg, dtype)
+    lens = [70, 1, 33, 64, 5, 90, 32]
+    reqs = {i + 1: tokens(cfg, n, seed=10 + i) for i, n in enumerate(lens)}
+    want = {i: reference(cfg, W, t) for i, t in reqs.items()}
+    e, t = engine(cfg, W, device, dtype, tokens=288), Tally(dtype)
+    rng = np.random.default_rng(0)
+    at, live, waiting = {}, [], list(reqs)
+    while waiting or live:
+        while waiting and len(live) < 4:
+            live.append(waiting.pop(0))
+            at[live[-1]] = 0
+        ents, end, spans = [], [], []
+        for r in live:
+            if len(ents) and rng.random() < 0.25:
+                continue                        # left out of this step
+            left = len(reqs[r]) - at[r]
+            n = int(min(left, rng.choice([1, 1, 2, 3, 17, 32, 40])))
+            ents.append((r, reqs[r][at[r]:at[r] + n], list(range(n))))
+            spans.append((r, at[r], n))
+            at[r] += n
+            if at[r] == len(reqs[r]):
+                end.append(r)
+        y = e.feed(ents, end)
+        k = 0
+        for r, a, n in spans:
+            t.add(y[k:k + n], want[r][a:a + n], f"request {r} at {a}")
+            k += n
+        live = [r for r in live if r not in end]
+    t.done()
+    assert e.sched.kv_usage == 0.0
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_request_alone_and_in_a_batch_agree(device, dtype):
+    cfg = CASES["beyond"]
+    W = weights_for(cfg, dtype)
+    toks = [tokens(cfg, n, seed=20 + n) for n in (3, 65, 40)]
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    alone = [e.feed([(9, x, list(range(len(x))))], [9]) for x in toks]
+    both = e.feed([(i + 1, x, list(range(len(x)))) for i, x in enumerate(toks)], [1, 2, 3])
+    t.add(both, torch.cat(alone))
+    t.done()
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_long_decoding(device, dtype):
+    """Decoded tokens pass over the chunks and pages of the prompt."""
+    cfg = CASES["mixed"]
+    W = weights_for(cfg, dtype)
+    toks = tokens(cfg, 240, seed=50)
+    want = reference(cfg, W, toks)
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    e.feed([(1, toks[:30], [])])
+    for i in range(30, 240):
+        y = e.feed([(1, toks[i:i + 1], [0] if i % 5 == 4 or i < 80 else [])])
+        if y.shape[0]:
+            t.add(y, want[i:i + 1], f"at {i}")
+    t.done()
+
+
+def sharp_chunk(chunk, back):
+    """One layer whose attention looks for the token ``back`` places back and
+    hardly anything else: constant queries and keys, and a rotation of the query
+    that makes that distance the best match."""
+    R = 32
+    rot = dict(base=float(3 * chunk), dims=R, scaling=dict(factor=1.5))
+    left = dict(heads=1, kv_heads=1, dim=R, vdim=16, mask=dict(size=chunk), rot=rot, scale=3.0)
+    cfg = config([par(None, left, memory(1, 8, 8), (1.0, 0.0))], width=32, vocab=40)
+    W = {k: v.float() for k, v in weights(cfg, 3).items()}
+    a = oracle.frequencies(rot).float() * back
+    # carried by an embedding column all tokens share
+    W["embed"][:, 0] = 4.0
+    x = "l0.mix.left."
+    for n in "qk":
+        W[x + n], W[x + n + ".b"] = torch.zeros(R, 32), torch.zeros(R)
+        W[x + n + ".norm"] = torch.ones(R)
+    W[x + "q"][:, 0] = torch.cat([a.cos(), -a.sin()])         # turned back by that many
+    W[x + "k"][:R // 2, 0] = 1.0
+    W[x + "talk"], W[x + "temp"] = torch.ones(1, 1), torch.ones(1)
+    W[x + "sink"] = torch.full((1,), 2.0)
+    return cfg, {k: v.to(torch.bfloat16) for k, v in W.items()}
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+@pytest.mark.parametrize("chunk", [31, 32, 33, 64, 65])
+def test_the_edge_of_a_chunk(chunk, device, dtype):
+    """Rows look for the token half a chunk back: in the chunk's second half it
+    is there, in the first it is the other side of the edge.  Around page
+    borders, in prompts, portions and decoding: a chunk one off moves the logits,
+    and so does no chunk."""
+    back = chunk // 2
+    cfg, W = sharp_chunk(chunk, back)
+    n = 2 * chunk + 40
+    toks = tokens(cfg, n, seed=9)
+    want = oracle.forward(cfg, W, toks)
+    p = torch.arange(n)
+    for size in (chunk - 1, chunk + 1, 4 * n):
+        c = json.loads(json.dumps(cfg))
+        c["layers"][0]["mixer"]["left"]["mask"]["size"] = size
+        e = errors(oracle.forward(c, W, toks), want)
+        # rows whose token is hidden by one of both chunkings only
+        seen = lambda s: (p - back >= 0) & (p // s == (p - back) // s)
+        assert float(e[seen(chunk) != seen(size)].quantile(0.25)) > 0.15   # the weights show it
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    t.add(e.feed([(1, toks, list(range(n)))], [1]), want, "whole")
+    at = 0
+    for k in (chunk - 1, 1, 1, 2, 5, 30):
+        t.add(e.feed([(2, toks[at:at + k], list(range(k)))]), want[at:at + k], f"portion {at}")
+        at += k
+    for i in range(at, n):
+        t.add(e.feed([(2, toks[i:i + 1], [0])]), want[i:i + 1], f"decoded {i}")
+    t.done()
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_a_token_far_back(device, dtype):
+    """The memory carries a distant token across chunks: one token of a prompt is
+    exchanged, and every later position must move as the reference's does, in
+    the prompt and over portions and decoding."""
+    cfg = config([par(None, attention(chunk=3), memory(2, 16, 16), (0.5, 1.0))] * 2)
+    W = dict(weights(cfg, 12))
+    for i in range(2):
+        x = f"l{i}.mix.right."
+        W[x + "f"], W[x + "f.b"] = W[x + "f"] * 0, W[x + "f.b"] * 0 + 6.5     # hardly any decay
+        W[x + "i"] = W[x + "i"] * 0.1
+    a = tokens(cfg, 200, seed=13)
+    b = a[:3] + [(a[3] + 1) % cfg["vocab"]] + a[4:]
+    want = [oracle.forward(cfg, W, x) for x in (a, b)]
+    e = errors(want[0], want[1])
+    assert float(e[20:60].median()) > 0.1 and float(e[150:].median()) > 0.04
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    for k, x in enumerate((a, b)):
+        y = [e.feed([(k, x[i:j], list(range(j - i)))]) for i, j in ((0, 70), (70, 72), (72, 180))]
+        y += [e.feed([(k, x[i:i + 1], [0])]) for i in range(180, 200)]
+        t.add(torch.cat(y), want[k], f"text {k}")
+        e.feed([], [k])
+    t.done()
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_the_first_tokens(device, dtype):
+    """Sequences of one to a few tokens, where the memory's maximum starts and the
+    sink weighs most: alone, in one batch, decoded."""
+    cfg = CASES["mixed"]
+    W = weights_for(cfg, dtype)
+    toks = [tokens(cfg, n, seed=70 + n) for n in (1, 2, 3, 5)]
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    y = e.feed([(i + 1, x, list(range(len(x)))) for i, x in enumerate(toks)], [1, 2, 3, 4])
+    t.add(y, torch.cat([reference(cfg, W, x) for x in toks]), "batch")
+    for i in range(5):
+        t.add(e.feed([(9, toks[3][i:i + 1], [0])]), reference(cfg, W, toks[3])[i:i + 1], "decoded")
+    t.done()
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_generation_is_greedy_of_the_reference(device, dtype):
+    """The engine's own entry point: batches of unequal prompts through the
+    scheduler, the sampler and (on the GPU) the captured decode graphs."""
+    cfg = CASES["mixed"]
+    W = weights_for(cfg, dtype, 4)
+    e = engine(cfg, W, device, dtype, graphs=device == "cuda")
+    prompts = [tokens(cfg, n, seed=30 + n) for n in (1, 5, 40, 66, 2, 31)]
+    new = 24
+    outs = e.generate(prompts, SamplingParams(temperature=0, max_tokens=new, ignore_eos=True))
+    for p, o in zip(prompts, outs):
+        assert len(o) == new
+        lg = oracle.forward(cfg, W, p + o)[len(p) - 1:-1]
+        short = lg.max(-1).values - lg[torch.arange(new), torch.tensor(o)]
+        # a token may only differ from the reference's where that is a near tie
+        bad = int((short > 4 * TOL[dtype] * float(lg.std())).sum())
+        assert bad <= STRAY[dtype] * new
+    if device == "cuda":
+        assert e.stats["graph_steps"] > 0
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_preemption_recomputes_the_state(device, dtype):
+    """A pool too small for every request: preempted sequences lose pages and
+    slot and come back through a recomputed prompt."""
+    cfg = CASES["mixed"]
+    W = weights_for(cfg, dtype, 6)
+    e = engine(cfg, W, device, dtype, tokens=192, graphs=device == "cuda")
+    prompts = [tokens(cfg, 50, seed=40 + i) for i in range(4)]
+    outs = e.generate(prompts, SamplingParams(temperature=0, max_tokens=30, ignore_eos=True))
+    assert e.sched.preemptions > 0
+    for p, o in zip(prompts, outs):
+        lg = oracle.forward(cfg, W, p + o)[len(p) - 1:-1]
+        short = lg.max(-1).values - lg[torch.arange(len(o)), torch.tensor(o)]
+        assert len(o) == 30
+        assert int((short > 4 * TOL[dtype] * float(lg.std())).sum()) <= STRAY[dtype] * 30
+
+
+@GPU
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_captured_graphs_replay_what_eager_steps_compute(dtype):
+    """The same streams through captured decode graphs and through eager steps,
+    in batches that grow and shrink between replays."""
+    cfg = CASES["fast"]
+    W = weights_for(cfg, dtype, 8)
+    prompts = [tokens(cfg, n, seed=60 + n) for n in (4, 35, 1, 140, 20, 9)]
+    sp = SamplingParams(temperature=0, max_tokens=20, ignore_eos=True)
+    outs = []
+    for graphs in (True, False):
+        e = engine(cfg, W, "cuda", dtype, seqs=3, graphs=graphs)
+        outs.append(e.generate(prompts, sp))
+    assert outs[0] == outs[1]
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_a_planted_mistake_shows(device, dtype):
+    """The weights of the tests are sharp enough: the reference with one
+    mechanism wrong is far outside the tolerance the product meets."""
+    cfg = CASES["mixed"]
+    W = weights_for(cfg, dtype)
+    toks = tokens(cfg, 70)
+    got = engine(cfg, W, device, dtype).feed([(1, toks, list(range(70)))])
+    t = Tally(dtype)
+    t.add(got, reference(cfg, W, toks))
+    t.done()
+
+    def changed(fn):
+        c = json.loads(json.dumps(cfg))
+        fn(c)
+        return c, W
+    left, right = (lambda c, n=n: c["layers"][1]["mixer"][n] for n in ("left", "right"))
+
+    def tensor(name, fn):
+        return cfg, {**W, name: fn(W[name].float()).to(torch.bfloat16)}
+    x, y = "l1.mix.left.", "l1.mix.right."
+    wrong = {
+        "left scale": changed(lambda c: c["layers"][1]["mixer"].update(left_scale=1.6)),
+        "right scale": changed(lambda c: c["layers"][1]["mixer"].update(right_scale=0.4)),
+        "rotation": changed(lambda c: left(c)["rot"].update(base=50.0)),
+        "rotated channels": changed(lambda c: left(c)["rot"].update(dims=24)),
+        "length scaling": changed(lambda c: left(c)["rot"]["scaling"].update(factor=1.0)),
+        "attention scale": changed(lambda c: left(c).update(scale=1.2)),
+        "chunk": changed(lambda c: left(c)["mask"].update(size=20)),
+        "cap": changed(lambda c: right(c).update(gate_cap=1.0)),
+        "top": changed(lambda c: c["layers"][1]["mlp"]["router"].update(top=1)),
+        "groups": changed(lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(keep=1)),
+        "correction": tensor("l1.mlp.correction", lambda t: t * 0),
+        "sink": tensor(x + "sink", lambda t: t * 0 - 9.0),
+        "talk": tensor(x + "talk", lambda t: torch.eye(t.shape[0])),
+        "talk transposed": tensor(x + "talk", lambda t: t.t().contiguous()),
+        "temperature": tensor(x + "temp", lambda t: t * 0 + 1.0),
+        "query bias": tensor(x + "q.b", lambda t: t * 0),
+        "query norm": tensor(x + "q.norm", lambda t: t * 0 + 1.0),
+        "key norm": tensor(x + "k.norm", lambda t: t * 0 + 1.0),
+        "value bias": tensor(x + "v.b", lambda t: t * 0),
+        "attention gate": tensor(x + "g", lambda t: t * 0),
+        "output bias": tensor(x + "o.b", lambda t: t * 0),
+        "input gate": tensor(y + "i", lambda t: t * 0),
+        "forget gate": tensor(y + "f.b", lambda t: t - 2.0),
+        "memory gain": tensor(y + "norm", lambda t: t * 0 + 1.0),
+        "memory gate": tensor(y + "g", lambda t: t * 0),
+        "up bias": tensor("l0.mlp.up.b", lambda t: t * 0),
+        "down bias": tensor("l0.mlp.down.b", lambda t: t * 0),
+        "mixer norm": tensor("l1.norm1", lambda t: t * 0 + 1.0),
+        "feed-forward norm": tensor("l0.norm2", lambda t: t * 0 + 1.0),
+    }
+    if dtype == "bfloat16":            # calm routers rank the groups by the correction alone
+        del wrong["groups"]
+    for name, (c, w) in wrong.items():
+        e = errors(got, oracle.forward(c, w, toks))
+        assert float(e.quantile(0.75)) > SHOWS[dtype], f"{name}: {float(e.quantile(0.75)):.4f}"
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_residual_after_every_layer(device, dtype):
+    cfg = CASES["mixed"]
+    toks = tokens(cfg, 40, seed=2)
+    W = weights_for(cfg, dtype)
+    e = engine(cfg, W, device, dtype)
+    got, run = [], e.model.forward
+
+    def forward(*a, **k):
+        return run(*a, layers_out=got, **k)
+    e.model.forward = forward
+    e.feed([(1, toks, [0])])
+    want = []
+    oracle.forward(cfg, W, toks, want)
+    assert len(got) == len(want) == len(cfg["layers"])
+    for a, b in zip(got, want):
+        e_ = ((a.cpu().double() - b).pow(2).mean(-1).sqrt() / b.std())
+        assert float(e_.median()) < TOL[dtype] / 2
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_a_wide_shared_expert(device, dtype):
+    cfg = config([par(moe(ff=20, shared=1100)), par(dense())])
+    W = weights_for(cfg, dtype)
+    toks = tokens(cfg, 40, seed=4)
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    y = [e.feed([(1, toks[a:b], list(range(b - a)))]) for a, b in ((0, 17), (17, 18), (18, 40))]
+    t.add(torch.cat(y), reference(cfg, W, toks))
+    t.done()
+
+
+# ------------------------------------------------- configuration, loading ----
+def test_checkpoint_directory_round_trip(tmp_path):
+    cfg = CASES["mixed"]
+    W = weights(cfg)
+    pc = product_config(cfg)
+    assert {k: tuple(v) for k, v in tensor_shapes(pc).items()} == shapes(cfg)
+    save_layer_list(W, pc, str(tmp_path))
+    back = mc.resolve(str(tmp_path))
+    assert back.family == "zovozen" and model_class(back) is ZovozenModel
+    assert (back.layers, back.vocab_size, back.hidden_size, back.rms_eps) == \
+        (pc.layers, pc.vocab_size, pc.hidden_size, pc.rms_eps)
+    W2 = load_weights(str(tmp_path), back, "cpu")
+    assert all(torch.equal(W[k], W2[k]) for k in W)
+    assert back.params == sum(t.numel() for t in W.values())
+    save_layer_list(dict(W, embed=W["embed"][:-1]), pc, str(tmp_path))
+    with pytest.raises(ValueError, match="embed"):
+        load_weights(str(tmp_path), back, "cpu")
+
+
+def test_unknown_mechanisms_are_refused():
+    with pytest.raises(ValueError, match="mixer"):
+        product_config(config([{**par(), "type": "retention"}]))
+    with pytest.raises(ValueError, match="feed-forward"):
+        product_config(config([par({**dense(), "kind": "glu"})]))
+    for bad in (par(None, attention(chunk=0)), par(None, attention(heads=3)),
+                par(None, attention(dims=26)), par(None, attention(dims=5)),
+                par(None, None, memory(cap=0.0)), par(moe(top=10)), par(moe(groups=4)),
+                par(moe(keep=4)), par(moe(top=4, keep=1)), par(moe(identity=-1))):
+        with pytest.raises(ValueError):
+            ZovozenModel(product_config(config([bad])), "cpu")
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+def test_what_a_configuration_may_leave_out(device, dtype):
+    """No rotation, no chunks, no scaling, no groups, no identity experts, no
+    shared expert, no feed-forward."""
+    left = attention()
+    del left["rot"], left["mask"]
+    plain = attention(chunk=20)
+    del plain["rot"]["scaling"]
+    f = moe(5, 0, 2)
+    del f["router"]["groups"], f["router"]["identity"], f["shared"]
+    cfg = config([par(f, left), par(None, plain)])
+    full = json.loads(json.dumps(cfg))          # the same in full, for the reference
+    full["layers"][0]["mixer"]["left"].update(mask=dict(size=1000), rot=dict(base=1.0, dims=2, scaling=dict(
+        factor=1e30)))
+    W = weights_for(cfg, dtype)
+    toks = tokens(cfg, 60)
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    y = [e.feed([(1, toks[a:b], list(range(b - a)))]) for a, b in ((0, 35), (35, 36), (36, 60))]
+    t.add(torch.cat(y), oracle.forward(full, W, toks))
+    t.done()
+
+
+def test_presets_and_layer_subsets():
+    full = mc.resolve("zovozen-8b")
+    assert 7.0 < full.params_b < 8.5
+    assert mc.resolve("zovozen-8b@L3").num_layers == 3
+    e = LLMEngine(EngineConfig(model="tiny-zovozen", max_num_seqs=2, max_batched_tokens=64,
+                               max_model_len=128, use_graphs=False), device="cpu")
+    out = e.generate([[1, 2, 3], [9] * 40], SamplingParams(temperature=0.8, seed=3, max_tokens=5,
+                                                          ignore_eos=True))
+    assert [len(o) for o in out] == [5, 5] and e.sched.prefix_hits == 0
+    assert e.model.weight_bytes() > 0
+
+
+@pytest.mark.parametrize("device,dtype", RUNS)
+@pytest.mark.parametrize("layers", [[par()], [par(moe()), par(dense(), attention(8, 4, 16, 16, 300, 16))]],
+                         ids=["one layer", "unequal caches"])
+def test_models_of_few_layers(layers, device, dtype):
+    cfg = config(layers)
+    W = weights_for(cfg, dtype)
+    toks = tokens(cfg, 47)
+    e, t = engine(cfg, W, device, dtype), Tally(dtype)
+    y = torch.cat([e.feed([(1, toks[:20], list(range(20)))]),
+                   e.feed([(1, toks[20:], list(range(27)))])])
+    t.add(y, reference(cfg, W, toks))
+    t.done()
+
+
+def test_trace_replay(tmp_path):
+    from llm_mcp_amd.engine import trace
+    cfg = CASES["mixed"]
+    W = weights_for(cfg, "float32")
+    save_layer_list(W, product_config(cfg), str(tmp_path / "m"))
+    e = trace.build_engine(str(tmp_path / "m"), "float32", 130, 4, "cpu")
+    toks = tokens(cfg, 40)
+    want = reference(cfg, W, toks)
+    out = tmp_path / "out"
+    out.mkdir()
+    lines = [json.dumps(s) + "\n" for s in (
+        {"step": 0, "entries": [{"id": "x", "tokens": toks[:11], "want": [10, 3]}], "end": []},
+        {"step": 1, "entries": [{"id": "y", "tokens": toks[:2], "want": [1]},
+                                {"id": "x", "tokens": toks[11:], "want": [0, 28]}],
+         "end": ["x", "y"]})]
+    said = []
+    trace.replay(e, lines, str(out), said.append)
+    assert said == ["done 0", "done 1"]
+    t = Tally("float32")
+    for step, places in ((0, [10, 3]), (1, [1, 11, 39])):
+        got = np.fromfile(out / f"{step}.f32", "<f4").reshape(-1, cfg["vocab"])
+        t.add(torch.from_numpy(got.copy()), want[places])
+    t.done()
