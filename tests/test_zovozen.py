@@ -22,7 +22,7 @@ RUNS = [pytest.param("cpu", "float32", id="cpu-fp32"),
         pytest.param("cuda", "float32", id="gpu-fp32", marks=GPU),
         pytest.param("cuda", "bfloat16", id="gpu-bf16", marks=GPU)]
 # rms error over the vocabulary, relative to the logits' own rms
-TOL = {"float32": 5e-5, "bfloat16": 0.08}
+TOL = {"float32": 1.2e-4, "bfloat16": 0.08}
 # what a mistake must move (the upper quarter of the positions)
 SHOWS = {"float32": 0.02, "bfloat16": 0.04}
 # positions that may be over: a dot product with the memory's n that nearly cancels

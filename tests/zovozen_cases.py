@@ -104,7 +104,8 @@ def weights(cfg, seed=0, calm=False):
     from 1, mixed heads, sinks that weigh, corrections that outweigh scores,
     memories that neither vanish nor hold.  ``calm``: routers whose choices stay
     clear of ties (a choice that falls the other way in bf16 moves every later
-    token)."""
+    token), memories whose queries resemble the keys (the divisor n q of others
+    nearly cancels now and then)."""
     g = torch.Generator().manual_seed(seed)
     out = {}
     for name, s in shapes(cfg).items():
@@ -131,6 +132,9 @@ def weights(cfg, seed=0, calm=False):
         elif name != "embed":
             t = 1.5 * t / math.sqrt(s[-1])
         out[name] = t.to(torch.bfloat16)
+        if calm and name.endswith("right.k"):
+            q = name[:-1] + "q"
+            out[q] = (0.5 * out[q].float() + t).to(torch.bfloat16)
     return out
 
 
