@@ -356,6 +356,11 @@ __global__ void __launch_bounds__(64 * TW, 2) talk_prefill_kernel(
 }
 
 // ---------------------------------------------------------------- decode ----
+// keys per partition: whole pages, at most max_parts partitions
+__device__ __forceinline__ int decode_part(int n, int part_tokens, int max_parts) {
+  return max(part_tokens, ((n + max_parts - 1) / max_parts + BS - 1) / BS * BS);
+}
+
 // grid (max_parts, rows), block 64 * min(8, Hkv); KPW: key heads per wave
 template <int HD, int KPW>
 __global__ void __launch_bounds__(512) talk_decode_kernel(TalkArgs a, const int* __restrict__ ctx_lens,
@@ -366,7 +371,7 @@ __global__ void __launch_bounds__(512) talk_decode_kernel(TalkArgs a, const int*
   constexpr int KS = HD / 32, NT = HD / 16;
   const int b = blockIdx.y, p = blockIdx.x;
   const int ctx = ctx_lens[b], lo = chunk_first(a.chunk, ctx - 1), base = lo / BS * BS;
-  const int part = effective_part(ctx - base, part_tokens, max_parts);
+  const int part = decode_part(ctx - base, part_tokens, max_parts);
   const int nparts = (ctx - base + part - 1) / part;
   if (p >= nparts) return;
   const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
@@ -517,7 +522,7 @@ __global__ void __launch_bounds__(64) talk_reduce_kernel(TalkArgs a, const int* 
                                                          int part_tokens, int max_parts) {
   const int h = blockIdx.x, b = blockIdx.y, d = 4 * threadIdx.x;
   const int ctx = ctx_lens[b], n = ctx - chunk_first(a.chunk, ctx - 1) / BS * BS;
-  const int part = effective_part(n, part_tokens, max_parts);
+  const int part = decode_part(n, part_tokens, max_parts);
   const int nparts = (n + part - 1) / part;
   if (nparts <= 1) return;
   const long at = ((long)b * a.Hq + h) * max_parts;

@@ -553,7 +553,7 @@ class Talk:
 
 TALK_QT = 8                     # query rows per prefill workgroup (talk.hip)
 TALK_MAX_HEADS = 32             # heads of the MFMA kernels (head sizes 64, 128)
-TALK_PART = 128                 # least keys of a decode partition
+TALK_PART = 64                  # least keys of a decode partition
 
 
 def talk_tiles(qlens, ctx, chunk: int) -> np.ndarray:
